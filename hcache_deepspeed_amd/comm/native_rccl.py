@@ -2,7 +2,7 @@
 
 ``RcclCommunicator(group)`` creates ONE private RCCL communicator for a ``torch.distributed`` group: rank 0 of the
 group draws the unique id in C++, it is broadcast once over the existing process group, and every rank calls
-``ncclCommInitRank`` on its current HIP device. The C++ side issues on a high-priority communication stream (from torch's
+``ncclCommInitRank`` on its current HIP device. The C++ side issues on its own communication stream (from torch's
 stream pool) and keeps a ring of completion events:
 
 * every collective is ordered after the work queued on the caller's stream by a GPU-side event wait (no host sync),
@@ -78,7 +78,7 @@ class RcclCommunicator:
         self.world = tdist.get_world_size(group) if tdist.is_initialized() else 1
         from .setup import collective_setup
         # torch's pooled streams are never destroyed, so record_stream() events on it outlive this object
-        self.stream = torch.cuda.Stream(priority=-1)
+        self.stream = torch.cuda.Stream()
         self._h = None
 
         # failure-symmetric (comm/setup.py): rank 0's unique id travels in the same all_gather_object that agrees on

@@ -4,7 +4,7 @@
 // z1.cpp:72 (a private ncclComm_t with ncclAllGather / ncclReduceScatter / ncclAllReduce on dedicated streams),
 // SURVEY.md §2.10 N20 and §5.8 "Native path". Not a translation: this layer owns
 //   * the RCCL communicator (one per process group, created from a unique id that python broadcasts once),
-//   * ONE high-priority communication HIP stream per communicator, so collectives never queue behind compute
+//   * ONE communication HIP stream per communicator, so collectives never queue behind compute
 //     (created by torch's stream pool and passed in: torch never destroys pooled streams, so the caching
 //     allocator's record_stream events on it stay valid after the communicator is gone),
 //   * a ring of completion events: every collective first waits (on the GPU, hipStreamWaitEvent) for the caller's
@@ -122,7 +122,7 @@ HDS_EXPORT int hds_rccl_unique_id(char* out128) {
   return rc;
 }
 
-// Create the communicator on the CURRENT HIP device (python sets it), issuing on `stream` (a high-priority stream
+// Create the communicator on the CURRENT HIP device (python sets it), issuing on `stream` (a stream
 // owned by the caller). Returns a handle or null (*err set).
 HDS_EXPORT void* hds_rccl_init(const char* id128, int nranks, int rank, void* stream, int* err) {
   *err = 3;

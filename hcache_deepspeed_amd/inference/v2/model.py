@@ -89,7 +89,7 @@ class RaggedTransformer:
         else:
             self.cos = self.sin = None
         self.kv_cache = None
-        self.copy_stream = torch.cuda.Stream(device, priority=-1) if device.type == "cuda" else None
+        self.copy_stream = torch.cuda.Stream(device) if device.type == "cuda" else None
         self._decode_graphs = {}
         self._graph_pool = None
         import os as _os

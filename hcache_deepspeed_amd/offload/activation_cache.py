@@ -141,12 +141,12 @@ class HostActivationCache:
         self.keep = int(min_layers_resident)
         self.prefetch_layers = int(prefetch_layers)
         self.pool = PinnedPool()
-        # high priority: HIP maps streams onto GPU_MAX_HW_QUEUES (4) hardware queues round-robin, and a copy that
-        # lands in the compute stream's queue cannot start before every kernel queued ahead of it has finished
-        self.stream = torch.cuda.Stream(device, priority=-1) if device.type == "cuda" else None
+        # copy streams keep the default priority, like every stream of the package: queues of different priorities
+        # have hung on MI355X
+        self.stream = torch.cuda.Stream(device) if device.type == "cuda" else None
         # backward prefetches get their own stream: on the D2H stream they queued behind the forward's spill backlog
         # (up to the copy window) and the first recomputed block of a 128k ckpt_offload step waited 191 ms for them
-        self.h2d_stream = torch.cuda.Stream(device, priority=-1) if device.type == "cuda" else None
+        self.h2d_stream = torch.cuda.Stream(device) if device.type == "cuda" else None
         self.cur_layer = -1
         self.n_layers = 0
         self.by_layer = {}

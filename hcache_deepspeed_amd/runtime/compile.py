@@ -126,7 +126,7 @@ def compile_engine(engine, backend="native", compile_kwargs=None, schedule=None)
     t0 = time.perf_counter()
     if cfg.native_comm and engine.optimizer is not None and hasattr(engine.optimizer, "enable_native_comm"):
         # DeepCompile's private-communicator path (reference csrc/compile/deepcompile.cpp): ZeRO all-gathers and
-        # reduce-scatters go through the C++ RCCL executor (comm/native_rccl.py) on its own priority stream
+        # reduce-scatters go through the C++ RCCL executor (comm/native_rccl.py) on its own stream
         engine.optimizer.enable_native_comm()
     times["native_comm"] = time.perf_counter() - t0
     t0 = time.perf_counter()

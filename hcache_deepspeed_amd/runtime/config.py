@@ -12,8 +12,7 @@ MI355X-specific knobs live under ``"mi355x"``::
         "zero3_prefetch_depth": 2,      # units all-gathered ahead of compute
         "zero3_max_reduce_inflight": 2, # gradient reduce-scatters in flight before the oldest is retired
         "host_act_cache": {"enabled": false, "slots": 8, "slot_mb": 512, "min_layers_resident": 2},
-        "fused_lm_head_ce": true,
-        "comm_high_priority": true      # ZeRO-3 AG/RS communicators on high-priority streams
+        "fused_lm_head_ce": true
     }
 """
 import copy
@@ -213,9 +212,6 @@ class MI355XConfig:
     # turns instead of overlapping (profiles/r6/overlap_step/)
     overlap_step: bool = False
     fused_lm_head_ce: bool = True
-    # ZeRO-3 all-gather / reduce-scatter communicators run their RCCL kernels on high-priority HIP streams, so
-    # the few workgroups a collective needs are dispatched ahead of queued GEMM tiles (overlap under full load)
-    comm_high_priority: bool = True
     # per-step exposed-communication / busbw accounting of the ZeRO collectives (runtime/zero/comm_stats.py)
     comm_stats: bool = False
     # ZeRO-3 unit collectives: "auto" measures rccl / native / symmetric per size class at dp > 1 and routes each
@@ -363,7 +359,6 @@ class DeepSpeedConfig:
             direct_wgrad=bool(m.get("direct_wgrad", True)),
             overlap_step=bool(m.get("overlap_step", False)),
             fused_lm_head_ce=bool(m.get("fused_lm_head_ce", True)),
-            comm_high_priority=bool(m.get("comm_high_priority", True)),
             host_act_cache=HostActCacheConfig(**{f.name: hac[f.name]
                                                  for f in fields(HostActCacheConfig) if f.name in hac}))
 

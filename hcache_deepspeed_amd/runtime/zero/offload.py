@@ -95,10 +95,8 @@ class OffloadZeroOptimizer(ZeroOptimizer):
             s.states = {k: None for k in s.states}
         elif self.n_off > 0:
             self._compact_device_part()
-        # copy streams at high priority: a stream that shares a hardware queue with the compute stream (HIP
-        # spreads streams over GPU_MAX_HW_QUEUES=4 queues) cannot start a copy before the kernels queued ahead
-        self.copy_stream = torch.cuda.Stream(self.device, priority=-1) if self.device.type == "cuda" else None  # D2H
-        self.h2d_stream = torch.cuda.Stream(self.device, priority=-1) if self.device.type == "cuda" else None  # H2D
+        self.copy_stream = torch.cuda.Stream(self.device) if self.device.type == "cuda" else None  # D2H
+        self.h2d_stream = torch.cuda.Stream(self.device) if self.device.type == "cuda" else None  # H2D
         log_dist(f"ZeRO-Offload: {self.n_off / 1e6:.1f}M of {n / 1e6:.1f}M elements on {self.offload_device} "
                  f"(sub-group {self.sub / 1e6:.1f}M)" + (", parameters on NVMe" if self.nvme_param else ""),
                  ranks=[0])

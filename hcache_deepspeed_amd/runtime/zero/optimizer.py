@@ -246,9 +246,8 @@ class ZeroOptimizer:
                     torch.distributed.get_process_group_ranks(dp_group)) if self.dp_world > 1 else [dist.get_rank()]
         self._setup_zeropp(dp_ranks)
         if self.stage == 3 and self.dp_world > 1 and not self.mics:
-            hp = bool(getattr(self.mi, "comm_high_priority", True))
-            self.ag_group = dist.new_group(ranks=dp_ranks, high_priority=hp)
-            self.rs_group = dist.new_group(ranks=dp_ranks, high_priority=hp)
+            self.ag_group = dist.new_group(ranks=dp_ranks)
+            self.rs_group = dist.new_group(ranks=dp_ranks)
 
         op = self.zcfg.offload_param
         self.offload_param = bool(op.enabled) and self.stage == 3
@@ -256,7 +255,7 @@ class ZeroOptimizer:
         self.nvme_param = self.offload_param and op.device == "nvme"
         self.param_swapper = None
         if self.offload_param and self.device.type == "cuda":
-            self.param_h2d_stream = torch.cuda.Stream(self.device, priority=-1)
+            self.param_h2d_stream = torch.cuda.Stream(self.device)
         else:
             self.param_h2d_stream = None
         self.state_offload = None  # DeepCompile offload_adam_states executor (runtime/zero/state_offload.py)
@@ -994,7 +993,7 @@ class ZeroOptimizer:
         self.offload_param = True
         self.param_offload_gpu_step = True
         if cuda:
-            self.param_h2d_stream = torch.cuda.Stream(self.device, priority=-1)
+            self.param_h2d_stream = torch.cuda.Stream(self.device)
             self._lp_d2h_stream = torch.cuda.Stream(self.device)
         log_dist(f"offload_parameters: {s.numel * host.element_size() / 2**30:.2f} GiB of parameter shards on the "
                  f"host", ranks=[0])
@@ -1052,7 +1051,7 @@ class ZeroOptimizer:
     def enable_symmetric_comm(self, cap_limit_bytes=1 << 30):
         """``compile.symmetric_memory``: unit all-gathers / reduce-scatters of intra-node groups run as one-kernel
         direct-read collectives over symmetric (IPC-mapped, uncached) buffers (comm/symmetric.py) on two dedicated
-        priority streams -- the reference's SymmetricMemory all-gather (csrc/compile/z3.cpp:91-110). Each buffer is
+        streams -- the reference's SymmetricMemory all-gather (csrc/compile/z3.cpp:91-110). Each buffer is
         sized for the largest unit collective of its group (up to ``cap_limit_bytes``; larger units keep RCCL).
         Collective: every rank must call it. Returns False (RCCL kept) on CPU or for groups of > 8 ranks."""
         from ...comm import symmetric
@@ -1079,10 +1078,10 @@ class ZeroOptimizer:
         return True
 
     def _install_symm(self, bufs):
-        """Symmetric buffers {(kind, id(group)): SymmetricMemory} for the unit collectives, their priority streams and
+        """Symmetric buffers {(kind, id(group)): SymmetricMemory} for the unit collectives, their streams and
         the device error flag the step folds (see below)."""
         self._symm = dict(bufs)
-        self._symm_streams = {k: torch.cuda.Stream(device=self.device, priority=-1) for k in ("ag", "rs")}
+        self._symm_streams = {k: torch.cuda.Stream(device=self.device) for k in ("ag", "rs")}
         # a timed-out exchange raises this device flag (symm_comm.hip): step() folds it, reduced over the data-parallel
         # group, into the skip flag -- the step that consumed stale peer data never updates the weights -- and raises
         # at the next step on every rank (read from pinned memory once the copy has landed: no extra host sync)

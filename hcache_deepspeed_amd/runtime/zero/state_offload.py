@@ -11,7 +11,7 @@ into two separately allocated pieces:
 
 * the head [0, a) stays on the device for good (``store.states[k]`` / ``store.master`` ARE the heads while split);
 * the tail [a, n) lives in pinned host memory between ``step()`` and the late backward of the next step: one D2H per
-  state on a high-priority copy stream right after the step (overlapping the next forward), its device buffer
+  state on a copy stream right after the step (overlapping the next forward), its device buffer
   released the moment the DMA drains; the reload is issued at the backward trace position the pass picks
   (``compile/passes.plan_state_reload``) or as soon as the HBM the backward has freed holds it.
 
@@ -68,8 +68,8 @@ class OptimizerStateOffload:
         self.chunk_bytes = max(256, int(float(chunk_mb) * 2**20))
         dev = zopt.device
         self.cuda = dev.type == "cuda"
-        self.stream = torch.cuda.Stream(dev, priority=-1) if self.cuda else None  # offload (D2H)
-        self.reload_stream = torch.cuda.Stream(dev, priority=-1) if self.cuda else None  # reload (H2D)
+        self.stream = torch.cuda.Stream(dev) if self.cuda else None  # offload (D2H)
+        self.reload_stream = torch.cuda.Stream(dev) if self.cuda else None  # reload (H2D)
         self.host = {}  # key -> pinned tail [n - a]
         self.tail = {}  # key -> [device chunk or None (off the device)] per tail chunk
         self.events = {}  # (key, chunk) -> last D2H / H2D event of that chunk

@@ -7,7 +7,7 @@ landed on: at data-parallel size > 1 the optimizer measures, for every unit all-
 every group, the three transports this framework has,
 
 * ``rccl``      -- torch.distributed (backend "nccl" = RCCL over xGMI; gloo on CPU dry runs),
-* ``native``    -- the private C++ RCCL communicator on a priority stream (comm/native_rccl.py),
+* ``native``    -- the private C++ RCCL communicator on a stream of its own (comm/native_rccl.py),
 * ``symmetric`` -- one-kernel direct-read collectives over IPC-mapped buffers (comm/symmetric.py, one node only),
 
 and routes each size class to the fastest. Every decision is COLLECTIVE: a candidate is usable only if it set up and

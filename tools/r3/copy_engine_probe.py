@@ -1,7 +1,7 @@
 """Which engine runs a side-stream host<->device copy, and what it costs the compute stream.
 
 For each host buffer kind (torch pinned, hipHostMalloc portable) and direction, time: the copy alone, a GEMM loop
-alone, and both concurrently (copy on a high-priority side stream). A copy executed by SDMA leaves the GEMMs at
+alone, and both concurrently (copy on a side stream). A copy executed by SDMA leaves the GEMMs at
 their solo speed; one executed as a blit kernel (``__amd_rocclr_copyBuffer``, visible in a kernel trace) takes CUs
 from them. Prints one JSON line per case plus the HIP/HSA environment.
 """
@@ -35,7 +35,7 @@ def main():
     src = torch.randn(n, device=dev, dtype=torch.bfloat16)
     hosts = {"torch_pinned": torch.empty(n, dtype=torch.bfloat16, pin_memory=True),
              "hipHostMalloc": pinned_empty((n, ), torch.bfloat16)}
-    side = torch.cuda.Stream(priority=-1)
+    side = torch.cuda.Stream()
 
     def gemms(k=40):
         for _ in range(k):
