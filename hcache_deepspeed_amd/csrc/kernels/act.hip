@@ -97,6 +97,28 @@ __global__ __launch_bounds__(256) void glu_fwd(const T* __restrict__ gu, T* __re
   }
 }
 
+// the same on strided rows of any width (serving: the result goes into a column block of a wider matrix)
+template <typename T, int A, int V>
+__global__ __launch_bounds__(256) void glu_rows(const T* __restrict__ gu, int64_t ld, T* __restrict__ y, int64_t ldo,
+                                                int64_t rows, int I) {
+  const int vpr = I / V;
+  const int64_t total = rows * vpr;
+  for (int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * 256) {
+    const int64_t r = total < (int64_t)0x7fffffff ? (unsigned)idx / (unsigned)vpr : idx / vpr;
+    const int c = (int)(idx - r * vpr) * V;
+    if constexpr (V == 8) {
+      float g[8], u[8], o[8];
+      Vec8<T>::load(gu + r * ld + c, g);
+      Vec8<T>::load(gu + r * ld + I + c, u);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = act_f<A>(g[j]) * u[j];
+      Vec8<T>::store(y + r * ldo + c, o);
+    } else {
+      y[r * ldo + c] = from_f<T>(act_f<A>(to_f(gu[r * ld + c])) * to_f(gu[r * ld + I + c]));
+    }
+  }
+}
+
 template <typename T, int A>
 __global__ __launch_bounds__(256) void glu_bwd(const T* __restrict__ dy, const T* __restrict__ gu,
                                                T* __restrict__ dgu, int64_t rows, int I) {
@@ -385,6 +407,34 @@ HDS_EXPORT int hds_glu_fwd(int dtype, int act, const void* gu, void* y, int64_t 
     dim3 grid(stream_grid(rows * (I / 8), 256)), block(256);
     DT_SWITCH(dtype, ACT_SWITCH(act, glu_fwd, T, grid, block, 0, st, (const T*)gu, (T*)y, rows, I));
   }
+  return hipGetLastError();
+}
+
+// gu: [rows, ld] with the gate in columns [0, I) and up in [I, 2I); y: [rows, ldo]
+HDS_EXPORT int hds_glu_rows(int dtype, int act, const void* gu, int64_t ld, void* y, int64_t ldo, int64_t rows, int I,
+                            hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (I < 1 || ld < 2 * (int64_t)I || ldo < I || act < 0 || act > kIdentity) return hipErrorInvalidValue;
+  const bool v8 = I % 8 == 0 && ld % 8 == 0 && ldo % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)y % 16 == 0;
+  const dim3 grid(stream_grid(rows * (v8 ? I / 8 : I), 256)), block(256);
+#define HDS_GR(TT, AA)                                                                                            \
+  case AA:                                                                                                        \
+    if (v8)                                                                                                       \
+      hipLaunchKernelGGL((glu_rows<TT, AA, 8>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I);     \
+    else                                                                                                          \
+      hipLaunchKernelGGL((glu_rows<TT, AA, 1>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I);     \
+    break;
+#define HDS_GRA(TT) \
+  switch (act) { HDS_GR(TT, kSilu) HDS_GR(TT, kGeluTanh) HDS_GR(TT, kRelu) HDS_GR(TT, kGeluErf) HDS_GR(TT, kIdentity) }
+  if (dtype == kBF16) {
+    HDS_GRA(bf16)
+  } else if (dtype == kF32) {
+    HDS_GRA(float)
+  } else {
+    return hipErrorInvalidValue;
+  }
+#undef HDS_GRA
+#undef HDS_GR
   return hipGetLastError();
 }
 

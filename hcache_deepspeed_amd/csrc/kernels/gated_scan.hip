@@ -1,0 +1,223 @@
+// Gated linear recurrence of a recurrent mixer (minGRU): element by element over time, in 32-bit,
+//
+//   z = sigmoid(a + ba),  u = b + bb,  v = u + 1/2 (u >= 0) or sigmoid(u) (u < 0)
+//   S_t = (1 - z) S_(t-1) + z v,       out_t = S_t * silu(c)
+//
+// with a | b | c the three column blocks of one projection row. The state of a sequence is one 32-bit row in its slot;
+// a sequence whose `seen` is 0 starts from zero whatever the slot holds.
+//
+// Short steps (decode, small portions) run one thread per channel over the new tokens. Prompts are cut into chunks of
+// kChunk tokens: pass 1 reduces every chunk to S_out = A S_in + B, pass 2 walks the chunks of a sequence and leaves
+// each chunk's S_in (and the sequence's new state), pass 3 replays the chunks from it. No workgroup waits for another.
+#include "hds_common.h"
+
+namespace {
+using namespace hds;
+
+constexpr int kChunk = 32;
+
+template <typename T, int V>
+__device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
+  if constexpr (V == 1) {
+    v[0] = to_f(*p);
+  } else if constexpr (sizeof(T) == 2) {
+    const bf16x4 r = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = (float)r[i];
+  } else {
+    const f32x4 r = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = r[i];
+  }
+}
+template <typename T, int V>
+__device__ __forceinline__ void stv(T* p, const float (&v)[V]) {
+  if constexpr (V == 1) {
+    *p = from_f<T>(v[0]);
+  } else if constexpr (sizeof(T) == 2) {
+    bf16x4 r;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) r[i] = (bf16)v[i];
+    *reinterpret_cast<bf16x4*>(p) = r;
+  } else {
+    *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+  }
+}
+
+// sigmoid(x) and 1 - sigmoid(x), neither by cancellation
+__device__ __forceinline__ void sigmoid2(float x, float& s, float& c) {
+  const float e = __expf(-fabsf(x));
+  const float r = 1.f / (1.f + e);
+  s = x >= 0.f ? r : e * r;
+  c = x >= 0.f ? e * r : r;
+}
+__device__ __forceinline__ void gates(float a, float b, float& keep, float& add) {
+  float z, us, uc;
+  sigmoid2(a, z, keep);
+  sigmoid2(b, us, uc);
+  add = z * (b >= 0.f ? b + 0.5f : us);
+}
+__device__ __forceinline__ float silu(float x) {
+  float s, c;
+  sigmoid2(x, s, c);
+  return x * s;
+}
+
+template <typename T>
+struct ScanParams {
+  const T* in;       // [tokens, ld]: a at column 0, b at W, c at 2 W
+  int64_t ld;
+  const float* ba;   // [W]
+  const float* bb;
+  T* out;            // [tokens, ldo]
+  int64_t ldo;
+  float* state;      // [slots] x slot_stride
+  int64_t slot_stride;
+  const int* slots;
+  const int* seq_meta;
+  float* ws;         // [S, chunks, 2, W]
+  int W, chunks;
+};
+
+// pass 0: whole sequences serially; pass 1: chunk reductions; pass 3: chunk replays
+template <typename T, int V, int PASS>
+__global__ __launch_bounds__(64) void scan_kernel(ScanParams<T> p) {
+  const int c = (blockIdx.x * 64 + threadIdx.x) * V;
+  if (c >= p.W) return;
+  const int seq = blockIdx.z, ch = blockIdx.y;
+  const int q0 = p.seq_meta[3 * seq], n = p.seq_meta[3 * seq + 1], seen = p.seq_meta[3 * seq + 2];
+  const int t0 = PASS == 0 ? 0 : ch * kChunk;
+  if (t0 >= n) return;
+  const int t1 = PASS == 0 ? n : min(n, t0 + kChunk);
+  float ba[V], bb[V], s[V], A[V];
+  ldv<float, V>(p.ba + c, ba);
+  ldv<float, V>(p.bb + c, bb);
+  float* st = p.state + (PASS == 0 ? (int64_t)p.slots[seq] * p.slot_stride + c : 0);
+  float* ws = PASS == 0 ? nullptr : p.ws + (((int64_t)seq * p.chunks + ch) * 2) * p.W + c;
+#pragma unroll
+  for (int i = 0; i < V; ++i) {
+    s[i] = 0.f;
+    A[i] = 1.f;
+  }
+  if (PASS == 0 && seen > 0) ldv<float, V>(st, s);
+  if (PASS == 3) ldv<float, V>(ws + p.W, s);
+  const T* in = p.in + (int64_t)(q0 + t0) * p.ld + c;
+  T* out = p.out + (int64_t)(q0 + t0) * p.ldo + c;
+  auto step = [&](const float (&a)[V], const float (&b)[V], const float (&g)[V], T* o) {
+    float y[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      float keep, add;
+      gates(a[i] + ba[i], b[i] + bb[i], keep, add);
+      s[i] = keep * s[i] + add;
+      if (PASS == 1) A[i] *= keep;
+      if (PASS != 1) y[i] = s[i] * silu(g[i]);
+    }
+    if (PASS != 1) stv<T, V>(o, y);
+  };
+  constexpr int U = 4;
+  int t = t0;
+  for (; t + U <= t1; t += U) {
+    float a[U][V], b[U][V], g[U][V];
+#pragma unroll
+    for (int k = 0; k < U; ++k) {
+      ldv<T, V>(in + k * p.ld, a[k]);
+      ldv<T, V>(in + k * p.ld + p.W, b[k]);
+      if (PASS != 1) ldv<T, V>(in + k * p.ld + 2 * p.W, g[k]);
+    }
+#pragma unroll
+    for (int k = 0; k < U; ++k) step(a[k], b[k], g[k], out + k * p.ldo);
+    in += U * p.ld;
+    out += U * p.ldo;
+  }
+  for (; t < t1; ++t) {
+    float a[V], b[V], g[V];
+    ldv<T, V>(in, a);
+    ldv<T, V>(in + p.W, b);
+    if (PASS != 1) ldv<T, V>(in + 2 * p.W, g);
+    step(a, b, g, out);
+    in += p.ld;
+    out += p.ldo;
+  }
+  if (PASS == 0) stv<float, V>(st, s);
+  if (PASS == 1) {
+    stv<float, V>(ws, A);
+    stv<float, V>(ws + p.W, s);
+  }
+}
+
+// pass 2: ws[., 1] becomes the state a chunk starts from; the sequence's last state goes to its slot
+template <typename T>
+__global__ __launch_bounds__(64) void scan_carry_kernel(ScanParams<T> p) {
+  const int c = blockIdx.x * 64 + threadIdx.x;
+  if (c >= p.W) return;
+  const int seq = blockIdx.y;
+  const int n = p.seq_meta[3 * seq + 1], seen = p.seq_meta[3 * seq + 2];
+  if (n <= 0) return;
+  const int nc = (n + kChunk - 1) / kChunk;
+  float* st = p.state + (int64_t)p.slots[seq] * p.slot_stride + c;
+  float s = seen > 0 ? *st : 0.f;
+  float* ws = p.ws + (int64_t)seq * p.chunks * 2 * p.W + c;
+  constexpr int U = 8;
+  for (int k0 = 0; k0 < nc; k0 += U) {
+    float A[U], B[U];
+#pragma unroll
+    for (int k = 0; k < U; ++k) {
+      const int64_t o = (int64_t)(k0 + k) * 2 * p.W;
+      A[k] = k0 + k < nc ? ws[o] : 1.f;
+      B[k] = k0 + k < nc ? ws[o + p.W] : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < U; ++k) {
+      if (k0 + k < nc) ws[(int64_t)(k0 + k) * 2 * p.W + p.W] = s;
+      s = A[k] * s + B[k];
+    }
+  }
+  *st = s;
+}
+
+template <typename T, int V>
+int launch_scan(const ScanParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
+  const int cb = (p.W + 64 * V - 1) / (64 * V);
+  if (p.ws == nullptr) {
+    hipLaunchKernelGGL((scan_kernel<T, V, 0>), dim3(cb, 1, n_seqs), dim3(64), 0, st, p);
+    return hipGetLastError();
+  }
+  const dim3 grid(cb, (max_new + kChunk - 1) / kChunk, n_seqs);
+  hipLaunchKernelGGL((scan_kernel<T, V, 1>), grid, dim3(64), 0, st, p);
+  hipLaunchKernelGGL((scan_carry_kernel<T>), dim3((p.W + 63) / 64, n_seqs), dim3(64), 0, st, p);
+  hipLaunchKernelGGL((scan_kernel<T, V, 3>), grid, dim3(64), 0, st, p);
+  return hipGetLastError();
+}
+
+template <typename T>
+int scan(const ScanParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
+  if (p.W % 4 == 0 && p.ld % 4 == 0 && p.ldo % 4 == 0 && p.slot_stride % 4 == 0 && (uintptr_t)p.in % 16 == 0 &&
+      (uintptr_t)p.out % 16 == 0 && (uintptr_t)p.state % 16 == 0)
+    return launch_scan<T, 4>(p, n_seqs, max_new, st);
+  return launch_scan<T, 1>(p, n_seqs, max_new, st);
+}
+
+}  // namespace
+
+HDS_EXPORT int hds_gated_scan_chunk() { return kChunk; }
+
+// ws: null -> every sequence serially; else n_seqs * chunks * 2 * W floats with chunks = ceil(max_new / kChunk)
+HDS_EXPORT int hds_gated_scan(int dtype, const void* in, int64_t ld, const float* ba, const float* bb, void* out,
+                              int64_t ldo, float* state, int64_t slot_stride, const int* slots, const int* seq_meta,
+                              float* ws, int n_seqs, int max_new, int W, hipStream_t st) {
+  if (n_seqs <= 0 || max_new <= 0) return 0;
+  if (W < 1 || ld < 3 * (int64_t)W || ldo < W || !state || !slots || n_seqs > 65535) return hipErrorInvalidValue;
+  const int chunks = (max_new + kChunk - 1) / kChunk;
+  if (chunks > 65535) return hipErrorInvalidValue;
+  if (dtype == kBF16) {
+    ScanParams<bf16> p{(const bf16*)in, ld, ba, bb, (bf16*)out, ldo, state, slot_stride, slots, seq_meta, ws, W, chunks};
+    return scan(p, n_seqs, max_new, st);
+  }
+  if (dtype == kF32) {
+    ScanParams<float> p{(const float*)in, ld, ba, bb, (float*)out, ldo, state, slot_stride, slots, seq_meta, ws, W,
+                        chunks};
+    return scan(p, n_seqs, max_new, st);
+  }
+  return hipErrorInvalidValue;
+}

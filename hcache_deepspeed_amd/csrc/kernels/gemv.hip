@@ -99,9 +99,15 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const bf16* __restrict__
 // serial prologue cost what a separate RMSNorm launch did (fused qkv 15.4 us vs 10.9 us plain GEMV + 4.6 us norm).
 // Workgroup 0 also writes r (the new residual stream) and, when asked, x (the normed rows: HCache's hidden-state
 // latents) once its waves know rstd.
-// GLU: the weight is [gate; up] ([2I, K]) and the output y[M, I] = bf16(act(bf16(x.g_j)) * bf16(x.u_j)) (silu): a wave
+// GLU: the weight is [gate; up] ([2I, K]) and the output y[M, I] = bf16(act(bf16(x.g_j)) * bf16(x.u_j)): a wave
 // owns R output columns and streams their gate AND up rows, so the [M, 2I] intermediate never exists.
 __device__ __forceinline__ float silu_f(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
+// the gate's activation, by the codes of act.hip: 0 silu, 1 gelu_tanh, 2 relu
+__device__ __forceinline__ float gate_f(float v, int act) {
+  if (act == 2) return fmaxf(v, 0.f);
+  if (act == 1) return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+  return silu_f(v);
+}
 
 // r = bf16(h + res) (h without res) for 8 elements at k
 __device__ __forceinline__ bf16x8 load_r(const bf16* __restrict__ h, const bf16* __restrict__ res, int64_t off, int k) {
@@ -138,8 +144,8 @@ template <int MAXM, int R, bool NORM, bool GLU>
 __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16* __restrict__ h, const bf16* __restrict__ res,
                                                          const bf16* __restrict__ gamma, float eps,
                                                          const bf16* __restrict__ w, bf16* __restrict__ y,
-                                                         bf16* __restrict__ r_out, bf16* __restrict__ x_out, int M,
-                                                         int N, int K, int64_t ldh, int64_t ldy) {
+                                                         bf16* __restrict__ r_out, bf16* __restrict__ x_out, int act,
+                                                         int M, int N, int K, int64_t ldh, int64_t ldy) {
   const int lane = threadIdx.x & 63;
   const int wid = threadIdx.x >> 6;
   const int n0 = (blockIdx.x * 4 + wid) * R;  // output columns [n0, n0 + R)
@@ -220,7 +226,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16* __restrict_
         const float v = rstd[m] * wave_sum(acc[r][m]);
         if constexpr (GLU) {
           const float u = rstd[m] * wave_sum(acc[R + r][m]);
-          if (lane == 0) y[m * ldy + n0 + r] = (bf16)(silu_f((float)(bf16)v) * (float)(bf16)u);
+          if (lane == 0) y[m * ldy + n0 + r] = (bf16)(gate_f((float)(bf16)v, act) * (float)(bf16)u);
         } else {
           if (lane == 0) y[m * ldy + n0 + r] = (bf16)v;
         }
@@ -295,7 +301,102 @@ __global__ __launch_bounds__(256) void skinny_mfma_kernel(const bf16* __restrict
 
 int g_skinny_u = 16;
 
+// ---------------------------------------------------------------------------------------------------------------
+// One decode step of the gated recurrence (gated_scan.hip) with its projection: a wave owns one channel j and streams
+// the three weight rows j, N + j, 2N + j (update gate, candidate, output gate) against up to MAXM token rows, each of
+// another sequence; lane 0 then advances the channel's 32-bit state of every row and writes S * silu(c). The projected
+// values are rounded to bf16 first, as the separate projection stores them.
+__device__ __forceinline__ void sigmoid2_f(float x, float& s, float& c) {
+  const float e = __expf(-fabsf(x)), r = 1.f / (1.f + e);
+  s = x >= 0.f ? r : e * r;
+  c = x >= 0.f ? e * r : r;
+}
+
+template <int MAXM>
+__global__ __launch_bounds__(256) void gemv_recur_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
+                                                         const float* __restrict__ ba, const float* __restrict__ bb,
+                                                         bf16* __restrict__ y, float* __restrict__ state,
+                                                         int64_t slot_stride, const int* __restrict__ slots,
+                                                         const int* __restrict__ seq_meta, int M, int N, int K,
+                                                         int64_t ldx, int64_t ldy) {
+  const int lane = threadIdx.x & 63;
+  const int j = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (j >= N) return;
+  float acc[3][MAXM];
+#pragma unroll
+  for (int r = 0; r < 3; ++r)
+#pragma unroll
+    for (int m = 0; m < MAXM; ++m) acc[r][m] = 0.f;
+  const bf16* wr[3];
+#pragma unroll
+  for (int r = 0; r < 3; ++r) wr[r] = w + ((int64_t)r * N + j) * K;
+  int k0 = 8 * lane;
+  for (; k0 + 512 < K; k0 += 1024) {
+    bf16x8 wa[3], wb[3];
+#pragma unroll
+    for (int r = 0; r < 3; ++r) {
+      wa[r] = *reinterpret_cast<const bf16x8*>(wr[r] + k0);
+      wb[r] = *reinterpret_cast<const bf16x8*>(wr[r] + k0 + 512);
+    }
+#pragma unroll
+    for (int m = 0; m < MAXM; ++m) {
+      if (m < M) {
+        const bf16x8 xa = *reinterpret_cast<const bf16x8*>(x + m * ldx + k0);
+        const bf16x8 xb = *reinterpret_cast<const bf16x8*>(x + m * ldx + k0 + 512);
+#pragma unroll
+        for (int r = 0; r < 3; ++r) acc[r][m] = dot8(xb, wb[r], dot8(xa, wa[r], acc[r][m]));
+      }
+    }
+  }
+  if (k0 < K) {
+    bf16x8 wa[3];
+#pragma unroll
+    for (int r = 0; r < 3; ++r) wa[r] = *reinterpret_cast<const bf16x8*>(wr[r] + k0);
+#pragma unroll
+    for (int m = 0; m < MAXM; ++m) {
+      if (m < M) {
+        const bf16x8 xa = *reinterpret_cast<const bf16x8*>(x + m * ldx + k0);
+#pragma unroll
+        for (int r = 0; r < 3; ++r) acc[r][m] = dot8(xa, wa[r], acc[r][m]);
+      }
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < MAXM; ++m) {
+    if (m < M) {
+      const float a = (float)(bf16)wave_sum(acc[0][m]) + ba[j], b = (float)(bf16)wave_sum(acc[1][m]) + bb[j];
+      const float g = (float)(bf16)wave_sum(acc[2][m]);
+      if (lane == 0) {
+        float* st = state + (int64_t)slots[m] * slot_stride + j;
+        const float s0 = seq_meta[3 * m + 2] > 0 ? *st : 0.f;
+        float z, keep, us, uc, gs, gc;
+        sigmoid2_f(a, z, keep);
+        sigmoid2_f(b, us, uc);
+        sigmoid2_f(g, gs, gc);
+        const float s = keep * s0 + z * (b >= 0.f ? b + 0.5f : us);
+        *st = s;
+        y[m * ldy + j] = (bf16)(s * g * gs);
+      }
+    }
+  }
+}
+
 }  // namespace
+
+// A decode step of the recurrence for M <= 8 sequences (row m of x is the one new token of sequence m): w is [3N, K]
+// (update gate, candidate, output gate rows), y [M, N] with row stride ldy. K % 8 == 0, 16-B aligned x and w.
+HDS_EXPORT int hds_gemv_recur_bf16(const void* x, const void* w, const float* ba, const float* bb, void* y,
+                                   float* state, int64_t slot_stride, const int* slots, const int* seq_meta, int M,
+                                   int N, int K, int64_t ldx, int64_t ldy, hipStream_t st) {
+  if (M < 1 || M > 8 || N < 1 || K < 8 || K % 8 || ldx % 8 || ldx < K || ldy < N || !state || !slots || !seq_meta)
+    return hipErrorInvalidValue;
+#define HDS_RC(MM)                                                                                                   \
+  hipLaunchKernelGGL(gemv_recur_kernel<MM>, dim3((N + 3) / 4), dim3(256), 0, st, (const bf16*)x, (const bf16*)w, ba, \
+                     bb, (bf16*)y, state, slot_stride, slots, seq_meta, M, N, K, ldx, ldy)
+  if (M == 1) HDS_RC(1); else if (M <= 2) HDS_RC(2); else if (M <= 4) HDS_RC(4); else HDS_RC(8);
+#undef HDS_RC
+  return hipGetLastError();
+}
 
 // Skinny matrix-core GEMM (skinny_mfma_kernel): 1 <= M <= 16, K % 128 == 0, 16-B aligned rows
 HDS_EXPORT int hds_skinny_gemm_bf16(const void* x, const void* w, const void* bias, void* y, int M, int N, int K,
@@ -320,20 +421,21 @@ HDS_EXPORT int hds_skinny_set_unroll(int u) {
   return prev;
 }
 
-// Fused decode GEMV (see gemv_fused_kernel): y[M, N] = norm(h (+ res)) . W^T, or with glu != 0, y[M, N] =
-// silu(x . Wg^T) * (x . Wu^T) for W = [Wg; Wu] of 2N rows (x normed when gamma is given, else h itself). r_out /
+// Fused decode GEMV (see gemv_fused_kernel): y[M, N] = norm(h (+ res)) . W^T, or with glu = 1 + activation code
+// (0 silu, 1 gelu_tanh, 2 relu), y[M, N] = act(x . Wg^T) * (x . Wu^T) for W = [Wg; Wu] of 2N rows (x normed when gamma is given, else h itself). r_out /
 // x_out (workgroup 0, with gamma): the new residual rows and the normed rows. ldh: row stride of h / res / r_out /
 // x_out (elements); ldy: row stride of y. Shapes: M <= 8, K % 8 == 0, 16-B aligned operands (checked by the caller).
 HDS_EXPORT int hds_gemv_fused_bf16(const void* h, const void* res, const void* gamma, float eps, const void* w,
                                    void* y, void* r_out, void* x_out, int glu, int M, int N, int K, int64_t ldh,
                                    int64_t ldy, hipStream_t st) {
-  if (M < 1 || M > 8 || N < 1 || K < 8 || K % 8 || ldh % 8) return hipErrorInvalidValue;
+  if (M < 1 || M > 8 || N < 1 || K < 8 || K % 8 || ldh % 8 || glu < 0 || glu > 3) return hipErrorInvalidValue;
+  const int act = glu - 1;
   if (gamma == nullptr && (r_out != nullptr || x_out != nullptr || res != nullptr)) return hipErrorInvalidValue;
   const int R = N >= 8192 ? (glu ? 2 : 4) : (N >= 4096 ? 2 : 1);
 #define HDS_GF(MM, RR, NN, GG)                                                                                   \
   hipLaunchKernelGGL((gemv_fused_kernel<MM, RR, NN, GG>), dim3((N + 4 * RR - 1) / (4 * RR)), dim3(256), 0, st,  \
                      (const bf16*)h, (const bf16*)res, (const bf16*)gamma, eps, (const bf16*)w, (bf16*)y,      \
-                     (bf16*)r_out, (bf16*)x_out, M, N, K, ldh, ldy)
+                     (bf16*)r_out, (bf16*)x_out, act, M, N, K, ldh, ldy)
 #define HDS_GFM(RR, NN, GG)                                                                                    \
   if (M == 1) HDS_GF(1, RR, NN, GG); else if (M <= 2) HDS_GF(2, RR, NN, GG);                                   \
   else if (M <= 4) HDS_GF(4, RR, NN, GG); else HDS_GF(8, RR, NN, GG);

@@ -41,6 +41,11 @@ class ArchSpec:
     tie_embeddings: bool = False
     lm_head_bias: bool = False
     moe: Optional[dict] = None         # {num_experts, top_k, normalize, shared}
+    # layers of several kinds (hybrid.HybridTransformer): one entry per layer, {"mixer": {"type", sizes ...},
+    # "mlp": {"ff", "act"} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
+    layers: Optional[list] = None
+    loop: Optional[dict] = None
+    input_conv_taps: int = 1
     extra: dict = field(default_factory=dict)
 
     # LlamaConfig-compatible aliases used by the engine / KV cache sizing
@@ -60,7 +65,73 @@ def _g(hf, *names, default=None):
     return default
 
 
+def run_order(spec):
+    """Layer index of every layer run, in order (looped layers appear once per pass)."""
+    n, lp = len(spec.layers), spec.loop
+    if not lp:
+        return list(range(n))
+    a, b = lp["start"], lp["stop"]
+    return list(range(a)) + list(range(a, b)) * lp["times"] + list(range(b, n))
+
+
+# ---------------------------------------------------------------------------------------------
+# Gofasun: minGRU and latent-attention mixers beside a ReLU-gated MLP in parallel (two scalar-gain RMS norms of the
+# same residual), a short causal convolution in front of every sublayer, optionally looped layers
+# ---------------------------------------------------------------------------------------------
+def _gofasun_mixer(kind, m):
+    if kind == "mingru":
+        return {"type": kind, "width": int(m["width"])}
+    if kind == "latent_attention":
+        rot, mask = m.get("rot") or {}, m.get("mask") or {}
+        return {"type": kind, "heads": int(m["heads"]), "dim": int(m["dim"]), "rot_dim": int(m["rot_dim"]),
+                "rot_dims": int(rot.get("dims", m["rot_dim"])), "rope_base": float(rot.get("base", 10000.0)),
+                "kv_rank": int(m["kv_rank"]), "vdim": int(m["vdim"]), "window": int(mask.get("size") or 0),
+                "scale": float(m["scale"])}
+    raise NotImplementedError(f"Gofasun mixer {kind!r}")
+
+
+def spec_gofasun(cfg):
+    layers = []
+    for e in cfg["layers"]:
+        mlp = e.get("mlp")
+        if mlp is not None and mlp.get("kind", "dense") != "dense":
+            raise NotImplementedError(f"Gofasun feed-forward {mlp['kind']!r}")
+        layers.append({"mixer": _gofasun_mixer(e["type"], e["mixer"]),
+                       "mlp": None if mlp is None else {"ff": int(mlp["ff"]), "act": "relu"}})
+    lp = cfg.get("loop")
+    loop = {k: int(lp[k]) for k in ("start", "stop", "times")} if lp else None
+    heads = max((x["mixer"].get("heads", 1) for x in layers), default=1)
+    return ArchSpec(model_type="gofasun", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                    num_hidden_layers=len(layers), num_attention_heads=heads, num_key_value_heads=heads,
+                    head_dim=max((x["mixer"].get("dim", 0) + x["mixer"].get("rot_dim", 0) for x in layers), default=0),
+                    intermediate_size=max((x["mlp"]["ff"] for x in layers if x["mlp"]), default=0), norm="rms",
+                    norm_eps=float(cfg["norm"]["eps"]), act="relu", gated=True, parallel="two_ln", layers=layers,
+                    loop=loop, input_conv_taps=int((cfg.get("canon") or {}).get("taps", 1)))
+
+
+def convert_gofasun(sd, spec):
+    out = {"embed": sd["embed"], "final.w": sd["final.norm"], "lm_head.w": sd["head"], "layers": []}
+    for i, e in enumerate(spec.layers):
+        p = f"l{i}."
+        L = {"mix": {k[len(p) + 4:]: v for k, v in sd.items() if k.startswith(p + "mix.")},
+             "ln1.w": sd[p + "norm1"], "conv1.w": sd.get(p + "canon1")}
+        if e["mlp"] is not None:
+            L.update({"ln2.w": sd[p + "norm2"], "conv2.w": sd.get(p + "canon2"), "gate.w": sd[p + "mlp.gate"],
+                      "up.w": sd[p + "mlp.up"], "down.w": sd[p + "mlp.down"]})
+        out["layers"].append(L)
+    return out
+
+
+# config.json's "architecture" / "model_type" -> (config reader, weight converter)
+ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun)}
+
+
 def spec_from_hf(hf):
+    name = str(hf.get("model_type") or hf.get("architecture") or "").lower()
+    if name in ARCHITECTURES:
+        return ARCHITECTURES[name][0](hf)
+    if "model_type" not in hf and hf.get("architecture"):
+        raise NotImplementedError(f"architecture {hf['architecture']} is not supported by the serving engine")
     rp = hf.get("rope_parameters")
     if isinstance(rp, dict):  # transformers>=5 nests the RoPE fields
         flat = {k: rp[k] for k in ("rope_theta", "partial_rotary_factor") if k in rp}
@@ -140,6 +211,8 @@ def _experts(sd, m, E, gate, up, down):
 def convert_hf(sd, spec):
     """HF state dict -> {"embed", "pos_embed", "final.w", "final.b", "lm_head.w", "lm_head.b", "layers": [...]}"""
     mt = spec.model_type
+    if mt in ARCHITECTURES:
+        return ARCHITECTURES[mt][1](sd, spec)
     out = {"layers": []}
     g = sd.get
     if mt in ("llama", "mistral", "qwen2", "mixtral", "qwen2_moe", "phi3"):

@@ -19,8 +19,9 @@ import torch
 
 from ... import comm as dist
 from ...utils.logging import log_dist
+from .hybrid import HybridTransformer
 from .model import RaggedTransformer
-from .ragged import BlockedKVCache, DSStateManager, DSStateManagerConfig, RaggedBatchWrapper
+from .ragged import (BlockedKVCache, DSStateManager, DSStateManagerConfig, RaggedBatchWrapper, SequenceStatePool)
 
 
 class SchedulingResult(Enum):
@@ -73,13 +74,17 @@ class InferenceEngineV2:
         if not isinstance(model_config, ArchSpec):  # this framework's Llama / Mixtral training configs
             model_config = spec_from_llama_config(model_config)
             weights = convert_own_llama(weights, model_config)
-        self._model = RaggedTransformer(model_config, weights, device, dtype, tp_group=self._base_mp_group,
-                                        latent_mode=self._config.latent_mode, engine_config=self._config)
+        cls = RaggedTransformer if model_config.layers is None else HybridTransformer
+        self._model = cls(model_config, weights, device, dtype, tp_group=self._base_mp_group,
+                          latent_mode=self._config.latent_mode, engine_config=self._config)
         sm = self._config.state_manager
+        floats = self._model.state_floats()
+        self._states = SequenceStatePool(sm.max_tracked_sequences, floats, device) if floats else None
         kvc = self._model.kv_cache_config()
         self._kv = BlockedKVCache(kvc["num_layers"], kvc["n_kv_heads"], kvc["head_dim"], sm.kv_block_size, dtype,
-                                  device, sm.memory_config, tp_group=self._base_mp_group, num_blocks=num_kv_blocks)
-        self._model.set_kv_cache(self._kv)
+                                  device, sm.memory_config, tp_group=self._base_mp_group, num_blocks=num_kv_blocks,
+                                  row_widths=kvc.get("row_widths"))
+        self._model.set_kv_cache(self._kv, self._states)
         self._state_manager = DSStateManager(sm, self._kv)
         self._batch = RaggedBatchWrapper(sm, device, self._state_manager.max_blocks_per_seq)
         from ...ops.paged import ROWS_PER_ATOM
@@ -116,9 +121,12 @@ class InferenceEngineV2:
 
     # ------------------------------------------------------------------------------------------
     def put(self, batch_uids: Iterable[int], batch_tokens: Iterable[torch.Tensor], do_checks: bool = True,
-            capture_latents: bool = True, sync_latents: Optional[bool] = None
+            capture_latents: bool = True, sync_latents: Optional[bool] = None,
+            logits_at: Optional[Iterable[Iterable[int]]] = None
             ) -> Tuple[torch.Tensor, List[Optional[torch.Tensor]]]:
         """One ragged forward. Returns logits [n_seqs, V] and, per sequence, its latents [L, n_tokens, W] (host).
+        ``logits_at``: for each sequence the places among its new tokens whose logits are wanted (possibly none); the
+        logits then have one row per wanted place, in that order, instead of one per sequence.
         ``sync_latents=False``: the host does not wait for the latent copies (no per-forward synchronize, reference
         engine_v2.py:131-189 keeps its host free the same way); call ``wait_latents()`` (or check
         ``latents_ready()``) before reading them -- ``restore_kv`` / ``evict`` wait on their own; HIP-graph decode
@@ -133,11 +141,12 @@ class InferenceEngineV2:
                 raise SchedulingError(res)
         sm, batch = self._state_manager, self._batch
         batch.clear()
-        for uid, tokens in zip(batch_uids, batch_tokens):
+        places = [None] * len(batch_uids) if logits_at is None else [list(p) for p in logits_at]
+        for uid, tokens, want in zip(batch_uids, batch_tokens, places):
             seq = sm.get_or_create_sequence(uid)
             sm.maybe_allocate_kv(seq, tokens.numel())
             seq.pre_forward(tokens.numel())
-            batch.insert_sequence(seq, tokens, do_checks=do_checks)
+            batch.insert_sequence(seq, tokens, do_checks=do_checks, logits_at=want)
         batch.finalize()
         if self._model.decode_graph_eligible(batch, capture_latents):
             # HIP-graph decode step (latents, if captured, land in the graph's device ring)
@@ -200,15 +209,29 @@ class InferenceEngineV2:
         if not lat:
             return
         batch.finalize()
+        if self._states is not None:
+            for uid in restored:
+                seq = sm.get_sequence(uid)
+                st = seq.evicted_state
+                if st is None or seq.seen_tokens or st[0] != seq.in_flight_tokens:
+                    raise RuntimeError(f"sequence {uid}: its recurrent state was saved at "
+                                       f"{st[0] if st else 'no'} tokens; restore exactly those")
         self._model.restore_kv(batch, lat)  # per-sequence pinned pieces, copied straight to the device
         for uid in restored:
-            sm.get_sequence(uid).post_forward()
+            seq = sm.get_sequence(uid)
+            if self._states is not None:
+                self._states.load(seq.tracking_id, seq.evicted_state[1])
+                seq.evicted_state = None
+            seq.post_forward()
 
     def evict(self, uid):
-        """Free a sequence's KV blocks but keep tracking it (its tokens/latents live on the host)."""
+        """Free a sequence's KV blocks but keep tracking it (its tokens/latents live on the host, and so does a copy of
+        its recurrent state, if the model has any)."""
         seq = self._state_manager.get_sequence(uid)
         self.wait_latents()
         if seq is not None:
+            if self._states is not None and seq.seen_tokens:
+                seq.evicted_state = (seq.seen_tokens, self._states.export(seq.tracking_id))
             self._state_manager.free_kv(seq)
             seq.seen_tokens = 0
 
@@ -288,12 +311,15 @@ class InferenceEngineV2:
             json.dump(meta, f, default=str)
 
     # ------------------------------------------------------------------------------------------
-    def generate(self, uid, prompt, max_new_tokens=16):
-        """Greedy decoding helper (prefill + decode through ``put``)."""
+    def generate(self, uid, prompt, max_new_tokens=16, do_sample=False, temperature=1.0, top_k=0, top_p=1.0,
+                 generator=None):
+        """Decoding helper (prefill + decode through ``put``): greedy, or temperature / top-k / nucleus sampling with
+        ``do_sample`` (models/generation.py)."""
+        from ...models.generation import _sample
         logits, _ = self.put([uid], [prompt], capture_latents=False)
         out = []
         for _ in range(max_new_tokens):
-            nxt = int(logits[0].argmax())
+            nxt = int(_sample(logits[:1].float(), do_sample, temperature, top_k, top_p, generator))
             out.append(nxt)
             logits, _ = self.put([uid], [torch.tensor([nxt])], capture_latents=False)
         return out
@@ -308,11 +334,11 @@ def build_engine_from_model(model, engine_config=None, device=None, num_kv_block
     return InferenceEngineV2(cfg, sd, engine_config, device=device, num_kv_blocks=num_kv_blocks)
 
 
-def build_hf_engine(path, engine_config=None, debug_level=None, device=None):
+def build_hf_engine(path, engine_config=None, debug_level=None, device=None, num_kv_blocks=None):
     """Serving engine from a HuggingFace checkpoint directory (config.json + *.safetensors / *.bin).
 
     Supported ``model_type``: llama, mistral, mixtral, qwen, qwen2, qwen2_moe, phi, phi3, falcon, opt
-    (reference inference/v2/engine_factory.py:69-130)."""
+    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun."""
     from .arch import convert_hf, spec_from_hf
     with open(os.path.join(path, "config.json")) as f:
         hf = json.load(f)
@@ -327,7 +353,7 @@ def build_hf_engine(path, engine_config=None, debug_level=None, device=None):
             sd.update(torch.load(full, map_location="cpu", weights_only=True))
     if isinstance(engine_config, dict):
         engine_config = RaggedInferenceEngineConfig.from_dict(engine_config)
-    return InferenceEngineV2(spec, convert_hf(sd, spec), engine_config, device=device)
+    return InferenceEngineV2(spec, convert_hf(sd, spec), engine_config, device=device, num_kv_blocks=num_kv_blocks)
 
 
 def build_engine_from_hf_model(hf_model, engine_config=None, device=None, num_kv_blocks=None):

@@ -1,0 +1,232 @@
+"""Decoder whose layers mix tokens in different ways: recurrent layers beside latent attention, each next to a gated MLP
+that reads the same residual (parallel block, two norms), a causal convolution in front of every sublayer, and
+optionally a run of layers that is passed several times with the same weights.
+
+Driven by :class:`arch.ArchSpec` ``layers`` / ``loop`` / ``input_conv_taps`` and served by the same engine, paged cache,
+batch metadata and decode graphs as :class:`model.RaggedTransformer`. What differs from it:
+
+* the residual stream is 32-bit; a layer is: input norm (residual add + norm + convolutions, one kernel), the mixer and
+  the gated MLP into two column blocks of one matrix, and ONE output projection [W_o | W_down] of that matrix;
+* every layer *run* (a pass of a looped layer counts) has its own paged cache rows and its own part of the sequence's
+  state row (``ragged.SequenceStatePool``): convolution tails and recurrent states, float32;
+* HCache latents are the attention runs' cached rows themselves, side by side ([1, tokens, sum of row widths]): they
+  are already the compressed form. ``restore_kv`` scatters them back; the state row travels with ``evict``.
+"""
+import torch
+
+from ...ops.input_norm import norm_rows
+from ...ops.latent_attention import copy_rows
+from ...ops.rope import rope_tables
+from .arch import run_order
+from .model import RaggedTransformer, _Layer
+from .modules import (DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig, DSUnembedConfig,
+                      instantiate_gated_mlp, instantiate_input_norm, instantiate_linear, instantiate_mixer,
+                      instantiate_unembed)
+from .modules.implementations import _PackedWeight
+
+
+class _Run:
+    """One pass of one layer: where its cached rows and its states are."""
+    __slots__ = ("layer", "cache", "tail", "state")
+
+    def __init__(self, layer, cache, tail, state):
+        self.layer, self.cache, self.tail, self.state = layer, cache, tail, state
+
+
+class HybridTransformer(RaggedTransformer):
+    # kernel sources this class runs on, for builds of just those (ops/build.py)
+    KERNEL_SOURCES = ("act.hip", "gated_scan.hip", "gemv.hip", "input_norm.hip", "latent_attn.hip")
+
+    def __init__(self, spec, weights, device, dtype=torch.bfloat16, tp_group=None, latent_mode="hidden",
+                 engine_config=None):
+        self._init_runtime(spec, device, dtype, tp_group)
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise NotImplementedError(f"{spec.model_type}: dtype {dtype} (bf16 or fp32)")
+        if latent_mode not in ("auto", "hidden", "kv"):
+            raise NotImplementedError(f"{spec.model_type}: latent_mode {latent_mode!r}; latents are the cached rows")
+        self.latent_mode = "kv"
+        self.n_q = self.n_kv = 1  # the batch's attention atoms are not used
+        self.max_positions = max(8192, getattr(getattr(engine_config, "state_manager", None), "max_context", 0))
+        self._build_modules(engine_config)
+        self._load(weights)
+        self._plan_runs()
+
+    # ------------------------------------------------------------------------------------------
+    def _build_modules(self, ec):
+        spec, H = self.spec, self.spec.hidden_size
+        self.norm_mod = instantiate_input_norm(
+            DSInputNormConfig(H, "rms", spec.norm_eps, spec.input_conv_taps, self.dtype), ec)
+        self.unembed_mod = instantiate_unembed(DSUnembedConfig(model_dim=H, vocab_size=spec.vocab_size,
+                                                               norm_type="rms"), ec)
+        self.mixers, self.mlps, self.linears = [], [], []
+        for e in spec.layers:
+            mix = instantiate_mixer(DSMixerConfig(e["mixer"]["type"], H, e["mixer"], spec.norm_eps, self.tp,
+                                                  self.dtype), ec)
+            ff = e["mlp"]["ff"] if e["mlp"] else 0
+            assert ff % self.tp == 0, "the feed-forward width must divide the tensor-parallel size"
+            ff //= self.tp
+            mlp = instantiate_gated_mlp(DSGatedMLPConfig(H, ff, e["mlp"]["act"]), ec) if e["mlp"] else None
+            lins = {"in.w": instantiate_linear(DSLinearConfig(H, mix.in_width), ec),
+                    "out.w": instantiate_linear(DSLinearConfig(mix.out_width + ff, H), ec)}
+            if mlp is not None:
+                lins["up.w"] = instantiate_linear(DSLinearConfig(H, 2 * ff), ec)
+            if hasattr(mix, "bind_tables"):
+                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base,
+                                             device=self.device))
+            self.mixers.append(mix)
+            self.mlps.append((mlp, ff))
+            self.linears.append(lins)
+
+    def _transform(self, L):
+        for k, mod in self.linears[len(self.layers)].items():
+            L.w[k] = mod.transform_param(L.w[k])
+
+    def _f32(self, x):
+        return None if x is None else x.to(device=self.device, dtype=torch.float32).contiguous()
+
+    def _load(self, sd):
+        if sd.get("__presharded__"):
+            return self._load_presharded(sd)
+        t, f, r = self._t, self._f32, self.tp_rank
+        self.embed, self.final_w = t(sd["embed"]), f(sd["final.w"].reshape(-1))
+        self.pos_embed = self.final_b = self.lm_head_b = None
+        lm = sd["lm_head.w"]
+        self.vocab = lm.shape[0]
+        vs = -(-self.vocab // self.tp)
+        shard = lm[r * vs:(r + 1) * vs]
+        if shard.shape[0] < vs:  # equal row counts on every rank; the padding columns are cut at ``vocab``
+            shard = torch.cat([shard, shard.new_zeros(vs - shard.shape[0], shard.shape[1])])
+        self.lm_head = t(shard)
+        self.layers = []
+        for i, Ls in enumerate(sd["layers"]):
+            L = _Layer()
+            mw = self.mixers[i].shard(Ls["mix"], self._rows, self._cols)
+            o = mw.pop("o.w")
+            for k, v in mw.items():
+                L.w[k] = f(v) if v.dtype == torch.float32 and v.dim() == 1 else t(v)
+            for k in ("1", "2"):
+                if Ls.get(f"ln{k}.w") is not None:
+                    L.w[f"ln{k}.w"] = f(Ls[f"ln{k}.w"].reshape(-1))
+                    cw = Ls.get(f"conv{k}.w")
+                    L.w[f"conv{k}.w"] = None if cw is None else f(cw.t())  # [taps, W]
+            if self.mlps[i][0] is not None:
+                L.w["up.w"] = t(torch.cat([self._rows(Ls["gate.w"]), self._rows(Ls["up.w"])]))
+                o = torch.cat([o, self._cols(Ls["down.w"])], 1)
+            L.w["out.w"] = t(o)
+            self._transform(L)
+            self.layers.append(L)
+
+    def _load_presharded(self, sd):
+        t, f = self._t, self._f32
+        self.embed, self.final_w, self.lm_head = t(sd["embed"]), f(sd["final.w"]), t(sd["lm_head.w"])
+        self.pos_embed = self.final_b = self.lm_head_b = None
+        self.vocab = self.spec.vocab_size
+        self.layers = []
+        for Ls in sd["layers"]:
+            L = _Layer()
+            for k, v in Ls.items():
+                if isinstance(v, dict):
+                    L.w[k] = _PackedWeight(v["q"].to(self.device), v["scales"].to(self.device),
+                                           *[int(i) for i in v["meta"]])
+                else:
+                    L.w[k] = f(v) if v.dtype == torch.float32 and k not in ("in.w", "up.w", "out.w", "ukv.w") else t(v)
+            self._transform(L)
+            self.layers.append(L)
+
+    def _plan_runs(self):
+        self.runs, off = [], 0
+        self.row_widths = []
+        for li in run_order(self.spec):
+            mix = self.mixers[li]
+            tail, off = off, off + self.norm_mod.state_floats()
+            st, off = off, off + mix.state_floats()
+            cache = None
+            if mix.cache_row:
+                cache = len(self.row_widths)
+                self.row_widths.append(mix.cache_row)
+            self.runs.append(_Run(li, cache, tail, st))
+        self._state_floats = off
+
+    # ------------------------------------------------------------------------------------------
+    def kv_cache_config(self):
+        return dict(num_layers=len(self.row_widths), n_kv_heads=1, head_dim=0, row_widths=self.row_widths)
+
+    def state_floats(self):
+        return max(1, self._state_floats)
+
+    def save_state(self, batch):
+        return self.state_pool.data.index_select(0, batch.slots.long())
+
+    def load_state(self, batch, snapshot):
+        self.state_pool.data.index_copy_(0, batch.slots.long(), snapshot)
+
+    def decode_graph_eligible(self, batch, capture_latents):
+        return self.dtype == torch.bfloat16 and super().decode_graph_eligible(batch, capture_latents)
+
+    # ------------------------------------------------------------------------------------------
+    def _layer(self, run, x, delta, batch):
+        """One layer run: (new residual, this layer's output, to be added by whoever reads the residual next)."""
+        i = run.layer
+        L, mix, (mlp, ff), lins = self.layers[i], self.mixers[i], self.mlps[i], self.linears[i]
+        state = self.state_pool.data
+        gains, convs = [L["ln1.w"]], [L["conv1.w"]]
+        if mlp is not None:
+            gains.append(L["ln2.w"])
+            convs.append(L["conv2.w"])
+        x, ys = self.norm_mod(x, delta, gains, convs, batch, state, run.tail, embed=self.embed)
+        mid = torch.empty(batch.current_tokens, mix.out_width + ff, dtype=self.dtype, device=self.device)
+        mix(ys[0], L, lins["in.w"], mid[:, :mix.out_width], batch,
+            None if run.cache is None else self.kv_cache.get_cache(run.cache), state, run.state)
+        if mlp is not None:
+            mlp(ys[1], L["up.w"], lins["up.w"], mid[:, mix.out_width:])
+        return x, self._allreduce(lins["out.w"](mid, L["out.w"]))
+
+    @torch.no_grad()
+    def forward(self, batch, capture_latents=True, sync_latents=True, sink=None):
+        """Logits of the wanted rows and the latents ([1, T, W] on the host, or None); see the base class."""
+        T = batch.current_tokens
+        x = delta = None
+        for run in self.runs:
+            x, delta = self._layer(run, x, delta, batch)
+        idx = batch.last_token_idx
+        if idx.numel():
+            hl = norm_rows(x, delta, idx, self.final_w, self.spec.norm_eps)
+            logits = self.unembed_mod.project(hl, self.lm_head, None, self.tp_group, self.vocab)
+        else:
+            logits = torch.empty(0, self.vocab, dtype=self.dtype, device=self.device)
+        lat, events = None, []
+        if capture_latents:
+            rows = torch.empty(T, self.latent_width(), dtype=self.dtype, device=self.device)
+            self._each_cache(lambda c, r: copy_rows(c, r, batch.tok_seq, batch.tok_pos, batch.block_tables), rows)
+            if sink is not None:
+                sink(0, rows)
+            elif self.latent_width() == 0:
+                lat = torch.empty(1, T, 0, dtype=self.dtype)
+            else:
+                lat = self._latent_buffer(1, T)
+                self._d2h(rows, lat[0], events)
+        self.latent_event = events[-1] if events else None
+        if events and sync_latents:
+            events[-1].synchronize()
+        return logits, lat
+
+    def _each_cache(self, fn, rows):
+        o = 0
+        for c, w in enumerate(self.row_widths):
+            fn(self.kv_cache.get_cache(c), rows[:, o:o + w])
+            o += w
+
+    def latent_layers(self):
+        return 1
+
+    def latent_width(self):
+        return sum(self.row_widths)
+
+    @torch.no_grad()
+    def restore_kv(self, batch, latents):
+        """Scatter the sequences' cached rows (host latents, [1, n, W] pieces in batch order) back into their pages."""
+        pieces = list(latents) if isinstance(latents, (list, tuple)) else [latents]
+        assert sum(p.shape[1] for p in pieces) == batch.current_tokens, "latents must cover exactly the batch's tokens"
+        rows = torch.cat([p[0].to(self.device, non_blocking=True) for p in pieces])
+        self._each_cache(lambda c, r: copy_rows(c, r, batch.tok_seq, batch.tok_pos, batch.block_tables,
+                                                to_cache=True), rows)

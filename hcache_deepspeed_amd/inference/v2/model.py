@@ -61,12 +61,7 @@ class RaggedTransformer:
 
     def __init__(self, spec, weights, device, dtype=torch.bfloat16, tp_group=None, latent_mode="hidden",
                  engine_config=None):
-        self.cfg = self.spec = spec
-        self.device = device
-        self.dtype = dtype
-        self.tp_group = tp_group
-        self.tp = dist.get_world_size(tp_group) if tp_group is not None else 1
-        self.tp_rank = dist.get_rank(tp_group) if tp_group is not None else 0
+        self._init_runtime(spec, device, dtype, tp_group)
         # "auto": the smaller lossless latent per token-layer -- pre-RoPE K|V for GQA models (2*Hkv*D < H), the hidden
         # state otherwise (HCache's byte advantage, MHA)
         if latent_mode == "auto":
@@ -88,11 +83,18 @@ class RaggedTransformer:
                                              spec.rope_scaling, device=device)
         else:
             self.cos = self.sin = None
+
+    def _init_runtime(self, spec, device, dtype, tp_group):
+        self.cfg = self.spec = spec
+        self.device = device
+        self.dtype = dtype
+        self.tp_group = tp_group
+        self.tp = dist.get_world_size(tp_group) if tp_group is not None else 1
+        self.tp_rank = dist.get_rank(tp_group) if tp_group is not None else 0
         self.kv_cache = None
         self.copy_stream = torch.cuda.Stream(device) if device.type == "cuda" else None
         self._decode_graphs = {}
         self._graph_pool = None
-        import os as _os
         # HCache latents inside the decode graph (device ring drained every `decode_latent_ring_steps` steps)
         self.decode_graph_latents = _os.environ.get("HDS_V2_DECODE_GRAPH_LATENTS", "1") == "1"
         self.decode_latent_ring_steps = int(_os.environ.get("HDS_V2_LATENT_RING_STEPS", "16"))
@@ -240,8 +242,20 @@ class RaggedTransformer:
     def kv_cache_config(self):
         return dict(num_layers=self.spec.num_hidden_layers, n_kv_heads=self.n_kv, head_dim=self.d)
 
-    def set_kv_cache(self, kv_cache):
+    def state_floats(self):
+        """float32 values of unpaged per-sequence state (recurrent layers); 0: the paged cache holds everything."""
+        return 0
+
+    def set_kv_cache(self, kv_cache, state_pool=None):
         self.kv_cache = kv_cache
+        self.state_pool = state_pool
+
+    def save_state(self, batch):
+        """Device copy of the unpaged state of the batch's sequences (None without any)."""
+        return None
+
+    def load_state(self, batch, snapshot):
+        pass
 
     def _allreduce(self, x):
         if self.tp > 1:
@@ -324,7 +338,7 @@ class RaggedTransformer:
                 or self.spec.moe is not None or self.decode_graph_max_batch <= 0):
             return False
         S = batch.current_sequences
-        return (0 < S <= self.decode_graph_max_batch and batch.current_tokens == S
+        return (batch.logits_of_last_tokens and 0 < S <= self.decode_graph_max_batch and batch.current_tokens == S
                 and getattr(batch, "atoms", None) is not None and getattr(batch, "_dev_meta", None) is not None)
 
     @torch.no_grad()
@@ -342,7 +356,7 @@ class RaggedTransformer:
         key = (B, bool(capture_latents))
         g = self._decode_graphs.get(key)
         n = batch.seq_meta.numel() + batch.tok_seq.numel() + batch.tok_pos.numel() + batch.last_token_idx.numel() \
-            + batch.block_tables.numel() + batch.atoms.numel()
+            + batch.block_tables.numel() + batch.atoms.numel() + batch.slots.numel()
         if g is None:
             ring = _LatentRing(self, B, self.decode_latent_ring_steps) if capture_latents else None
             g = self._decode_graphs[key] = _DecodeGraph(self, batch, n, ring)
@@ -442,6 +456,10 @@ class RaggedTransformer:
     _latent_pool = None
 
     INT8_GROUP = 128  # hidden_int8: one fp32 scale per 128 channels (3 % of the bytes)
+
+    def latent_layers(self):
+        """Leading dimension of the latents ([latent_layers, tokens, latent_width])."""
+        return self.spec.num_hidden_layers
 
     def latent_width(self):
         """Elements of one token-layer latent (bytes for the quantized modes)."""
@@ -597,7 +615,7 @@ class _LatentRing:
     def __init__(self, model, B, steps):
         self.model = model
         self.R = max(1, int(steps))
-        L = model.spec.num_hidden_layers
+        L = model.latent_layers()
         self.dtype = torch.uint8 if model.latent_mode in ("hidden_fp8", "hidden_int8") else model.dtype
         self.shape = (L, B, model.latent_width())
         self.dev = torch.empty((2 * self.R, ) + self.shape, dtype=self.dtype, device=model.device)
@@ -712,6 +730,10 @@ class _DecodeGraph:
         sb.block_tables = take(B * mb, (B, mb))
         sb.atoms = take(3 * A, (A, 3))
         sb.n_atoms = A
+        sb.slots = take(B, (B, ))
+        sb.max_new = 1
+        sb.plans = {}
+        sb.logits_of_last_tokens = True
         sb.current_tokens = B
         sb.current_sequences = B
         sb.seq_meta_host = None
@@ -727,8 +749,11 @@ class _DecodeGraph:
         cap = self.ring is not None
         sink = self.ring.sink if cap else None
         with torch.cuda.stream(side):
-            # warm-up: hipBLASLt / GEMV handles, KV (idempotent); its latents go to the slot the replay rewrites
+            # warm-up: hipBLASLt / GEMV handles, KV (idempotent; recurrent state is put back); its latents go to the
+            # slot the replay rewrites
+            snap = model.save_state(self.batch)
             model.forward(self.batch, capture_latents=cap, sink=sink)
+            model.load_state(self.batch, snap)
         cur.wait_stream(side)
         if model._graph_pool is None:
             model._graph_pool = torch.cuda.graph_pool_handle()

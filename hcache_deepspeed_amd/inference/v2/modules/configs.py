@@ -51,6 +51,32 @@ class DSNormConfig:
 
 
 @dataclass
+class DSInputNormConfig:
+    channels: int
+    type: str = "rms"
+    eps: float = 1e-6
+    conv_taps: int = 1  # 1: the current token only
+    input_dtype: torch.dtype = torch.bfloat16
+
+
+@dataclass
+class DSMixerConfig:
+    type: str            # registered mixer name
+    model_dim: int
+    params: dict         # the mixer's sizes and constants
+    eps: float = 1e-6    # of norms inside the mixer
+    tp: int = 1
+    input_dtype: torch.dtype = torch.bfloat16
+
+
+@dataclass
+class DSGatedMLPConfig:
+    model_dim: int
+    intermediate_features: int
+    activation: str = "silu"
+
+
+@dataclass
 class DSEmbeddingsConfig:
     residual_dtype: torch.dtype = torch.bfloat16
     embedding_dim: int = 0

@@ -2,9 +2,10 @@
 :36-195). The engine config's ``quantization.quantization_mode`` picks the weight-only linear ("wf6af16" -> FP6,
 "int8"/"int4" -> group INT); everything else has one MI355X implementation per interface today, chosen here so
 that adding a variant (e.g. an FP8 prefill GEMM) touches only this file and the registry."""
-from .configs import (DSEmbeddingsConfig, DSLinearConfig, DSMoEConfig, DSNormConfig, DSSelfAttentionConfig,
-                      DSUnembedConfig)
-from .interfaces import (DSEmbeddingRegistry, DSLinearRegistry, DSMoERegistry, DSPostNormRegistry, DSPreNormRegistry,
+from .configs import (DSEmbeddingsConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig,
+                      DSMoEConfig, DSNormConfig, DSSelfAttentionConfig, DSUnembedConfig)
+from .interfaces import (DSEmbeddingRegistry, DSGatedMLPRegistry, DSInputNormRegistry, DSLinearRegistry,
+                         DSMixerRegistry, DSMoERegistry, DSPostNormRegistry, DSPreNormRegistry,
                          DSSelfAttentionRegistry, DSUnembedRegistry)
 from .module_registry import ConfigBundle
 from . import implementations  # noqa: F401  (registers the implementations)
@@ -53,6 +54,18 @@ def instantiate_post_norm(norm_config: DSNormConfig, engine_config=None):
 def instantiate_pre_norm(norm_config: DSNormConfig, engine_config=None):
     name = "ds_pre_rms" if norm_config.type == "rms" else "ds_pre_ln"
     return DSPreNormRegistry.instantiate_config(ConfigBundle(name, norm_config))
+
+
+def instantiate_input_norm(config: DSInputNormConfig, engine_config=None):
+    return DSInputNormRegistry.instantiate_config(ConfigBundle("rms_input_conv", config))
+
+
+def instantiate_mixer(config: DSMixerConfig, engine_config=None):
+    return DSMixerRegistry.instantiate_config(ConfigBundle(config.type, config))
+
+
+def instantiate_gated_mlp(config: DSGatedMLPConfig, engine_config=None):
+    return DSGatedMLPRegistry.instantiate_config(ConfigBundle("gated_mlp_rows", config))
 
 
 def instantiate_unembed(unembed_config: DSUnembedConfig, engine_config=None):

@@ -13,13 +13,18 @@ import torch
 import torch.nn.functional as F
 
 from .... import comm as dist
-from ....ops.activations import bias_act, glu
+from ....ops.activations import bias_act, glu, glu_rows
+from ....ops.gated_scan import gated_scan, recur_step, recur_step_ok
+from ....ops.gemv import glu_gemv
 from ....ops.grouped_gemm import moe_ffn_dropless
+from ....ops.input_norm import input_norm
+from ....ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
 from ....ops.moe import moe_combine, moe_dispatch, topk_assign, topk_route
 from ....ops.norm import layer_norm, rms_norm
 from ....ops.paged import kv_rope_scatter, paged_attention
 from ....ops.quantizer import fp6_linear, int_linear, quantize, quantize_minifloat
-from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSLinearBase, DSLinearRegistry, DSMoEBase,
+from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSGatedMLPBase, DSGatedMLPRegistry, DSInputNormBase,
+                         DSInputNormRegistry, DSLinearBase, DSLinearRegistry, DSMixerBase, DSMixerRegistry, DSMoEBase,
                          DSMoERegistry, DSPostNormBase, DSPostNormRegistry, DSPreNormBase, DSPreNormRegistry,
                          DSSelfAttentionBase, DSSelfAttentionRegistry, DSUnembedBase, DSUnembedRegistry)
 
@@ -278,6 +283,10 @@ class RaggedUnembed(DSUnembedBase):
                 hl, _ = layer_norm(hidden[idx], final_w, final_b, norm_eps, residual[idx])
         else:
             hl = hidden[idx] + residual[idx]
+        return self.project(hl, lm_head, lm_head_b, tp_group, vocab)
+
+    def project(self, hl, lm_head, lm_head_b=None, tp_group=None, vocab=None):
+        """Logits of already normed rows."""
         logits = F.linear(hl, lm_head, lm_head_b)
         tp = dist.get_world_size(tp_group) if tp_group is not None else 1
         if tp > 1:
@@ -285,3 +294,135 @@ class RaggedUnembed(DSUnembedBase):
             dist.all_gather(parts, logits, group=tp_group)
             logits = torch.cat(parts, -1)[:, :vocab]
         return logits
+
+
+# ---------------------------------------------------------------------------------------------------------------
+# layers with a 32-bit residual stream and mixers of several kinds
+# ---------------------------------------------------------------------------------------------------------------
+@DSInputNormRegistry.register_module
+class RmsInputConv(DSInputNormBase):
+    """Residual add, RMS norm with scalar or vector gains and a causal input convolution per sublayer, one kernel."""
+
+    @staticmethod
+    def name():
+        return "rms_input_conv"
+
+    @staticmethod
+    def supports_config(c):
+        return c.type == "rms" and 1 <= c.conv_taps <= 16
+
+    def state_floats(self):
+        n = (self._config.conv_taps - 1) * self._config.channels
+        return -(-n // 4) * 4
+
+    def forward(self, x, delta, gains, convs, batch, state, offset, embed=None):
+        c = self._config
+        return input_norm(x, delta, gains, convs, c.eps, c.conv_taps, batch, state, offset, c.input_dtype, embed)
+
+
+def _is_plain(lin):
+    return isinstance(lin, BlasFPLinear)
+
+
+@DSMixerRegistry.register_module
+class MinGRUMixer(DSMixerBase):
+    """Gated linear recurrence whose gates read the current token only (ops/gated_scan.py)."""
+
+    FUSED_ROWS = 4  # decode batches of at most this many sequences run projection and recurrence in one kernel
+
+    @staticmethod
+    def name():
+        return "mingru"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        assert config.params["width"] % config.tp == 0, "the recurrence's width must divide the tensor-parallel size"
+        self.width = self.out_width = config.params["width"] // config.tp
+        self.in_width = 3 * self.width
+
+    def state_floats(self):
+        return -(-self.width // 4) * 4
+
+    def shard(self, w, rows, cols):
+        return {"in.w": torch.cat([rows(w["z"]), rows(w["x"]), rows(w["g"])]), "o.w": cols(w["o"]),
+                "z.b": rows(w["z.b"]).float(), "x.b": rows(w["x.b"]).float()}
+
+    def forward(self, x, w, lin, out, batch, cache, state, offset):
+        if batch.max_new == 1 and _is_plain(lin) and recur_step_ok(x, w["in.w"], self.FUSED_ROWS) and \
+                x.shape[0] == batch.current_sequences:
+            return recur_step(x, w["in.w"], w["z.b"], w["x.b"], out, batch, state, offset)
+        return gated_scan(lin(x, w["in.w"]), w["z.b"], w["x.b"], out, batch, state, offset)
+
+
+@DSMixerRegistry.register_module
+class LatentAttentionMixer(DSMixerBase):
+    """Attention over compressed K/V rows, sliding window, interleaved rotation of a shared key part
+    (ops/latent_attention.py). Heads are sharded over the tensor-parallel group, the latent is computed on every
+    rank."""
+
+    @staticmethod
+    def name():
+        return "latent_attention"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        p = config.params
+        assert p["heads"] % config.tp == 0, "attention heads must divide the tensor-parallel size"
+        self.shape = LatentShape(heads=p["heads"] // config.tp, dim=p["dim"], rot=p["rot_dim"], rot_dims=p["rot_dims"],
+                                 rank=p["kv_rank"], vdim=p["vdim"], window=p["window"], scale=p["scale"],
+                                 eps=config.eps)
+        self.rope_base = p["rope_base"]
+        self.out_width = self.shape.heads * self.shape.vdim
+        self.in_width = self.shape.q_width + self.shape.row
+        self.cache_row = self.shape.row
+        self.cos = self.sin = None
+
+    def bind_tables(self, cos, sin):
+        self.cos, self.sin = cos, sin
+
+    def shard(self, w, rows, cols):
+        # q, uk, uv are laid out head by head: equal row slices are whole heads
+        return {"in.w": torch.cat([rows(w["q"]), w["dkv"]]), "o.w": cols(w["o"]),
+                "ukv.w": torch.cat([rows(w["uk"]), rows(w["uv"])]), "dkv.norm": w["dkv.norm"].float()}
+
+    def _plan(self, batch):
+        sh = self.shape
+        if batch.max_new == 1:
+            expand = False
+        else:
+            expand = can_expand(sh, self._config.input_dtype) if batch.tok_pos.is_cuda else False
+        key = (sh.window, expand)
+        plan = batch.plans.get(key)
+        if plan is None:
+            plan = batch.plans[key] = make_plan(batch.seq_meta_host if expand else [], batch.current_tokens, sh.window,
+                                                expand, batch.tok_pos.device)
+        return plan
+
+    def forward(self, x, w, lin, out, batch, cache, state, offset):
+        sh = self.shape
+        ukv = w["ukv.w"]
+        uk = ukv[:sh.heads * sh.dim].view(sh.heads, sh.dim, sh.rank)
+        uv = ukv[sh.heads * sh.dim:].view(sh.heads, sh.vdim, sh.rank)
+        return latent_attention(lin(x, w["in.w"]), sh, w["dkv.norm"], uk, uv, ukv, self.cos, self.sin, cache, batch,
+                                self._plan(batch), out)
+
+
+@DSGatedMLPRegistry.register_module
+class GatedMLPRows(DSGatedMLPBase):
+    """act(x gate^T) * (x up^T) into a column block: one GEMV for decode rows, else projection + activation kernel."""
+
+    FUSED_ROWS = 1
+
+    @staticmethod
+    def name():
+        return "gated_mlp_rows"
+
+    @staticmethod
+    def supports_config(c):
+        return c.activation in _PLAIN_ACTS
+
+    def forward(self, x, w, lin, out):
+        act = self._config.activation
+        if x.shape[0] <= self.FUSED_ROWS and _is_plain(lin) and glu_gemv(x, w, act, out):
+            return out
+        return glu_rows(lin(x, w), act, out)

@@ -32,6 +32,26 @@ class DSUnembedBase(DSModuleBase):
     token [n_seqs, V_local]."""
 
 
+class DSInputNormBase(DSModuleBase):
+    """forward(x32, delta, gains, convs, batch, state, offset, embed) -> (new 32-bit residual, [one row matrix per
+    gain]); ``state_floats()`` per sequence."""
+
+
+class DSMixerBase(DSModuleBase):
+    """Token mixer of one layer. ``in_width`` / ``out_width`` (this rank's); ``cache_row``: values a token stores in
+    the paged cache; ``state_floats()``: unpaged float32 state per sequence; ``shard(weights, rows, cols)`` -> this
+    rank's weights, with the input projection "in.w" and the output projection "o.w";
+    forward(x, weights, lin, out, batch, cache, state, offset) fills ``out`` [T, out_width]."""
+    cache_row = 0
+
+    def state_floats(self):
+        return 0
+
+
+class DSGatedMLPBase(DSModuleBase):
+    """forward(x [T, in], w [gate; up], lin, out [T, I])."""
+
+
 def _registry(base):
 
     class _R(DSModuleRegistryBase):
@@ -52,3 +72,6 @@ DSPreNormRegistry = _registry(DSPreNormBase)
 DSPostNormRegistry = _registry(DSPostNormBase)
 DSEmbeddingRegistry = _registry(DSEmbeddingBase)
 DSUnembedRegistry = _registry(DSUnembedBase)
+DSInputNormRegistry = _registry(DSInputNormBase)
+DSMixerRegistry = _registry(DSMixerBase)
+DSGatedMLPRegistry = _registry(DSGatedMLPBase)

@@ -95,6 +95,7 @@ class DSSequenceDescriptor:
         self.tracking_id = tracking_id
         self.seen_tokens = 0
         self.in_flight_tokens = 0
+        self.evicted_state = None  # (tokens seen, host copy of the state row) of an evicted sequence
         self._blocks: List[int] = []
         self.max_blocks = max_blocks
 
@@ -129,12 +130,15 @@ class DSSequenceDescriptor:
 # KV cache
 # -----------------------------------------------------------------------------------------------
 class BlockedKVCache:
-    """Per-layer paged K/V storage: ``cache[layer]`` is [num_blocks, block_size, 2, n_kv_heads, head_dim]."""
+    """Per-layer paged K/V storage: ``cache[layer]`` is [num_blocks, block_size, 2, n_kv_heads, head_dim], or, with
+    ``row_widths`` (one number per cached layer: what a token stores there, e.g. a compressed K/V row),
+    [num_blocks, block_size, row_widths[layer]]. One block table serves every layer."""
 
     def __init__(self, num_layers, n_kv_heads, head_dim, block_size, dtype, device, memory_config, tp_group=None,
-                 num_blocks=None):
+                 num_blocks=None, row_widths=None):
         self.num_layers, self.n_kv_heads, self.head_dim, self.block_size = num_layers, n_kv_heads, head_dim, block_size
-        per_block = num_layers * block_size * 2 * n_kv_heads * head_dim * torch.tensor([], dtype=dtype).element_size()
+        row = num_layers * 2 * n_kv_heads * head_dim if row_widths is None else sum(row_widths)
+        per_block = max(1, block_size * row * torch.tensor([], dtype=dtype).element_size())
         if num_blocks is None:
             if device.type == "cuda":
                 free, _ = torch.cuda.mem_get_info(device)
@@ -144,12 +148,15 @@ class BlockedKVCache:
                     budget = min(free, memory_config.size)
             else:
                 budget = memory_config.size if memory_config.mode == "allocate" else 256 * 2**20
-            num_blocks = max(1, budget // per_block)
+            num_blocks = max(1, min(budget // per_block, 1 << 22))
             if tp_group is not None and dist.get_world_size(tp_group) > 1:
                 t = torch.tensor([num_blocks], device=device if device.type == "cuda" else "cpu")
                 dist.all_reduce(t, op=dist.ReduceOp.MIN, group=tp_group)
                 num_blocks = int(t.item())
         self.num_blocks = int(num_blocks)
+        if row_widths is not None:
+            self.cache = [torch.zeros(self.num_blocks, block_size, w, dtype=dtype, device=device) for w in row_widths]
+            return
         self.cache = torch.zeros(num_layers, self.num_blocks, block_size, 2, n_kv_heads, head_dim, dtype=dtype,
                                  device=device)
 
@@ -158,6 +165,22 @@ class BlockedKVCache:
 
     def offload(self, blocks):
         raise NotImplementedError("use the HCache latent path (put() -> latents, restore_kv()) to move KV off-GPU")
+
+
+class SequenceStatePool:
+    """Fixed-size per-sequence state that is not paged (recurrent states, convolution tails): one float32 row per
+    tracked sequence, indexed by the descriptor's ``tracking_id``. A row is not cleared when its slot is reused: the
+    kernels take a sequence without earlier tokens as starting from zero."""
+
+    def __init__(self, num_slots, floats_per_slot, device):
+        self.floats = int(floats_per_slot)
+        self.data = torch.zeros(num_slots, max(4, -(-self.floats // 4) * 4), dtype=torch.float32, device=device)
+
+    def export(self, slot):
+        return self.data[slot].to("cpu", copy=True)
+
+    def load(self, slot, row):
+        self.data[slot].copy_(row)
 
 
 # -----------------------------------------------------------------------------------------------
@@ -239,19 +262,26 @@ class RaggedBatchWrapper:
         self._seqs: List[DSSequenceDescriptor] = []
         self._tokens: List[torch.Tensor] = []
         self.seq_meta_host = []  # (q_start, n_new, seen)
+        self._logit_rows = None  # explicit logits rows (default: each sequence's last token)
         self.current_tokens = 0
 
     @property
     def current_sequences(self):
         return len(self._seqs)
 
-    def insert_sequence(self, seq: DSSequenceDescriptor, tokens: torch.Tensor, do_checks=True):
+    def insert_sequence(self, seq: DSSequenceDescriptor, tokens: torch.Tensor, do_checks=True, logits_at=None):
+        """``logits_at``: the places among ``tokens`` whose logits are wanted (default: the last one); given for one
+        sequence of a batch it must be given for all of them."""
         n = int(tokens.numel())
         if do_checks:
             if self.current_tokens + n > self._config.max_ragged_batch_size:
                 raise RuntimeError("ragged batch token budget exceeded")
             if len(self._seqs) + 1 > self._config.max_ragged_sequence_count:
                 raise RuntimeError("ragged batch sequence budget exceeded")
+        if logits_at is not None:
+            if any(not 0 <= int(i) < n for i in logits_at):
+                raise ValueError(f"logits_at outside the sequence's {n} new tokens")
+            self._logit_rows = (self._logit_rows or []) + [self.current_tokens + int(i) for i in logits_at]
         self.seq_meta_host.append((self.current_tokens, n, seq.seen_tokens))
         self._seqs.append(seq)
         self._tokens.append(tokens.reshape(-1).to(torch.int64))
@@ -296,12 +326,17 @@ class RaggedBatchWrapper:
         need = ctypes.c_int64(0)
         lib.hds_ragged_meta_build(P(n_new), P(seen), S, P(flat), P(off), mb, n_q, n_kv, rpa, None, 0,
                                   ctypes.byref(need))
-        si, host = self._pinned_slot(int(need.value))
+        # after the builder's part: the sequences' state slots, then explicit logits rows
+        extra = [seq.tracking_id for seq in self._seqs] + (self._logit_rows or [])
+        si, host = self._pinned_slot(int(need.value) + len(extra))
         A = lib.hds_ragged_meta_build(P(n_new), P(seen), S, P(flat), P(off), mb, n_q, n_kv, rpa,
                                       ctypes.c_void_p(host.data_ptr()), host.numel(), ctypes.byref(need))
         if A < 0:
             raise RuntimeError(f"ragged metadata builder failed ({A})")
         n = int(need.value)
+        if extra:
+            host.numpy()[n:n + len(extra)] = extra
+        n += len(extra)
         dev_buf = self.__dict__.get("_dev_meta")
         if dev_buf is None or dev_buf.numel() < n:
             dev_buf = self._dev_meta = torch.empty(max(n, 4096), dtype=torch.int32, device=self.device)
@@ -328,6 +363,14 @@ class RaggedBatchWrapper:
         self.block_tables = take(S * mb, (S, mb))
         self.atoms = take(3 * A, (A, 3)) if hasattr(self, "_geom") else None
         self.n_atoms = int(A) if hasattr(self, "_geom") else None
+        if self.atoms is None:
+            take(3 * A, (3 * A, ))
+        self.slots = take(S, (S, ))
+        self.slots_host = [seq.tracking_id for seq in self._seqs]
+        self.max_new = int(n_new.max()) if S else 0
+        self.plans = {}
+        if self._logit_rows is not None:
+            self.last_token_idx = take(len(self._logit_rows), (-1, ))
         self.tables_host = host[4 * S + 2 * T:4 * S + 2 * T + S * mb].view(S, mb).clone() if S else \
             torch.zeros(1, mb, dtype=torch.int32)
         if S == 0:  # keep 1-row shapes for empty batches (kernels never run on them)
@@ -343,3 +386,8 @@ class RaggedBatchWrapper:
     @property
     def _inflight_seq_descriptors_shadow(self):
         return [(q0, nn, seen, 0) for (q0, nn, seen) in self.seq_meta_host]
+
+    @property
+    def logits_of_last_tokens(self):
+        """Logits are wanted for exactly each sequence's last token."""
+        return self._logit_rows is None or self._logit_rows == [q0 + n - 1 for (q0, n, _) in self.seq_meta_host]

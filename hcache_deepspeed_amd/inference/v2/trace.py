@@ -1,0 +1,85 @@
+"""Trace replay: feed given token ids through a served model step by step and write the logits that are asked for.
+
+    bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N < steps.jsonl
+
+One JSON object a line on standard input is one step, i.e. one ragged batch through the engine's ``put``:
+
+    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+
+``entries``: requests with their next tokens and the places among them whose logits are wanted; ``end``: requests that
+are finished after the step (``flush``). A step with wanted places writes ``OUT/<step>.f32``: little-endian float32
+[wanted, vocab] in the order of the entries and of ``want``. Every step answers ``done <step>`` on standard output.
+
+The KV pool is made for ``--max-tokens`` tokens and the engine tracks at most ``--max-requests`` (4) requests, so pages
+and state slots are used again. Nothing is sampled."""
+import argparse
+import json
+import os
+import sys
+
+
+def build_engine(model_dir, dtype, max_tokens, max_requests=4, block_size=64, device=None):
+    from .engine import build_hf_engine
+    blocks = -(-max_tokens // block_size)
+    conf = {"dtype": {"bfloat16": "bf16", "float32": "fp32"}[dtype],
+            "state_manager": {"max_context": blocks * block_size, "max_ragged_batch_size": blocks * block_size,
+                              "max_tracked_sequences": max_requests, "kv_block_size": block_size}}
+    return build_hf_engine(model_dir, conf, device=device, num_kv_blocks=blocks)
+
+
+def run_step(engine, step, out_dir):
+    """One step; returns the logits [wanted, vocab] (float32, host) or None."""
+    import torch
+    logits = None
+    entries = step.get("entries") or []
+    if entries:
+        wanted = [list(e.get("want") or []) for e in entries]
+        got, _ = engine.put([e["id"] for e in entries], [torch.tensor(e["tokens"], dtype=torch.int64) for e in entries],
+                            capture_latents=False, logits_at=wanted)
+        if any(wanted):
+            logits = got.float().cpu()
+            path = os.path.join(out_dir, f"{step['step']}.f32")
+            with open(path, "wb") as f:
+                f.write(logits.numpy().astype("<f4").tobytes())
+    for uid in step.get("end") or []:
+        engine.flush(uid)
+    return logits
+
+
+def _load_needed_kernels(model_dir):
+    """Compile (first call of a checkout) only the kernels the model's class runs on."""
+    from ...ops import native
+    from .arch import spec_from_hf
+    from .hybrid import HybridTransformer
+    with open(os.path.join(model_dir, "config.json")) as f:
+        spec = spec_from_hf(json.load(f))
+    native.load_kernels(only=HybridTransformer.KERNEL_SOURCES if spec.layers is not None else None)
+
+
+def main(argv=None):
+    ap = argparse.ArgumentParser(prog="trace_run", description="Replay a token trace through the serving engine.")
+    ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
+    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16")
+    ap.add_argument("--out", required=True, help="folder the logits are written to")
+    ap.add_argument("--max-tokens", type=int, required=True, help="most tokens live requests hold at any time")
+    ap.add_argument("--max-requests", type=int, default=4, help="most requests live at any time")
+    args = ap.parse_args(argv)
+    import torch
+    if not torch.cuda.is_available():
+        print("trace_run: no GPU", file=sys.stderr)
+        return 2
+    torch.backends.cuda.matmul.allow_tf32 = False
+    torch.set_float32_matmul_precision("highest")
+    _load_needed_kernels(args.model)
+    engine = build_engine(args.model, args.dtype, args.max_tokens, args.max_requests)
+    os.makedirs(args.out, exist_ok=True)
+    for line in sys.stdin:
+        if line.strip():
+            step = json.loads(line)
+            run_step(engine, step, args.out)
+            print(f"done {step['step']}", flush=True)
+    return 0
+
+
+if __name__ == "__main__":
+    sys.exit(main())

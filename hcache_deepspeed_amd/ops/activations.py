@@ -168,3 +168,16 @@ class _BiasActFn(torch.autograd.Function):
 
 def bias_act(x, bias=None, act="gelu"):
     return _BiasActFn.apply(x, bias, act_code(act))
+
+
+def glu_rows(gu, act, out):
+    """``glu`` without autograd into ``out`` [T, I], a (possibly strided) column block; any width."""
+    I = out.shape[1]
+    a = act_code(act)
+    if native.use_native(gu):
+        assert gu.stride(1) == 1 and out.stride(1) == 1 and gu.dtype == out.dtype
+        native.check(native.kernels().hds_glu_rows(native.dt(gu), a, gu.data_ptr(), gu.stride(0), out.data_ptr(),
+                                                   out.stride(0), gu.shape[0], I, native.stream()), "glu_rows")
+        return out
+    out.copy_(_ref_act(gu[:, :I].float(), a) * gu[:, I:].float())
+    return out

@@ -57,7 +57,7 @@ def _digest(paths, extra):
     h = hashlib.sha256()
     for p in paths:
         with open(p, "rb") as f:
-            h.update(p.encode())
+            h.update(os.path.relpath(p, PKG_DIR).encode())
             h.update(f.read())
     h.update(" ".join(extra).encode())
     return h.hexdigest()
@@ -75,17 +75,35 @@ def _stamp_ok(lib, digest):
     return os.path.exists(lib) and os.path.exists(st) and open(st).read().strip() == digest
 
 
-def build_kernels(force=False, jobs=None, verbose=False, file_flags=None, out=None):
+def subset_lib(only):
+    """Path of the library that holds just the kernel sources ``only`` (file names)."""
+    tag = hashlib.sha256(" ".join(sorted(only)).encode()).hexdigest()[:8]
+    return os.path.join(LIB_DIR, f"libhds_kernels_part_{tag}.so")
+
+
+def kernels_current():
+    """The full kernel library is built from the sources as they are."""
+    return _stamp_ok(KERNEL_LIB, _kernel_digest(_sources("kernels", (".hip",)), FILE_FLAGS))
+
+
+def _kernel_digest(srcs, file_flags):
+    return _digest(srcs + _sources("kernels", (".h",)),
+                   HIPCC_FLAGS + sorted(f"{k}:{' '.join(v)}" for k, v in file_flags.items()))
+
+
+def build_kernels(force=False, jobs=None, verbose=False, file_flags=None, out=None, only=None):
     """``file_flags`` / ``out``: an A/B build with different per-source flags into another path (loaded with
-    HDS_KERNEL_LIB=<out>); the default build uses FILE_FLAGS into _lib/libhds_kernels.so."""
+    HDS_KERNEL_LIB=<out>); the default build uses FILE_FLAGS into _lib/libhds_kernels.so. ``only``: a library of just
+    these sources (``subset_lib``), for a program that needs one model's kernels and should not wait for the rest."""
     file_flags = FILE_FLAGS if file_flags is None else file_flags
+    if only is not None:
+        out = out or subset_lib(only)
     lib_path = out or KERNEL_LIB
-    srcs = _sources("kernels", (".hip",))
-    hdrs = _sources("kernels", (".h",))
-    digest = _digest(srcs + hdrs, HIPCC_FLAGS + sorted(f"{k}:{' '.join(v)}" for k, v in file_flags.items()))
+    srcs = [s for s in _sources("kernels", (".hip",)) if only is None or os.path.basename(s) in only]
+    digest = _kernel_digest(srcs, file_flags)
     if not force and _stamp_ok(lib_path, digest):
         return lib_path
-    bdir = BUILD_DIR if out is None else BUILD_DIR + "_ab"
+    bdir = BUILD_DIR if out is None else BUILD_DIR + ("_ab" if only is None else "_part")
     os.makedirs(bdir, exist_ok=True)
     os.makedirs(os.path.dirname(lib_path), exist_ok=True)
     hipcc = os.path.join(ROCM, "bin", "hipcc")

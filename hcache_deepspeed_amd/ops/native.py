@@ -26,6 +26,20 @@ _KERNEL_SIGS = {
     "hds_rope": "ii" + "pppp" + "l" + "iii" + "l" + "ii" + "f" + "s",
     "hds_glu_fwd": "iipplis",
     "hds_glu_bwd": "iippplis",
+    "hds_glu_rows": "ii" + "plpl" + "li" + "s",
+    "hds_input_norm": "i" + "ppppp" + "pipp" + "pipp" + "p" + "l" + "pp" + "iiiii" + "f" + "s",
+    "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
+    "hds_gated_scan_chunk": "",
+    "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "ppp" + "iii" + "s",
+    "hds_gemv_recur_bf16": "ppppp" + "pl" + "pp" + "iii" + "ll" + "s",
+    "hds_latent_prep": "i" + "pl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
+    "hds_latent_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
+    "hds_latent_decode_mfma_ok": "ii",
+    "hds_latent_decode_splits": "iii",
+    "hds_latent_decode": "i" + "p" * 8 + "i" * 8 + "f" + "i" + "s",
+    "hds_latent_combine": "i" + "ppppp" + "l" + "iiiii" + "s",
+    "hds_latent_prefill_ok": "iiii",
+    "hds_latent_prefill": "plplplpl" + "p" + "i" * 8 + "f" + "s",
     "hds_glu_fwd_t": "i" + "ppp" + "ii" + "s",
     "hds_glu_bwd_t": "i" + "pppp" + "ii" + "s",
     "hds_bias_act_fwd": "iippplis",
@@ -140,8 +154,10 @@ def kernel_lib_path():
     return _build.KERNEL_LIB
 
 
-def load_kernels(build_if_missing=True):
-    """Load (building first if needed) the HIP kernel library. Returns None when unavailable."""
+def load_kernels(build_if_missing=True, only=None):
+    """Load (building first if needed) the HIP kernel library. Returns None when unavailable. ``only``: kernel source
+    names; if the full library is not built, a library of just these is built and loaded instead (a process that
+    serves one model). The first load of a process decides."""
     global _klib
     if _klib is not None:
         return _klib
@@ -151,7 +167,10 @@ def load_kernels(build_if_missing=True):
         path = os.environ.get("HDS_KERNEL_LIB") or _build.KERNEL_LIB  # override: an A/B build (ops/build.py)
         if build_if_missing and os.environ.get("HDS_NO_BUILD", "0") != "1" and not os.environ.get("HDS_KERNEL_LIB"):
             try:
-                path = _build.build_kernels()
+                part = only is not None and not _build.kernels_current()
+                if part:
+                    path = _build.subset_lib(only)
+                path = _build.build_kernels(only=only if part else None)
             except Exception:
                 if not os.path.exists(path):
                     raise
@@ -159,6 +178,14 @@ def load_kernels(build_if_missing=True):
             return None
         lib = ctypes.CDLL(path, mode=ctypes.RTLD_GLOBAL)
         _bind(lib, _KERNEL_SIGS)
+        _klib_init(lib)
+        _klib = lib
+        return _klib
+
+
+def _klib_init(lib):
+    """Process-wide kernel variants (of the sources the library holds)."""
+    if hasattr(lib, "hds_attn_fwd"):
         # FlashAttention backward with LDS reads pipelined two MFMAs ahead (csrc/kernels/flash_attn.hip PIPE; 2 = + uniform-
         # base LDS-DMA staging of full tiles: 3.80 vs 3.85 ms, profiles/r3/fa_bwd_pipe2_r3q.txt)
         lib.hds_attn_bwd_pipe(int(os.environ.get("HDS_ATTN_BWD_PIPE", "2")))
@@ -168,10 +195,9 @@ def load_kernels(build_if_missing=True):
         check(lib.hds_attn_fwd_variant(fwd_variant_default()), "hds_attn_fwd_variant")
         # FlashAttention backward dQ kernel (hds_attn_bwd_dq_variant; 1 = one wave per SIMD, 64 rows per wave)
         lib.hds_attn_bwd_dq_variant(int(os.environ.get("HDS_ATTN_DQ_VAR", "0")))
+    if hasattr(lib, "hds_skinny_set_unroll"):
         # skinny GEMM weight loads in flight per lane (16: B = 4 decode 925 vs 881 tok/s with 8, profiles/r6/skinny_u)
         lib.hds_skinny_set_unroll(int(os.environ.get("HDS_SKINNY_U", "16")))
-        _klib = lib
-        return _klib
 
 
 # FlashAttention forward variants of the shipped library (flash_attn.hip hds_attn_fwd_variant): 20 the default, 5 the
