@@ -243,8 +243,9 @@ SHAPES = {"odd": (3, 5, 6, 4, 7, 9, 11), "plain-prefill": (2, 8, 8, 8, 24, 24, 1
 
 def _attention_case(name):
     H, dim, rot, rd, rank, vd, win = SHAPES[name]
-    sh = LatentShape(heads=H, dim=dim, rot=rot, rot_dims=rd, rank=rank, vdim=vd, window=win, scale=0.3, eps=1e-4)
-    m = {"heads": H, "dim": dim, "rot_dim": rot, "vdim": vd, "kv_rank": rank, "scale": 0.3,
+    scale = min(0.3, 2.0 / math.sqrt(dim + rot))
+    sh = LatentShape(heads=H, dim=dim, rot=rot, rot_dims=rd, rank=rank, vdim=vd, window=win, scale=scale, eps=1e-4)
+    m = {"heads": H, "dim": dim, "rot_dim": rot, "vdim": vd, "kv_rank": rank, "scale": scale,
          "rot": {"dims": rd, "base": 700.0}, "mask": {"size": win or 10**9}}
     return sh, m
 
