@@ -111,9 +111,21 @@ def main():
     ap.add_argument("--comm-timing", action="store_true",
                     help="N>1: TORCH_NCCL_ENABLE_TIMING=1 for the whole run (in-step RCCL busbw in extra.comm; adds two "
                          "events per collective to the timed steps too)")
+    ap.add_argument("--serving", default=None, metavar="MODELS",
+                    help="instead of the training step: prefill and decode throughput of the ragged serving engine, "
+                    "comma-separated from llama, gofasun, gofasun-mingru, gofasun-latent (one JSON line each)")
+    ap.add_argument("--serving-sizes", default="2048,4096", help="layer widths of --serving")
+    ap.add_argument("--serving-layers", type=int, default=8)
+    ap.add_argument("--serving-prompt", type=int, default=4096)
+    ap.add_argument("--serving-batches", default="1,4,16", help="decode batch sizes of --serving")
     ap.add_argument("--deepcompile", action="store_true",
                     help="engine.compile() with DeepCompile: profiled ZeRO-3 gather schedule (selective gather + prefetch)")
     args = ap.parse_args()
+    if args.serving:
+        from hcache_deepspeed_amd.benchmarks import serving
+        serving.run(args.serving.split(","), args.serving_sizes.split(","), args.serving_layers, args.serving_prompt,
+                    [int(b) for b in args.serving_batches.split(",")], steps=32)
+        return
     if os.environ.get("HDS_HANG_DUMP"):
         # diagnosis of a stuck run: every N seconds print the Python stacks of all threads to stderr
         import faulthandler

@@ -1,0 +1,124 @@
+"""Prefill and decode throughput of the ragged serving engine on random weights of a real model's layer sizes: the hybrid
+design (Gofasun) next to the dense Llama layout at equal width, depth, feed-forward and head count
+(``bench.py --serving``). One JSON line per measurement."""
+import json
+import time
+
+import torch
+
+# name -> (width, ff, heads, kv heads of the dense model)
+SIZES = {"2048": (2048, 5632, 16, 4), "4096": (4096, 14336, 32, 8)}
+VOCAB = 32000
+HEAD, ROT, WINDOW = 128, 64, 4096
+
+
+def _rand(gen, dev, *shape, scale=None):
+    s = shape[-1]**-0.5 if scale is None else scale
+    return (torch.randn(*shape, generator=gen, device=dev, dtype=torch.float32) * s).to(torch.bfloat16)
+
+
+def dense_model(size, layers, dev, max_context):
+    from ..inference.v2.arch import ArchSpec
+    W, ff, nq, nkv = SIZES[size]
+    g = torch.Generator(device=dev).manual_seed(0)
+    spec = ArchSpec("llama", VOCAB, W, layers, nq, nkv, HEAD, ff, norm_eps=1e-5, max_position_embeddings=max_context)
+    one = torch.ones(W, device=dev, dtype=torch.bfloat16)
+    lay = [{"ln1.w": one, "ln2.w": one, "qkv.w": _rand(g, dev, (nq + 2 * nkv) * HEAD, W),
+            "o.w": _rand(g, dev, W, nq * HEAD), "up.w": _rand(g, dev, 2 * ff, W), "down.w": _rand(g, dev, W, ff)}
+           for _ in range(layers)]
+    return spec, {"embed": _rand(g, dev, VOCAB, W), "final.w": one, "lm_head.w": _rand(g, dev, VOCAB, W),
+                  "layers": lay}
+
+
+def gofasun_model(size, layers, dev, kinds=("mingru", "latent_attention")):
+    from ..inference.v2.arch import convert_hf, spec_from_hf
+    W, ff, H, _ = SIZES[size]
+    rank = W // 8
+    mixers = {"mingru": {"width": W},
+              "latent_attention": {"heads": H, "dim": HEAD, "rot_dim": ROT, "kv_rank": rank, "vdim": HEAD,
+                                   "scale": (HEAD + ROT)**-0.5, "rot": {"base": 10000.0, "dims": ROT},
+                                   "mask": {"size": WINDOW}}}
+    cfg = {"architecture": "Gofasun", "vocab": VOCAB, "width": W, "canon": {"taps": 4}, "norm": {"eps": 1e-5},
+           "loop": None,
+           "layers": [{"type": kinds[i % len(kinds)], "mixer": mixers[kinds[i % len(kinds)]],
+                       "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]}
+    g = torch.Generator(device=dev).manual_seed(0)
+    w = {"embed": _rand(g, dev, VOCAB, W), "head": _rand(g, dev, VOCAB, W), "final.norm": torch.ones((), device=dev)}
+    for i, e in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        for k in ("1", "2"):
+            w[p + "norm" + k] = torch.ones((), device=dev)
+            w[p + "canon" + k] = _rand(g, dev, W, cfg["canon"]["taps"], scale=0.1)
+        shapes = {"mlp.gate": (ff, W), "mlp.up": (ff, W), "mlp.down": (W, ff)}
+        if e["type"] == "mingru":
+            shapes.update({"mix.z": (W, W), "mix.x": (W, W), "mix.g": (W, W), "mix.o": (W, W)})
+            w[p + "mix.z.b"] = _rand(g, dev, W, scale=1.0)
+            w[p + "mix.x.b"] = _rand(g, dev, W, scale=1.0)
+        else:
+            shapes.update({"mix.q": (H * (HEAD + ROT), W), "mix.dkv": (rank + ROT, W), "mix.uk": (H * HEAD, rank),
+                           "mix.uv": (H * HEAD, rank), "mix.o": (W, H * HEAD)})
+            w[p + "mix.dkv.norm"] = torch.ones(rank, device=dev)
+        for k, s in shapes.items():
+            w[p + k] = _rand(g, dev, *s)
+    spec = spec_from_hf(cfg)
+    return spec, convert_hf(w, spec)
+
+
+def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
+    from ..inference.v2.engine import InferenceEngineV2, RaggedInferenceEngineConfig
+    if kind == "llama":
+        spec, w = dense_model(size, layers, dev, max_context)
+    else:
+        kinds = {"gofasun": ("mingru", "latent_attention"), "gofasun-mingru": ("mingru", ),
+                 "gofasun-latent": ("latent_attention", )}[kind]
+        spec, w = gofasun_model(size, layers, dev, kinds)
+    conf = RaggedInferenceEngineConfig.from_dict(dict(
+        dtype="bf16", state_manager=dict(max_context=max_context, max_ragged_batch_size=max_batch_tokens,
+                                         max_tracked_sequences=max(4, batch), kv_block_size=64)))
+    return InferenceEngineV2(spec, w, conf, device=dev, num_kv_blocks=batch * (-(-max_context // 64)))
+
+
+def _time(fn, steps, warmup):
+    for _ in range(warmup):
+        fn()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / steps
+
+
+def measure(kind, size, layers, dev, prompt, batches, steps, warmup):
+    g = torch.Generator().manual_seed(1)
+    top = max(batches)
+    ctx = prompt + 64 * (1 + (2 * (steps + warmup) + 8) // 64)
+    eng = _engine(kind, size, layers, dev, top, ctx, prompt)
+    ids = torch.randint(0, VOCAB, (prompt, ), generator=g)
+    base = {"model": kind, "width": int(size), "layers": layers}
+
+    def prefill():
+        eng.put(["p"], [ids], capture_latents=False)
+        eng.flush("p")
+
+    dt = _time(prefill, max(2, steps // 4), 2)
+    yield dict(base, phase="prefill", tokens=prompt, ms=round(dt * 1e3, 3), tok_per_s=round(prompt / dt, 1))
+    for B in batches:
+        uids = list(range(B))
+        for u in uids:
+            eng.put([u], [ids], capture_latents=False)
+        tok = [torch.tensor([5 + u]) for u in uids]
+        dt = _time(lambda: eng.put(uids, tok, capture_latents=False), steps, warmup)
+        for u in uids:
+            eng.flush(u)
+        yield dict(base, phase="decode", batch=B, context=prompt, ms=round(dt * 1e3, 3), tok_per_s=round(B / dt, 1))
+
+
+def run(models=("llama", "gofasun"), sizes=("2048", "4096"), layers=8, prompt=4096, batches=(1, 4, 16), steps=32,
+        warmup=4):
+    dev = torch.device("cuda", 0)
+    for size in sizes:
+        for kind in models:
+            for rec in measure(kind, size, layers, dev, prompt, batches, steps, warmup):
+                print(json.dumps(rec), flush=True)
+            torch.cuda.empty_cache()
