@@ -44,23 +44,22 @@ __device__ __forceinline__ void stv(T* p, const float (&v)[V]) {
   }
 }
 
-// sigmoid(x) and 1 - sigmoid(x), neither by cancellation
-__device__ __forceinline__ void sigmoid2(float x, float& s, float& c) {
-  const float e = __expf(-fabsf(x));
-  const float r = 1.f / (1.f + e);
-  s = x >= 0.f ? r : e * r;
-  c = x >= 0.f ? e * r : r;
-}
-__device__ __forceinline__ void gates(float a, float b, float& keep, float& add) {
-  float z, us, uc;
-  sigmoid2(a, z, keep);
-  sigmoid2(b, us, uc);
-  add = z * (b >= 0.f ? b + 0.5f : us);
-}
-__device__ __forceinline__ float silu(float x) {
-  float s, c;
-  sigmoid2(x, s, c);
-  return x * s;
+// 1 - z, z * v and (with OUT) g * sigmoid(g). Every sigmoid is 1 / (1 + e) or e / (1 + e) with e = exp(-|x|) <= 1 (no
+// cancellation, no overflow); one reciprocal of the product of the 1 + e serves all of them.
+template <bool OUT>
+__device__ __forceinline__ void gates(float a, float b, float g, float& keep, float& add, float& og) {
+  const float ea = __expf(-fabsf(a)), eb = __expf(-fabsf(b)), eg = OUT ? __expf(-fabsf(g)) : 0.f;
+  const float pa = 1.f + ea, pb = 1.f + eb, pg = 1.f + eg;
+  const float r = __builtin_amdgcn_rcpf(OUT ? pa * pb * pg : pa * pb);
+  const float ra = OUT ? r * (pb * pg) : r * pb;
+  const float rb = OUT ? r * (pa * pg) : r * pa;
+  keep = a >= 0.f ? ea * ra : ra;
+  const float z = a >= 0.f ? ra : ea * ra;
+  add = z * (b >= 0.f ? b + 0.5f : eb * rb);
+  if (OUT) {
+    const float rg = g * (r * (pa * pb));
+    og = g >= 0.f ? rg : eg * rg;
+  }
 }
 
 template <typename T>
@@ -107,11 +106,11 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanParams<T> p) {
     float y[V];
 #pragma unroll
     for (int i = 0; i < V; ++i) {
-      float keep, add;
-      gates(a[i] + ba[i], b[i] + bb[i], keep, add);
+      float keep, add, og;
+      gates<PASS != 1>(a[i] + ba[i], b[i] + bb[i], g[i], keep, add, og);
       s[i] = keep * s[i] + add;
       if (PASS == 1) A[i] *= keep;
-      if (PASS != 1) y[i] = s[i] * silu(g[i]);
+      if (PASS != 1) y[i] = s[i] * og;
     }
     if (PASS != 1) stv<T, V>(o, y);
   };
@@ -158,7 +157,7 @@ __global__ __launch_bounds__(64) void scan_carry_kernel(ScanParams<T> p) {
   float* st = p.state + (int64_t)p.slots[seq] * p.slot_stride + c;
   float s = seen > 0 ? *st : 0.f;
   float* ws = p.ws + (int64_t)seq * p.chunks * 2 * p.W + c;
-  constexpr int U = 8;
+  constexpr int U = 32;
   for (int k0 = 0; k0 < nc; k0 += U) {
     float A[U], B[U];
 #pragma unroll

@@ -47,6 +47,7 @@ template <> struct VecN<bf16, 4> {
   }
 };
 
+constexpr int kU = 4;         // loads in flight per lane and operand
 constexpr int kMaxRows = 64;  // rows a workgroup holds statistics of: R + 2 (taps - 1) at most
 
 template <typename T>
@@ -124,12 +125,19 @@ __global__ __launch_bounds__(NT) void input_norm_kernel(InputNormParams<T> p) {
       const bool own = r >= halo && r < halo + rows;
       const int row = q0 + i;
       float ss = 0.f;
-      for (int c = lane * V; c < p.W; c += 64 * V) {
-        float v[V];
-        load_sum<T, V>(p, row, c, v);
+      for (int c0 = lane * V; c0 < p.W; c0 += 64 * V * kU) {
+        float v[kU][V];
 #pragma unroll
-        for (int k = 0; k < V; ++k) ss += v[k] * v[k];
-        if (own) VecN<float, V>::store(p.x_out + (int64_t)row * p.W + c, v);
+        for (int k = 0; k < kU; ++k)
+          if (c0 + 64 * V * k < p.W) load_sum<T, V>(p, row, c0 + 64 * V * k, v[k]);
+#pragma unroll
+        for (int k = 0; k < kU; ++k) {
+          const int c = c0 + 64 * V * k;
+          if (c >= p.W) continue;
+#pragma unroll
+          for (int i2 = 0; i2 < V; ++i2) ss += v[k][i2] * v[k][i2];
+          if (own) VecN<float, V>::store(p.x_out + (int64_t)row * p.W + c, v[k]);
+        }
       }
       ss = wave_sum(ss);
       if (lane == 0) s_rstd[r] = 1.f / sqrtf(ss / (float)p.W + p.eps);
@@ -172,33 +180,41 @@ __global__ __launch_bounds__(NT) void input_norm_kernel(InputNormParams<T> p) {
         if (k <= m && p.w[o] != nullptr) VecN<float, V>::load(p.w[o] + (int64_t)(m - k) * p.W + c, w[o][k]);
       }
     }
-    for (int r = 0; r < rows; ++r) {
-      const int row = q0 + start + r;
-      float u[V];
-      load_sum<T, V>(p, row, c, u);
-      const float rs = s_rstd[halo + r];
+    for (int r0 = 0; r0 < rows; r0 += kU) {
+      float us[kU][V];
 #pragma unroll
-      for (int i = 0; i < V; ++i) u[i] *= rs;
+      for (int b = 0; b < kU; ++b)
+        if (r0 + b < rows) load_sum<T, V>(p, q0 + start + r0 + b, c, us[b]);
 #pragma unroll
-      for (int o = 0; o < 2; ++o) {
-        if (o >= nout) break;
-        float y[V];
+      for (int b = 0; b < kU; ++b) {
+        const int r = r0 + b;
+        if (r >= rows) break;
+        const int row = q0 + start + r;
+        float (&u)[V] = us[b];
+        const float rs = s_rstd[halo + r];
 #pragma unroll
-        for (int i = 0; i < V; ++i) {
-          float a = u[i] + w[o][0][i] * u[i];
+        for (int i = 0; i < V; ++i) u[i] *= rs;
 #pragma unroll
-          for (int k = 0; k < M; ++k) a += w[o][k + 1][i] * hist[k][i];
-          y[i] = a * g[o][i];
+        for (int o = 0; o < 2; ++o) {
+          if (o >= nout) break;
+          float y[V];
+#pragma unroll
+          for (int i = 0; i < V; ++i) {
+            float a = u[i] + w[o][0][i] * u[i];
+#pragma unroll
+            for (int k = 0; k < M; ++k) a += w[o][k + 1][i] * hist[k][i];
+            y[i] = a * g[o][i];
+          }
+          VecN<T, V>::store(p.y[o] + (int64_t)row * p.W + c, y);
         }
-        VecN<T, V>::store(p.y[o] + (int64_t)row * p.W + c, y);
-      }
 #pragma unroll
-      for (int k = M - 1; k > 0; --k)
+        for (int k = M - 1; k > 0; --k)
 #pragma unroll
-        for (int i = 0; i < V; ++i) hist[k][i] = hist[k - 1][i];
-      if (M > 0) {
+          for (int i = 0; i < V; ++i) hist[k][i] = hist[k - 1][i];
+        if (M > 0) {
 #pragma unroll
-        for (int i = 0; i < V; ++i) hist[0][i] = u[i];
+          for (int i = 0; i < V; ++i) hist[0][i] = u[i];
+        }
       }
     }
     if (first && m > 0) {
@@ -219,6 +235,78 @@ __global__ __launch_bounds__(NT) void input_norm_kernel(InputNormParams<T> p) {
         VecN<float, V>::store(tail + (int64_t)e * p.W + c, u);
       }
     }
+  }
+}
+
+// One new token per sequence: a workgroup of 1024 threads a row, P * 4 columns a thread. Everything the row needs is
+// requested before the reduction, so the step is one memory round trip and one barrier long.
+template <typename T, int M, int P>
+__global__ __launch_bounds__(1024) void input_norm_step_kernel(InputNormParams<T> p) {
+  __shared__ float s_part[16];
+  const int seq = blockIdx.x;
+  if (p.seq_meta[3 * seq + 1] <= 0) return;
+  const int row = p.seq_meta[3 * seq], seen = p.seq_meta[3 * seq + 2];
+  const int m = p.taps - 1;
+  float* tail = M > 0 ? p.tail + (int64_t)p.slots[seq] * p.slot_stride : nullptr;
+  const int nout = p.y[1] != nullptr ? 2 : 1;
+  float u[P][4], hist[P][M > 0 ? M : 1][4], w[P][2][M + 1][4], g[P][2][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int q = 0; q < P; ++q) {
+    const int c = (q * 1024 + threadIdx.x) * 4;
+    if (c >= p.W) continue;
+    load_sum<T, 4>(p, row, c, u[q]);
+#pragma unroll
+    for (int k = 0; k < M; ++k) {  // hist[k]: k + 1 back; entries before the sequence's start are zero
+#pragma unroll
+      for (int i = 0; i < 4; ++i) hist[q][k][i] = 0.f;
+      if (k < m && seen - 1 - k >= 0) VecN<float, 4>::load(tail + (int64_t)(m - 1 - k) * p.W + c, hist[q][k]);
+    }
+#pragma unroll
+    for (int o = 0; o < 2; ++o) {
+      if (o >= nout) break;
+#pragma unroll
+      for (int k = 0; k <= M; ++k) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) w[q][o][k][i] = 0.f;
+        if (k <= m && p.w[o] != nullptr) VecN<float, 4>::load(p.w[o] + (int64_t)(m - k) * p.W + c, w[q][o][k]);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) g[q][o][i] = p.g[o][p.gs[o] ? c + i : 0];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ss += u[q][i] * u[q][i];
+  }
+  ss = wave_sum(ss);
+  if ((threadIdx.x & 63) == 0) s_part[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) ss += s_part[i];
+  const float rs = 1.f / sqrtf(ss / (float)p.W + p.eps);
+#pragma unroll
+  for (int q = 0; q < P; ++q) {
+    const int c = (q * 1024 + threadIdx.x) * 4;
+    if (c >= p.W) continue;
+    VecN<float, 4>::store(p.x_out + (int64_t)row * p.W + c, u[q]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u[q][i] *= rs;
+#pragma unroll
+    for (int o = 0; o < 2; ++o) {
+      if (o >= nout) break;
+      float y[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float a = u[q][i] + w[q][o][0][i] * u[q][i];
+#pragma unroll
+        for (int k = 0; k < M; ++k) a += w[q][o][k + 1][i] * hist[q][k][i];
+        y[i] = a * g[q][o][i];
+      }
+      VecN<T, 4>::store(p.y[o] + (int64_t)row * p.W + c, y);
+    }
+#pragma unroll
+    for (int k = 0; k < M; ++k)
+      if (k < m) VecN<float, 4>::store(tail + (int64_t)(m - 1 - k) * p.W + c, k == 0 ? u[q] : hist[q][k > 0 ? k - 1 : 0]);
   }
 }
 
@@ -252,13 +340,18 @@ template <typename T, int V, int NT>
 int launch_input_norm(const InputNormParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
   const dim3 grid((max_new + p.R - 1) / p.R, n_seqs);
   const int m = p.taps - 1;
+  if constexpr (V == 1) {
+    if (m > 3) {
+      if (m <= 7) hipLaunchKernelGGL((input_norm_kernel<T, 1, 7, NT>), grid, dim3(NT), 0, st, p);
+      else hipLaunchKernelGGL((input_norm_kernel<T, 1, 15, NT>), grid, dim3(NT), 0, st, p);
+      return hipGetLastError();
+    }
+  }
 #define HDS_IN(MM) hipLaunchKernelGGL((input_norm_kernel<T, V, MM, NT>), grid, dim3(NT), 0, st, p)
   if (m == 0) HDS_IN(0);
   else if (m == 1) HDS_IN(1);
   else if (m == 2) HDS_IN(2);
-  else if (m == 3) HDS_IN(3);
-  else if (m <= 7) HDS_IN(7);
-  else HDS_IN(15);
+  else HDS_IN(3);
 #undef HDS_IN
   return hipGetLastError();
 }
@@ -266,11 +359,15 @@ int launch_input_norm(const InputNormParams<T>& p, int n_seqs, int max_new, hipS
 template <typename T>
 int input_norm(const InputNormParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
   const bool v4 = p.W % 4 == 0 && p.slot_stride % 4 == 0;
-  if (max_new == 1) {
-    if (v4) return launch_input_norm<T, 4, 512>(p, n_seqs, max_new, st);
-    return launch_input_norm<T, 1, 512>(p, n_seqs, max_new, st);
+  if (max_new == 1 && v4 && p.taps <= 4 && p.W <= 8192) {
+#define HDS_IS(MM)                                                                                              \
+  if (p.W <= 4096) hipLaunchKernelGGL((input_norm_step_kernel<T, MM, 1>), dim3(n_seqs), dim3(1024), 0, st, p); \
+  else hipLaunchKernelGGL((input_norm_step_kernel<T, MM, 2>), dim3(n_seqs), dim3(1024), 0, st, p)
+    if (p.taps == 1) { HDS_IS(0); } else if (p.taps == 2) { HDS_IS(1); } else if (p.taps == 3) { HDS_IS(2); } else { HDS_IS(3); }
+#undef HDS_IS
+    return hipGetLastError();
   }
-  if (v4) return launch_input_norm<T, 4, 256>(p, n_seqs, max_new, st);
+  if (v4 && p.taps <= 4) return launch_input_norm<T, 4, 512>(p, n_seqs, max_new, st);
   return launch_input_norm<T, 1, 256>(p, n_seqs, max_new, st);
 }
 

@@ -51,10 +51,156 @@ __device__ __forceinline__ float rotated(const T* v, int e, int rdims, const flo
   return (e & 1) ? x * cc + y * ss : x * cc - y * ss;
 }
 
-constexpr int kAbsTok = 4;  // absorbed tokens that share one read of W_uk[h]
+// 8 elements e .. e + 7 of a rotated part (rdims and e multiples of 8)
+template <typename T>
+__device__ __forceinline__ void rotate8(float (&v)[8], int e, int rdims, const float* c, const float* s) {
+  if (e >= rdims) return;
+  const f32x4 cc = *reinterpret_cast<const f32x4*>(c + e / 2), sn = *reinterpret_cast<const f32x4*>(s + e / 2);
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float a = v[2 * k], b = v[2 * k + 1];
+    v[2 * k] = a * cc[k] - b * sn[k];
+    v[2 * k + 1] = b * cc[k] + a * sn[k];
+  }
+}
 
-// workgroups [0, n_tok): one token each (norm, rotation, scatter, q of expanded tokens rotated in place);
-// then ceil(n_abs / kAbsTok) x H: absorption
+constexpr int kAbsTok = 4;    // absorbed tokens that share one read of W_uk[h]
+constexpr int kAbsCols = 128; // latent columns of an absorption workgroup (vector path)
+
+// Vector path (all part sizes multiples of 8, rank <= 2048). Workgroups [0, n_tok): one token each (norm, rotation,
+// scatter, q of expanded tokens rotated in place); then one per (head, kAbsCols columns, kAbsTok absorbed tokens).
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
+  extern __shared__ float sm[];
+  const int qh = p.dim + p.rot, row_w = p.rank + p.rot;
+  const int half = p.rdims / 2;
+  if ((int)blockIdx.x < p.n_tok) {
+    const int t = blockIdx.x;
+    const int pos = min(p.tok_pos[t], p.n_pos - 1);
+    const float* ct = p.cos_t + (int64_t)pos * half;
+    const float* st = p.sin_t + (int64_t)pos * half;
+    T* row = p.qd + (int64_t)t * p.ld;
+    const T* c = row + (int64_t)p.H * qh;
+    const int nc = row_w / 8;
+    const int i = threadIdx.x;  // chunk of the row; rows of more than 256 chunks loop below for the rotated part only
+    float v[8];
+    float ss = 0.f;
+    if (8 * i < p.rank) {
+      Vec8<T>::load(c + 8 * i, v);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) ss += v[k] * v[k];
+    }
+    const int blk = p.tables[(int64_t)p.tok_seq[t] * p.max_blocks + pos / p.block_size];
+    T* dst = p.cache + ((int64_t)blk * p.block_size + pos % p.block_size) * row_w;
+    const int wr = p.ws_row != nullptr ? p.ws_row[t] : -1;
+    T* dst2 = wr >= 0 ? p.ws + (int64_t)wr * row_w : nullptr;
+    if (wr >= 0) {
+      const int nq = p.rdims / 8;
+      for (int q = threadIdx.x; q < p.H * nq; q += 256) {
+        const int h = q / nq, e = 8 * (q - h * nq);
+        T* a = row + (int64_t)h * qh + p.dim + e;
+        float x[8];
+        Vec8<T>::load(a, x);
+        rotate8<T>(x, e, p.rdims, ct, st);
+        Vec8<T>::store(a, x);
+      }
+    }
+    ss = block_sum<256>(ss, sm);
+    const float rs = 1.f / sqrtf(ss / (float)p.rank + p.eps);
+    if (8 * i < p.rank) {
+      float n[8];
+      Vec8<float>::load(p.norm + 8 * i, n);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] *= rs * n[k];
+      Vec8<T>::store(dst + 8 * i, v);
+      if (dst2 != nullptr) Vec8<T>::store(dst2 + 8 * i, v);
+    }
+    for (int j = p.rank / 8 + threadIdx.x; j < nc; j += 256) {
+      Vec8<T>::load(c + 8 * j, v);
+      rotate8<T>(v, 8 * j - p.rank, p.rdims, ct, st);
+      Vec8<T>::store(dst + 8 * j, v);
+      if (dst2 != nullptr) Vec8<T>::store(dst2 + 8 * j, v);
+    }
+    return;
+  }
+  const int ncb = (p.rank + kAbsCols - 1) / kAbsCols;
+  int w = blockIdx.x - p.n_tok;
+  const int h = w % p.H;
+  w /= p.H;
+  const int cb = w % ncb, a0 = (w / ncb) * kAbsTok;
+  const int na = min(kAbsTok, p.n_abs - a0);
+  float* sq = sm;                         // [kAbsTok][dim]
+  float* red = sm + kAbsTok * p.dim;      // [4 waves][kAbsTok][kAbsCols]
+  for (int i = threadIdx.x; i < kAbsTok * p.dim; i += 256) {
+    const int a = i / p.dim, d = i - a * p.dim;
+    float v = 0.f;
+    if (a < na) {
+      const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
+      v = to_f(p.qd[(int64_t)t * p.ld + (int64_t)h * qh + d]);
+    }
+    sq[i] = v;
+  }
+  if (cb == 0) {
+    const int nr = p.rot / 8;
+    for (int i = threadIdx.x; i < na * nr; i += 256) {
+      const int a = i / nr, e = 8 * (i - a * nr);
+      const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
+      const int pos = min(p.tok_pos[t], p.n_pos - 1);
+      float x[8];
+      Vec8<T>::load(p.qd + (int64_t)t * p.ld + (int64_t)h * qh + p.dim + e, x);
+      rotate8<T>(x, e, p.rdims, p.cos_t + (int64_t)pos * half, p.sin_t + (int64_t)pos * half);
+      Vec8<T>::store(p.qa + ((int64_t)(a0 + a) * p.H + h) * row_w + p.rank + e, x);
+    }
+  }
+  // 16 lanes cover the columns, the other 16 lane groups of the workgroup take every 16th row of W_uk[h]
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int col = cb * kAbsCols + 8 * (lane & 15), dg = wid * 4 + (lane >> 4);
+  const bool col_ok = col < p.rank;
+  const T* uk = p.uk + (int64_t)h * p.dim * p.rank + (col_ok ? col : 0);
+  float acc[kAbsTok][8];
+#pragma unroll
+  for (int a = 0; a < kAbsTok; ++a)
+#pragma unroll
+    for (int k = 0; k < 8; ++k) acc[a][k] = 0.f;
+  __syncthreads();
+  for (int d0 = dg; d0 < p.dim; d0 += 128) {
+    float u[8][8];
+#pragma unroll
+    for (int b = 0; b < 8; ++b)
+      if (d0 + 16 * b < p.dim) Vec8<T>::load(uk + (int64_t)(d0 + 16 * b) * p.rank, u[b]);
+#pragma unroll
+    for (int b = 0; b < 8; ++b) {
+      const int d = d0 + 16 * b;
+      if (d >= p.dim) break;
+#pragma unroll
+      for (int a = 0; a < kAbsTok; ++a) {
+        const float q = sq[a * p.dim + d];
+#pragma unroll
+        for (int k = 0; k < 8; ++k) acc[a][k] += q * u[b][k];
+      }
+    }
+  }
+#pragma unroll
+  for (int a = 0; a < kAbsTok; ++a)
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      float v = acc[a][k];
+      v += __shfl_xor(v, 16, 64);
+      v += __shfl_xor(v, 32, 64);
+      if (lane < 16) red[(wid * kAbsTok + a) * kAbsCols + 8 * lane + k] = v;
+    }
+  __syncthreads();
+  for (int i = threadIdx.x; i < na * kAbsCols; i += 256) {
+    const int a = i / kAbsCols, cc = i - a * kAbsCols;
+    if (cb * kAbsCols + cc >= p.rank) continue;
+    float v = 0.f;
+#pragma unroll
+    for (int x = 0; x < 4; ++x) v += red[(x * kAbsTok + a) * kAbsCols + cc];
+    p.qa[((int64_t)(a0 + a) * p.H + h) * row_w + cb * kAbsCols + cc] = from_f<T>(v);
+  }
+}
+
+// any sizes; workgroups [0, n_tok): one token each, then ceil(n_abs / kAbsTok) x H: absorption
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(PrepParams<T> p) {
   extern __shared__ float sm[];
@@ -150,6 +296,13 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(T* __restrict__ cache,
   const int p = pos[i];
   T* c = cache + ((int64_t)tables[(int64_t)seq[i] * max_blocks + p / block_size] * block_size + p % block_size) * W;
   T* r = rows + (int64_t)(dst_row != nullptr ? dst_row[i] : i) * ld;
+  constexpr int V = 16 / sizeof(T);
+  if (W % V == 0 && ((uintptr_t)rows | (uintptr_t)(ld * sizeof(T))) % 16 == 0) {
+    const u32x4* src = reinterpret_cast<const u32x4*>(TO_CACHE ? r : c);
+    u32x4* dst = reinterpret_cast<u32x4*>(TO_CACHE ? c : r);
+    for (int k = lane; k < W / V; k += 64) dst[k] = src[k];
+    return;
+  }
   for (int k = lane; k < W; k += 64) {
     if (TO_CACHE) c[k] = r[k]; else r[k] = c[k];
   }
@@ -238,59 +391,75 @@ __global__ __launch_bounds__(256) void latent_decode_plain_kernel(DecodeParams<T
   }
 }
 
-// bf16, rank and rot multiples of 8: 16 heads of one absorbed row on the matrix cores, 64 keys a tile. The key tile is
-// one LDS image read by rows for the scores (A = keys, B = q: the accumulator column is the head) and transposed for
-// the weighted sum (A = weights, B = latent columns). NB: 16-column blocks of the latent per wave.
+// bf16, rank and rot multiples of 8: 16 HG heads of one absorbed row on the matrix cores, 64 keys a tile. The key tile
+// is one LDS image read by rows for the scores (A = keys, B = q: the accumulator column is the head) and transposed for
+// the weighted sum (A = weights, B = latent columns). Four waves per group of 16 heads: each takes 16 keys of the
+// scores, then every fourth 16-column block of the latent (NB of them at most). A thread stages NCH 16-byte chunks of
+// one key row and requests the next tile's before it computes on this one.
 constexpr int kTK = 64;
 
-template <int NB>
-__global__ __launch_bounds__(256) void latent_decode_mfma_kernel(DecodeParams<bf16> p) {
+template <int HG, int NCH, int NB>
+__global__ __launch_bounds__(256 * HG) void latent_decode_mfma_kernel(DecodeParams<bf16> p) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
+  constexpr int NT = 256 * HG, TPR = 4 * HG;    // threads; of them on one key row
   const int row_w = p.rank + p.rot;
   const int kd = (row_w + 31) & ~31;            // contraction length, zero padded
   const int ldk = kd + 8;                       // LDS row stride (elements)
   bf16* sk = reinterpret_cast<bf16*>(lds);      // [kTK][ldk]
-  bf16* sq = sk + kTK * ldk;                    // [16][ldk]
-  bf16* sp = sq + 16 * ldk;                     // [16][kTK + 8]
-  float* smax = reinterpret_cast<float*>(sp + 16 * (kTK + 8));  // [4][16]
-  float* ssum = smax + 64;                      // [4][16]
-  const int split = blockIdx.x, h0 = blockIdx.y * 16, a = blockIdx.z;
+  bf16* sq = sk + kTK * ldk;                    // [16 HG][ldk]
+  const int lane = threadIdx.x & 63, hg = threadIdx.x >> 8, w = (threadIdx.x >> 6) & 3;
+  bf16* sp = sq + 16 * HG * ldk + hg * 16 * (kTK + 8);  // [HG][16][kTK + 8]
+  float* smax = reinterpret_cast<float*>(sq + 16 * HG * ldk + HG * 16 * (kTK + 8)) + hg * 128;  // [HG][4][16]
+  float* ssum = smax + 64;                              // [HG][4][16]
+  const int split = blockIdx.x, hb = blockIdx.y * 16 * HG, a = blockIdx.z;
+  const int h0 = hb + 16 * hg;
   const int t = p.atok != nullptr ? p.atok[a] : a;
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int l15 = lane & 15, g = lane >> 4;
   int j0, j1;
   key_range(p, t, split, j0, j1);
   const int* table = p.tables + (int64_t)p.tok_seq[t] * p.max_blocks;
   const int nch = row_w / 8, nchp = kd / 8;
   const bf16x8 zero = {};
-  for (int i = threadIdx.x; i < 16 * nchp; i += 256) {
+  const int kr = threadIdx.x / TPR, kc = threadIdx.x % TPR;
+  bf16x8 pf[NCH];
+  auto fetch = [&](int jb) {
+    const int j = jb + kr;
+    const bool ok = j < j1;
+    const bf16* src = p.cache;
+    if (ok) src += ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * row_w;
+#pragma unroll
+    for (int k = 0; k < NCH; ++k) {
+      const int c = kc + TPR * k;
+      pf[k] = zero;
+      if (ok && c < nch) pf[k] = *reinterpret_cast<const bf16x8*>(src + 8 * c);
+    }
+  };
+  if (j0 < j1) fetch(j0);
+  for (int i = threadIdx.x; i < 16 * HG * nchp; i += NT) {
     const int r = i / nchp, c = i - r * nchp;
     bf16x8 v = zero;
-    if (h0 + r < p.H && c < nch)
-      v = *reinterpret_cast<const bf16x8*>(p.qa + ((int64_t)a * p.H + h0 + r) * row_w + 8 * c);
+    if (hb + r < p.H && c < nch)
+      v = *reinterpret_cast<const bf16x8*>(p.qa + ((int64_t)a * p.H + hb + r) * row_w + 8 * c);
     *reinterpret_cast<bf16x8*>(sq + r * ldk + 8 * c) = v;
   }
   f32x4 o[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b) o[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;  // of head l15 (replicated over the lane groups and waves)
+  float m = -INFINITY, l = 0.f;  // of head l15 (replicated over the lane groups and the head group's waves)
   const float c2 = p.scale * kLog2e;
   for (int jb = j0; jb < j1; jb += kTK) {
-    __syncthreads();  // the previous tile is read out (and q is staged)
-    for (int i = threadIdx.x; i < kTK * nchp; i += 256) {
-      const int r = i / nchp, c = i - r * nchp;
-      const int j = jb + r;
-      bf16x8 v = zero;
-      if (j < j1 && c < nch)
-        v = *reinterpret_cast<const bf16x8*>(
-            p.cache + ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * row_w + 8 * c);
-      *reinterpret_cast<bf16x8*>(sk + r * ldk + 8 * c) = v;
+    if (jb > j0) __syncthreads();  // the previous tile is read out
+#pragma unroll
+    for (int k = 0; k < NCH; ++k) {
+      const int c = kc + TPR * k;
+      if (c < nchp) *reinterpret_cast<bf16x8*>(sk + kr * ldk + 8 * c) = pf[k];
     }
     __syncthreads();
+    if (jb + kTK < j1) fetch(jb + kTK);
     f32x4 s = {0.f, 0.f, 0.f, 0.f};  // keys 16 w + 4 g + r of head l15
     const bf16* ka = sk + (16 * w + l15) * ldk + 8 * g;
-    const bf16* qb = sq + l15 * ldk + 8 * g;
-#pragma unroll 4
+    const bf16* qb = sq + (16 * hg + l15) * ldk + 8 * g;
+#pragma unroll 6
     for (int k = 0; k < kd; k += 32)
       s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ka + k),
                                                   *reinterpret_cast<const bf16x8*>(qb + k), s, 0, 0, 0);
@@ -366,75 +535,96 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(DecodeParams<bf
   }
 }
 
-// merges the splits of one (absorbed row, head) and applies W_uv[h]
-template <typename T>
+// Merges the splits of TG absorbed rows of one head and applies kUvRows rows of W_uv[h] to them (grid: heads, row groups,
+// slices of W_uv[h]; every slice merges for itself).
+constexpr int kUvRows = 32;
+
+template <typename T, int TG>
 __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml,
                                                              const T* __restrict__ uv, const int* __restrict__ atok,
-                                                             T* __restrict__ out, int64_t ldo, int H, int rank, int vd,
-                                                             int splits) {
-  extern __shared__ float so[];  // [rank]
-  __shared__ float sa[64];
-  const int h = blockIdx.x, a = blockIdx.y;
+                                                             T* __restrict__ out, int64_t ldo, int n_abs, int H,
+                                                             int rank, int vd, int splits) {
+  extern __shared__ float so[];  // [TG][rank]
+  __shared__ float sa[TG][64];
+  const int h = blockIdx.x, a0 = blockIdx.y * TG;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
-  const int64_t pi = ((int64_t)a * H + h) * splits;
-  if (w == 0) {
+  for (int x = w; x < TG; x += 4) {
+    const int64_t pi = ((int64_t)min(a0 + x, n_abs - 1) * H + h) * splits;
     const float m = lane < splits ? part_ml[2 * (pi + lane)] : -INFINITY;
     const float l = lane < splits ? part_ml[2 * (pi + lane) + 1] : 0.f;
     const float mm = wave_max(m);
     const float e = m == -INFINITY ? 0.f : __expf(m - mm);
     const float tot = wave_sum(l * e);
-    sa[lane] = tot > 0.f ? e / tot : 0.f;
+    sa[x][lane] = tot > 0.f ? e / tot : 0.f;
   }
   __syncthreads();
-  for (int i = threadIdx.x; i < rank; i += 256) {
-    float o = 0.f;
-    const float* po = part_o + pi * rank + i;
-    int s = 0;
-    for (; s + 8 <= splits; s += 8) {
-      float v[8];
 #pragma unroll
-      for (int k = 0; k < 8; ++k) v[k] = po[(int64_t)(s + k) * rank];
+  for (int x = 0; x < TG; ++x) {
+    const float* pb = part_o + ((int64_t)min(a0 + x, n_abs - 1) * H + h) * splits * rank;
+    for (int i = threadIdx.x; i < rank; i += 256) {
+      float o = 0.f;
+      const float* po = pb + i;
+      for (int s = 0; s < splits; s += 16) {
+        float v[16];
 #pragma unroll
-      for (int k = 0; k < 8; ++k) o += sa[s + k] != 0.f ? v[k] * sa[s + k] : 0.f;
-    }
-    for (; s < splits; ++s) o += sa[s] != 0.f ? po[(int64_t)s * rank] * sa[s] : 0.f;
-    so[i] = o;
-  }
-  __syncthreads();
-  const int64_t t = atok != nullptr ? atok[a] : a;
-  const T* u = uv + (int64_t)h * vd * rank;
-  const bool vec = rank % 8 == 0;
-  for (int r0 = w * 4; r0 < vd; r0 += 16) {  // a wave takes 4 value rows at a time
-    float acc[4] = {0.f, 0.f, 0.f, 0.f};
-    if (vec) {
-      for (int i = lane * 8; i < rank; i += 512) {
-        float x[8];
+        for (int k = 0; k < 16; ++k) v[k] = s + k < splits ? po[(int64_t)(s + k) * rank] : 0.f;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = so[i + e];
-#pragma unroll
-        for (int k = 0; k < 4; ++k) {
-          float y[8];
-          Vec8<T>::load(u + (int64_t)min(r0 + k, vd - 1) * rank + i, y);
-#pragma unroll
-          for (int e = 0; e < 8; ++e) acc[k] += x[e] * y[e];
-        }
+        for (int k = 0; k < 16; ++k) o += s + k < splits ? v[k] * sa[x][s + k] : 0.f;
       }
-    } else {
-      for (int i = lane; i < rank; i += 64)
-#pragma unroll
-        for (int k = 0; k < 4; ++k) acc[k] += so[i] * to_f(u[(int64_t)min(r0 + k, vd - 1) * rank + i]);
+      so[x * rank + i] = o;
     }
+  }
+  __syncthreads();
+  const T* u = uv + (int64_t)h * vd * rank;
+  const int r0 = blockIdx.z * kUvRows + w * 8;  // a wave takes 8 value rows
+  if (r0 >= vd) return;
+  float acc[8][TG];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const float v = wave_sum(acc[k]);
-      if (lane == 0 && r0 + k < vd) out[t * ldo + (int64_t)h * vd + r0 + k] = from_f<T>(v);
+  for (int k = 0; k < 8; ++k)
+#pragma unroll
+    for (int x = 0; x < TG; ++x) acc[k][x] = 0.f;
+  if (rank % 8 == 0) {
+    for (int i = lane * 8; i < rank; i += 512) {
+      float y[8][8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) Vec8<T>::load(u + (int64_t)min(r0 + k, vd - 1) * rank + i, y[k]);
+#pragma unroll
+      for (int x = 0; x < TG; ++x) {
+        float z[8];
+        Vec8<float>::load(so + x * rank + i, z);
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) acc[k][x] += z[e] * y[k][e];
+      }
+    }
+  } else {
+    for (int i = lane; i < rank; i += 64)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const float y = to_f(u[(int64_t)min(r0 + k, vd - 1) * rank + i]);
+#pragma unroll
+        for (int x = 0; x < TG; ++x) acc[k][x] += so[x * rank + i] * y;
+      }
+  }
+#pragma unroll
+  for (int x = 0; x < TG; ++x) {
+    float mine = 0.f;  // lane k keeps row r0 + k
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const float v = wave_sum(acc[k][x]);
+      mine = lane == k ? v : mine;
+    }
+    if (a0 + x < n_abs && lane < 8 && r0 + lane < vd) {
+      const int64_t t = atok != nullptr ? atok[a0 + x] : a0 + x;
+      out[t * ldo + (int64_t)h * vd + r0 + lane] = from_f<T>(mine);
     }
   }
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// expanded form: flash attention over gathered keys, 128 query rows of one (sequence, head) a workgroup
+// expanded form: flash attention over gathered keys, 32 query rows of one (sequence, head) a wave
 // ---------------------------------------------------------------------------------------------------------------
 struct PrefillParams {
   const bf16* q;       // [tokens, ld]: head h at column h * dk, rotated
@@ -453,8 +643,10 @@ struct PrefillParams {
 constexpr int BN = 64;
 
 // DK / DV: LDS and register room; the runtime dk, vd (multiples of 16) may be smaller
-template <int DK, int DV>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
+// NW waves of 32 query rows; FULL: dk == DK and vd == DV
+template <int DK, int DV, int NW, bool FULL>
+__global__ __launch_bounds__(64 * NW) void latent_prefill_kernel(PrefillParams p) {
+  constexpr int RB = 32 * NW;
   constexpr int KS = DK / 16, DT = DV / 32;
   constexpr int TK = Dim<DK>::TILE, TV = Dim<DV>::TILE;
   extern __shared__ __attribute__((aligned(1024))) char smem[];  // K[2], V[2]
@@ -463,7 +655,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
   const int* md = p.meta + 4 * blockIdx.z;
   const int q0 = md[0], n_new = md[1], ws0 = md[2], past = md[3];
   // the last row blocks see the most keys: they start first
-  const int row_start = ((int)gridDim.x - 1 - (int)blockIdx.x) * 128;
+  const int row_start = ((int)gridDim.x - 1 - (int)blockIdx.x) * RB;
   if (row_start >= n_new) return;
   const int head = blockIdx.y;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, h = lane >> 5;
@@ -478,10 +670,10 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       qf[ks] = bf16x8{};
-      if (16 * ks < p.dk) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 16 * ks);
+      if (FULL || 16 * ks < p.dk) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 16 * ks);
     }
   }
-  const int last_row = min(row_start + 128, n_new) - 1;
+  const int last_row = min(row_start + RB, n_new) - 1;
   const int ctx = past + last_row + 1;
   const int kt_end = (ctx + BN - 1) / BN;
   int kt_begin = 0;
@@ -493,15 +685,15 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
   const bf16* vbase = p.kv + (int64_t)p.H * p.dim + (int64_t)head * p.vd;
   auto stage = [&](int kt, int buf) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int n = w * 4 + i;
+    for (int i = 0; i < 16 / NW; ++i) {
+      const int n = w * (16 / NW) + i;
       const int row = 4 * n + (lane >> 4);
       const int key = min(kt * BN + row, ctx - 1);
       const int64_t kr = ws0 + key;
 #pragma unroll
       for (int cc = 0; cc < Dim<DK>::NT; ++cc) {
         const int ch = 16 * cc + ((lane & 15) ^ swz(row));
-        if (8 * ch < p.dk) {
+        if (FULL ? 8 * ch < DK : 8 * ch < p.dk) {
           const bf16* src = 8 * ch < p.dim ? kbase + kr * p.ldkv + 8 * ch : p.kr + kr * p.ldr + (8 * ch - p.dim);
           __builtin_amdgcn_global_load_lds((gbl_void*)src, (lds_void*)(sK + buf * TK + cc * 16384 + n * 1024), 16, 0, 0);
         }
@@ -509,7 +701,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
 #pragma unroll
       for (int cc = 0; cc < Dim<DV>::NT; ++cc) {
         const int ch = 16 * cc + ((lane & 15) ^ swz(row));
-        if (8 * ch < p.vd)
+        if (FULL ? 8 * ch < DV : 8 * ch < p.vd)
           __builtin_amdgcn_global_load_lds((gbl_void*)(vbase + kr * p.ldkv + 8 * ch),
                                            (lds_void*)(sV + buf * TV + cc * 16384 + n * 1024), 16, 0, 0);
       }
@@ -540,7 +732,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
         s[t] = f32x16{};
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks)
-          if (16 * ks < p.dk) s[t] = mfma(rows_d(Kt, 32 * t, ks), qf[ks], s[t]);
+          if (FULL || 16 * ks < p.dk) s[t] = mfma(rows_d(Kt, 32 * t, ks), qf[ks], s[t]);
       }
       float tmax = -INFINITY;
 #pragma unroll
@@ -578,7 +770,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
       const bf16x8 pb[4] = {acc_to_b<0>(s[0]), acc_to_b<1>(s[0]), acc_to_b<0>(s[1]), acc_to_b<1>(s[1])};
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt)
-        if (32 * dt < p.vd) {
+        if (FULL || 32 * dt < p.vd) {
 #pragma unroll
           for (int st = 0; st < 4; ++st) o[dt] = mfma(tr_d(Vt, st, dt), pb[st], o[dt]);
         }
@@ -590,7 +782,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
     bf16* op = p.out + (int64_t)(q0 + tok) * p.ldo + (int64_t)head * p.vd;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      if (32 * dt + 32 <= p.vd) {
+      if (FULL || 32 * dt + 32 <= p.vd) {
         store_row_block<DV>(op, o[dt], dt, h, inv);
       } else if (32 * dt < p.vd) {  // vd = 32 k + 16: the first half of the block
 #pragma unroll
@@ -605,30 +797,49 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(PrefillParams p) {
   }
 }
 
-template <int DK, int DV>
-int launch_prefill(const PrefillParams& p, int n_pre, int max_new, hipStream_t st) {
+template <int DK, int DV, int NW, bool FULL>
+int launch_prefill_as(const PrefillParams& p, int n_pre, int max_new, hipStream_t st) {
   constexpr int bytes = 2 * (Dim<DK>::TILE + Dim<DV>::TILE);
   static_assert(bytes <= 160 * 1024, "LDS");
-  static const hipError_t attr = hipFuncSetAttribute((const void*)latent_prefill_kernel<DK, DV>,
+  static const hipError_t attr = hipFuncSetAttribute((const void*)latent_prefill_kernel<DK, DV, NW, FULL>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
   if (attr != hipSuccess) return attr;
-  hipLaunchKernelGGL((latent_prefill_kernel<DK, DV>), dim3((max_new + 127) / 128, p.H, n_pre), dim3(256), bytes, st, p);
+  hipLaunchKernelGGL((latent_prefill_kernel<DK, DV, NW, FULL>), dim3((max_new + 32 * NW - 1) / (32 * NW), p.H, n_pre),
+                     dim3(64 * NW), bytes, st, p);
   return hipGetLastError();
 }
 
-size_t decode_lds(int rank, int rot) {
-  const int kd = (rank + rot + 31) & ~31;
-  return (size_t)(kTK + 16) * (kd + 8) * 2 + 16 * (kTK + 8) * 2 + 128 * 4;
+template <int DK, int DV>
+int launch_prefill(const PrefillParams& p, int n_pre, int max_new, hipStream_t st) {
+  if constexpr (DK <= 192) {  // registers for two waves per SIMD
+    if (max_new > 128) {
+      if (p.dk == DK && p.vd == DV) return launch_prefill_as<DK, DV, 8, true>(p, n_pre, max_new, st);
+      return launch_prefill_as<DK, DV, 8, false>(p, n_pre, max_new, st);
+    }
+  }
+  return launch_prefill_as<DK, DV, 4, false>(p, n_pre, max_new, st);
 }
 
-template <int NB>
+size_t decode_lds(int rank, int rot, int hg) {
+  const int kd = (rank + rot + 31) & ~31;
+  return (size_t)(kTK + 16 * hg) * (kd + 8) * 2 + hg * (16 * (kTK + 8) * 2 + 128 * 4);
+}
+
+template <int HG, int NCH, int NB>
 int launch_decode(const DecodeParams<bf16>& p, int n_abs, hipStream_t st) {
-  const size_t lds = decode_lds(p.rank, p.rot);
-  static const hipError_t attr = hipFuncSetAttribute((const void*)latent_decode_mfma_kernel<NB>,
+  const size_t lds = decode_lds(p.rank, p.rot, HG);
+  static const hipError_t attr = hipFuncSetAttribute((const void*)latent_decode_mfma_kernel<HG, NCH, NB>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
   if (attr != hipSuccess) return attr;
-  hipLaunchKernelGGL(latent_decode_mfma_kernel<NB>, dim3(p.splits, (p.H + 15) / 16, n_abs), dim3(256), lds, st, p);
+  hipLaunchKernelGGL((latent_decode_mfma_kernel<HG, NCH, NB>),
+                     dim3(p.splits, (p.H + 16 * HG - 1) / (16 * HG), n_abs), dim3(256 * HG), lds, st, p);
   return hipGetLastError();
+}
+
+// heads of one workgroup / 16
+int decode_hg(int H, int rank, int rot) {
+  const int kd = (rank + rot + 31) & ~31;
+  return H > 16 && kd <= 640 && rank <= 512 ? 2 : 1;
 }
 
 }  // namespace
@@ -642,15 +853,21 @@ HDS_EXPORT int hds_latent_prep(int dtype, void* qd, int64_t ld, const float* nor
   if (H < 1 || dim < 0 || rot < 0 || rdims < 0 || rdims > rot || rdims % 2 || rank < 1 || n_pos < 1 || n_abs < 0 ||
       n_abs > n_tok || block_size < 1 || ld < (int64_t)H * (dim + rot) + rank + rot || (n_abs > 0 && (!qa || !uk)))
     return hipErrorInvalidValue;
-  const int64_t grid = n_tok + (int64_t)((n_abs + kAbsTok - 1) / kAbsTok) * H;
-  const size_t lds = sizeof(float) * (kAbsTok * dim > 16 ? kAbsTok * dim : 16);
+  const bool v8 = dim % 8 == 0 && rot % 8 == 0 && rdims % 8 == 0 && rank % 8 == 0 && rank <= 2048 && ld % 8 == 0 &&
+                  (uintptr_t)qd % 16 == 0 && (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0;
+  const int64_t cblocks = v8 ? (rank + kAbsCols - 1) / kAbsCols : 1;
+  const int64_t grid = n_tok + (int64_t)((n_abs + kAbsTok - 1) / kAbsTok) * H * cblocks;
+  const size_t lds = sizeof(float) * (kAbsTok * dim + 16 + (v8 ? 4 * kAbsTok * kAbsCols : 0));
   if (grid > 0x7fffffff || lds > 64 * 1024) return hipErrorInvalidValue;
 #define HDS_LP(TT)                                                                                                   \
   {                                                                                                                  \
     PrepParams<TT> p{(TT*)qd, ld, norm, cos_t, sin_t, (TT*)cache, tok_seq, tok_pos, tables, ws_row, (TT*)ws,       \
                      (const TT*)uk, atok, (TT*)qa, n_tok, n_abs, n_pos, max_blocks, block_size, H, dim, rot, rdims, \
                      rank, eps};                                                                                     \
-    hipLaunchKernelGGL(latent_prep_kernel<TT>, dim3((unsigned)grid), dim3(256), lds, st, p);                         \
+    if (v8)                                                                                                          \
+      hipLaunchKernelGGL(latent_prep8_kernel<TT>, dim3((unsigned)grid), dim3(256), lds, st, p);                      \
+    else                                                                                                             \
+      hipLaunchKernelGGL(latent_prep_kernel<TT>, dim3((unsigned)grid), dim3(256), lds, st, p);                       \
   }
   if (dtype == kBF16) HDS_LP(bf16) else if (dtype == kF32) HDS_LP(float) else return hipErrorInvalidValue;
 #undef HDS_LP
@@ -677,14 +894,16 @@ HDS_EXPORT int hds_latent_rows(int dtype, int to_cache, void* cache, void* rows,
 }
 
 HDS_EXPORT int hds_latent_decode_mfma_ok(int rank, int rot) {
-  return rank % 8 == 0 && rot % 8 == 0 && rank >= 8 && rank <= 1024 && decode_lds(rank, rot) <= 160 * 1024;
+  return rank % 8 == 0 && rot % 8 == 0 && rank >= 8 && rank + rot <= 960;
 }
 
-// key splits of one absorbed row: enough workgroups for the chip, >= 32 keys each, <= 64 (one wave merges them)
-HDS_EXPORT int hds_latent_decode_splits(int n_abs, int head_groups, int max_keys) {
-  const int64_t groups = (int64_t)n_abs * head_groups;
-  int64_t s = (512 + groups - 1) / groups;
-  const int by_len = (max_keys + 31) / 32;
+// key splits of one absorbed row: about one workgroup per CU, >= 128 keys each (the partial sums of a split are as
+// large as 128 cached rows of a wide latent), <= 64 (one wave merges them)
+HDS_EXPORT int hds_latent_decode_splits(int n_abs, int H, int rank, int rot, int mfma, int max_keys) {
+  const int per = mfma ? 16 * decode_hg(H, rank, rot) : 1;
+  const int64_t groups = (int64_t)n_abs * ((H + per - 1) / per);
+  int64_t s = (256 + groups - 1) / groups;
+  const int by_len = (max_keys + 127) / 128;
   s = s < by_len ? s : by_len;
   return s < 1 ? 1 : (s > 64 ? 64 : (int)s);
 }
@@ -701,11 +920,12 @@ HDS_EXPORT int hds_latent_decode(int dtype, const void* qa, const void* cache, f
     if (dtype != kBF16 || !hds_latent_decode_mfma_ok(rank, rot)) return hipErrorInvalidValue;
     DecodeParams<bf16> p{(const bf16*)qa, (const bf16*)cache, part_o, part_ml, atok, tok_seq, tok_pos, tables,
                          max_blocks, block_size, H, rank, rot, splits, window, scale};
-    if (rank <= 64) return launch_decode<1>(p, n_abs, st);
-    if (rank <= 128) return launch_decode<2>(p, n_abs, st);
-    if (rank <= 256) return launch_decode<4>(p, n_abs, st);
-    if (rank <= 512) return launch_decode<8>(p, n_abs, st);
-    return launch_decode<16>(p, n_abs, st);
+    const int kd = (rank + rot + 31) & ~31;
+    const bool two = decode_hg(H, rank, rot) == 2;
+    if (kd <= 128) return two ? launch_decode<2, 2, 2>(p, n_abs, st) : launch_decode<1, 4, 2>(p, n_abs, st);
+    if (kd <= 320 && rank <= 256) return two ? launch_decode<2, 5, 4>(p, n_abs, st) : launch_decode<1, 10, 4>(p, n_abs, st);
+    if (kd <= 640 && rank <= 512) return two ? launch_decode<2, 10, 8>(p, n_abs, st) : launch_decode<1, 20, 8>(p, n_abs, st);
+    return launch_decode<1, 30, 15>(p, n_abs, st);
   }
   const size_t lds = sizeof(float) * (size_t)(2 * rank + rot + kGenKeys);
   if (lds > 64 * 1024) return hipErrorInvalidValue;
@@ -725,15 +945,19 @@ HDS_EXPORT int hds_latent_combine(int dtype, const float* part_o, const float* p
                                   int splits, hipStream_t st) {
   if (n_abs <= 0) return 0;
   if (splits < 1 || splits > 64 || vd < 1 || n_abs > 65535 || rank > 8192) return hipErrorInvalidValue;
-  const dim3 grid(H, n_abs);
-  if (dtype == kBF16)
-    hipLaunchKernelGGL(latent_combine_kernel<bf16>, grid, dim3(256), rank * sizeof(float), st, part_o, part_ml,
-                       (const bf16*)uv, atok, (bf16*)out, ldo, H, rank, vd, splits);
-  else if (dtype == kF32)
-    hipLaunchKernelGGL(latent_combine_kernel<float>, grid, dim3(256), rank * sizeof(float), st, part_o, part_ml,
-                       (const float*)uv, atok, (float*)out, ldo, H, rank, vd, splits);
-  else
+#define HDS_LC(TT, TG)                                                                                               \
+  hipLaunchKernelGGL((latent_combine_kernel<TT, TG>), dim3(H, (n_abs + TG - 1) / TG, (vd + kUvRows - 1) / kUvRows), \
+                     dim3(256), TG * rank * sizeof(float), st, part_o, part_ml, (const TT*)uv, atok, (TT*)out, ldo, \
+                     n_abs, H, rank, vd, splits)
+  const bool four = n_abs >= 4 && rank <= 2048;
+  if (dtype == kBF16) {
+    if (four) HDS_LC(bf16, 4); else HDS_LC(bf16, 1);
+  } else if (dtype == kF32) {
+    if (four) HDS_LC(float, 4); else HDS_LC(float, 1);
+  } else {
     return hipErrorInvalidValue;
+  }
+#undef HDS_LC
   return hipGetLastError();
 }
 

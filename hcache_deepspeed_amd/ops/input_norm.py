@@ -9,14 +9,13 @@ import torch
 from . import native
 
 MAX_TAPS = 16
-_MAX_ROWS = 64
 
 
 def _rows_per_group(taps, max_new, n_tokens):
     if max_new == 1:
         return 1
-    r = 4 if n_tokens <= 2048 else 16
-    return max(r, taps - 1)
+    # rows plus history fill the workgroup's 8 waves once (short steps) or twice
+    return max((8 if n_tokens <= 2048 else 16) - (taps - 1), taps - 1, 1)
 
 
 def input_norm(x, delta, gains, convs, eps, taps, batch, state, offset, dtype, embed=None):

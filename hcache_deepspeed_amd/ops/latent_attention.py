@@ -150,7 +150,7 @@ def latent_attention(qd, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, pla
         mfma = int(qd.dtype == torch.bfloat16 and bool(lib.hds_latent_decode_mfma_ok(sh.rank, sh.rot)))
         cap = mb * bs
         keys = min(cap, sh.window) if sh.window else cap
-        splits = lib.hds_latent_decode_splits(n_abs, -(-H // 16) if mfma else H, keys)
+        splits = lib.hds_latent_decode_splits(n_abs, H, sh.rank, sh.rot, mfma, keys)
         part_o = torch.empty(n_abs * H * splits * sh.rank, dtype=torch.float32, device=dev)
         part_ml = torch.empty(n_abs * H * splits * 2, dtype=torch.float32, device=dev)
         native.check(

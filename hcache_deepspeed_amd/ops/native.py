@@ -35,7 +35,7 @@ _KERNEL_SIGS = {
     "hds_latent_prep": "i" + "pl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
     "hds_latent_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
     "hds_latent_decode_mfma_ok": "ii",
-    "hds_latent_decode_splits": "iii",
+    "hds_latent_decode_splits": "iiiiii",
     "hds_latent_decode": "i" + "p" * 8 + "i" * 8 + "f" + "i" + "s",
     "hds_latent_combine": "i" + "ppppp" + "l" + "iiiii" + "s",
     "hds_latent_prefill_ok": "iiii",
