@@ -7,7 +7,7 @@
 // a sequence whose `seen` is 0 starts from zero whatever the slot holds.
 //
 // Short steps (decode, small portions) run one thread per channel over the new tokens. Prompts are cut into chunks of
-// kChunk tokens: pass 1 reduces every chunk to S_out = A S_in + B, pass 2 walks the chunks of a sequence and leaves
+// kChunk tokens: pass 1 reduces every chunk to S_out = A S_in + B, pass 2 composes the chunks of a sequence and leaves
 // each chunk's S_in (and the sequence's new state), pass 3 replays the chunks from it. No workgroup waits for another.
 #include "hds_common.h"
 
@@ -15,11 +15,20 @@ namespace {
 using namespace hds;
 
 constexpr int kChunk = 32;
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 
 template <typename T, int V>
 __device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
   if constexpr (V == 1) {
     v[0] = to_f(*p);
+  } else if constexpr (V == 2 && sizeof(T) == 2) {
+    const bf16x2 r = *reinterpret_cast<const bf16x2*>(p);
+    v[0] = (float)r[0];
+    v[1] = (float)r[1];
+  } else if constexpr (V == 2) {
+    const float2 r = *reinterpret_cast<const float2*>(p);
+    v[0] = r.x;
+    v[1] = r.y;
   } else if constexpr (sizeof(T) == 2) {
     const bf16x4 r = *reinterpret_cast<const bf16x4*>(p);
 #pragma unroll
@@ -34,6 +43,10 @@ template <typename T, int V>
 __device__ __forceinline__ void stv(T* p, const float (&v)[V]) {
   if constexpr (V == 1) {
     *p = from_f<T>(v[0]);
+  } else if constexpr (V == 2 && sizeof(T) == 2) {
+    *reinterpret_cast<bf16x2*>(p) = bf16x2{(bf16)v[0], (bf16)v[1]};
+  } else if constexpr (V == 2) {
+    *reinterpret_cast<float2*>(p) = make_float2(v[0], v[1]);
   } else if constexpr (sizeof(T) == 2) {
     bf16x4 r;
 #pragma unroll
@@ -74,7 +87,7 @@ struct ScanParams {
   int64_t slot_stride;
   const int* slots;
   const int* seq_meta;
-  float* ws;         // [S, chunks, 2, W]
+  float* ws;         // [S, W / V, chunks, 2 V]: A then B (after pass 2: the chunk's S_in) of V channels
   int W, chunks;
 };
 
@@ -92,14 +105,14 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanParams<T> p) {
   ldv<float, V>(p.ba + c, ba);
   ldv<float, V>(p.bb + c, bb);
   float* st = p.state + (PASS == 0 ? (int64_t)p.slots[seq] * p.slot_stride + c : 0);
-  float* ws = PASS == 0 ? nullptr : p.ws + (((int64_t)seq * p.chunks + ch) * 2) * p.W + c;
+  float* ws = PASS == 0 ? nullptr : p.ws + (((int64_t)seq * (p.W / V) + c / V) * p.chunks + ch) * (2 * V);
 #pragma unroll
   for (int i = 0; i < V; ++i) {
     s[i] = 0.f;
     A[i] = 1.f;
   }
   if (PASS == 0 && seen > 0) ldv<float, V>(st, s);
-  if (PASS == 3) ldv<float, V>(ws + p.W, s);
+  if (PASS == 3) ldv<float, V>(ws + V, s);
   const T* in = p.in + (int64_t)(q0 + t0) * p.ld + c;
   T* out = p.out + (int64_t)(q0 + t0) * p.ldo + c;
   auto step = [&](const float (&a)[V], const float (&b)[V], const float (&g)[V], T* o) {
@@ -114,7 +127,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanParams<T> p) {
     }
     if (PASS != 1) stv<T, V>(o, y);
   };
-  constexpr int U = 4;
+  constexpr int U = 8;
   int t = t0;
   for (; t + U <= t1; t += U) {
     float a[U][V], b[U][V], g[U][V];
@@ -141,38 +154,54 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanParams<T> p) {
   if (PASS == 0) stv<float, V>(st, s);
   if (PASS == 1) {
     stv<float, V>(ws, A);
-    stv<float, V>(ws + p.W, s);
+    stv<float, V>(ws + V, s);
   }
 }
 
-// pass 2: ws[., 1] becomes the state a chunk starts from; the sequence's last state goes to its slot
-template <typename T>
+// pass 2: a wave per V channels of a sequence, a chunk per lane: prefix composition of the chunks' maps S -> A S + B by
+// shuffles, 64 chunks at a time; every chunk's S_in goes back to ws, the last state to the sequence's slot
+template <typename T, int V>
 __global__ __launch_bounds__(64) void scan_carry_kernel(ScanParams<T> p) {
-  const int c = blockIdx.x * 64 + threadIdx.x;
-  if (c >= p.W) return;
+  const int c = blockIdx.x * V, lane = threadIdx.x;
   const int seq = blockIdx.y;
   const int n = p.seq_meta[3 * seq + 1], seen = p.seq_meta[3 * seq + 2];
   if (n <= 0) return;
   const int nc = (n + kChunk - 1) / kChunk;
   float* st = p.state + (int64_t)p.slots[seq] * p.slot_stride + c;
-  float s = seen > 0 ? *st : 0.f;
-  float* ws = p.ws + (int64_t)seq * p.chunks * 2 * p.W + c;
-  constexpr int U = 32;
-  for (int k0 = 0; k0 < nc; k0 += U) {
-    float A[U], B[U];
+  float s[V];
 #pragma unroll
-    for (int k = 0; k < U; ++k) {
-      const int64_t o = (int64_t)(k0 + k) * 2 * p.W;
-      A[k] = k0 + k < nc ? ws[o] : 1.f;
-      B[k] = k0 + k < nc ? ws[o + p.W] : 0.f;
+  for (int i = 0; i < V; ++i) s[i] = 0.f;
+  if (seen > 0) ldv<float, V>(st, s);
+  float* ws = p.ws + ((int64_t)seq * (p.W / V) + blockIdx.x) * p.chunks * (2 * V);
+  for (int k0 = 0; k0 < nc; k0 += 64) {
+    const int k = k0 + lane;
+    float A[V], B[V], in[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      A[i] = 1.f;
+      B[i] = 0.f;
+    }
+    if (k < nc) {
+      ldv<float, V>(ws + (int64_t)k * 2 * V, A);
+      ldv<float, V>(ws + (int64_t)k * 2 * V + V, B);
     }
 #pragma unroll
-    for (int k = 0; k < U; ++k) {
-      if (k0 + k < nc) ws[(int64_t)(k0 + k) * 2 * p.W + p.W] = s;
-      s = A[k] * s + B[k];
+    for (int i = 0; i < V; ++i) {
+#pragma unroll
+      for (int d = 1; d < 64; d <<= 1) {
+        const float pa = __shfl_up(A[i], d, 64), pb = __shfl_up(B[i], d, 64);
+        if (lane >= d) {
+          B[i] = A[i] * pb + B[i];
+          A[i] *= pa;
+        }
+      }
+      const float ea = __shfl_up(A[i], 1, 64), eb = __shfl_up(B[i], 1, 64);
+      in[i] = lane == 0 ? s[i] : ea * s[i] + eb;
+      s[i] = __shfl(A[i], 63, 64) * s[i] + __shfl(B[i], 63, 64);
     }
+    if (k < nc) stv<float, V>(ws + (int64_t)k * 2 * V + V, in);
   }
-  *st = s;
+  if (lane == 0) stv<float, V>(st, s);
 }
 
 template <typename T, int V>
@@ -184,7 +213,7 @@ int launch_scan(const ScanParams<T>& p, int n_seqs, int max_new, hipStream_t st)
   }
   const dim3 grid(cb, (max_new + kChunk - 1) / kChunk, n_seqs);
   hipLaunchKernelGGL((scan_kernel<T, V, 1>), grid, dim3(64), 0, st, p);
-  hipLaunchKernelGGL((scan_carry_kernel<T>), dim3((p.W + 63) / 64, n_seqs), dim3(64), 0, st, p);
+  hipLaunchKernelGGL((scan_carry_kernel<T, V>), dim3(p.W / V, n_seqs), dim3(64), 0, st, p);
   hipLaunchKernelGGL((scan_kernel<T, V, 3>), grid, dim3(64), 0, st, p);
   return hipGetLastError();
 }
@@ -193,7 +222,7 @@ template <typename T>
 int scan(const ScanParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
   if (p.W % 4 == 0 && p.ld % 4 == 0 && p.ldo % 4 == 0 && p.slot_stride % 4 == 0 && (uintptr_t)p.in % 16 == 0 &&
       (uintptr_t)p.out % 16 == 0 && (uintptr_t)p.state % 16 == 0)
-    return launch_scan<T, 4>(p, n_seqs, max_new, st);
+    return p.ws == nullptr ? launch_scan<T, 4>(p, n_seqs, max_new, st) : launch_scan<T, 2>(p, n_seqs, max_new, st);
   return launch_scan<T, 1>(p, n_seqs, max_new, st);
 }
 

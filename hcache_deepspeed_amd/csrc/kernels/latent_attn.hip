@@ -68,8 +68,9 @@ constexpr int kAbsTok = 4;    // absorbed tokens that share one read of W_uk[h]
 constexpr int kAbsCols = 128; // latent columns of an absorption workgroup (vector path)
 
 // Vector path (all part sizes multiples of 8, rank <= 2048). Workgroups [0, n_tok): one token each (norm, rotation,
-// scatter, q of expanded tokens rotated in place); then one per (head, kAbsCols columns, kAbsTok absorbed tokens).
-template <typename T>
+// scatter, q of expanded tokens rotated in place); then one per (head, kAbsCols columns, TG absorbed tokens).
+// TG: absorbed tokens a workgroup takes; 0: none in the batch.
+template <typename T, int TG>
 __global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
   extern __shared__ float sm[];
   const int qh = p.dim + p.rot, row_w = p.rank + p.rot;
@@ -123,80 +124,85 @@ __global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
     }
     return;
   }
-  const int ncb = (p.rank + kAbsCols - 1) / kAbsCols;
-  int w = blockIdx.x - p.n_tok;
-  const int h = w % p.H;
-  w /= p.H;
-  const int cb = w % ncb, a0 = (w / ncb) * kAbsTok;
-  const int na = min(kAbsTok, p.n_abs - a0);
-  float* sq = sm;                         // [kAbsTok][dim]
-  float* red = sm + kAbsTok * p.dim;      // [4 waves][kAbsTok][kAbsCols]
-  for (int i = threadIdx.x; i < kAbsTok * p.dim; i += 256) {
-    const int a = i / p.dim, d = i - a * p.dim;
-    float v = 0.f;
-    if (a < na) {
-      const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
-      v = to_f(p.qd[(int64_t)t * p.ld + (int64_t)h * qh + d]);
-    }
-    sq[i] = v;
-  }
-  if (cb == 0) {
-    const int nr = p.rot / 8;
-    for (int i = threadIdx.x; i < na * nr; i += 256) {
-      const int a = i / nr, e = 8 * (i - a * nr);
-      const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
-      const int pos = min(p.tok_pos[t], p.n_pos - 1);
-      float x[8];
-      Vec8<T>::load(p.qd + (int64_t)t * p.ld + (int64_t)h * qh + p.dim + e, x);
-      rotate8<T>(x, e, p.rdims, p.cos_t + (int64_t)pos * half, p.sin_t + (int64_t)pos * half);
-      Vec8<T>::store(p.qa + ((int64_t)(a0 + a) * p.H + h) * row_w + p.rank + e, x);
-    }
-  }
-  // 16 lanes cover the columns, the other 16 lane groups of the workgroup take every 16th row of W_uk[h]
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  const int col = cb * kAbsCols + 8 * (lane & 15), dg = wid * 4 + (lane >> 4);
-  const bool col_ok = col < p.rank;
-  const T* uk = p.uk + (int64_t)h * p.dim * p.rank + (col_ok ? col : 0);
-  float acc[kAbsTok][8];
-#pragma unroll
-  for (int a = 0; a < kAbsTok; ++a)
-#pragma unroll
-    for (int k = 0; k < 8; ++k) acc[a][k] = 0.f;
-  __syncthreads();
-  for (int d0 = dg; d0 < p.dim; d0 += 128) {
+  if constexpr (TG > 0) {
+    const int ncb = (p.rank + kAbsCols - 1) / kAbsCols;
+    int w = blockIdx.x - p.n_tok;
+    const int h = w % p.H;
+    w /= p.H;
+    const int cb = w % ncb, a0 = (w / ncb) * TG;
+    const int na = min(TG, p.n_abs - a0);
+    float* sq = sm;                    // [TG][dim]
+    float* red = sm + TG * p.dim;      // [4 waves][TG][kAbsCols]
+    // 16 lanes cover the columns, the 16 lane groups of the workgroup take every 16th row of W_uk[h]
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int col = cb * kAbsCols + 8 * (lane & 15), dg = wid * 4 + (lane >> 4);
+    const T* uk = p.uk + (int64_t)h * p.dim * p.rank + (col < p.rank ? col : 0);
     float u[8][8];
+    auto fetch = [&](int d0) {
 #pragma unroll
-    for (int b = 0; b < 8; ++b)
-      if (d0 + 16 * b < p.dim) Vec8<T>::load(uk + (int64_t)(d0 + 16 * b) * p.rank, u[b]);
-#pragma unroll
-    for (int b = 0; b < 8; ++b) {
-      const int d = d0 + 16 * b;
-      if (d >= p.dim) break;
-#pragma unroll
-      for (int a = 0; a < kAbsTok; ++a) {
-        const float q = sq[a * p.dim + d];
-#pragma unroll
-        for (int k = 0; k < 8; ++k) acc[a][k] += q * u[b][k];
+      for (int b = 0; b < 8; ++b)
+        if (d0 + 16 * b < p.dim) Vec8<T>::load(uk + (int64_t)(d0 + 16 * b) * p.rank, u[b]);
+    };
+    fetch(dg);
+    for (int i = threadIdx.x; i < TG * p.dim; i += 256) {
+      const int a = i / p.dim, d = i - a * p.dim;
+      float v = 0.f;
+      if (a < na) {
+        const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
+        v = to_f(p.qd[(int64_t)t * p.ld + (int64_t)h * qh + d]);
+      }
+      sq[i] = v;
+    }
+    if (cb == 0) {
+      const int nr = p.rot / 8;
+      for (int i = threadIdx.x; i < na * nr; i += 256) {
+        const int a = i / nr, e = 8 * (i - a * nr);
+        const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
+        const int pos = min(p.tok_pos[t], p.n_pos - 1);
+        float x[8];
+        Vec8<T>::load(p.qd + (int64_t)t * p.ld + (int64_t)h * qh + p.dim + e, x);
+        rotate8<T>(x, e, p.rdims, p.cos_t + (int64_t)pos * half, p.sin_t + (int64_t)pos * half);
+        Vec8<T>::store(p.qa + ((int64_t)(a0 + a) * p.H + h) * row_w + p.rank + e, x);
       }
     }
-  }
+    float acc[TG][8];
 #pragma unroll
-  for (int a = 0; a < kAbsTok; ++a)
+    for (int a = 0; a < TG; ++a)
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
-      float v = acc[a][k];
-      v += __shfl_xor(v, 16, 64);
-      v += __shfl_xor(v, 32, 64);
-      if (lane < 16) red[(wid * kAbsTok + a) * kAbsCols + 8 * lane + k] = v;
+      for (int k = 0; k < 8; ++k) acc[a][k] = 0.f;
+    __syncthreads();
+    for (int d0 = dg; d0 < p.dim; d0 += 128) {
+      if (d0 != dg) fetch(d0);
+#pragma unroll
+      for (int b = 0; b < 8; ++b) {
+        const int d = d0 + 16 * b;
+        if (d >= p.dim) break;
+#pragma unroll
+        for (int a = 0; a < TG; ++a) {
+          const float q = sq[a * p.dim + d];
+#pragma unroll
+          for (int k = 0; k < 8; ++k) acc[a][k] += q * u[b][k];
+        }
+      }
     }
-  __syncthreads();
-  for (int i = threadIdx.x; i < na * kAbsCols; i += 256) {
-    const int a = i / kAbsCols, cc = i - a * kAbsCols;
-    if (cb * kAbsCols + cc >= p.rank) continue;
-    float v = 0.f;
 #pragma unroll
-    for (int x = 0; x < 4; ++x) v += red[(x * kAbsTok + a) * kAbsCols + cc];
-    p.qa[((int64_t)(a0 + a) * p.H + h) * row_w + cb * kAbsCols + cc] = from_f<T>(v);
+    for (int a = 0; a < TG; ++a)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        float v = acc[a][k];
+        v += __shfl_xor(v, 16, 64);
+        v += __shfl_xor(v, 32, 64);
+        if (lane < 16) red[(wid * TG + a) * kAbsCols + 8 * lane + k] = v;
+      }
+    __syncthreads();
+    for (int i = threadIdx.x; i < na * kAbsCols; i += 256) {
+      const int a = i / kAbsCols, cc = i - a * kAbsCols;
+      if (cb * kAbsCols + cc >= p.rank) continue;
+      float v = 0.f;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) v += red[(x * TG + a) * kAbsCols + cc];
+      p.qa[((int64_t)(a0 + a) * p.H + h) * row_w + cb * kAbsCols + cc] = from_f<T>(v);
+    }
   }
 }
 
@@ -559,20 +565,30 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __rest
     sa[x][lane] = tot > 0.f ? e / tot : 0.f;
   }
   __syncthreads();
-#pragma unroll
-  for (int x = 0; x < TG; ++x) {
-    const float* pb = part_o + ((int64_t)min(a0 + x, n_abs - 1) * H + h) * splits * rank;
-    for (int i = threadIdx.x; i < rank; i += 256) {
-      float o = 0.f;
-      const float* po = pb + i;
+  if (rank % 4 == 0) {
+    const int rq = rank / 4;
+    for (int j = threadIdx.x; j < TG * rq; j += 256) {
+      const int x = j / rq, i = 4 * (j - x * rq);
+      const float* po = part_o + ((int64_t)min(a0 + x, n_abs - 1) * H + h) * splits * rank + i;
+      f32x4 o = {0.f, 0.f, 0.f, 0.f};
       for (int s = 0; s < splits; s += 16) {
-        float v[16];
+        f32x4 v[16];
 #pragma unroll
-        for (int k = 0; k < 16; ++k) v[k] = s + k < splits ? po[(int64_t)(s + k) * rank] : 0.f;
+        for (int k = 0; k < 16; ++k)
+          if (s + k < splits) v[k] = *reinterpret_cast<const f32x4*>(po + (int64_t)(s + k) * rank);
 #pragma unroll
-        for (int k = 0; k < 16; ++k) o += s + k < splits ? v[k] * sa[x][s + k] : 0.f;
+        for (int k = 0; k < 16; ++k)
+          if (s + k < splits) o += v[k] * sa[x][s + k];
       }
-      so[x * rank + i] = o;
+      *reinterpret_cast<f32x4*>(so + x * rank + i) = o;
+    }
+  } else {
+    for (int j = threadIdx.x; j < TG * rank; j += 256) {
+      const int x = j / rank, i = j - x * rank;
+      const float* po = part_o + ((int64_t)min(a0 + x, n_abs - 1) * H + h) * splits * rank + i;
+      float o = 0.f;
+      for (int s = 0; s < splits; ++s) o += po[(int64_t)s * rank] * sa[x][s];
+      so[j] = o;
     }
   }
   __syncthreads();
@@ -856,7 +872,8 @@ HDS_EXPORT int hds_latent_prep(int dtype, void* qd, int64_t ld, const float* nor
   const bool v8 = dim % 8 == 0 && rot % 8 == 0 && rdims % 8 == 0 && rank % 8 == 0 && rank <= 2048 && ld % 8 == 0 &&
                   (uintptr_t)qd % 16 == 0 && (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0;
   const int64_t cblocks = v8 ? (rank + kAbsCols - 1) / kAbsCols : 1;
-  const int64_t grid = n_tok + (int64_t)((n_abs + kAbsTok - 1) / kAbsTok) * H * cblocks;
+  const int tg = v8 && n_abs == 1 ? 1 : kAbsTok;
+  const int64_t grid = n_tok + (int64_t)((n_abs + tg - 1) / tg) * H * cblocks;
   const size_t lds = sizeof(float) * (kAbsTok * dim + 16 + (v8 ? 4 * kAbsTok * kAbsCols : 0));
   if (grid > 0x7fffffff || lds > 64 * 1024) return hipErrorInvalidValue;
 #define HDS_LP(TT)                                                                                                   \
@@ -864,8 +881,12 @@ HDS_EXPORT int hds_latent_prep(int dtype, void* qd, int64_t ld, const float* nor
     PrepParams<TT> p{(TT*)qd, ld, norm, cos_t, sin_t, (TT*)cache, tok_seq, tok_pos, tables, ws_row, (TT*)ws,       \
                      (const TT*)uk, atok, (TT*)qa, n_tok, n_abs, n_pos, max_blocks, block_size, H, dim, rot, rdims, \
                      rank, eps};                                                                                     \
-    if (v8)                                                                                                          \
-      hipLaunchKernelGGL(latent_prep8_kernel<TT>, dim3((unsigned)grid), dim3(256), lds, st, p);                      \
+    if (v8 && n_abs == 0)                                                                                            \
+      hipLaunchKernelGGL((latent_prep8_kernel<TT, 0>), dim3((unsigned)grid), dim3(256), 64, st, p);                  \
+    else if (v8 && n_abs == 1)                                                                                       \
+      hipLaunchKernelGGL((latent_prep8_kernel<TT, 1>), dim3((unsigned)grid), dim3(256), lds, st, p);                 \
+    else if (v8)                                                                                                     \
+      hipLaunchKernelGGL((latent_prep8_kernel<TT, kAbsTok>), dim3((unsigned)grid), dim3(256), lds, st, p);           \
     else                                                                                                             \
       hipLaunchKernelGGL(latent_prep_kernel<TT>, dim3((unsigned)grid), dim3(256), lds, st, p);                       \
   }
