@@ -5,8 +5,6 @@ import torch
 
 from . import native
 
-_CHUNKED_FROM = 64  # longest portion one thread per channel walks alone
-
 
 def gated_scan(proj, bias_z, bias_x, out, batch, state, offset):
     """proj: [T, 3 W] (update gate | candidate | output gate); out: [T, W] view with unit column stride;
@@ -14,16 +12,12 @@ def gated_scan(proj, bias_z, bias_x, out, batch, state, offset):
     W = out.shape[1]
     if native.use_native(proj):
         assert proj.stride(1) == 1 and out.stride(1) == 1 and out.dtype == proj.dtype
-        lib = native.kernels()
-        ws = None
-        if batch.max_new > _CHUNKED_FROM:
-            chunks = -(-batch.max_new // lib.hds_gated_scan_chunk())
-            ws = torch.empty(batch.current_sequences * chunks * 2 * W, dtype=torch.float32, device=proj.device)
         native.check(
-            lib.hds_gated_scan(native.dt(proj), proj.data_ptr(), proj.stride(0), bias_z.data_ptr(), bias_x.data_ptr(),
-                               out.data_ptr(), out.stride(0), state.data_ptr() + 4 * offset, state.stride(0),
-                               batch.slots.data_ptr(), batch.seq_meta.data_ptr(), native.ptr(ws),
-                               batch.current_sequences, batch.max_new, W, native.stream()), "gated_scan")
+            native.kernels().hds_gated_scan(native.dt(proj), proj.data_ptr(), proj.stride(0), bias_z.data_ptr(),
+                                            bias_x.data_ptr(), out.data_ptr(), out.stride(0),
+                                            state.data_ptr() + 4 * offset, state.stride(0), batch.slots.data_ptr(),
+                                            batch.seq_meta.data_ptr(), batch.current_sequences, batch.max_new, W,
+                                            native.stream()), "gated_scan")
         return out
     a, b, g = proj.float().split(W, 1)
     a, b = a + bias_z, b + bias_x

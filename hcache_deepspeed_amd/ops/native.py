@@ -29,8 +29,7 @@ _KERNEL_SIGS = {
     "hds_glu_rows": "ii" + "plpl" + "li" + "s",
     "hds_input_norm": "i" + "ppppp" + "pipp" + "pipp" + "p" + "l" + "pp" + "iiiii" + "f" + "s",
     "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
-    "hds_gated_scan_chunk": "",
-    "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "ppp" + "iii" + "s",
+    "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "pp" + "iii" + "s",
     "hds_gemv_recur_bf16": "ppppp" + "pl" + "pp" + "iii" + "ll" + "s",
     "hds_latent_prep": "i" + "pl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
     "hds_latent_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
