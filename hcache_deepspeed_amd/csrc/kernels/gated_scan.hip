@@ -9,7 +9,7 @@
 // Short steps (decode, small portions) run one thread per V channels over the new tokens. Longer portions run a
 // workgroup per 16 channels: 64 thread groups take G consecutive tokens each, keep their gates in registers, compose
 // them to one map S -> A S + B, find the state they start from over the wave (shuffles) and the workgroup (LDS), and
-// write their outputs. Every value is read once and every gate evaluated once; the next 64 G tokens are requested before
+// write their outputs. Every value is read and every gate evaluated once; the next 64 G tokens are requested before
 // this step's are worked on.
 #include "hds_common.h"
 
@@ -114,11 +114,12 @@ __global__ __launch_bounds__(64) void scan_serial_kernel(ScanParams<T> p) {
   if (n > 0) stv<float, V>(st, s);
 }
 
-constexpr int kCols = 16, kGroups = 64;
+constexpr int kCols = 16, kThreads = 1024;  // channels and threads of a workgroup
 
+// one channel and G consecutive tokens a thread; row offsets of a sequence fit 32 bits
 template <typename T, int G>
-__global__ __launch_bounds__(kCols * kGroups) void scan_block_kernel(ScanParams<T> p) {
-  constexpr int NW = kCols * kGroups / 64, STEP = kGroups * G;
+__global__ __launch_bounds__(kThreads) void scan_block_kernel(ScanParams<T> p) {
+  constexpr int NW = kThreads / 64, STEP = kThreads / kCols * G;
   __shared__ float sA[2][NW][kCols], sB[2][NW][kCols];
   // neighbouring channel blocks share cache lines: keep them on one XCD (workgroups go round-robin over the 8)
   const int nb = gridDim.x, bx = nb % 8 == 0 ? (blockIdx.x & 7) * (nb / 8) + (blockIdx.x >> 3) : blockIdx.x;
@@ -132,26 +133,34 @@ __global__ __launch_bounds__(kCols * kGroups) void scan_block_kernel(ScanParams<
   float* st = p.state + (int64_t)p.slots[seq] * p.slot_stride + c;
   const float ba = p.ba[c], bb = p.bb[c];
   float s = seen > 0 ? *st : 0.f;  // the state before this step, the same in every thread of a channel
+  const T* in_a = p.in + (int64_t)q0 * p.ld;
+  const T* in_b = in_a + p.W;
+  const T* in_g = in_b + p.W;
+  T* out = p.out + (int64_t)q0 * p.ldo;
+  const uint32_t ld = (uint32_t)p.ld, ldo = (uint32_t)p.ldo;
   T ra[G], rb[G], rg[G];
   auto fetch = [&](int t0) {
+    const int t = t0 + grp * G;
+    const bool full = t0 + STEP <= n;
+    uint32_t o = (uint32_t)t * ld + c;
 #pragma unroll
     for (int k = 0; k < G; ++k) {
-      const int t = min(t0 + grp * G + k, n - 1);
-      const T* in = p.in + (int64_t)(q0 + t) * p.ld + c;
-      ra[k] = in[0];
-      rb[k] = in[p.W];
-      rg[k] = in[2 * p.W];
+      if (!full) o = (uint32_t)min(t + k, n - 1) * ld + c;
+      ra[k] = in_a[o];
+      rb[k] = in_b[o];
+      rg[k] = in_g[o];
+      o += ld;
     }
   };
   fetch(0);
   for (int t0 = 0, it = 0; t0 < n; t0 += STEP, ++it) {
-    const int tb = t0 + grp * G;
+    const int left = n - (t0 + grp * G);  // tokens this thread has
     float keep[G], add[G], og[G];
     float A = 1.f, B = 0.f;
 #pragma unroll
     for (int k = 0; k < G; ++k) {
       gates(to_f(ra[k]) + ba, to_f(rb[k]) + bb, to_f(rg[k]), keep[k], add[k], og[k]);
-      if (tb + k >= n) {
+      if (k >= left) {
         keep[k] = 1.f;
         add[k] = 0.f;
       }
@@ -180,16 +189,18 @@ __global__ __launch_bounds__(kCols * kGroups) void scan_block_kernel(ScanParams<
     }
     __syncthreads();  // one barrier a step: the other buffer is written next
     float sw = s;
-#pragma unroll
+#pragma unroll 4
     for (int i = 0; i < NW; ++i) {
       if (i == w) sw = s;
       s = sA[buf][i][cl] * s + sB[buf][i][cl];
     }
     float cur = ea * sw + eb;
+    uint32_t o = (uint32_t)(t0 + grp * G) * ldo + c;
 #pragma unroll
     for (int k = 0; k < G; ++k) {
       cur = keep[k] * cur + add[k];
-      if (ok && tb + k < n) p.out[(int64_t)(q0 + tb + k) * p.ldo + c] = from_f<T>(cur * og[k]);
+      if (ok && k < left) out[o] = from_f<T>(cur * og[k]);
+      o += ldo;
     }
   }
   if (ok && grp == 0) *st = s;
@@ -197,12 +208,14 @@ __global__ __launch_bounds__(kCols * kGroups) void scan_block_kernel(ScanParams<
 
 template <typename T>
 int scan(const ScanParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
-  if (max_new > 32) {
+  // (steps whose rows span 2^31 bytes and more: one thread per channel, 64-bit offsets)
+  const int64_t span = (int64_t)max_new * (p.ld > p.ldo ? p.ld : p.ldo) * (int64_t)sizeof(T);
+  if (max_new > 32 && span < (int64_t)0x7fffffff) {
     const dim3 grid((p.W + kCols - 1) / kCols, n_seqs);
-    if (max_new <= 4 * kGroups)
-      hipLaunchKernelGGL((scan_block_kernel<T, 4>), grid, dim3(kCols * kGroups), 0, st, p);
+    if (max_new <= 1024)
+      hipLaunchKernelGGL((scan_block_kernel<T, 4>), grid, dim3(kThreads), 0, st, p);
     else
-      hipLaunchKernelGGL((scan_block_kernel<T, 8>), grid, dim3(kCols * kGroups), 0, st, p);
+      hipLaunchKernelGGL((scan_block_kernel<T, 8>), grid, dim3(kThreads), 0, st, p);
     return hipGetLastError();
   }
   if (p.W % 4 == 0 && p.ld % 4 == 0 && p.ldo % 4 == 0 && p.slot_stride % 4 == 0 && (uintptr_t)p.in % 16 == 0 &&
