@@ -27,6 +27,9 @@ OPS = {
     "cross_entropy": ("kernels", "hds_xent"),
     "paged_attention (ragged)": ("kernels", "hds_paged_attn"),
     "kv_rotary_scatter (HCache restore)": ("kernels", "hds_kv_rope_scatter"),
+    "latent_attention (ragged)": ("kernels", "hds_latent_decode"),
+    "gated_scan (minGRU)": ("kernels", "hds_gated_scan"),
+    "input_norm (norm + input convolution)": ("kernels", "hds_input_norm"),
     "moe_scatter / moe_gather": ("kernels", "hds_moe_dispatch"),
     "quantizer (int8/int4)": ("kernels", "hds_quant_int"),
     "fp_quantizer (fp8)": ("kernels", "hds_quant_fp8"),

@@ -200,6 +200,10 @@ class InferenceEngineV2:
             n = tokens.numel() if isinstance(tokens, torch.Tensor) else len(tokens)
             assert latents.shape[1] == n, "latents must cover exactly the tokens being restored"
             seq = sm.get_or_create_sequence(uid)
+            if self._states is not None and (seq.evicted_state is None or seq.seen_tokens
+                                             or seq.evicted_state[0] != n):
+                at = seq.evicted_state[0] if seq.evicted_state else "no"
+                raise RuntimeError(f"sequence {uid}: its recurrent state was saved at {at} tokens; restore exactly those")
             sm.maybe_allocate_kv(seq, n)
             seq.pre_forward(n)
             batch.insert_sequence(seq, tokens if isinstance(tokens, torch.Tensor) else torch.tensor(tokens),
@@ -209,13 +213,6 @@ class InferenceEngineV2:
         if not lat:
             return
         batch.finalize()
-        if self._states is not None:
-            for uid in restored:
-                seq = sm.get_sequence(uid)
-                st = seq.evicted_state
-                if st is None or seq.seen_tokens or st[0] != seq.in_flight_tokens:
-                    raise RuntimeError(f"sequence {uid}: its recurrent state was saved at "
-                                       f"{st[0] if st else 'no'} tokens; restore exactly those")
         self._model.restore_kv(batch, lat)  # per-sequence pinned pieces, copied straight to the device
         for uid in restored:
             seq = sm.get_sequence(uid)

@@ -1,17 +1,14 @@
-"""Trace replay: feed given token ids through a served model step by step and write the logits that are asked for.
+"""Trace replay: given token ids go through a served model, one ragged batch a step, and chosen logits go to files.
 
     bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N < steps.jsonl
 
-One JSON object a line on standard input is one step, i.e. one ragged batch through the engine's ``put``:
+Standard input holds a step per line, a JSON object that becomes one call of the engine's ``put``:
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 7, "entries": [{"id": "r1", "tokens": [11, 4], "want": [1]}, {"id": "r2", "tokens": [9]}], "end": ["r1"]}
 
-``entries``: requests with their next tokens and the places among them whose logits are wanted; ``end``: requests that
-are finished after the step (``flush``). A step with wanted places writes ``OUT/<step>.f32``: little-endian float32
-[wanted, vocab] in the order of the entries and of ``want``. Every step answers ``done <step>`` on standard output.
-
-The KV pool is made for ``--max-tokens`` tokens and the engine tracks at most ``--max-requests`` (4) requests, so pages
-and state slots are used again. Nothing is sampled."""
+``want`` are places among an entry's tokens; the logits there, as little-endian float32 rows in entry and ``want`` order,
+are written to ``OUT/<step>.f32``. Requests in ``end`` are flushed after the step. ``done <step>`` on standard output
+answers each step. ``--max-tokens`` and ``--max-requests`` size the KV pool and the state slots; nothing is sampled."""
 import argparse
 import json
 import os
@@ -61,8 +58,8 @@ def main(argv=None):
     ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
     ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16")
     ap.add_argument("--out", required=True, help="folder the logits are written to")
-    ap.add_argument("--max-tokens", type=int, required=True, help="most tokens live requests hold at any time")
-    ap.add_argument("--max-requests", type=int, default=4, help="most requests live at any time")
+    ap.add_argument("--max-tokens", type=int, required=True, help="size of the KV pool in tokens (rounded up to pages)")
+    ap.add_argument("--max-requests", type=int, default=4, help="state slots")
     args = ap.parse_args(argv)
     import torch
     if not torch.cuda.is_available():

@@ -35,8 +35,9 @@ class LatentShape:
         return self.heads * (self.dim + self.rot)
 
 
-# portions of at most this many tokens run absorbed
-ABSORB_MAX = 4
+# Portions of at most this many tokens run absorbed: each re-reads the visible rows, which costs less than expanding them
+# once (a product over the whole window) up to some twenty tokens
+ABSORB_MAX = 16
 
 
 @dataclass

@@ -536,7 +536,6 @@ def test_evict_and_restore(run, name):
     lat = torch.cat(lats, 1)
     with pytest.raises(RuntimeError):
         eng.restore_kv([1], [torch.tensor(s[:32])], [lat[:, :32]])
-    eng.state_manager.free_kv(eng.state_manager.get_sequence(1))
     eng.restore_kv([1], [torch.tensor(s[:33])], [lat])
     got = [eng.put([1], [torch.tensor(s[33 + i:34 + i])], capture_latents=False)[0].double().cpu() for i in range(7)]
     check_logits(torch.cat(got), oracle_logits(name, s)[33:], run[1])
@@ -670,6 +669,26 @@ def test_trace_replay(run, tmp_path):
     want = torch.stack([oracle_logits("mixed", b + [3])[70], oracle_logits("mixed", a)[30]])
     check_logits(read(2), want, run[1])
     check_logits(read(3), oracle_logits("mixed", a)[:1], run[1])
+
+
+def test_kernel_sources_of_the_model_class_are_complete():
+    """A library of HybridTransformer.KERNEL_SOURCES alone exports every entry point the class's ops call."""
+    import os
+    import re
+
+    from hcache_deepspeed_amd.inference.v2.hybrid import HybridTransformer
+    from hcache_deepspeed_amd.ops import build, gated_scan, gemv, input_norm, latent_attention
+    have = ""
+    for f in HybridTransformer.KERNEL_SOURCES:
+        with open(os.path.join(build.CSRC, "kernels", f)) as fh:
+            have += fh.read()
+    used = {"hds_glu_rows"}
+    for mod in (gated_scan, gemv, input_norm, latent_attention):
+        with open(mod.__file__) as fh:
+            used |= set(re.findall(r"\)?\.(hds_\w+)\(", fh.read()))
+    assert len(used) > 12
+    for name in used:
+        assert re.search(rf"HDS_EXPORT int {name}\(", have), name
 
 
 def test_checkpoint_folder_and_registry(tmp_path):
