@@ -238,7 +238,9 @@ def test_gated_mlp_rows(run, act, T, I):
 SHAPES = {"odd": (3, 5, 6, 4, 7, 9, 11), "plain-prefill": (2, 8, 8, 8, 24, 24, 19), "mfma": (5, 24, 8, 8, 40, 16, 21),
           "mfma-rot-rest": (17, 40, 24, 12, 72, 48, 64), "no-window": (2, 32, 16, 16, 96, 80, 0),
           "wide": (2, 128, 64, 64, 264, 128, 130), "widest": (1, 192, 64, 64, 520, 208, 70),
-          "window-1": (2, 16, 16, 16, 32, 32, 1)}
+          "window-1": (2, 16, 16, 16, 32, 32, 1), "18-heads": (18, 16, 16, 16, 200, 16, 40),
+          "20-heads": (20, 16, 8, 8, 400, 16, 50), "full-64": (2, 48, 16, 16, 64, 64, 100),
+          "full-128": (2, 64, 64, 64, 72, 128, 90)}
 
 
 def _attention_case(name):
@@ -300,6 +302,21 @@ def test_latent_attention(run, name, sizes):
     w = _attention_weights(sh, dtype)
     qds = [rnd(n, sh.q_width + sh.row, seed=40 + n).to(dtype).double() for n in (75, 2, 49)]
     got = _run_attention(sh, m, qds, w, sizes, dev, dtype)
+    for g, qd in zip(got, qds):
+        close(g, _oracle_attention(sh, m, qd, w), dtype, bf16=2e-2)
+
+
+@pytest.mark.parametrize("name", ["mfma", "no-window", "wide", "full-64", "full-128"])
+@pytest.mark.parametrize("sizes", [[1000], [190]])
+def test_latent_attention_long_prompts(run, name, sizes):
+    """Portions of several row blocks, with earlier keys before them."""
+    dev, dtype = run
+    if dev.type == "cpu":
+        pytest.skip("the CPU implementation has one form")
+    sh, m = _attention_case(name)
+    w = _attention_weights(sh, dtype)
+    qds = [rnd(n, sh.q_width + sh.row, seed=60 + n).to(dtype).double() for n in (330, 141)]
+    got = _run_attention(sh, m, qds, w, sizes, dev, dtype, block_size=64)
     for g, qd in zip(got, qds):
         close(g, _oracle_attention(sh, m, qd, w), dtype, bf16=2e-2)
 
