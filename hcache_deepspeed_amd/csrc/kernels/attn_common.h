@@ -241,6 +241,27 @@ __device__ __forceinline__ void stage_tile_d(char* tile, RowPtr row_ptr) {
   }
 }
 
+// stage_tile_d for rows of nch 16-byte chunks, nch known at run time and at most D / 8; the other chunks of the tile keep
+// what they hold
+template <int NW, int D, typename RowPtr>
+__device__ __forceinline__ void stage_tile_n(char* tile, RowPtr row_ptr, int nch) {
+  const int lane = threadIdx.x & 63;
+  const int w = threadIdx.x >> 6;
+#pragma unroll
+  for (int c = 0; c < Dim<D>::NT; ++c) {
+#pragma unroll
+    for (int i = 0; i < 16 / NW; ++i) {
+      const int n = w * (16 / NW) + i;
+      const int row = 4 * n + (lane >> 4);
+      const int ch = (lane & 15) ^ swz(row);
+      if (16 * c + ch < nch) {
+        const char* src = (const char*)(row_ptr(row) + 128 * c) + ch * 16;
+        __builtin_amdgcn_global_load_lds((gbl_void*)src, (lds_void*)(tile + c * 16384 + n * 1024), 16, 0, 0);
+      }
+    }
+  }
+}
+
 // Same as stage_tile_d, but staged by a GROUP of NWG waves: wi = this wave's index inside the group.
 template <int NWG, int D, typename RowPtr>
 __device__ __forceinline__ void stage_tile_dw(char* tile, RowPtr row_ptr, int wi) {
@@ -307,6 +328,19 @@ __device__ __forceinline__ void store_row_block(bf16* dst, const f32x16& acc, in
   }
 }
 
+// the same for a row of n columns known at run time (n % 8 == 0, dst 8-B aligned)
+__device__ __forceinline__ void store_row_block_n(bf16* dst, const f32x16& acc, int dt, int h, float mul, int n) {
+#pragma unroll
+  for (int g = 0; g < 4; ++g) {
+    const int col = 32 * dt + 8 * g + 4 * h;
+    if (col < n) {
+      bf16x4 v4;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v4[j] = (bf16)(acc[4 * g + j] * mul);
+      *reinterpret_cast<bf16x4*>(dst + col) = v4;
+    }
+  }
+}
 
 }  // namespace attn
 }  // namespace hds

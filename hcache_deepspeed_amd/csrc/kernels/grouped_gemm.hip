@@ -16,6 +16,9 @@
 //   * both operands are K-contiguous, staged by LDS-DMA (global_load_lds_dwordx4) into the XOR-swizzled
 //     64 x 256 B tiles of attn_common.h (conflict-free ds_read_b128 A/B fragments), double-buffered:
 //     the next K tile streams in while the current one feeds the MFMAs;
+//   * options (serving, hds_experts_gemm): X rows read through an index list instead of being permuted first; W = [gate;
+//     up] with the activation silu(gate) * up in the epilogue -- a wave then holds the accumulators of the same features
+//     of both halves; a tile list made elsewhere (experts.hip);
 //   * blockIdx.x walks N tiles fastest so the (consecutively dispatched, XCD-round-robin) blocks of one
 //     token tile share the X tile in L2 while W[e] streams.
 #include "attn_common.h"
@@ -50,7 +53,12 @@ __global__ __launch_bounds__(64) void gg_plan_kernel(const int* __restrict__ off
   if (lane == 0) *n_tiles = base < max_tiles ? base : max_tiles;
 }
 
-__global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
+__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
+
+// GATHER: row r of the sorted order is x[src[r]] (n_src rows of x). GLU: w holds 2N rows per expert, gate then up.
+template <bool GATHER, bool GLU>
+__global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, int64_t ldx,
+                                                 const int* __restrict__ src, int n_src, const bf16* __restrict__ w,
                                                  bf16* __restrict__ y, const int* __restrict__ offs,
                                                  const int* __restrict__ tile_e, const int* __restrict__ tile_m,
                                                  const int* __restrict__ n_tiles, int T, int N, int K, int ldy) {
@@ -60,20 +68,32 @@ __global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, con
   const int m0 = tile_m[t];
   const int row0 = min(max(offs[e], 0), T);
   const int rows = min(max(offs[e + 1], row0), T) - row0;  // >= 1: the plan only emits tiles of non-empty experts
-  const int n0 = blockIdx.x * BN;
+  const int n0 = blockIdx.x * (GLU ? BN / 2 : BN);
 
   __shared__ __attribute__((aligned(16))) char smem[2 * 65536];
+  __shared__ int s_src[GATHER ? BM : 1];
   // buffer b: W tile halves at [b*64K, +16K, ...], X tile halves at [b*64K + 32K, +16K]
-  const bf16* wb = w + (int64_t)e * N * K + (int64_t)n0 * K;
-  const bf16* xb = x + (int64_t)row0 * K;
+  const bf16* wb = w + (int64_t)e * (GLU ? 2 : 1) * N * K + (int64_t)n0 * K;
+  const int64_t whalf = (int64_t)(GLU ? N : 64) * K;  // second half of the W tile: the up rows, or the next 64 rows
+  const bf16* xb = x + (int64_t)row0 * ldx;
+  if constexpr (GATHER) {
+    for (int r = threadIdx.x; r < BM; r += 256)
+      s_src[r] = min(max(src[row0 + min(m0 + r, rows - 1)], 0), n_src - 1);
+    __syncthreads();
+  }
   auto wrow = [&](int half, int kt) {
-    return [=](int r) { return wb + (int64_t)(64 * half + r) * K + (int64_t)kt * BK; };
+    return [=](int r) { return wb + half * whalf + (int64_t)r * K + (int64_t)kt * BK; };
   };
   auto xrow = [&](int half, int kt) {
+    const int* sp = s_src;
     return [=](int r) {
-      int m = m0 + 64 * half + r;
-      m = m < rows ? m : rows - 1;
-      return xb + (int64_t)m * K + (int64_t)kt * BK;
+      if constexpr (GATHER) {
+        return x + (int64_t)sp[64 * half + r] * ldx + (int64_t)kt * BK;
+      } else {
+        int m = m0 + 64 * half + r;
+        m = m < rows ? m : rows - 1;
+        return xb + (int64_t)m * ldx + (int64_t)kt * BK;
+      }
     };
   };
   auto stage = [&](int buf, int kt) {
@@ -98,11 +118,13 @@ __global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, con
   for (int kt = 0; kt < KT; ++kt) {
     const int buf = kt & 1;
     if (kt + 1 < KT) stage(buf ^ 1, kt + 1);
-    const char* Wt = smem + buf * 65536 + wn * 16384;
+    // GLU: the wave's two row blocks are the same 32 features of the gate and of the up half
+    const char* Wt = smem + buf * 65536 + (GLU ? 0 : wn * 16384);
     const char* Xt = smem + buf * 65536 + 32768 + wm * 16384;
 #pragma unroll
     for (int ks = 0; ks < 8; ++ks) {
-      const bf16x8 a0 = read_rows(Wt, 0, ks), a1 = read_rows(Wt, 32, ks);
+      const bf16x8 a0 = read_rows(Wt, GLU ? 32 * wn : 0, ks);
+      const bf16x8 a1 = GLU ? read_rows(Wt + 16384, 32 * wn, ks) : read_rows(Wt, 32, ks);
       const bf16x8 b0 = read_rows(Xt, 0, ks), b1 = read_rows(Xt, 32, ks);
       acc[0][0] = mfma(a0, b0, acc[0][0]);
       acc[0][1] = mfma(a0, b1, acc[0][1]);
@@ -119,7 +141,17 @@ __global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, con
   for (int j = 0; j < 2; ++j) {
     const int m = m0 + 64 * wm + 32 * j + (lane & 31);
     if (m >= rows) continue;
-    bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + 64 * wn;
+    bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + (GLU ? 32 : 64) * wn;
+    if constexpr (GLU) {
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        bf16x4 v;
+#pragma unroll
+        for (int q = 0; q < 4; ++q) v[q] = (bf16)silu_mul(acc[0][j][4 * g + q], acc[1][j][4 * g + q]);
+        *reinterpret_cast<bf16x4*>(yr + acc_row(4 * g, h)) = v;
+      }
+      continue;
+    }
 #pragma unroll
     for (int i = 0; i < 2; ++i)
 #pragma unroll
@@ -167,8 +199,10 @@ __device__ __forceinline__ bf16x8 frag128(const char* lds, int row0, int ks) {
   return *reinterpret_cast<const bf16x8*>(lds + off128(row0 + (lane & 31), 2 * ks + (lane >> 5)));
 }
 
-__global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
-                                                     bf16* __restrict__ y, const int* __restrict__ offs,
+template <bool GATHER, bool GLU>
+__global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x, int64_t ldx,
+                                                     const int* __restrict__ src, int n_src,
+                                                     const bf16* __restrict__ w, bf16* __restrict__ y, const int* __restrict__ offs,
                                                      const int* __restrict__ tile_e, const int* __restrict__ tile_m,
                                                      const int* __restrict__ n_tiles, int T, int N, int K, int ldy,
                                                      int ntn) {
@@ -184,23 +218,36 @@ __global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x,
   const int gsz = min(GT, mt - grp * GT);
   const int t = grp * GT + rem % gsz;
   if (t >= *n_tiles) return;  // block-uniform exit before any barrier
-  const int n0 = (rem / gsz) * BN2;
+  const int n0 = (rem / gsz) * (GLU ? BN2 / 2 : BN2);
   const int e = tile_e[t];
   const int m0 = tile_m[t];
   const int row0 = min(max(offs[e], 0), T);
   const int rows = min(max(offs[e + 1], row0), T) - row0;
 
   __shared__ __attribute__((aligned(16))) char smem[2 * 65536];  // [buf][W 32 KB | X 32 KB]
-  const bf16* wb = w + (int64_t)e * N * K + (int64_t)n0 * K;
-  const bf16* xb = x + (int64_t)row0 * K;
+  __shared__ int s_src[GATHER ? BM2 : 1];
+  const bf16* wb = w + (int64_t)e * (GLU ? 2 : 1) * N * K + (int64_t)n0 * K;
+  const bf16* xb = x + (int64_t)row0 * ldx;
+  if constexpr (GATHER) {
+    if (threadIdx.x < BM2)
+      s_src[threadIdx.x] = min(max(src[row0 + min(m0 + (int)threadIdx.x, rows - 1)], 0), n_src - 1);
+    __syncthreads();
+  }
   auto stage = [&](int buf, int kt) {
     char* s = smem + buf * 65536;
     const int64_t k0 = (int64_t)kt * BK2;
-    stage128<8, 256>(s, [=](int rr) { return wb + (int64_t)rr * K + k0; });
+    const int* sp = s_src;
+    // GLU: tile rows 0-127 are gate features, 128-255 the same features of the up half
+    const int64_t up = GLU ? (int64_t)(N - 128) * K : 0;
+    stage128<8, 256>(s, [=](int rr) { return wb + (int64_t)rr * K + k0 + (GLU && rr >= 128 ? up : 0); });
     stage128<8, 256>(s + 32768, [=](int rr) {
-      int m = m0 + rr;
-      m = m < rows ? m : rows - 1;
-      return xb + (int64_t)m * K + k0;
+      if constexpr (GATHER) {
+        return x + (int64_t)sp[rr] * ldx + k0;
+      } else {
+        int m = m0 + rr;
+        m = m < rows ? m : rows - 1;
+        return xb + (int64_t)m * ldx + k0;
+      }
     });
   };
 
@@ -218,13 +265,13 @@ __global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x,
   for (int kt = 0; kt < KT; ++kt) {
     const int buf = kt & 1;
     if (kt + 1 < KT) stage(buf ^ 1, kt + 1);
-    const char* Wt = smem + buf * 65536 + wn * 128 * 128;
+    const char* Wt = smem + buf * 65536 + wn * (GLU ? 64 : 128) * 128;
     const char* Xt = smem + buf * 65536 + 32768 + wm * 64 * 128;
 #pragma unroll
     for (int ks = 0; ks < 4; ++ks) {
       bf16x8 a[4], b[2];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) a[i] = frag128(Wt, 32 * i, ks);
+      for (int i = 0; i < 4; ++i) a[i] = frag128(Wt, GLU ? 32 * (i & 1) + 128 * (i >> 1) : 32 * i, ks);
 #pragma unroll
       for (int j = 0; j < 2; ++j) b[j] = frag128(Xt, 32 * j, ks);
 #pragma unroll
@@ -241,7 +288,19 @@ __global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x,
   for (int j = 0; j < 2; ++j) {
     const int m = m0 + 64 * wm + 32 * j + (lane & 31);
     if (m >= rows) continue;
-    bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + 128 * wn;
+    bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + (GLU ? 64 : 128) * wn;
+    if constexpr (GLU) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          bf16x4 v;
+#pragma unroll
+          for (int q = 0; q < 4; ++q) v[q] = (bf16)silu_mul(acc[i][j][4 * g + q], acc[i + 2][j][4 * g + q]);
+          *reinterpret_cast<bf16x4*>(yr + 32 * i + acc_row(4 * g, h)) = v;
+        }
+      continue;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -276,12 +335,43 @@ HDS_EXPORT int hds_grouped_gemm(const void* x, const void* w, void* y, const int
     const int max_tiles = (T + BM2 - 1) / BM2 + E;  // <= cap
     const int ntn = N / BN2;
     hipLaunchKernelGGL(gg_plan_kernel<BM2>, dim3(1), dim3(64), 0, st, offs, E, T, tile_e, tile_m, n_tiles, max_tiles);
-    hipLaunchKernelGGL(gg_big_kernel, dim3(ntn * max_tiles), dim3(512), 0, st, (const bf16*)x, (const bf16*)w,
-                       (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, ntn);
+    hipLaunchKernelGGL((gg_big_kernel<false, false>), dim3(ntn * max_tiles), dim3(512), 0, st, (const bf16*)x, K,
+                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, ntn);
   } else {
     hipLaunchKernelGGL(gg_plan_kernel<BM>, dim3(1), dim3(64), 0, st, offs, E, T, tile_e, tile_m, n_tiles, cap);
-    hipLaunchKernelGGL(gg_kernel, dim3(N / BN, cap), dim3(256), 0, st, (const bf16*)x, (const bf16*)w, (bf16*)y,
-                       offs, tile_e, tile_m, n_tiles, T, N, K, ldy);
+    hipLaunchKernelGGL((gg_kernel<false, false>), dim3(N / BN, cap), dim3(256), 0, st, (const bf16*)x, K,
+                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy);
   }
+  return hipGetLastError();
+}
+
+// Rows of a tile for T rows over E experts and N columns (what hds_experts_gemm wants its tile list to be made for)
+HDS_EXPORT int hds_experts_gemm_tile(int T, int N, int E) { return N % BN2 == 0 && T >= BM2 * E ? BM2 : BM; }
+
+// Grouped product of sorted rows with a ready tile list (tm = 128 or 256 rows, see hds_experts_gemm_tile; at most
+// max_tiles entries, the number on the device). src: row of x [n_src, ldx] for every sorted row, or null: x is sorted.
+// glu: w [E, 2N, K] is gate rows then up rows and y = silu(gate) * up. T: upper bound of the rows. K % 128 == 0; N a
+// multiple of the tile's columns (128, 256; half of that with glu).
+HDS_EXPORT int hds_experts_gemm(const void* x, int64_t ldx, const int* src, int n_src, const void* w, void* y, int ldy,
+                                const int* offs, const int* tile_e, const int* tile_m, const int* n_tiles,
+                                int max_tiles, int tm, int T, int N, int K, int E, int glu, hipStream_t st) {
+  if (T <= 0 || E <= 0) return 0;
+  const int cols = (tm == BM2 ? BN2 : BN) / (glu ? 2 : 1);
+  if ((tm != BM && tm != BM2) || N % cols || K % BK || ldx < K || ldx % 8 || ldy < N || ldy % 8 || max_tiles < 1 ||
+      max_tiles > 65535 || (src != nullptr && n_src < 1))
+    return hipErrorInvalidValue;
+#define HDS_EG(GA, GL)                                                                                               \
+  if (tm == BM2)                                                                                                     \
+    hipLaunchKernelGGL((gg_big_kernel<GA, GL>), dim3(N / cols * max_tiles), dim3(512), 0, st, (const bf16*)x, ldx,  \
+                       src, n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, N / cols); \
+  else                                                                                                               \
+    hipLaunchKernelGGL((gg_kernel<GA, GL>), dim3(N / cols, max_tiles), dim3(256), 0, st, (const bf16*)x, ldx, src,  \
+                       n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy)
+  if (src != nullptr) {
+    if (glu) { HDS_EG(true, true); } else { HDS_EG(true, false); }
+  } else {
+    if (glu) { HDS_EG(false, true); } else { HDS_EG(false, false); }
+  }
+#undef HDS_EG
   return hipGetLastError();
 }

@@ -82,6 +82,40 @@ template <> struct Vec8<float> {
   }
 };
 
+// V consecutive elements as floats
+template <typename T, int V> struct VecN;
+template <typename T> struct VecN<T, 1> {
+  __device__ __forceinline__ static void load(const T* p, float (&v)[1]) { v[0] = to_f(*p); }
+  __device__ __forceinline__ static void store(T* p, const float (&v)[1]) { *p = from_f<T>(v[0]); }
+};
+template <> struct VecN<float, 4> {
+  __device__ __forceinline__ static void load(const float* p, float (&v)[4]) {
+    const f32x4 r = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = r[i];
+  }
+  __device__ __forceinline__ static void store(float* p, const float (&v)[4]) {
+    *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+  }
+};
+template <> struct VecN<bf16, 4> {
+  __device__ __forceinline__ static void load(const bf16* p, float (&v)[4]) {
+    const bf16x4 r = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = (float)r[i];
+  }
+  __device__ __forceinline__ static void store(bf16* p, const float (&v)[4]) {
+    bf16x4 r;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) r[i] = (bf16)v[i];
+    *reinterpret_cast<bf16x4*>(p) = r;
+  }
+};
+template <typename T> struct VecN<T, 8> {
+  __device__ __forceinline__ static void load(const T* p, float (&v)[8]) { Vec8<T>::load(p, v); }
+  __device__ __forceinline__ static void store(T* p, const float (&v)[8]) { Vec8<T>::store(p, v); }
+};
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o >= 1; o >>= 1) v += __shfl_xor(v, o, 64);

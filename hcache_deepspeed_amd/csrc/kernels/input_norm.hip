@@ -18,35 +18,6 @@
 namespace {
 using namespace hds;
 
-template <typename T, int V> struct VecN;
-template <typename T> struct VecN<T, 1> {
-  __device__ __forceinline__ static void load(const T* p, float (&v)[1]) { v[0] = to_f(*p); }
-  __device__ __forceinline__ static void store(T* p, const float (&v)[1]) { *p = from_f<T>(v[0]); }
-};
-template <> struct VecN<float, 4> {
-  __device__ __forceinline__ static void load(const float* p, float (&v)[4]) {
-    const f32x4 r = *reinterpret_cast<const f32x4*>(p);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = r[i];
-  }
-  __device__ __forceinline__ static void store(float* p, const float (&v)[4]) {
-    *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
-  }
-};
-template <> struct VecN<bf16, 4> {
-  __device__ __forceinline__ static void load(const bf16* p, float (&v)[4]) {
-    const bf16x4 r = *reinterpret_cast<const bf16x4*>(p);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = (float)r[i];
-  }
-  __device__ __forceinline__ static void store(bf16* p, const float (&v)[4]) {
-    bf16x4 r;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) r[i] = (bf16)v[i];
-    *reinterpret_cast<bf16x4*>(p) = r;
-  }
-};
-
 constexpr int kU = 4;         // loads in flight per lane and operand
 constexpr int kMaxRows = 64;  // rows a workgroup holds statistics of: R + 2 (taps - 1) at most
 
@@ -310,32 +281,6 @@ __global__ __launch_bounds__(1024) void input_norm_step_kernel(InputNormParams<T
   }
 }
 
-// y[i] = g * norm(x[idx[i]] + delta[idx[i]]): the output norm of the rows whose logits are asked for
-template <typename T, int V>
-__global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ x, const T* __restrict__ delta,
-                                                        const int* __restrict__ idx, const float* __restrict__ g,
-                                                        int gs, T* __restrict__ y, int W, float eps) {
-  __shared__ float red[4];
-  const int64_t row = idx[blockIdx.x];
-  float ss = 0.f;
-  for (int c = threadIdx.x * V; c < W; c += 256 * V) {
-    float v[V], d[V];
-    VecN<float, V>::load(x + row * W + c, v);
-    VecN<T, V>::load(delta + row * W + c, d);
-#pragma unroll
-    for (int i = 0; i < V; ++i) ss += (v[i] + d[i]) * (v[i] + d[i]);
-  }
-  const float rs = 1.f / sqrtf(block_sum<256>(ss, red) / (float)W + eps);
-  for (int c = threadIdx.x * V; c < W; c += 256 * V) {
-    float v[V], d[V];
-    VecN<float, V>::load(x + row * W + c, v);
-    VecN<T, V>::load(delta + row * W + c, d);
-#pragma unroll
-    for (int i = 0; i < V; ++i) v[i] = (v[i] + d[i]) * rs * g[gs ? c + i : 0];
-    VecN<T, V>::store(y + (int64_t)blockIdx.x * W + c, v);
-  }
-}
-
 template <typename T, int V, int NT>
 int launch_input_norm(const InputNormParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
   const dim3 grid((max_new + p.R - 1) / p.R, n_seqs);
@@ -398,22 +343,4 @@ HDS_EXPORT int hds_input_norm(int dtype, const float* x, const void* embed, cons
     return input_norm(p, n_seqs, max_new, st);
   }
   return hipErrorInvalidValue;
-}
-
-HDS_EXPORT int hds_norm_rows(int dtype, const float* x, const void* delta, const int* idx, const float* g, int gs,
-                             void* y, int n_rows, int W, float eps, hipStream_t st) {
-  if (n_rows <= 0) return 0;
-  const bool v4 = W % 4 == 0;
-#define HDS_NR(TT, VV)                                                                                             \
-  hipLaunchKernelGGL((norm_rows_kernel<TT, VV>), dim3(n_rows), dim3(256), 0, st, x, (const TT*)delta, idx, g, gs, \
-                     (TT*)y, W, eps)
-  if (dtype == kBF16) {
-    if (v4) HDS_NR(bf16, 4); else HDS_NR(bf16, 1);
-  } else if (dtype == kF32) {
-    if (v4) HDS_NR(float, 4); else HDS_NR(float, 1);
-  } else {
-    return hipErrorInvalidValue;
-  }
-#undef HDS_NR
-  return hipGetLastError();
 }

@@ -7,17 +7,24 @@
 // library in the reference).
 //
 // Cache layout per layer (same as the reference BlockedKVCache): [num_blocks, block_size, 2, Hkv, D]
-// (K then V for each slot). Any block_size works: every staged tile row computes its own
+// (K then V for each slot). Key and value heads may differ in size: a slot is then [Hkv * DK | Hkv * DV], the same
+// layout when DK == DV. Any block_size works: every staged tile row computes its own
 // (block, slot) address, and LDS-DMA takes a per-lane global source address.
 //
 // Head dims: every multiple of 16 up to 256 that flash_attn.hip instantiates (HDS_PAGED_DIMS below), via the
-// generic tile helpers of attn_common.h. The RoPE scatter takes any head_dim % 4 == 0 with a rotary prefix
+// generic tile helpers of attn_common.h; other sizes that are multiples of 8 run the same kernel on zero-padded tiles,
+// float32 and everything else a plain kernel. The RoPE scatter takes any head_dim % 4 == 0 with a rotary prefix
 // of rot_dim (% 8 == 0) dims -- partial rotary (Phi, GPT-NeoX) rotates the prefix and copies the rest.
 //
 // Attention work unit ("atom"): (sequence, kv head, 128 packed rows). Rows pack the G = Hq/Hkv
 // query heads that share a kv head with the tokens of the chunk (row = token * G + head_in_group),
 // so K/V of a kv head are read ONCE for all of its query heads -- for decode (1 token) one wave
 // serves the whole GQA group from a single pass over the sequence's KV blocks.
+//
+// Options of all attention kernels: a sliding window; a sink, one learned score per query head that joins the softmax
+// denominator but has no key and no value; an output gate, one value per token and query head whose sigmoid multiplies
+// the head's output. head_norm_scatter is the counterpart of the RoPE scatter for heads that are RMS-normed and not
+// rotated.
 #include "attn_common.h"
 
 using namespace hds;
@@ -110,27 +117,121 @@ __global__ __launch_bounds__(256) void kv_rope_scatter_kernel(T* __restrict__ qk
 }
 
 // ------------------------------------------------------------------------------------------
+// per-head RMS norm of q (in place) and k (into the cache) + V copy into the cache
+// ------------------------------------------------------------------------------------------
+template <typename T>
+struct HeadNormParams {
+  T* qkv;  // [tokens, ld]: hq query heads of dk, hkv key heads of dk, hkv value heads of dv
+  int64_t ld;
+  const float* qn;  // [dk] or null: q stays as it is
+  const float* kn;
+  T* cache;
+  const int* tok_seq;
+  const int* tok_pos;
+  const int* tables;
+  int n_tok, max_blocks, block_size, hq, hkv, dk, dv;
+  float eps;
+};
+
+template <typename T>
+__device__ __forceinline__ T* cache_slot(const HeadNormParams<T>& p, int t) {
+  const int pos = p.tok_pos[t];
+  const int blk = p.tables[(int64_t)p.tok_seq[t] * p.max_blocks + pos / p.block_size];
+  return p.cache + ((int64_t)blk * p.block_size + pos % p.block_size) * p.hkv * (p.dk + p.dv);
+}
+
+// LPH lanes per head, 8 elements each (dk, dv and ld multiples of 8)
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void head_norm_scatter8_kernel(HeadNormParams<T> p) {
+  constexpr int HPB = 256 / LPH;
+  const int heads = p.hq + 2 * p.hkv;
+  const int64_t item = (int64_t)blockIdx.x * HPB + threadIdx.x / LPH;
+  const int c = 8 * (threadIdx.x % LPH);
+  const bool live = item < (int64_t)p.n_tok * heads;  // no early exit: the lanes of a head reduce together
+  const int t = live ? (int)(item / heads) : 0, h = live ? (int)(item - (int64_t)t * heads) : 0;
+  const bool is_v = h >= p.hq + p.hkv;
+  const int d = is_v ? p.dv : p.dk;
+  const int off = is_v ? (p.hq + p.hkv) * p.dk + (h - p.hq - p.hkv) * p.dv : h * p.dk;
+  const bool ok = live && c < d;
+  T* src = p.qkv + (int64_t)t * p.ld + off + c;
+  float v[8];
+  float ss = 0.f;
+  if (ok) {
+    Vec8<T>::load(src, v);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
+  }
+#pragma unroll
+  for (int o = LPH / 2; o >= 1; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  if (!ok) return;
+  const float* w = is_v ? nullptr : (h < p.hq ? p.qn : p.kn);
+  if (w != nullptr) {
+    const float rs = 1.f / sqrtf(ss / (float)p.dk + p.eps);
+    float n[8];
+    Vec8<float>::load(w + c, n);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= rs * n[i];
+  }
+  if (h < p.hq) {
+    if (w != nullptr) Vec8<T>::store(src, v);
+  } else {
+    Vec8<T>::store(cache_slot(p, t) + off - p.hq * p.dk + c, v);
+  }
+}
+
+// any sizes: one wave per head
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_scatter_kernel(HeadNormParams<T> p) {
+  const int heads = p.hq + 2 * p.hkv;
+  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (int64_t)p.n_tok * heads) return;
+  const int lane = threadIdx.x & 63, t = (int)(item / heads), h = (int)(item - (int64_t)t * heads);
+  const bool is_v = h >= p.hq + p.hkv;
+  const int d = is_v ? p.dv : p.dk;
+  const int off = is_v ? (p.hq + p.hkv) * p.dk + (h - p.hq - p.hkv) * p.dv : h * p.dk;
+  T* src = p.qkv + (int64_t)t * p.ld + off;
+  const float* w = is_v ? nullptr : (h < p.hq ? p.qn : p.kn);
+  T* dst = h < p.hq ? src : cache_slot(p, t) + off - p.hq * p.dk;
+  float rs = 1.f;
+  if (w != nullptr) {
+    float ss = 0.f;
+    for (int i = lane; i < d; i += 64) ss += to_f(src[i]) * to_f(src[i]);
+    rs = 1.f / sqrtf(wave_sum(ss) / (float)d + p.eps);
+  }
+  for (int i = lane; i < d; i += 64) dst[i] = from_f<T>(w != nullptr ? to_f(src[i]) * rs * w[i] : to_f(src[i]));
+}
+
+// ------------------------------------------------------------------------------------------
 // paged attention (ragged prefill + decode)
 // ------------------------------------------------------------------------------------------
+__device__ __forceinline__ float gate_of(float g) { return 1.f / (1.f + __expf(-g)); }
+
 struct PagedParams {
-  const bf16* q;  // [T, Hq, D] rows with token stride sq
+  const bf16* q;  // [T, Hq, DK] rows with token stride sq
   int64_t sq;
-  const bf16* cache;  // layer base: [num_blocks, block_size, 2, Hkv, D]
-  bf16* o;            // [T, Hq, D] contiguous
+  const bf16* cache;  // layer base: [num_blocks, block_size, Hkv * DK | Hkv * DV]
+  bf16* o;            // [T, Hq, DV] rows with token stride so
+  int64_t so;
   const int* atoms;   // [n_atoms][3] = {seq, kv_head, row_start}
   const int* seq_meta;  // [n_seqs][3] = {q_start, n_new, seen}
   const int* block_tables;
   int max_blocks;
   int block_size;
   int hq, hkv;
+  int dk, dv;  // read by the padded kernels only
   float scale;
   int window;
+  const float* sink;  // [Hq] or null
+  const bf16* gate;   // [T, Hq] with token stride sg, or null
+  int64_t sg;
 };
 
-template <int D, int NW>
+// DK / DV: head sizes, or with PAD their upper bounds (tiles zero-padded to them; the sizes are multiples of 8)
+template <int DK, int DV, int NW, bool PAD>
 __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
-  constexpr int KS = Dim<D>::KS, DT = Dim<D>::DT, TL = Dim<D>::TILE;
-  __shared__ __attribute__((aligned(16))) char smem[4 * TL];  // K[2], V[2]
+  constexpr int KS = Dim<DK>::KS, DT = Dim<DV>::DT, TLK = Dim<DK>::TILE, TLV = Dim<DV>::TILE;
+  __shared__ __attribute__((aligned(16))) char smem[2 * TLK + 2 * TLV];  // K[2], V[2]
+  const int dk = PAD ? p.dk : DK, dv = PAD ? p.dv : DV;
   const int* at = p.atoms + blockIdx.x * 3;
   const int seq = at[0], hk = at[1], row_start = at[2];
   const int q_start = p.seq_meta[seq * 3], n_new = p.seq_meta[seq * 3 + 1], seen = p.seq_meta[seq * 3 + 2];
@@ -144,13 +245,24 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
   const int qpos = seen + tok;  // absolute position of this row's query
   const float c = p.scale * kLog2e;
   const int* table = p.block_tables + (int64_t)seq * p.max_blocks;
-  const int64_t kv_row = 2LL * p.hkv * D;  // elements between consecutive slots
+  const int64_t kv_row = (int64_t)p.hkv * (dk + dv);  // elements between consecutive slots
 
+  if constexpr (PAD) {  // staging fills the chunks below dk / dv only: the rest stays zero
+    for (int i = threadIdx.x; i < (2 * TLK + 2 * TLV) / 16; i += 64 * NW) reinterpret_cast<u32x4*>(smem)[i] = u32x4{};
+    __syncthreads();
+  }
   bf16x8 qf[KS];
   {
-    const bf16* qp = p.q + (int64_t)(q_start + tok) * p.sq + (int64_t)head * D + 8 * h;
+    const bf16* qp = p.q + (int64_t)(q_start + tok) * p.sq + (int64_t)head * dk + 8 * h;
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 16 * ks);
+    for (int ks = 0; ks < KS; ++ks) {
+      if constexpr (PAD) {
+        qf[ks] = bf16x8{};
+        if (16 * ks + 8 * h < dk) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 16 * ks);
+      } else {
+        qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 16 * ks);
+      }
+    }
   }
   // last query position covered by this workgroup (rows are token-major)
   const int last_row = min(row_start + 32 * NW, n_rows) - 1;
@@ -162,14 +274,23 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
     const int first = seen + (row_start / G) - p.window + 1;
     kt_begin = first > 0 ? first / BN : 0;
   }
-  auto rowp = [&](int kt, int kv) {
+  auto rowp = [&](int kt, int off) {
     return [=](int row) {
       int pos = kt * BN + row;
       pos = pos < ctx ? pos : ctx - 1;
       const int blk = table[pos / p.block_size];
-      return p.cache + ((int64_t)blk * p.block_size + pos % p.block_size) * kv_row + (int64_t)kv * p.hkv * D +
-             (int64_t)hk * D;
+      return p.cache + ((int64_t)blk * p.block_size + pos % p.block_size) * kv_row + off;
     };
+  };
+  const int koff = hk * dk, voff = p.hkv * dk + hk * dv;
+  auto stage = [&](int buf, int kt) {
+    if constexpr (PAD) {
+      stage_tile_n<NW, DK>(smem + buf * TLK, rowp(kt, koff), dk / 8);
+      stage_tile_n<NW, DV>(smem + 2 * TLK + buf * TLV, rowp(kt, voff), dv / 8);
+    } else {
+      stage_tile_d<NW, DK>(smem + buf * TLK, rowp(kt, koff));
+      stage_tile_d<NW, DV>(smem + 2 * TLK + buf * TLV, rowp(kt, voff));
+    }
   };
   const int w_row_lo = row_start + 32 * w;
   const int w_qpos_lo = seen + min(w_row_lo, n_rows - 1) / G;
@@ -179,19 +300,20 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
   f32x16 o[DT];
 #pragma unroll
   for (int i = 0; i < DT; ++i) o[i] = f32x16{};
+  // the sink is a key of its own score and no value, seen before all others
   float m = -INFINITY, l = 0.f;
+  if (p.sink != nullptr) {
+    m = p.sink[head] * kLog2e;
+    l = 1.f;
+  }
 
-  stage_tile_d<NW, D>(smem, rowp(kt_begin, 0));
-  stage_tile_d<NW, D>(smem + 2 * TL, rowp(kt_begin, 1));
+  stage(0, kt_begin);
   __syncthreads();
   for (int kt = kt_begin; kt < kt_end; ++kt) {
     const int buf = (kt - kt_begin) & 1;
-    const char* Kt = smem + buf * TL;
-    const char* Vt = smem + 2 * TL + buf * TL;
-    if (kt + 1 < kt_end) {
-      stage_tile_d<NW, D>(smem + (buf ^ 1) * TL, rowp(kt + 1, 0));
-      stage_tile_d<NW, D>(smem + 2 * TL + (buf ^ 1) * TL, rowp(kt + 1, 1));
-    }
+    const char* Kt = smem + buf * TLK;
+    const char* Vt = smem + 2 * TLK + buf * TLV;
+    if (kt + 1 < kt_end) stage(buf ^ 1, kt + 1);
     const int k0 = kt * BN;
     bool skip = !wave_active || k0 > w_qpos_hi;
     if (p.window > 0 && k0 + BN - 1 <= w_qpos_lo - p.window) skip = true;
@@ -243,45 +365,93 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
     __syncthreads();
   }
   if (row_ok) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    bf16* op = p.o + ((int64_t)(q_start + tok) * p.hq + head) * D;
+    float inv = l > 0.f ? 1.f / l : 0.f;
+    if (p.gate != nullptr) inv *= gate_of((float)p.gate[(int64_t)(q_start + tok) * p.sg + head]);
+    bf16* op = p.o + (int64_t)(q_start + tok) * p.so + (int64_t)head * dv;
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) store_row_block<D>(op, o[dt], dt, h, inv);
+    for (int dt = 0; dt < DT; ++dt) {
+      if constexpr (PAD) store_row_block_n(op, o[dt], dt, h, inv, dv);
+      else store_row_block<DV>(op, o[dt], dt, h, inv);
+    }
   }
 }
 
 // ------------------------------------------------------------------------------------------
-// decode-only batches: split-K ("flash decoding") over the paged cache
+// single tokens: split-K ("flash decoding") over the paged cache
 // ------------------------------------------------------------------------------------------
-// One new token per sequence: the atom kernel above would run one 4-wave workgroup per (sequence, kv head) --
+// The atom kernel above would run one 4-wave workgroup per (sequence, kv head) for a lone new token --
 // 8 workgroups for a single Llama-3-8B sequence, each walking the whole context on a mostly empty 128-row MFMA tile
 // (35 us per layer at 540 keys, profiles/r3). Decode is a K/V stream, so this kernel is built like decode_attn.hip:
-// grid (splits, Hkv, n_seqs), a workgroup serves all G query heads of its kv head from ONE read of its key range,
-// 16-B loads with LPK = D / 8 lanes per key, online softmax in registers, lane groups and waves merged by
-// max / rescale, splits merged by a combine kernel through fp32 partials. The key range comes from the device-side
-// sequence metadata (seen + 1 keys), so one launch shape serves every step of a HIP-graph decode.
+// grid (splits, Hkv x blocks of GM query heads, tokens), a workgroup serves its query heads from ONE read of its key
+// range, 16-B loads with LPK lanes per key (8 elements of a key and of a value each), the next keys requested before
+// this iteration's are used, online softmax in registers, lane groups and waves merged by max / rescale, splits merged
+// by a combine kernel through fp32 partials. The key range comes from device-side metadata (and covers only the
+// window), so one launch shape serves every step of a HIP-graph decode.
 constexpr int kDecGMax = 8;
 
+template <typename T>
 struct PagedDecodeParams {
-  const bf16* q;  // [T, Hq, D] rows with token stride sq
+  const T* q;  // [T, Hq, DK] rows with token stride sq
   int64_t sq;
-  const bf16* cache;  // [num_blocks, block_size, 2, Hkv, D]
-  bf16* o;            // [T, Hq, D]
-  float* part_o;      // [n_seqs, Hq, splits, D]
-  float* part_ml;     // [n_seqs, Hq, splits, 2]
-  const int* seq_meta;  // [n_seqs][3] = {q_start, n_new (1), seen}
+  const T* cache;  // [num_blocks, block_size, Hkv * DK | Hkv * DV]
+  T* o;            // [T, Hq, DV] rows with token stride so
+  int64_t so;
+  float* part_o;   // [n, Hq, splits, DV]
+  float* part_ml;  // [n, Hq, splits, 2]
+  // the n tokens: seq_meta [n][3] = {q_start, n_new (1), seen}, one sequence each; or, with seq_meta null, rows
+  // toks[i] (null: i) of the step's tok_seq / tok_pos
+  const int* seq_meta;
+  const int* toks;
+  const int* tok_seq;
+  const int* tok_pos;
   const int* block_tables;
-  int max_blocks, block_size, hq, hkv, splits;
+  int max_blocks, block_size, hq, hkv, dk, dv, splits;
   float scale;
   int window;
-  // splits > 1: one int per (sequence, kv head), zero between launches. Non-null: the last workgroup of a
-  // (sequence, kv head) to finish merges the splits itself (no combine launch) and resets its counter to 0, so a
+  const float* sink;  // [Hq] or null
+  const T* gate;      // [T, Hq] with token stride sg, or null
+  int64_t sg;
+  // splits > 1: one int per (token, kv head), zero between launches. Non-null: the last workgroup of a
+  // (token, kv head) to finish merges the splits itself (no combine launch) and resets its counter to 0, so a
   // HIP-graph replay finds it zeroed again.
   int* counters;
 };
 
-template <int D>
-__device__ __forceinline__ void decode_merge_splits(const PagedDecodeParams& p, int b, int h, int d, int q_start) {
+struct DecodeToken {
+  int row, seq, pos;
+};
+
+template <typename T>
+__device__ __forceinline__ DecodeToken decode_token(const PagedDecodeParams<T>& p, int b) {
+  if (p.seq_meta != nullptr) return {p.seq_meta[3 * b], b, p.seq_meta[3 * b + 2]};
+  const int t = p.toks != nullptr ? p.toks[b] : b;
+  return {t, p.tok_seq[t], p.tok_pos[t]};
+}
+
+// this split's keys: an equal share of what the token sees
+template <typename T>
+__device__ __forceinline__ void decode_keys(const PagedDecodeParams<T>& p, int pos, int split, int& j0, int& j1) {
+  const int lo = p.window > 0 ? max(0, pos + 1 - p.window) : 0;
+  const int per = (pos + 1 - lo + p.splits - 1) / p.splits;
+  j0 = lo + split * per;
+  j1 = min(pos + 1, j0 + per);
+}
+
+// factor of head h's weighted value sum whose softmax so far has maximum m and denominator l
+template <typename T>
+__device__ __forceinline__ float decode_factor(const PagedDecodeParams<T>& p, int row, int h, float m, float l) {
+  float f = 1.f;
+  if (p.sink != nullptr) {
+    const float mm = fmaxf(m, p.sink[h]);
+    f = m == -INFINITY ? 0.f : __expf(m - mm);
+    l = l * f + __expf(p.sink[h] - mm);
+  }
+  f = l > 0.f ? f / l : 0.f;
+  return p.gate != nullptr ? f * gate_of(to_f(p.gate[(int64_t)row * p.sg + h])) : f;
+}
+
+template <typename T>
+__device__ __forceinline__ void decode_merge_splits(const PagedDecodeParams<T>& p, int b, int h, int d, int row) {
   const float* pm = p.part_ml + ((int64_t)b * p.hq + h) * p.splits * 2;
   float mm = -INFINITY;
   for (int s = 0; s < p.splits; ++s) mm = fmaxf(mm, pm[2 * s]);
@@ -289,58 +459,71 @@ __device__ __forceinline__ void decode_merge_splits(const PagedDecodeParams& p, 
   for (int s = 0; s < p.splits; ++s) {
     const float a = mm == -INFINITY ? 0.f : __expf(pm[2 * s] - mm);
     ll += pm[2 * s + 1] * a;
-    oo += p.part_o[(((int64_t)b * p.hq + h) * p.splits + s) * D + d] * a;
+    oo += p.part_o[(((int64_t)b * p.hq + h) * p.splits + s) * p.dv + d] * a;
   }
-  p.o[((int64_t)q_start * p.hq + h) * D + d] = (bf16)(ll > 0.f ? oo / ll : 0.f);
+  p.o[(int64_t)row * p.so + (int64_t)h * p.dv + d] = from_f<T>(oo * decode_factor(p, row, h, mm, ll));
 }
 
-template <int D>
-__global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) {
-  constexpr int LPK = D / 8, KPW = 64 / LPK;
-  __shared__ float red[4][kDecGMax][2 + D];
-  const int split = blockIdx.x, hk = blockIdx.y, b = blockIdx.z;
-  const int G = p.hq / p.hkv;
+template <int LPK, int GM>
+__global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf16> p) {
+  constexpr int KPW = 64 / LPK;
+  __shared__ float red[4][GM][2 + 8 * LPK];
+  const int G = p.hq / p.hkv, gb = (G + GM - 1) / GM;
+  const int split = blockIdx.x, hk = blockIdx.y / gb, g0 = (blockIdx.y % gb) * GM, b = blockIdx.z;
+  const int gn = min(GM, G - g0), h0 = hk * G + g0;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int kl = lane / LPK, c = lane % LPK;
-  const int q_start = p.seq_meta[3 * b], ctx = p.seq_meta[3 * b + 2] + 1;
-  const int jb = p.window > 0 ? max(0, ctx - p.window) : 0;
-  const int kps = (ctx + p.splits - 1) / p.splits;
-  const int j0 = split * kps, j1 = min(ctx, j0 + kps);
-  const int* table = p.block_tables + (int64_t)b * p.max_blocks;
-  const int64_t kv_row = 2LL * p.hkv * D;
+  const DecodeToken tk = decode_token(p, b);
+  int j0, j1;
+  decode_keys(p, tk.pos, split, j0, j1);
+  const int* table = p.block_tables + (int64_t)tk.seq * p.max_blocks;
+  const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
+  const bool k_on = 8 * c < p.dk, v_on = 8 * c < p.dv;
+  const bf16* kbase = p.cache + (int64_t)hk * p.dk + c * 8;
+  const bf16* vbase = p.cache + (int64_t)p.hkv * p.dk + (int64_t)hk * p.dv + c * 8;
 
-  float qv[kDecGMax][8];
+  float qv[GM][8];
 #pragma unroll
-  for (int g = 0; g < kDecGMax; ++g) {
-    if (g < G) {
-      Vec8<bf16>::load(p.q + (int64_t)q_start * p.sq + (int64_t)(hk * G + g) * D + c * 8, qv[g]);
+  for (int g = 0; g < GM; ++g) {
+    if (g < gn && k_on) {
+      Vec8<bf16>::load(p.q + (int64_t)tk.row * p.sq + (int64_t)(h0 + g) * p.dk + c * 8, qv[g]);
 #pragma unroll
       for (int e = 0; e < 8; ++e) qv[g][e] *= p.scale;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) qv[g][e] = 0.f;
     }
   }
-  float m[kDecGMax], l[kDecGMax], acc[kDecGMax][8];
+  float m[GM], l[GM], acc[GM][8];
 #pragma unroll
-  for (int g = 0; g < kDecGMax; ++g) {
+  for (int g = 0; g < GM; ++g) {
     m[g] = -INFINITY;
     l[g] = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; ++e) acc[g][e] = 0.f;
   }
-  for (int j = j0 + w * KPW + kl; j - kl < j1; j += 4 * KPW) {
-    const bool ok = j < j1 && j >= jb;
-    float kv[8] = {}, vv[8] = {};
-    if (ok) {
-      const int blk = table[j / p.block_size];
-      const bf16* kb = p.cache + ((int64_t)blk * p.block_size + j % p.block_size) * kv_row + (int64_t)hk * D + c * 8;
-      Vec8<bf16>::load(kb, kv);
-      Vec8<bf16>::load(kb + (int64_t)p.hkv * D, vv);
+  bf16x8 kn = {}, vn = {};
+  auto fetch = [&](int j) {
+    kn = bf16x8{};
+    vn = bf16x8{};
+    if (j < j1) {
+      const int64_t r = ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * kv_row;
+      if (k_on) kn = *reinterpret_cast<const bf16x8*>(kbase + r);
+      if (v_on) vn = *reinterpret_cast<const bf16x8*>(vbase + r);
     }
+  };
+  int j = j0 + w * KPW + kl;
+  fetch(j);
+  for (; j - kl < j1; j += 4 * KPW) {
+    const bool ok = j < j1;
+    const bf16x8 kc = kn, vc = vn;
+    fetch(j + 4 * KPW);
 #pragma unroll
-    for (int g = 0; g < kDecGMax; ++g) {
-      if (g >= G) break;
+    for (int g = 0; g < GM; ++g) {
+      if (g >= gn) break;
       float sc = 0.f;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) sc += qv[g][e] * kv[e];
+      for (int e = 0; e < 8; ++e) sc += qv[g][e] * (float)kc[e];
 #pragma unroll
       for (int off = LPK / 2; off >= 1; off >>= 1) sc += __shfl_xor(sc, off, 64);
       sc = ok ? sc : -INFINITY;
@@ -349,13 +532,13 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) 
       const float a = none ? 1.f : __expf(m[g] - mn), e_s = none ? 0.f : __expf(sc - mn);
       l[g] = l[g] * a + e_s;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[g][e] = acc[g][e] * a + e_s * vv[e];
+      for (int e = 0; e < 8; ++e) acc[g][e] = acc[g][e] * a + e_s * (float)vc[e];
       m[g] = mn;
     }
   }
 #pragma unroll
-  for (int g = 0; g < kDecGMax; ++g) {
-    if (g >= G) break;
+  for (int g = 0; g < GM; ++g) {
+    if (g >= gn) break;
 #pragma unroll
     for (int off = LPK; off < 64; off <<= 1) {
       const float mo = __shfl_xor(m[g], off, 64), lo = __shfl_xor(l[g], off, 64);
@@ -369,8 +552,8 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) 
   }
   if (kl == 0) {
 #pragma unroll
-    for (int g = 0; g < kDecGMax; ++g) {
-      if (g >= G) break;
+    for (int g = 0; g < GM; ++g) {
+      if (g >= gn) break;
       if (c == 0) {
         red[w][g][0] = m[g];
         red[w][g][1] = l[g];
@@ -380,7 +563,7 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) 
     }
   }
   __syncthreads();
-  for (int t = threadIdx.x; t < G * LPK; t += 256) {
+  for (int t = threadIdx.x; t < gn * LPK; t += 256) {
     const int g = t / LPK, cc = t % LPK;
     float mm = -INFINITY;
     for (int ww = 0; ww < 4; ++ww) mm = fmaxf(mm, red[ww][g][0]);
@@ -391,20 +574,18 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) 
 #pragma unroll
       for (int e = 0; e < 8; ++e) oo[e] += red[ww][g][2 + cc * 8 + e] * a;
     }
-    const int h = hk * G + g;
+    const int h = h0 + g;
     if (p.splits == 1) {
-      const float inv = ll > 0.f ? 1.f / ll : 0.f;
+      const float f = decode_factor(p, tk.row, h, mm, ll);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) oo[e] *= inv;
-      Vec8<bf16>::store(p.o + ((int64_t)q_start * p.hq + h) * D + cc * 8, oo);
+      for (int e = 0; e < 8; ++e) oo[e] *= f;
+      if (8 * cc < p.dv) Vec8<bf16>::store(p.o + (int64_t)tk.row * p.so + (int64_t)h * p.dv + cc * 8, oo);
     } else {
-      float* po = p.part_o + (((int64_t)b * p.hq + h) * p.splits + split) * D + cc * 8;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) po[e] = oo[e];
+      const int64_t pi = ((int64_t)b * p.hq + h) * p.splits + split;
+      if (8 * cc < p.dv) Vec8<float>::store(p.part_o + pi * p.dv + cc * 8, oo);
       if (cc == 0) {
-        float* pm = p.part_ml + (((int64_t)b * p.hq + h) * p.splits + split) * 2;
-        pm[0] = mm;
-        pm[1] = ll;
+        p.part_ml[2 * pi] = mm;
+        p.part_ml[2 * pi + 1] = ll;
       }
     }
   }
@@ -418,30 +599,95 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams p) 
     __syncthreads();
     if (!s_last) return;
     __threadfence();
-    for (int t = threadIdx.x; t < G * D; t += 256) decode_merge_splits<D>(p, b, hk * G + t / D, t % D, q_start);
+    for (int t = threadIdx.x; t < gn * p.dv; t += 256) decode_merge_splits(p, b, h0 + t / p.dv, t % p.dv, tk.row);
     if (threadIdx.x == 0) p.counters[b * p.hkv + hk] = 0;
   }
 }
 
-// One workgroup of D threads per (sequence, q head): the split maxima / sums are loaded once, one per thread, into LDS
+// any type and sizes: one workgroup per (split, query head, token); a wave's lanes share the dims of a key, then every
+// thread owns output columns
+constexpr int kPlainKeys = 64;
+
+template <typename T>
+__global__ __launch_bounds__(256) void paged_plain_kernel(PagedDecodeParams<T> p) {
+  extern __shared__ float sm[];  // q [dk], acc [dv], scores / weights [kPlainKeys]
+  float* sq = sm;
+  float* acc = sm + p.dk;
+  float* ss = acc + p.dv;
+  const int split = blockIdx.x, h = blockIdx.y, b = blockIdx.z, hk = h / (p.hq / p.hkv);
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const DecodeToken tk = decode_token(p, b);
+  int j0, j1;
+  decode_keys(p, tk.pos, split, j0, j1);
+  const int* table = p.block_tables + (int64_t)tk.seq * p.max_blocks;
+  const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
+  auto slot = [&](int j) {
+    return p.cache + ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * kv_row;
+  };
+  for (int i = threadIdx.x; i < p.dk; i += 256) sq[i] = to_f(p.q[(int64_t)tk.row * p.sq + (int64_t)h * p.dk + i]);
+  for (int i = threadIdx.x; i < p.dv; i += 256) acc[i] = 0.f;
+  __syncthreads();
+  float m = -INFINITY, l = 0.f;
+  for (int jb = j0; jb < j1; jb += kPlainKeys) {
+    const int nk = min(kPlainKeys, j1 - jb);
+    for (int k = w; k < nk; k += 4) {
+      const T* kr = slot(jb + k) + (int64_t)hk * p.dk;
+      float s = 0.f;
+      for (int i = lane; i < p.dk; i += 64) s += sq[i] * to_f(kr[i]);
+      s = wave_sum(s);
+      if (lane == 0) ss[k] = s * p.scale;
+    }
+    __syncthreads();
+    float mt = m;
+    for (int k = 0; k < nk; ++k) mt = fmaxf(mt, ss[k]);
+    __syncthreads();
+    if ((int)threadIdx.x < nk) ss[threadIdx.x] = __expf(ss[threadIdx.x] - mt);
+    __syncthreads();
+    const float alpha = __expf(m - mt);  // 0 at the first tile
+    m = mt;
+    float sum = 0.f;
+    for (int k = 0; k < nk; ++k) sum += ss[k];
+    l = l * alpha + sum;
+    for (int i = threadIdx.x; i < p.dv; i += 256) {
+      float o = acc[i] * alpha;
+      for (int k = 0; k < nk; ++k) o += ss[k] * to_f(slot(jb + k)[p.hkv * p.dk + hk * p.dv + i]);
+      acc[i] = o;
+    }
+    __syncthreads();
+  }
+  const int64_t pi = ((int64_t)b * p.hq + h) * p.splits + split;
+  if (p.splits == 1) {
+    const float f = decode_factor(p, tk.row, h, m, l);
+    for (int i = threadIdx.x; i < p.dv; i += 256)
+      p.o[(int64_t)tk.row * p.so + (int64_t)h * p.dv + i] = from_f<T>(acc[i] * f);
+    return;
+  }
+  for (int i = threadIdx.x; i < p.dv; i += 256) p.part_o[pi * p.dv + i] = acc[i];
+  if (threadIdx.x == 0) {
+    p.part_ml[2 * pi] = m;
+    p.part_ml[2 * pi + 1] = l;
+  }
+}
+
+// One workgroup per (token, q head): the split maxima / sums are loaded once, one per thread, into LDS
 // (one memory round trip instead of a dependent walk over the splits), then every thread merges its output column
-// over the splits from partial-o values it requested before the barrier (splits <= 64 <= D).
-template <int D>
-__global__ __launch_bounds__(D) void paged_decode_combine_kernel(PagedDecodeParams p) {
+// over the splits from partial-o values it requested before the barrier (splits <= 64 <= threads).
+template <typename T>
+__global__ __launch_bounds__(256) void paged_decode_combine_kernel(PagedDecodeParams<T> p) {
   __shared__ float s_m[64], s_l[64];
   const int bh = blockIdx.x, b = bh / p.hq, h = bh % p.hq;
-  const int d = threadIdx.x;
+  const int d0 = threadIdx.x, dl = min(d0, p.dv - 1);
   // every load is issued before the barrier: the partial-o column (its addresses need no split stat) and the output
   // row overlap the stats' round trip instead of following it
-  const float* po = p.part_o + (int64_t)bh * p.splits * D + d;
+  const float* po = p.part_o + (int64_t)bh * p.splits * p.dv;
   float pov[64];
 #pragma unroll
-  for (int s = 0; s < 64; ++s) pov[s] = s < p.splits ? po[(int64_t)s * D] : 0.f;
-  const int row = p.seq_meta[3 * b];
+  for (int s = 0; s < 64; ++s) pov[s] = s < p.splits ? po[(int64_t)s * p.dv + dl] : 0.f;
+  const int row = decode_token(p, b).row;
   const float* pm = p.part_ml + (int64_t)bh * p.splits * 2;
-  if (d < p.splits) {
-    s_m[d] = pm[2 * d];
-    s_l[d] = pm[2 * d + 1];
+  if (d0 < p.splits) {
+    s_m[d0] = pm[2 * d0];
+    s_l[d0] = pm[2 * d0 + 1];
   }
   __syncthreads();
   float mm = -INFINITY;
@@ -455,7 +701,55 @@ __global__ __launch_bounds__(D) void paged_decode_combine_kernel(PagedDecodePara
       oo += pov[s] * a;
     }
   }
-  p.o[((int64_t)row * p.hq + h) * D + d] = (bf16)(ll > 0.f ? oo / ll : 0.f);
+  const float f = decode_factor(p, row, h, mm, ll);
+  T* op = p.o + (int64_t)row * p.so + (int64_t)h * p.dv;
+  if (d0 < p.dv) op[d0] = from_f<T>(oo * f);
+  for (int d = d0 + blockDim.x; d < p.dv; d += blockDim.x) {  // heads wider than the workgroup
+    oo = 0.f;
+    for (int s = 0; s < p.splits; ++s) oo += po[(int64_t)s * p.dv + d] * (mm == -INFINITY ? 0.f : __expf(s_m[s] - mm));
+    op[d] = from_f<T>(oo * f);
+  }
+}
+
+template <typename T>
+void launch_combine(const PagedDecodeParams<T>& p, int n, hipStream_t st) {
+  const int threads = p.dv >= 256 ? 256 : (p.dv + 63) / 64 * 64;
+  hipLaunchKernelGGL(paged_decode_combine_kernel<T>, dim3(n * p.hq), dim3(threads), 0, st, p);
+}
+
+template <int LPK>
+int launch_decode(const PagedDecodeParams<bf16>& p, int n, hipStream_t st) {
+  const int G = p.hq / p.hkv;
+#define HDS_DEC(GM)                                                                                                 \
+  hipLaunchKernelGGL((paged_decode_kernel<LPK, GM>), dim3(p.splits, p.hkv * ((G + GM - 1) / GM), n), dim3(256), 0, st, p)
+  if (G == 1) HDS_DEC(1); else if (G == 2) HDS_DEC(2); else if (G <= 4) HDS_DEC(4); else HDS_DEC(8);
+#undef HDS_DEC
+  if (p.splits > 1 && p.counters == nullptr) launch_combine(p, n, st);
+  return hipGetLastError();
+}
+
+template <typename T>
+int launch_plain(const PagedDecodeParams<T>& p, int n, hipStream_t st) {
+  const size_t lds = (p.dk + p.dv + kPlainKeys) * sizeof(float);
+  if (lds > 64 * 1024 || p.hq > 65535) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(paged_plain_kernel<T>, dim3(p.splits, p.hq, n), dim3(256), lds, st, p);
+  if (p.splits > 1) launch_combine(p, n, st);
+  return hipGetLastError();
+}
+
+template <typename T>
+int launch_head_norm(const HeadNormParams<T>& p, hipStream_t st) {
+  const int64_t items = (int64_t)p.n_tok * (p.hq + 2 * p.hkv);
+  const int d = p.dk > p.dv ? p.dk : p.dv;
+  if (p.dk % 8 || p.dv % 8 || p.ld % 8 || d > 512) {
+    hipLaunchKernelGGL(head_norm_scatter_kernel<T>, dim3((items + 3) / 4), dim3(256), 0, st, p);
+    return hipGetLastError();
+  }
+#define HDS_HN(L) \
+  hipLaunchKernelGGL((head_norm_scatter8_kernel<T, L>), dim3((items + 256 / L - 1) / (256 / L)), dim3(256), 0, st, p)
+  if (d <= 64) HDS_HN(8); else if (d <= 128) HDS_HN(16); else if (d <= 256) HDS_HN(32); else HDS_HN(64);
+#undef HDS_HN
+  return hipGetLastError();
 }
 
 }  // namespace
@@ -485,30 +779,61 @@ HDS_EXPORT int hds_kv_rope_scatter(int dtype, void* qkv, int64_t sq, void* cache
   return hipGetLastError();
 }
 
-// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]
-HDS_EXPORT int hds_paged_attn(const void* q, int64_t sq, const void* cache, void* o, const int* atoms, int n_atoms,
-                              const int* seq_meta, const int* block_tables, int max_blocks, int block_size, int hq,
-                              int hkv, int head_dim, float scale, int window, hipStream_t st) {
-  if (hq % hkv) return hipErrorInvalidValue;
+// q heads normed in place, k heads normed into the cache, v heads copied there; qn / kn null: no norm
+HDS_EXPORT int hds_head_norm_scatter(int dtype, void* qkv, int64_t ld, const float* qn, const float* kn, void* cache,
+                                     const int* tok_seq, const int* tok_pos, const int* block_tables, int n_tok,
+                                     int max_blocks, int block_size, int hq, int hkv, int dk, int dv, float eps,
+                                     hipStream_t st) {
+  if (n_tok <= 0) return 0;
+  if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || ld < (int64_t)(hq + hkv) * dk + (int64_t)hkv * dv)
+    return hipErrorInvalidValue;
+  if (dtype == kBF16)
+    return launch_head_norm(HeadNormParams<bf16>{(bf16*)qkv, ld, qn, kn, (bf16*)cache, tok_seq, tok_pos, block_tables,
+                                                 n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps}, st);
+  if (dtype == kF32)
+    return launch_head_norm(HeadNormParams<float>{(float*)qkv, ld, qn, kn, (float*)cache, tok_seq, tok_pos,
+                                                  block_tables, n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps},
+                            st);
+  return hipErrorInvalidValue;
+}
+
+// bf16 head sizes the atom kernel takes (16-B rows; the caller checks sq and the q / o alignment)
+HDS_EXPORT int hds_paged_attn_supported(int dk, int dv) {
+  return dk >= 8 && dv >= 8 && dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256;
+}
+
+// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]; sink [hq] and gate [tokens, hq] may be null
+HDS_EXPORT int hds_paged_attn(const void* q, int64_t sq, const void* cache, void* o, int64_t so, const int* atoms,
+                              int n_atoms, const int* seq_meta, const int* block_tables, int max_blocks,
+                              int block_size, int hq, int hkv, int dk, int dv, float scale, int window,
+                              const float* sink, const void* gate, int64_t sg, hipStream_t st) {
+  if (hq < 1 || hkv < 1 || hq % hkv || sq % 8 || so % 4 || !hds_paged_attn_supported(dk, dv))
+    return hipErrorInvalidValue;
   if (n_atoms <= 0) return 0;
-  PagedParams p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, atoms, seq_meta, block_tables, max_blocks,
-                block_size, hq, hkv, scale, window};
-#define HDS_CASE(d)                                                                          \
-  if (head_dim == d) {                                                                       \
-    hipLaunchKernelGGL((paged_attn_kernel<d, 4>), dim3(n_atoms), dim3(256), 0, st, p);       \
-    return hipGetLastError();                                                                \
+  PagedParams p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, atoms, seq_meta, block_tables, max_blocks,
+                block_size, hq, hkv, dk, dv, scale, window, sink, (const bf16*)gate, sg};
+#define HDS_CASE(d)                                                                                    \
+  if (dk == d && dv == d) {                                                                            \
+    hipLaunchKernelGGL((paged_attn_kernel<d, d, 4, false>), dim3(n_atoms), dim3(256), 0, st, p);       \
+    return hipGetLastError();                                                                          \
   }
   HDS_PAGED_DIMS(HDS_CASE)
 #undef HDS_CASE
+#define HDS_PAD(a, b)                                                                                  \
+  if (dk <= a && dv <= b) {                                                                            \
+    hipLaunchKernelGGL((paged_attn_kernel<a, b, 4, true>), dim3(n_atoms), dim3(256), 0, st, p);        \
+    return hipGetLastError();                                                                          \
+  }
+  HDS_PAD(64, 64) HDS_PAD(64, 128) HDS_PAD(64, 256) HDS_PAD(128, 64) HDS_PAD(128, 128) HDS_PAD(128, 256)
+  HDS_PAD(256, 64) HDS_PAD(256, 128) HDS_PAD(256, 256)
+#undef HDS_PAD
   return hipErrorInvalidValue;
 }
 
 HDS_EXPORT int hds_paged_rows_per_atom() { return 128; }
 
-// decode-only batches (every sequence has exactly one new token)
-HDS_EXPORT int hds_paged_decode_supported(int head_dim, int G) {
-  return (head_dim == 64 || head_dim == 128 || head_dim == 256) && G >= 1 && G <= kDecGMax;
-}
+// the vectorised single-token kernel (bf16): any group size, head sizes that are multiples of 8 up to 256
+HDS_EXPORT int hds_paged_decode_supported(int dk, int dv) { return hds_paged_attn_supported(dk, dv); }
 
 // key splits for n_seqs sequences of at most max_ctx keys: >= 2 workgroups per CU overall, >= 32 keys per split
 HDS_EXPORT int hds_paged_decode_splits(int n_seqs, int hkv, int max_ctx) {
@@ -519,30 +844,41 @@ HDS_EXPORT int hds_paged_decode_splits(int n_seqs, int hkv, int max_ctx) {
   return splits < 1 ? 1 : (splits > 64 ? 64 : splits);
 }
 
-// counters: null -> the splits are merged by a second (combine) launch; else n_seqs * hkv zeroed ints and the last
-// workgroup of each (sequence, kv head) merges them in the same launch (see paged_decode_kernel)
-HDS_EXPORT int hds_paged_decode(const void* q, int64_t sq, const void* cache, void* o, float* part_o, float* part_ml,
-                                const int* seq_meta, const int* block_tables, int max_blocks, int block_size,
-                                int n_seqs, int hq, int hkv, int head_dim, int splits, float scale, int window,
-                                int* counters, hipStream_t st) {
-  if (n_seqs <= 0) return 0;
-  if (hq % hkv || !hds_paged_decode_supported(head_dim, hq / hkv) || splits < 1 || splits > 64 ||
+// Single tokens. seq_meta: one sequence with one new token each (n of them); null: the n tokens toks (null: 0 .. n - 1)
+// of a step described by tok_seq / tok_pos. plain: the kernel for any type and size (always for float32).
+// counters: null -> the splits are merged by a second (combine) launch; else n * hkv zeroed ints and the last
+// workgroup of each (token, kv head) merges them in the same launch (at most kDecGMax query heads per kv head)
+HDS_EXPORT int hds_paged_decode(int dtype, int plain, const void* q, int64_t sq, const void* cache, void* o, int64_t so,
+                                float* part_o, float* part_ml, const int* seq_meta, const int* toks,
+                                const int* tok_seq, const int* tok_pos, const int* block_tables, int max_blocks,
+                                int block_size, int n, int hq, int hkv, int dk, int dv, int splits, float scale,
+                                int window, const float* sink, const void* gate, int64_t sg, int* counters,
+                                hipStream_t st) {
+  if (n <= 0) return 0;
+  if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || splits < 1 || splits > 64 || n > 65535 ||
+      (seq_meta == nullptr && (tok_seq == nullptr || tok_pos == nullptr)) ||
       (splits > 1 && (!part_o || !part_ml)))  // <= 64: the combine kernel stages the split stats in LDS
     return hipErrorInvalidValue;
-  PagedDecodeParams p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, part_o, part_ml, seq_meta, block_tables,
-                      max_blocks, block_size, hq, hkv, splits, scale, window, counters};
-  const dim3 grid(splits, hkv, n_seqs);
-  switch (head_dim) {
-#define HDS_DEC(d)                                                                                            \
-  case d:                                                                                                     \
-    hipLaunchKernelGGL(paged_decode_kernel<d>, grid, dim3(256), 0, st, p);                                    \
-    if (splits > 1 && counters == nullptr)                                                                    \
-      hipLaunchKernelGGL(paged_decode_combine_kernel<d>, dim3(n_seqs * hq), dim3(d), 0, st, p);               \
-    break;
-    HDS_DEC(64)
-    HDS_DEC(128)
-    HDS_DEC(256)
-#undef HDS_DEC
+  if (dtype == kF32) {
+    return launch_plain(PagedDecodeParams<float>{(const float*)q, sq, (const float*)cache, (float*)o, so, part_o,
+                                                 part_ml, seq_meta, toks, tok_seq, tok_pos, block_tables, max_blocks,
+                                                 block_size, hq, hkv, dk, dv, splits, scale, window, sink,
+                                                 (const float*)gate, sg, nullptr}, n, st);
   }
-  return hipGetLastError();
+  if (dtype != kBF16) return hipErrorInvalidValue;
+  PagedDecodeParams<bf16> p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, part_o, part_ml, seq_meta, toks,
+                            tok_seq, tok_pos, block_tables, max_blocks, block_size, hq, hkv, dk, dv, splits, scale,
+                            window, sink, (const bf16*)gate, sg, counters};
+  if (plain) {
+    p.counters = nullptr;
+    return launch_plain(p, n, st);
+  }
+  if (!hds_paged_decode_supported(dk, dv) || sq % 8 || so % 8 || hkv > 65535 / kDecGMax ||
+      (counters != nullptr && hq / hkv > kDecGMax))
+    return hipErrorInvalidValue;
+  const int d = dk > dv ? dk : dv;
+  if (d <= 32) return launch_decode<4>(p, n, st);
+  if (d <= 64) return launch_decode<8>(p, n, st);
+  if (d <= 128) return launch_decode<16>(p, n, st);
+  return launch_decode<32>(p, n, st);
 }

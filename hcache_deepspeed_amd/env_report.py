@@ -30,6 +30,8 @@ OPS = {
     "latent_attention (ragged)": ("kernels", "hds_latent_decode"),
     "gated_scan (minGRU)": ("kernels", "hds_gated_scan"),
     "input_norm (norm + input convolution)": ("kernels", "hds_input_norm"),
+    "residual_norm (norm on a sublayer's output)": ("kernels", "hds_residual_norm"),
+    "routed experts (router, grouped / skinny products)": ("kernels", "hds_experts_skinny"),
     "moe_scatter / moe_gather": ("kernels", "hds_moe_dispatch"),
     "quantizer (int8/int4)": ("kernels", "hds_quant_int"),
     "fp_quantizer (fp8)": ("kernels", "hds_quant_fp8"),

@@ -41,11 +41,15 @@ class ArchSpec:
     tie_embeddings: bool = False
     lm_head_bias: bool = False
     moe: Optional[dict] = None         # {num_experts, top_k, normalize, shared}
-    # layers of several kinds (hybrid.HybridTransformer): one entry per layer, {"mixer": {"type", sizes ...},
-    # "mlp": {"ff", "act"} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
+    # layers listed one by one (hybrid.py): one entry per layer with weights, {"mixer": {"type", sizes ...}, "mlp":
+    # {"ff", "act"}, {"ff", "act", "shared_ff", "router": {...}} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
     layers: Optional[list] = None
     loop: Optional[dict] = None
+    order: Optional[list] = None       # the layer every layer run uses (None: each once, with ``loop``)
     input_conv_taps: int = 1
+    norm_place: str = "pre"            # pre: sublayers read the normed residual | post: their output is normed
+    embed_scale: float = 1.0
+    logit_scale: float = 1.0
     extra: dict = field(default_factory=dict)
 
     # LlamaConfig-compatible aliases used by the engine / KV cache sizing
@@ -66,7 +70,9 @@ def _g(hf, *names, default=None):
 
 
 def run_order(spec):
-    """Layer index of every layer run, in order (looped layers appear once per pass)."""
+    """Layer index of every layer run, in order (looped and shared layers appear once per pass)."""
+    if spec.order is not None:
+        return list(spec.order)
     n, lp = len(spec.layers), spec.loop
     if not lp:
         return list(range(n))
@@ -122,8 +128,75 @@ def convert_gofasun(sd, spec):
     return out
 
 
+# ---------------------------------------------------------------------------------------------
+# Buvuzen: grouped-query attention without rotation (query / key norms, sliding window, sink, output gate) and routed
+# experts, the norms on the sublayers' outputs; layers may share another layer's weights
+# ---------------------------------------------------------------------------------------------
+def _buvuzen_layer(e, index):
+    if e["type"] != "attention":
+        raise NotImplementedError(f"Buvuzen mixer {e['type']!r}")
+    m, mlp = e["mixer"], e.get("mlp")
+    mixer = {"type": "attention", "heads": int(m["heads"]), "kv_heads": int(m["kv_heads"]), "dim": int(m["dim"]),
+             "vdim": int(m["vdim"]), "window": int((m.get("mask") or {}).get("size") or 0), "scale": float(m["scale"]),
+             "gated": True}
+    if mlp is not None:
+        if mlp.get("kind", "moe") != "moe":
+            raise NotImplementedError(f"Buvuzen feed-forward {mlp['kind']!r}")
+        r = mlp["router"]
+        g = r.get("groups") or {}
+        mlp = {"kind": "moe", "ff": int(mlp["expert"]["ff"]), "shared_ff": int((mlp.get("shared") or {}).get("ff", 0)),
+               "act": "silu", "router": {"experts": int(r["experts"]), "identity": int(r.get("identity") or 0),
+                                         "top": int(r["top"]), "groups": int(g.get("count", 1)),
+                                         "keep": int(g.get("keep", 1)), "scale": float(r.get("scale", 1.0))}}
+    return {"mixer": mixer, "mlp": mlp, "source": index}
+
+
+def spec_buvuzen(cfg):
+    entries, layers, place, order = cfg["layers"], [], {}, []
+    for i, e in enumerate(entries):
+        at, hops = i, 0
+        while entries[at].get("weights_of") is not None:
+            at, hops = int(entries[at]["weights_of"]), hops + 1
+            if not 0 <= at < len(entries) or hops > len(entries):
+                raise ValueError(f"layer {i}: weights_of leads to no layer with weights")
+        if at not in place:
+            place[at] = len(layers)
+            layers.append(_buvuzen_layer(entries[at], at))
+        order.append(place[at])
+    heads = max(x["mixer"]["heads"] for x in layers)
+    return ArchSpec(model_type="buvuzen", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                    num_hidden_layers=len(order), num_attention_heads=heads,
+                    num_key_value_heads=max(x["mixer"]["kv_heads"] for x in layers),
+                    head_dim=max(x["mixer"]["dim"] for x in layers),
+                    intermediate_size=max((x["mlp"]["ff"] for x in layers if x["mlp"]), default=0), norm="rms",
+                    norm_eps=float(cfg["norm"]["eps"]), act="silu", gated=True, pos="none", layers=layers, order=order,
+                    norm_place="post", embed_scale=float(cfg["embedding"]["scale"]),
+                    logit_scale=float(cfg["logit_scale"]))
+
+
+def convert_buvuzen(sd, spec):
+    def gain(name):  # norm weights are stored around zero
+        return 1 + sd[name].float()
+
+    out = {"embed": sd["embed"], "final.w": gain("final.norm"), "lm_head.w": sd["head"], "layers": []}
+    for e in spec.layers:
+        p = f"l{e['source']}."
+        L = {"mix": {k[len(p) + 4:]: v for k, v in sd.items() if k.startswith(p + "mix.")}, "ln1.w": gain(p + "norm1")}
+        if e["mlp"] is not None:
+            m = p + "mlp."
+            L["ln2.w"] = gain(p + "norm2")
+            L["experts"] = {k: torch.stack([sd[f"{m}e{x}.{k}"] for x in range(e["mlp"]["router"]["experts"])])
+                            for k in ("gate", "up", "down")}
+            names = ["router", "correction"]
+            if e["mlp"]["shared_ff"]:
+                names += ["shared.gate", "shared.up", "shared.down", "shared.sg"]
+            L["experts"].update({k: sd[m + k] for k in names})
+        out["layers"].append(L)
+    return out
+
+
 # config.json's "architecture" / "model_type" -> (config reader, weight converter)
-ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun)}
+ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun), "buvuzen": (spec_buvuzen, convert_buvuzen)}
 
 
 def spec_from_hf(hf):

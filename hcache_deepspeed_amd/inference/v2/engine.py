@@ -19,7 +19,7 @@ import torch
 
 from ... import comm as dist
 from ...utils.logging import log_dist
-from .hybrid import HybridTransformer
+from .hybrid import HybridTransformer, PostNormTransformer
 from .model import RaggedTransformer
 from .ragged import (BlockedKVCache, DSStateManager, DSStateManagerConfig, RaggedBatchWrapper, SequenceStatePool)
 
@@ -59,6 +59,13 @@ class RaggedInferenceEngineConfig:
         return cfg
 
 
+def transformer_class(spec):
+    """The model implementation that serves an ArchSpec."""
+    if spec.layers is None:
+        return RaggedTransformer
+    return PostNormTransformer if spec.norm_place == "post" else HybridTransformer
+
+
 class InferenceEngineV2:
 
     def __init__(self, model_config, weights, engine_config: RaggedInferenceEngineConfig = None, device=None,
@@ -74,9 +81,10 @@ class InferenceEngineV2:
         if not isinstance(model_config, ArchSpec):  # this framework's Llama / Mixtral training configs
             model_config = spec_from_llama_config(model_config)
             weights = convert_own_llama(weights, model_config)
-        cls = RaggedTransformer if model_config.layers is None else HybridTransformer
-        self._model = cls(model_config, weights, device, dtype, tp_group=self._base_mp_group,
-                          latent_mode=self._config.latent_mode, engine_config=self._config)
+        self._model = transformer_class(model_config)(model_config, weights, device, dtype,
+                                                      tp_group=self._base_mp_group,
+                                                      latent_mode=self._config.latent_mode,
+                                                      engine_config=self._config)
         sm = self._config.state_manager
         floats = self._model.state_floats()
         self._states = SequenceStatePool(sm.max_tracked_sequences, floats, device) if floats else None
@@ -335,7 +343,7 @@ def build_hf_engine(path, engine_config=None, debug_level=None, device=None, num
     """Serving engine from a HuggingFace checkpoint directory (config.json + *.safetensors / *.bin).
 
     Supported ``model_type``: llama, mistral, mixtral, qwen, qwen2, qwen2_moe, phi, phi3, falcon, opt
-    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun."""
+    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun, Buvuzen."""
     from .arch import convert_hf, spec_from_hf
     with open(os.path.join(path, "config.json")) as f:
         hf = json.load(f)

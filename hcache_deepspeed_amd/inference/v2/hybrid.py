@@ -1,26 +1,33 @@
-"""Decoder whose layers mix tokens in different ways: recurrent layers beside latent attention, each next to a gated MLP
-that reads the same residual (parallel block, two norms), a causal convolution in front of every sublayer, and
-optionally a run of layers that is passed several times with the same weights.
+"""Decoders whose layers are listed one by one in :class:`arch.ArchSpec` ``layers``: mixers of several kinds, layers that
+run more than once with the same weights (``loop`` / ``order``), a 32-bit residual stream. Served by the same engine,
+paged cache, batch metadata and decode graphs as :class:`model.RaggedTransformer`. Two layer forms:
 
-Driven by :class:`arch.ArchSpec` ``layers`` / ``loop`` / ``input_conv_taps`` and served by the same engine, paged cache,
-batch metadata and decode graphs as :class:`model.RaggedTransformer`. What differs from it:
+* :class:`HybridTransformer` (``norm_place`` "pre"): mixer and gated MLP read the same residual (parallel block, two
+  norms), with a causal convolution in front of every sublayer. A layer is: input norm (residual add + norm +
+  convolutions, one kernel), the mixer and the gated MLP into two column blocks of one matrix, and ONE output projection
+  [W_o | W_down] of that matrix;
+* :class:`PostNormTransformer` ("post"): mixer, then expert layer, each reading the residual itself; the norm is on their
+  outputs. A layer is: mixer and its output projection, norm + residual add (one kernel), router and experts, and one
+  kernel that sums the experts' outputs, norms the sum and adds it.
 
-* the residual stream is 32-bit; a layer is: input norm (residual add + norm + convolutions, one kernel), the mixer and
-  the gated MLP into two column blocks of one matrix, and ONE output projection [W_o | W_down] of that matrix;
-* every layer *run* (a pass of a looped layer counts) has its own paged cache rows and its own part of the sequence's
+Common to both:
+
+* every layer *run* (a pass of a looped or shared layer counts) has its own paged cache rows and its own part of the sequence's
   state row (``ragged.SequenceStatePool``): convolution tails and recurrent states, float32;
 * HCache latents are the attention runs' cached rows themselves, side by side ([1, tokens, sum of row widths]): they
   are already the compressed form. ``restore_kv`` scatters them back; the state row travels with ``evict``.
 """
 import torch
 
-from ...ops.input_norm import norm_rows
-from ...ops.latent_attention import copy_rows
+from ...ops.experts import RouterShape
+from ...ops.output_norm import norm_rows
+from ...ops.paged import copy_rows
 from ...ops.rope import rope_tables
 from .arch import run_order
 from .model import RaggedTransformer, _Layer
-from .modules import (DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig, DSUnembedConfig,
-                      instantiate_gated_mlp, instantiate_input_norm, instantiate_linear, instantiate_mixer,
+from .modules import (DSExpertLayerConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig,
+                      DSNormConfig, DSUnembedConfig, instantiate_expert_layer, instantiate_gated_mlp,
+                      instantiate_input_norm, instantiate_linear, instantiate_mixer, instantiate_output_norm,
                       instantiate_unembed)
 from .modules.implementations import _PackedWeight
 
@@ -33,9 +40,14 @@ class _Run:
         self.layer, self.cache, self.tail, self.state = layer, cache, tail, state
 
 
+# weights kept in the engine's dtype; every other float32 tensor stays float32
+_MATRICES = ("in.w", "up.w", "out.w", "ukv.w", "router.w", "w13", "w2", "ws13", "ws2")
+
+
 class HybridTransformer(RaggedTransformer):
     # kernel sources this class runs on, for builds of just those (ops/build.py)
-    KERNEL_SOURCES = ("act.hip", "gated_scan.hip", "gemv.hip", "input_norm.hip", "latent_attn.hip")
+    KERNEL_SOURCES = ("act.hip", "gated_scan.hip", "gemv.hip", "input_norm.hip", "latent_attn.hip", "output_norm.hip",
+                      "paged_rows.hip")
 
     def __init__(self, spec, weights, device, dtype=torch.bfloat16, tp_group=None, latent_mode="hidden",
                  engine_config=None):
@@ -54,14 +66,23 @@ class HybridTransformer(RaggedTransformer):
     # ------------------------------------------------------------------------------------------
     def _build_modules(self, ec):
         spec, H = self.spec, self.spec.hidden_size
-        self.norm_mod = instantiate_input_norm(
-            DSInputNormConfig(H, "rms", spec.norm_eps, spec.input_conv_taps, self.dtype), ec)
         self.unembed_mod = instantiate_unembed(DSUnembedConfig(model_dim=H, vocab_size=spec.vocab_size,
                                                                norm_type="rms"), ec)
         self.mixers, self.mlps, self.linears = [], [], []
         for e in spec.layers:
             mix = instantiate_mixer(DSMixerConfig(e["mixer"]["type"], H, e["mixer"], spec.norm_eps, self.tp,
                                                   self.dtype), ec)
+            if hasattr(mix, "bind_tables"):
+                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base,
+                                             device=self.device))
+            self.mixers.append(mix)
+        self._build_layers(ec)
+
+    def _build_layers(self, ec):
+        spec, H = self.spec, self.spec.hidden_size
+        self.norm_mod = instantiate_input_norm(
+            DSInputNormConfig(H, "rms", spec.norm_eps, spec.input_conv_taps, self.dtype), ec)
+        for e, mix in zip(spec.layers, self.mixers):
             ff = e["mlp"]["ff"] if e["mlp"] else 0
             assert ff % self.tp == 0, "the feed-forward width must divide the tensor-parallel size"
             ff //= self.tp
@@ -70,10 +91,6 @@ class HybridTransformer(RaggedTransformer):
                     "out.w": instantiate_linear(DSLinearConfig(mix.out_width + ff, H), ec)}
             if mlp is not None:
                 lins["up.w"] = instantiate_linear(DSLinearConfig(H, 2 * ff), ec)
-            if hasattr(mix, "bind_tables"):
-                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base,
-                                             device=self.device))
-            self.mixers.append(mix)
             self.mlps.append((mlp, ff))
             self.linears.append(lins)
 
@@ -102,19 +119,27 @@ class HybridTransformer(RaggedTransformer):
             L = _Layer()
             mw = self.mixers[i].shard(Ls["mix"], self._rows, self._cols)
             o = mw.pop("o.w")
-            for k, v in mw.items():
-                L.w[k] = f(v) if v.dtype == torch.float32 and v.dim() == 1 else t(v)
+            self._put(L, mw)
             for k in ("1", "2"):
                 if Ls.get(f"ln{k}.w") is not None:
                     L.w[f"ln{k}.w"] = f(Ls[f"ln{k}.w"].reshape(-1))
-                    cw = Ls.get(f"conv{k}.w")
-                    L.w[f"conv{k}.w"] = None if cw is None else f(cw.t())  # [taps, W]
-            if self.mlps[i][0] is not None:
-                L.w["up.w"] = t(torch.cat([self._rows(Ls["gate.w"]), self._rows(Ls["up.w"])]))
-                o = torch.cat([o, self._cols(Ls["down.w"])], 1)
-            L.w["out.w"] = t(o)
+            L.w["out.w"] = t(self._load_layer(i, L, Ls, o))
             self._transform(L)
             self.layers.append(L)
+
+    def _put(self, L, weights):
+        for k, v in weights.items():
+            L.w[k] = self._t(v) if v is None or k in _MATRICES or v.dtype != torch.float32 else self._f32(v)
+
+    def _load_layer(self, i, L, Ls, o):
+        """The layer's other weights; returns the output projection (the mixer's ``o`` with what joins it)."""
+        for k in ("1", "2"):
+            cw = Ls.get(f"conv{k}.w")
+            L.w[f"conv{k}.w"] = None if cw is None else self._f32(cw.t())  # [taps, W]
+        if self.mlps[i][0] is None:
+            return o
+        L.w["up.w"] = self._t(torch.cat([self._rows(Ls["gate.w"]), self._rows(Ls["up.w"])]))
+        return torch.cat([o, self._cols(Ls["down.w"])], 1)
 
     def _load_presharded(self, sd):
         t, f = self._t, self._f32
@@ -129,7 +154,7 @@ class HybridTransformer(RaggedTransformer):
                     L.w[k] = _PackedWeight(v["q"].to(self.device), v["scales"].to(self.device),
                                            *[int(i) for i in v["meta"]])
                 else:
-                    L.w[k] = f(v) if v.dtype == torch.float32 and k not in ("in.w", "up.w", "out.w", "ukv.w") else t(v)
+                    self._put(L, {k: v})
             self._transform(L)
             self.layers.append(L)
 
@@ -138,7 +163,7 @@ class HybridTransformer(RaggedTransformer):
         self.row_widths = []
         for li in run_order(self.spec):
             mix = self.mixers[li]
-            tail, off = off, off + self.norm_mod.state_floats()
+            tail, off = off, off + self._norm_state_floats()
             st, off = off, off + mix.state_floats()
             cache = None
             if mix.cache_row:
@@ -147,36 +172,56 @@ class HybridTransformer(RaggedTransformer):
             self.runs.append(_Run(li, cache, tail, st))
         self._state_floats = off
 
+    def _norm_state_floats(self):
+        return self.norm_mod.state_floats()
+
     # ------------------------------------------------------------------------------------------
     def kv_cache_config(self):
         return dict(num_layers=len(self.row_widths), n_kv_heads=1, head_dim=0, row_widths=self.row_widths)
 
     def state_floats(self):
-        return max(1, self._state_floats)
+        return self._state_floats
 
     def save_state(self, batch):
-        return self.state_pool.data.index_select(0, batch.slots.long())
+        return None if self.state_pool is None else self.state_pool.data.index_select(0, batch.slots.long())
 
     def load_state(self, batch, snapshot):
-        self.state_pool.data.index_copy_(0, batch.slots.long(), snapshot)
+        if snapshot is not None:
+            self.state_pool.data.index_copy_(0, batch.slots.long(), snapshot)
 
     def decode_graph_eligible(self, batch, capture_latents):
         return self.dtype == torch.bfloat16 and super().decode_graph_eligible(batch, capture_latents)
 
     # ------------------------------------------------------------------------------------------
-    def _layer(self, run, x, delta, batch):
+    # the residual stream: a pair that _start makes, every layer run maps to the next one, and _final reads
+    def _start(self, batch):
+        return None, None
+
+    def _final(self, stream, idx):
+        """The output norm of rows ``idx``, as the unembedding reads them."""
+        x, delta = stream
+        return norm_rows(x, delta, idx, self.final_w, self.spec.norm_eps)
+
+    def _mix(self, run, x, out, batch):
+        i = run.layer
+        self.mixers[i](x, self.layers[i], self.linears[i]["in.w"], out, batch,
+                       None if run.cache is None else self.kv_cache.get_cache(run.cache), self._state(), run.state)
+
+    def _state(self):
+        return None if self.state_pool is None else self.state_pool.data
+
+    def _layer(self, run, stream, batch):
         """One layer run: (new residual, this layer's output, to be added by whoever reads the residual next)."""
         i = run.layer
+        x, delta = stream
         L, mix, (mlp, ff), lins = self.layers[i], self.mixers[i], self.mlps[i], self.linears[i]
-        state = self.state_pool.data
         gains, convs = [L["ln1.w"]], [L["conv1.w"]]
         if mlp is not None:
             gains.append(L["ln2.w"])
             convs.append(L["conv2.w"])
-        x, ys = self.norm_mod(x, delta, gains, convs, batch, state, run.tail, embed=self.embed)
+        x, ys = self.norm_mod(x, delta, gains, convs, batch, self._state(), run.tail, embed=self.embed)
         mid = torch.empty(batch.current_tokens, mix.out_width + ff, dtype=self.dtype, device=self.device)
-        mix(ys[0], L, lins["in.w"], mid[:, :mix.out_width], batch,
-            None if run.cache is None else self.kv_cache.get_cache(run.cache), state, run.state)
+        self._mix(run, ys[0], mid[:, :mix.out_width], batch)
         if mlp is not None:
             mlp(ys[1], L["up.w"], lins["up.w"], mid[:, mix.out_width:])
         return x, self._allreduce(lins["out.w"](mid, L["out.w"]))
@@ -185,13 +230,12 @@ class HybridTransformer(RaggedTransformer):
     def forward(self, batch, capture_latents=True, sync_latents=True, sink=None):
         """Logits of the wanted rows and the latents ([1, T, W] on the host, or None); see the base class."""
         T = batch.current_tokens
-        x = delta = None
+        stream = self._start(batch)
         for run in self.runs:
-            x, delta = self._layer(run, x, delta, batch)
+            stream = self._layer(run, stream, batch)
         idx = batch.last_token_idx
         if idx.numel():
-            hl = norm_rows(x, delta, idx, self.final_w, self.spec.norm_eps)
-            logits = self.unembed_mod.project(hl, self.lm_head, None, self.tp_group, self.vocab)
+            logits = self.unembed_mod.project(self._final(stream, idx), self.lm_head, None, self.tp_group, self.vocab)
         else:
             logits = torch.empty(0, self.vocab, dtype=self.dtype, device=self.device)
         lat, events = None, []
@@ -230,3 +274,50 @@ class HybridTransformer(RaggedTransformer):
         rows = torch.cat([p[0].to(self.device, non_blocking=True) for p in pieces])
         self._each_cache(lambda c, r: copy_rows(c, r, batch.tok_seq, batch.tok_pos, batch.block_tables,
                                                 to_cache=True), rows)
+
+
+class PostNormTransformer(HybridTransformer):
+    """Layers with the norm on their sublayers' outputs and routed experts: x += n1(mixer(x)), x += n2(experts(x))."""
+    KERNEL_SOURCES = ("act.hip", "experts.hip", "gemv.hip", "grouped_gemm.hip", "output_norm.hip", "paged_attn.hip",
+                      "paged_rows.hip")
+
+    def _build_layers(self, ec):
+        spec, H = self.spec, self.spec.hidden_size
+        self.norm_mod = instantiate_output_norm(DSNormConfig(H, "rms", spec.norm_eps, torch.float32, self.dtype), ec)
+        for e, mix in zip(spec.layers, self.mixers):
+            m = e["mlp"]
+            self.mlps.append(None if m is None else instantiate_expert_layer(
+                DSExpertLayerConfig(H, m["ff"], RouterShape(**m["router"]), m["shared_ff"], self.tp, self.dtype), ec))
+            self.linears.append({"in.w": instantiate_linear(DSLinearConfig(H, mix.in_width), ec),
+                                 "out.w": instantiate_linear(DSLinearConfig(mix.out_width, H), ec)})
+
+    def _load_layer(self, i, L, Ls, o):
+        if self.mlps[i] is not None:
+            self._put(L, self.mlps[i].shard(Ls["experts"], self._rows, self._cols))
+        return o
+
+    def _norm_state_floats(self):
+        return 0
+
+    # the stream: (32-bit residual, the rows a sublayer reads)
+    def _start(self, batch):
+        return self.norm_mod.start(self.embed, batch.input_ids, self.spec.embed_scale)
+
+    def _final(self, stream, idx):
+        if not hasattr(self, "_final_gain"):
+            self._final_gain = self.final_w * self.spec.logit_scale
+        return norm_rows(stream[0], None, idx, self._final_gain, self.spec.norm_eps, self.dtype)
+
+    def _layer(self, run, stream, batch):
+        i = run.layer
+        L, mix, moe = self.layers[i], self.mixers[i], self.mlps[i]
+        x, rows = stream
+        mid = torch.empty(batch.current_tokens, mix.out_width, dtype=self.dtype, device=self.device)
+        self._mix(run, rows[:, :x.shape[1]], mid, batch)
+        x, rows = self.norm_mod(x, self._allreduce(self.linears[i]["out.w"](mid, L["out.w"])), L["ln1.w"])
+        if moe is None:
+            return x, rows
+        parts = moe(rows, L, self.tp_rank)
+        if self.tp > 1:
+            parts = self._allreduce(moe.total(x, parts))
+        return self.norm_mod(x, parts, L["ln2.w"])

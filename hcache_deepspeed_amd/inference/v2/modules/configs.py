@@ -5,6 +5,8 @@ from typing import Optional
 
 import torch
 
+from ....ops.experts import RouterShape
+
 
 @dataclass
 class DSSelfAttentionConfig:
@@ -65,6 +67,16 @@ class DSMixerConfig:
     model_dim: int
     params: dict         # the mixer's sizes and constants
     eps: float = 1e-6    # of norms inside the mixer
+    tp: int = 1
+    input_dtype: torch.dtype = torch.bfloat16
+
+
+@dataclass
+class DSExpertLayerConfig:
+    model_dim: int
+    intermediate_features: int
+    router: "RouterShape"  # ops/experts.py: numbers of experts, identity experts, groups, ...
+    shared_features: int = 0  # 0: no shared expert
     tp: int = 1
     input_dtype: torch.dtype = torch.bfloat16
 

@@ -2,11 +2,11 @@
 :36-195). The engine config's ``quantization.quantization_mode`` picks the weight-only linear ("wf6af16" -> FP6,
 "int8"/"int4" -> group INT); everything else has one MI355X implementation per interface today, chosen here so
 that adding a variant (e.g. an FP8 prefill GEMM) touches only this file and the registry."""
-from .configs import (DSEmbeddingsConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig,
-                      DSMoEConfig, DSNormConfig, DSSelfAttentionConfig, DSUnembedConfig)
-from .interfaces import (DSEmbeddingRegistry, DSGatedMLPRegistry, DSInputNormRegistry, DSLinearRegistry,
-                         DSMixerRegistry, DSMoERegistry, DSPostNormRegistry, DSPreNormRegistry,
-                         DSSelfAttentionRegistry, DSUnembedRegistry)
+from .configs import (DSEmbeddingsConfig, DSExpertLayerConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig,
+                      DSMixerConfig, DSMoEConfig, DSNormConfig, DSSelfAttentionConfig, DSUnembedConfig)
+from .interfaces import (DSEmbeddingRegistry, DSExpertLayerRegistry, DSGatedMLPRegistry, DSInputNormRegistry,
+                         DSLinearRegistry, DSMixerRegistry, DSMoERegistry, DSOutputNormRegistry, DSPostNormRegistry,
+                         DSPreNormRegistry, DSSelfAttentionRegistry, DSUnembedRegistry)
 from .module_registry import ConfigBundle
 from . import implementations  # noqa: F401  (registers the implementations)
 
@@ -66,6 +66,14 @@ def instantiate_mixer(config: DSMixerConfig, engine_config=None):
 
 def instantiate_gated_mlp(config: DSGatedMLPConfig, engine_config=None):
     return DSGatedMLPRegistry.instantiate_config(ConfigBundle("gated_mlp_rows", config))
+
+
+def instantiate_output_norm(config: DSNormConfig, engine_config=None):
+    return DSOutputNormRegistry.instantiate_config(ConfigBundle("rms_residual", config))
+
+
+def instantiate_expert_layer(config: DSExpertLayerConfig, engine_config=None):
+    return DSExpertLayerRegistry.instantiate_config(ConfigBundle("routed_experts", config))
 
 
 def instantiate_unembed(unembed_config: DSUnembedConfig, engine_config=None):

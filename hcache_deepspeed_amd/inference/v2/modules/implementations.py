@@ -14,6 +14,7 @@ import torch.nn.functional as F
 
 from .... import comm as dist
 from ....ops.activations import bias_act, glu, glu_rows
+from ....ops.experts import PAD, routed_experts
 from ....ops.gated_scan import gated_scan, recur_step, recur_step_ok
 from ....ops.gemv import glu_gemv
 from ....ops.grouped_gemm import moe_ffn_dropless
@@ -21,12 +22,15 @@ from ....ops.input_norm import input_norm
 from ....ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
 from ....ops.moe import moe_combine, moe_dispatch, topk_assign, topk_route
 from ....ops.norm import layer_norm, rms_norm
-from ....ops.paged import kv_rope_scatter, paged_attention
+from ....ops.output_norm import embed_rows, padded, residual_norm, sum_experts
+from ....ops.paged import (HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
+                           paged_attention)
 from ....ops.quantizer import fp6_linear, int_linear, quantize, quantize_minifloat
-from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSGatedMLPBase, DSGatedMLPRegistry, DSInputNormBase,
-                         DSInputNormRegistry, DSLinearBase, DSLinearRegistry, DSMixerBase, DSMixerRegistry, DSMoEBase,
-                         DSMoERegistry, DSPostNormBase, DSPostNormRegistry, DSPreNormBase, DSPreNormRegistry,
-                         DSSelfAttentionBase, DSSelfAttentionRegistry, DSUnembedBase, DSUnembedRegistry)
+from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSExpertLayerBase, DSExpertLayerRegistry, DSGatedMLPBase,
+                         DSGatedMLPRegistry, DSInputNormBase, DSInputNormRegistry, DSLinearBase, DSLinearRegistry,
+                         DSMixerBase, DSMixerRegistry, DSMoEBase, DSMoERegistry, DSOutputNormBase, DSOutputNormRegistry,
+                         DSPostNormBase, DSPostNormRegistry, DSPreNormBase, DSPreNormRegistry, DSSelfAttentionBase,
+                         DSSelfAttentionRegistry, DSUnembedBase, DSUnembedRegistry)
 
 _PLAIN_ACTS = ("gelu", "gelu_tanh", "relu", "silu")
 
@@ -405,6 +409,118 @@ class LatentAttentionMixer(DSMixerBase):
         uv = ukv[sh.heads * sh.dim:].view(sh.heads, sh.vdim, sh.rank)
         return latent_attention(lin(x, w["in.w"]), sh, w["dkv.norm"], uk, uv, ukv, self.cos, self.sin, cache, batch,
                                 self._plan(batch), out)
+
+
+@DSMixerRegistry.register_module
+class HeadAttentionMixer(DSMixerBase):
+    """Grouped-query attention without rotation: sliding window, optional query / key norms, sink and output gate
+    (ops/paged.py ``head_attention``). Heads are sharded over the tensor-parallel group."""
+
+    @staticmethod
+    def name():
+        return "attention"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        p, tp = config.params, config.tp
+        if p["heads"] % tp or p["kv_heads"] % tp or p["heads"] % p["kv_heads"]:
+            raise ValueError(f"{p['heads']} / {p['kv_heads']} heads: not groups of equal size on {tp} ranks")
+        self.shape = HeadShape(heads=p["heads"] // tp, kv_heads=p["kv_heads"] // tp, dim=p["dim"], vdim=p["vdim"],
+                               window=p["window"], scale=p["scale"], eps=config.eps, gated=p["gated"])
+        self.out_width = self.shape.heads * p["vdim"]
+        self.in_width = padded(self.shape.width, 8)  # 16-byte rows
+        self.cache_row = self.shape.row
+
+    def shard(self, w, rows, cols):
+        # q, k, v, g and the sink are laid out head by head: equal slices are whole heads
+        parts = [rows(w[k]) for k in (("q", "k", "v", "g") if self.shape.gated else ("q", "k", "v"))]
+        fill = self.in_width - self.shape.width
+        if fill:
+            parts.append(parts[0].new_zeros(fill, parts[0].shape[1]))
+        out = {"in.w": torch.cat(parts), "o.w": cols(w["o"])}
+        for k in ("q.norm", "k.norm"):
+            out[k] = w[k].float() if k in w else None
+        out["sink"] = rows(w["sink"]).float() if "sink" in w else None
+        return out
+
+    def _plan(self, batch):
+        sh = self.shape
+        blocks = batch.max_new > 1 and batch.tok_pos.is_cuda and head_blocks_ok(sh, self._config.input_dtype)
+        key = ("heads", sh.heads, sh.kv_heads, blocks)
+        plan = batch.plans.get(key)
+        if plan is None:
+            plan = batch.plans[key] = make_head_plan(batch.seq_meta_host if blocks else [], batch.current_tokens,
+                                                     sh.heads, sh.kv_heads, blocks, batch.tok_pos.device)
+        return plan
+
+    def forward(self, x, w, lin, out, batch, cache, state, offset):
+        return head_attention(lin(x, w["in.w"]), self.shape, w["q.norm"], w["k.norm"], w["sink"], cache, batch,
+                              self._plan(batch), out)
+
+
+@DSOutputNormRegistry.register_module
+class RmsResidual(DSOutputNormBase):
+    """32-bit residual, RMS norm of what is added to it; bf16 rows come zero-padded to the expert products' tile."""
+
+    @staticmethod
+    def name():
+        return "rms_residual"
+
+    @staticmethod
+    def supports_config(c):
+        return c.type == "rms"
+
+    def _pad(self):
+        return PAD if self._config.input_dtype == torch.bfloat16 else 1
+
+    def start(self, embed, ids, scale):
+        return embed_rows(embed, ids, scale, self._config.input_dtype, self._pad())
+
+    def forward(self, x, delta, gain):
+        return residual_norm(x, delta, gain, self._config.eps, self._config.input_dtype, self._pad())
+
+
+@DSExpertLayerRegistry.register_module
+class RoutedExperts(DSExpertLayerBase):
+    """Group-limited top-k experts with identity experts and a gated shared expert (ops/experts.py). Every expert's
+    feed-forward width is sharded over the tensor-parallel group; bf16 weights are zero-padded to the products' tile."""
+
+    @staticmethod
+    def name():
+        return "routed_experts"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        config.router.check()
+        if config.intermediate_features % config.tp or config.shared_features % config.tp:
+            raise ValueError("the experts' widths must divide the tensor-parallel size")
+
+    def _fit(self, w):
+        """w zero-padded at the end of its last two dimensions."""
+        if self._config.input_dtype != torch.bfloat16:
+            return w
+        add = [padded(n, PAD) - n for n in w.shape[-2:]]
+        return F.pad(w, (0, add[1], 0, add[0])) if any(add) else w
+
+    def _gate_up(self, gate, up, rows):
+        # ``rows`` slices the first dimension
+        gate, up = (rows(t.transpose(0, -2)).transpose(0, -2) for t in (gate, up))
+        return torch.cat([self._fit(gate), self._fit(up)], -2)
+
+    def shard(self, w, rows, cols):
+        fit, shared = self._fit, self._config.shared_features > 0
+        router = torch.cat([w["router"], w["shared.sg"]]) if shared else w["router"]
+        n = router.shape[0]
+        return {"router.w": fit(router)[:n], "router.c": w["correction"].float(),
+                "w13": self._gate_up(w["gate"], w["up"], rows), "w2": fit(cols(w["down"])),
+                "ws13": self._gate_up(w["shared.gate"], w["shared.up"], rows) if shared else None,
+                "ws2": fit(cols(w["shared.down"])) if shared else None}
+
+    def forward(self, x, w, rank=0):
+        return routed_experts(x, w, self._config.router, identity=rank == 0)
+
+    def total(self, x32, parts):
+        return sum_experts(x32, parts, self._config.input_dtype)
 
 
 @DSGatedMLPRegistry.register_module

@@ -48,6 +48,16 @@ class DSMixerBase(DSModuleBase):
         return 0
 
 
+class DSOutputNormBase(DSModuleBase):
+    """forward(x32, delta, gain) -> (x32 + gain * norm(delta), the rows the next sublayer reads); delta: a matrix or the
+    parts an expert layer returns. ``start(embed, ids, scale)`` -> the same pair for the step's tokens."""
+
+
+class DSExpertLayerBase(DSModuleBase):
+    """forward(x, weights, rank) -> the output in parts for DSOutputNormBase; ``shard(weights, rows, cols)`` -> this
+    rank's weights."""
+
+
 class DSGatedMLPBase(DSModuleBase):
     """forward(x [T, in], w [gate; up], lin, out [T, I])."""
 
@@ -75,3 +85,5 @@ DSUnembedRegistry = _registry(DSUnembedBase)
 DSInputNormRegistry = _registry(DSInputNormBase)
 DSMixerRegistry = _registry(DSMixerBase)
 DSGatedMLPRegistry = _registry(DSGatedMLPBase)
+DSOutputNormRegistry = _registry(DSOutputNormBase)
+DSExpertLayerRegistry = _registry(DSExpertLayerBase)

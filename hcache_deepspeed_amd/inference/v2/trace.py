@@ -47,10 +47,10 @@ def _load_needed_kernels(model_dir):
     """Compile (first call of a checkout) only the kernels the model's class runs on."""
     from ...ops import native
     from .arch import spec_from_hf
-    from .hybrid import HybridTransformer
+    from .engine import transformer_class
     with open(os.path.join(model_dir, "config.json")) as f:
         spec = spec_from_hf(json.load(f))
-    native.load_kernels(only=HybridTransformer.KERNEL_SOURCES if spec.layers is not None else None)
+    native.load_kernels(only=getattr(transformer_class(spec), "KERNEL_SOURCES", None))
 
 
 def main(argv=None):

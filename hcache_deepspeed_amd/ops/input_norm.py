@@ -2,11 +2,11 @@
 
 ``input_norm`` adds the previous layer's output to the residual, RMS-norms the row once and writes, for each of up to
 two sublayers k, ``h_k + conv_k(h_k)`` with ``h_k = g_k * norm(x)``; the last ``taps - 1`` normed rows of every
-sequence live in its state slot. ``norm_rows`` is the output norm of selected rows. CPU tensors run the torch
-implementation below."""
+sequence live in its state slot. CPU tensors run the torch implementation below."""
 import torch
 
 from . import native
+from .output_norm import norm_rows  # noqa: F401  (the norm at the other end of the stream)
 
 MAX_TAPS = 16
 
@@ -67,18 +67,3 @@ def input_norm(x, delta, gains, convs, eps, taps, batch, state, offset, dtype, e
                     h += w[j] * full[j:j + n]
             y[q0:q0 + n] = (h * g).to(dtype)
     return x_out, ys
-
-
-def norm_rows(x, delta, idx, gain, eps):
-    """g * norm(x[idx] + delta[idx]) in delta's dtype: [len(idx), W]. idx: int32."""
-    W = x.shape[1]
-    y = torch.empty(idx.numel(), W, dtype=delta.dtype, device=x.device)
-    if native.use_native(x):
-        native.check(
-            native.kernels().hds_norm_rows(native.dt(delta), x.data_ptr(), delta.data_ptr(), idx.data_ptr(),
-                                           gain.data_ptr(), int(gain.numel() > 1), y.data_ptr(), idx.numel(), W,
-                                           float(eps), native.stream()), "norm_rows")
-        return y
-    h = x[idx.long()] + delta[idx.long()].float()
-    y.copy_(h / torch.sqrt((h * h).mean(-1, keepdim=True) + eps) * gain)
-    return y

@@ -12,6 +12,7 @@ import torch
 import torch.nn.functional as F
 
 from . import native
+from .paged import copy_rows
 
 
 @dataclass(frozen=True)
@@ -94,28 +95,6 @@ def make_plan(seq_meta_host, n_tokens, window, expand, device, absorb_max=None):
                       g_dst=views[5])
     plan._keep = host  # pinned source of an asynchronous copy
     return plan
-
-
-def copy_rows(cache, rows, seq, pos, tables, dst_row=None, to_cache=False):
-    """Rows of ``cache`` [blocks, block_size, W] at (seq[i], pos[i]) -> ``rows[dst_row[i] or i]``, or back."""
-    n, W, bs = seq.numel(), cache.shape[2], cache.shape[1]
-    if n == 0:
-        return
-    if native.use_native(cache):
-        assert rows.dtype == cache.dtype and rows.stride(1) == 1 and rows.shape[1] == W
-        native.check(
-            native.kernels().hds_latent_rows(native.dt(cache), int(to_cache), cache.data_ptr(), rows.data_ptr(),
-                                             rows.stride(0), seq.data_ptr(), pos.data_ptr(), native.ptr(dst_row),
-                                             tables.data_ptr(), tables.shape[1], bs, W, n, native.stream()),
-            "latent_rows")
-        return
-    p = pos.long()
-    blk = tables[seq.long(), p // bs].long()
-    dst = torch.arange(n) if dst_row is None else dst_row.long()
-    if to_cache:
-        cache[blk, p % bs] = rows[dst].to(cache.dtype)
-    else:
-        rows[dst] = cache[blk, p % bs].to(rows.dtype)
 
 
 def _rot(v, cos, sin, rdims):

@@ -28,11 +28,21 @@ _KERNEL_SIGS = {
     "hds_glu_bwd": "iippplis",
     "hds_glu_rows": "ii" + "plpl" + "li" + "s",
     "hds_input_norm": "i" + "ppppp" + "pipp" + "pipp" + "p" + "l" + "pp" + "iiiii" + "f" + "s",
+    "hds_residual_norm": "i" + "ppp" + "l" + "pl" + "p" + "ii" + "f" + "s",
+    "hds_experts_norm": "i" + "ppp" + "l" + "pp" + "pl" + "ppp" + "pl" + "pl" + "iiiii" + "f" + "s",
+    "hds_embed_rows": "i" + "pp" + "f" + "pp" + "l" + "iii" + "s",
+    "hds_router_logits": "pl" + "p" + "pl" + "iii" + "s",
+    "hds_router_select": "pl" + "ppp" + "iiiii" + "f" + "s",
+    "hds_expert_sort": "p" + "iii" + "ppp" + "i" + "ppp" + "i" + "s",
+    "hds_experts_skinny_max": "",
+    "hds_experts_skinny": "i" + "pl" + "p" + "pl" + "p" + "iiiii" + "pl" + "p" + "pl" + "iii" + "s",
+    "hds_experts_gemm_f32": "pl" + "p" + "pl" + "ppppp" + "iiii" + "s",
+    "hds_experts_gemm_tile": "iii",
+    "hds_experts_gemm": "pl" + "pi" + "pp" + "i" + "pppp" + "iiiiiii" + "s",
     "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
     "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "pp" + "iii" + "s",
     "hds_gemv_recur_bf16": "ppppp" + "pl" + "pp" + "iii" + "ll" + "s",
     "hds_latent_prep": "i" + "pl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
-    "hds_latent_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
     "hds_latent_decode_mfma_ok": "ii",
     "hds_latent_decode_splits": "iiiiii",
     "hds_latent_decode": "i" + "p" * 8 + "i" * 8 + "f" + "i" + "s",
@@ -65,7 +75,10 @@ _KERNEL_SIGS = {
     "hds_bsattn_fwd": "p" * 8 + "i" * 7 + "f" + "i" + "s",
     "hds_bsattn_bwd": "p" * 15 + "i" * 7 + "f" + "i" + "s",
     "hds_kv_rope_scatter": "i" + "p" + "l" + "pppp" + "i" + "pp" + "i" * 8 + "s",
-    "hds_paged_attn": "p" + "l" + "ppp" + "i" + "pp" + "i" * 5 + "f" + "i" + "s",
+    "hds_head_norm_scatter": "i" + "pl" + "pppppp" + "iiiiiii" + "f" + "s",
+    "hds_paged_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
+    "hds_paged_attn_supported": "ii",
+    "hds_paged_attn": "pl" + "p" + "pl" + "pi" + "pp" + "i" * 6 + "f" + "i" + "pp" + "l" + "s",
     "hds_paged_rows_per_atom": "",
     "hds_moe_dispatch": "i" + "pppp" + "iiii" + "s",
     "hds_moe_dispatch_bwd": "i" + "pppp" + "iiii" + "s",
@@ -112,7 +125,7 @@ _KERNEL_SIGS = {
     "hds_nhwc_bias_add": "i" + "ppppp" + "l" + "ii" + "s",
     "hds_paged_decode_supported": "ii",
     "hds_paged_decode_splits": "iii",
-    "hds_paged_decode": "p" + "l" + "pppp" + "pp" + "iiiiiii" + "f" + "i" + "p" + "s",
+    "hds_paged_decode": "ii" + "pl" + "p" + "pl" + "pp" + "ppppp" + "i" * 8 + "f" + "i" + "pp" + "l" + "p" + "s",
     "hds_copy_d2h": "pp" + "l" + "i" + "s",
     "hds_latent_slot_store": "p" + "l" + "pp" + "l" + "i" + "l" + "s",
     "hds_slot_advance": "p" + "i" + "s",

@@ -1,9 +1,13 @@
-"""Paged-KV serving ops: fused RoPE + KV scatter, ragged paged attention (HIP, csrc/kernels/paged_attn.hip).
+"""Paged-KV serving ops: fused RoPE + KV scatter, ragged paged attention (HIP, csrc/kernels/paged_attn.hip), and
+``head_attention``: attention with normed unrotated heads, a window, a sink and an output gate over the same kernels.
 
 Reference parity: inference/v2/kernels/ragged_ops/linear_blocked_kv_rotary (``LinearBlockedKVCopy``,
 ``BlockedRotaryEmbeddings``) and ragged_ops/blocked_flash (``BlockedFlashAttn``) + atom_builder.
 CPU tensors run torch references (used by the CPU test-suite and as the GPU numerics oracle).
 """
+from dataclasses import dataclass
+from typing import Optional
+
 import torch
 
 from . import native
@@ -106,24 +110,27 @@ def paged_attention(q, cache, atoms, n_atoms, seq_meta, block_tables, n_q, n_kv,
         if not kernel_head_dim_ok(D) or q.dtype != torch.bfloat16:
             raise NotImplementedError(f"paged_attention: head_dim {D} / {q.dtype} has no HIP kernel")
         lib = native.kernels()
-        if decode and lib.hds_paged_decode_supported(D, n_q // n_kv):
+        if decode:
             n_seqs = T
-            splits = lib.hds_paged_decode_splits(n_seqs, n_kv, block_tables.shape[1] * cache.shape[1])
+            keys = block_tables.shape[1] * cache.shape[1]
+            splits = lib.hds_paged_decode_splits(n_seqs, n_kv, min(keys, window) if window else keys)
             part_o = part_ml = None
             if splits > 1:
                 part_o = torch.empty(n_seqs * n_q * splits * D, device=q.device, dtype=torch.float32)
                 part_ml = torch.empty(n_seqs * n_q * splits * 2, device=q.device, dtype=torch.float32)
+            counters = _merge_counters(q.device, n_seqs * n_kv) if splits > 1 and n_q // n_kv <= 8 else None
             native.check(
-                lib.hds_paged_decode(q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(), native.ptr(part_o),
-                                     native.ptr(part_ml), seq_meta.data_ptr(), block_tables.data_ptr(),
-                                     block_tables.shape[1], cache.shape[1], n_seqs, n_q, n_kv, D, splits, float(scale),
-                                     int(window), _merge_counters(q.device, n_seqs * n_kv) if splits > 1 else None,
+                lib.hds_paged_decode(native.dt(q), 0, q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(),
+                                     n_q * D, native.ptr(part_o), native.ptr(part_ml), seq_meta.data_ptr(), None, None,
+                                     None, block_tables.data_ptr(), block_tables.shape[1], cache.shape[1], n_seqs, n_q,
+                                     n_kv, D, D, splits, float(scale), int(window), None, None, 0, counters,
                                      native.stream()), "paged_decode")
             return o
         native.check(
-            lib.hds_paged_attn(q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(), atoms.data_ptr(), n_atoms,
-                               seq_meta.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], cache.shape[1],
-                               n_q, n_kv, D, float(scale), int(window), native.stream()), "paged_attn")
+            lib.hds_paged_attn(q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(), n_q * D, atoms.data_ptr(),
+                               n_atoms, seq_meta.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
+                               cache.shape[1], n_q, n_kv, D, D, float(scale), int(window), None, None, 0,
+                               native.stream()), "paged_attn")
         return o
     meta = seq_meta_host if seq_meta_host is not None else seq_meta.tolist()
     tables = block_tables_host if block_tables_host is not None else block_tables
@@ -148,3 +155,173 @@ def paged_attention(q, cache, atoms, n_atoms, seq_meta, block_tables, n_q, n_kv,
         sc = sc.masked_fill(mask[None], float("-inf"))
         o[q0:q0 + n_new] = torch.einsum("htc,chd->thd", torch.softmax(sc, -1), vv).to(o.dtype)
     return o
+
+
+def copy_rows(cache, rows, seq, pos, tables, dst_row=None, to_cache=False):
+    """Rows of ``cache`` [blocks, block_size, W] at (seq[i], pos[i]) -> ``rows[dst_row[i] or i]``, or back."""
+    n, W, bs = seq.numel(), cache.shape[2], cache.shape[1]
+    if n == 0:
+        return
+    if native.use_native(cache):
+        assert rows.dtype == cache.dtype and rows.stride(1) == 1 and rows.shape[1] == W
+        native.check(
+            native.kernels().hds_paged_rows(native.dt(cache), int(to_cache), cache.data_ptr(), rows.data_ptr(),
+                                            rows.stride(0), seq.data_ptr(), pos.data_ptr(), native.ptr(dst_row),
+                                            tables.data_ptr(), tables.shape[1], bs, W, n, native.stream()),
+            "paged_rows")
+        return
+    p = pos.long()
+    blk = tables[seq.long(), p // bs].long()
+    dst = torch.arange(n) if dst_row is None else dst_row.long()
+    if to_cache:
+        cache[blk, p % bs] = rows[dst].to(cache.dtype)
+    else:
+        rows[dst] = cache[blk, p % bs].to(rows.dtype)
+
+
+# -----------------------------------------------------------------------------------------------------------------
+# normed heads, window, sink, output gate
+# -----------------------------------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class HeadShape:
+    heads: int
+    kv_heads: int
+    dim: int        # of a query / key head
+    vdim: int       # of a value head
+    window: int     # 0: every earlier token
+    scale: float
+    eps: float      # of the query / key norms
+    gated: bool     # the projection ends with one gate column per query head
+
+    @property
+    def row(self):
+        return self.kv_heads * (self.dim + self.vdim)
+
+    @property
+    def qkv_width(self):
+        return self.heads * self.dim + self.row
+
+    @property
+    def width(self):
+        return self.qkv_width + (self.heads if self.gated else 0)
+
+
+# Sequences with at most this many new tokens run token by token on the split-key kernel, the others in row blocks on
+# the matrix cores
+DECODE_MAX = 8
+
+
+@dataclass
+class HeadPlan:
+    """Which tokens of a step run one by one, and the row blocks of the other sequences."""
+    n_dec: int
+    toks: Optional[torch.Tensor] = None   # None: every token, in order
+    n_atoms: int = 0
+    atoms: Optional[torch.Tensor] = None  # [n_atoms, 3] sequence, kv head, first row
+
+
+def make_head_plan(seq_meta_host, n_tokens, heads, kv_heads, blocks, device, decode_max=None):
+    """The plan of one batch for layers with these head counts; one host-to-device copy, shared by the layers.
+    ``blocks`` False: every token runs one by one."""
+    decode_max = DECODE_MAX if decode_max is None else decode_max
+    if not blocks or all(n <= decode_max for (_, n, _) in seq_meta_host):
+        return HeadPlan(n_tokens)
+    toks, atoms, G = [], [], heads // kv_heads
+    for s, (q0, n, _) in enumerate(seq_meta_host):
+        if n <= decode_max:
+            toks += range(q0, q0 + n)
+            continue
+        # the last rows of a portion see the most keys: start them first
+        starts = range(0, n * G, ROWS_PER_ATOM)[::-1]
+        atoms += [(s, hk, r0) for r0 in starts for hk in range(kv_heads)]
+    flat = torch.tensor([v for a in atoms for v in a] + toks, dtype=torch.int32)
+    if device.type == "cuda":
+        flat = flat.pin_memory()
+    dev = flat.to(device, non_blocking=True)
+    k = 3 * len(atoms)
+    plan = HeadPlan(len(toks), dev[k:], len(atoms), dev[:k].view(-1, 3))
+    plan._keep = flat  # pinned source of an asynchronous copy
+    return plan
+
+
+def head_blocks_ok(shape, dtype):
+    """Do the matrix-core and vector kernels take these heads (else the plain kernel)?"""
+    return dtype == torch.bfloat16 and bool(native.kernels().hds_paged_attn_supported(shape.dim, shape.vdim))
+
+
+def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out):
+    """qkv: [T, >= shape.width] projection, row by row q heads | k heads | v heads | gates (consumed). q_norm / k_norm:
+    [dim] float32 or None; sink: [heads] float32 or None; cache: [blocks, block_size, shape.row]. Appends the step's keys
+    and values to ``cache`` and writes the gated heads into ``out`` [T, heads * vdim] (unit column stride)."""
+    sh, T = shape, qkv.shape[0]
+    if not native.use_native(qkv):
+        return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out)
+    lib, st, dt = native.kernels(), native.stream(), native.dt(qkv)
+    bs, tab = cache.shape[1], batch.block_tables
+    mb = tab.shape[1]
+    assert qkv.stride(1) == 1 and out.stride(1) == 1 and cache.dtype == qkv.dtype == out.dtype
+    assert cache.shape[2] == sh.row and qkv.shape[1] >= sh.width and out.shape[1] == sh.heads * sh.vdim
+    native.check(
+        lib.hds_head_norm_scatter(dt, qkv.data_ptr(), qkv.stride(0), native.ptr(q_norm), native.ptr(k_norm),
+                                  cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(),
+                                  T, mb, bs, sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.eps), st),
+        "head_norm_scatter")
+    gate = qkv.data_ptr() + qkv.element_size() * sh.qkv_width if sh.gated else None
+    fast = head_blocks_ok(sh, qkv.dtype) and qkv.stride(0) % 8 == 0 and out.stride(0) % 8 == 0 and \
+        qkv.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0
+    assert fast or not plan.n_atoms
+    if plan.n_dec:
+        n = plan.n_dec
+        keys = min(mb * bs, sh.window) if sh.window else mb * bs
+        splits = lib.hds_paged_decode_splits(n, sh.kv_heads if fast else sh.heads, keys)
+        part_o = part_ml = None
+        if splits > 1:
+            part_o = torch.empty(n * sh.heads * splits * sh.vdim, device=qkv.device, dtype=torch.float32)
+            part_ml = torch.empty(n * sh.heads * splits * 2, device=qkv.device, dtype=torch.float32)
+        native.check(
+            lib.hds_paged_decode(dt, int(not fast), qkv.data_ptr(), qkv.stride(0), cache.data_ptr(), out.data_ptr(),
+                                 out.stride(0), native.ptr(part_o), native.ptr(part_ml), None, native.ptr(plan.toks),
+                                 batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(), mb, bs, n,
+                                 sh.heads, sh.kv_heads, sh.dim, sh.vdim, splits, float(sh.scale), sh.window,
+                                 native.ptr(sink), gate, qkv.stride(0), None, st), "paged_decode")
+    if plan.n_atoms:
+        native.check(
+            lib.hds_paged_attn(qkv.data_ptr(), qkv.stride(0), cache.data_ptr(), out.data_ptr(), out.stride(0),
+                               plan.atoms.data_ptr(), plan.n_atoms, batch.seq_meta.data_ptr(), tab.data_ptr(), mb, bs,
+                               sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, native.ptr(sink),
+                               gate, qkv.stride(0), st), "paged_attn")
+    return out
+
+
+def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out):
+    T, H, G = qkv.shape[0], sh.heads, sh.kv_heads
+
+    def normed(v, w):
+        return v if w is None else v / torch.sqrt((v * v).mean(-1, keepdim=True) + sh.eps) * w
+
+    q, k, v = qkv[:, :sh.qkv_width].float().split([H * sh.dim, G * sh.dim, G * sh.vdim], 1)
+    q = normed(q.reshape(T, H, sh.dim), q_norm)
+    k = normed(k.reshape(T, G, sh.dim), k_norm).reshape(T, -1)
+    copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
+    gate = torch.sigmoid(qkv[:, sh.qkv_width:sh.width].float()) if sh.gated else torch.ones(T, H)
+    bs = cache.shape[1]
+    for s, (q0, n, seen) in enumerate(batch.seq_meta_host):
+        if n == 0:
+            continue
+        lo = max(0, seen - sh.window + 1) if sh.window else 0
+        j = torch.arange(lo, seen + n)
+        rows = cache[batch.block_tables[s, j // bs].long(), j % bs].float()
+        kk = rows[:, :G * sh.dim].view(-1, G, sh.dim).repeat_interleave(H // G, 1)
+        vv = rows[:, G * sh.dim:].reshape(-1, G, sh.vdim).repeat_interleave(H // G, 1)
+        sc = torch.einsum("thd,jhd->htj", q[q0:q0 + n], kk) * sh.scale
+        i = seen + torch.arange(n)
+        hide = j[None] > i[:, None]
+        if sh.window:
+            hide |= j[None] <= i[:, None] - sh.window
+        sc = sc.masked_fill(hide[None], float("-inf"))
+        if sink is not None:
+            sc = torch.cat([sc, sink.view(H, 1, 1).expand(H, n, 1)], -1)
+        p = torch.softmax(sc, -1)[..., :j.numel()]
+        o = torch.einsum("htj,jhd->thd", p, vv) * gate[q0:q0 + n, :, None]
+        out[q0:q0 + n] = o.reshape(n, -1).to(out.dtype)
+    return out
