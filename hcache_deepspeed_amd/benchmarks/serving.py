@@ -1,6 +1,7 @@
 """Prefill and decode throughput of the ragged serving engine on random weights of a real model's layer sizes: the hybrid
-design (Gofasun) next to the dense Llama layout at equal width, depth, feed-forward and head count
-(``bench.py --serving``). One JSON line per measurement."""
+design (Gofasun) next to the dense Llama layout at equal width, depth, feed-forward and head count, and the post-norm
+routed design (Buvuzen) next to the Qwen2-MoE layout at equal width, depth, heads and experts (``bench.py --serving``).
+One JSON line per measurement."""
 import json
 import time
 
@@ -8,6 +9,8 @@ import torch
 
 # name -> (width, ff, heads, kv heads of the dense model)
 SIZES = {"2048": (2048, 5632, 16, 4), "4096": (4096, 14336, 32, 8)}
+# name -> (experts, chosen experts, expert ff, shared expert ff) of the routed models
+EXPERTS = {"2048": (64, 6, 1024, 2048), "4096": (64, 4, 2048, 4096)}
 VOCAB = 32000
 HEAD, ROT, WINDOW = 128, 64, 4096
 
@@ -64,10 +67,62 @@ def gofasun_model(size, layers, dev, kinds=("mingru", "latent_attention")):
     return spec, convert_hf(w, spec)
 
 
+def moe_model(size, layers, dev, max_context):
+    from ..inference.v2.arch import ArchSpec
+    W, _, nq, nkv = SIZES[size]
+    E, top, ff, sh = EXPERTS[size]
+    g = torch.Generator(device=dev).manual_seed(0)
+    spec = ArchSpec("qwen2_moe", VOCAB, W, layers, nq, nkv, HEAD, ff, norm_eps=1e-5, sliding_window=WINDOW,
+                    max_position_embeddings=max_context,
+                    moe=dict(num_experts=E, top_k=top, normalize=False, shared=True, shared_intermediate_size=sh))
+    one = torch.ones(W, device=dev, dtype=torch.bfloat16)
+    lay = [{"ln1.w": one, "ln2.w": one, "qkv.w": _rand(g, dev, (nq + 2 * nkv) * HEAD, W),
+            "o.w": _rand(g, dev, W, nq * HEAD), "router.w": _rand(g, dev, E, W), "w13": _rand(g, dev, E, 2 * ff, W),
+            "w2": _rand(g, dev, E, W, ff), "shared.w13": _rand(g, dev, 2 * sh, W), "shared.w2": _rand(g, dev, W, sh),
+            "shared_gate.w": _rand(g, dev, 1, W)} for _ in range(layers)]
+    return spec, {"embed": _rand(g, dev, VOCAB, W), "final.w": one, "lm_head.w": _rand(g, dev, VOCAB, W),
+                  "layers": lay}
+
+
+def buvuzen_model(size, layers, dev):
+    from ..inference.v2.arch import convert_hf, spec_from_hf
+    W, _, nq, nkv = SIZES[size]
+    E, top, ff, sh = EXPERTS[size]
+    layer = {"type": "attention",
+             "mixer": {"heads": nq, "kv_heads": nkv, "dim": HEAD, "vdim": HEAD, "scale": HEAD**-0.5,
+                       "mask": {"size": WINDOW}},
+             "mlp": {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": sh},
+                     "router": {"experts": E, "identity": 0, "top": top, "groups": {"count": 8, "keep": 4},
+                                "scale": 2.0}}}
+    cfg = {"architecture": "Buvuzen", "vocab": VOCAB, "width": W, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+           "logit_scale": 1.0, "layers": [layer] * layers}
+    g = torch.Generator(device=dev).manual_seed(0)
+    w = {"embed": _rand(g, dev, VOCAB, W), "head": _rand(g, dev, VOCAB, W), "final.norm": torch.zeros(W, device=dev)}
+    for i in range(layers):
+        p = f"l{i}."
+        for k, n in (("norm1", W), ("norm2", W), ("mix.sink", nq), ("mlp.correction", E)):
+            w[p + k] = torch.zeros(n, device=dev)
+        for k in ("mix.q.norm", "mix.k.norm"):
+            w[p + k] = torch.ones(HEAD, device=dev)
+        shapes = {"mix.q": (nq * HEAD, W), "mix.k": (nkv * HEAD, W), "mix.v": (nkv * HEAD, W), "mix.g": (nq, W),
+                  "mix.o": (W, nq * HEAD), "mlp.router": (E, W), "mlp.shared.gate": (sh, W), "mlp.shared.up": (sh, W),
+                  "mlp.shared.down": (W, sh), "mlp.shared.sg": (1, W)}
+        for e in range(E):
+            shapes.update({f"mlp.e{e}.gate": (ff, W), f"mlp.e{e}.up": (ff, W), f"mlp.e{e}.down": (W, ff)})
+        for k, s in shapes.items():
+            w[p + k] = _rand(g, dev, *s)
+    spec = spec_from_hf(cfg)
+    return spec, convert_hf(w, spec)
+
+
 def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
     from ..inference.v2.engine import InferenceEngineV2, RaggedInferenceEngineConfig
     if kind == "llama":
         spec, w = dense_model(size, layers, dev, max_context)
+    elif kind == "qwen2-moe":
+        spec, w = moe_model(size, layers, dev, max_context)
+    elif kind == "buvuzen":
+        spec, w = buvuzen_model(size, layers, dev)
     else:
         kinds = {"gofasun": ("mingru", "latent_attention"), "gofasun-mingru": ("mingru", ),
                  "gofasun-latent": ("latent_attention", )}[kind]
