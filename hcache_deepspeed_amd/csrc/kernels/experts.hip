@@ -18,61 +18,62 @@ using namespace hds;
 // ---------------------------------------------------------------------------------------------------------------
 // router
 // ---------------------------------------------------------------------------------------------------------------
-// logits[T, R] = x[T, K] . w[R, K]^T in 32-bit. A workgroup: 16 router rows x 16 TT tokens, its four waves split K
-// (K % 128 == 0). mfma_f32_16x16x32_bf16 with A = router rows, B = tokens (accumulator column = token).
-template <int TT>
-__global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restrict__ x, int64_t ldx,
+// logits[T, R] = x[T, K] . w[R, K]^T in 32-bit. A workgroup: 16 RT router rows x 16 tokens, its NW waves take every
+// NW-th 32 of K (K % 32 == 0). mfma_f32_16x16x32_bf16 with A = router rows, B = tokens (accumulator column = token).
+// Long steps use a large RT (the tokens are read once for most routers), short ones spread over workgroups.
+template <int RT, int NW>
+__global__ __launch_bounds__(64 * NW) void router_logits_kernel(const bf16* __restrict__ x, int64_t ldx,
                                                             const bf16* __restrict__ w, float* __restrict__ z,
                                                             int64_t ldz, int T, int R, int K) {
-  __shared__ f32x4 red[3][TT][64];
+  __shared__ f32x4 red[NW - 1][RT][64];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  const int r0 = blockIdx.x * 16, t0 = blockIdx.y * 16 * TT;
-  const int kq = K >> 2, kb = wid * kq + 8 * (lane >> 4);
-  const bf16* wp = w + (int64_t)min(r0 + (lane & 15), R - 1) * K + kb;
-  const bf16* xp[TT];
+  const int r0 = blockIdx.x * 16 * RT, t0 = blockIdx.y * 16;
+  const int kb = 8 * (lane >> 4);
+  const bf16* wp[RT];
 #pragma unroll
-  for (int i = 0; i < TT; ++i) xp[i] = x + (int64_t)min(t0 + 16 * i + (lane & 15), T - 1) * ldx + kb;
-  f32x4 acc[TT];
+  for (int i = 0; i < RT; ++i) wp[i] = w + (int64_t)min(r0 + 16 * i + (lane & 15), R - 1) * K + kb;
+  const bf16* xp = x + (int64_t)min(t0 + (lane & 15), T - 1) * ldx + kb;
+  f32x4 acc[RT];
 #pragma unroll
-  for (int i = 0; i < TT; ++i) acc[i] = f32x4{};
-  constexpr int U = TT == 1 ? 8 : 2;
-  int k = 0;
-  for (; k + 32 * U <= kq; k += 32 * U) {
-    bf16x8 a[U], b[U][TT];
+  for (int i = 0; i < RT; ++i) acc[i] = f32x4{};
+  constexpr int U = RT == 1 ? 8 : 4, S = 32 * NW;
+  int k = 32 * wid;
+  for (; k + S * (U - 1) < K; k += S * U) {
+    bf16x8 a[U][RT], b[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      a[u] = *reinterpret_cast<const bf16x8*>(wp + k + 32 * u);
+      b[u] = *reinterpret_cast<const bf16x8*>(xp + k + S * u);
 #pragma unroll
-      for (int i = 0; i < TT; ++i) b[u][i] = *reinterpret_cast<const bf16x8*>(xp[i] + k + 32 * u);
+      for (int i = 0; i < RT; ++i) a[u][i] = *reinterpret_cast<const bf16x8*>(wp[i] + k + S * u);
     }
 #pragma unroll
     for (int u = 0; u < U; ++u)
 #pragma unroll
-      for (int i = 0; i < TT; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u], b[u][i], acc[i], 0, 0, 0);
+      for (int i = 0; i < RT; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u][i], b[u], acc[i], 0, 0, 0);
   }
-  for (; k < kq; k += 32) {
-    const bf16x8 a = *reinterpret_cast<const bf16x8*>(wp + k);
+  for (; k < K; k += S) {
+    const bf16x8 b = *reinterpret_cast<const bf16x8*>(xp + k);
 #pragma unroll
-    for (int i = 0; i < TT; ++i) {
-      const bf16x8 b = *reinterpret_cast<const bf16x8*>(xp[i] + k);
+    for (int i = 0; i < RT; ++i) {
+      const bf16x8 a = *reinterpret_cast<const bf16x8*>(wp[i] + k);
       acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[i], 0, 0, 0);
     }
   }
   if (wid > 0) {
 #pragma unroll
-    for (int i = 0; i < TT; ++i) red[wid - 1][i][lane] = acc[i];
+    for (int i = 0; i < RT; ++i) red[wid - 1][i][lane] = acc[i];
   }
   __syncthreads();
   if (wid > 0) return;
+  const int t = t0 + (lane & 15);
+  if (t >= T) return;
 #pragma unroll
-  for (int i = 0; i < TT; ++i) {
+  for (int i = 0; i < RT; ++i) {
 #pragma unroll
-    for (int v = 0; v < 3; ++v) acc[i] += red[v][i][lane];
-    const int t = t0 + 16 * i + (lane & 15);
-    if (t >= T) continue;
+    for (int v = 0; v < NW - 1; ++v) acc[i] += red[v][i][lane];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int n = r0 + 4 * (lane >> 4) + r;
+      const int n = r0 + 16 * i + 4 * (lane >> 4) + r;
       if (n < R) z[(int64_t)t * ldz + n] = acc[i][r];
     }
   }
@@ -91,7 +92,13 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
   }
 }
 
-// One wave per token; lane l holds entries l + 64 q of the N = experts + identities. groups <= 64.
+// Entry v of lane l (uniform), for every lane
+__device__ __forceinline__ float of_lane(float v, int l) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), l));
+}
+
+// One wave per token; lane l holds entries l + 64 q of the N = experts + identities. groups <= 64. Up to 128 entries every
+// lane ranks its own against all others (readlane, no dependent steps); more are picked one by one.
 template <int Q>
 __global__ __launch_bounds__(256) void router_select_kernel(const float* __restrict__ z, int64_t ldz,
                                                             const float* __restrict__ correction,
@@ -120,6 +127,59 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     const int e = lane + 64 * q;
     s[q] *= inv;
     c[q] = e < N ? s[q] + correction[e] : -INFINITY;
+    if (c[q] != c[q]) c[q] = -3.0e38f;  // rank a NaN last: every choice stays a valid index
+  }
+  if constexpr (Q <= 2) {
+    // how many entries go before entry e: greater ones, and equal ones of a smaller index
+    auto ranks = [&](int (&rank)[Q]) {
+#pragma unroll
+      for (int q = 0; q < Q; ++q) rank[q] = 0;
+#pragma unroll
+      for (int o = 0; o < Q; ++o) {
+        const int nl = min(64, N - 64 * o);
+        for (int l = 0; l < nl; ++l) {
+          const float v = of_lane(c[o], l);
+#pragma unroll
+          for (int q = 0; q < Q; ++q) rank[q] += v > c[q] || (v == c[q] && l + 64 * o < lane + 64 * q);
+        }
+      }
+    };
+    int rank[Q];
+    if (keep < groups) {
+      const int size = N / groups;
+      int group[Q], before[Q];
+      float best[Q];
+#pragma unroll
+      for (int q = 0; q < Q; ++q) {
+        group[q] = (lane + 64 * q) / size;
+        best[q] = -INFINITY;
+        before[q] = 0;
+      }
+      for (int g = 0; g < groups; ++g) {  // group g's largest score: its own entries learn it, all others compare
+        float top_g = -INFINITY;
+        for (int e = g * size; e < (g + 1) * size; ++e) top_g = fmaxf(top_g, of_lane(Q == 2 && e >= 64 ? c[Q - 1] : c[0], e & 63));
+#pragma unroll
+        for (int q = 0; q < Q; ++q)
+          if (group[q] == g) best[q] = top_g;
+      }
+      for (int g = 0; g < groups; ++g) {
+        const int e = g * size;
+        const float top_g = of_lane(Q == 2 && e >= 64 ? best[Q - 1] : best[0], e & 63);
+#pragma unroll
+        for (int q = 0; q < Q; ++q) before[q] += top_g > best[q] || (top_g == best[q] && g < group[q]);
+      }
+#pragma unroll
+      for (int q = 0; q < Q; ++q)
+        if (before[q] >= keep) c[q] = -INFINITY;
+    }
+    ranks(rank);
+#pragma unroll
+    for (int q = 0; q < Q; ++q)
+      if (lane + 64 * q < N && rank[q] < top) {
+        expert[(int64_t)t * top + rank[q]] = lane + 64 * q;
+        weight[(int64_t)t * top + rank[q]] = s[q] * scale;
+      }
+    return;
   }
   if (keep < groups) {
     const int size = N / groups;
@@ -188,9 +248,16 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   count[tid] = 0;
   __syncthreads();
-  for (int a = tid; a < n; a += 1024) {
-    const int e = expert[a];
-    row[a] = e >= 0 && e < E ? atomicAdd(&count[e], 1) : -1;
+  constexpr int U = 8;  // choices of a thread at a time: their loads and counts overlap
+  for (int a0 = tid; a0 < n; a0 += 1024 * U) {
+    int e[U], r[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) e[u] = a0 + 1024 * u < n ? expert[a0 + 1024 * u] : -1;
+#pragma unroll
+    for (int u = 0; u < U; ++u) r[u] = e[u] >= 0 && e[u] < E ? atomicAdd(&count[e[u]], 1) : -1;
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (a0 + 1024 * u < n) row[a0 + 1024 * u] = r[u];
   }
   __syncthreads();
   // exclusive sums of the counts and of the tile counts over the experts (thread = expert)
@@ -231,12 +298,21 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
       }
     }
   }
-  for (int a = tid; a < n; a += 1024) {
-    const int r0 = row[a];
-    if (r0 < 0) continue;
-    const int r = start[expert[a]] + r0;
-    row[a] = r;
-    token[r] = a / k;
+  for (int a0 = tid; a0 < n; a0 += 1024 * U) {
+    int e[U], r[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int a = min(a0 + 1024 * u, n - 1);
+      e[u] = expert[a];
+      r[u] = row[a];  // written by this thread above
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int a = a0 + 1024 * u;
+      if (a >= n || r[u] < 0) continue;
+      row[a] = start[e[u]] + r[u];
+      token[start[e[u]] + r[u]] = a / k;
+    }
   }
 }
 
@@ -429,12 +505,11 @@ HDS_EXPORT int hds_router_logits(const void* x, int64_t ldx, const void* w, floa
                                  hipStream_t st) {
   if (T <= 0) return 0;
   if (R < 1 || K < 128 || K % 128 || ldx % 8 || ldx < K || ldz < R) return hipErrorInvalidValue;
-  if (T >= 512)
-    hipLaunchKernelGGL(router_logits_kernel<4>, dim3((R + 15) / 16, (T + 63) / 64), dim3(256), 0, st, (const bf16*)x,
-                       ldx, (const bf16*)w, z, ldz, T, R, K);
-  else
-    hipLaunchKernelGGL(router_logits_kernel<1>, dim3((R + 15) / 16, (T + 15) / 16), dim3(256), 0, st, (const bf16*)x,
-                       ldx, (const bf16*)w, z, ldz, T, R, K);
+#define HDS_RL(RT, NW)                                                                                               \
+  hipLaunchKernelGGL((router_logits_kernel<RT, NW>), dim3((R + 16 * RT - 1) / (16 * RT), (T + 15) / 16),            \
+                     dim3(64 * NW), 0, st, (const bf16*)x, ldx, (const bf16*)w, z, ldz, T, R, K)
+  if (T >= 512) HDS_RL(5, 8); else if (T > 64) HDS_RL(1, 4); else HDS_RL(1, 16);
+#undef HDS_RL
   return hipGetLastError();
 }
 

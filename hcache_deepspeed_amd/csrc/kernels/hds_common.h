@@ -127,6 +127,24 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// v of another lane by DPP: 0xB1 / 0x4E exchange with the lane 1 / 2 away, 0x141 / 0x140 mirror groups of 8 / 16
+template <int CTRL>
+__device__ __forceinline__ float dpp_f(float v) {
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
+}
+// Sum over aligned groups of N lanes (a power of two up to 64), in every lane
+template <int N>
+__device__ __forceinline__ float group_sum(float v) {
+  if constexpr (N >= 2) v += dpp_f<0xB1>(v);
+  if constexpr (N >= 4) v += dpp_f<0x4E>(v);
+  if constexpr (N >= 8) v += dpp_f<0x141>(v);   // the quads' sums: mirroring 8 lanes swaps them
+  if constexpr (N >= 16) v += dpp_f<0x140>(v);
+  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
 // Block-wide sum for blockDim.x == NT (multiple of 64). `red` must hold NT/64 floats.
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red) {

@@ -52,7 +52,7 @@ __device__ __forceinline__ void load_delta(const ResidualNormParams<T>& p, int t
     const int a = t * p.k + j, e = p.expert[a];
     float v[V];
     if (e < p.E) {
-      VecN<T, V>::load(p.y + (int64_t)(p.row != nullptr ? p.row[a] : a) * p.ldy + c, v);
+      VecN<T, V>::load(p.y + (int64_t)(p.row != nullptr ? max(p.row[a], 0) : a) * p.ldy + c, v);
     } else {
       if (!p.identity) continue;
       VecN<float, V>::load(p.x + (int64_t)t * p.W + c, v);
@@ -70,12 +70,12 @@ __device__ __forceinline__ void load_delta(const ResidualNormParams<T>& p, int t
   }
 }
 
-// RT threads a row (a whole wave or the workgroup), a row of at most NC * V * RT elements in registers
-template <typename T, int V, int NC, int RT>
+// one workgroup a row, the row (at most NC * V * 256 elements) in registers
+template <typename T, int V, int NC>
 __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormParams<T> p) {
   __shared__ float red[4];
-  const int t = blockIdx.x * (256 / RT) + threadIdx.x / RT, i0 = threadIdx.x % RT;
-  if (RT == 64 && t >= p.n) return;  // whole waves; with RT = 256 the grid is exact
+  constexpr int RT = 256;
+  const int t = blockIdx.x, i0 = threadIdx.x;
   float d[NC][V], x[NC][V];
   float ss = 0.f;
 #pragma unroll
@@ -96,8 +96,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormParams<T
     }
     return;
   }
-  ss = RT == 64 ? wave_sum(ss) : block_sum<256>(ss, red);
-  const float rs = 1.f / sqrtf(ss / (float)p.W + p.eps);
+  const float rs = 1.f / sqrtf(block_sum<256>(ss, red) / (float)p.W + p.eps);
 #pragma unroll
   for (int q = 0; q < NC; ++q) {
     const int c = (i0 + q * RT) * V;
@@ -144,14 +143,9 @@ __global__ __launch_bounds__(256) void residual_norm_any_kernel(ResidualNormPara
 template <typename T>
 int launch_residual_norm(const ResidualNormParams<T>& p, hipStream_t st) {
   const bool v8 = p.W % 8 == 0 && p.ldb % 8 == 0 && p.ldd % 8 == 0 && p.ldy % 8 == 0 && p.lds % 8 == 0;
-  // a wave per row once there are enough rows to fill the chip with waves
-#define HDS_RN(NC, RT)                                                                                              \
-  hipLaunchKernelGGL((residual_norm_kernel<T, 8, NC, RT>), dim3((p.n + 256 / RT - 1) / (256 / RT)), dim3(256), 0, st, p)
-  if (v8 && p.n >= 1024 && p.W <= 4096) {
-    if (p.W <= 1024) HDS_RN(2, 64); else if (p.W <= 2048) HDS_RN(4, 64); else HDS_RN(8, 64);
-  } else if (v8 && p.W <= 16384) {
-    if (p.W <= 2048) HDS_RN(1, 256); else if (p.W <= 4096) HDS_RN(2, 256); else if (p.W <= 8192) HDS_RN(4, 256);
-    else HDS_RN(8, 256);
+#define HDS_RN(NC) hipLaunchKernelGGL((residual_norm_kernel<T, 8, NC>), dim3(p.n), dim3(256), 0, st, p)
+  if (v8 && p.W <= 16384) {
+    if (p.W <= 2048) HDS_RN(1); else if (p.W <= 4096) HDS_RN(2); else if (p.W <= 8192) HDS_RN(4); else HDS_RN(8);
   } else {
     const size_t lds = (4 + (size_t)p.W) * sizeof(float);
     if (lds > 64 * 1024) return hipErrorInvalidValue;

@@ -204,6 +204,25 @@ __global__ __launch_bounds__(256) void head_norm_scatter_kernel(HeadNormParams<T
 // ------------------------------------------------------------------------------------------
 // paged attention (ragged prefill + decode)
 // ------------------------------------------------------------------------------------------
+// A sequence's slots: position -> (block, slot) without an integer division per access. The reciprocal is exact for
+// positions below 2^32 / block_size (longer tables divide).
+struct PageTable {
+  const int* table;
+  int size;
+  uint32_t inv;  // 0: divide
+  __device__ __forceinline__ PageTable(const int* t, int block_size, int max_blocks) : table(t), size(block_size) {
+    inv = 0xFFFFFFFFu / (uint32_t)block_size + 1u;  // 0 for blocks of one slot
+    if ((uint64_t)max_blocks * block_size * block_size >> 32) inv = 0;
+  }
+  __device__ __forceinline__ int block(int pos) const {
+    return inv != 0 ? (int)__umulhi((uint32_t)pos, inv) : pos / size;
+  }
+  __device__ __forceinline__ int64_t slot(int pos) const {
+    const int b = block(pos);
+    return (int64_t)table[b] * size + (pos - b * size);
+  }
+};
+
 __device__ __forceinline__ float gate_of(float g) { return 1.f / (1.f + __expf(-g)); }
 
 struct PagedParams {
@@ -227,8 +246,12 @@ struct PagedParams {
 };
 
 // DK / DV: head sizes, or with PAD their upper bounds (tiles zero-padded to them; the sizes are multiples of 8)
+// Two workgroups per CU where their LDS fits
+template <int DK, int DV>
+constexpr int atom_waves() { return Dim<DK>::TILE + Dim<DV>::TILE <= 32768 ? 2 : 1; }
+
 template <int DK, int DV, int NW, bool PAD>
-__global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
+__global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_kernel(PagedParams p) {
   constexpr int KS = Dim<DK>::KS, DT = Dim<DV>::DT, TLK = Dim<DK>::TILE, TLV = Dim<DV>::TILE;
   __shared__ __attribute__((aligned(16))) char smem[2 * TLK + 2 * TLV];  // K[2], V[2]
   const int dk = PAD ? p.dk : DK, dv = PAD ? p.dv : DV;
@@ -383,8 +406,8 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_kernel(PagedParams p) {
 // 8 workgroups for a single Llama-3-8B sequence, each walking the whole context on a mostly empty 128-row MFMA tile
 // (35 us per layer at 540 keys, profiles/r3). Decode is a K/V stream, so this kernel is built like decode_attn.hip:
 // grid (splits, Hkv x blocks of GM query heads, tokens), a workgroup serves its query heads from ONE read of its key
-// range, 16-B loads with LPK lanes per key (8 elements of a key and of a value each), the next keys requested before
-// this iteration's are used, online softmax in registers, lane groups and waves merged by max / rescale, splits merged
+// range, 16-B loads with LPK lanes per key (8 elements of a key and of a value each), U keys per lane group in
+// flight while as many are used (the stream is bound by the bytes in flight), online softmax in registers, lane groups and waves merged by max / rescale, splits merged
 // by a combine kernel through fp32 partials. The key range comes from device-side metadata (and covers only the
 // window), so one launch shape serves every step of a HIP-graph decode.
 constexpr int kDecGMax = 8;
@@ -464,9 +487,19 @@ __device__ __forceinline__ void decode_merge_splits(const PagedDecodeParams<T>& 
   p.o[(int64_t)row * p.so + (int64_t)h * p.dv + d] = from_f<T>(oo * decode_factor(p, row, h, mm, ll));
 }
 
+__device__ __forceinline__ float dot8(const bf16x8& a, const bf16x8& b) {
+  typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+  float c = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    c = __builtin_amdgcn_fdot2_f32_bf16(bf16x2{a[2 * j], a[2 * j + 1]}, bf16x2{b[2 * j], b[2 * j + 1]}, c, false);
+  return c;
+}
+
 template <int LPK, int GM>
 __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf16> p) {
   constexpr int KPW = 64 / LPK;
+  constexpr int U = GM >= 8 ? 2 : 4;  // (registers)
   __shared__ float red[4][GM][2 + 8 * LPK];
   const int G = p.hq / p.hkv, gb = (G + GM - 1) / GM;
   const int split = blockIdx.x, hk = blockIdx.y / gb, g0 = (blockIdx.y % gb) * GM, b = blockIdx.z;
@@ -476,23 +509,19 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
   const DecodeToken tk = decode_token(p, b);
   int j0, j1;
   decode_keys(p, tk.pos, split, j0, j1);
-  const int* table = p.block_tables + (int64_t)tk.seq * p.max_blocks;
+  const PageTable pages(p.block_tables + (int64_t)tk.seq * p.max_blocks, p.block_size, p.max_blocks);
   const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
+  // lanes past a head's size read its start: their q is zero, their value columns are not stored
   const bool k_on = 8 * c < p.dk, v_on = 8 * c < p.dv;
-  const bf16* kbase = p.cache + (int64_t)hk * p.dk + c * 8;
-  const bf16* vbase = p.cache + (int64_t)p.hkv * p.dk + (int64_t)hk * p.dv + c * 8;
+  const bf16* kbase = p.cache + (int64_t)hk * p.dk + (k_on ? c * 8 : 0);
+  const bf16* vbase = p.cache + (int64_t)p.hkv * p.dk + (int64_t)hk * p.dv + (v_on ? c * 8 : 0);
 
-  float qv[GM][8];
+  bf16x8 qv[GM];
 #pragma unroll
   for (int g = 0; g < GM; ++g) {
-    if (g < gn && k_on) {
-      Vec8<bf16>::load(p.q + (int64_t)tk.row * p.sq + (int64_t)(h0 + g) * p.dk + c * 8, qv[g]);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) qv[g][e] *= p.scale;
-    } else {
-#pragma unroll
-      for (int e = 0; e < 8; ++e) qv[g][e] = 0.f;
-    }
+    qv[g] = bf16x8{};
+    if (g < gn && k_on)
+      qv[g] = *reinterpret_cast<const bf16x8*>(p.q + (int64_t)tk.row * p.sq + (int64_t)(h0 + g) * p.dk + c * 8);
   }
   float m[GM], l[GM], acc[GM][8];
 #pragma unroll
@@ -502,37 +531,53 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
 #pragma unroll
     for (int e = 0; e < 8; ++e) acc[g][e] = 0.f;
   }
-  bf16x8 kn = {}, vn = {};
+  bf16x8 kn[U], vn[U];
+  constexpr int STEP = 4 * KPW;  // keys between a lane group's consecutive ones
+  // all block numbers, then all rows: two round trips for U keys. Keys past the end read the last one (weight zero).
   auto fetch = [&](int j) {
-    kn = bf16x8{};
-    vn = bf16x8{};
-    if (j < j1) {
-      const int64_t r = ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * kv_row;
-      if (k_on) kn = *reinterpret_cast<const bf16x8*>(kbase + r);
-      if (v_on) vn = *reinterpret_cast<const bf16x8*>(vbase + r);
+    int64_t r[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) r[u] = pages.slot(min(j + u * STEP, j1 - 1)) * kv_row;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      kn[u] = *reinterpret_cast<const bf16x8*>(kbase + r[u]);
+      vn[u] = *reinterpret_cast<const bf16x8*>(vbase + r[u]);
     }
   };
   int j = j0 + w * KPW + kl;
   fetch(j);
-  for (; j - kl < j1; j += 4 * KPW) {
-    const bool ok = j < j1;
-    const bf16x8 kc = kn, vc = vn;
-    fetch(j + 4 * KPW);
+  for (; j - kl < j1; j += U * STEP) {
+    bf16x8 kc[U], vc[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      kc[u] = kn[u];
+      vc[u] = vn[u];
+    }
+    fetch(j + U * STEP);
 #pragma unroll
     for (int g = 0; g < GM; ++g) {
       if (g >= gn) break;
-      float sc = 0.f;
+      float sc[U];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) sc += qv[g][e] * (float)kc[e];
+      for (int u = 0; u < U; ++u) sc[u] = group_sum<LPK>(dot8(qv[g], kc[u])) * p.scale;
+      float mn = m[g];
 #pragma unroll
-      for (int off = LPK / 2; off >= 1; off >>= 1) sc += __shfl_xor(sc, off, 64);
-      sc = ok ? sc : -INFINITY;
-      const float mn = fmaxf(m[g], sc);
+      for (int u = 0; u < U; ++u) {
+        sc[u] = j + u * STEP < j1 ? sc[u] : -INFINITY;
+        mn = fmaxf(mn, sc[u]);
+      }
       const bool none = mn == -INFINITY;
-      const float a = none ? 1.f : __expf(m[g] - mn), e_s = none ? 0.f : __expf(sc - mn);
-      l[g] = l[g] * a + e_s;
+      const float a = none ? 1.f : __expf(m[g] - mn);
+      l[g] *= a;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[g][e] = acc[g][e] * a + e_s * (float)vc[e];
+      for (int e = 0; e < 8; ++e) acc[g][e] *= a;
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const float e_s = none ? 0.f : __expf(sc[u] - mn);
+        l[g] += e_s;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[g][e] += e_s * (float)vc[u][e];
+      }
       m[g] = mn;
     }
   }
@@ -619,11 +664,9 @@ __global__ __launch_bounds__(256) void paged_plain_kernel(PagedDecodeParams<T> p
   const DecodeToken tk = decode_token(p, b);
   int j0, j1;
   decode_keys(p, tk.pos, split, j0, j1);
-  const int* table = p.block_tables + (int64_t)tk.seq * p.max_blocks;
+  const PageTable pages(p.block_tables + (int64_t)tk.seq * p.max_blocks, p.block_size, p.max_blocks);
   const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
-  auto slot = [&](int j) {
-    return p.cache + ((int64_t)table[j / p.block_size] * p.block_size + j % p.block_size) * kv_row;
-  };
+  auto slot = [&](int j) { return p.cache + pages.slot(j) * kv_row; };
   for (int i = threadIdx.x; i < p.dk; i += 256) sq[i] = to_f(p.q[(int64_t)tk.row * p.sq + (int64_t)h * p.dk + i]);
   for (int i = threadIdx.x; i < p.dv; i += 256) acc[i] = 0.f;
   __syncthreads();
