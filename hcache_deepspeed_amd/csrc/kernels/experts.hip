@@ -136,8 +136,9 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
       for (int q = 0; q < Q; ++q) rank[q] = 0;
 #pragma unroll
       for (int o = 0; o < Q; ++o) {
-        const int nl = min(64, N - 64 * o);
-        for (int l = 0; l < nl; ++l) {
+        // (lanes past the N entries hold -infinity: they come before none of them)
+#pragma unroll 16
+        for (int l = 0; l < 64; ++l) {
           const float v = of_lane(c[o], l);
 #pragma unroll
           for (int q = 0; q < Q; ++q) rank[q] += v > c[q] || (v == c[q] && l + 64 * o < lane + 64 * q);
@@ -157,7 +158,8 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
       }
       for (int g = 0; g < groups; ++g) {  // group g's largest score: its own entries learn it, all others compare
         float top_g = -INFINITY;
-        for (int e = g * size; e < (g + 1) * size; ++e) top_g = fmaxf(top_g, of_lane(Q == 2 && e >= 64 ? c[Q - 1] : c[0], e & 63));
+        for (int e = g * size; e < (g + 1) * size; ++e)
+          top_g = fmaxf(top_g, of_lane(Q == 2 && e >= 64 ? c[Q - 1] : c[0], e & 63));
 #pragma unroll
         for (int q = 0; q < Q; ++q)
           if (group[q] == g) best[q] = top_g;
