@@ -156,16 +156,19 @@ int launch_residual_norm(const ResidualNormParams<T>& p, hipStream_t st) {
 }
 
 // x = embed[id] * scale, and its rounded copy
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const T* __restrict__ embed, const int64_t* __restrict__ ids,
                                                          float scale, float* __restrict__ x, T* __restrict__ xb,
                                                          int64_t ldb, int W, int vocab) {
   const int64_t t = blockIdx.x;
   const int64_t id = min(max(ids[t], (int64_t)0), (int64_t)vocab - 1);
-  for (int c = threadIdx.x; c < W; c += 256) {
-    const float v = to_f(embed[id * W + c]) * scale;
-    x[t * W + c] = v;
-    if (xb != nullptr) xb[t * ldb + c] = from_f<T>(v);
+  for (int c = threadIdx.x * V; c < W; c += 256 * V) {
+    float v[V];
+    VecN<T, V>::load(embed + id * W + c, v);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] *= scale;
+    VecN<float, V>::store(x + t * W + c, v);
+    if (xb != nullptr) VecN<T, V>::store(xb + t * ldb + c, v);
   }
   if (xb != nullptr)
     for (int c = W + threadIdx.x; c < ldb; c += 256) xb[t * ldb + c] = from_f<T>(0.f);
@@ -246,14 +249,18 @@ HDS_EXPORT int hds_embed_rows(int dtype, const void* embed, const int64_t* ids, 
                               int64_t ldb, int n, int W, int vocab, hipStream_t st) {
   if (n <= 0) return 0;
   if (W < 1 || vocab < 1 || (xb != nullptr && ldb < W)) return hipErrorInvalidValue;
-  if (dtype == kBF16)
-    hipLaunchKernelGGL(embed_rows_kernel<bf16>, dim3(n), dim3(256), 0, st, (const bf16*)embed, ids, scale, x, (bf16*)xb,
-                       ldb, W, vocab);
-  else if (dtype == kF32)
-    hipLaunchKernelGGL(embed_rows_kernel<float>, dim3(n), dim3(256), 0, st, (const float*)embed, ids, scale, x,
-                       (float*)xb, ldb, W, vocab);
-  else
+  const bool v8 = W % 8 == 0 && ldb % 8 == 0;
+#define HDS_ER(TT, VV)                                                                                             \
+  hipLaunchKernelGGL((embed_rows_kernel<TT, VV>), dim3(n), dim3(256), 0, st, (const TT*)embed, ids, scale, x,     \
+                     (TT*)xb, ldb, W, vocab)
+  if (dtype == kBF16) {
+    if (v8) HDS_ER(bf16, 8); else HDS_ER(bf16, 1);
+  } else if (dtype == kF32) {
+    if (v8) HDS_ER(float, 8); else HDS_ER(float, 1);
+  } else {
     return hipErrorInvalidValue;
+  }
+#undef HDS_ER
   return hipGetLastError();
 }
 
