@@ -17,7 +17,8 @@ using namespace hds;
 
 namespace {
 
-enum Act : int { kSilu = 0, kGeluTanh = 1, kRelu = 2, kGeluErf = 3, kIdentity = 4 };
+// kClamped: gated units only, g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit) and u' = clamp(u, -limit, limit)
+enum Act : int { kSilu = 0, kGeluTanh = 1, kRelu = 2, kGeluErf = 3, kIdentity = 4, kClamped = 5 };
 
 template <int A>
 __device__ __forceinline__ float act_f(float x) {
@@ -97,10 +98,21 @@ __global__ __launch_bounds__(256) void glu_fwd(const T* __restrict__ gu, T* __re
   }
 }
 
+template <int A>
+__device__ __forceinline__ float gated_f(float g, float u, float limit) {
+  if constexpr (A == kClamped) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __expf(-1.702f * g)) * (u + 1.f);
+  } else {
+    return act_f<A>(g) * u;
+  }
+}
+
 // the same on strided rows of any width (serving: the result goes into a column block of a wider matrix)
 template <typename T, int A, int V>
 __global__ __launch_bounds__(256) void glu_rows(const T* __restrict__ gu, int64_t ld, T* __restrict__ y, int64_t ldo,
-                                                int64_t rows, int I) {
+                                                int64_t rows, int I, float limit) {
   const int vpr = I / V;
   const int64_t total = rows * vpr;
   for (int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * 256) {
@@ -111,10 +123,10 @@ __global__ __launch_bounds__(256) void glu_rows(const T* __restrict__ gu, int64_
       Vec8<T>::load(gu + r * ld + c, g);
       Vec8<T>::load(gu + r * ld + I + c, u);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) o[j] = act_f<A>(g[j]) * u[j];
+      for (int j = 0; j < 8; ++j) o[j] = gated_f<A>(g[j], u[j], limit);
       Vec8<T>::store(y + r * ldo + c, o);
     } else {
-      y[r * ldo + c] = from_f<T>(act_f<A>(to_f(gu[r * ld + c])) * to_f(gu[r * ld + I + c]));
+      y[r * ldo + c] = from_f<T>(gated_f<A>(to_f(gu[r * ld + c]), to_f(gu[r * ld + I + c]), limit));
     }
   }
 }
@@ -410,22 +422,23 @@ HDS_EXPORT int hds_glu_fwd(int dtype, int act, const void* gu, void* y, int64_t 
   return hipGetLastError();
 }
 
-// gu: [rows, ld] with the gate in columns [0, I) and up in [I, 2I); y: [rows, ldo]
+// gu: [rows, ld] with the gate in columns [0, I) and up in [I, 2I); y: [rows, ldo]; limit: of kClamped
 HDS_EXPORT int hds_glu_rows(int dtype, int act, const void* gu, int64_t ld, void* y, int64_t ldo, int64_t rows, int I,
-                            hipStream_t st) {
+                            float limit, hipStream_t st) {
   if (rows <= 0) return 0;
-  if (I < 1 || ld < 2 * (int64_t)I || ldo < I || act < 0 || act > kIdentity) return hipErrorInvalidValue;
+  if (I < 1 || ld < 2 * (int64_t)I || ldo < I || act < 0 || act > kClamped) return hipErrorInvalidValue;
   const bool v8 = I % 8 == 0 && ld % 8 == 0 && ldo % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)y % 16 == 0;
   const dim3 grid(stream_grid(rows * (v8 ? I / 8 : I), 256)), block(256);
 #define HDS_GR(TT, AA)                                                                                            \
   case AA:                                                                                                        \
     if (v8)                                                                                                       \
-      hipLaunchKernelGGL((glu_rows<TT, AA, 8>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I);     \
+      hipLaunchKernelGGL((glu_rows<TT, AA, 8>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I, limit); \
     else                                                                                                          \
-      hipLaunchKernelGGL((glu_rows<TT, AA, 1>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I);     \
+      hipLaunchKernelGGL((glu_rows<TT, AA, 1>), grid, block, 0, st, (const TT*)gu, ld, (TT*)y, ldo, rows, I, limit); \
     break;
 #define HDS_GRA(TT) \
-  switch (act) { HDS_GR(TT, kSilu) HDS_GR(TT, kGeluTanh) HDS_GR(TT, kRelu) HDS_GR(TT, kGeluErf) HDS_GR(TT, kIdentity) }
+  switch (act) { HDS_GR(TT, kSilu) HDS_GR(TT, kGeluTanh) HDS_GR(TT, kRelu) HDS_GR(TT, kGeluErf) HDS_GR(TT, kIdentity) \
+    HDS_GR(TT, kClamped) }
   if (dtype == kBF16) {
     HDS_GRA(bf16)
   } else if (dtype == kF32) {

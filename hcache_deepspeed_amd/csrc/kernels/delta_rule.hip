@@ -1,0 +1,590 @@
+// Gated delta rule of a recurrent mixer over ragged batches. A head h carries a 32-bit state S [dk, dv]; per token
+//
+//   x      = silu(conv(x))                        for the channels of q, k and v: causal, depthwise, `taps` wide
+//   q, k   = q / |q| * dk^(-1/2),  k / |k|        |x| = sqrt(sum(x^2) + 1e-6); query / key head h / (H / G)
+//   beta   = sigmoid(b),  g = exp(-exp(A) * softplus(a + dt))
+//   S      = g S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q
+//   out    = o / sqrt(mean(o^2) + eps) * w * silu(gate)
+//
+// One projection row holds, column block by column block, q [G dk] | k [G dk] | v [H dv] | gate [H dv] | b [H] | a [H].
+// A sequence's slot holds S of all heads and then the convolution's last inputs as a ring: the input of position p is
+// entry p % taps, [taps, C] with C = 2 G dk + H dv. (With taps - 1 of them in use, a step of one token reads other entries
+// than it writes, so the workgroups of heads that share a key head need no order among them.) A sequence whose `seen` is
+// 0 starts from zero whatever the slot holds.
+//
+// Single tokens run one kernel, a workgroup per (sequence, head): delta_step. Portions run delta_conv (convolutions,
+// factors of the unit norms, log decays and betas), a scan over the tokens, and delta_out (norm and gate of the heads).
+#include "hds_common.h"
+
+namespace {
+using namespace hds;
+
+constexpr float kUnitEps = 1e-6f;
+
+__device__ __forceinline__ float sigmoid_f(float x) {
+  const float e = expf(-fabsf(x)), r = 1.f / (1.f + e);
+  return x >= 0.f ? r : e * r;
+}
+__device__ __forceinline__ float silu_f(float x) { return x * sigmoid_f(x); }
+__device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+template <typename T>
+__device__ __forceinline__ float rounded(float x) { return to_f(from_f<T>(x)); }
+
+struct DeltaDims {
+  int H, G, dk, dv, taps;
+  int64_t ld;  // row stride of the projection
+  __device__ __host__ __forceinline__ int k0() const { return G * dk; }
+  __device__ __host__ __forceinline__ int v0() const { return 2 * G * dk; }
+  __device__ __host__ __forceinline__ int C() const { return 2 * G * dk + H * dv; }      // convolved channels
+  __device__ __host__ __forceinline__ int b0() const { return 2 * G * dk + 2 * H * dv; }
+  __device__ __host__ __forceinline__ int64_t states() const { return (int64_t)H * dk * dv; }
+};
+
+template <typename T>
+struct DeltaParams {
+  DeltaDims d;
+  const T* proj;        // [tokens, d.ld]
+  const float* cw;      // [taps, C], the last row is the current token's
+  const float* a_log;   // [H]
+  const float* dt;      // [H]
+  const float* norm;    // [dv]
+  float* state;         // [slots] x slot_stride
+  int64_t slot_stride;
+  const int* slots;
+  const int* seq_meta;  // [sequences][3] = {first row, new tokens, seen}
+  const int* seqs;      // the sequences this launch works on; null: 0, 1, ..
+  T* y;                 // [tokens, C] convolved channels
+  float* rn;            // [tokens, 2 G] factors of q (with dk^(-1/2)) and k
+  float* gb;            // [tokens, H, 2] log decay, beta
+  float* o;             // [tokens, H, dv] read-outs
+  T* out;               // [tokens, ldo]
+  int64_t ldo;
+  int n_tok;
+  float eps;
+};
+
+struct Seq {
+  int q0, n, seen, slot;
+};
+template <typename T>
+__device__ __forceinline__ Seq seq_of(const DeltaParams<T>& p, int i) {
+  const int s = p.seqs != nullptr ? p.seqs[i] : i;
+  return {p.seq_meta[3 * s], p.seq_meta[3 * s + 1], p.seq_meta[3 * s + 2], p.slots[s]};
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// convolutions, unit norms, decays
+// ---------------------------------------------------------------------------------------------------------------
+// heads in channel order: G query heads, G key heads, H value heads
+__device__ __forceinline__ void unit_of(const DeltaDims& d, int u, int& c0, int& width) {
+  width = u < 2 * d.G ? d.dk : d.dv;
+  c0 = u < 2 * d.G ? u * d.dk : d.v0() + (u - 2 * d.G) * d.dv;
+}
+
+template <typename T>
+__device__ __forceinline__ void write_gates(const DeltaParams<T>& p, const Seq& s, int t0, int rows) {
+  for (int i = threadIdx.x; i < rows * p.d.H; i += blockDim.x) {
+    const int t = s.q0 + t0 + i / p.d.H, h = i % p.d.H;
+    const T* row = p.proj + (int64_t)t * p.d.ld + p.d.b0();
+    float* gb = p.gb + 2 * ((int64_t)t * p.d.H + h);
+    gb[0] = -expf(p.a_log[h]) * softplus_f(to_f(row[p.d.H + h]) + p.dt[h]);
+    gb[1] = sigmoid_f(to_f(row[h]));
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ void write_factor(const DeltaParams<T>& p, int t, int u, float ss) {
+  if (u < 2 * p.d.G)
+    p.rn[(int64_t)t * 2 * p.d.G + u] = 1.f / sqrtf(ss + kUnitEps) * (u < p.d.G ? 1.f / sqrtf((float)p.d.dk) : 1.f);
+}
+
+// The workgroup of a sequence's first tokens is the only one that reads the ring (R >= taps - 1) and writes it last.
+// LPU lanes a head, 8 channels each; M >= taps - 1 rows of history in registers (dk, dv, ld, C multiples of 8)
+template <typename T, int LPU, int M>
+__global__ __launch_bounds__(256) void delta_conv8_kernel(DeltaParams<T> p, int R) {
+  const Seq s = seq_of(p, blockIdx.z);
+  const int start = blockIdx.x * R;
+  if (start >= s.n) return;
+  const int rows = min(R, s.n - start), m = p.d.taps - 1;
+  if (blockIdx.y == 0) write_gates(p, s, start, rows);
+  const int u = blockIdx.y * (256 / LPU) + threadIdx.x / LPU;
+  const bool live = u < 2 * p.d.G + p.d.H;
+  int c0, width;
+  unit_of(p.d, live ? u : 0, c0, width);
+  const int e = 8 * (threadIdx.x % LPU);
+  const bool ok = live && e < width;
+  const int c = c0 + (ok ? e : 0);
+  float* ring = p.state + (int64_t)s.slot * p.slot_stride + p.d.states() + c;
+  const T* in = p.proj + (int64_t)s.q0 * p.d.ld + c;
+  const int C = p.d.C();
+  float w[M + 1][8], hist[M + 1][8];  // [k]: k + 1 back for hist, k back for w
+#pragma unroll
+  for (int k = 0; k <= M; ++k) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) w[k][i] = hist[k][i] = 0.f;
+    if (k <= m) Vec8<float>::load(p.cw + (int64_t)(m - k) * C + c, w[k]);
+    if (k < m) {
+      const int i0 = start - 1 - k, pos = s.seen + i0;
+      if (i0 >= 0) Vec8<T>::load(in + (int64_t)i0 * p.d.ld, hist[k]);
+      else if (pos >= 0) Vec8<float>::load(ring + (int64_t)(pos % p.d.taps) * C, hist[k]);
+    }
+  }
+  float x[8];
+  Vec8<T>::load(in + (int64_t)start * p.d.ld, x);
+  for (int r = 0; r < rows; ++r) {
+    float nx[8];
+    if (r + 1 < rows) Vec8<T>::load(in + (int64_t)(start + r + 1) * p.d.ld, nx);
+    float y[8], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      float a = w[0][i] * x[i];
+#pragma unroll
+      for (int k = 0; k < M; ++k) a += w[k + 1][i] * hist[k][i];
+      y[i] = rounded<T>(silu_f(rounded<T>(a)));
+      ss += ok ? y[i] * y[i] : 0.f;
+    }
+    const int t = s.q0 + start + r;
+    if (ok) Vec8<T>::store(p.y + (int64_t)t * C + c, y);
+    ss = group_sum<LPU>(ss);
+    if (ok && e == 0) write_factor(p, t, u, ss);
+#pragma unroll
+    for (int k = M - 1; k > 0; --k)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) hist[k][i] = hist[k - 1][i];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      hist[0][i] = x[i];
+      if (r + 1 < rows) x[i] = nx[i];
+    }
+  }
+  if (blockIdx.x == 0 && ok)
+    for (int i0 = max(s.n - m, 0); i0 < s.n; ++i0) {
+      float v[8];
+      Vec8<T>::load(in + (int64_t)i0 * p.d.ld, v);
+      Vec8<float>::store(ring + (int64_t)((s.seen + i0) % p.d.taps) * C, v);
+    }
+}
+
+// any sizes: one wave a head
+template <typename T>
+__global__ __launch_bounds__(256) void delta_conv_kernel(DeltaParams<T> p, int R) {
+  const Seq s = seq_of(p, blockIdx.z);
+  const int start = blockIdx.x * R;
+  if (start >= s.n) return;
+  const int rows = min(R, s.n - start), m = p.d.taps - 1;
+  if (blockIdx.y == 0) write_gates(p, s, start, rows);
+  const int u = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (u >= 2 * p.d.G + p.d.H) return;
+  int c0, width;
+  unit_of(p.d, u, c0, width);
+  float* ring = p.state + (int64_t)s.slot * p.slot_stride + p.d.states();
+  const T* in = p.proj + (int64_t)s.q0 * p.d.ld;
+  const int C = p.d.C();
+  for (int r = 0; r < rows; ++r) {
+    float ss = 0.f;
+    for (int c = c0 + lane; c < c0 + width; c += 64) {
+      float a = 0.f;
+      for (int k = 0; k <= m; ++k) {
+        const int i0 = start + r - k, pos = s.seen + i0;
+        if (pos < 0) break;
+        const float v = i0 >= 0 ? to_f(in[(int64_t)i0 * p.d.ld + c]) : ring[(int64_t)(pos % p.d.taps) * C + c];
+        a += p.cw[(int64_t)(m - k) * C + c] * v;
+      }
+      const float y = rounded<T>(silu_f(rounded<T>(a)));
+      p.y[(int64_t)(s.q0 + start + r) * C + c] = from_f<T>(y);
+      ss += y * y;
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) write_factor(p, s.q0 + start + r, u, ss);
+  }
+  if (blockIdx.x == 0)
+    for (int c = c0 + lane; c < c0 + width; c += 64)
+      for (int i0 = max(s.n - m, 0); i0 < s.n; ++i0)
+        ring[(int64_t)((s.seen + i0) % p.d.taps) * C + c] = to_f(in[(int64_t)i0 * p.d.ld + c]);
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// scan, token by token: a workgroup per 64 columns of one head's state, R rows of it in each wave's registers
+// ---------------------------------------------------------------------------------------------------------------
+constexpr int kScanTok = 8;  // tokens staged at a time
+
+template <typename T, int R>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams<T> p) {
+  __shared__ float sq[2][kScanTok][4 * R], sk[2][kScanTok][4 * R];
+  __shared__ float part[2][4][2][64];
+  __shared__ float sg[2][kScanTok][3];  // decay, beta, k . q
+  const Seq s = seq_of(p, blockIdx.z);
+  if (s.n <= 0) return;
+  const int h = blockIdx.y, hk = h / (p.d.H / p.d.G);
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int col = blockIdx.x * 64 + lane, dk = p.d.dk, dv = p.d.dv, C = p.d.C();
+  const bool ok = col < dv;
+  const int cc = ok ? col : dv - 1;
+  float* st = p.state + (int64_t)s.slot * p.slot_stride + (int64_t)h * dk * dv + cc;
+  float S[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int row = w * R + r;
+    S[r] = s.seen > 0 && row < dk ? st[(int64_t)row * dv] : 0.f;
+  }
+  // unit vectors of kScanTok tokens; wave w prepares tokens w, w + 4, ..
+  auto stage = [&](int buf, int t0) {
+    for (int i = w; i < kScanTok; i += 4) {
+      if (t0 + i >= s.n) break;
+      const int64_t t = s.q0 + t0 + i;
+      const T* y = p.y + t * C;
+      const float rq = p.rn[t * 2 * p.d.G + hk], rk = p.rn[t * 2 * p.d.G + p.d.G + hk];
+      float kq = 0.f;
+      for (int e = lane; e < 4 * R; e += 64) {
+        const float q = e < dk ? to_f(y[hk * dk + e]) * rq : 0.f;
+        const float k = e < dk ? to_f(y[p.d.k0() + hk * dk + e]) * rk : 0.f;
+        sq[buf][i][e] = q;
+        sk[buf][i][e] = k;
+        kq += k * q;
+      }
+      kq = wave_sum(kq);
+      if (lane == 0) {
+        sg[buf][i][0] = expf(p.gb[2 * (t * p.d.H + h)]);
+        sg[buf][i][1] = p.gb[2 * (t * p.d.H + h) + 1];
+        sg[buf][i][2] = kq;
+      }
+    }
+  };
+  stage(0, 0);
+  __syncthreads();
+  for (int t0 = 0; t0 < s.n; t0 += kScanTok) {
+    const int buf = (t0 / kScanTok) & 1, nt = min(kScanTok, s.n - t0);
+    if (t0 + kScanTok < s.n) stage(buf ^ 1, t0 + kScanTok);
+    float vn = to_f(p.y[(int64_t)(s.q0 + t0) * C + p.d.v0() + h * dv + cc]);
+    for (int i = 0; i < nt; ++i) {
+      const float v = vn;
+      if (i + 1 < nt) vn = to_f(p.y[(int64_t)(s.q0 + t0 + i + 1) * C + p.d.v0() + h * dv + cc]);
+      float ks = 0.f, qs = 0.f;
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        ks += S[r] * sk[buf][i][w * R + r];
+        qs += S[r] * sq[buf][i][w * R + r];
+      }
+      const int pb = (t0 + i) & 1;
+      part[pb][w][0][lane] = ks;
+      part[pb][w][1][lane] = qs;
+      __syncthreads();  // one a token: the other part buffer is written next
+      ks = part[pb][0][0][lane] + part[pb][1][0][lane] + part[pb][2][0][lane] + part[pb][3][0][lane];
+      qs = part[pb][0][1][lane] + part[pb][1][1][lane] + part[pb][2][1][lane] + part[pb][3][1][lane];
+      const float g = sg[buf][i][0], u = sg[buf][i][1] * (v - g * ks);
+#pragma unroll
+      for (int r = 0; r < R; ++r) S[r] = g * S[r] + sk[buf][i][w * R + r] * u;
+      if (w == 0 && ok) p.o[((int64_t)(s.q0 + t0 + i) * p.d.H + h) * dv + col] = g * qs + sg[buf][i][2] * u;
+    }
+    __syncthreads();
+  }
+  if (ok)
+#pragma unroll
+    for (int r = 0; r < R; ++r)
+      if (w * R + r < dk) st[(int64_t)(w * R + r) * dv] = S[r];
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// norm and gate of the heads
+// ---------------------------------------------------------------------------------------------------------------
+template <typename T>
+__device__ __forceinline__ bool out_item(const DeltaParams<T>& p, int64_t item, int R, int& t, int& h) {
+  const Seq s = seq_of(p, blockIdx.z);
+  const int start = blockIdx.x * R;
+  const int i = start + (int)(item / p.d.H);
+  h = (int)(item % p.d.H);
+  t = s.q0 + i;
+  return i < min(s.n, start + R);
+}
+
+// LPU lanes a head, 8 values each; a workgroup takes R tokens
+template <typename T, int LPU>
+__global__ __launch_bounds__(256) void delta_out8_kernel(DeltaParams<T> p, int R) {
+  const int e = 8 * (threadIdx.x % LPU), dv = p.d.dv;
+  if (blockIdx.x * R >= seq_of(p, blockIdx.z).n) return;
+  float nw[8];
+  if (e < dv) Vec8<float>::load(p.norm + e, nw);
+  for (int64_t item = threadIdx.x / LPU; item < (int64_t)R * p.d.H; item += 256 / LPU) {
+    int t, h;
+    const bool ok = out_item(p, item, R, t, h) && e < dv;
+    float o[8], g[8], ss = 0.f;
+    if (ok) {
+      Vec8<float>::load(p.o + ((int64_t)t * p.d.H + h) * dv + e, o);
+      Vec8<T>::load(p.proj + (int64_t)t * p.d.ld + p.d.C() + h * dv + e, g);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += o[i] * o[i];
+    }
+    ss = group_sum<LPU>(ss);
+    if (!ok) continue;
+    const float rs = 1.f / sqrtf(ss / (float)dv + p.eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] *= rs * nw[i] * silu_f(g[i]);
+    Vec8<T>::store(p.out + (int64_t)t * p.ldo + h * dv + e, o);
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams<T> p, int R) {
+  const int lane = threadIdx.x & 63, dv = p.d.dv;
+  for (int64_t item = threadIdx.x >> 6; item < (int64_t)R * p.d.H; item += 4) {
+    int t, h;
+    if (!out_item(p, item, R, t, h)) break;
+    const float* o = p.o + ((int64_t)t * p.d.H + h) * dv;
+    const T* g = p.proj + (int64_t)t * p.d.ld + p.d.C() + h * dv;
+    float ss = 0.f;
+    for (int e = lane; e < dv; e += 64) ss += o[e] * o[e];
+    const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dv + p.eps);
+    for (int e = lane; e < dv; e += 64)
+      p.out[(int64_t)t * p.ldo + h * dv + e] = from_f<T>(o[e] * rs * p.norm[e] * silu_f(to_f(g[e])));
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// one token per sequence: everything from the projection to the gated output in a workgroup per (head, sequence)
+// ---------------------------------------------------------------------------------------------------------------
+// A thread keeps 4 columns of RPT rows of S. S^T k and S^T q come from one pass over the old state:
+// o = g S^T q + (k . q) u.
+template <typename T, int RPT, int NT>
+__global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
+  constexpr int NW = NT / 64;
+  extern __shared__ float sm[];
+  const DeltaDims& d = p.d;
+  const int dk = d.dk, dv = d.dv, C = d.C(), cq = dv / 4;
+  const int RG = NT / cq;                     // row groups
+  const bool fold = (cq & (cq - 1)) == 0 && cq <= 64;  // the row groups of a wave reduce by lane exchange
+  const int P = fold ? NW : RG;
+  float* part = sm;                           // [P][2][dv]
+  float* su = part + 2 * P * dv;              // [dv]
+  float* so = su + dv;                        // [dv]
+  float* sq = so + dv;                        // [dk], then k [dk] and v [dv]
+  float* sk = sq + dk;
+  float* sv = sk + dk;
+  const int h = blockIdx.x, hk = h / (d.H / d.G);
+  const Seq s = seq_of(p, blockIdx.y);
+  if (s.n != 1) return;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int c4 = threadIdx.x % cq, rg = threadIdx.x / cq;
+  const bool act = rg < RG;
+  float* st = p.state + (int64_t)s.slot * p.slot_stride;
+  float* Sp = st + ((int64_t)h * dk) * dv + 4 * c4;
+  f32x4 S[RPT];
+#pragma unroll
+  for (int r = 0; r < RPT; ++r) {
+    S[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int row = rg + r * RG;
+    if (act && s.seen > 0 && row < dk) S[r] = *reinterpret_cast<const f32x4*>(Sp + (int64_t)row * dv);
+  }
+  const T* row = p.proj + (int64_t)s.q0 * d.ld;
+  const float beta = sigmoid_f(to_f(row[d.b0() + h]));
+  const float g = expf(-expf(p.a_log[h]) * softplus_f(to_f(row[d.b0() + d.H + h]) + p.dt[h]));
+  // convolutions of this head's channels
+  float* ring = st + d.states();
+  for (int i = threadIdx.x; i < 2 * dk + dv; i += NT) {
+    const int c = i < dk ? hk * dk + i : (i < 2 * dk ? d.k0() + hk * dk + i - dk : d.v0() + h * dv + i - 2 * dk);
+    const float x = to_f(row[c]);
+    float a = p.cw[(int64_t)(d.taps - 1) * C + c] * x;
+    for (int k = 1; k < d.taps; ++k)
+      if (s.seen - k >= 0) a += p.cw[(int64_t)(d.taps - 1 - k) * C + c] * ring[(int64_t)((s.seen - k) % d.taps) * C + c];
+    sq[i] = rounded<T>(silu_f(rounded<T>(a)));
+    if (i >= 2 * dk || h % (d.H / d.G) == 0) ring[(int64_t)(s.seen % d.taps) * C + c] = x;
+  }
+  __syncthreads();
+  float qq = 0.f, kk = 0.f, kq = 0.f;
+  for (int e = lane; e < dk; e += 64) {
+    qq += sq[e] * sq[e];
+    kk += sk[e] * sk[e];
+    kq += sk[e] * sq[e];
+  }
+  const float rq = 1.f / sqrtf(wave_sum(qq) + kUnitEps) / sqrtf((float)dk), rk = 1.f / sqrtf(wave_sum(kk) + kUnitEps);
+  kq = wave_sum(kq) * rq * rk;
+  f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < RPT; ++r) {
+    const int e = rg + r * RG;
+    if (act && e < dk) {
+      ks += S[r] * sk[e];
+      qs += S[r] * sq[e];
+    }
+  }
+  if (fold) {
+    for (int off = cq; off < 64; off <<= 1)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        ks[i] += __shfl_xor(ks[i], off, 64);
+        qs[i] += __shfl_xor(qs[i], off, 64);
+      }
+    if (lane < cq) {
+      *reinterpret_cast<f32x4*>(part + (2 * w) * dv + 4 * c4) = ks;
+      *reinterpret_cast<f32x4*>(part + (2 * w + 1) * dv + 4 * c4) = qs;
+    }
+  } else if (act) {
+    *reinterpret_cast<f32x4*>(part + (2 * rg) * dv + 4 * c4) = ks;
+    *reinterpret_cast<f32x4*>(part + (2 * rg + 1) * dv + 4 * c4) = qs;
+  }
+  __syncthreads();
+  for (int c = threadIdx.x; c < dv; c += NT) {
+    float a = 0.f, b = 0.f;
+    for (int i = 0; i < P; ++i) {
+      a += part[(2 * i) * dv + c];
+      b += part[(2 * i + 1) * dv + c];
+    }
+    const float u = beta * (sv[c] - g * rk * a);
+    su[c] = u;
+    so[c] = g * rq * b + kq * u;
+  }
+  __syncthreads();
+  if (act) {
+    const f32x4 u = *reinterpret_cast<const f32x4*>(su + 4 * c4);
+#pragma unroll
+    for (int r = 0; r < RPT; ++r) {
+      const int e = rg + r * RG;
+      if (e < dk) *reinterpret_cast<f32x4*>(Sp + (int64_t)e * dv) = g * S[r] + (rk * sk[e]) * u;
+    }
+  }
+  if (w * 64 < dv) {
+    float ss = 0.f;
+    for (int c = lane; c < dv; c += 64) ss += so[c] * so[c];
+    const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dv + p.eps);
+    for (int c = threadIdx.x; c < dv; c += NT)
+      p.out[(int64_t)s.q0 * p.ldo + h * dv + c] =
+          from_f<T>(so[c] * rs * p.norm[c] * silu_f(to_f(row[C + h * dv + c])));
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+template <typename T>
+int launch_conv(const DeltaParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
+  const DeltaDims& d = p.d;
+  int R = max_new > 1024 ? 32 : 16;
+  if (R < d.taps - 1) R = d.taps - 1;
+  const int units = 2 * d.G + d.H, w = d.dk > d.dv ? d.dk : d.dv;
+  const int blocks = (max_new + R - 1) / R;
+  if (d.dk % 8 || d.dv % 8 || d.ld % 8 || d.taps > 8 || w > 512 || p.slot_stride % 4 || (uintptr_t)p.state % 16 ||
+      (uintptr_t)p.proj % 16 || d.states() % 4) {
+    hipLaunchKernelGGL(delta_conv_kernel<T>, dim3(blocks, (units + 3) / 4, n_seqs), dim3(256), 0, st, p, R);
+    return hipGetLastError();
+  }
+#define HDS_DC(L, MM)                                                                                              \
+  hipLaunchKernelGGL((delta_conv8_kernel<T, L, MM>), dim3(blocks, (units + 256 / L - 1) / (256 / L), n_seqs),     \
+                     dim3(256), 0, st, p, R)
+#define HDS_DCM(L) { if (d.taps <= 4) HDS_DC(L, 3); else HDS_DC(L, 7); }
+  if (w <= 64) HDS_DCM(8) else if (w <= 128) HDS_DCM(16) else if (w <= 256) HDS_DCM(32) else HDS_DCM(64)
+#undef HDS_DCM
+#undef HDS_DC
+  return hipGetLastError();
+}
+
+template <typename T>
+int launch_out(const DeltaParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
+  const int dv = p.d.dv, R = 4;
+  const dim3 grid((max_new + R - 1) / R, 1, n_seqs);
+  if (dv % 8 || dv > 512 || p.d.ld % 8 || p.d.C() % 8 || p.ldo % 8 || (uintptr_t)p.out % 16 || (uintptr_t)p.proj % 16) {
+    hipLaunchKernelGGL(delta_out_kernel<T>, grid, dim3(256), 0, st, p, R);
+    return hipGetLastError();
+  }
+#define HDS_DO(L) hipLaunchKernelGGL((delta_out8_kernel<T, L>), grid, dim3(256), 0, st, p, R)
+  if (dv <= 64) HDS_DO(8); else if (dv <= 128) HDS_DO(16); else if (dv <= 256) HDS_DO(32); else HDS_DO(64);
+#undef HDS_DO
+  return hipGetLastError();
+}
+
+template <typename T>
+int launch_scan(const DeltaParams<T>& p, int n_seqs, hipStream_t st) {
+  const dim3 grid((p.d.dv + 63) / 64, p.d.H, n_seqs);
+#define HDS_DS(RR) hipLaunchKernelGGL((delta_scan_kernel<T, RR>), grid, dim3(256), 0, st, p)
+  const int dk = p.d.dk;
+  if (dk <= 32) HDS_DS(8); else if (dk <= 64) HDS_DS(16); else if (dk <= 128) HDS_DS(32); else if (dk <= 256) HDS_DS(64);
+  else HDS_DS(128);
+#undef HDS_DS
+  return hipGetLastError();
+}
+
+// threads and rows a thread of delta_step; 0: the kernel does not take these sizes
+int step_shape(int dk, int dv, int& nt) {
+  if (dv % 4 || dv > 1024) return 0;
+  nt = (int64_t)dk * dv <= 4096 ? 256 : 1024;
+  if (dv / 4 > nt) nt = 1024;
+  const int rg = nt / (dv / 4), rows = (dk + rg - 1) / rg;
+  return rows <= 16 ? rows : 0;
+}
+size_t step_lds(int dk, int dv, int nt) {
+  const int cq = dv / 4, rg = nt / cq;
+  const bool fold = (cq & (cq - 1)) == 0 && cq <= 64;
+  return sizeof(float) * (2 * (size_t)dk + 3 * dv + 2 * (size_t)(fold ? nt / 64 : rg) * dv);
+}
+
+template <typename T>
+int launch_step(const DeltaParams<T>& p, int n_seqs, hipStream_t st) {
+  int nt = 0;
+  const int rows = step_shape(p.d.dk, p.d.dv, nt);
+  const size_t lds = rows ? step_lds(p.d.dk, p.d.dv, nt) : 0;
+  if (rows == 0 || lds > 64 * 1024 || p.slot_stride % 4 || (uintptr_t)p.state % 16) return hipErrorInvalidValue;
+#define HDS_DT(RR, NN) hipLaunchKernelGGL((delta_step_kernel<T, RR, NN>), dim3(p.d.H, n_seqs), dim3(NN), lds, st, p)
+#define HDS_DTN(NN)                                                                                      \
+  {                                                                                                      \
+    if (rows <= 1) HDS_DT(1, NN); else if (rows <= 2) HDS_DT(2, NN); else if (rows <= 4) HDS_DT(4, NN); \
+    else if (rows <= 8) HDS_DT(8, NN); else HDS_DT(16, NN);                                              \
+  }
+  if (nt == 256) HDS_DTN(256) else HDS_DTN(1024)
+#undef HDS_DTN
+#undef HDS_DT
+  return hipGetLastError();
+}
+
+bool dims_ok(const DeltaDims& d) {
+  return d.H >= 1 && d.G >= 1 && d.H % d.G == 0 && d.dk >= 1 && d.dk <= 512 && d.dv >= 1 && d.taps >= 1 &&
+         d.taps <= 256 && d.H <= 65535 && d.ld >= (int64_t)d.b0() + 2 * d.H;
+}
+
+}  // namespace
+
+// heads of these sizes run delta_step (else single tokens run like portions)
+HDS_EXPORT int hds_delta_step_ok(int dk, int dv) {
+  int nt = 0;
+  return dk >= 1 && dv >= 1 && step_shape(dk, dv, nt) > 0 && step_lds(dk, dv, nt) <= 64 * 1024;
+}
+
+// the sequences' one new token each
+HDS_EXPORT int hds_delta_step(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
+                              const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
+                              const int* seq_meta, const int* seqs, void* out, int64_t ldo, int n_seqs, int H, int G,
+                              int dk, int dv, int taps, float eps, hipStream_t st) {
+  if (n_seqs <= 0) return 0;
+  const DeltaDims d{H, G, dk, dv, taps, ld};
+  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || ldo < (int64_t)H * dv ||
+      slot_stride < d.states() + (int64_t)taps * d.C())
+    return hipErrorInvalidValue;
+#define HDS_DX(TT)                                                                                                 \
+  return launch_step(DeltaParams<TT>{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, \
+                                     seqs, nullptr, nullptr, nullptr, nullptr, (TT*)out, ldo, 0, eps}, n_seqs, st)
+  if (dtype == kBF16) HDS_DX(bf16);
+  if (dtype == kF32) HDS_DX(float);
+#undef HDS_DX
+  return hipErrorInvalidValue;
+}
+
+// Portions of at most max_new tokens. y [tokens, C], rn [tokens, 2 G], gb [tokens, H, 2] and o [tokens, H, dv] are
+// scratch memory with a row for every token of the step.
+HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
+                              const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
+                              const int* seq_meta, const int* seqs, void* y, float* rn, float* gb, float* o, void* out,
+                              int64_t ldo, int n_seqs, int max_new, int H, int G, int dk, int dv, int taps, float eps,
+                              hipStream_t st) {
+  if (n_seqs <= 0 || max_new <= 0) return 0;
+  const DeltaDims d{H, G, dk, dv, taps, ld};
+  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || !y || !rn || !gb || !o || ldo < (int64_t)H * dv ||
+      slot_stride < d.states() + (int64_t)taps * d.C())
+    return hipErrorInvalidValue;
+#define HDS_DX(TT)                                                                                                   \
+  {                                                                                                                  \
+    const DeltaParams<TT> p{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, seqs,     \
+                            (TT*)y, rn, gb, o, (TT*)out, ldo, 0, eps};                                               \
+    if (int e = launch_conv(p, n_seqs, max_new, st)) return e;                                                       \
+    if (int e = launch_scan(p, n_seqs, st)) return e;                                                                \
+    return launch_out(p, n_seqs, max_new, st);                                                                       \
+  }
+  if (dtype == kBF16) HDS_DX(bf16)
+  if (dtype == kF32) HDS_DX(float)
+#undef HDS_DX
+  return hipErrorInvalidValue;
+}

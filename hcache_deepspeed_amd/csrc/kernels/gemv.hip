@@ -102,11 +102,16 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const bf16* __restrict__
 // GLU: the weight is [gate; up] ([2I, K]) and the output y[M, I] = bf16(act(bf16(x.g_j)) * bf16(x.u_j)): a wave
 // owns R output columns and streams their gate AND up rows, so the [M, 2I] intermediate never exists.
 __device__ __forceinline__ float silu_f(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
-// the gate's activation, by the codes of act.hip: 0 silu, 1 gelu_tanh, 2 relu
+// gated unit, by the codes of act.hip: 0 silu, 1 gelu_tanh, 2 relu, 5 the clamped form with its limit
 __device__ __forceinline__ float gate_f(float v, int act) {
   if (act == 2) return fmaxf(v, 0.f);
   if (act == 1) return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
   return silu_f(v);
+}
+__device__ __forceinline__ float gated_f(float g, float u, int act, float limit) {
+  if (act != 5) return gate_f(g, act) * u;
+  g = fminf(g, limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-1.702f * g)) * (fminf(fmaxf(u, -limit), limit) + 1.f);
 }
 
 // r = bf16(h + res) (h without res) for 8 elements at k
@@ -145,7 +150,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16* __restrict_
                                                          const bf16* __restrict__ gamma, float eps,
                                                          const bf16* __restrict__ w, bf16* __restrict__ y,
                                                          bf16* __restrict__ r_out, bf16* __restrict__ x_out, int act,
-                                                         int M, int N, int K, int64_t ldh, int64_t ldy) {
+                                                         float limit, int M, int N, int K, int64_t ldh, int64_t ldy) {
   const int lane = threadIdx.x & 63;
   const int wid = threadIdx.x >> 6;
   const int n0 = (blockIdx.x * 4 + wid) * R;  // output columns [n0, n0 + R)
@@ -226,7 +231,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16* __restrict_
         const float v = rstd[m] * wave_sum(acc[r][m]);
         if constexpr (GLU) {
           const float u = rstd[m] * wave_sum(acc[R + r][m]);
-          if (lane == 0) y[m * ldy + n0 + r] = (bf16)(gate_f((float)(bf16)v, act) * (float)(bf16)u);
+          if (lane == 0) y[m * ldy + n0 + r] = (bf16)gated_f((float)(bf16)v, (float)(bf16)u, act, limit);
         } else {
           if (lane == 0) y[m * ldy + n0 + r] = (bf16)v;
         }
@@ -422,20 +427,20 @@ HDS_EXPORT int hds_skinny_set_unroll(int u) {
 }
 
 // Fused decode GEMV (see gemv_fused_kernel): y[M, N] = norm(h (+ res)) . W^T, or with glu = 1 + activation code
-// (0 silu, 1 gelu_tanh, 2 relu), y[M, N] = act(x . Wg^T) * (x . Wu^T) for W = [Wg; Wu] of 2N rows (x normed when gamma is given, else h itself). r_out /
+// (0 silu, 1 gelu_tanh, 2 relu, 5 the clamped gate with its limit), y[M, N] = act(x . Wg^T) * (x . Wu^T) for W = [Wg; Wu] of 2N rows (x normed when gamma is given, else h itself). r_out /
 // x_out (workgroup 0, with gamma): the new residual rows and the normed rows. ldh: row stride of h / res / r_out /
 // x_out (elements); ldy: row stride of y. Shapes: M <= 8, K % 8 == 0, 16-B aligned operands (checked by the caller).
 HDS_EXPORT int hds_gemv_fused_bf16(const void* h, const void* res, const void* gamma, float eps, const void* w,
-                                   void* y, void* r_out, void* x_out, int glu, int M, int N, int K, int64_t ldh,
-                                   int64_t ldy, hipStream_t st) {
-  if (M < 1 || M > 8 || N < 1 || K < 8 || K % 8 || ldh % 8 || glu < 0 || glu > 3) return hipErrorInvalidValue;
+                                   void* y, void* r_out, void* x_out, int glu, float limit, int M, int N, int K,
+                                   int64_t ldh, int64_t ldy, hipStream_t st) {
+  if (M < 1 || M > 8 || N < 1 || K < 8 || K % 8 || ldh % 8 || glu < 0 || glu > 6 || glu == 4 || glu == 5) return hipErrorInvalidValue;
   const int act = glu - 1;
   if (gamma == nullptr && (r_out != nullptr || x_out != nullptr || res != nullptr)) return hipErrorInvalidValue;
   const int R = N >= 8192 ? (glu ? 2 : 4) : (N >= 4096 ? 2 : 1);
 #define HDS_GF(MM, RR, NN, GG)                                                                                   \
   hipLaunchKernelGGL((gemv_fused_kernel<MM, RR, NN, GG>), dim3((N + 4 * RR - 1) / (4 * RR)), dim3(256), 0, st,  \
                      (const bf16*)h, (const bf16*)res, (const bf16*)gamma, eps, (const bf16*)w, (bf16*)y,      \
-                     (bf16*)r_out, (bf16*)x_out, act, M, N, K, ldh, ldy)
+                     (bf16*)r_out, (bf16*)x_out, act, limit, M, N, K, ldh, ldy)
 #define HDS_GFM(RR, NN, GG)                                                                                    \
   if (M == 1) HDS_GF(1, RR, NN, GG); else if (M <= 2) HDS_GF(2, RR, NN, GG);                                   \
   else if (M <= 4) HDS_GF(4, RR, NN, GG); else HDS_GF(8, RR, NN, GG);

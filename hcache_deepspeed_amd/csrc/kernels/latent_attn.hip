@@ -3,6 +3,8 @@
 //
 //   score(i, j, h) = scale * (q_nope[i, h] . W_uk[h] c_j + q_rot[i, h] . r_j),  0 <= i - j < window (0: no window)
 //
+// and optionally a gate per token and head whose sigmoid multiplies the head's output.
+//
 // Two forms of the same product, chosen per sequence of a step:
 //   * absorbed (single tokens, short portions): W_uk[h]^T q_nope is formed once per token and head, scores and the
 //     weighted sum run on the cached rows themselves (read once for all heads), W_uv[h] is applied to the sum;
@@ -21,10 +23,14 @@ namespace {
 
 constexpr float kLog2e = 1.4426950408889634f;
 
+__device__ __forceinline__ float gate_of(float g) { return 1.f / (1.f + __expf(-g)); }
+
 template <typename T>
 struct PrepParams {
-  T* qd;                  // [tokens, ld]: per head q [dim | rot], then c [rank], then r [rot]
-  int64_t ld;
+  T* q;                   // [tokens, ldq]: per head [dim | rot]
+  int64_t ldq;
+  const T* c;             // [tokens, ldc]: latent [rank], then the shared key part [rot]
+  int64_t ldc;
   const float* norm;      // [rank]
   const float* cos_t;     // [positions, rd / 2]
   const float* sin_t;
@@ -80,8 +86,8 @@ __global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
     const int pos = min(p.tok_pos[t], p.n_pos - 1);
     const float* ct = p.cos_t + (int64_t)pos * half;
     const float* st = p.sin_t + (int64_t)pos * half;
-    T* row = p.qd + (int64_t)t * p.ld;
-    const T* c = row + (int64_t)p.H * qh;
+    T* row = p.q + (int64_t)t * p.ldq;
+    const T* c = p.c + (int64_t)t * p.ldc;
     const int nc = row_w / 8;
     const int i = threadIdx.x;  // chunk of the row; rows of more than 256 chunks loop below for the rotated part only
     float v[8];
@@ -149,7 +155,7 @@ __global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
       float v = 0.f;
       if (a < na) {
         const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
-        v = to_f(p.qd[(int64_t)t * p.ld + (int64_t)h * qh + d]);
+        v = to_f(p.q[(int64_t)t * p.ldq + (int64_t)h * qh + d]);
       }
       sq[i] = v;
     }
@@ -160,7 +166,7 @@ __global__ __launch_bounds__(256) void latent_prep8_kernel(PrepParams<T> p) {
         const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
         const int pos = min(p.tok_pos[t], p.n_pos - 1);
         float x[8];
-        Vec8<T>::load(p.qd + (int64_t)t * p.ld + (int64_t)h * qh + p.dim + e, x);
+        Vec8<T>::load(p.q + (int64_t)t * p.ldq + (int64_t)h * qh + p.dim + e, x);
         rotate8<T>(x, e, p.rdims, p.cos_t + (int64_t)pos * half, p.sin_t + (int64_t)pos * half);
         Vec8<T>::store(p.qa + ((int64_t)(a0 + a) * p.H + h) * row_w + p.rank + e, x);
       }
@@ -216,8 +222,8 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepParams<T> p) {
     const int pos = min(p.tok_pos[t], p.n_pos - 1);
     const float* ct = p.cos_t + (int64_t)pos * (p.rdims / 2);
     const float* st = p.sin_t + (int64_t)pos * (p.rdims / 2);
-    T* row = p.qd + (int64_t)t * p.ld;
-    const T* c = row + (int64_t)p.H * qh;
+    T* row = p.q + (int64_t)t * p.ldq;
+    const T* c = p.c + (int64_t)t * p.ldc;
     float ss = 0.f;
     for (int i = threadIdx.x; i < p.rank; i += 256) {
       const float v = to_f(c[i]);
@@ -252,7 +258,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepParams<T> p) {
   for (int i = threadIdx.x; i < na * p.dim; i += 256) {
     const int a = i / p.dim, d = i - a * p.dim;
     const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
-    sm[i] = to_f(p.qd[(int64_t)t * p.ld + (int64_t)h * qh + d]);
+    sm[i] = to_f(p.q[(int64_t)t * p.ldq + (int64_t)h * qh + d]);
   }
   for (int i = na * p.dim + threadIdx.x; i < kAbsTok * p.dim; i += 256) sm[i] = 0.f;
   __syncthreads();
@@ -284,7 +290,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepParams<T> p) {
     const int a = i / p.rot, e = i - a * p.rot;
     const int t = p.atok != nullptr ? p.atok[a0 + a] : a0 + a;
     const int pos = min(p.tok_pos[t], p.n_pos - 1);
-    const T* v = p.qd + (int64_t)t * p.ld + (int64_t)h * qh + p.dim;
+    const T* v = p.q + (int64_t)t * p.ldq + (int64_t)h * qh + p.dim;
     p.qa[((int64_t)(a0 + a) * p.H + h) * row_w + p.rank + e] =
         from_f<T>(rotated(v, e, p.rdims, p.cos_t + (int64_t)pos * (p.rdims / 2), p.sin_t + (int64_t)pos * (p.rdims / 2)));
   }
@@ -525,7 +531,8 @@ template <typename T, int TG>
 __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml,
                                                              const T* __restrict__ uv, const int* __restrict__ atok,
-                                                             T* __restrict__ out, int64_t ldo, int n_abs, int H,
+                                                             T* __restrict__ out, int64_t ldo,
+                                                             const T* __restrict__ gate, int64_t ldg, int n_abs, int H,
                                                              int rank, int vd, int splits) {
   extern __shared__ float so[];  // [TG][rank]
   __shared__ float sa[TG][64];
@@ -610,6 +617,7 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __rest
     }
     if (a0 + x < n_abs && lane < 8 && r0 + lane < vd) {
       const int64_t t = atok != nullptr ? atok[a0 + x] : a0 + x;
+      if (gate != nullptr) mine *= gate_of(to_f(gate[t * ldg + h]));
       out[t * ldo + (int64_t)h * vd + r0 + lane] = from_f<T>(mine);
     }
   }
@@ -627,6 +635,8 @@ struct PrefillParams {
   int64_t ldr;
   bf16* out;           // [tokens, ldo]: head h at column h * vd
   int64_t ldo;
+  const bf16* gate;    // [tokens, H] with row stride ldg (the head's output times its sigmoid), or null
+  int64_t ldg;
   const int* meta;     // [n_pre][4] = {q_start, n_new, ws_row of the first key, keys before the first new token}
   int H, dim, dk, vd, window;
   float scale;
@@ -770,7 +780,8 @@ __global__ __launch_bounds__(64 * NW) void latent_prefill_kernel(PrefillParams p
     __syncthreads();
   }
   if (row_ok) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
+    float inv = l > 0.f ? 1.f / l : 0.f;
+    if (p.gate != nullptr) inv *= gate_of((float)p.gate[(int64_t)(q0 + tok) * p.ldg + head]);
     bf16* op = p.out + (int64_t)(q0 + tok) * p.ldo + (int64_t)head * p.vd;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -836,17 +847,17 @@ int decode_hg(int H, int rank, int rot) {
 
 }  // namespace
 
-HDS_EXPORT int hds_latent_prep(int dtype, void* qd, int64_t ld, const float* norm, const float* cos_t,
-                               const float* sin_t, void* cache, const int* tok_seq, const int* tok_pos,
+HDS_EXPORT int hds_latent_prep(int dtype, void* q, int64_t ldq, const void* c, int64_t ldc, const float* norm,
+                               const float* cos_t, const float* sin_t, void* cache, const int* tok_seq, const int* tok_pos,
                                const int* tables, const int* ws_row, void* ws, const void* uk, const int* atok,
                                void* qa, int n_tok, int n_abs, int n_pos, int max_blocks, int block_size, int H,
                                int dim, int rot, int rdims, int rank, float eps, hipStream_t st) {
   if (n_tok <= 0) return 0;
   if (H < 1 || dim < 0 || rot < 0 || rdims < 0 || rdims > rot || rdims % 2 || rank < 1 || n_pos < 1 || n_abs < 0 ||
-      n_abs > n_tok || block_size < 1 || ld < (int64_t)H * (dim + rot) + rank + rot || (n_abs > 0 && (!qa || !uk)))
+      n_abs > n_tok || block_size < 1 || ldq < (int64_t)H * (dim + rot) || ldc < rank + rot || (n_abs > 0 && (!qa || !uk)))
     return hipErrorInvalidValue;
-  const bool v8 = dim % 8 == 0 && rot % 8 == 0 && rdims % 8 == 0 && rank % 8 == 0 && rank <= 2048 && ld % 8 == 0 &&
-                  (uintptr_t)qd % 16 == 0 && (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0;
+  const bool v8 = dim % 8 == 0 && rot % 8 == 0 && rdims % 8 == 0 && rank % 8 == 0 && rank <= 2048 && ldq % 8 == 0 && ldc % 8 == 0 &&
+                  (uintptr_t)q % 16 == 0 && (uintptr_t)c % 16 == 0 && (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0;
   const int64_t cblocks = v8 ? (rank + kAbsCols - 1) / kAbsCols : 1;
   const int tg = v8 && n_abs == 1 ? 1 : kAbsTok;
   const int64_t grid = n_tok + (int64_t)((n_abs + tg - 1) / tg) * H * cblocks;
@@ -854,8 +865,8 @@ HDS_EXPORT int hds_latent_prep(int dtype, void* qd, int64_t ld, const float* nor
   if (grid > 0x7fffffff || lds > 64 * 1024) return hipErrorInvalidValue;
 #define HDS_LP(TT)                                                                                                   \
   {                                                                                                                  \
-    PrepParams<TT> p{(TT*)qd, ld, norm, cos_t, sin_t, (TT*)cache, tok_seq, tok_pos, tables, ws_row, (TT*)ws,       \
-                     (const TT*)uk, atok, (TT*)qa, n_tok, n_abs, n_pos, max_blocks, block_size, H, dim, rot, rdims, \
+    PrepParams<TT> p{(TT*)q, ldq, (const TT*)c, ldc, norm, cos_t, sin_t, (TT*)cache, tok_seq, tok_pos, tables,       \
+                     ws_row, (TT*)ws, (const TT*)uk, atok, (TT*)qa, n_tok, n_abs, n_pos, max_blocks, block_size, H, dim, rot, rdims, \
                      rank, eps};                                                                                     \
     if (v8 && n_abs == 0)                                                                                            \
       hipLaunchKernelGGL((latent_prep8_kernel<TT, 0>), dim3((unsigned)grid), dim3(256), 64, st, p);                  \
@@ -919,14 +930,14 @@ HDS_EXPORT int hds_latent_decode(int dtype, const void* qa, const void* cache, f
 }
 
 HDS_EXPORT int hds_latent_combine(int dtype, const float* part_o, const float* part_ml, const void* uv,
-                                  const int* atok, void* out, int64_t ldo, int n_abs, int H, int rank, int vd,
-                                  int splits, hipStream_t st) {
+                                  const int* atok, void* out, int64_t ldo, const void* gate, int64_t ldg, int n_abs,
+                                  int H, int rank, int vd, int splits, hipStream_t st) {
   if (n_abs <= 0) return 0;
   if (splits < 1 || splits > 64 || vd < 1 || n_abs > 65535 || rank > 8192) return hipErrorInvalidValue;
 #define HDS_LC(TT, TG)                                                                                               \
   hipLaunchKernelGGL((latent_combine_kernel<TT, TG>), dim3(H, (n_abs + TG - 1) / TG, (vd + kUvRows - 1) / kUvRows), \
                      dim3(256), TG * rank * sizeof(float), st, part_o, part_ml, (const TT*)uv, atok, (TT*)out, ldo, \
-                     n_abs, H, rank, vd, splits)
+                     (const TT*)gate, ldg, n_abs, H, rank, vd, splits)
   const bool four = n_abs >= 4 && rank <= 2048;
   if (dtype == kBF16) {
     if (four) HDS_LC(bf16, 4); else HDS_LC(bf16, 1);
@@ -947,13 +958,14 @@ HDS_EXPORT int hds_latent_prefill_ok(int dim, int rot, int rank, int vd) {
 }
 
 HDS_EXPORT int hds_latent_prefill(const void* q, int64_t ldq, const void* kv, int64_t ldkv, const void* kr,
-                                  int64_t ldr, void* out, int64_t ldo, const int* meta, int n_pre, int max_new, int H,
-                                  int dim, int rot, int rank, int vd, int window, float scale, hipStream_t st) {
+                                  int64_t ldr, void* out, int64_t ldo, const void* gate, int64_t ldg, const int* meta,
+                                  int n_pre, int max_new, int H, int dim, int rot, int rank, int vd, int window,
+                                  float scale, hipStream_t st) {
   if (n_pre <= 0 || max_new <= 0) return 0;
   if (!hds_latent_prefill_ok(dim, rot, rank, vd) || ldq % 8 || ldkv % 8 || ldr % 8 || ldo % 8 || H > 65535 ||
       n_pre > 65535 || window < 0)
     return hipErrorInvalidValue;
-  PrefillParams p{(const bf16*)q, ldq, (const bf16*)kv, ldkv, (const bf16*)kr, ldr, (bf16*)out, ldo, meta, H, dim,
+  PrefillParams p{(const bf16*)q, ldq, (const bf16*)kv, ldkv, (const bf16*)kr, ldr, (bf16*)out, ldo, (const bf16*)gate, ldg, meta, H, dim,
                   dim + rot, vd, window, scale};
   const int dk = dim + rot;
   if (dk <= 64 && vd <= 64) return launch_prefill<64, 64>(p, n_pre, max_new, st);

@@ -21,10 +21,11 @@
 // so K/V of a kv head are read ONCE for all of its query heads -- for decode (1 token) one wave
 // serves the whole GQA group from a single pass over the sequence's KV blocks.
 //
-// Options of all attention kernels: a sliding window; a sink, one learned score per query head that joins the softmax
-// denominator but has no key and no value; an output gate, one value per token and query head whose sigmoid multiplies
-// the head's output. head_norm_scatter is the counterpart of the RoPE scatter for heads that are RMS-normed and not
-// rotated.
+// Options of all attention kernels: a sliding window; chunks, runs of positions counted from the sequence's start that see
+// only themselves; a soft cap of the scores, cap * tanh(score / cap); a sink, one score per query head that joins the
+// softmax denominator but has no key and no value; an output gate, one value per token and query head (or per element of
+// the head's output) whose sigmoid multiplies it. head_norm_scatter is the counterpart of the RoPE scatter for heads that
+// are not rotated: optional RMS norms of q and k, optional mixing of the values with another layer's.
 #include "attn_common.h"
 
 using namespace hds;
@@ -131,6 +132,9 @@ struct HeadNormParams {
   const int* tables;
   int n_tok, max_blocks, block_size, hq, hkv, dk, dv;
   float eps;
+  const T* v0;  // [tokens, ldv0] values of another layer, or null: v <- v + mix * (v0 - v)
+  int64_t ldv0;
+  const float* mix;
 };
 
 template <typename T>
@@ -172,6 +176,13 @@ __global__ __launch_bounds__(256) void head_norm_scatter8_kernel(HeadNormParams<
 #pragma unroll
     for (int i = 0; i < 8; ++i) v[i] *= rs * n[i];
   }
+  if (is_v && p.v0 != nullptr) {
+    const float lam = *p.mix;
+    float o[8];
+    Vec8<T>::load(p.v0 + (int64_t)t * p.ldv0 + (h - p.hq - p.hkv) * p.dv + c, o);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = (1.f - lam) * v[i] + lam * o[i];
+  }
   if (h < p.hq) {
     if (w != nullptr) Vec8<T>::store(src, v);
   } else {
@@ -197,6 +208,12 @@ __global__ __launch_bounds__(256) void head_norm_scatter_kernel(HeadNormParams<T
     float ss = 0.f;
     for (int i = lane; i < d; i += 64) ss += to_f(src[i]) * to_f(src[i]);
     rs = 1.f / sqrtf(wave_sum(ss) / (float)d + p.eps);
+  }
+  if (is_v && p.v0 != nullptr) {
+    const float lam = *p.mix;
+    const T* o = p.v0 + (int64_t)t * p.ldv0 + (h - p.hq - p.hkv) * p.dv;
+    for (int i = lane; i < d; i += 64) dst[i] = from_f<T>((1.f - lam) * to_f(src[i]) + lam * to_f(o[i]));
+    return;
   }
   for (int i = lane; i < d; i += 64) dst[i] = from_f<T>(w != nullptr ? to_f(src[i]) * rs * w[i] : to_f(src[i]));
 }
@@ -225,6 +242,21 @@ struct PageTable {
 
 __device__ __forceinline__ float gate_of(float g) { return 1.f / (1.f + __expf(-g)); }
 
+// cap * tanh(x / cap)
+__device__ __forceinline__ float soft_cap(float x, float cap) { return cap * tanhf(x / cap); }
+// the same in the log2 domain of the matrix-core kernel: cap2 = cap * log2(e), inv2 = 2 / cap, x and the result scaled by
+// log2(e); tanh(y) = 1 - 2 / (exp(2 y) + 1)
+__device__ __forceinline__ float soft_cap2(float x, float cap2, float inv2) {
+  return cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(fast_exp2(x * inv2) + 1.f);
+}
+
+// the first position that position pos sees (window, chunk: 0 for none)
+__device__ __forceinline__ int first_key(int pos, int window, int chunk) {
+  int lo = window > 0 ? max(0, pos + 1 - window) : 0;
+  if (chunk > 0) lo = max(lo, pos - pos % chunk);
+  return lo;
+}
+
 struct PagedParams {
   const bf16* q;  // [T, Hq, DK] rows with token stride sq
   int64_t sq;
@@ -239,10 +271,12 @@ struct PagedParams {
   int hq, hkv;
   int dk, dv;  // read by the padded kernels only
   float scale;
-  int window;
+  int window, chunk;
+  float softcap;      // 0: none
   const float* sink;  // [Hq] or null
-  const bf16* gate;   // [T, Hq] with token stride sg, or null
+  const bf16* gate;   // [T, Hq * gw] with token stride sg, or null
   int64_t sg;
+  int gw;             // 1: a gate per head, dv: one per element
 };
 
 // DK / DV: head sizes, or with PAD their upper bounds (tiles zero-padded to them; the sizes are multiples of 8)
@@ -267,6 +301,8 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
   const int tok = rr / G, head = hk * G + rr % G;
   const int qpos = seen + tok;  // absolute position of this row's query
   const float c = p.scale * kLog2e;
+  const bool bounded = p.window > 0 || p.chunk > 0;
+  const int lo = first_key(qpos, p.window, p.chunk);
   const int* table = p.block_tables + (int64_t)seq * p.max_blocks;
   const int64_t kv_row = (int64_t)p.hkv * (dk + dv);  // elements between consecutive slots
 
@@ -292,11 +328,7 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
   const int wg_qpos_max = seen + last_row / G;
   const int ctx = wg_qpos_max + 1;
   const int kt_end = (ctx + BN - 1) / BN;
-  int kt_begin = 0;
-  if (p.window > 0) {
-    const int first = seen + (row_start / G) - p.window + 1;
-    kt_begin = first > 0 ? first / BN : 0;
-  }
+  const int kt_begin = bounded ? first_key(seen + row_start / G, p.window, p.chunk) / BN : 0;
   auto rowp = [&](int kt, int off) {
     return [=](int row) {
       int pos = kt * BN + row;
@@ -319,6 +351,7 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
   const int w_qpos_lo = seen + min(w_row_lo, n_rows - 1) / G;
   const int w_qpos_hi = seen + min(w_row_lo + 31, n_rows - 1) / G;
   const bool wave_active = w_row_lo < n_rows;
+  const int w_lo = bounded ? first_key(w_qpos_lo, p.window, p.chunk) : 0;
 
   f32x16 o[DT];
 #pragma unroll
@@ -339,7 +372,7 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
     if (kt + 1 < kt_end) stage(buf ^ 1, kt + 1);
     const int k0 = kt * BN;
     bool skip = !wave_active || k0 > w_qpos_hi;
-    if (p.window > 0 && k0 + BN - 1 <= w_qpos_lo - p.window) skip = true;
+    if (k0 + BN - 1 < w_lo) skip = true;
     if (!skip) {
       f32x16 s[2];
 #pragma unroll
@@ -348,6 +381,13 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) s[t] = mfma(rows_d(Kt, 32 * t, ks), qf[ks], s[t]);
       }
+      if (p.softcap > 0.f) {  // (s * c holds the score times log2(e))
+        const float cap2 = p.softcap * kLog2e / c, inv2 = 2.f * c / p.softcap;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) s[t][r] = soft_cap2(s[t][r], cap2, inv2);
+      }
       float tmax = -INFINITY;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
@@ -355,7 +395,7 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
         for (int r = 0; r < 16; ++r) {
           const int kp = k0 + 32 * t + acc_row(r, h);
           float x = s[t][r] * c;
-          if (kp > qpos || !row_ok || (p.window > 0 && kp <= qpos - p.window)) x = -INFINITY;
+          if (kp > qpos || !row_ok || kp < lo) x = -INFINITY;
           s[t][r] = x;
           tmax = fmaxf(tmax, x);
         }
@@ -389,7 +429,22 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
   }
   if (row_ok) {
     float inv = l > 0.f ? 1.f / l : 0.f;
-    if (p.gate != nullptr) inv *= gate_of((float)p.gate[(int64_t)(q_start + tok) * p.sg + head]);
+    const bf16* gp = p.gate == nullptr ? nullptr : p.gate + (int64_t)(q_start + tok) * p.sg + (int64_t)head * p.gw;
+    if (gp != nullptr && p.gw == 1) {
+      inv *= gate_of((float)*gp);
+    } else if (gp != nullptr) {  // registers 4 g .. 4 g + 3 of a block are neighbouring columns
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          const int col = 32 * dt + 8 * g + 4 * h;
+          if (col < dv) {
+            const bf16x4 gv = *reinterpret_cast<const bf16x4*>(gp + col);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) o[dt][4 * g + j] *= gate_of((float)gv[j]);
+          }
+        }
+    }
     bf16* op = p.o + (int64_t)(q_start + tok) * p.so + (int64_t)head * dv;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -430,10 +485,12 @@ struct PagedDecodeParams {
   const int* block_tables;
   int max_blocks, block_size, hq, hkv, dk, dv, splits;
   float scale;
-  int window;
+  int window, chunk;
+  float softcap;      // 0: none
   const float* sink;  // [Hq] or null
-  const T* gate;      // [T, Hq] with token stride sg, or null
+  const T* gate;      // [T, Hq * gw] with token stride sg, or null
   int64_t sg;
+  int gw;             // 1: a gate per head, dv: one per element
   // splits > 1: one int per (token, kv head), zero between launches. Non-null: the last workgroup of a
   // (token, kv head) to finish merges the splits itself (no combine launch) and resets its counter to 0, so a
   // HIP-graph replay finds it zeroed again.
@@ -454,7 +511,7 @@ __device__ __forceinline__ DecodeToken decode_token(const PagedDecodeParams<T>& 
 // this split's keys: an equal share of what the token sees
 template <typename T>
 __device__ __forceinline__ void decode_keys(const PagedDecodeParams<T>& p, int pos, int split, int& j0, int& j1) {
-  const int lo = p.window > 0 ? max(0, pos + 1 - p.window) : 0;
+  const int lo = first_key(pos, p.window, p.chunk);
   const int per = (pos + 1 - lo + p.splits - 1) / p.splits;
   j0 = lo + split * per;
   j1 = min(pos + 1, j0 + per);
@@ -470,7 +527,13 @@ __device__ __forceinline__ float decode_factor(const PagedDecodeParams<T>& p, in
     l = l * f + __expf(p.sink[h] - mm);
   }
   f = l > 0.f ? f / l : 0.f;
-  return p.gate != nullptr ? f * gate_of(to_f(p.gate[(int64_t)row * p.sg + h])) : f;
+  return p.gate != nullptr && p.gw == 1 ? f * gate_of(to_f(p.gate[(int64_t)row * p.sg + h])) : f;
+}
+
+// gate of element d of head h's output, where every element has its own (else 1; the head's gate is in decode_factor)
+template <typename T>
+__device__ __forceinline__ float decode_gate(const PagedDecodeParams<T>& p, int row, int h, int d) {
+  return p.gate != nullptr && p.gw > 1 ? gate_of(to_f(p.gate[(int64_t)row * p.sg + (int64_t)h * p.gw + d])) : 1.f;
 }
 
 template <typename T>
@@ -484,7 +547,8 @@ __device__ __forceinline__ void decode_merge_splits(const PagedDecodeParams<T>& 
     ll += pm[2 * s + 1] * a;
     oo += p.part_o[(((int64_t)b * p.hq + h) * p.splits + s) * p.dv + d] * a;
   }
-  p.o[(int64_t)row * p.so + (int64_t)h * p.dv + d] = from_f<T>(oo * decode_factor(p, row, h, mm, ll));
+  p.o[(int64_t)row * p.so + (int64_t)h * p.dv + d] =
+      from_f<T>(oo * decode_factor(p, row, h, mm, ll) * decode_gate(p, row, h, d));
 }
 
 __device__ __forceinline__ float dot8(const bf16x8& a, const bf16x8& b) {
@@ -560,6 +624,11 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
       float sc[U];
 #pragma unroll
       for (int u = 0; u < U; ++u) sc[u] = group_sum<LPK>(dot8(qv[g], kc[u])) * p.scale;
+      if (p.softcap > 0.f) {
+        const float cap2 = p.softcap * kLog2e, inv2 = 2.f / p.softcap;
+#pragma unroll
+        for (int u = 0; u < U; ++u) sc[u] = soft_cap2(sc[u] * kLog2e, cap2, inv2) / kLog2e;
+      }
       float mn = m[g];
 #pragma unroll
       for (int u = 0; u < U; ++u) {
@@ -624,6 +693,9 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
       const float f = decode_factor(p, tk.row, h, mm, ll);
 #pragma unroll
       for (int e = 0; e < 8; ++e) oo[e] *= f;
+      if (p.gw > 1 && 8 * cc < p.dv)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) oo[e] *= decode_gate(p, tk.row, h, 8 * cc + e);
       if (8 * cc < p.dv) Vec8<bf16>::store(p.o + (int64_t)tk.row * p.so + (int64_t)h * p.dv + cc * 8, oo);
     } else {
       const int64_t pi = ((int64_t)b * p.hq + h) * p.splits + split;
@@ -678,7 +750,7 @@ __global__ __launch_bounds__(256) void paged_plain_kernel(PagedDecodeParams<T> p
       float s = 0.f;
       for (int i = lane; i < p.dk; i += 64) s += sq[i] * to_f(kr[i]);
       s = wave_sum(s);
-      if (lane == 0) ss[k] = s * p.scale;
+      if (lane == 0) ss[k] = p.softcap > 0.f ? soft_cap(s * p.scale, p.softcap) : s * p.scale;
     }
     __syncthreads();
     float mt = m;
@@ -702,7 +774,7 @@ __global__ __launch_bounds__(256) void paged_plain_kernel(PagedDecodeParams<T> p
   if (p.splits == 1) {
     const float f = decode_factor(p, tk.row, h, m, l);
     for (int i = threadIdx.x; i < p.dv; i += 256)
-      p.o[(int64_t)tk.row * p.so + (int64_t)h * p.dv + i] = from_f<T>(acc[i] * f);
+      p.o[(int64_t)tk.row * p.so + (int64_t)h * p.dv + i] = from_f<T>(acc[i] * f * decode_gate(p, tk.row, h, i));
     return;
   }
   for (int i = threadIdx.x; i < p.dv; i += 256) p.part_o[pi * p.dv + i] = acc[i];
@@ -727,6 +799,7 @@ __global__ __launch_bounds__(256) void paged_decode_combine_kernel(PagedDecodePa
 #pragma unroll
   for (int s = 0; s < 64; ++s) pov[s] = s < p.splits ? po[(int64_t)s * p.dv + dl] : 0.f;
   const int row = decode_token(p, b).row;
+  const float gate0 = decode_gate(p, row, h, dl);
   const float* pm = p.part_ml + (int64_t)bh * p.splits * 2;
   if (d0 < p.splits) {
     s_m[d0] = pm[2 * d0];
@@ -746,11 +819,11 @@ __global__ __launch_bounds__(256) void paged_decode_combine_kernel(PagedDecodePa
   }
   const float f = decode_factor(p, row, h, mm, ll);
   T* op = p.o + (int64_t)row * p.so + (int64_t)h * p.dv;
-  if (d0 < p.dv) op[d0] = from_f<T>(oo * f);
+  if (d0 < p.dv) op[d0] = from_f<T>(oo * f * gate0);
   for (int d = d0 + blockDim.x; d < p.dv; d += blockDim.x) {  // heads wider than the workgroup
     oo = 0.f;
     for (int s = 0; s < p.splits; ++s) oo += po[(int64_t)s * p.dv + d] * (mm == -INFINITY ? 0.f : __expf(s_m[s] - mm));
-    op[d] = from_f<T>(oo * f);
+    op[d] = from_f<T>(oo * f * decode_gate(p, row, h, d));
   }
 }
 
@@ -784,7 +857,7 @@ template <typename T>
 int launch_head_norm(const HeadNormParams<T>& p, hipStream_t st) {
   const int64_t items = (int64_t)p.n_tok * (p.hq + 2 * p.hkv);
   const int d = p.dk > p.dv ? p.dk : p.dv;
-  if (p.dk % 8 || p.dv % 8 || p.ld % 8 || d > 512) {
+  if (p.dk % 8 || p.dv % 8 || p.ld % 8 || d > 512 || (p.v0 != nullptr && (p.ldv0 % 8 || (uintptr_t)p.v0 % 16))) {
     hipLaunchKernelGGL(head_norm_scatter_kernel<T>, dim3((items + 3) / 4), dim3(256), 0, st, p);
     return hipGetLastError();
   }
@@ -822,21 +895,24 @@ HDS_EXPORT int hds_kv_rope_scatter(int dtype, void* qkv, int64_t sq, void* cache
   return hipGetLastError();
 }
 
-// q heads normed in place, k heads normed into the cache, v heads copied there; qn / kn null: no norm
+// q heads normed in place, k heads normed into the cache, v heads copied there; qn / kn null: no norm. v0: values
+// [n_tok, hkv * dv] with row stride ldv0 of which the share *mix goes into v; null: v as it is
 HDS_EXPORT int hds_head_norm_scatter(int dtype, void* qkv, int64_t ld, const float* qn, const float* kn, void* cache,
                                      const int* tok_seq, const int* tok_pos, const int* block_tables, int n_tok,
                                      int max_blocks, int block_size, int hq, int hkv, int dk, int dv, float eps,
-                                     hipStream_t st) {
+                                     const void* v0, int64_t ldv0, const float* mix, hipStream_t st) {
   if (n_tok <= 0) return 0;
-  if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || ld < (int64_t)(hq + hkv) * dk + (int64_t)hkv * dv)
+  if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || ld < (int64_t)(hq + hkv) * dk + (int64_t)hkv * dv ||
+      (v0 != nullptr && (mix == nullptr || ldv0 < (int64_t)hkv * dv)))
     return hipErrorInvalidValue;
   if (dtype == kBF16)
     return launch_head_norm(HeadNormParams<bf16>{(bf16*)qkv, ld, qn, kn, (bf16*)cache, tok_seq, tok_pos, block_tables,
-                                                 n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps}, st);
+                                                 n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps, (const bf16*)v0, ldv0,
+                                                 mix}, st);
   if (dtype == kF32)
     return launch_head_norm(HeadNormParams<float>{(float*)qkv, ld, qn, kn, (float*)cache, tok_seq, tok_pos,
-                                                  block_tables, n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps},
-                            st);
+                                                  block_tables, n_tok, max_blocks, block_size, hq, hkv, dk, dv, eps,
+                                                  (const float*)v0, ldv0, mix}, st);
   return hipErrorInvalidValue;
 }
 
@@ -845,16 +921,18 @@ HDS_EXPORT int hds_paged_attn_supported(int dk, int dv) {
   return dk >= 8 && dv >= 8 && dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256;
 }
 
-// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]; sink [hq] and gate [tokens, hq] may be null
+// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]; window, chunk and softcap: 0 for none; sink [hq]
+// and gate [tokens, hq * gw] (gw 1 or dv) may be null
 HDS_EXPORT int hds_paged_attn(const void* q, int64_t sq, const void* cache, void* o, int64_t so, const int* atoms,
                               int n_atoms, const int* seq_meta, const int* block_tables, int max_blocks,
-                              int block_size, int hq, int hkv, int dk, int dv, float scale, int window,
-                              const float* sink, const void* gate, int64_t sg, hipStream_t st) {
-  if (hq < 1 || hkv < 1 || hq % hkv || sq % 8 || so % 4 || !hds_paged_attn_supported(dk, dv))
+                              int block_size, int hq, int hkv, int dk, int dv, float scale, int window, int chunk,
+                              float softcap, const float* sink, const void* gate, int64_t sg, int gw, hipStream_t st) {
+  if (hq < 1 || hkv < 1 || hq % hkv || sq % 8 || so % 4 || !hds_paged_attn_supported(dk, dv) || window < 0 ||
+      chunk < 0 || (gate != nullptr && gw != 1 && (gw != dv || sg % 4 || (uintptr_t)gate % 8)))
     return hipErrorInvalidValue;
   if (n_atoms <= 0) return 0;
   PagedParams p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, atoms, seq_meta, block_tables, max_blocks,
-                block_size, hq, hkv, dk, dv, scale, window, sink, (const bf16*)gate, sg};
+                block_size, hq, hkv, dk, dv, scale, window, chunk, softcap, sink, (const bf16*)gate, sg, gw};
 #define HDS_CASE(d)                                                                                    \
   if (dk == d && dv == d) {                                                                            \
     hipLaunchKernelGGL((paged_attn_kernel<d, d, 4, false>), dim3(n_atoms), dim3(256), 0, st, p);       \
@@ -895,23 +973,24 @@ HDS_EXPORT int hds_paged_decode(int dtype, int plain, const void* q, int64_t sq,
                                 float* part_o, float* part_ml, const int* seq_meta, const int* toks,
                                 const int* tok_seq, const int* tok_pos, const int* block_tables, int max_blocks,
                                 int block_size, int n, int hq, int hkv, int dk, int dv, int splits, float scale,
-                                int window, const float* sink, const void* gate, int64_t sg, int* counters,
-                                hipStream_t st) {
+                                int window, int chunk, float softcap, const float* sink, const void* gate, int64_t sg,
+                                int gw, int* counters, hipStream_t st) {
   if (n <= 0) return 0;
   if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || splits < 1 || splits > 64 || n > 65535 ||
+      window < 0 || chunk < 0 || (gate != nullptr && gw != 1 && gw != dv) ||
       (seq_meta == nullptr && (tok_seq == nullptr || tok_pos == nullptr)) ||
       (splits > 1 && (!part_o || !part_ml)))  // <= 64: the combine kernel stages the split stats in LDS
     return hipErrorInvalidValue;
   if (dtype == kF32) {
     return launch_plain(PagedDecodeParams<float>{(const float*)q, sq, (const float*)cache, (float*)o, so, part_o,
                                                  part_ml, seq_meta, toks, tok_seq, tok_pos, block_tables, max_blocks,
-                                                 block_size, hq, hkv, dk, dv, splits, scale, window, sink,
-                                                 (const float*)gate, sg, nullptr}, n, st);
+                                                 block_size, hq, hkv, dk, dv, splits, scale, window, chunk, softcap,
+                                                 sink, (const float*)gate, sg, gw, nullptr}, n, st);
   }
   if (dtype != kBF16) return hipErrorInvalidValue;
   PagedDecodeParams<bf16> p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, part_o, part_ml, seq_meta, toks,
                             tok_seq, tok_pos, block_tables, max_blocks, block_size, hq, hkv, dk, dv, splits, scale,
-                            window, sink, (const bf16*)gate, sg, counters};
+                            window, chunk, softcap, sink, (const bf16*)gate, sg, gw, counters};
   if (plain) {
     p.counters = nullptr;
     return launch_plain(p, n, st);

@@ -42,14 +42,15 @@ class ArchSpec:
     lm_head_bias: bool = False
     moe: Optional[dict] = None         # {num_experts, top_k, normalize, shared}
     # layers listed one by one (hybrid.py): one entry per layer with weights, {"mixer": {"type", sizes ...}, "mlp":
-    # {"ff", "act"}, {"ff", "act", "shared_ff", "router": {...}} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
+    # {"ff", "act"[, "limit"]}, {"ff", "act", "shared_ff", "router": {...}} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
     layers: Optional[list] = None
     loop: Optional[dict] = None
     order: Optional[list] = None       # the layer every layer run uses (None: each once, with ``loop``)
     input_conv_taps: int = 1
-    norm_place: str = "pre"            # pre: sublayers read the normed residual | post: their output is normed
+    norm_place: str = "pre"            # pre: sublayers read the normed residual | post: their output is normed | both
     embed_scale: float = 1.0
     logit_scale: float = 1.0
+    logit_softcap: float = 0.0         # logits <- cap * tanh(logits / cap); 0: none
     extra: dict = field(default_factory=dict)
 
     # LlamaConfig-compatible aliases used by the engine / KV cache sizing
@@ -195,8 +196,70 @@ def convert_buvuzen(sd, spec):
     return out
 
 
+# ---------------------------------------------------------------------------------------------
+# Fifotar: gated delta rule, latent attention (queries through a latent too, YaRN, a gate per head) and chunked
+# grouped-query attention (soft cap, zero sink, mixed values, a gate per element) before a clamped gated MLP, a norm on
+# both sides of every sublayer, tied embeddings, soft-capped logits
+# ---------------------------------------------------------------------------------------------
+def _fifotar_mixer(kind, m, value_source):
+    """The mixer's sizes; ``value_source``: an earlier layer has left its values."""
+    if kind == "delta":
+        return {"type": kind, **{k: int(m[k]) for k in ("heads", "kv_heads", "dim", "vdim", "conv")}}
+    if kind == "latent_attention":
+        rot = m["rot"]
+        sc = rot.get("scaling")
+        if sc is not None:
+            sc = {"rope_type": "yarn", "factor": float(sc["factor"]), "beta_fast": float(sc["fast"]),
+                  "beta_slow": float(sc["slow"]), "original_max_position_embeddings": float(sc["original"])}
+        return {"type": kind, **{k: int(m[k]) for k in ("heads", "dim", "rot_dim", "kv_rank", "q_rank", "vdim")},
+                "rot_dims": int(rot.get("dims", m["rot_dim"])), "rope_base": float(rot["base"]), "rope_scaling": sc,
+                "rot_layout": "half", "window": 0, "scale": float(m["scale"]), "gated": True}
+    if kind == "attention":
+        mix = ("mix" if value_source else "source") if m.get("v_mix") else None
+        return {"type": kind, **{k: int(m[k]) for k in ("heads", "kv_heads", "dim", "vdim")}, "window": 0,
+                "chunk": int((m.get("mask") or {}).get("size") or 0), "scale": float(m["scale"]),
+                "softcap": float(m.get("softcap") or 0.0), "gated": True, "gate_elements": True, "zero_sink": True,
+                "value_mix": mix}
+    raise NotImplementedError(f"Fifotar mixer {kind!r}")
+
+
+def spec_fifotar(cfg):
+    layers, source = [], False
+    for e in cfg["layers"]:
+        mlp = e.get("mlp")
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise NotImplementedError(f"Fifotar feed-forward {mlp['kind']!r}")
+            mlp = {"ff": int(mlp["ff"]), "act": "clamped", "limit": float(mlp["limit"])}
+        layers.append({"mixer": _fifotar_mixer(e["type"], e["mixer"], source), "mlp": mlp})
+        source |= layers[-1]["mixer"].get("value_mix") is not None
+    return ArchSpec(model_type="fifotar", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                    num_hidden_layers=len(layers), num_attention_heads=max(x["mixer"]["heads"] for x in layers),
+                    num_key_value_heads=max(x["mixer"].get("kv_heads", 1) for x in layers),
+                    head_dim=max(x["mixer"]["dim"] + x["mixer"].get("rot_dim", 0) for x in layers),
+                    intermediate_size=max((x["mlp"]["ff"] for x in layers if x["mlp"]), default=0), norm="rms",
+                    norm_eps=float(cfg["norm"]["eps"]), act="clamped", gated=True, layers=layers, norm_place="both",
+                    embed_scale=float(cfg["embedding"]["scale"]), logit_softcap=float(cfg.get("logit_softcap") or 0.0),
+                    tie_embeddings=True, extra={"residual_mult": float(cfg["residual_mult"])})
+
+
+def convert_fifotar(sd, spec):
+    mult = spec.extra["residual_mult"]
+    out = {"embed": sd["embed"], "final.w": sd["final.norm"], "lm_head.w": sd["embed"], "layers": []}
+    for i, e in enumerate(spec.layers):
+        p = f"l{i}."
+        L = {"mix": {k[len(p) + 4:]: v for k, v in sd.items() if k.startswith(p + "mix.")},
+             "ln1.w": sd[p + "norm1"], "ln1b.w": sd[p + "norm1b"].float() * mult}
+        if e["mlp"] is not None:
+            L.update({"ln2.w": sd[p + "norm2"], "ln2b.w": sd[p + "norm2b"].float() * mult,
+                      "gate.w": sd[p + "mlp.gate"], "up.w": sd[p + "mlp.up"], "down.w": sd[p + "mlp.down"]})
+        out["layers"].append(L)
+    return out
+
+
 # config.json's "architecture" / "model_type" -> (config reader, weight converter)
-ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun), "buvuzen": (spec_buvuzen, convert_buvuzen)}
+ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun), "buvuzen": (spec_buvuzen, convert_buvuzen),
+                 "fifotar": (spec_fifotar, convert_fifotar)}
 
 
 def spec_from_hf(hf):

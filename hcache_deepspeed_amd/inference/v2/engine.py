@@ -19,7 +19,7 @@ import torch
 
 from ... import comm as dist
 from ...utils.logging import log_dist
-from .hybrid import HybridTransformer, PostNormTransformer
+from .hybrid import HybridTransformer, PostNormTransformer, SandwichTransformer
 from .model import RaggedTransformer
 from .ragged import (BlockedKVCache, DSStateManager, DSStateManagerConfig, RaggedBatchWrapper, SequenceStatePool)
 
@@ -63,7 +63,7 @@ def transformer_class(spec):
     """The model implementation that serves an ArchSpec."""
     if spec.layers is None:
         return RaggedTransformer
-    return PostNormTransformer if spec.norm_place == "post" else HybridTransformer
+    return {"pre": HybridTransformer, "post": PostNormTransformer, "both": SandwichTransformer}[spec.norm_place]
 
 
 class InferenceEngineV2:
@@ -343,7 +343,7 @@ def build_hf_engine(path, engine_config=None, debug_level=None, device=None, num
     """Serving engine from a HuggingFace checkpoint directory (config.json + *.safetensors / *.bin).
 
     Supported ``model_type``: llama, mistral, mixtral, qwen, qwen2, qwen2_moe, phi, phi3, falcon, opt
-    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun, Buvuzen."""
+    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun, Buvuzen, Fifotar."""
     from .arch import convert_hf, spec_from_hf
     with open(os.path.join(path, "config.json")) as f:
         hf = json.load(f)

@@ -1,6 +1,6 @@
 """Decoders whose layers are listed one by one in :class:`arch.ArchSpec` ``layers``: mixers of several kinds, layers that
 run more than once with the same weights (``loop`` / ``order``), a 32-bit residual stream. Served by the same engine,
-paged cache, batch metadata and decode graphs as :class:`model.RaggedTransformer`. Two layer forms:
+paged cache, batch metadata and decode graphs as :class:`model.RaggedTransformer`. Three layer forms:
 
 * :class:`HybridTransformer` (``norm_place`` "pre"): mixer and gated MLP read the same residual (parallel block, two
   norms), with a causal convolution in front of every sublayer. A layer is: input norm (residual add + norm +
@@ -9,8 +9,10 @@ paged cache, batch metadata and decode graphs as :class:`model.RaggedTransformer
 * :class:`PostNormTransformer` ("post"): mixer, then expert layer, each reading the residual itself; the norm is on their
   outputs. A layer is: mixer and its output projection, norm + residual add (one kernel), router and experts, and one
   kernel that sums the experts' outputs, norms the sum and adds it.
+* :class:`SandwichTransformer` ("both"): mixer, then gated MLP, each between a norm of its input and a norm of its output.
+  One kernel between two sublayers norms the first one's output, adds it to the residual and norms the sum for the next.
 
-Common to both:
+Common to all:
 
 * every layer *run* (a pass of a looped or shared layer counts) has its own paged cache rows and its own part of the sequence's
   state row (``ragged.SequenceStatePool``): convolution tails and recurrent states, float32;
@@ -28,7 +30,7 @@ from .model import RaggedTransformer, _Layer
 from .modules import (DSExpertLayerConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig,
                       DSNormConfig, DSUnembedConfig, instantiate_expert_layer, instantiate_gated_mlp,
                       instantiate_input_norm, instantiate_linear, instantiate_mixer, instantiate_output_norm,
-                      instantiate_unembed)
+                      instantiate_sandwich_norm, instantiate_unembed)
 from .modules.implementations import _PackedWeight
 
 
@@ -41,7 +43,7 @@ class _Run:
 
 
 # weights kept in the engine's dtype; every other float32 tensor stays float32
-_MATRICES = ("in.w", "up.w", "out.w", "ukv.w", "router.w", "w13", "w2", "ws13", "ws2")
+_MATRICES = ("in.w", "up.w", "out.w", "down.w", "uq.w", "ukv.w", "router.w", "w13", "w2", "ws13", "ws2")
 
 
 class HybridTransformer(RaggedTransformer):
@@ -67,16 +69,18 @@ class HybridTransformer(RaggedTransformer):
     def _build_modules(self, ec):
         spec, H = self.spec, self.spec.hidden_size
         self.unembed_mod = instantiate_unembed(DSUnembedConfig(model_dim=H, vocab_size=spec.vocab_size,
-                                                               norm_type="rms"), ec)
+                                                               norm_type="rms", softcap=spec.logit_softcap), ec)
         self.mixers, self.mlps, self.linears = [], [], []
         for e in spec.layers:
             mix = instantiate_mixer(DSMixerConfig(e["mixer"]["type"], H, e["mixer"], spec.norm_eps, self.tp,
                                                   self.dtype), ec)
             if hasattr(mix, "bind_tables"):
-                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base,
+                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base, mix.rope_scaling,
                                              device=self.device))
             self.mixers.append(mix)
         self._build_layers(ec)
+        for lins, mix in zip(self.linears, self.mixers):
+            lins.update({k: instantiate_linear(DSLinearConfig(*io), ec) for k, io in mix.extra_linears().items()})
 
     def _build_layers(self, ec):
         spec, H = self.spec, self.spec.hidden_size
@@ -113,14 +117,15 @@ class HybridTransformer(RaggedTransformer):
         shard = lm[r * vs:(r + 1) * vs]
         if shard.shape[0] < vs:  # equal row counts on every rank; the padding columns are cut at ``vocab``
             shard = torch.cat([shard, shard.new_zeros(vs - shard.shape[0], shard.shape[1])])
-        self.lm_head = t(shard)
+        self.lm_head = self.embed if shard is sd["embed"] or shard.data_ptr() == sd["embed"].data_ptr() and \
+            shard.shape == sd["embed"].shape else t(shard)
         self.layers = []
         for i, Ls in enumerate(sd["layers"]):
             L = _Layer()
             mw = self.mixers[i].shard(Ls["mix"], self._rows, self._cols)
             o = mw.pop("o.w")
             self._put(L, mw)
-            for k in ("1", "2"):
+            for k in ("1", "2", "1b", "2b"):
                 if Ls.get(f"ln{k}.w") is not None:
                     L.w[f"ln{k}.w"] = f(Ls[f"ln{k}.w"].reshape(-1))
             L.w["out.w"] = t(self._load_layer(i, L, Ls, o))
@@ -204,7 +209,7 @@ class HybridTransformer(RaggedTransformer):
 
     def _mix(self, run, x, out, batch):
         i = run.layer
-        self.mixers[i](x, self.layers[i], self.linears[i]["in.w"], out, batch,
+        self.mixers[i](x, self.layers[i], self.linears[i], out, batch,
                        None if run.cache is None else self.kv_cache.get_cache(run.cache), self._state(), run.state)
 
     def _state(self):
@@ -230,6 +235,7 @@ class HybridTransformer(RaggedTransformer):
     def forward(self, batch, capture_latents=True, sync_latents=True, sink=None):
         """Logits of the wanted rows and the latents ([1, T, W] on the host, or None); see the base class."""
         T = batch.current_tokens
+        batch.carry.clear()
         stream = self._start(batch)
         for run in self.runs:
             stream = self._layer(run, stream, batch)
@@ -321,3 +327,59 @@ class PostNormTransformer(HybridTransformer):
         if self.tp > 1:
             parts = self._allreduce(moe.total(x, parts))
         return self.norm_mod(x, parts, L["ln2.w"])
+
+
+class SandwichTransformer(HybridTransformer):
+    """Layers with a norm on both sides of every sublayer: x += n1b(mixer(n1(x))), x += n2b(mlp(n2(x))); the factor of the
+    residual sum is part of the gains of n1b and n2b."""
+    KERNEL_SOURCES = ("act.hip", "delta_rule.hip", "gemv.hip", "latent_attn.hip", "output_norm.hip", "paged_attn.hip",
+                      "paged_rows.hip")
+
+    def _build_layers(self, ec):
+        spec, H = self.spec, self.spec.hidden_size
+        self.norm_mod = instantiate_sandwich_norm(DSNormConfig(H, "rms", spec.norm_eps, torch.float32, self.dtype), ec)
+        for e, mix in zip(spec.layers, self.mixers):
+            m = e["mlp"]
+            lins = {"in.w": instantiate_linear(DSLinearConfig(H, mix.in_width), ec),
+                    "out.w": instantiate_linear(DSLinearConfig(mix.out_width, H), ec)}
+            mlp, ff = None, 0
+            if m is not None:
+                assert m["ff"] % self.tp == 0, "the feed-forward width must divide the tensor-parallel size"
+                ff = m["ff"] // self.tp
+                mlp = instantiate_gated_mlp(DSGatedMLPConfig(H, ff, m["act"], m.get("limit", 0.0)), ec)
+                lins["up.w"] = instantiate_linear(DSLinearConfig(H, 2 * ff), ec)
+                lins["down.w"] = instantiate_linear(DSLinearConfig(ff, H), ec)
+            self.mlps.append((mlp, ff))
+            self.linears.append(lins)
+
+    def _load_layer(self, i, L, Ls, o):
+        if self.mlps[i][0] is not None:
+            L.w["up.w"] = self._t(torch.cat([self._rows(Ls["gate.w"]), self._rows(Ls["up.w"])]))
+            L.w["down.w"] = self._t(self._cols(Ls["down.w"]))
+        return o
+
+    def _norm_state_floats(self):
+        return 0
+
+    # the stream: (32-bit residual or None at the start, the last sublayer's output, the gain of its norm)
+    def _start(self, batch):
+        self._rows_in = (self.embed, batch.input_ids, self.spec.embed_scale)
+        return None, None, None
+
+    def _final(self, stream, idx):
+        return self.norm_mod(*stream, self.final_w, embed=self._rows_in, idx=idx)[1]
+
+    def _layer(self, run, stream, batch):
+        i = run.layer
+        L, mix, (mlp, ff), lins = self.layers[i], self.mixers[i], self.mlps[i], self.linears[i]
+        T = batch.current_tokens
+        x, rows = self.norm_mod(*stream, L["ln1.w"], embed=self._rows_in)
+        mid = torch.empty(T, mix.out_width, dtype=self.dtype, device=self.device)
+        self._mix(run, rows, mid, batch)
+        y = self._allreduce(lins["out.w"](mid, L["out.w"]))
+        if mlp is None:
+            return x, y, L["ln1b.w"]
+        x, rows = self.norm_mod(x, y, L["ln1b.w"], L["ln2.w"])
+        h = torch.empty(T, ff, dtype=self.dtype, device=self.device)
+        mlp(rows, L["up.w"], lins["up.w"], h)
+        return x, self._allreduce(lins["down.w"](h, L["down.w"])), L["ln2b.w"]

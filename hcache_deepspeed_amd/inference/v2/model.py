@@ -733,6 +733,7 @@ class _DecodeGraph:
         sb.slots = take(B, (B, ))
         sb.max_new = 1
         sb.plans = {}
+        sb.carry = {}
         sb.logits_of_last_tokens = True
         sb.current_tokens = B
         sb.current_sequences = B

@@ -86,6 +86,7 @@ class DSGatedMLPConfig:
     model_dim: int
     intermediate_features: int
     activation: str = "silu"
+    limit: float = 0.0  # of the activation "clamped"
 
 
 @dataclass
@@ -102,4 +103,5 @@ class DSUnembedConfig:
     dtype: torch.dtype = torch.bfloat16
     model_dim: int = 0
     vocab_size: int = 0
+    softcap: float = 0.0  # logits <- softcap * tanh(logits / softcap); 0: none
     norm_type: Optional[str] = "rms"  # final norm fused in front of the vocab GEMM (None: none)

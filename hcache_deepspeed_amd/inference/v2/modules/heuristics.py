@@ -6,7 +6,7 @@ from .configs import (DSEmbeddingsConfig, DSExpertLayerConfig, DSGatedMLPConfig,
                       DSMixerConfig, DSMoEConfig, DSNormConfig, DSSelfAttentionConfig, DSUnembedConfig)
 from .interfaces import (DSEmbeddingRegistry, DSExpertLayerRegistry, DSGatedMLPRegistry, DSInputNormRegistry,
                          DSLinearRegistry, DSMixerRegistry, DSMoERegistry, DSOutputNormRegistry, DSPostNormRegistry,
-                         DSPreNormRegistry, DSSelfAttentionRegistry, DSUnembedRegistry)
+                         DSPreNormRegistry, DSSandwichNormRegistry, DSSelfAttentionRegistry, DSUnembedRegistry)
 from .module_registry import ConfigBundle
 from . import implementations  # noqa: F401  (registers the implementations)
 
@@ -70,6 +70,10 @@ def instantiate_gated_mlp(config: DSGatedMLPConfig, engine_config=None):
 
 def instantiate_output_norm(config: DSNormConfig, engine_config=None):
     return DSOutputNormRegistry.instantiate_config(ConfigBundle("rms_residual", config))
+
+
+def instantiate_sandwich_norm(config: DSNormConfig, engine_config=None):
+    return DSSandwichNormRegistry.instantiate_config(ConfigBundle("rms_sandwich", config))
 
 
 def instantiate_expert_layer(config: DSExpertLayerConfig, engine_config=None):

@@ -14,6 +14,7 @@ import torch.nn.functional as F
 
 from .... import comm as dist
 from ....ops.activations import bias_act, glu, glu_rows
+from ....ops.delta_rule import DeltaShape, delta_rule, make_delta_plan, step_ok
 from ....ops.experts import PAD, routed_experts
 from ....ops.gated_scan import gated_scan, recur_step, recur_step_ok
 from ....ops.gemv import glu_gemv
@@ -22,15 +23,17 @@ from ....ops.input_norm import input_norm
 from ....ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
 from ....ops.moe import moe_combine, moe_dispatch, topk_assign, topk_route
 from ....ops.norm import layer_norm, rms_norm
-from ....ops.output_norm import embed_rows, padded, residual_norm, sum_experts
+from ....ops.output_norm import (embed_rows, padded, residual_norm, rms_rows, sandwich_norm, softcap_,
+                                 sum_experts)
 from ....ops.paged import (HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
                            paged_attention)
 from ....ops.quantizer import fp6_linear, int_linear, quantize, quantize_minifloat
 from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSExpertLayerBase, DSExpertLayerRegistry, DSGatedMLPBase,
                          DSGatedMLPRegistry, DSInputNormBase, DSInputNormRegistry, DSLinearBase, DSLinearRegistry,
                          DSMixerBase, DSMixerRegistry, DSMoEBase, DSMoERegistry, DSOutputNormBase, DSOutputNormRegistry,
-                         DSPostNormBase, DSPostNormRegistry, DSPreNormBase, DSPreNormRegistry, DSSelfAttentionBase,
-                         DSSelfAttentionRegistry, DSUnembedBase, DSUnembedRegistry)
+                         DSPostNormBase, DSPostNormRegistry, DSPreNormBase, DSPreNormRegistry, DSSandwichNormBase,
+                         DSSandwichNormRegistry, DSSelfAttentionBase, DSSelfAttentionRegistry, DSUnembedBase,
+                         DSUnembedRegistry)
 
 _PLAIN_ACTS = ("gelu", "gelu_tanh", "relu", "silu")
 
@@ -296,8 +299,8 @@ class RaggedUnembed(DSUnembedBase):
         if tp > 1:
             parts = [torch.empty_like(logits) for _ in range(tp)]
             dist.all_gather(parts, logits, group=tp_group)
-            logits = torch.cat(parts, -1)[:, :vocab]
-        return logits
+            logits = torch.cat(parts, -1)[:, :vocab].contiguous()
+        return softcap_(logits, self._config.softcap) if self._config.softcap else logits
 
 
 # ---------------------------------------------------------------------------------------------------------------
@@ -351,7 +354,8 @@ class MinGRUMixer(DSMixerBase):
         return {"in.w": torch.cat([rows(w["z"]), rows(w["x"]), rows(w["g"])]), "o.w": cols(w["o"]),
                 "z.b": rows(w["z.b"]).float(), "x.b": rows(w["x.b"]).float()}
 
-    def forward(self, x, w, lin, out, batch, cache, state, offset):
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
+        lin = lins["in.w"]
         if batch.max_new == 1 and _is_plain(lin) and recur_step_ok(x, w["in.w"], self.FUSED_ROWS) and \
                 x.shape[0] == batch.current_sequences:
             return recur_step(x, w["in.w"], w["z.b"], w["x.b"], out, batch, state, offset)
@@ -360,9 +364,10 @@ class MinGRUMixer(DSMixerBase):
 
 @DSMixerRegistry.register_module
 class LatentAttentionMixer(DSMixerBase):
-    """Attention over compressed K/V rows, sliding window, interleaved rotation of a shared key part
-    (ops/latent_attention.py). Heads are sharded over the tensor-parallel group, the latent is computed on every
-    rank."""
+    """Attention over compressed K/V rows, sliding window, rotation of a shared key part, optionally queries through a
+    latent of their own and a gate per head (ops/latent_attention.py). Heads are sharded over the tensor-parallel group,
+    the latents are computed on every rank. The kernels turn neighbouring dimensions; the "half" rotation, which pairs i
+    with i + rot_dims / 2, becomes that by reordering the rotated rows of the query and key weights."""
 
     @staticmethod
     def name():
@@ -374,20 +379,47 @@ class LatentAttentionMixer(DSMixerBase):
         assert p["heads"] % config.tp == 0, "attention heads must divide the tensor-parallel size"
         self.shape = LatentShape(heads=p["heads"] // config.tp, dim=p["dim"], rot=p["rot_dim"], rot_dims=p["rot_dims"],
                                  rank=p["kv_rank"], vdim=p["vdim"], window=p["window"], scale=p["scale"],
-                                 eps=config.eps)
-        self.rope_base = p["rope_base"]
+                                 eps=config.eps, gated=p.get("gated", False))
+        self.rope_base, self.rope_scaling = p["rope_base"], p.get("rope_scaling")
+        self.half = p.get("rot_layout", "interleaved") == "half"
+        self.q_rank = p.get("q_rank", 0)  # 0: queries straight from the input
         self.out_width = self.shape.heads * self.shape.vdim
-        self.in_width = self.shape.q_width + self.shape.row
+        self.width = (self.q_rank or self.shape.q_width) + self.shape.row + (self.shape.heads if self.shape.gated else 0)
+        self.in_width = padded(self.width, 8) if self.q_rank or self.shape.gated else self.width
         self.cache_row = self.shape.row
         self.cos = self.sin = None
+
+    def extra_linears(self):
+        return {"uq.w": (self.q_rank, self.shape.q_width)} if self.q_rank else {}
+
+    def _turned(self, w):
+        """w [..., rot, in]: the rotated rows in the kernels' order."""
+        n = self.shape.rot_dims
+        if not self.half:
+            return w
+        order = [i for j in range(n // 2) for i in (j, j + n // 2)] + list(range(n, self.shape.rot))
+        return w[..., order, :]
 
     def bind_tables(self, cos, sin):
         self.cos, self.sin = cos, sin
 
     def shard(self, w, rows, cols):
-        # q, uk, uv are laid out head by head: equal row slices are whole heads
-        return {"in.w": torch.cat([rows(w["q"]), w["dkv"]]), "o.w": cols(w["o"]),
-                "ukv.w": torch.cat([rows(w["uk"]), rows(w["uv"])]), "dkv.norm": w["dkv.norm"].float()}
+        # q, uk, uv and the gate are laid out head by head: equal row slices are whole heads
+        sh = self.shape
+        q = rows(w["uq"] if self.q_rank else w["q"])
+        q = q.reshape(sh.heads, sh.dim + sh.rot, -1)
+        q = torch.cat([q[:, :sh.dim], self._turned(q[:, sh.dim:])], 1).reshape(sh.q_width, -1)
+        parts = [w["dq"] if self.q_rank else q, w["dkv"][:sh.rank], self._turned(w["dkv"][sh.rank:])]
+        if sh.gated:
+            parts.append(rows(w["g"]))
+        out = {"o.w": cols(w["o"]), "ukv.w": torch.cat([rows(w["uk"]), rows(w["uv"])]),
+               "dkv.norm": w["dkv.norm"].float()}
+        if self.q_rank:
+            out["uq.w"], out["dq.norm"] = q, w["dq.norm"].float()
+        if self.in_width > self.width:
+            parts.append(q.new_zeros(self.in_width - self.width, parts[0].shape[1]))
+        out["in.w"] = torch.cat(parts)
+        return out
 
     def _plan(self, batch):
         sh = self.shape
@@ -402,19 +434,27 @@ class LatentAttentionMixer(DSMixerBase):
                                                 expand, batch.tok_pos.device)
         return plan
 
-    def forward(self, x, w, lin, out, batch, cache, state, offset):
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
         sh = self.shape
         ukv = w["ukv.w"]
         uk = ukv[:sh.heads * sh.dim].view(sh.heads, sh.dim, sh.rank)
         uv = ukv[sh.heads * sh.dim:].view(sh.heads, sh.vdim, sh.rank)
-        return latent_attention(lin(x, w["in.w"]), sh, w["dkv.norm"], uk, uv, ukv, self.cos, self.sin, cache, batch,
-                                self._plan(batch), out)
+        y = lins["in.w"](x, w["in.w"])
+        n = self.q_rank or sh.q_width
+        q, ckr = y[:, :n], y[:, n:n + sh.row]
+        gate = y[:, n + sh.row:self.width] if sh.gated else None
+        if self.q_rank:
+            q = lins["uq.w"](rms_rows(q, w["dq.norm"], sh.eps), w["uq.w"])
+        return latent_attention(q, ckr, sh, w["dkv.norm"], uk, uv, ukv, self.cos, self.sin, cache, batch,
+                                self._plan(batch), out, gate)
 
 
 @DSMixerRegistry.register_module
 class HeadAttentionMixer(DSMixerBase):
-    """Grouped-query attention without rotation: sliding window, optional query / key norms, sink and output gate
-    (ops/paged.py ``head_attention``). Heads are sharded over the tensor-parallel group."""
+    """Grouped-query attention without rotation: sliding window or chunks, soft cap, optional query / key norms, sink (learned
+    or of score zero), output gate per head or element, and values mixed with those of an earlier layer (``value_mix``:
+    "source" leaves its values for the later ones of the step, "mix" takes them). ops/paged.py ``head_attention``. Heads
+    are sharded over the tensor-parallel group."""
 
     @staticmethod
     def name():
@@ -426,7 +466,11 @@ class HeadAttentionMixer(DSMixerBase):
         if p["heads"] % tp or p["kv_heads"] % tp or p["heads"] % p["kv_heads"]:
             raise ValueError(f"{p['heads']} / {p['kv_heads']} heads: not groups of equal size on {tp} ranks")
         self.shape = HeadShape(heads=p["heads"] // tp, kv_heads=p["kv_heads"] // tp, dim=p["dim"], vdim=p["vdim"],
-                               window=p["window"], scale=p["scale"], eps=config.eps, gated=p["gated"])
+                               window=p["window"], scale=p["scale"], eps=config.eps, gated=p["gated"],
+                               gate_width=p["vdim"] if p.get("gate_elements") else 1, chunk=p.get("chunk", 0),
+                               softcap=p.get("softcap", 0.0))
+        self.value_mix = p.get("value_mix")
+        self.zero_sink = p.get("zero_sink", False)
         self.out_width = self.shape.heads * p["vdim"]
         self.in_width = padded(self.shape.width, 8)  # 16-byte rows
         self.cache_row = self.shape.row
@@ -441,6 +485,10 @@ class HeadAttentionMixer(DSMixerBase):
         for k in ("q.norm", "k.norm"):
             out[k] = w[k].float() if k in w else None
         out["sink"] = rows(w["sink"]).float() if "sink" in w else None
+        if self.zero_sink:
+            out["sink"] = torch.zeros(self.shape.heads)
+        if self.value_mix == "mix":
+            out["vmix"] = w["vmix"].reshape(1).float()
         return out
 
     def _plan(self, batch):
@@ -453,9 +501,60 @@ class HeadAttentionMixer(DSMixerBase):
                                                      sh.heads, sh.kv_heads, blocks, batch.tok_pos.device)
         return plan
 
-    def forward(self, x, w, lin, out, batch, cache, state, offset):
-        return head_attention(lin(x, w["in.w"]), self.shape, w["q.norm"], w["k.norm"], w["sink"], cache, batch,
-                              self._plan(batch), out)
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
+        sh = self.shape
+        qkv = lins["in.w"](x, w["in.w"])
+        own = qkv[:, sh.qkv_width - sh.kv_heads * sh.vdim:sh.qkv_width]
+        if self.value_mix == "source":
+            batch.carry["values"] = own
+        first = batch.carry["values"] if self.value_mix == "mix" else None
+        return head_attention(qkv, sh, w["q.norm"], w["k.norm"], w["sink"], cache, batch, self._plan(batch), out, first,
+                              w["vmix"])
+
+
+@DSMixerRegistry.register_module
+class DeltaMixer(DSMixerBase):
+    """Gated delta rule with short convolutions (ops/delta_rule.py). Heads are sharded over the tensor-parallel group."""
+
+    @staticmethod
+    def name():
+        return "delta"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        p, tp = config.params, config.tp
+        if p["heads"] % tp or p["kv_heads"] % tp or p["heads"] % p["kv_heads"]:
+            raise ValueError(f"{p['heads']} / {p['kv_heads']} heads: not groups of equal size on {tp} ranks")
+        self.shape = DeltaShape(heads=p["heads"] // tp, kv_heads=p["kv_heads"] // tp, dim=p["dim"], vdim=p["vdim"],
+                                taps=p["conv"], eps=config.eps)
+        self.out_width = self.shape.heads * self.shape.vdim
+        self.in_width = padded(self.shape.width, 8)
+
+    def state_floats(self):
+        return padded(self.shape.state_floats, 4)
+
+    def shard(self, w, rows, cols):
+        # everything is laid out head by head: equal slices are whole heads
+        parts = [rows(w[k]) for k in ("q", "k", "v", "g", "b", "a")]
+        fill = self.in_width - self.shape.width
+        if fill:
+            parts.append(parts[0].new_zeros(fill, parts[0].shape[1]))
+        conv = torch.cat([rows(w[k + ".conv"]) for k in ("q", "k", "v")])
+        return {"in.w": torch.cat(parts), "o.w": cols(w["o"]), "conv.w": conv.float().t().contiguous(),
+                "A_log": rows(w["A_log"]).float(), "dt_bias": rows(w["dt_bias"]).float(), "norm": w["norm"].float()}
+
+    def _plan(self, batch):
+        single = batch.tok_pos.is_cuda and step_ok(self.shape)
+        key = ("delta", single)
+        plan = batch.plans.get(key)
+        if plan is None:
+            plan = batch.plans[key] = make_delta_plan(batch.seq_meta_host, batch.current_sequences, batch.max_new, single,
+                                                      batch.tok_pos.device)
+        return plan
+
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
+        return delta_rule(lins["in.w"](x, w["in.w"]), self.shape, w["conv.w"], w["A_log"], w["dt_bias"], w["norm"],
+                          state, offset, batch, self._plan(batch), out)
 
 
 @DSOutputNormRegistry.register_module
@@ -478,6 +577,22 @@ class RmsResidual(DSOutputNormBase):
 
     def forward(self, x, delta, gain):
         return residual_norm(x, delta, gain, self._config.eps, self._config.input_dtype, self._pad())
+
+
+@DSSandwichNormRegistry.register_module
+class RmsSandwich(DSSandwichNormBase):
+    """32-bit residual, RMS norms on both sides of every sublayer; the step between two sublayers is one kernel."""
+
+    @staticmethod
+    def name():
+        return "rms_sandwich"
+
+    @staticmethod
+    def supports_config(c):
+        return c.type == "rms"
+
+    def forward(self, x, delta, gain, next_gain, embed=None, idx=None):
+        return sandwich_norm(x, delta, gain, next_gain, self._config.eps, self._config.input_dtype, embed, idx)
 
 
 @DSExpertLayerRegistry.register_module
@@ -525,7 +640,8 @@ class RoutedExperts(DSExpertLayerBase):
 
 @DSGatedMLPRegistry.register_module
 class GatedMLPRows(DSGatedMLPBase):
-    """act(x gate^T) * (x up^T) into a column block: one GEMV for decode rows, else projection + activation kernel."""
+    """act(x gate^T) * (x up^T), or the clamped unit, into a column block: one GEMV for decode rows, else projection +
+    activation kernel."""
 
     FUSED_ROWS = 1
 
@@ -535,10 +651,10 @@ class GatedMLPRows(DSGatedMLPBase):
 
     @staticmethod
     def supports_config(c):
-        return c.activation in _PLAIN_ACTS
+        return c.activation in _PLAIN_ACTS + ("clamped", )
 
     def forward(self, x, w, lin, out):
-        act = self._config.activation
-        if x.shape[0] <= self.FUSED_ROWS and _is_plain(lin) and glu_gemv(x, w, act, out):
+        act, limit = self._config.activation, self._config.limit
+        if x.shape[0] <= self.FUSED_ROWS and _is_plain(lin) and glu_gemv(x, w, act, out, limit):
             return out
-        return glu_rows(lin(x, w), act, out)
+        return glu_rows(lin(x, w), act, out, limit)

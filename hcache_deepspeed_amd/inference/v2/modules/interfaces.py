@@ -40,17 +40,26 @@ class DSInputNormBase(DSModuleBase):
 class DSMixerBase(DSModuleBase):
     """Token mixer of one layer. ``in_width`` / ``out_width`` (this rank's); ``cache_row``: values a token stores in
     the paged cache; ``state_floats()``: unpaged float32 state per sequence; ``shard(weights, rows, cols)`` -> this
-    rank's weights, with the input projection "in.w" and the output projection "o.w";
-    forward(x, weights, lin, out, batch, cache, state, offset) fills ``out`` [T, out_width]."""
+    rank's weights, with the input projection "in.w" and the output projection "o.w"; ``extra_linears()``: further
+    products, name -> (in, out); forward(x, weights, lins, out, batch, cache, state, offset) fills ``out`` [T, out_width],
+    ``lins`` holds the linear modules by weight name, ``batch.carry`` what layers of a step hand to later ones."""
     cache_row = 0
 
     def state_floats(self):
         return 0
 
+    def extra_linears(self):
+        return {}
+
 
 class DSOutputNormBase(DSModuleBase):
     """forward(x32, delta, gain) -> (x32 + gain * norm(delta), the rows the next sublayer reads); delta: a matrix or the
     parts an expert layer returns. ``start(embed, ids, scale)`` -> the same pair for the step's tokens."""
+
+
+class DSSandwichNormBase(DSModuleBase):
+    """forward(x32, delta, gain, next_gain, embed, idx) -> (x32 + gain * norm(delta), next_gain * norm(of that)); x32 None:
+    the stream starts from ``embed`` (table, ids, scale); ``idx``: the second result of these rows only."""
 
 
 class DSExpertLayerBase(DSModuleBase):
@@ -86,4 +95,5 @@ DSInputNormRegistry = _registry(DSInputNormBase)
 DSMixerRegistry = _registry(DSMixerBase)
 DSGatedMLPRegistry = _registry(DSGatedMLPBase)
 DSOutputNormRegistry = _registry(DSOutputNormBase)
+DSSandwichNormRegistry = _registry(DSSandwichNormBase)
 DSExpertLayerRegistry = _registry(DSExpertLayerBase)

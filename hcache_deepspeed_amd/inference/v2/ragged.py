@@ -369,6 +369,7 @@ class RaggedBatchWrapper:
         self.slots_host = [seq.tracking_id for seq in self._seqs]
         self.max_new = int(n_new.max()) if S else 0
         self.plans = {}
+        self.carry = {}
         if self._logit_rows is not None:
             self.last_token_idx = take(len(self._logit_rows), (-1, ))
         self.tables_host = host[4 * S + 2 * T:4 * S + 2 * T + S * mb].view(S, mb).clone() if S else \

@@ -10,8 +10,9 @@ from . import native
 from ..offload import act_plan as _ap
 
 SILU, GELU_TANH, RELU, GELU, IDENTITY = 0, 1, 2, 3, 4
+CLAMPED = 5  # of gated units only (glu_rows): see clamped_unit
 _NAMES = {"silu": SILU, "swish": SILU, "gelu_tanh": GELU_TANH, "gelu_new": GELU_TANH, "gelu_pytorch_tanh": GELU_TANH,
-          "relu": RELU, "gelu": GELU, "identity": IDENTITY}
+          "relu": RELU, "gelu": GELU, "identity": IDENTITY, "clamped": CLAMPED}
 
 
 def act_code(name):
@@ -170,14 +171,23 @@ def bias_act(x, bias=None, act="gelu"):
     return _BiasActFn.apply(x, bias, act_code(act))
 
 
-def glu_rows(gu, act, out):
-    """``glu`` without autograd into ``out`` [T, I], a (possibly strided) column block; any width."""
+def clamped_unit(g, u, limit):
+    """g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit)."""
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return g * torch.sigmoid(1.702 * g) * (u + 1)
+
+
+def glu_rows(gu, act, out, limit=0.0):
+    """``glu`` without autograd into ``out`` [T, I], a (possibly strided) column block; any width. ``act`` "clamped":
+    ``clamped_unit`` with ``limit``."""
     I = out.shape[1]
     a = act_code(act)
     if native.use_native(gu):
         assert gu.stride(1) == 1 and out.stride(1) == 1 and gu.dtype == out.dtype
         native.check(native.kernels().hds_glu_rows(native.dt(gu), a, gu.data_ptr(), gu.stride(0), out.data_ptr(),
-                                                   out.stride(0), gu.shape[0], I, native.stream()), "glu_rows")
+                                                   out.stride(0), gu.shape[0], I, float(limit), native.stream()),
+                     "glu_rows")
         return out
-    out.copy_(_ref_act(gu[:, :I].float(), a) * gu[:, I:].float())
+    g, u = gu[:, :I].float(), gu[:, I:].float()
+    out.copy_(clamped_unit(g, u, limit) if a == CLAMPED else _ref_act(g, a) * u)
     return out

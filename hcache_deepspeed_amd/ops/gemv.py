@@ -136,7 +136,7 @@ def fused_gemv(h, w, res=None, gamma=None, eps=1e-5, glu=False, want_x=False, x_
             x = x_out.view(h2.shape) if ok_out else torch.empty_like(h2)
         native.check(native.kernels().hds_gemv_fused_bf16(
             h2.data_ptr(), native.ptr(res2), native.ptr(gamma), float(eps), w.data_ptr(), y.data_ptr(),
-            native.ptr(r if res2 is not None else None), native.ptr(x), int(bool(glu)), M, N, K, K, N,
+            native.ptr(r if res2 is not None else None), native.ptr(x), int(bool(glu)), 0.0, M, N, K, K, N,
             native.stream()), "gemv_fused_bf16")
         if gamma is None:
             x = h2
@@ -144,16 +144,17 @@ def fused_gemv(h, w, res=None, gamma=None, eps=1e-5, glu=False, want_x=False, x_
     return (y.view(*lead, N), r.view(shape), None if x is None or not want_x else x.view(shape))
 
 
-_GLU_GEMV_ACTS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
+_GLU_GEMV_ACTS = {"silu": 0, "gelu_tanh": 1, "relu": 2, "clamped": 5}
 
 
-def glu_gemv(x2, w, act, out):
-    """act(x . gate^T) * (x . up^T) of decode rows into ``out`` [M, I] (strided column block) in one kernel; ``w`` is
+def glu_gemv(x2, w, act, out, limit=0.0):
+    """act(x . gate^T) * (x . up^T) (or the clamped unit) of decode rows into ``out`` [M, I] (strided column block) in one kernel; ``w`` is
     [gate; up]. Returns False, with nothing written, for rows or weights the kernel does not take."""
     if act not in _GLU_GEMV_ACTS or not torch.is_tensor(w) or not fused_ok(x2, w, None, True):
         return False
     M, K = x2.shape
     native.check(native.kernels().hds_gemv_fused_bf16(x2.data_ptr(), None, None, 0.0, w.data_ptr(), out.data_ptr(),
-                                                      None, None, 1 + _GLU_GEMV_ACTS[act], M, w.shape[0] // 2, K,
+                                                      None, None, 1 + _GLU_GEMV_ACTS[act], float(limit), M,
+                                                      w.shape[0] // 2, K,
                                                       x2.stride(0), out.stride(0), native.stream()), "glu_gemv")
     return True

@@ -26,6 +26,7 @@ class LatentShape:
     window: int     # 0: every earlier token
     scale: float
     eps: float
+    gated: bool = False  # a gate per token and head multiplies the head's output
 
     @property
     def row(self):
@@ -106,28 +107,32 @@ def _rot(v, cos, sin, rdims):
     return out
 
 
-def latent_attention(qd, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, plan, out):
-    """qd: [T, q_width + rank + rot] projection (q heads, latent, shared key part; consumed). norm_w: [rank] float32;
-    uk: [H, dim, rank]; uv: [H, vdim, rank]; ukv: the two stacked, [H (dim + vdim), rank]. Appends the step's rows to
-    ``cache`` and writes the heads' values into ``out`` [T, H vdim] (unit column stride)."""
-    if not native.use_native(qd):
-        return _latent_attention_cpu(qd, shape, norm_w, uk, uv, cos, sin, cache, batch, out)
+def latent_attention(q, ckr, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, plan, out, gate=None):
+    """q: [T, q_width] projected query heads (consumed); ckr: [T, rank + rot] latent and shared key part. norm_w: [rank]
+    float32; uk: [H, dim, rank]; uv: [H, vdim, rank]; ukv: the two stacked, [H (dim + vdim), rank]; gate: [T, H] or None.
+    Appends the step's rows to ``cache`` and writes the heads' values into ``out`` [T, H vdim] (unit column strides)."""
+    assert (gate is not None) == shape.gated
+    if not native.use_native(q):
+        return _latent_attention_cpu(q, ckr, shape, norm_w, uk, uv, cos, sin, cache, batch, out, gate)
     sh, lib = shape, native.kernels()
-    T, dt, dev = qd.shape[0], native.dt(qd), qd.device
+    T, dt, dev = q.shape[0], native.dt(q), q.device
     H, bs, mb = sh.heads, cache.shape[1], batch.block_tables.shape[1]
-    assert qd.stride(1) == 1 and out.stride(1) == 1 and cache.dtype == qd.dtype == out.dtype
+    assert q.stride(1) == 1 and ckr.stride(1) == 1 and out.stride(1) == 1
+    assert cache.dtype == q.dtype == out.dtype == ckr.dtype and q.shape[1] == sh.q_width and ckr.shape[1] == sh.row
+    assert gate is None or (gate.dtype == q.dtype and gate.shape == (T, H) and gate.stride(1) == 1)
+    gp, ldg = native.ptr(gate), 0 if gate is None else gate.stride(0)
     assert cache.shape[2] == sh.row and cos.shape[1] == sh.rot_dims // 2
     n_abs = plan.n_abs
-    qa = torch.empty(n_abs, H, sh.row, dtype=qd.dtype, device=dev) if n_abs else None
-    ws = torch.empty(plan.ws_rows, sh.row, dtype=qd.dtype, device=dev) if plan.n_pre else None
+    qa = torch.empty(n_abs, H, sh.row, dtype=q.dtype, device=dev) if n_abs else None
+    ws = torch.empty(plan.ws_rows, sh.row, dtype=q.dtype, device=dev) if plan.n_pre else None
     native.check(
-        lib.hds_latent_prep(dt, qd.data_ptr(), qd.stride(0), norm_w.data_ptr(), cos.data_ptr(), sin.data_ptr(),
-                            cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(),
+        lib.hds_latent_prep(dt, q.data_ptr(), q.stride(0), ckr.data_ptr(), ckr.stride(0), norm_w.data_ptr(),
+                            cos.data_ptr(), sin.data_ptr(), cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(),
                             batch.block_tables.data_ptr(), native.ptr(plan.ws_row), native.ptr(ws), uk.data_ptr(),
                             native.ptr(plan.atok), native.ptr(qa), T, n_abs, cos.shape[0], mb, bs, H, sh.dim, sh.rot,
                             sh.rot_dims, sh.rank, float(sh.eps), native.stream()), "latent_prep")
     if n_abs:
-        mfma = int(qd.dtype == torch.bfloat16 and bool(lib.hds_latent_decode_mfma_ok(sh.rank, sh.rot)))
+        mfma = int(q.dtype == torch.bfloat16 and bool(lib.hds_latent_decode_mfma_ok(sh.rank, sh.rot)))
         cap = mb * bs
         keys = min(cap, sh.window) if sh.window else cap
         splits = lib.hds_latent_decode_splits(n_abs, H, sh.rank, sh.rot, mfma, keys)
@@ -140,7 +145,7 @@ def latent_attention(qd, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, pla
                                   float(sh.scale), mfma, native.stream()), "latent_decode")
         native.check(
             lib.hds_latent_combine(dt, part_o.data_ptr(), part_ml.data_ptr(), uv.data_ptr(), native.ptr(plan.atok),
-                                   out.data_ptr(), out.stride(0), n_abs, H, sh.rank, sh.vdim, splits,
+                                   out.data_ptr(), out.stride(0), gp, ldg, n_abs, H, sh.rank, sh.vdim, splits,
                                    native.stream()), "latent_combine")
     if plan.n_pre:
         copy_rows(cache, ws, plan.g_seq, plan.g_pos, batch.block_tables, plan.g_dst)
@@ -148,10 +153,11 @@ def latent_attention(qd, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, pla
         kr = ws[:, sh.rank:]
         o = out if out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0 else \
             torch.empty(T, out.shape[1], dtype=out.dtype, device=dev)
-        q = qd if qd.stride(0) % 8 == 0 else qd.narrow(1, 0, sh.q_width).contiguous()
+        if q.stride(0) % 8 or q.data_ptr() % 16:
+            q = q.clone(memory_format=torch.contiguous_format)
         native.check(
             lib.hds_latent_prefill(q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), kr.data_ptr(),
-                                   kr.stride(0), o.data_ptr(), o.stride(0), plan.meta.data_ptr(), plan.n_pre,
+                                   kr.stride(0), o.data_ptr(), o.stride(0), gp, ldg, plan.meta.data_ptr(), plan.n_pre,
                                    plan.max_pre, H, sh.dim, sh.rot, sh.rank, sh.vdim, sh.window, float(sh.scale),
                                    native.stream()), "latent_prefill")
         if o is not out:
@@ -160,12 +166,11 @@ def latent_attention(qd, shape, norm_w, uk, uv, ukv, cos, sin, cache, batch, pla
     return out
 
 
-def _latent_attention_cpu(qd, sh, norm_w, uk, uv, cos, sin, cache, batch, out):
-    H, dh, T = sh.heads, sh.dim + sh.rot, qd.shape[0]
+def _latent_attention_cpu(q, ckr, sh, norm_w, uk, uv, cos, sin, cache, batch, out, gate):
+    H, dh, T = sh.heads, sh.dim + sh.rot, q.shape[0]
     pos = batch.tok_pos.long()
-    q = qd[:, :sh.q_width].float().view(T, H, dh)
-    c = qd[:, sh.q_width:sh.q_width + sh.rank].float()
-    kr = qd[:, sh.q_width + sh.rank:].float()
+    q = q.float().reshape(T, H, dh)
+    c, kr = ckr.float().split([sh.rank, sh.rot], 1)
     c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + sh.eps) * norm_w
     row = torch.cat([c, _rot(kr, cos[pos], sin[pos], sh.rot_dims)], 1).to(cache.dtype)
     copy_rows(cache, row, batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
@@ -186,5 +191,8 @@ def _latent_attention_cpu(qd, sh, norm_w, uk, uv, cos, sin, cache, batch, out):
             hide |= j[None] <= i[:, None] - sh.window
         p = torch.softmax(sc.masked_fill(hide[None], float("-inf")), -1)
         o = torch.einsum("htj,jr->thr", p, k[:, :sh.rank])
-        out[q0:q0 + n] = torch.einsum("thr,hvr->thv", o, uv.float()).reshape(n, -1).to(out.dtype)
+        o = torch.einsum("thr,hvr->thv", o, uv.float())
+        if gate is not None:
+            o = o * torch.sigmoid(gate[q0:q0 + n].float())[..., None]
+        out[q0:q0 + n] = o.reshape(n, -1).to(out.dtype)
     return out

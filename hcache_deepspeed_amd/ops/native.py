@@ -26,9 +26,12 @@ _KERNEL_SIGS = {
     "hds_rope": "ii" + "pppp" + "l" + "iii" + "l" + "ii" + "f" + "s",
     "hds_glu_fwd": "iipplis",
     "hds_glu_bwd": "iippplis",
-    "hds_glu_rows": "ii" + "plpl" + "li" + "s",
+    "hds_glu_rows": "ii" + "plpl" + "li" + "f" + "s",
     "hds_input_norm": "i" + "ppppp" + "pipp" + "pipp" + "p" + "l" + "pp" + "iiiii" + "f" + "s",
     "hds_residual_norm": "i" + "ppp" + "l" + "pl" + "p" + "ii" + "f" + "s",
+    "hds_sandwich_norm": "i" + "ppp" + "f" + "pl" + "ppppp" + "iii" + "f" + "s",
+    "hds_row_norm": "i" + "pl" + "ppl" + "ii" + "f" + "s",
+    "hds_softcap": "i" + "p" + "l" + "f" + "s",
     "hds_experts_norm": "i" + "ppp" + "l" + "pp" + "pl" + "ppp" + "pl" + "pl" + "iiiii" + "f" + "s",
     "hds_embed_rows": "i" + "pp" + "f" + "pp" + "l" + "iii" + "s",
     "hds_router_logits": "pl" + "p" + "pl" + "iii" + "s",
@@ -41,14 +44,17 @@ _KERNEL_SIGS = {
     "hds_experts_gemm": "pl" + "pi" + "pp" + "i" + "pppp" + "iiiiiii" + "s",
     "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
     "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "pp" + "iii" + "s",
+    "hds_delta_step_ok": "ii",
+    "hds_delta_step": "i" + "pl" + "pppp" + "pl" + "ppp" + "pl" + "iiiiii" + "f" + "s",
+    "hds_delta_scan": "i" + "pl" + "pppp" + "pl" + "ppp" + "pppp" + "pl" + "i" * 7 + "f" + "s",
     "hds_gemv_recur_bf16": "ppppp" + "pl" + "pp" + "iii" + "ll" + "s",
-    "hds_latent_prep": "i" + "pl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
+    "hds_latent_prep": "i" + "plpl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
     "hds_latent_decode_mfma_ok": "ii",
     "hds_latent_decode_splits": "iiiiii",
     "hds_latent_decode": "i" + "p" * 8 + "i" * 8 + "f" + "i" + "s",
-    "hds_latent_combine": "i" + "ppppp" + "l" + "iiiii" + "s",
+    "hds_latent_combine": "i" + "ppppp" + "l" + "pl" + "iiiii" + "s",
     "hds_latent_prefill_ok": "iiii",
-    "hds_latent_prefill": "plplplpl" + "p" + "i" * 8 + "f" + "s",
+    "hds_latent_prefill": "plplplplpl" + "p" + "i" * 8 + "f" + "s",
     "hds_glu_fwd_t": "i" + "ppp" + "ii" + "s",
     "hds_glu_bwd_t": "i" + "pppp" + "ii" + "s",
     "hds_bias_act_fwd": "iippplis",
@@ -75,10 +81,10 @@ _KERNEL_SIGS = {
     "hds_bsattn_fwd": "p" * 8 + "i" * 7 + "f" + "i" + "s",
     "hds_bsattn_bwd": "p" * 15 + "i" * 7 + "f" + "i" + "s",
     "hds_kv_rope_scatter": "i" + "p" + "l" + "pppp" + "i" + "pp" + "i" * 8 + "s",
-    "hds_head_norm_scatter": "i" + "pl" + "pppppp" + "iiiiiii" + "f" + "s",
+    "hds_head_norm_scatter": "i" + "pl" + "pppppp" + "iiiiiii" + "f" + "plp" + "s",
     "hds_paged_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
     "hds_paged_attn_supported": "ii",
-    "hds_paged_attn": "pl" + "p" + "pl" + "pi" + "pp" + "i" * 6 + "f" + "i" + "pp" + "l" + "s",
+    "hds_paged_attn": "pl" + "p" + "pl" + "pi" + "pp" + "i" * 6 + "f" + "ii" + "f" + "pp" + "li" + "s",
     "hds_paged_rows_per_atom": "",
     "hds_moe_dispatch": "i" + "pppp" + "iiii" + "s",
     "hds_moe_dispatch_bwd": "i" + "pppp" + "iiii" + "s",
@@ -97,7 +103,7 @@ _KERNEL_SIGS = {
     "hds_transpose_bf16_var": "pp" + "ii" + "l" + "i" + "s",
     "hds_gemv_bf16_supported": "iii",
     "hds_gemv_bf16": "pppp" + "iii" + "ll" + "s",
-    "hds_gemv_fused_bf16": "ppp" + "f" + "pppp" + "iiii" + "ll" + "s",
+    "hds_gemv_fused_bf16": "ppp" + "f" + "pppp" + "if" + "iii" + "ll" + "s",
     "hds_skinny_gemm_bf16": "pppp" + "iii" + "ll" + "s",
     "hds_skinny_set_unroll": "i",
     "hds_wmix_splits": "iii",
@@ -125,7 +131,7 @@ _KERNEL_SIGS = {
     "hds_nhwc_bias_add": "i" + "ppppp" + "l" + "ii" + "s",
     "hds_paged_decode_supported": "ii",
     "hds_paged_decode_splits": "iii",
-    "hds_paged_decode": "ii" + "pl" + "p" + "pl" + "pp" + "ppppp" + "i" * 8 + "f" + "i" + "pp" + "l" + "p" + "s",
+    "hds_paged_decode": "ii" + "pl" + "p" + "pl" + "pp" + "ppppp" + "i" * 8 + "f" + "ii" + "f" + "pp" + "li" + "p" + "s",
     "hds_copy_d2h": "pp" + "l" + "i" + "s",
     "hds_latent_slot_store": "p" + "l" + "pp" + "l" + "i" + "l" + "s",
     "hds_slot_advance": "p" + "i" + "s",

@@ -4,7 +4,9 @@
 plain matrix or an :class:`ops.experts.ExpertSum`, the parts of a routed expert layer's output, which the kernel sums on
 the way in. It returns the new residual and the rows the next sublayer reads: rounded to the activations' type and
 zero-padded to a multiple of ``pad`` columns (the 32-bit rows themselves where that changes nothing). ``embed_rows``
-starts the stream, ``norm_rows`` is the output norm of selected rows. CPU tensors run the torch implementations."""
+starts the stream, ``norm_rows`` is the output norm of selected rows. ``sandwich_norm`` is the step between two sublayers
+with a norm on both sides: the residual sum of the first one's normed output and the second one's norm in one kernel.
+``rms_rows`` norms column blocks, ``softcap_`` bounds logits. CPU tensors run the torch implementations."""
 import torch
 
 from . import native
@@ -106,3 +108,59 @@ def norm_rows(x, delta, idx, gain, eps, dtype=None):
         h = h + delta[idx.long()].float()
     y.copy_(h / torch.sqrt((h * h).mean(-1, keepdim=True) + eps) * gain)
     return y
+
+
+def _rms(x, eps):
+    return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+
+def sandwich_norm(x, delta, gain, next_gain, eps, dtype, embed=None, idx=None):
+    """(x' = x + gain * norm(delta), next_gain * norm(x') in ``dtype``). x: [T, W] float32, updated in place; or None, then
+    ``embed`` = (table, ids, scale) starts the stream. delta: [T, W] of ``dtype`` or None (x' = x). gains: [W] float32.
+    ``idx`` (int32): only these rows, and the first result is None."""
+    table, ids, scale = embed if x is None else (None, None, 1.0)
+    W = table.shape[1] if x is None else x.shape[1]
+    n = idx.numel() if idx is not None else (ids.numel() if x is None else x.shape[0])
+    dev = table.device if x is None else x.device
+    out = None if idx is not None else (x if x is not None else torch.empty(n, W, dtype=torch.float32, device=dev))
+    y = torch.empty(n, W, dtype=dtype, device=dev)
+    if native.use_native(y):
+        assert delta is None or (delta.dtype == dtype and delta.stride(1) == 1 and gain.numel() == W)
+        assert next_gain.numel() == W and (x is None or x.is_contiguous()) and (table is None or table.dtype == dtype)
+        native.check(
+            native.kernels().hds_sandwich_norm(
+                native.dt(dtype), native.ptr(x), native.ptr(table), native.ptr(ids), float(scale), native.ptr(delta),
+                0 if delta is None else delta.stride(0), native.ptr(gain), next_gain.data_ptr(), native.ptr(idx),
+                native.ptr(out), y.data_ptr(), n, W, 0 if table is None else table.shape[0], float(eps),
+                native.stream()), "sandwich_norm")
+        return out, y
+    h = table[ids].float() * scale if x is None else x
+    if idx is not None:
+        h, delta = h[idx.long()], None if delta is None else delta[idx.long()]
+    if delta is not None:
+        h = h + gain * _rms(delta.float(), eps)
+    if out is not None:
+        out.copy_(h)
+    return out, y.copy_(next_gain * _rms(h, eps))
+
+
+def rms_rows(x, gain, eps):
+    """gain * norm(x) of rows [T, W] (any row stride), contiguous."""
+    y = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    if native.use_native(x):
+        assert x.stride(1) == 1 and gain.numel() == x.shape[1]
+        native.check(
+            native.kernels().hds_row_norm(native.dt(x), x.data_ptr(), x.stride(0), gain.data_ptr(), y.data_ptr(),
+                                          y.stride(0), x.shape[0], x.shape[1], float(eps), native.stream()), "row_norm")
+        return y
+    return y.copy_(gain * _rms(x.float(), eps))
+
+
+def softcap_(x, cap):
+    """cap * tanh(x / cap) in place (contiguous)."""
+    if native.use_native(x):
+        assert x.is_contiguous()
+        native.check(native.kernels().hds_softcap(native.dt(x), x.data_ptr(), x.numel(), float(cap), native.stream()),
+                     "softcap")
+        return x
+    return x.copy_(cap * torch.tanh(x.float() / cap))

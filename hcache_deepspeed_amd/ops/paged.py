@@ -1,5 +1,6 @@
 """Paged-KV serving ops: fused RoPE + KV scatter, ragged paged attention (HIP, csrc/kernels/paged_attn.hip), and
-``head_attention``: attention with normed unrotated heads, a window, a sink and an output gate over the same kernels.
+``head_attention``: attention with unrotated heads (optionally normed), a window or chunks, a soft cap, a sink, value mixing
+and an output gate over the same kernels.
 
 Reference parity: inference/v2/kernels/ragged_ops/linear_blocked_kv_rotary (``LinearBlockedKVCopy``,
 ``BlockedRotaryEmbeddings``) and ragged_ops/blocked_flash (``BlockedFlashAttn``) + atom_builder.
@@ -123,13 +124,13 @@ def paged_attention(q, cache, atoms, n_atoms, seq_meta, block_tables, n_q, n_kv,
                 lib.hds_paged_decode(native.dt(q), 0, q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(),
                                      n_q * D, native.ptr(part_o), native.ptr(part_ml), seq_meta.data_ptr(), None, None,
                                      None, block_tables.data_ptr(), block_tables.shape[1], cache.shape[1], n_seqs, n_q,
-                                     n_kv, D, D, splits, float(scale), int(window), None, None, 0, counters,
+                                     n_kv, D, D, splits, float(scale), int(window), 0, 0.0, None, None, 0, 1, counters,
                                      native.stream()), "paged_decode")
             return o
         native.check(
             lib.hds_paged_attn(q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(), n_q * D, atoms.data_ptr(),
                                n_atoms, seq_meta.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
-                               cache.shape[1], n_q, n_kv, D, D, float(scale), int(window), None, None, 0,
+                               cache.shape[1], n_q, n_kv, D, D, float(scale), int(window), 0, 0.0, None, None, 0, 1,
                                native.stream()), "paged_attn")
         return o
     meta = seq_meta_host if seq_meta_host is not None else seq_meta.tolist()
@@ -180,7 +181,7 @@ def copy_rows(cache, rows, seq, pos, tables, dst_row=None, to_cache=False):
 
 
 # -----------------------------------------------------------------------------------------------------------------
-# normed heads, window, sink, output gate
+# unrotated heads: norms, window, chunks, soft cap, sink, value mixing, output gate
 # -----------------------------------------------------------------------------------------------------------------
 @dataclass(frozen=True)
 class HeadShape:
@@ -191,11 +192,20 @@ class HeadShape:
     window: int     # 0: every earlier token
     scale: float
     eps: float      # of the query / key norms
-    gated: bool     # the projection ends with one gate column per query head
+    gated: bool     # the projection ends with gate columns, one per query head
+    gate_width: int = 1   # .. or, vdim: one per element of the heads' outputs
+    chunk: int = 0        # positions see their own run of this many, counted from the sequence's start; 0: no chunks
+    softcap: float = 0.0  # 0: none
 
     @property
     def row(self):
         return self.kv_heads * (self.dim + self.vdim)
+
+    @property
+    def span(self):
+        """The most keys a position sees; 0: no bound."""
+        bounds = [b for b in (self.window, self.chunk) if b]
+        return min(bounds) if bounds else 0
 
     @property
     def qkv_width(self):
@@ -203,7 +213,7 @@ class HeadShape:
 
     @property
     def width(self):
-        return self.qkv_width + (self.heads if self.gated else 0)
+        return self.qkv_width + (self.heads * self.gate_width if self.gated else 0)
 
 
 # Sequences with at most this many new tokens run token by token on the split-key kernel, the others in row blocks on
@@ -249,13 +259,14 @@ def head_blocks_ok(shape, dtype):
     return dtype == torch.bfloat16 and bool(native.kernels().hds_paged_attn_supported(shape.dim, shape.vdim))
 
 
-def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out):
+def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, values=None, mix=None):
     """qkv: [T, >= shape.width] projection, row by row q heads | k heads | v heads | gates (consumed). q_norm / k_norm:
     [dim] float32 or None; sink: [heads] float32 or None; cache: [blocks, block_size, shape.row]. Appends the step's keys
-    and values to ``cache`` and writes the gated heads into ``out`` [T, heads * vdim] (unit column stride)."""
+    and values to ``cache`` and writes the gated heads into ``out`` [T, heads * vdim] (unit column stride). ``values``:
+    [T, kv_heads * vdim] values of another layer, of which the share ``mix`` ([1] float32) goes into this layer's."""
     sh, T = shape, qkv.shape[0]
     if not native.use_native(qkv):
-        return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out)
+        return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values, mix)
     lib, st, dt = native.kernels(), native.stream(), native.dt(qkv)
     bs, tab = cache.shape[1], batch.block_tables
     mb = tab.shape[1]
@@ -264,15 +275,18 @@ def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out):
     native.check(
         lib.hds_head_norm_scatter(dt, qkv.data_ptr(), qkv.stride(0), native.ptr(q_norm), native.ptr(k_norm),
                                   cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(),
-                                  T, mb, bs, sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.eps), st),
+                                  T, mb, bs, sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.eps),
+                                  native.ptr(values), 0 if values is None else values.stride(0),
+                                  None if values is None else mix.data_ptr(), st),
         "head_norm_scatter")
     gate = qkv.data_ptr() + qkv.element_size() * sh.qkv_width if sh.gated else None
+    assert values is None or (values.shape == (T, sh.kv_heads * sh.vdim) and values.dtype == qkv.dtype)
     fast = head_blocks_ok(sh, qkv.dtype) and qkv.stride(0) % 8 == 0 and out.stride(0) % 8 == 0 and \
         qkv.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0
     assert fast or not plan.n_atoms
     if plan.n_dec:
         n = plan.n_dec
-        keys = min(mb * bs, sh.window) if sh.window else mb * bs
+        keys = min(mb * bs, sh.span) if sh.span else mb * bs
         splits = lib.hds_paged_decode_splits(n, sh.kv_heads if fast else sh.heads, keys)
         part_o = part_ml = None
         if splits > 1:
@@ -283,17 +297,19 @@ def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out):
                                  out.stride(0), native.ptr(part_o), native.ptr(part_ml), None, native.ptr(plan.toks),
                                  batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(), mb, bs, n,
                                  sh.heads, sh.kv_heads, sh.dim, sh.vdim, splits, float(sh.scale), sh.window,
-                                 native.ptr(sink), gate, qkv.stride(0), None, st), "paged_decode")
+                                 sh.chunk, float(sh.softcap), native.ptr(sink), gate, qkv.stride(0), sh.gate_width,
+                                 None, st), "paged_decode")
     if plan.n_atoms:
         native.check(
             lib.hds_paged_attn(qkv.data_ptr(), qkv.stride(0), cache.data_ptr(), out.data_ptr(), out.stride(0),
                                plan.atoms.data_ptr(), plan.n_atoms, batch.seq_meta.data_ptr(), tab.data_ptr(), mb, bs,
-                               sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, native.ptr(sink),
-                               gate, qkv.stride(0), st), "paged_attn")
+                               sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, sh.chunk,
+                               float(sh.softcap), native.ptr(sink), gate, qkv.stride(0), sh.gate_width, st),
+            "paged_attn")
     return out
 
 
-def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out):
+def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values=None, mix=None):
     T, H, G = qkv.shape[0], sh.heads, sh.kv_heads
 
     def normed(v, w):
@@ -302,26 +318,36 @@ def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out):
     q, k, v = qkv[:, :sh.qkv_width].float().split([H * sh.dim, G * sh.dim, G * sh.vdim], 1)
     q = normed(q.reshape(T, H, sh.dim), q_norm)
     k = normed(k.reshape(T, G, sh.dim), k_norm).reshape(T, -1)
+    if values is not None:
+        v = (1 - mix) * v + mix * values.float()
     copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
-    gate = torch.sigmoid(qkv[:, sh.qkv_width:sh.width].float()) if sh.gated else torch.ones(T, H)
+    gate = torch.ones(T, H, 1)
+    if sh.gated:
+        gate = torch.sigmoid(qkv[:, sh.qkv_width:sh.width].float()).reshape(T, H, sh.gate_width)
     bs = cache.shape[1]
     for s, (q0, n, seen) in enumerate(batch.seq_meta_host):
         if n == 0:
             continue
         lo = max(0, seen - sh.window + 1) if sh.window else 0
+        if sh.chunk:
+            lo = max(lo, seen - seen % sh.chunk)
         j = torch.arange(lo, seen + n)
         rows = cache[batch.block_tables[s, j // bs].long(), j % bs].float()
         kk = rows[:, :G * sh.dim].view(-1, G, sh.dim).repeat_interleave(H // G, 1)
         vv = rows[:, G * sh.dim:].reshape(-1, G, sh.vdim).repeat_interleave(H // G, 1)
         sc = torch.einsum("thd,jhd->htj", q[q0:q0 + n], kk) * sh.scale
+        if sh.softcap:
+            sc = sh.softcap * torch.tanh(sc / sh.softcap)
         i = seen + torch.arange(n)
         hide = j[None] > i[:, None]
         if sh.window:
             hide |= j[None] <= i[:, None] - sh.window
+        if sh.chunk:
+            hide |= j[None] < (i - i % sh.chunk)[:, None]
         sc = sc.masked_fill(hide[None], float("-inf"))
         if sink is not None:
             sc = torch.cat([sc, sink.view(H, 1, 1).expand(H, n, 1)], -1)
         p = torch.softmax(sc, -1)[..., :j.numel()]
-        o = torch.einsum("htj,jhd->thd", p, vv) * gate[q0:q0 + n, :, None]
+        o = torch.einsum("htj,jhd->thd", p, vv) * gate[q0:q0 + n]
         out[q0:q0 + n] = o.reshape(n, -1).to(out.dtype)
     return out

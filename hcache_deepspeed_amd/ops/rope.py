@@ -3,7 +3,7 @@
 Reference parity: ``apply_rotary_pos_emb`` (csrc/transformer/inference/csrc/apply_rotary_pos_emb.cu,
 ops/transformer/inference/op_binding) and the rotary part of ``kv_rotary_pos_kernel``
 (inference/v2/kernels/ragged_ops/linear_blocked_kv_rotary). Supports Llama-3 frequency scaling
-(rope_type="llama3") and linear scaling.
+(rope_type="llama3"), YaRN (rope_type="yarn") and linear scaling.
 """
 import math
 
@@ -31,7 +31,27 @@ def rope_inv_freq(rot_dim, base=10000.0, scaling=None):
             scaled = torch.where(wl > lo_wl, inv / factor, inv)
             mid = (wl <= lo_wl) & (wl >= hi_wl)
             inv = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
+        elif kind == "yarn":
+            # pairs that turn more than beta_fast times over the original context keep their frequency, those that turn
+            # less than beta_slow times get it divided by the factor, a linear ramp over the pairs between
+            old = float(scaling["original_max_position_embeddings"])
+
+            def pair_of(turns):
+                return rot_dim * math.log(old / (2 * math.pi * turns)) / (2 * math.log(base))
+
+            lo = max(math.floor(pair_of(float(scaling.get("beta_fast", 32.0)))), 0)
+            hi = min(math.ceil(pair_of(float(scaling.get("beta_slow", 1.0)))), rot_dim - 1)
+            ramp = ((torch.arange(rot_dim // 2, dtype=torch.float64) - lo) / max(hi - lo, 1e-3)).clamp(0, 1)
+            inv = inv / float(scaling["factor"]) * ramp + inv * (1 - ramp)
     return inv
+
+
+def rope_amplitude(scaling=None):
+    """What cos and sin are multiplied with (YaRN: 0.1 ln(factor) + 1, or its attention_factor)."""
+    if not scaling or scaling.get("rope_type", scaling.get("type")) != "yarn":
+        return 1.0
+    given = scaling.get("attention_factor")
+    return 0.1 * math.log(float(scaling["factor"])) + 1.0 if given is None else float(given)
 
 
 def rope_tables(max_pos, rot_dim, base=10000.0, scaling=None, device="cpu"):
@@ -41,8 +61,8 @@ def rope_tables(max_pos, rot_dim, base=10000.0, scaling=None, device="cpu"):
     if t is None:
         inv = rope_inv_freq(rot_dim, base, scaling)
         pos = torch.arange(max_pos, dtype=torch.float64)
-        ang = torch.outer(pos, inv)
-        t = (ang.cos().float().contiguous().to(device), ang.sin().float().contiguous().to(device))
+        ang, amp = torch.outer(pos, inv), rope_amplitude(scaling)
+        t = tuple((amp * f).float().contiguous().to(device) for f in (ang.cos(), ang.sin()))
         _CACHE[key] = t
     return t
 

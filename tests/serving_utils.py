@@ -62,6 +62,7 @@ class Pages:
         b.block_tables = torch.stack([self.tables[s] for s, _, _ in seqs]).to(self.device).contiguous()
         b.slots_host = [self.slots[s] for s, _, _ in seqs]
         b.slots, b.max_new, b.plans = i32(b.slots_host), max(n for _, n, _ in seqs), {}
+        b.carry = {}
         return b
 
 

@@ -187,8 +187,8 @@ def _run_attention(sh, m, qds, w, sizes, dev, dtype, absorb_max=None, block_size
         out = torch.zeros(qd.shape[0], sh.heads * sh.vdim + 8, dtype=dtype, device=dev)
         expand = dev.type == "cuda" and can_expand(sh, dtype)
         plan = make_plan(b.seq_meta_host, b.current_tokens, sh.window, expand, dev, absorb_max)
-        latent_attention(qd, sh, w["dkv.norm"].float().to(dev), uk, uv, ukv, cos, sin, pages.cache, b, plan,
-                         out[:, :sh.heads * sh.vdim])
+        latent_attention(qd[:, :sh.q_width], qd[:, sh.q_width:], sh, w["dkv.norm"].float().to(dev), uk, uv, ukv, cos, sin,
+                         pages.cache, b, plan, out[:, :sh.heads * sh.vdim])
         assert (out[:, sh.heads * sh.vdim:] == 0).all()
         for i, (s, n, _) in enumerate(step):
             q0 = b.seq_meta_host[i][0]
