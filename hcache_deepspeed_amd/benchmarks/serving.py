@@ -1,7 +1,7 @@
 """Prefill and decode throughput of the ragged serving engine on random weights of a real model's layer sizes: the hybrid
-design (Gofasun) next to the dense Llama layout at equal width, depth, feed-forward and head count, and the post-norm
-routed design (Buvuzen) next to the Qwen2-MoE layout at equal width, depth, heads and experts (``bench.py --serving``).
-One JSON line per measurement."""
+designs (Gofasun, Fifotar) next to the dense Llama layout at equal width, depth, feed-forward and head count, and the
+post-norm routed design (Buvuzen) next to the Qwen2-MoE layout at equal width, depth, heads and experts
+(``bench.py --serving``). One JSON line per measurement."""
 import json
 import time
 
@@ -115,6 +115,54 @@ def buvuzen_model(size, layers, dev):
     return spec, convert_hf(w, spec)
 
 
+FIFOTAR = ("attention", "delta", "latent_attention", "delta")
+
+
+def fifotar_model(size, layers, dev, kinds=FIFOTAR):
+    from ..inference.v2.arch import convert_hf, spec_from_hf
+    W, ff, H, G = SIZES[size]
+    rank, qrank, taps = W // 8, W // 4, 4
+    mixers = {"delta": {"heads": H, "kv_heads": H // 2, "dim": HEAD, "vdim": HEAD, "conv": taps},
+              "latent_attention": {"heads": H, "dim": HEAD, "rot_dim": ROT, "kv_rank": rank, "q_rank": qrank,
+                                   "vdim": HEAD, "scale": (HEAD + ROT)**-0.5,
+                                   "rot": {"base": 500000.0, "dims": ROT, "scaling": {
+                                       "factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 4096}}},
+              # as many keys as the other models see
+              "attention": {"heads": H, "kv_heads": G, "dim": HEAD, "vdim": HEAD, "scale": HEAD**-0.5, "softcap": 50.0,
+                            "v_mix": True, "mask": {"size": 2 * WINDOW}}}
+    cfg = {"architecture": "Fifotar", "vocab": VOCAB, "width": W, "norm": {"eps": 1e-5}, "embedding": {"scale": W**0.5},
+           "residual_mult": 0.5, "logit_softcap": 30.0,
+           "layers": [{"type": kinds[i % len(kinds)], "mixer": mixers[kinds[i % len(kinds)]],
+                       "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}} for i in range(layers)]}
+    g = torch.Generator(device=dev).manual_seed(0)
+    w = {"embed": _rand(g, dev, VOCAB, W), "final.norm": torch.ones(W, device=dev)}
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        for k in ("norm1", "norm1b", "norm2", "norm2b"):
+            w[p + k] = torch.ones(W, device=dev)
+        shapes = {"mlp.gate": (ff, W), "mlp.up": (ff, W), "mlp.down": (W, ff), "mix.o": (W, H * HEAD)}
+        if e["type"] == "delta":
+            D = H // 2 * HEAD
+            shapes.update({"mix.q": (D, W), "mix.k": (D, W), "mix.v": (H * HEAD, W), "mix.g": (H * HEAD, W),
+                           "mix.b": (H, W), "mix.a": (H, W)})
+            for k, n in (("q", D), ("k", D), ("v", H * HEAD)):
+                w[f"{p}mix.{k}.conv"] = _rand(g, dev, n, taps, scale=0.5)
+            w[p + "mix.A_log"], w[p + "mix.dt_bias"] = _rand(g, dev, H, scale=1.0), _rand(g, dev, H, scale=1.0)
+            w[p + "mix.norm"] = torch.ones(HEAD, device=dev)
+        elif e["type"] == "latent_attention":
+            shapes.update({"mix.dq": (qrank, W), "mix.uq": (H * (HEAD + ROT), qrank), "mix.dkv": (rank + ROT, W),
+                           "mix.uk": (H * HEAD, rank), "mix.uv": (H * HEAD, rank), "mix.g": (H, W)})
+            w[p + "mix.dq.norm"], w[p + "mix.dkv.norm"] = torch.ones(qrank, device=dev), torch.ones(rank, device=dev)
+        else:
+            shapes.update({"mix.q": (H * HEAD, W), "mix.k": (G * HEAD, W), "mix.v": (G * HEAD, W),
+                           "mix.g": (H * HEAD, W)})
+            w[p + "mix.vmix"] = torch.tensor(0.5, device=dev)
+        for k, s in shapes.items():
+            w[p + k] = _rand(g, dev, *s)
+    spec = spec_from_hf(cfg)
+    return spec, convert_hf(w, spec)
+
+
 def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
     from ..inference.v2.engine import InferenceEngineV2, RaggedInferenceEngineConfig
     if kind == "llama":
@@ -123,6 +171,10 @@ def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
         spec, w = moe_model(size, layers, dev, max_context)
     elif kind == "buvuzen":
         spec, w = buvuzen_model(size, layers, dev)
+    elif kind.startswith("fifotar"):
+        kinds = {"fifotar": FIFOTAR, "fifotar-delta": ("delta", ), "fifotar-latent": ("latent_attention", ),
+                 "fifotar-attention": ("attention", )}[kind]
+        spec, w = fifotar_model(size, layers, dev, kinds)
     else:
         kinds = {"gofasun": ("mingru", "latent_attention"), "gofasun-mingru": ("mingru", ),
                  "gofasun-latent": ("latent_attention", )}[kind]

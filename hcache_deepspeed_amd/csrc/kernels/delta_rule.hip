@@ -14,6 +14,10 @@
 //
 // Single tokens run one kernel, a workgroup per (sequence, head): delta_step. Portions run delta_conv (convolutions,
 // factors of the unit norms, log decays and betas), a scan over the tokens, and delta_out (norm and gate of the heads).
+// The scan goes token by token (delta_scan: short portions, 32-bit engines, any sizes) or by chunks on the matrix cores
+// (delta_chunk_prep, delta_chunk_scan).
+#include <type_traits>
+
 #include "hds_common.h"
 
 namespace {
@@ -285,6 +289,316 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams<T> p) {
 }
 
 // ---------------------------------------------------------------------------------------------------------------
+// scan by chunks of 64 tokens
+// ---------------------------------------------------------------------------------------------------------------
+// With G_i the sum of the log decays of a chunk's tokens up to i, S the state before the chunk and u_i as above,
+//
+//   (1 + L) U = beta V - diag(beta e^G) K S,      L_ij = beta_i e^(G_i - G_j) k_i . k_j   (j < i)
+//   O         = diag(e^G) Q S + A U,              A_ij = e^(G_i - G_j) q_i . k_j          (j <= i)
+//   S        <- e^G_last S + sum_j e^(G_last - G_j) k_j u_j^T
+//
+// delta_chunk_prep, all chunks at once: 16 x 16 blocks of -L below the diagonal, the inverses of the diagonal blocks of
+// 1 + L, the blocks of A, and the factors per token. delta_chunk_scan, a wave per 16 columns of a head's state: walks the
+// chunks with S in registers. Everything is 32-bit: q and k are bfloat16 up to a 32-bit factor per token, so products
+// among them are exact on the bfloat16 matrix cores; S and U enter their products with q and k as sums of three bfloat16
+// numbers (24 bits); the blocks of L and A multiply U on the 32-bit matrix cores.
+//
+// An accumulator tile (lane: column l & 15, rows 4 (l >> 4) + r) is the right operand of the next product as it is, if the
+// left operand takes its contraction index in the same order: f32 step r contracts rows 4 (l >> 4) + r of a 16-row block,
+// a bf16 step the rows 4 (l >> 4) .. + 3 of two blocks.
+constexpr int kChunk = 64, kBlocks = 10;                              // lower 16 x 16 blocks
+constexpr int kChunkFloats = 2 * kBlocks * 256 + 5 * kChunk;          // per chunk and head
+__device__ __forceinline__ constexpr int block_at(int b, int j) { return b * (b + 1) / 2 + j; }
+
+struct ChunkWs {
+  float* base;  // [chunks, H, kChunkFloats]; the chunks of sequence i start at q0 / 64 + i (they do not overlap)
+  __device__ __forceinline__ float* at(const Seq& s, int i, int chunk, int h, int H) const {
+    return base + ((int64_t)(s.q0 / kChunk + i + chunk) * H + h) * kChunkFloats;
+  }
+};
+
+// KS: key dims / 32 (dk a multiple of 8, zero-filled to 32 KS)
+template <int KS>
+__global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16> p, ChunkWs ws) {
+  __shared__ float sl[4][16][17];
+  const Seq s = seq_of(p, blockIdx.z);
+  const int chunk = blockIdx.x, h = blockIdx.y;
+  if (chunk * kChunk >= s.n) return;
+  const DeltaDims& d = p.d;
+  const int hk = h / (d.H / d.G), C = d.C();
+  const int lane = threadIdx.x & 63, b = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
+  const int left = s.n - chunk * kChunk;  // tokens from the chunk's start on
+  const int64_t t0 = s.q0 + chunk * kChunk;
+  float* out = ws.at(s, blockIdx.z, chunk, h, d.H);
+  float G = 0.f, beta = 0.f, rq = 0.f, rk = 0.f;  // of token `lane`; missing tokens change nothing
+  if (lane < left) {
+    const float* gb = p.gb + 2 * ((t0 + lane) * d.H + h);
+    G = gb[0];
+    beta = gb[1];
+    rq = p.rn[(t0 + lane) * 2 * d.G + hk];
+    rk = p.rn[(t0 + lane) * 2 * d.G + d.G + hk];
+  }
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const float v = __shfl_up(G, o, 64);
+    if (lane >= o) G += v;
+  }
+  const float last = __shfl(G, 63, 64);
+  if (b == 0) {
+    float* sc = out + 2 * kBlocks * 256 + lane;
+    const float eg = expf(G);
+    sc[0] = beta * eg * rk;
+    sc[kChunk] = beta;
+    sc[2 * kChunk] = eg * rq;
+    sc[3 * kChunk] = expf(last - G) * rk;
+    sc[4 * kChunk] = expf(last);
+  }
+  auto frag = [&](int blk, int base, int ks) {  // rows 16 blk + l15 of q or k
+    const int e = 32 * ks + 8 * g;
+    bf16x8 v = {};
+    if (e < d.dk) v = *reinterpret_cast<const bf16x8*>(p.y + (t0 + min(16 * blk + l15, left - 1)) * C + base + hk * d.dk + e);
+    return v;
+  };
+  bf16x8 kb[KS], qb[KS];
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) {
+    kb[ks] = frag(b, d.k0(), ks);
+    qb[ks] = frag(b, 0, ks);
+  }
+  float Gi[4], bi[4], qi[4], ki[4];  // of the rows 16 b + 4 g + r
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int i = 16 * b + 4 * g + r;
+    Gi[r] = __shfl(G, i, 64);
+    bi[r] = __shfl(beta, i, 64);
+    qi[r] = __shfl(rq, i, 64);
+    ki[r] = __shfl(rk, i, 64);
+  }
+  for (int j = 0; j <= b; ++j) {
+    f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bf16x8 kj = frag(j, d.k0(), ks);
+      kk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kb[ks], kj, kk, 0, 0, 0);
+      qk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qb[ks], kj, qk, 0, 0, 0);
+    }
+    const float Gj = __shfl(G, 16 * j + l15, 64), kj = __shfl(rk, 16 * j + l15, 64);
+    float* m1 = out + block_at(b, j) * 256 + l15;
+    float* am = m1 + kBlocks * 256;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = 4 * g + r;
+      const bool below = j < b || row > l15, on = below || row == l15;
+      const float e = on ? expf(Gi[r] - Gj) * kj : 0.f;
+      am[row * 16] = e * qi[r] * qk[r];
+      const float l = below ? bi[r] * e * ki[r] * kk[r] : 0.f;
+      if (j < b) m1[row * 16] = -l;
+      else sl[b][row][l15] = l;
+    }
+  }
+  __syncthreads();
+  if (lane < 16) {  // column l15 of (1 + L_bb)^-1 by forward substitution
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == l15 ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) v -= sl[b][i][j] * x[j];
+      x[i] = v;
+      out[block_at(b, b) * 256 + i * 16 + l15] = v;
+    }
+  }
+}
+
+// x = h + m + l to 24 bits
+__device__ __forceinline__ void split3(const float (&x)[8], bf16x8& h, bf16x8& m, bf16x8& l) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    h[i] = (bf16)x[i];
+    const float r = x[i] - (float)h[i];
+    m[i] = (bf16)r;
+    l[i] = (bf16)(r - (float)m[i]);
+  }
+}
+__device__ __forceinline__ void split_tiles(const f32x4& a, const f32x4& b, bf16x8& h, bf16x8& m, bf16x8& l) {
+  const float x[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+  split3(x, h, m, l);
+}
+__device__ __forceinline__ f32x4 mfma3(const bf16x8& a, const bf16x8& h, const bf16x8& m, const bf16x8& l, f32x4 c) {
+  c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, l, c, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, m, c, 0, 0, 0);
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, h, c, 0, 0, 0);
+}
+__device__ __forceinline__ f32x4 mfma_f32(const f32x4& a, const f32x4& b, f32x4 c) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], c, 0, 0, 0);
+  return c;
+}
+__device__ __forceinline__ bf16x4 read_tr4(const bf16* a) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4*)a);
+}
+
+template <int KS>
+struct ChunkTile {
+  static constexpr int kLd = 32 * KS + 8, kLdv = 64 + 8;             // row strides (elements)
+  static constexpr int kQ = kChunk * kLd, kV = 2 * kChunk * kLd;     // offsets of q and v after k
+  static constexpr int kSize = kV + kChunk * kLdv;
+};
+
+template <int KS>
+__global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf16> p, ChunkWs ws) {
+  using Tile = ChunkTile<KS>;
+  constexpr int LD = Tile::kLd, LDV = Tile::kLdv;
+  constexpr int CK = kChunk * 4 * KS / 256, CV = kChunk * 8 / 256;  // 16-byte pieces a thread stages of k (and q), of v
+  extern __shared__ __attribute__((aligned(16))) bf16 lds[];        // two tiles
+  const Seq s = seq_of(p, blockIdx.z);
+  if (s.n <= 0) return;
+  const DeltaDims& d = p.d;
+  const int h = blockIdx.y, hk = h / (d.H / d.G), C = d.C(), dv = d.dv;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
+  const int c0 = blockIdx.x * 64, col = c0 + 16 * w + l15;
+  const bool active = c0 + 16 * w < dv, ok = col < dv;
+  float* st = p.state + (int64_t)s.slot * p.slot_stride + (int64_t)h * d.dk * dv;
+  f32x4 S[2 * KS];
+#pragma unroll
+  for (int t = 0; t < 2 * KS; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = 16 * t + 4 * g + r;
+      S[t][r] = s.seen > 0 && ok && row < d.dk ? st[(int64_t)row * dv + col] : 0.f;
+    }
+  const bf16x8 zero = {};
+  bf16x8 nk[CK], nq[CK], nv[CV];
+  auto fetch = [&](int chunk) {
+    const int64_t t0 = s.q0 + chunk * kChunk;
+    const int left = s.n - chunk * kChunk;
+#pragma unroll
+    for (int i = 0; i < CK; ++i) {
+      const int x = threadIdx.x + 256 * i, row = x / (4 * KS), e = 8 * (x % (4 * KS));
+      nk[i] = nq[i] = zero;
+      if (row < left && e < d.dk) {
+        const bf16* y = p.y + (t0 + row) * C + hk * d.dk + e;
+        nq[i] = *reinterpret_cast<const bf16x8*>(y);
+        nk[i] = *reinterpret_cast<const bf16x8*>(y + d.k0());
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < CV; ++i) {
+      const int x = threadIdx.x + 256 * i, row = x / 8, e = c0 + 8 * (x % 8);
+      nv[i] = zero;
+      if (row < left && e < dv) nv[i] = *reinterpret_cast<const bf16x8*>(p.y + (t0 + row) * C + d.v0() + h * dv + e);
+    }
+  };
+  auto put = [&](bf16* tile) {
+#pragma unroll
+    for (int i = 0; i < CK; ++i) {
+      const int x = threadIdx.x + 256 * i, at = x / (4 * KS) * LD + 8 * (x % (4 * KS));
+      *reinterpret_cast<bf16x8*>(tile + at) = nk[i];
+      *reinterpret_cast<bf16x8*>(tile + Tile::kQ + at) = nq[i];
+    }
+#pragma unroll
+    for (int i = 0; i < CV; ++i) {
+      const int x = threadIdx.x + 256 * i;
+      *reinterpret_cast<bf16x8*>(tile + Tile::kV + x / 8 * LDV + 8 * (x % 8)) = nv[i];
+    }
+  };
+  const int chunks = (s.n + kChunk - 1) / kChunk;
+  fetch(0);
+  put(lds);
+  __syncthreads();
+  for (int ch = 0; ch < chunks; ++ch) {
+    const bf16* tile = lds + (ch & 1) * Tile::kSize;
+    if (active) {
+      const float* cw = ws.at(s, blockIdx.z, ch, h, d.H);
+      f32x4 M1[kBlocks], A[kBlocks], sc[4][4];
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          sc[k][b] = *reinterpret_cast<const f32x4*>(cw + 2 * kBlocks * 256 + k * kChunk + 16 * b + 4 * g);
+      const float keep = cw[2 * kBlocks * 256 + 4 * kChunk];
+#pragma unroll
+      for (int x = 0; x < kBlocks; ++x) M1[x] = *reinterpret_cast<const f32x4*>(cw + x * 256 + l15 * 16 + 4 * g);
+#pragma unroll
+      for (int x = 0; x < kBlocks; ++x)
+        A[x] = *reinterpret_cast<const f32x4*>(cw + (kBlocks + x) * 256 + l15 * 16 + 4 * g);
+      if (ch + 1 < chunks) fetch(ch + 1);
+      f32x4 U[4], O[4];  // K S, then u; Q S, then o
+#pragma unroll
+      for (int b = 0; b < 4; ++b) U[b] = O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        bf16x8 sh, sm, sl;
+        split_tiles(S[2 * ks], S[2 * ks + 1], sh, sm, sl);
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+          const bf16* kr = tile + (16 * b + l15) * LD + 32 * ks + 4 * g;
+          const bf16x4 k0 = *reinterpret_cast<const bf16x4*>(kr), k1 = *reinterpret_cast<const bf16x4*>(kr + 16);
+          const bf16x4 q0 = *reinterpret_cast<const bf16x4*>(kr + Tile::kQ);
+          const bf16x4 q1 = *reinterpret_cast<const bf16x4*>(kr + Tile::kQ + 16);
+          U[b] = mfma3(__builtin_shufflevector(k0, k1, 0, 1, 2, 3, 4, 5, 6, 7), sh, sm, sl, U[b]);
+          O[b] = mfma3(__builtin_shufflevector(q0, q1, 0, 1, 2, 3, 4, 5, 6, 7), sh, sm, sl, O[b]);
+        }
+      }
+      const int q = l15 >> 2, pp = l15 & 3;
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        const bf16x4 v = read_tr4(tile + Tile::kV + (16 * b + 4 * g + q) * LDV + 16 * w + 4 * pp);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) U[b][r] = sc[1][b][r] * (float)v[r] - sc[0][b][r] * U[b][r];
+#pragma unroll
+        for (int j = 0; j < b; ++j) U[b] = mfma_f32(M1[block_at(b, j)], U[j], U[b]);
+        U[b] = mfma_f32(M1[block_at(b, b)], U[b], f32x4{0.f, 0.f, 0.f, 0.f});
+      }
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        O[b] *= sc[2][b];
+#pragma unroll
+        for (int j = 0; j <= b; ++j) O[b] = mfma_f32(A[block_at(b, j)], U[j], O[b]);
+      }
+#pragma unroll
+      for (int t = 0; t < 2 * KS; ++t) S[t] *= keep;
+#pragma unroll
+      for (int b = 0; b < 4; ++b) U[b] *= sc[3][b];
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf) {
+        bf16x8 uh, um, ul;
+        split_tiles(U[2 * hf], U[2 * hf + 1], uh, um, ul);
+#pragma unroll
+        for (int t = 0; t < 2 * KS; ++t) {
+          const bf16* kc = tile + (32 * hf + 4 * g + q) * LD + 16 * t + 4 * pp;
+          const bf16x4 lo = read_tr4(kc), hi = read_tr4(kc + 16 * LD);
+          S[t] = mfma3(__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7), uh, um, ul, S[t]);
+        }
+      }
+      if (ok) {
+        const int left = s.n - ch * kChunk;
+        float* o = p.o + ((int64_t)(s.q0 + ch * kChunk) * d.H + h) * dv + col;
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int i = 16 * b + 4 * g + r;
+            if (i < left) o[(int64_t)i * d.H * dv] = O[b][r];
+          }
+      }
+    } else if (ch + 1 < chunks) {
+      fetch(ch + 1);
+    }
+    if (ch + 1 < chunks) put(lds + ((ch + 1) & 1) * Tile::kSize);  // the tile before this one: nobody reads it any more
+    __syncthreads();
+  }
+  if (ok)
+#pragma unroll
+    for (int t = 0; t < 2 * KS; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = 16 * t + 4 * g + r;
+        if (row < d.dk) st[(int64_t)row * dv + col] = S[t][r];
+      }
+}
+
+// ---------------------------------------------------------------------------------------------------------------
 // norm and gate of the heads
 // ---------------------------------------------------------------------------------------------------------------
 template <typename T>
@@ -499,6 +813,27 @@ int launch_scan(const DeltaParams<T>& p, int n_seqs, hipStream_t st) {
   return hipGetLastError();
 }
 
+bool chunk_ok(int dtype, int dk, int dv) { return dtype == kBF16 && dk % 8 == 0 && dv % 8 == 0 && dk <= 128; }
+
+template <int KS>
+int launch_chunks_as(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, int max_new, hipStream_t st) {
+  constexpr int lds = 2 * ChunkTile<KS>::kSize * sizeof(bf16);
+  static_assert(lds <= 160 * 1024, "LDS");
+  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_scan_kernel<KS>,
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  if (attr != hipSuccess) return attr;
+  hipLaunchKernelGGL(delta_chunk_prep_kernel<KS>, dim3((max_new + kChunk - 1) / kChunk, p.d.H, n_seqs), dim3(256), 0, st,
+                     p, ws);
+  hipLaunchKernelGGL(delta_chunk_scan_kernel<KS>, dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p, ws);
+  return hipGetLastError();
+}
+
+int launch_chunks(const DeltaParams<bf16>& p, float* ws, int n_seqs, int max_new, hipStream_t st) {
+  if (p.d.dk <= 32) return launch_chunks_as<1>(p, ChunkWs{ws}, n_seqs, max_new, st);
+  if (p.d.dk <= 64) return launch_chunks_as<2>(p, ChunkWs{ws}, n_seqs, max_new, st);
+  return launch_chunks_as<4>(p, ChunkWs{ws}, n_seqs, max_new, st);
+}
+
 // threads and rows a thread of delta_step; 0: the kernel does not take these sizes
 int step_shape(int dk, int dv, int& nt) {
   if (dv % 4 || dv > 1024) return 0;
@@ -563,12 +898,18 @@ HDS_EXPORT int hds_delta_step(int dtype, const void* proj, int64_t ld, const flo
   return hipErrorInvalidValue;
 }
 
+// floats of the chunk scan's scratch memory per chunk and head (a step of n tokens has up to n / 64 + n_seqs chunks);
+// 0: heads of these sizes and this type are scanned token by token
+HDS_EXPORT int hds_delta_chunk_floats(int dtype, int dk, int dv) { return chunk_ok(dtype, dk, dv) ? kChunkFloats : 0; }
+HDS_EXPORT int hds_delta_chunk_tokens() { return kChunk; }
+
 // Portions of at most max_new tokens. y [tokens, C], rn [tokens, 2 G], gb [tokens, H, 2] and o [tokens, H, dv] are
-// scratch memory with a row for every token of the step.
+// scratch memory with a row for every token of the step; chunks: scratch memory of the chunk scan (the sequences ascend in
+// the step's rows), or null: token by token.
 HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
                               const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
-                              const int* seq_meta, const int* seqs, void* y, float* rn, float* gb, float* o, void* out,
-                              int64_t ldo, int n_seqs, int max_new, int H, int G, int dk, int dv, int taps, float eps,
+                              const int* seq_meta, const int* seqs, void* y, float* rn, float* gb, float* o, float* chunks,
+                              void* out, int64_t ldo, int n_seqs, int max_new, int H, int G, int dk, int dv, int taps, float eps,
                               hipStream_t st) {
   if (n_seqs <= 0 || max_new <= 0) return 0;
   const DeltaDims d{H, G, dk, dv, taps, ld};
@@ -580,9 +921,15 @@ HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const flo
     const DeltaParams<TT> p{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, seqs,     \
                             (TT*)y, rn, gb, o, (TT*)out, ldo, 0, eps};                                               \
     if (int e = launch_conv(p, n_seqs, max_new, st)) return e;                                                       \
-    if (int e = launch_scan(p, n_seqs, st)) return e;                                                                \
+    if (int e = scan(p)) return e;                                                                                   \
     return launch_out(p, n_seqs, max_new, st);                                                                       \
   }
+  const auto scan = [&](const auto& p) -> int {
+    if constexpr (std::is_same<decltype(p.proj), const bf16*>::value)
+      if (chunks != nullptr) return launch_chunks(p, chunks, n_seqs, max_new, st);
+    return launch_scan(p, n_seqs, st);
+  };
+  if (chunks != nullptr && !chunk_ok(dtype, dk, dv)) return hipErrorInvalidValue;
   if (dtype == kBF16) HDS_DX(bf16)
   if (dtype == kF32) HDS_DX(float)
 #undef HDS_DX

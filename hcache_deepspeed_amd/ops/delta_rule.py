@@ -13,6 +13,9 @@ from . import native
 
 UNIT_EPS = 1e-6
 
+# Portions of a step are scanned by chunks on the matrix cores if one of them has more than this many tokens
+SERIAL_MAX = 16
+
 
 @dataclass(frozen=True)
 class DeltaShape:
@@ -68,6 +71,12 @@ def make_delta_plan(seq_meta_host, n_seqs, max_new, single, device):
     return plan
 
 
+def _chunk_floats(sh, dtype, n_tok, n_seqs):
+    lib = native.kernels()
+    per = lib.hds_delta_chunk_floats(native.dt(dtype), sh.dim, sh.vdim)
+    return (n_tok // lib.hds_delta_chunk_tokens() + n_seqs) * sh.heads * per
+
+
 def delta_rule(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch, plan, out):
     """proj: [T, >= shape.width]; conv_w: [taps, channels], the last row is the current token's; a_log, dt_bias: [heads];
     norm_w: [vdim], all float32. ``state[slot, offset:offset + shape.state_floats]`` is read and advanced; ``out``
@@ -92,9 +101,11 @@ def delta_rule(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch
         y = torch.empty(T, sh.channels, dtype=proj.dtype, device=dev)
         rn, gb = torch.empty(T, 2 * sh.kv_heads, **f32), torch.empty(T, sh.heads, 2, **f32)
         o = torch.empty(T, sh.heads, sh.vdim, **f32)
+        n_ws = _chunk_floats(sh, proj.dtype, T, plan.n_scan) if plan.max_new > SERIAL_MAX else 0
+        ws = torch.empty(n_ws, **f32) if n_ws else None
         native.check(
             lib.hds_delta_scan(*head, native.ptr(plan.scan), y.data_ptr(), rn.data_ptr(), gb.data_ptr(), o.data_ptr(),
-                               out.data_ptr(), out.stride(0), plan.n_scan, plan.max_new, *dims), "delta_scan")
+                               native.ptr(ws), out.data_ptr(), out.stride(0), plan.n_scan, plan.max_new, *dims), "delta_scan")
     return out
 
 
