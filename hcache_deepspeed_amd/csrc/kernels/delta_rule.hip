@@ -31,6 +31,12 @@ __device__ __forceinline__ float sigmoid_f(float x) {
 }
 __device__ __forceinline__ float silu_f(float x) { return x * sigmoid_f(x); }
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+// of activations and output gates (rounded to T)
+template <typename T>
+__device__ __forceinline__ float silu_act(float x) {
+  if constexpr (sizeof(T) == 2) return x * __builtin_amdgcn_rcpf(1.f + __expf(-x));
+  return silu_f(x);
+}
 template <typename T>
 __device__ __forceinline__ float rounded(float x) { return to_f(from_f<T>(x)); }
 
@@ -133,32 +139,43 @@ __global__ __launch_bounds__(256) void delta_conv8_kernel(DeltaParams<T> p, int 
       else if (pos >= 0) Vec8<float>::load(ring + (int64_t)(pos % p.d.taps) * C, hist[k]);
     }
   }
-  float x[8];
-  Vec8<T>::load(in + (int64_t)start * p.d.ld, x);
-  for (int r = 0; r < rows; ++r) {
-    float nx[8];
-    if (r + 1 < rows) Vec8<T>::load(in + (int64_t)(start + r + 1) * p.d.ld, nx);
-    float y[8], ss = 0.f;
+  constexpr int U = 4;  // rows in flight, and as many requested ahead
+  float nx[U][8];
+  auto fetch = [&](int r) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      float a = w[0][i] * x[i];
+    for (int k = 0; k < U; ++k) Vec8<T>::load(in + (int64_t)(start + min(r + k, rows - 1)) * p.d.ld, nx[k]);
+  };
+  fetch(0);
+  for (int r0 = 0; r0 < rows; r0 += U) {
+    float xs[U][8];
 #pragma unroll
-      for (int k = 0; k < M; ++k) a += w[k + 1][i] * hist[k][i];
-      y[i] = rounded<T>(silu_f(rounded<T>(a)));
-      ss += ok ? y[i] * y[i] : 0.f;
-    }
-    const int t = s.q0 + start + r;
-    if (ok) Vec8<T>::store(p.y + (int64_t)t * C + c, y);
-    ss = group_sum<LPU>(ss);
-    if (ok && e == 0) write_factor(p, t, u, ss);
+    for (int k = 0; k < U; ++k)
 #pragma unroll
-    for (int k = M - 1; k > 0; --k)
+      for (int i = 0; i < 8; ++i) xs[k][i] = nx[k][i];
+    if (r0 + U < rows) fetch(r0 + U);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) hist[k][i] = hist[k - 1][i];
+    for (int b = 0; b < U; ++b) {
+      float y[8], ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      hist[0][i] = x[i];
-      if (r + 1 < rows) x[i] = nx[i];
+      for (int i = 0; i < 8; ++i) {
+        float a = w[0][i] * xs[b][i];
+#pragma unroll
+        for (int k = 0; k < M; ++k) a += w[k + 1][i] * hist[k][i];
+        y[i] = rounded<T>(silu_act<T>(rounded<T>(a)));
+        ss += ok ? y[i] * y[i] : 0.f;
+      }
+      const int t = s.q0 + start + r0 + b;
+      ss = group_sum<LPU>(ss);
+      if (ok && r0 + b < rows) {
+        Vec8<T>::store(p.y + (int64_t)t * C + c, y);
+        if (e == 0) write_factor(p, t, u, ss);
+      }
+#pragma unroll
+      for (int k = M - 1; k > 0; --k)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) hist[k][i] = hist[k - 1][i];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) hist[0][i] = xs[b][i];
     }
   }
   if (blockIdx.x == 0 && ok)
@@ -194,7 +211,7 @@ __global__ __launch_bounds__(256) void delta_conv_kernel(DeltaParams<T> p, int R
         const float v = i0 >= 0 ? to_f(in[(int64_t)i0 * p.d.ld + c]) : ring[(int64_t)(pos % p.d.taps) * C + c];
         a += p.cw[(int64_t)(m - k) * C + c] * v;
       }
-      const float y = rounded<T>(silu_f(rounded<T>(a)));
+      const float y = rounded<T>(silu_act<T>(rounded<T>(a)));
       p.y[(int64_t)(s.q0 + start + r) * C + c] = from_f<T>(y);
       ss += y * y;
     }
@@ -305,7 +322,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams<T> p) {
 //
 // An accumulator tile (lane: column l & 15, rows 4 (l >> 4) + r) is the right operand of the next product as it is, if the
 // left operand takes its contraction index in the same order: f32 step r contracts rows 4 (l >> 4) + r of a 16-row block,
-// a bf16 step the rows 4 (l >> 4) .. + 3 of two blocks.
+// a bf16 step over tokens the rows 4 (l >> 4) .. + 3 of two blocks. The rows of S are dealt to the tiles such that a bf16
+// step over them takes 8 neighbours.
 constexpr int kChunk = 64, kBlocks = 10;                              // lower 16 x 16 blocks
 constexpr int kChunkFloats = 2 * kBlocks * 256 + 5 * kChunk;          // per chunk and head
 __device__ __forceinline__ constexpr int block_at(int b, int j) { return b * (b + 1) / 2 + j; }
@@ -410,6 +428,10 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16>
   }
 }
 
+// row of S in register r of accumulator tile t: 8 neighbouring rows of two tiles are the 8 contraction indices a lane of the
+// bfloat16 products holds
+__device__ __forceinline__ int state_row(int t, int g, int r) { return 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r; }
+
 // x = h + m + l to 24 bits
 __device__ __forceinline__ void split3(const float (&x)[8], bf16x8& h, bf16x8& m, bf16x8& l) {
 #pragma unroll
@@ -424,33 +446,29 @@ __device__ __forceinline__ void split_tiles(const f32x4& a, const f32x4& b, bf16
   const float x[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
   split3(x, h, m, l);
 }
-__device__ __forceinline__ f32x4 mfma3(const bf16x8& a, const bf16x8& h, const bf16x8& m, const bf16x8& l, f32x4 c) {
-  c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, l, c, 0, 0, 0);
-  c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, m, c, 0, 0, 0);
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, h, c, 0, 0, 0);
-}
 __device__ __forceinline__ f32x4 mfma_f32(const f32x4& a, const f32x4& b, f32x4 c) {
 #pragma unroll
   for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], c, 0, 0, 0);
   return c;
 }
-__device__ __forceinline__ bf16x4 read_tr4(const bf16* a) {
+__device__ __forceinline__ bf16x4 read_tr4(const char* a) {
   return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4*)a);
 }
 
-template <int KS>
-struct ChunkTile {
-  static constexpr int kLd = 32 * KS + 8, kLdv = 64 + 8;             // row strides (elements)
-  static constexpr int kQ = kChunk * kLd, kV = 2 * kChunk * kLd;     // offsets of q and v after k
-  static constexpr int kSize = kV + kChunk * kLdv;
-};
+// LDS image of a chunk, filled by direct loads (a wave instruction writes 64 lanes x 16 bytes in a row, so rows have no
+// padding; 16-byte pieces are swapped within a row instead, by the row number): k and q as 64 rows of 256 bytes, 64 columns
+// of v as 64 rows of 128 bytes, the chunk's blocks and factors as they are.
+constexpr int kTileQ = 16384, kTileV = 32768, kTileW = 40960, kTileBytes = kTileW + 4 * kChunkFloats;
+__device__ __forceinline__ int row_off(int row, int piece) { return row * 256 + 16 * (piece ^ (((row & 3) << 2) | ((row >> 2) & 3))); }
+__device__ __forceinline__ int v_off(int row, int piece) { return row * 128 + 16 * (piece ^ (row & 7)); }
+__device__ __forceinline__ void direct_load(const void* src, char* dst) {
+  __builtin_amdgcn_global_load_lds((__attribute__((address_space(1))) const void*)src,
+                                   (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
+}
 
 template <int KS>
 __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf16> p, ChunkWs ws) {
-  using Tile = ChunkTile<KS>;
-  constexpr int LD = Tile::kLd, LDV = Tile::kLdv;
-  constexpr int CK = kChunk * 4 * KS / 256, CV = kChunk * 8 / 256;  // 16-byte pieces a thread stages of k (and q), of v
-  extern __shared__ __attribute__((aligned(16))) bf16 lds[];        // two tiles
+  extern __shared__ __attribute__((aligned(1024))) char lds[];  // two chunks
   const Seq s = seq_of(p, blockIdx.z);
   if (s.n <= 0) return;
   const DeltaDims& d = p.d;
@@ -464,136 +482,210 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
   for (int t = 0; t < 2 * KS; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int row = 16 * t + 4 * g + r;
+      const int row = state_row(t, g, r);
       S[t][r] = s.seen > 0 && ok && row < d.dk ? st[(int64_t)row * dv + col] : 0.f;
     }
-  const bf16x8 zero = {};
-  bf16x8 nk[CK], nq[CK], nv[CV];
+  // Rows past the end repeat the last one: their factors are zero. Key columns past dk stay zero: a row of S there would
+  // take part otherwise.
+  const bf16* yq = p.y + (int64_t)s.q0 * C + hk * d.dk;
+  const bf16* yv = p.y + (int64_t)s.q0 * C + d.v0() + h * dv + c0;
   auto fetch = [&](int chunk) {
-    const int64_t t0 = s.q0 + chunk * kChunk;
-    const int left = s.n - chunk * kChunk;
+    char* tile = lds + (chunk & 1) * kTileBytes;
+    const int last = s.n - 1 - chunk * kChunk;
+    const int64_t at = (int64_t)chunk * kChunk * C;
 #pragma unroll
-    for (int i = 0; i < CK; ++i) {
-      const int x = threadIdx.x + 256 * i, row = x / (4 * KS), e = 8 * (x % (4 * KS));
-      nk[i] = nq[i] = zero;
-      if (row < left && e < d.dk) {
-        const bf16* y = p.y + (t0 + row) * C + hk * d.dk + e;
-        nq[i] = *reinterpret_cast<const bf16x8*>(y);
-        nk[i] = *reinterpret_cast<const bf16x8*>(y + d.k0());
+    for (int i = 0; i < 4; ++i) {  // 4 rows an instruction
+      const int n = 4 * w + i, row = 4 * n + (lane >> 4);
+      const int e = 8 * ((lane & 15) ^ (((row & 3) << 2) | ((row >> 2) & 3)));
+      const bf16* src = yq + at + (uint32_t)(min(row, last) * C + e);
+      if (e < d.dk) {
+        direct_load(src + d.k0(), tile + n * 1024);
+        direct_load(src, tile + kTileQ + n * 1024);
       }
     }
 #pragma unroll
-    for (int i = 0; i < CV; ++i) {
-      const int x = threadIdx.x + 256 * i, row = x / 8, e = c0 + 8 * (x % 8);
-      nv[i] = zero;
-      if (row < left && e < dv) nv[i] = *reinterpret_cast<const bf16x8*>(p.y + (t0 + row) * C + d.v0() + h * dv + e);
+    for (int i = 0; i < 2; ++i) {  // 8 rows an instruction
+      const int n = 2 * w + i, row = 8 * n + (lane >> 3), e = 8 * ((lane & 7) ^ (row & 7));
+      if (c0 + e < dv) direct_load(yv + at + (uint32_t)(min(row, last) * C + e), tile + kTileV + n * 1024);
     }
-  };
-  auto put = [&](bf16* tile) {
+    const char* cw = reinterpret_cast<const char*>(ws.at(s, blockIdx.z, chunk, h, d.H)) + 16 * lane;
+    constexpr int kW = 4 * kChunkFloats;
 #pragma unroll
-    for (int i = 0; i < CK; ++i) {
-      const int x = threadIdx.x + 256 * i, at = x / (4 * KS) * LD + 8 * (x % (4 * KS));
-      *reinterpret_cast<bf16x8*>(tile + at) = nk[i];
-      *reinterpret_cast<bf16x8*>(tile + Tile::kQ + at) = nq[i];
-    }
-#pragma unroll
-    for (int i = 0; i < CV; ++i) {
-      const int x = threadIdx.x + 256 * i;
-      *reinterpret_cast<bf16x8*>(tile + Tile::kV + x / 8 * LDV + 8 * (x % 8)) = nv[i];
+    for (int i = 0; i < (kW + 4095) / 4096; ++i) {
+      const int n = 4 * i + w;
+      if (n * 1024 + 16 * lane < kW) direct_load(cw + n * 1024, tile + kTileW + n * 1024);
     }
   };
   const int chunks = (s.n + kChunk - 1) / kChunk;
+  if (d.dk < 32 * KS) {
+    for (int i = threadIdx.x; i < 2 * kTileBytes / 16; i += 256) reinterpret_cast<u32x4*>(lds)[i] = u32x4{};
+    __syncthreads();
+  }
+  // Offsets of this lane's reads in a tile. Row blocks and halves are 16-row steps, which leave the swap of the pieces as
+  // it is; another k step or key block flips bits of the offset.
+  const int q = l15 >> 2, pp = l15 & 3;
+  const int row_at = row_off(l15, g);           // ^ 64 ks; + 4096 b
+  const int col_at = row_off(4 * g + q, pp);    // ^ 64 (t >> 1); + 8 (t & 1), + 4096 per 16 tokens
+  const int v_at = kTileV + v_off(4 * g + q, 2 * w + (pp >> 1)) + 8 * (pp & 1);  // + 2048 b
   fetch(0);
-  put(lds);
   __syncthreads();
   for (int ch = 0; ch < chunks; ++ch) {
-    const bf16* tile = lds + (ch & 1) * Tile::kSize;
+    const char* tile = lds + (ch & 1) * kTileBytes;
     if (active) {
-      const float* cw = ws.at(s, blockIdx.z, ch, h, d.H);
-      f32x4 M1[kBlocks], A[kBlocks], sc[4][4];
+      const char* cw = tile + kTileW;
+      auto block = [&](int x) { return *reinterpret_cast<const f32x4*>(cw + x * 1024 + l15 * 64 + 16 * g); };
+      auto factor = [&](int k, int b) {
+        return *reinterpret_cast<const f32x4*>(cw + 2 * kBlocks * 1024 + k * 4 * kChunk + 64 * b + 16 * g);
+      };
+      const float keep = *reinterpret_cast<const float*>(cw + 2 * kBlocks * 1024 + 16 * kChunk);
+      // Operands are read from LDS one step ahead of the products that use them, products of different accumulators follow
+      // one another, and the splits of the next operands lie between them: the scheduling barriers keep it so.
+      bf16x4 v[4];
 #pragma unroll
-      for (int b = 0; b < 4; ++b)
-#pragma unroll
-        for (int k = 0; k < 4; ++k)
-          sc[k][b] = *reinterpret_cast<const f32x4*>(cw + 2 * kBlocks * 256 + k * kChunk + 16 * b + 4 * g);
-      const float keep = cw[2 * kBlocks * 256 + 4 * kChunk];
-#pragma unroll
-      for (int x = 0; x < kBlocks; ++x) M1[x] = *reinterpret_cast<const f32x4*>(cw + x * 256 + l15 * 16 + 4 * g);
-#pragma unroll
-      for (int x = 0; x < kBlocks; ++x)
-        A[x] = *reinterpret_cast<const f32x4*>(cw + (kBlocks + x) * 256 + l15 * 16 + 4 * g);
-      if (ch + 1 < chunks) fetch(ch + 1);
-      f32x4 U[4], O[4];  // K S, then u; Q S, then o
-#pragma unroll
-      for (int b = 0; b < 4; ++b) U[b] = O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        bf16x8 sh, sm, sl;
-        split_tiles(S[2 * ks], S[2 * ks + 1], sh, sm, sl);
+      for (int b = 0; b < 4; ++b) v[b] = read_tr4(tile + v_at + 2048 * b);
+      bf16x8 kf[2][4], qf[2][4];
+      auto rows = [&](int ks, bf16x8 (&kk)[4], bf16x8 (&qq)[4]) {
+        const char* p0 = tile + (row_at ^ (64 * ks));
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
-          const bf16* kr = tile + (16 * b + l15) * LD + 32 * ks + 4 * g;
-          const bf16x4 k0 = *reinterpret_cast<const bf16x4*>(kr), k1 = *reinterpret_cast<const bf16x4*>(kr + 16);
-          const bf16x4 q0 = *reinterpret_cast<const bf16x4*>(kr + Tile::kQ);
-          const bf16x4 q1 = *reinterpret_cast<const bf16x4*>(kr + Tile::kQ + 16);
-          U[b] = mfma3(__builtin_shufflevector(k0, k1, 0, 1, 2, 3, 4, 5, 6, 7), sh, sm, sl, U[b]);
-          O[b] = mfma3(__builtin_shufflevector(q0, q1, 0, 1, 2, 3, 4, 5, 6, 7), sh, sm, sl, O[b]);
+          kk[b] = *reinterpret_cast<const bf16x8*>(p0 + 4096 * b);
+          qq[b] = *reinterpret_cast<const bf16x8*>(p0 + kTileQ + 4096 * b);
+        }
+      };
+      rows(0, kf[0], qf[0]);
+      // the next chunk's loads go out before this chunk's work (transposed reads wait for direct loads before them: the
+      // ones below find them done)
+      __builtin_amdgcn_sched_barrier(0);
+      if (ch + 1 < chunks) fetch(ch + 1);
+      f32x4 U[4], O[4];  // K S, then u; Q S, then o
+      bf16x8 sp[2][3];
+      split_tiles(S[0], S[1], sp[0][0], sp[0][1], sp[0][2]);
+#pragma unroll
+      for (int b = 0; b < 4; ++b) U[b] = O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+      f32x4 M1[4][4], A[4][4], f0[4], f1[4];  // [row block][column block]
+      auto column = [&](int j) {
+#pragma unroll
+        for (int b = j; b < 4; ++b) {
+          M1[b][j] = block(block_at(b, j));
+          A[b][j] = block(kBlocks + block_at(b, j));
+        }
+      };
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        __builtin_amdgcn_sched_barrier(0);
+        if (ks + 1 < KS) {
+          rows(ks + 1, kf[(ks + 1) & 1], qf[(ks + 1) & 1]);
+        } else {
+#pragma unroll
+          for (int b = 0; b < 4; ++b) {
+            f0[b] = factor(0, b);
+            f1[b] = factor(1, b);
+          }
+          column(0);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int k = 2; k >= 0; --k) {  // the smallest piece first
+#pragma unroll
+          for (int b = 0; b < 4; ++b) {
+            U[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][b], sp[ks & 1][k], U[b], 0, 0, 0);
+            O[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ks & 1][b], sp[ks & 1][k], O[b], 0, 0, 0);
+          }
+        }
+        if (ks + 1 < KS) {
+          bf16x8(&n)[3] = sp[(ks + 1) & 1];
+          split_tiles(S[2 * ks + 2], S[2 * ks + 3], n[0], n[1], n[2]);
+        }
+#pragma unroll
+        for (int i = 0; i < 24; ++i) {
+          __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);  // a product,
+          __builtin_amdgcn_sched_group_barrier(0x002, 3, 0);  // vector instructions under it
         }
       }
-      const int q = l15 >> 2, pp = l15 & 3;
-#pragma unroll
-      for (int b = 0; b < 4; ++b) {
-        const bf16x4 v = read_tr4(tile + Tile::kV + (16 * b + 4 * g + q) * LDV + 16 * w + 4 * pp);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) U[b][r] = sc[1][b][r] * (float)v[r] - sc[0][b][r] * U[b][r];
-#pragma unroll
-        for (int j = 0; j < b; ++j) U[b] = mfma_f32(M1[block_at(b, j)], U[j], U[b]);
-        U[b] = mfma_f32(M1[block_at(b, b)], U[b], f32x4{0.f, 0.f, 0.f, 0.f});
-      }
-#pragma unroll
-      for (int b = 0; b < 4; ++b) {
-        O[b] *= sc[2][b];
-#pragma unroll
-        for (int j = 0; j <= b; ++j) O[b] = mfma_f32(A[block_at(b, j)], U[j], O[b]);
-      }
-#pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) S[t] *= keep;
-#pragma unroll
-      for (int b = 0; b < 4; ++b) U[b] *= sc[3][b];
-#pragma unroll
-      for (int hf = 0; hf < 2; ++hf) {
-        bf16x8 uh, um, ul;
-        split_tiles(U[2 * hf], U[2 * hf + 1], uh, um, ul);
+      __builtin_amdgcn_sched_barrier(0);
+      f32x4 f2[4], f3[4];
+      bf16x8 kt[2 * KS];  // transposed k: all key dims of 32 tokens
+      auto cols = [&](int hf) {
 #pragma unroll
         for (int t = 0; t < 2 * KS; ++t) {
-          const bf16* kc = tile + (32 * hf + 4 * g + q) * LD + 16 * t + 4 * pp;
-          const bf16x4 lo = read_tr4(kc), hi = read_tr4(kc + 16 * LD);
-          S[t] = mfma3(__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7), uh, um, ul, S[t]);
+          const char* p0 = tile + (col_at ^ (64 * (t >> 1))) + 8 * (t & 1) + 8192 * hf;
+          kt[t] = __builtin_shufflevector(read_tr4(p0), read_tr4(p0 + 4096), 0, 1, 2, 3, 4, 5, 6, 7);
         }
+      };
+      bf16x8 up[2][3];
+#pragma unroll
+      for (int b = 0; b < 4; ++b) f2[b] = factor(2, b);
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) U[b][r] = f1[b][r] * (float)v[b][r] - f0[b][r] * U[b][r];
+        O[b] *= f2[b];
       }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        __builtin_amdgcn_sched_barrier(0);
+        if (j < 3) column(j + 1);
+        f3[j] = factor(3, j);
+        if (j == 2) cols(0);
+        __builtin_amdgcn_sched_barrier(0);
+        U[j] = mfma_f32(M1[j][j], U[j], f32x4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+#pragma unroll
+          for (int b = j + 1; b < 4; ++b) U[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[b][j][r], U[j][r], U[b], 0, 0, 0);
+#pragma unroll
+          for (int b = j; b < 4; ++b) O[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(A[b][j][r], U[j][r], O[b], 0, 0, 0);
+        }
+        if (j == 0)
+#pragma unroll
+          for (int t = 0; t < 2 * KS; ++t) S[t] *= keep;
+        if (j == 2) split_tiles(U[0] * f3[0], U[1] * f3[1], up[0][0], up[0][1], up[0][2]);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int k = 2; k >= 0; --k)
+#pragma unroll
+        for (int t = 0; t < 2 * KS; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt[t], up[0][k], S[t], 0, 0, 0);
+      split_tiles(U[2] * f3[2], U[3] * f3[3], up[1][0], up[1][1], up[1][2]);
+#pragma unroll
+      for (int i = 0; i < 6 * KS; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+        __builtin_amdgcn_sched_group_barrier(0x002, 3, 0);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      cols(1);
+#pragma unroll
+      for (int k = 2; k >= 0; --k)
+#pragma unroll
+        for (int t = 0; t < 2 * KS; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt[t], up[1][k], S[t], 0, 0, 0);
       if (ok) {
         const int left = s.n - ch * kChunk;
         float* o = p.o + ((int64_t)(s.q0 + ch * kChunk) * d.H + h) * dv + col;
+        const uint32_t ld = (uint32_t)(d.H * dv);
+        if (left >= kChunk) {
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
+          for (int b = 0; b < 4; ++b)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int i = 16 * b + 4 * g + r;
-            if (i < left) o[(int64_t)i * d.H * dv] = O[b][r];
-          }
+            for (int r = 0; r < 4; ++r) o[(uint32_t)(16 * b + 4 * g + r) * ld] = O[b][r];
+        } else {
+#pragma unroll
+          for (int b = 0; b < 4; ++b)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              if (16 * b + 4 * g + r < left) o[(uint32_t)(16 * b + 4 * g + r) * ld] = O[b][r];
+        }
       }
     } else if (ch + 1 < chunks) {
       fetch(ch + 1);
     }
-    if (ch + 1 < chunks) put(lds + ((ch + 1) & 1) * Tile::kSize);  // the tile before this one: nobody reads it any more
-    __syncthreads();
+    __syncthreads();  // (also waits for the direct loads)
   }
   if (ok)
 #pragma unroll
     for (int t = 0; t < 2 * KS; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int row = 16 * t + 4 * g + r;
+        const int row = state_row(t, g, r);
         if (row < d.dk) st[(int64_t)row * dv + col] = S[t][r];
       }
 }
@@ -632,7 +724,7 @@ __global__ __launch_bounds__(256) void delta_out8_kernel(DeltaParams<T> p, int R
     if (!ok) continue;
     const float rs = 1.f / sqrtf(ss / (float)dv + p.eps);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) o[i] *= rs * nw[i] * silu_f(g[i]);
+    for (int i = 0; i < 8; ++i) o[i] *= rs * nw[i] * silu_act<T>(g[i]);
     Vec8<T>::store(p.out + (int64_t)t * p.ldo + h * dv + e, o);
   }
 }
@@ -649,7 +741,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams<T> p, int R)
     for (int e = lane; e < dv; e += 64) ss += o[e] * o[e];
     const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dv + p.eps);
     for (int e = lane; e < dv; e += 64)
-      p.out[(int64_t)t * p.ldo + h * dv + e] = from_f<T>(o[e] * rs * p.norm[e] * silu_f(to_f(g[e])));
+      p.out[(int64_t)t * p.ldo + h * dv + e] = from_f<T>(o[e] * rs * p.norm[e] * silu_act<T>(to_f(g[e])));
   }
 }
 
@@ -699,7 +791,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
     float a = p.cw[(int64_t)(d.taps - 1) * C + c] * x;
     for (int k = 1; k < d.taps; ++k)
       if (s.seen - k >= 0) a += p.cw[(int64_t)(d.taps - 1 - k) * C + c] * ring[(int64_t)((s.seen - k) % d.taps) * C + c];
-    sq[i] = rounded<T>(silu_f(rounded<T>(a)));
+    sq[i] = rounded<T>(silu_act<T>(rounded<T>(a)));
     if (i >= 2 * dk || h % (d.H / d.G) == 0) ring[(int64_t)(s.seen % d.taps) * C + c] = x;
   }
   __syncthreads();
@@ -761,7 +853,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
     const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dv + p.eps);
     for (int c = threadIdx.x; c < dv; c += NT)
       p.out[(int64_t)s.q0 * p.ldo + h * dv + c] =
-          from_f<T>(so[c] * rs * p.norm[c] * silu_f(to_f(row[C + h * dv + c])));
+          from_f<T>(so[c] * rs * p.norm[c] * silu_act<T>(to_f(row[C + h * dv + c])));
   }
 }
 
@@ -769,7 +861,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
 template <typename T>
 int launch_conv(const DeltaParams<T>& p, int n_seqs, int max_new, hipStream_t st) {
   const DeltaDims& d = p.d;
-  int R = max_new > 1024 ? 32 : 16;
+  int R = 16;
   if (R < d.taps - 1) R = d.taps - 1;
   const int units = 2 * d.G + d.H, w = d.dk > d.dv ? d.dk : d.dv;
   const int blocks = (max_new + R - 1) / R;
@@ -817,7 +909,7 @@ bool chunk_ok(int dtype, int dk, int dv) { return dtype == kBF16 && dk % 8 == 0 
 
 template <int KS>
 int launch_chunks_as(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, int max_new, hipStream_t st) {
-  constexpr int lds = 2 * ChunkTile<KS>::kSize * sizeof(bf16);
+  constexpr int lds = 2 * kTileBytes;
   static_assert(lds <= 160 * 1024, "LDS");
   static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_scan_kernel<KS>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, lds);

@@ -41,7 +41,9 @@ HIPCC_FLAGS = ["-O3", "-fPIC", "-std=c++17", f"--offload-arch={ARCH}", "-ffp-con
 FILE_FLAGS = {"flash_attn.hip": ["-fno-slp-vectorize"],
               # the one-wave-per-SIMD forward keeps S in VGPRs (builtin MFMAs, schedulable) and O in AGPRs (asm)
               "flash_attn_w64.hip": ["-fno-slp-vectorize", "-mllvm", "-amdgpu-mfma-vgpr-form"],
-              "flash_attn_bwd_w64.hip": ["-fno-slp-vectorize", "-mllvm", "-amdgpu-mfma-vgpr-form"]}
+              "flash_attn_bwd_w64.hip": ["-fno-slp-vectorize", "-mllvm", "-amdgpu-mfma-vgpr-form"],
+              # the chunk scan works on its accumulators with vector instructions too: no moves from and to AGPRs
+              "delta_rule.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
 HOST_FLAGS = ["-O3", "-fPIC", "-std=c++17", "-fopenmp", "-D__HIP_PLATFORM_AMD__", f"-I{ROCM}/include",
               "-Wall", "-Wno-unused-function", "-Wno-unused-variable"]
 
