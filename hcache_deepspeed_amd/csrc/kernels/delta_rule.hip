@@ -15,7 +15,7 @@
 // Single tokens run one kernel, a workgroup per (sequence, head): delta_step. Portions run delta_conv (convolutions,
 // factors of the unit norms, log decays and betas), a scan over the tokens, and delta_out (norm and gate of the heads).
 // The scan goes token by token (delta_scan: short portions, 32-bit engines, any sizes) or by chunks on the matrix cores
-// (delta_chunk_prep, delta_chunk_scan).
+// (delta_chunk_prep, delta_chunk_state, delta_chunk_out).
 #include <type_traits>
 
 #include "hds_common.h"
@@ -315,25 +315,31 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams<T> p) {
 //   S        <- e^G_last S + sum_j e^(G_last - G_j) k_j u_j^T
 //
 // delta_chunk_prep, all chunks at once: 16 x 16 blocks of -L below the diagonal, the inverses of the diagonal blocks of
-// 1 + L, the blocks of A, and the factors per token. delta_chunk_scan, a wave per 16 columns of a head's state: walks the
-// chunks with S in registers. Everything is 32-bit: q and k are bfloat16 up to a 32-bit factor per token, so products
-// among them are exact on the bfloat16 matrix cores; S and U enter their products with q and k as sums of three bfloat16
-// numbers (24 bits); the blocks of L and A multiply U on the 32-bit matrix cores.
+// 1 + L, the blocks of A, and the factors per token. delta_chunk_state, a wave per 16 columns of a head's state: walks the
+// chunks with S in registers and leaves every chunk's S and U. delta_chunk_out, all chunks at once: O, its norm and its
+// gate. Everything is 32-bit: q and k are bfloat16 up to a 32-bit factor per token, so products among them are exact on
+// the bfloat16 matrix cores; S and U enter their products with q and k as sums of three bfloat16 numbers (24 bits); the
+// blocks of L and A multiply U on the 32-bit matrix cores.
 //
 // An accumulator tile (lane: column l & 15, rows 4 (l >> 4) + r) is the right operand of the next product as it is, if the
 // left operand takes its contraction index in the same order: f32 step r contracts rows 4 (l >> 4) + r of a 16-row block,
 // a bf16 step over tokens the rows 4 (l >> 4) .. + 3 of two blocks. The rows of S are dealt to the tiles such that a bf16
 // step over them takes 8 neighbours.
-constexpr int kChunk = 64, kBlocks = 10;                              // lower 16 x 16 blocks
-constexpr int kChunkFloats = 2 * kBlocks * 256 + 5 * kChunk;          // per chunk and head
+constexpr int kChunk = 64, kBlocks = 10;                // lower 16 x 16 blocks
+constexpr int kWalkFloats = kBlocks * 256 + 5 * kChunk; // what the walk reads: blocks of L, factors
+constexpr int kFixedFloats = kWalkFloats + kBlocks * 256;
 __device__ __forceinline__ constexpr int block_at(int b, int j) { return b * (b + 1) / 2 + j; }
 
+// Scratch memory of a chunk and head: blocks of L | factors [5][64] | blocks of A, then per 16 columns of the state its
+// 2 KS tiles and U's 4 tiles as the lanes hold them. The chunks of sequence i start at q0 / 64 + i (they do not overlap).
 struct ChunkWs {
-  float* base;  // [chunks, H, kChunkFloats]; the chunks of sequence i start at q0 / 64 + i (they do not overlap)
+  float* base;
+  int64_t floats;  // per chunk and head
   __device__ __forceinline__ float* at(const Seq& s, int i, int chunk, int h, int H) const {
-    return base + ((int64_t)(s.q0 / kChunk + i + chunk) * H + h) * kChunkFloats;
+    return base + ((int64_t)(s.q0 / kChunk + i + chunk) * H + h) * floats;
   }
 };
+__device__ __host__ __forceinline__ constexpr int strip_floats(int ks) { return (2 * ks + 4) * 256; }
 
 // KS: key dims / 32 (dk a multiple of 8, zero-filled to 32 KS)
 template <int KS>
@@ -363,7 +369,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16>
   }
   const float last = __shfl(G, 63, 64);
   if (b == 0) {
-    float* sc = out + 2 * kBlocks * 256 + lane;
+    float* sc = out + kBlocks * 256 + lane;
     const float eg = expf(G);
     sc[0] = beta * eg * rk;
     sc[kChunk] = beta;
@@ -402,7 +408,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16>
     }
     const float Gj = __shfl(G, 16 * j + l15, 64), kj = __shfl(rk, 16 * j + l15, 64);
     float* m1 = out + block_at(b, j) * 256 + l15;
-    float* am = m1 + kBlocks * 256;
+    float* am = m1 + kWalkFloats;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = 4 * g + r;
@@ -432,34 +438,76 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16>
 // bfloat16 products holds
 __device__ __forceinline__ int state_row(int t, int g, int r) { return 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r; }
 
-// x = h + m + l to 24 bits
-__device__ __forceinline__ void split3(const float (&x)[8], bf16x8& h, bf16x8& m, bf16x8& l) {
-#pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    h[i] = (bf16)x[i];
-    const float r = x[i] - (float)h[i];
-    m[i] = (bf16)r;
-    l[i] = (bf16)(r - (float)m[i]);
-  }
-}
-__device__ __forceinline__ void split_tiles(const f32x4& a, const f32x4& b, bf16x8& h, bf16x8& m, bf16x8& l) {
-  const float x[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
-  split3(x, h, m, l);
-}
 __device__ __forceinline__ f32x4 mfma_f32(const f32x4& a, const f32x4& b, f32x4 c) {
 #pragma unroll
   for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], c, 0, 0, 0);
   return c;
 }
+// Transposed LDS reads as inline asm: in front of the builtin the compiler waits for every direct load and store under way
+// (it cannot tell that they go elsewhere). tr_wait is due before the values are used.
 __device__ __forceinline__ bf16x4 read_tr4(const char* a) {
-  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4*)a);
+  bf16x4 r;
+  asm volatile("ds_read_b64_tr_b16 %0, %1" : "=v"(r) : "v"((uint32_t)(uintptr_t)a) : "memory");
+  return r;
+}
+__device__ __forceinline__ void tr_wait(bf16x4& a, bf16x4& b) {
+  asm volatile("s_waitcnt lgkmcnt(0)" : "+v"(a), "+v"(b) : : "memory");
+}
+__device__ __forceinline__ f32x4 mfma_bf16(const bf16x8& a, const bf16x8& b, const f32x4& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+// Eight numbers as sums of three bfloat16 numbers (24 bits), in 12 steps of a few instructions, to lie between matrix
+// products
+struct Split {
+  u32x4 bits[3];  // high, middle, low
+  float r[8];
+  template <int STEP>
+  __device__ __forceinline__ void step(const f32x4& a, const f32x4& b) {
+    typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+    typedef float f32x2 __attribute__((ext_vector_type(2)));
+    constexpr int i = STEP / 3, k = STEP % 3;
+    const f32x2 x = k > 0 ? f32x2{r[2 * i], r[2 * i + 1]}
+                          : (i < 2 ? f32x2{a[2 * i & 3], a[(2 * i & 3) + 1]} : f32x2{b[2 * i & 3], b[(2 * i & 3) + 1]});
+    const uint32_t v = __builtin_bit_cast(uint32_t, __builtin_convertvector(x, bf16x2));
+    bits[k][i] = v;
+    if (k < 2) {
+      r[2 * i] = x[0] - __builtin_bit_cast(float, v << 16);
+      r[2 * i + 1] = x[1] - __builtin_bit_cast(float, v & 0xFFFF0000u);
+    }
+  }
+  __device__ __forceinline__ bf16x8 p(int k) const { return __builtin_bit_cast(bf16x8, bits[k]); }
+  __device__ __forceinline__ void all(const f32x4& a, const f32x4& b);
+};
+__device__ __forceinline__ void split_step(Split& s, int i, const f32x4& a, const f32x4& b) {
+  switch (i) {  // i: a constant after unrolling
+    case 0: s.step<0>(a, b); break;
+    case 1: s.step<1>(a, b); break;
+    case 2: s.step<2>(a, b); break;
+    case 3: s.step<3>(a, b); break;
+    case 4: s.step<4>(a, b); break;
+    case 5: s.step<5>(a, b); break;
+    case 6: s.step<6>(a, b); break;
+    case 7: s.step<7>(a, b); break;
+    case 8: s.step<8>(a, b); break;
+    case 9: s.step<9>(a, b); break;
+    case 10: s.step<10>(a, b); break;
+    case 11: s.step<11>(a, b); break;
+    default: break;
+  }
+}
+
+__device__ __forceinline__ void Split::all(const f32x4& a, const f32x4& b) {
+#pragma unroll
+  for (int i = 0; i < 12; ++i) split_step(*this, i, a, b);
 }
 
 // LDS image of a chunk, filled by direct loads (a wave instruction writes 64 lanes x 16 bytes in a row, so rows have no
-// padding; 16-byte pieces are swapped within a row instead, by the row number): k and q as 64 rows of 256 bytes, 64 columns
-// of v as 64 rows of 128 bytes, the chunk's blocks and factors as they are.
-constexpr int kTileQ = 16384, kTileV = 32768, kTileW = 40960, kTileBytes = kTileW + 4 * kChunkFloats;
-__device__ __forceinline__ int row_off(int row, int piece) { return row * 256 + 16 * (piece ^ (((row & 3) << 2) | ((row >> 2) & 3))); }
+// padding; 16-byte pieces are swapped within a row instead, by the row number): k as 64 rows of 256 bytes, 64 columns of v
+// as 64 rows of 128 bytes, the chunk's blocks and factors as they are.
+constexpr int kTileV = 16384, kTileW = 24576, kTileBytes = kTileW + (4 * kWalkFloats + 1023) / 1024 * 1024;
+__device__ __forceinline__ int piece_of(int row) { return ((row & 3) << 2) | ((row >> 2) & 3); }
+__device__ __forceinline__ int row_off(int row, int piece) { return row * 256 + 16 * (piece ^ piece_of(row)); }
 __device__ __forceinline__ int v_off(int row, int piece) { return row * 128 + 16 * (piece ^ (row & 7)); }
 __device__ __forceinline__ void direct_load(const void* src, char* dst) {
   __builtin_amdgcn_global_load_lds((__attribute__((address_space(1))) const void*)src,
@@ -467,7 +515,7 @@ __device__ __forceinline__ void direct_load(const void* src, char* dst) {
 }
 
 template <int KS>
-__global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf16> p, ChunkWs ws) {
+__global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<bf16> p, ChunkWs ws) {
   extern __shared__ __attribute__((aligned(1024))) char lds[];  // two chunks
   const Seq s = seq_of(p, blockIdx.z);
   if (s.n <= 0) return;
@@ -487,7 +535,7 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
     }
   // Rows past the end repeat the last one: their factors are zero. Key columns past dk stay zero: a row of S there would
   // take part otherwise.
-  const bf16* yq = p.y + (int64_t)s.q0 * C + hk * d.dk;
+  const bf16* yk = p.y + (int64_t)s.q0 * C + d.k0() + hk * d.dk;
   const bf16* yv = p.y + (int64_t)s.q0 * C + d.v0() + h * dv + c0;
   auto fetch = [&](int chunk) {
     char* tile = lds + (chunk & 1) * kTileBytes;
@@ -495,13 +543,8 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
     const int64_t at = (int64_t)chunk * kChunk * C;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {  // 4 rows an instruction
-      const int n = 4 * w + i, row = 4 * n + (lane >> 4);
-      const int e = 8 * ((lane & 15) ^ (((row & 3) << 2) | ((row >> 2) & 3)));
-      const bf16* src = yq + at + (uint32_t)(min(row, last) * C + e);
-      if (e < d.dk) {
-        direct_load(src + d.k0(), tile + n * 1024);
-        direct_load(src, tile + kTileQ + n * 1024);
-      }
+      const int n = 4 * w + i, row = 4 * n + (lane >> 4), e = 8 * ((lane & 15) ^ piece_of(row));
+      if (e < d.dk) direct_load(yk + at + (uint32_t)(min(row, last) * C + e), tile + n * 1024);
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {  // 8 rows an instruction
@@ -509,7 +552,7 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
       if (c0 + e < dv) direct_load(yv + at + (uint32_t)(min(row, last) * C + e), tile + kTileV + n * 1024);
     }
     const char* cw = reinterpret_cast<const char*>(ws.at(s, blockIdx.z, chunk, h, d.H)) + 16 * lane;
-    constexpr int kW = 4 * kChunkFloats;
+    constexpr int kW = 4 * kWalkFloats;
 #pragma unroll
     for (int i = 0; i < (kW + 4095) / 4096; ++i) {
       const int n = 4 * i + w;
@@ -528,157 +571,142 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
   const int col_at = row_off(4 * g + q, pp);    // ^ 64 (t >> 1); + 8 (t & 1), + 4096 per 16 tokens
   const int v_at = kTileV + v_off(4 * g + q, 2 * w + (pp >> 1)) + 8 * (pp & 1);  // + 2048 b
   fetch(0);
+  Split sp[2];
+  sp[0].all(S[0], S[1]);
   __syncthreads();
   for (int ch = 0; ch < chunks; ++ch) {
     const char* tile = lds + (ch & 1) * kTileBytes;
     if (active) {
       const char* cw = tile + kTileW;
-      auto block = [&](int x) { return *reinterpret_cast<const f32x4*>(cw + x * 1024 + l15 * 64 + 16 * g); };
-      auto factor = [&](int k, int b) {
-        return *reinterpret_cast<const f32x4*>(cw + 2 * kBlocks * 1024 + k * 4 * kChunk + 64 * b + 16 * g);
+      auto block = [&](int b, int j) {
+        return *reinterpret_cast<const f32x4*>(cw + block_at(b, j) * 1024 + l15 * 64 + 16 * g);
       };
-      const float keep = *reinterpret_cast<const float*>(cw + 2 * kBlocks * 1024 + 16 * kChunk);
+      auto factor = [&](int k, int b) {
+        return *reinterpret_cast<const f32x4*>(cw + kBlocks * 1024 + k * 4 * kChunk + 64 * b + 16 * g);
+      };
       // Operands are read from LDS one step ahead of the products that use them, products of different accumulators follow
       // one another, and the splits of the next operands lie between them: the scheduling barriers keep it so.
       bf16x4 v[4];
 #pragma unroll
       for (int b = 0; b < 4; ++b) v[b] = read_tr4(tile + v_at + 2048 * b);
-      bf16x8 kf[2][4], qf[2][4];
-      auto rows = [&](int ks, bf16x8 (&kk)[4], bf16x8 (&qq)[4]) {
-        const char* p0 = tile + (row_at ^ (64 * ks));
+      tr_wait(v[0], v[1]);
+      tr_wait(v[2], v[3]);
+      bf16x8 kf[2][4];
+      auto rows = [&](int ks, bf16x8 (&kk)[4]) {
 #pragma unroll
-        for (int b = 0; b < 4; ++b) {
-          kk[b] = *reinterpret_cast<const bf16x8*>(p0 + 4096 * b);
-          qq[b] = *reinterpret_cast<const bf16x8*>(p0 + kTileQ + 4096 * b);
-        }
+        for (int b = 0; b < 4; ++b) kk[b] = *reinterpret_cast<const bf16x8*>(tile + (row_at ^ (64 * ks)) + 4096 * b);
       };
-      rows(0, kf[0], qf[0]);
-      // the next chunk's loads go out before this chunk's work (transposed reads wait for direct loads before them: the
-      // ones below find them done)
+      rows(0, kf[0]);
+      // the next chunk's loads go out before this chunk's work
       __builtin_amdgcn_sched_barrier(0);
       if (ch + 1 < chunks) fetch(ch + 1);
-      f32x4 U[4], O[4];  // K S, then u; Q S, then o
-      bf16x8 sp[2][3];
-      split_tiles(S[0], S[1], sp[0][0], sp[0][1], sp[0][2]);
+      __builtin_amdgcn_sched_barrier(0);
+      float* keep_s = ws.at(s, blockIdx.z, ch, h, d.H) + kFixedFloats + (int64_t)(c0 / 16 + w) * strip_floats(KS) + 4 * lane;
 #pragma unroll
-      for (int b = 0; b < 4; ++b) U[b] = O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-      f32x4 M1[4][4], A[4][4], f0[4], f1[4];  // [row block][column block]
-      auto column = [&](int j) {
+      for (int t = 0; t < 2 * KS; ++t) *reinterpret_cast<f32x4*>(keep_s + 256 * t) = S[t];
+      f32x4 U[4];  // K S, then u
 #pragma unroll
-        for (int b = j; b < 4; ++b) {
-          M1[b][j] = block(block_at(b, j));
-          A[b][j] = block(kBlocks + block_at(b, j));
-        }
-      };
+      for (int b = 0; b < 4; ++b) U[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+      f32x4 M1[4][4], f0[4], f1[4], f3[4];  // [row block][column block]
+      const float keep = *reinterpret_cast<const float*>(cw + kBlocks * 1024 + 16 * kChunk);
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
         __builtin_amdgcn_sched_barrier(0);
         if (ks + 1 < KS) {
-          rows(ks + 1, kf[(ks + 1) & 1], qf[(ks + 1) & 1]);
+          rows(ks + 1, kf[(ks + 1) & 1]);
         } else {
 #pragma unroll
           for (int b = 0; b < 4; ++b) {
             f0[b] = factor(0, b);
             f1[b] = factor(1, b);
           }
-          column(0);
-        }
-        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int k = 2; k >= 0; --k) {  // the smallest piece first
+          for (int b = 0; b < 4; ++b)
 #pragma unroll
-          for (int b = 0; b < 4; ++b) {
-            U[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][b], sp[ks & 1][k], U[b], 0, 0, 0);
-            O[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ks & 1][b], sp[ks & 1][k], O[b], 0, 0, 0);
-          }
-        }
-        if (ks + 1 < KS) {
-          bf16x8(&n)[3] = sp[(ks + 1) & 1];
-          split_tiles(S[2 * ks + 2], S[2 * ks + 3], n[0], n[1], n[2]);
+            for (int j = 0; j <= b; ++j) M1[b][j] = block(b, j);
         }
 #pragma unroll
-        for (int i = 0; i < 24; ++i) {
-          __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);  // a product,
-          __builtin_amdgcn_sched_group_barrier(0x002, 3, 0);  // vector instructions under it
+        for (int i = 0; i < 12; ++i) {  // the smallest piece first
+          __builtin_amdgcn_sched_barrier(0);
+          U[i & 3] = mfma_bf16(kf[ks & 1][i & 3], sp[ks & 1].p(2 - i / 4), U[i & 3]);
+          if (ks + 1 < KS) split_step(sp[(ks + 1) & 1], i, S[2 * ks + 2], S[2 * ks + 3]);
         }
       }
       __builtin_amdgcn_sched_barrier(0);
-      f32x4 f2[4], f3[4];
-      bf16x8 kt[2 * KS];  // transposed k: all key dims of 32 tokens
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) U[b][r] = f1[b][r] * (float)v[b][r] - f0[b][r] * U[b][r];
+      bf16x4 kt[2][2 * KS][2];  // transposed k: all key dims of 32 tokens
       auto cols = [&](int hf) {
 #pragma unroll
         for (int t = 0; t < 2 * KS; ++t) {
           const char* p0 = tile + (col_at ^ (64 * (t >> 1))) + 8 * (t & 1) + 8192 * hf;
-          kt[t] = __builtin_shufflevector(read_tr4(p0), read_tr4(p0 + 4096), 0, 1, 2, 3, 4, 5, 6, 7);
+          kt[hf][t][0] = read_tr4(p0);
+          kt[hf][t][1] = read_tr4(p0 + 4096);
         }
       };
-      bf16x8 up[2][3];
-#pragma unroll
-      for (int b = 0; b < 4; ++b) f2[b] = factor(2, b);
-#pragma unroll
-      for (int b = 0; b < 4; ++b) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) U[b][r] = f1[b][r] * (float)v[b][r] - f0[b][r] * U[b][r];
-        O[b] *= f2[b];
-      }
+      auto key = [&](int hf, int t) {
+        return __builtin_shufflevector(kt[hf][t][0], kt[hf][t][1], 0, 1, 2, 3, 4, 5, 6, 7);
+      };
+      Split up[2];
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         __builtin_amdgcn_sched_barrier(0);
-        if (j < 3) column(j + 1);
         f3[j] = factor(3, j);
         if (j == 2) cols(0);
         __builtin_amdgcn_sched_barrier(0);
-        U[j] = mfma_f32(M1[j][j], U[j], f32x4{0.f, 0.f, 0.f, 0.f});
+        f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
+        x = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][0], U[j][0], x, 0, 0, 0);
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][1], U[j][1], y, 0, 0, 0);
+        x = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][2], U[j][2], x, 0, 0, 0);
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][3], U[j][3], y, 0, 0, 0);
+        if (j < 2)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
+          for (int t = KS * j; t < KS * (j + 1); ++t) S[t] *= keep;
+        U[j] = x + y;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
 #pragma unroll
           for (int b = j + 1; b < 4; ++b) U[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[b][j][r], U[j][r], U[b], 0, 0, 0);
-#pragma unroll
-          for (int b = j; b < 4; ++b) O[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(A[b][j][r], U[j][r], O[b], 0, 0, 0);
-        }
-        if (j == 0)
-#pragma unroll
-          for (int t = 0; t < 2 * KS; ++t) S[t] *= keep;
-        if (j == 2) split_tiles(U[0] * f3[0], U[1] * f3[1], up[0][0], up[0][1], up[0][2]);
+        *reinterpret_cast<f32x4*>(keep_s + 256 * (2 * KS + j)) = U[j];
+        U[j] *= f3[j];
+        if (j == 2) up[0].all(U[0], U[1]);
       }
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int k = 2; k >= 0; --k)
-#pragma unroll
-        for (int t = 0; t < 2 * KS; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt[t], up[0][k], S[t], 0, 0, 0);
-      split_tiles(U[2] * f3[2], U[3] * f3[3], up[1][0], up[1][1], up[1][2]);
-#pragma unroll
-      for (int i = 0; i < 6 * KS; ++i) {
-        __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
-        __builtin_amdgcn_sched_group_barrier(0x002, 3, 0);
-      }
-      __builtin_amdgcn_sched_barrier(0);
+      for (int t = 0; t < 2 * KS; ++t) tr_wait(kt[0][t][0], kt[0][t][1]);
       cols(1);
 #pragma unroll
-      for (int k = 2; k >= 0; --k)
+      for (int i = 0; i < 6 * KS; ++i) {
+        __builtin_amdgcn_sched_barrier(0);
+        S[i % (2 * KS)] = mfma_bf16(key(0, i % (2 * KS)), up[0].p(2 - i / (2 * KS)), S[i % (2 * KS)]);
+        if (KS >= 2) split_step(up[1], i, U[2], U[3]);
+      }
+      if (KS < 2) up[1].all(U[2], U[3]);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int t = 0; t < 2 * KS; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt[t], up[1][k], S[t], 0, 0, 0);
-      if (ok) {
-        const int left = s.n - ch * kChunk;
-        float* o = p.o + ((int64_t)(s.q0 + ch * kChunk) * d.H + h) * dv + col;
-        const uint32_t ld = (uint32_t)(d.H * dv);
-        if (left >= kChunk) {
+      for (int t = 0; t < 2 * KS; ++t) tr_wait(kt[1][t][0], kt[1][t][1]);
 #pragma unroll
-          for (int b = 0; b < 4; ++b)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) o[(uint32_t)(16 * b + 4 * g + r) * ld] = O[b][r];
-        } else {
-#pragma unroll
-          for (int b = 0; b < 4; ++b)
-#pragma unroll
-            for (int r = 0; r < 4; ++r)
-              if (16 * b + 4 * g + r < left) o[(uint32_t)(16 * b + 4 * g + r) * ld] = O[b][r];
+      for (int i = 0; i < 6 * KS; ++i) {
+        __builtin_amdgcn_sched_barrier(0);
+        S[i % (2 * KS)] = mfma_bf16(key(1, i % (2 * KS)), up[1].p(2 - i / (2 * KS)), S[i % (2 * KS)]);
+        if (i >= 4 * KS + 2) {  // S[0] and S[1] are done: the first operands of the next chunk
+          split_step(sp[0], 2 * (i - 4 * KS - 2), S[0], S[1]);
+          split_step(sp[0], 2 * (i - 4 * KS - 2) + 1, S[0], S[1]);
         }
       }
-    } else if (ch + 1 < chunks) {
-      fetch(ch + 1);
+#pragma unroll
+      for (int i = 4 * KS - 4; i < 12; ++i) split_step(sp[0], i, S[0], S[1]);
+      __builtin_amdgcn_sched_barrier(0);
+      // the direct loads went out before the stores of this chunk's S and U, which nobody here waits for
+      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(2 * KS + 4) : "memory");
+    } else {
+      if (ch + 1 < chunks) fetch(ch + 1);
+      asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" : : : "memory");
     }
-    __syncthreads();  // (also waits for the direct loads)
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" : : : "memory");
   }
   if (ok)
 #pragma unroll
@@ -688,6 +716,87 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_scan_kernel(DeltaParams<bf
         const int row = state_row(t, g, r);
         if (row < d.dk) st[(int64_t)row * dv + col] = S[t][r];
       }
+}
+
+// O = diag(e^G) Q S + A U of a chunk and head, its norm and gate. Eight waves share the head's columns, 16 at a time; then
+// LPU lanes a token, 8 columns each.
+template <int KS, int LPU>
+__global__ __launch_bounds__(512) void delta_chunk_out_kernel(DeltaParams<bf16> p, ChunkWs ws) {
+  extern __shared__ __attribute__((aligned(16))) float so[];  // [64][dv + 4]
+  const Seq s = seq_of(p, blockIdx.z);
+  const int chunk = blockIdx.x, h = blockIdx.y;
+  const int left = s.n - chunk * kChunk;
+  if (left <= 0) return;
+  const DeltaDims& d = p.d;
+  const int hk = h / (d.H / d.G), C = d.C(), dv = d.dv, ld = dv + 4;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
+  const int64_t t0 = s.q0 + chunk * kChunk;
+  const float* cw = ws.at(s, blockIdx.z, chunk, h, d.H);
+  const int strips = (dv + 15) / 16;
+  if (w < strips) {
+    bf16x8 qf[KS][4];
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        const int e = 32 * ks + 8 * g;
+        qf[ks][b] = bf16x8{};
+        if (e < d.dk) qf[ks][b] = *reinterpret_cast<const bf16x8*>(p.y + (t0 + min(16 * b + l15, left - 1)) * C + hk * d.dk + e);
+      }
+    for (int strip = w; strip < strips; strip += 8) {
+      const float* sw = cw + kFixedFloats + (int64_t)strip * strip_floats(KS) + 4 * lane;
+      f32x4 S[2 * KS], U[4], O[4];
+#pragma unroll
+      for (int t = 0; t < 2 * KS; ++t) S[t] = *reinterpret_cast<const f32x4*>(sw + 256 * t);
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        U[b] = *reinterpret_cast<const f32x4*>(sw + 256 * (2 * KS + b));
+        O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+      }
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        Split sp;
+        sp.all(S[2 * ks], S[2 * ks + 1]);
+#pragma unroll
+        for (int k = 2; k >= 0; --k)
+#pragma unroll
+          for (int b = 0; b < 4; ++b) O[b] = mfma_bf16(qf[ks][b], sp.p(k), O[b]);
+      }
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        O[b] *= *reinterpret_cast<const f32x4*>(cw + kBlocks * 256 + 2 * kChunk + 16 * b + 4 * g);
+#pragma unroll
+        for (int j = 0; j <= b; ++j)
+          O[b] = mfma_f32(*reinterpret_cast<const f32x4*>(cw + kWalkFloats + block_at(b, j) * 256 + l15 * 16 + 4 * g), U[j],
+                          O[b]);
+      }
+      if (16 * strip + l15 < dv)
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) so[(16 * b + 4 * g + r) * ld + 16 * strip + l15] = O[b][r];
+    }
+  }
+  __syncthreads();
+  const int e = 8 * (threadIdx.x % LPU);
+  float nw[8];
+  if (e < dv) Vec8<float>::load(p.norm + e, nw);
+  for (int i = threadIdx.x / LPU; i < kChunk; i += 512 / LPU) {
+    const bool on = i < left && e < dv;
+    float o[8], gt[8], ss = 0.f;
+    if (on) {
+      Vec8<float>::load(so + i * ld + e, o);
+      Vec8<bf16>::load(p.proj + (t0 + i) * d.ld + C + h * dv + e, gt);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) ss += o[x] * o[x];
+    }
+    ss = group_sum<LPU>(ss);
+    if (!on) continue;
+    const float rs = 1.f / sqrtf(ss / (float)dv + p.eps);
+#pragma unroll
+    for (int x = 0; x < 8; ++x) o[x] *= rs * nw[x] * silu_act<bf16>(gt[x]);
+    Vec8<bf16>::store(p.out + (t0 + i) * p.ldo + h * dv + e, o);
+  }
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -905,25 +1014,45 @@ int launch_scan(const DeltaParams<T>& p, int n_seqs, hipStream_t st) {
   return hipGetLastError();
 }
 
-bool chunk_ok(int dtype, int dk, int dv) { return dtype == kBF16 && dk % 8 == 0 && dv % 8 == 0 && dk <= 128; }
+bool chunk_ok(int dtype, int dk, int dv) {
+  return dtype == kBF16 && dk % 8 == 0 && dv % 8 == 0 && dk <= 128 && dv <= 512;
+}
+int chunk_ks(int dk) { return dk <= 32 ? 1 : dk <= 64 ? 2 : 4; }
+int chunk_floats(int dk, int dv) { return kFixedFloats + (dv + 15) / 16 * strip_floats(chunk_ks(dk)); }
+
+template <int KS, int LPU>
+int launch_chunk_out(const DeltaParams<bf16>& p, const ChunkWs& ws, dim3 grid, hipStream_t st) {
+  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_out_kernel<KS, LPU>,
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+  if (attr != hipSuccess) return attr;
+  hipLaunchKernelGGL((delta_chunk_out_kernel<KS, LPU>), grid, dim3(512), kChunk * (p.d.dv + 4) * sizeof(float), st, p, ws);
+  return hipGetLastError();
+}
 
 template <int KS>
 int launch_chunks_as(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, int max_new, hipStream_t st) {
   constexpr int lds = 2 * kTileBytes;
-  static_assert(lds <= 160 * 1024, "LDS");
-  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_scan_kernel<KS>,
+  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_state_kernel<KS>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   if (attr != hipSuccess) return attr;
-  hipLaunchKernelGGL(delta_chunk_prep_kernel<KS>, dim3((max_new + kChunk - 1) / kChunk, p.d.H, n_seqs), dim3(256), 0, st,
-                     p, ws);
-  hipLaunchKernelGGL(delta_chunk_scan_kernel<KS>, dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p, ws);
-  return hipGetLastError();
+  const dim3 grid((max_new + kChunk - 1) / kChunk, p.d.H, n_seqs);
+  hipLaunchKernelGGL(delta_chunk_prep_kernel<KS>, grid, dim3(256), 0, st, p, ws);
+  hipLaunchKernelGGL(delta_chunk_state_kernel<KS>, dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p, ws);
+  if (const hipError_t e = hipGetLastError()) return e;
+  if (p.d.dv <= 64) return launch_chunk_out<KS, 8>(p, ws, grid, st);
+  if (p.d.dv <= 128) return launch_chunk_out<KS, 16>(p, ws, grid, st);
+  if (p.d.dv <= 256) return launch_chunk_out<KS, 32>(p, ws, grid, st);
+  return launch_chunk_out<KS, 64>(p, ws, grid, st);
 }
 
-int launch_chunks(const DeltaParams<bf16>& p, float* ws, int n_seqs, int max_new, hipStream_t st) {
-  if (p.d.dk <= 32) return launch_chunks_as<1>(p, ChunkWs{ws}, n_seqs, max_new, st);
-  if (p.d.dk <= 64) return launch_chunks_as<2>(p, ChunkWs{ws}, n_seqs, max_new, st);
-  return launch_chunks_as<4>(p, ChunkWs{ws}, n_seqs, max_new, st);
+// the scan and what follows it
+int launch_chunks(const DeltaParams<bf16>& p, float* base, int n_seqs, int max_new, hipStream_t st) {
+  const ChunkWs ws{base, chunk_floats(p.d.dk, p.d.dv)};
+  switch (chunk_ks(p.d.dk)) {
+    case 1: return launch_chunks_as<1>(p, ws, n_seqs, max_new, st);
+    case 2: return launch_chunks_as<2>(p, ws, n_seqs, max_new, st);
+    default: return launch_chunks_as<4>(p, ws, n_seqs, max_new, st);
+  }
 }
 
 // threads and rows a thread of delta_step; 0: the kernel does not take these sizes
@@ -992,12 +1121,14 @@ HDS_EXPORT int hds_delta_step(int dtype, const void* proj, int64_t ld, const flo
 
 // floats of the chunk scan's scratch memory per chunk and head (a step of n tokens has up to n / 64 + n_seqs chunks);
 // 0: heads of these sizes and this type are scanned token by token
-HDS_EXPORT int hds_delta_chunk_floats(int dtype, int dk, int dv) { return chunk_ok(dtype, dk, dv) ? kChunkFloats : 0; }
+HDS_EXPORT int hds_delta_chunk_floats(int dtype, int dk, int dv) {
+  return chunk_ok(dtype, dk, dv) ? chunk_floats(dk, dv) : 0;
+}
 HDS_EXPORT int hds_delta_chunk_tokens() { return kChunk; }
 
-// Portions of at most max_new tokens. y [tokens, C], rn [tokens, 2 G], gb [tokens, H, 2] and o [tokens, H, dv] are
-// scratch memory with a row for every token of the step; chunks: scratch memory of the chunk scan (the sequences ascend in
-// the step's rows), or null: token by token.
+// Portions of at most max_new tokens. y [tokens, C], rn [tokens, 2 G] and gb [tokens, H, 2] are scratch memory with a row
+// for every token of the step. chunks: scratch memory of the scan by chunks (the sequences ascend in the step's rows; proj
+// and out rows 16-byte aligned); null: token by token, with o [tokens, H, dv] as scratch memory.
 HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
                               const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
                               const int* seq_meta, const int* seqs, void* y, float* rn, float* gb, float* o, float* chunks,
@@ -1005,7 +1136,7 @@ HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const flo
                               hipStream_t st) {
   if (n_seqs <= 0 || max_new <= 0) return 0;
   const DeltaDims d{H, G, dk, dv, taps, ld};
-  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || !y || !rn || !gb || !o || ldo < (int64_t)H * dv ||
+  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || !y || !rn || !gb || ldo < (int64_t)H * dv ||
       slot_stride < d.states() + (int64_t)taps * d.C())
     return hipErrorInvalidValue;
 #define HDS_DX(TT)                                                                                                   \
@@ -1013,15 +1144,17 @@ HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const flo
     const DeltaParams<TT> p{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, seqs,     \
                             (TT*)y, rn, gb, o, (TT*)out, ldo, 0, eps};                                               \
     if (int e = launch_conv(p, n_seqs, max_new, st)) return e;                                                       \
-    if (int e = scan(p)) return e;                                                                                   \
-    return launch_out(p, n_seqs, max_new, st);                                                                       \
+    return scan(p);                                                                                                  \
   }
   const auto scan = [&](const auto& p) -> int {
     if constexpr (std::is_same<decltype(p.proj), const bf16*>::value)
       if (chunks != nullptr) return launch_chunks(p, chunks, n_seqs, max_new, st);
-    return launch_scan(p, n_seqs, st);
+    if (int e = launch_scan(p, n_seqs, st)) return e;
+    return launch_out(p, n_seqs, max_new, st);
   };
-  if (chunks != nullptr && !chunk_ok(dtype, dk, dv)) return hipErrorInvalidValue;
+  if (chunks == nullptr && o == nullptr) return hipErrorInvalidValue;
+  if (chunks != nullptr && (!chunk_ok(dtype, dk, dv) || ld % 8 || ldo % 8 || (uintptr_t)proj % 16 || (uintptr_t)out % 16))
+    return hipErrorInvalidValue;
   if (dtype == kBF16) HDS_DX(bf16)
   if (dtype == kF32) HDS_DX(float)
 #undef HDS_DX

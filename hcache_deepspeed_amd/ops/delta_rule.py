@@ -100,11 +100,12 @@ def delta_rule(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch
         f32 = dict(dtype=torch.float32, device=dev)
         y = torch.empty(T, sh.channels, dtype=proj.dtype, device=dev)
         rn, gb = torch.empty(T, 2 * sh.kv_heads, **f32), torch.empty(T, sh.heads, 2, **f32)
-        o = torch.empty(T, sh.heads, sh.vdim, **f32)
-        n_ws = _chunk_floats(sh, proj.dtype, T, plan.n_scan) if plan.max_new > SERIAL_MAX else 0
+        aligned = all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (proj, out))
+        n_ws = _chunk_floats(sh, proj.dtype, T, plan.n_scan) if aligned and plan.max_new > SERIAL_MAX else 0
         ws = torch.empty(n_ws, **f32) if n_ws else None
+        o = None if n_ws else torch.empty(T, sh.heads, sh.vdim, **f32)
         native.check(
-            lib.hds_delta_scan(*head, native.ptr(plan.scan), y.data_ptr(), rn.data_ptr(), gb.data_ptr(), o.data_ptr(),
+            lib.hds_delta_scan(*head, native.ptr(plan.scan), y.data_ptr(), rn.data_ptr(), gb.data_ptr(), native.ptr(o),
                                native.ptr(ws), out.data_ptr(), out.stride(0), plan.n_scan, plan.max_new, *dims), "delta_scan")
     return out
 
