@@ -445,9 +445,10 @@ __device__ __forceinline__ f32x4 mfma_f32(const f32x4& a, const f32x4& b, f32x4 
 }
 // Transposed LDS reads as inline asm: in front of the builtin the compiler waits for every direct load and store under way
 // (it cannot tell that they go elsewhere). tr_wait is due before the values are used.
+template <int OFF>
 __device__ __forceinline__ bf16x4 read_tr4(const char* a) {
   bf16x4 r;
-  asm volatile("ds_read_b64_tr_b16 %0, %1" : "=v"(r) : "v"((uint32_t)(uintptr_t)a) : "memory");
+  asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(r) : "v"((uint32_t)(uintptr_t)a), "n"(OFF) : "memory");
   return r;
 }
 __device__ __forceinline__ void tr_wait(bf16x4& a, bf16x4& b) {
@@ -505,7 +506,8 @@ __device__ __forceinline__ void Split::all(const f32x4& a, const f32x4& b) {
 // LDS image of a chunk, filled by direct loads (a wave instruction writes 64 lanes x 16 bytes in a row, so rows have no
 // padding; 16-byte pieces are swapped within a row instead, by the row number): k as 64 rows of 256 bytes, 64 columns of v
 // as 64 rows of 128 bytes, the chunk's blocks and factors as they are.
-constexpr int kTileV = 16384, kTileW = 24576, kTileBytes = kTileW + (4 * kWalkFloats + 1023) / 1024 * 1024;
+constexpr int kTileV = 16384, kTileW = 24576, kTileBytes = kTileW + (4 * kWalkFloats + 4095) / 4096 * 4096;
+static_assert((4 * kWalkFloats + 4095) / 4096 * 4096 <= 4 * kFixedFloats, "reads past the entry");
 __device__ __forceinline__ int piece_of(int row) { return ((row & 3) << 2) | ((row >> 2) & 3); }
 __device__ __forceinline__ int row_off(int row, int piece) { return row * 256 + 16 * (piece ^ piece_of(row)); }
 __device__ __forceinline__ int v_off(int row, int piece) { return row * 128 + 16 * (piece ^ (row & 7)); }
@@ -514,16 +516,17 @@ __device__ __forceinline__ void direct_load(const void* src, char* dst) {
                                    (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
 }
 
-template <int KS>
+// FULL: dk == 32 KS and dv a multiple of 64 (no lane of a direct load is left out, which would split the schedule)
+template <int KS, bool FULL>
 __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<bf16> p, ChunkWs ws) {
-  extern __shared__ __attribute__((aligned(1024))) char lds[];  // two chunks
+  extern __shared__ __attribute__((aligned(1024))) char lds[];  // three chunks: this one, the next, the one on its way
   const Seq s = seq_of(p, blockIdx.z);
   if (s.n <= 0) return;
   const DeltaDims& d = p.d;
   const int h = blockIdx.y, hk = h / (d.H / d.G), C = d.C(), dv = d.dv;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
   const int c0 = blockIdx.x * 64, col = c0 + 16 * w + l15;
-  const bool active = c0 + 16 * w < dv, ok = col < dv;
+  const bool active = FULL || c0 + 16 * w < dv, ok = FULL || col < dv;
   float* st = p.state + (int64_t)s.slot * p.slot_stride + (int64_t)h * d.dk * dv;
   f32x4 S[2 * KS];
 #pragma unroll
@@ -537,31 +540,31 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   // take part otherwise.
   const bf16* yk = p.y + (int64_t)s.q0 * C + d.k0() + hk * d.dk;
   const bf16* yv = p.y + (int64_t)s.q0 * C + d.v0() + h * dv + c0;
-  auto fetch = [&](int chunk) {
-    char* tile = lds + (chunk & 1) * kTileBytes;
+  constexpr int kLoads = 6 + (4 * kWalkFloats + 4095) / 4096;  // direct loads a wave issues for a chunk
+  static_assert(kLoads == 9, "six between the products of K S, three later");
+  auto fetch_one = [&](int buffer, int chunk, int i) {
+    char* tile = lds + buffer * kTileBytes;
     const int last = s.n - 1 - chunk * kChunk;
     const int64_t at = (int64_t)chunk * kChunk * C;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {  // 4 rows an instruction
+    if (i < 4) {  // 4 rows of k an instruction
       const int n = 4 * w + i, row = 4 * n + (lane >> 4), e = 8 * ((lane & 15) ^ piece_of(row));
-      if (e < d.dk) direct_load(yk + at + (uint32_t)(min(row, last) * C + e), tile + n * 1024);
-    }
-#pragma unroll
-    for (int i = 0; i < 2; ++i) {  // 8 rows an instruction
-      const int n = 2 * w + i, row = 8 * n + (lane >> 3), e = 8 * ((lane & 7) ^ (row & 7));
-      if (c0 + e < dv) direct_load(yv + at + (uint32_t)(min(row, last) * C + e), tile + kTileV + n * 1024);
-    }
-    const char* cw = reinterpret_cast<const char*>(ws.at(s, blockIdx.z, chunk, h, d.H)) + 16 * lane;
-    constexpr int kW = 4 * kWalkFloats;
-#pragma unroll
-    for (int i = 0; i < (kW + 4095) / 4096; ++i) {
-      const int n = 4 * i + w;
-      if (n * 1024 + 16 * lane < kW) direct_load(cw + n * 1024, tile + kTileW + n * 1024);
+      if (FULL || e < d.dk) direct_load(yk + at + (uint32_t)(min(row, last) * C + e), tile + n * 1024);
+    } else if (i < 6) {  // 8 rows of v
+      const int n = 2 * w + i - 4, row = 8 * n + (lane >> 3), e = 8 * ((lane & 7) ^ (row & 7));
+      if (FULL || c0 + e < dv) direct_load(yv + at + (uint32_t)(min(row, last) * C + e), tile + kTileV + n * 1024);
+    } else {
+      const char* cw = reinterpret_cast<const char*>(ws.at(s, blockIdx.z, chunk, h, d.H)) + 16 * lane;
+      const int n = 4 * (i - 6) + w;  // (the last one reads into the blocks of A)
+      direct_load(cw + n * 1024, tile + kTileW + n * 1024);
     }
   };
+  auto fetch = [&](int buffer, int chunk) {
+#pragma unroll
+    for (int i = 0; i < kLoads; ++i) fetch_one(buffer, chunk, i);
+  };
   const int chunks = (s.n + kChunk - 1) / kChunk;
-  if (d.dk < 32 * KS) {
-    for (int i = threadIdx.x; i < 2 * kTileBytes / 16; i += 256) reinterpret_cast<u32x4*>(lds)[i] = u32x4{};
+  if (!FULL && d.dk < 32 * KS) {
+    for (int i = threadIdx.x; i < 3 * kTileBytes / 16; i += 256) reinterpret_cast<u32x4*>(lds)[i] = u32x4{};
     __syncthreads();
   }
   // Offsets of this lane's reads in a tile. Row blocks and halves are 16-row steps, which leave the swap of the pieces as
@@ -570,12 +573,16 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   const int row_at = row_off(l15, g);           // ^ 64 ks; + 4096 b
   const int col_at = row_off(4 * g + q, pp);    // ^ 64 (t >> 1); + 8 (t & 1), + 4096 per 16 tokens
   const int v_at = kTileV + v_off(4 * g + q, 2 * w + (pp >> 1)) + 8 * (pp & 1);  // + 2048 b
-  fetch(0);
+  fetch(0, 0);
+  fetch(1, min(1, chunks - 1));
   Split sp[2];
   sp[0].all(S[0], S[1]);
   __syncthreads();
+  int buffer = 0;
   for (int ch = 0; ch < chunks; ++ch) {
-    const char* tile = lds + (ch & 1) * kTileBytes;
+    const char* tile = lds + buffer * kTileBytes;
+    const int free = buffer == 0 ? 2 : buffer - 1;      // was read in the step before
+    const int next = min(ch + 2, chunks - 1);           // (the last one again: no branch)
     if (active) {
       const char* cw = tile + kTileW;
       auto block = [&](int b, int j) {
@@ -587,8 +594,10 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
       // Operands are read from LDS one step ahead of the products that use them, products of different accumulators follow
       // one another, and the splits of the next operands lie between them: the scheduling barriers keep it so.
       bf16x4 v[4];
-#pragma unroll
-      for (int b = 0; b < 4; ++b) v[b] = read_tr4(tile + v_at + 2048 * b);
+      v[0] = read_tr4<0>(tile + v_at);
+      v[1] = read_tr4<2048>(tile + v_at);
+      v[2] = read_tr4<4096>(tile + v_at);
+      v[3] = read_tr4<6144>(tile + v_at);
       tr_wait(v[0], v[1]);
       tr_wait(v[2], v[3]);
       bf16x8 kf[2][4];
@@ -597,13 +606,7 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
         for (int b = 0; b < 4; ++b) kk[b] = *reinterpret_cast<const bf16x8*>(tile + (row_at ^ (64 * ks)) + 4096 * b);
       };
       rows(0, kf[0]);
-      // the next chunk's loads go out before this chunk's work
-      __builtin_amdgcn_sched_barrier(0);
-      if (ch + 1 < chunks) fetch(ch + 1);
-      __builtin_amdgcn_sched_barrier(0);
       float* keep_s = ws.at(s, blockIdx.z, ch, h, d.H) + kFixedFloats + (int64_t)(c0 / 16 + w) * strip_floats(KS) + 4 * lane;
-#pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) *reinterpret_cast<f32x4*>(keep_s + 256 * t) = S[t];
       f32x4 U[4];  // K S, then u
 #pragma unroll
       for (int b = 0; b < 4; ++b) U[b] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -619,6 +622,7 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
           for (int b = 0; b < 4; ++b) {
             f0[b] = factor(0, b);
             f1[b] = factor(1, b);
+            f3[b] = factor(3, b);
           }
 #pragma unroll
           for (int b = 0; b < 4; ++b)
@@ -630,6 +634,8 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
           __builtin_amdgcn_sched_barrier(0);
           U[i & 3] = mfma_bf16(kf[ks & 1][i & 3], sp[ks & 1].p(2 - i / 4), U[i & 3]);
           if (ks + 1 < KS) split_step(sp[(ks + 1) & 1], i, S[2 * ks + 2], S[2 * ks + 3]);
+          // loads and stores are spread over the step: the wave would wait for a queue that is full
+          if ((12 * ks + i) % (2 * KS) == 2 * KS - 1) fetch_one(free, next, (12 * ks + i) / (2 * KS));  // 0 .. 5
         }
       }
       __builtin_amdgcn_sched_barrier(0);
@@ -641,9 +647,11 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
       auto cols = [&](int hf) {
 #pragma unroll
         for (int t = 0; t < 2 * KS; ++t) {
-          const char* p0 = tile + (col_at ^ (64 * (t >> 1))) + 8 * (t & 1) + 8192 * hf;
-          kt[hf][t][0] = read_tr4(p0);
-          kt[hf][t][1] = read_tr4(p0 + 4096);
+          const char* p0 = tile + (col_at ^ (64 * (t >> 1)));
+          kt[hf][t][0] = hf == 0 ? (t & 1 ? read_tr4<8>(p0) : read_tr4<0>(p0))
+                                 : (t & 1 ? read_tr4<8200>(p0) : read_tr4<8192>(p0));
+          kt[hf][t][1] = hf == 0 ? (t & 1 ? read_tr4<4104>(p0) : read_tr4<4096>(p0))
+                                 : (t & 1 ? read_tr4<12296>(p0) : read_tr4<12288>(p0));
         }
       };
       auto key = [&](int hf, int t) {
@@ -653,22 +661,25 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         __builtin_amdgcn_sched_barrier(0);
-        f3[j] = factor(3, j);
-        if (j == 2) cols(0);
+        if (j == 1) cols(0);
         __builtin_amdgcn_sched_barrier(0);
         f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
         x = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][0], U[j][0], x, 0, 0, 0);
         y = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][1], U[j][1], y, 0, 0, 0);
         x = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][2], U[j][2], x, 0, 0, 0);
         y = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[j][j][3], U[j][3], y, 0, 0, 0);
-        if (j < 2)
-#pragma unroll
-          for (int t = KS * j; t < KS * (j + 1); ++t) S[t] *= keep;
         U[j] = x + y;
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
+        for (int r = 0; r < 4; ++r) {
 #pragma unroll
           for (int b = j + 1; b < 4; ++b) U[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[b][j][r], U[j][r], U[b], 0, 0, 0);
+          const int t = j == 0 ? r : (j == 1 ? 4 + r : 2 * KS);  // S goes out, then decays
+          if (t < 2 * KS) {
+            *reinterpret_cast<f32x4*>(keep_s + 256 * t) = S[t];
+            S[t] *= keep;
+            __builtin_amdgcn_sched_barrier(0);
+          }
+        }
         *reinterpret_cast<f32x4*>(keep_s + 256 * (2 * KS + j)) = U[j];
         U[j] *= f3[j];
         if (j == 2) up[0].all(U[0], U[1]);
@@ -682,31 +693,35 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
         __builtin_amdgcn_sched_barrier(0);
         S[i % (2 * KS)] = mfma_bf16(key(0, i % (2 * KS)), up[0].p(2 - i / (2 * KS)), S[i % (2 * KS)]);
         if (KS >= 2) split_step(up[1], i, U[2], U[3]);
+        if (i % (2 * KS) == 0) fetch_one(free, next, 6 + i / (2 * KS));
       }
       if (KS < 2) up[1].all(U[2], U[3]);
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
       for (int t = 0; t < 2 * KS; ++t) tr_wait(kt[1][t][0], kt[1][t][1]);
+      // tiles 0 and 1 first: their sum is the first operand of the next chunk
 #pragma unroll
-      for (int i = 0; i < 6 * KS; ++i) {
+      for (int i = 0; i < 6; ++i) S[i & 1] = mfma_bf16(key(1, i & 1), up[1].p(2 - i / 2), S[i & 1]);
+      constexpr int R = 2 * KS - 2;  // the other tiles
+#pragma unroll
+      for (int i = 0; i < 3 * R; ++i) {
         __builtin_amdgcn_sched_barrier(0);
-        S[i % (2 * KS)] = mfma_bf16(key(1, i % (2 * KS)), up[1].p(2 - i / (2 * KS)), S[i % (2 * KS)]);
-        if (i >= 4 * KS + 2) {  // S[0] and S[1] are done: the first operands of the next chunk
-          split_step(sp[0], 2 * (i - 4 * KS - 2), S[0], S[1]);
-          split_step(sp[0], 2 * (i - 4 * KS - 2) + 1, S[0], S[1]);
-        }
+        S[2 + i % (R > 0 ? R : 1)] = mfma_bf16(key(1, 2 + i % (R > 0 ? R : 1)), up[1].p(2 - i / (R > 0 ? R : 1)),
+                                               S[2 + i % (R > 0 ? R : 1)]);
+        if (i >= 2) split_step(sp[0], i - 2, S[0], S[1]);
       }
 #pragma unroll
-      for (int i = 4 * KS - 4; i < 12; ++i) split_step(sp[0], i, S[0], S[1]);
+      for (int i = R > 0 ? 3 * R - 2 : 0; i < 12; ++i) split_step(sp[0], i, S[0], S[1]);
       __builtin_amdgcn_sched_barrier(0);
-      // the direct loads went out before the stores of this chunk's S and U, which nobody here waits for
-      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(2 * KS + 4) : "memory");
+      // the next chunk's loads went out a step ago: all but this step's loads and stores have to be done
+      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(kLoads + 2 * KS + 4) : "memory");
     } else {
-      if (ch + 1 < chunks) fetch(ch + 1);
-      asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" : : : "memory");
+      fetch(free, next);
+      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(kLoads) : "memory");
     }
     __builtin_amdgcn_s_barrier();
     asm volatile("" : : : "memory");
+    buffer = buffer == 2 ? 0 : buffer + 1;
   }
   if (ok)
 #pragma unroll
@@ -1029,16 +1044,26 @@ int launch_chunk_out(const DeltaParams<bf16>& p, const ChunkWs& ws, dim3 grid, h
   return hipGetLastError();
 }
 
-template <int KS>
-int launch_chunks_as(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, int max_new, hipStream_t st) {
-  constexpr int lds = 2 * kTileBytes;
-  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_state_kernel<KS>,
+template <int KS, bool FULL>
+int launch_chunk_state(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, hipStream_t st) {
+  constexpr int lds = 3 * kTileBytes;
+  static_assert(lds <= 160 * 1024, "LDS");
+  static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_state_kernel<KS, FULL>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   if (attr != hipSuccess) return attr;
+  hipLaunchKernelGGL((delta_chunk_state_kernel<KS, FULL>), dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p,
+                     ws);
+  return hipGetLastError();
+}
+
+template <int KS>
+int launch_chunks_as(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, int max_new, hipStream_t st) {
   const dim3 grid((max_new + kChunk - 1) / kChunk, p.d.H, n_seqs);
   hipLaunchKernelGGL(delta_chunk_prep_kernel<KS>, grid, dim3(256), 0, st, p, ws);
-  hipLaunchKernelGGL(delta_chunk_state_kernel<KS>, dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p, ws);
   if (const hipError_t e = hipGetLastError()) return e;
+  const bool full = p.d.dk == 32 * KS && p.d.dv % 64 == 0;
+  if (const int e = full ? launch_chunk_state<KS, true>(p, ws, n_seqs, st) : launch_chunk_state<KS, false>(p, ws, n_seqs, st))
+    return e;
   if (p.d.dv <= 64) return launch_chunk_out<KS, 8>(p, ws, grid, st);
   if (p.d.dv <= 128) return launch_chunk_out<KS, 16>(p, ws, grid, st);
   if (p.d.dv <= 256) return launch_chunk_out<KS, 32>(p, ws, grid, st);
