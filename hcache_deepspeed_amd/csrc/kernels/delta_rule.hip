@@ -438,11 +438,6 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaParams<bf16>
 // bfloat16 products holds
 __device__ __forceinline__ int state_row(int t, int g, int r) { return 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r; }
 
-__device__ __forceinline__ f32x4 mfma_f32(const f32x4& a, const f32x4& b, f32x4 c) {
-#pragma unroll
-  for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], c, 0, 0, 0);
-  return c;
-}
 // Transposed LDS reads as inline asm: in front of the builtin the compiler waits for every direct load and store under way
 // (it cannot tell that they go elsewhere). tr_wait is due before the values are used.
 template <int OFF>
@@ -736,7 +731,7 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
 // O = diag(e^G) Q S + A U of a chunk and head, its norm and gate. Eight waves share the head's columns, 16 at a time; then
 // LPU lanes a token, 8 columns each.
 template <int KS, int LPU>
-__global__ __launch_bounds__(512) void delta_chunk_out_kernel(DeltaParams<bf16> p, ChunkWs ws) {
+__global__ __launch_bounds__(512, 4) void delta_chunk_out_kernel(DeltaParams<bf16> p, ChunkWs ws) {
   extern __shared__ __attribute__((aligned(16))) float so[];  // [64][dv + 4]
   const Seq s = seq_of(p, blockIdx.z);
   const int chunk = blockIdx.x, h = blockIdx.y;
@@ -749,41 +744,62 @@ __global__ __launch_bounds__(512) void delta_chunk_out_kernel(DeltaParams<bf16> 
   const float* cw = ws.at(s, blockIdx.z, chunk, h, d.H);
   const int strips = (dv + 15) / 16;
   if (w < strips) {
-    bf16x8 qf[KS][4];
+    // rows past the end repeat the last one: they are not stored
+    const bf16* qr[4];
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-#pragma unroll
-      for (int b = 0; b < 4; ++b) {
-        const int e = 32 * ks + 8 * g;
-        qf[ks][b] = bf16x8{};
-        if (e < d.dk) qf[ks][b] = *reinterpret_cast<const bf16x8*>(p.y + (t0 + min(16 * b + l15, left - 1)) * C + hk * d.dk + e);
-      }
+    for (int b = 0; b < 4; ++b) qr[b] = p.y + (t0 + min(16 * b + l15, left - 1)) * C + hk * d.dk + 8 * g;
     for (int strip = w; strip < strips; strip += 8) {
       const float* sw = cw + kFixedFloats + (int64_t)strip * strip_floats(KS) + 4 * lane;
-      f32x4 S[2 * KS], U[4], O[4];
+      f32x4 U[4], O[4], S[2][2];
+      bf16x8 qf[2][4];
+      auto fetch = [&](int ks) {
+        S[ks & 1][0] = *reinterpret_cast<const f32x4*>(sw + 512 * ks);
+        S[ks & 1][1] = *reinterpret_cast<const f32x4*>(sw + 512 * ks + 256);
 #pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) S[t] = *reinterpret_cast<const f32x4*>(sw + 256 * t);
+        for (int b = 0; b < 4; ++b) {
+          qf[ks & 1][b] = bf16x8{};
+          if (32 * ks + 8 * g < d.dk) qf[ks & 1][b] = *reinterpret_cast<const bf16x8*>(qr[b] + 32 * ks);
+        }
+      };
+      fetch(0);
 #pragma unroll
-      for (int b = 0; b < 4; ++b) {
-        U[b] = *reinterpret_cast<const f32x4*>(sw + 256 * (2 * KS + b));
-        O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-      }
+      for (int b = 0; b < 4; ++b) O[b] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
+        if (ks + 1 < KS) {
+          fetch(ks + 1);
+        } else {
+#pragma unroll
+          for (int b = 0; b < 4; ++b) U[b] = *reinterpret_cast<const f32x4*>(sw + 256 * (2 * KS + b));
+        }
+        __builtin_amdgcn_sched_barrier(0);
         Split sp;
-        sp.all(S[2 * ks], S[2 * ks + 1]);
+        sp.all(S[ks & 1][0], S[ks & 1][1]);
 #pragma unroll
         for (int k = 2; k >= 0; --k)
 #pragma unroll
-          for (int b = 0; b < 4; ++b) O[b] = mfma_bf16(qf[ks][b], sp.p(k), O[b]);
+          for (int b = 0; b < 4; ++b) O[b] = mfma_bf16(qf[ks & 1][b], sp.p(k), O[b]);
+        __builtin_amdgcn_sched_barrier(0);
       }
+      auto block = [&](int b, int j) {
+        return *reinterpret_cast<const f32x4*>(cw + kWalkFloats + block_at(b, j) * 256 + l15 * 16 + 4 * g);
+      };
+      f32x4 A[2][4];
 #pragma unroll
       for (int b = 0; b < 4; ++b) {
+        A[0][b] = block(b, 0);
         O[b] *= *reinterpret_cast<const f32x4*>(cw + kBlocks * 256 + 2 * kChunk + 16 * b + 4 * g);
+      }
 #pragma unroll
-        for (int j = 0; j <= b; ++j)
-          O[b] = mfma_f32(*reinterpret_cast<const f32x4*>(cw + kWalkFloats + block_at(b, j) * 256 + l15 * 16 + 4 * g), U[j],
-                          O[b]);
+      for (int j = 0; j < 4; ++j) {
+#pragma unroll
+        for (int b = j + 1; b < 4; ++b) A[(j + 1) & 1][b] = block(b, j + 1);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int b = j; b < 4; ++b) O[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(A[j & 1][b][r], U[j][r], O[b], 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0);
       }
       if (16 * strip + l15 < dv)
 #pragma unroll
