@@ -890,8 +890,9 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams<T> p, int R)
 // ---------------------------------------------------------------------------------------------------------------
 // A thread keeps 4 columns of RPT rows of S. S^T k and S^T q come from one pass over the old state:
 // o = g S^T q + (k . q) u.
+// Loads go out in the order their values are needed: the convolution's, then S, then the norm's and the gate's.
 template <typename T, int RPT, int NT>
-__global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
+__global__ __launch_bounds__(NT, NT < 1024 ? 1 : (RPT <= 4 ? 8 : 4)) void delta_step_kernel(DeltaParams<T> p) {
   constexpr int NW = NT / 64;
   extern __shared__ float sm[];
   const DeltaDims& d = p.d;
@@ -913,26 +914,55 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
   const bool act = rg < RG;
   float* st = p.state + (int64_t)s.slot * p.slot_stride;
   float* Sp = st + ((int64_t)h * dk) * dv + 4 * c4;
+  const T* row = p.proj + (int64_t)s.q0 * d.ld;
+  float* ring = st + d.states();
+  const int now = s.seen % d.taps;  // ring entry of this token
+  constexpr int MT = 4;             // taps whose operands are requested together
+  auto channel = [&](int i) {
+    return i < dk ? hk * dk + i : (i < 2 * dk ? d.k0() + hk * dk + i - dk : d.v0() + h * dv + i - 2 * dk);
+  };
+  const int n_ch = 2 * dk + dv;
+  const int c_first = channel(min((int)threadIdx.x, n_ch - 1));
+  const bool few = d.taps <= MT;
+  float cw[MT], hist[MT];
+  if (few) {
+#pragma unroll
+    for (int k = 0; k < MT; ++k) {
+      cw[k] = k < d.taps ? p.cw[(int64_t)(d.taps - 1 - k) * C + c_first] : 0.f;
+      hist[k] = 0.f;
+      if (k == 0) hist[k] = to_f(row[c_first]);
+      else if (k < d.taps && s.seen >= k) hist[k] = ring[(int64_t)(now >= k ? now - k : now - k + d.taps) * C + c_first];
+    }
+  }
+  const float xb = to_f(row[d.b0() + h]), xa = to_f(row[d.b0() + d.H + h]), al = p.a_log[h], dt = p.dt[h];
   f32x4 S[RPT];
 #pragma unroll
   for (int r = 0; r < RPT; ++r) {
     S[r] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int row = rg + r * RG;
-    if (act && s.seen > 0 && row < dk) S[r] = *reinterpret_cast<const f32x4*>(Sp + (int64_t)row * dv);
+    const int e = rg + r * RG;
+    if (act && s.seen > 0 && e < dk) S[r] = *reinterpret_cast<const f32x4*>(Sp + (int64_t)e * dv);
   }
-  const T* row = p.proj + (int64_t)s.q0 * d.ld;
-  const float beta = sigmoid_f(to_f(row[d.b0() + h]));
-  const float g = expf(-expf(p.a_log[h]) * softplus_f(to_f(row[d.b0() + d.H + h]) + p.dt[h]));
+  const int o_first = min((int)threadIdx.x, dv - 1);
+  const float nw = p.norm[o_first], og = to_f(row[C + h * dv + o_first]);
+  const float beta = sigmoid_f(xb), g = expf(-expf(al) * softplus_f(xa + dt));
   // convolutions of this head's channels
-  float* ring = st + d.states();
-  for (int i = threadIdx.x; i < 2 * dk + dv; i += NT) {
-    const int c = i < dk ? hk * dk + i : (i < 2 * dk ? d.k0() + hk * dk + i - dk : d.v0() + h * dv + i - 2 * dk);
-    const float x = to_f(row[c]);
-    float a = p.cw[(int64_t)(d.taps - 1) * C + c] * x;
-    for (int k = 1; k < d.taps; ++k)
-      if (s.seen - k >= 0) a += p.cw[(int64_t)(d.taps - 1 - k) * C + c] * ring[(int64_t)((s.seen - k) % d.taps) * C + c];
+  for (int i = threadIdx.x; i < n_ch; i += NT) {
+    const int c = channel(i);
+    float x, a;
+    if (few && i == (int)threadIdx.x) {
+      x = hist[0];
+      a = cw[0] * x;
+#pragma unroll
+      for (int k = 1; k < MT; ++k) a += cw[k] * hist[k];
+    } else {
+      x = to_f(row[c]);
+      a = p.cw[(int64_t)(d.taps - 1) * C + c] * x;
+      for (int k = 1; k < d.taps; ++k)
+        if (s.seen >= k)
+          a += p.cw[(int64_t)(d.taps - 1 - k) * C + c] * ring[(int64_t)((s.seen - k) % d.taps) * C + c];
+    }
     sq[i] = rounded<T>(silu_act<T>(rounded<T>(a)));
-    if (i >= 2 * dk || h % (d.H / d.G) == 0) ring[(int64_t)(s.seen % d.taps) * C + c] = x;
+    if (i >= 2 * dk || h % (d.H / d.G) == 0) ring[(int64_t)now * C + c] = x;
   }
   __syncthreads();
   float qq = 0.f, kk = 0.f, kq = 0.f;
@@ -970,6 +1000,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
   __syncthreads();
   for (int c = threadIdx.x; c < dv; c += NT) {
     float a = 0.f, b = 0.f;
+#pragma unroll 8
     for (int i = 0; i < P; ++i) {
       a += part[(2 * i) * dv + c];
       b += part[(2 * i + 1) * dv + c];
@@ -992,8 +1023,9 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaParams<T> p) {
     for (int c = lane; c < dv; c += 64) ss += so[c] * so[c];
     const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dv + p.eps);
     for (int c = threadIdx.x; c < dv; c += NT)
-      p.out[(int64_t)s.q0 * p.ldo + h * dv + c] =
-          from_f<T>(so[c] * rs * p.norm[c] * silu_act<T>(to_f(row[C + h * dv + c])));
+      p.out[(int64_t)s.q0 * p.ldo + h * dv + c] = from_f<T>(
+          c == (int)threadIdx.x ? so[c] * rs * nw * silu_act<T>(og)
+                                : so[c] * rs * p.norm[c] * silu_act<T>(to_f(row[C + h * dv + c])));
   }
 }
 
