@@ -18,6 +18,7 @@ from hcache_deepspeed_amd.inference.v2.modules import (DSGatedMLPConfig, DSLinea
                                                        instantiate_gated_mlp, instantiate_linear, instantiate_mixer)
 from hcache_deepspeed_amd.ops import delta_rule as delta_op
 from hcache_deepspeed_amd.ops.delta_rule import DeltaShape, delta_rule, make_delta_plan, step_ok
+from hcache_deepspeed_amd.ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
 from hcache_deepspeed_amd.ops.output_norm import rms_rows, sandwich_norm, softcap_
 from hcache_deepspeed_amd.ops.paged import HeadShape, head_attention, head_blocks_ok, make_head_plan
 from hcache_deepspeed_amd.ops.rope import rope_amplitude, rope_inv_freq, rope_tables
@@ -387,6 +388,47 @@ def test_latent_attention(run, name, sizes):
         close(torch.cat(o), oracle.latent_attention(x, p, m, eps), dtype, f32=5e-5, bf16=4e-2)
 
 
+@pytest.mark.parametrize("name", ["exact", "odd"])
+@pytest.mark.parametrize("sizes", [[300], [1], [131, 2, 17]])
+def test_latent_attention_finds_one_key_at_any_distance(run, name, sizes):
+    """One latent's score towers over the others': every later query, next to it or hundreds of tokens on, gives back its
+    value times the head's gate, earlier ones do not see it."""
+    dev, dtype = run
+    H, d, r, rd, rank, _, e = LATENTS[name]
+    n = 300
+    sh = LatentShape(heads=H, dim=d, rot=r, rot_dims=rd, rank=rank, vdim=e, window=0, scale=0.5, eps=1e-6, gated=True)
+    cos, sin = rope_tables(512, rd, 1000.0, device=dev)
+    uk = torch.zeros(H, d, rank, dtype=torch.float64)
+    uk[:, 0, 0] = 1.0
+    uv = rnd(H, e, rank, seed=1)
+    ukv = torch.cat([uk.reshape(H * d, rank), uv.reshape(H * e, rank)]).to(dtype).to(dev)
+    for loud in (0, 1, 63, 64, 130):
+        q = torch.zeros(n, H, d + r, dtype=torch.float64)
+        q[:, :, 0] = 60.0
+        ckr = torch.zeros(n, rank + r, dtype=torch.float64)
+        ckr[:, 1:rank] = rnd(n, rank - 1, seed=loud + 2)
+        ckr[loud] = 0.0
+        ckr[loud, 0] = 3.0
+        gate = torch.full((n, H), 0.7, dtype=torch.float64)
+        pages = Pages(1, 5, 64, sh.row, [0], dev, dtype)
+        outs = []
+        for step in portions([n], sizes):
+            (_, k, p), = step
+            b = pages.batch(step)
+            t = lambda x: x[p:p + k].to(dtype).to(dev).contiguous()  # noqa: E731
+            out = torch.zeros(k, H * e, dtype=dtype, device=dev)
+            expand = dev.type == "cuda" and b.max_new > 1 and can_expand(sh, dtype)
+            plan = make_plan(b.seq_meta_host, k, 0, expand, dev)
+            latent_attention(t(q).view(k, -1), t(ckr), sh, torch.ones(rank, device=dev), ukv[:H * d].view(H, d, rank),
+                             ukv[H * d:].view(H, e, rank), ukv, cos, sin, pages.cache, b, plan, out, t(gate))
+            outs.append(out.double().cpu())
+        got = torch.cat(outs)
+        want = (uv[:, :, 0].to(dtype).double() * rank**0.5 * torch.sigmoid(torch.tensor(0.7))).reshape(-1)
+        for i in range(n):
+            same = float((got[i] - want).norm() / want.norm())
+            assert (same < 0.05) == (i >= loud), (loud, i, same)
+
+
 # -----------------------------------------------------------------------------------------------
 # norms, feed-forward, logits
 # -----------------------------------------------------------------------------------------------
@@ -481,6 +523,10 @@ CONFIGS = {
     "wide": dict(vocab=67, width=128, norm={"eps": 1e-6}, embedding={"scale": 5.0}, residual_mult=0.4,
                  logit_softcap=30.0, layers=[_lat(16, 64, 32, 128, 96, 64, _mlp(136)), _del(2, 1, 128, 128, 4),
                                              _att(8, 1, 128, 128, 64, _mlp(256))]),
+    # nothing that can be left out
+    "bare": dict(vocab=75, width=48, norm={"eps": 1e-5}, embedding={"scale": 3.0}, residual_mult=0.6, logit_softcap=None,
+                 layers=[dict(_att(4, 2, 16, 16, 8), mixer={"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 16, "scale": 0.3}),
+                         _lat(4, 16, 8, 24, 32, 24, sc=None), _del(3, 3, 16, 8, 2)]),
     # sizes the matrix-core and vector paths do not take
     "odd": dict(vocab=61, width=37, norm={"eps": 1e-6}, embedding={"scale": 5.0}, residual_mult=0.9, logit_softcap=11.0,
                 layers=[_del(3, 1, 5, 7, 3, _mlp(11)), _att(3, 1, 5, 7, 12), _lat(3, 5, 6, 9, 7, 7, _mlp(13)),
