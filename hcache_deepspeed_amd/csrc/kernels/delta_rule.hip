@@ -499,19 +499,28 @@ __device__ __forceinline__ void Split::all(const f32x4& a, const f32x4& b) {
 }
 
 // LDS image of a chunk, filled by direct loads (a wave instruction writes 64 lanes x 16 bytes in a row, so rows have no
-// padding; 16-byte pieces are swapped within a row instead, by the row number): k as 64 rows of 256 bytes, 64 columns of v
-// as 64 rows of 128 bytes, the chunk's blocks and factors as they are.
-constexpr int kTileV = 16384, kTileW = 24576, kTileBytes = kTileW + (4 * kWalkFloats + 4095) / 4096 * 4096;
+// padding; 16-byte pieces are swapped within a row instead, by the row number): k as 64 rows of 256 bytes, 64 / Z columns
+// of v as 64 rows, the chunk's blocks and factors as they are.
+constexpr int kTileV = 16384;
 static_assert((4 * kWalkFloats + 4095) / 4096 * 4096 <= 4 * kFixedFloats, "reads past the entry");
+template <int Z>
+struct ChunkTile {
+  static constexpr int kPieces = 8 / Z, kRowsV = 64 / kPieces;  // of v: pieces of a row, rows of a wave instruction
+  static constexpr int kW = kTileV + 64 * 16 * kPieces, kBytes = kW + (4 * kWalkFloats + 4095) / 4096 * 4096;
+  __device__ __forceinline__ static int swap(int row) { return Z == 1 ? row & 7 : (row >> 2) & 3; }
+  __device__ __forceinline__ static int off(int row, int piece) { return (row * kPieces + (piece ^ swap(row))) * 16; }
+};
 __device__ __forceinline__ int piece_of(int row) { return ((row & 3) << 2) | ((row >> 2) & 3); }
 __device__ __forceinline__ int row_off(int row, int piece) { return row * 256 + 16 * (piece ^ piece_of(row)); }
-__device__ __forceinline__ int v_off(int row, int piece) { return row * 128 + 16 * (piece ^ (row & 7)); }
 __device__ __forceinline__ void direct_load(const void* src, char* dst) {
   __builtin_amdgcn_global_load_lds((__attribute__((address_space(1))) const void*)src,
                                    (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
 }
 
-// FULL: dk == 32 KS and dv a multiple of 64 (no lane of a direct load is left out, which would split the schedule)
+// Z waves share 16 columns, each with its part of the key dims: they add up their parts of K S through LDS and then work out
+// the same U. (A wave's vector instructions do not run under its own matrix products, and there are fewer strips of columns
+// than SIMDs.) FULL: dk == 32 KS and dv a multiple of 64 (no lane of a direct load is left out, which would split the
+// schedule).
 template <int KS, bool FULL>
 __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<bf16> p, ChunkWs ws) {
   extern __shared__ __attribute__((aligned(1024))) char lds[];  // three chunks: this one, the next, the one on its way
@@ -520,37 +529,42 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   const DeltaDims& d = p.d;
   const int h = blockIdx.y, hk = h / (d.H / d.G), C = d.C(), dv = d.dv;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
-  const int c0 = blockIdx.x * 64, col = c0 + 16 * w + l15;
-  const bool active = FULL || c0 + 16 * w < dv, ok = FULL || col < dv;
+  constexpr int Z = KS > 1 ? 2 : 1, KZ = KS / Z, kStrips = 4 / Z;
+  using Tile = ChunkTile<Z>;
+  const int strip = w % kStrips, z = w / kStrips;
+  const int c0 = blockIdx.x * 16 * kStrips, col = c0 + 16 * strip + l15;
+  const bool active = FULL || c0 + 16 * strip < dv, ok = FULL || col < dv;
   float* st = p.state + (int64_t)s.slot * p.slot_stride + (int64_t)h * d.dk * dv;
-  f32x4 S[2 * KS];
+  f32x4 S[2 * KZ];
 #pragma unroll
-  for (int t = 0; t < 2 * KS; ++t)
+  for (int t = 0; t < 2 * KZ; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int row = state_row(t, g, r);
+      const int row = state_row(2 * KZ * z + t, g, r);
       S[t][r] = s.seen > 0 && ok && row < d.dk ? st[(int64_t)row * dv + col] : 0.f;
     }
   // Rows past the end repeat the last one: their factors are zero. Key columns past dk stay zero: a row of S there would
   // take part otherwise.
   const bf16* yk = p.y + (int64_t)s.q0 * C + d.k0() + hk * d.dk;
   const bf16* yv = p.y + (int64_t)s.q0 * C + d.v0() + h * dv + c0;
-  constexpr int kLoads = 6 + (4 * kWalkFloats + 4095) / 4096;  // direct loads a wave issues for a chunk
-  static_assert(kLoads == 9, "six between the products of K S, three later");
+  constexpr int kLoadsV = 2 / Z, kLoadsW = (4 * kWalkFloats + 4095) / 4096;
+  constexpr int kLoads = 4 + kLoadsV + kLoadsW;  // direct loads a wave issues for a chunk
+  static_assert(kLoadsW == 3, "the last three go out late");
   auto fetch_one = [&](int buffer, int chunk, int i) {
-    char* tile = lds + buffer * kTileBytes;
+    char* tile = lds + buffer * Tile::kBytes;
     const int last = s.n - 1 - chunk * kChunk;
     const int64_t at = (int64_t)chunk * kChunk * C;
     if (i < 4) {  // 4 rows of k an instruction
       const int n = 4 * w + i, row = 4 * n + (lane >> 4), e = 8 * ((lane & 15) ^ piece_of(row));
       if (FULL || e < d.dk) direct_load(yk + at + (uint32_t)(min(row, last) * C + e), tile + n * 1024);
-    } else if (i < 6) {  // 8 rows of v
-      const int n = 2 * w + i - 4, row = 8 * n + (lane >> 3), e = 8 * ((lane & 7) ^ (row & 7));
+    } else if (i < 4 + kLoadsV) {
+      const int n = kLoadsV * w + i - 4, row = n * Tile::kRowsV + lane / Tile::kPieces;
+      const int e = 8 * (lane % Tile::kPieces ^ Tile::swap(row));
       if (FULL || c0 + e < dv) direct_load(yv + at + (uint32_t)(min(row, last) * C + e), tile + kTileV + n * 1024);
     } else {
       const char* cw = reinterpret_cast<const char*>(ws.at(s, blockIdx.z, chunk, h, d.H)) + 16 * lane;
-      const int n = 4 * (i - 6) + w;  // (the last one reads into the blocks of A)
-      direct_load(cw + n * 1024, tile + kTileW + n * 1024);
+      const int n = 4 * (i - 4 - kLoadsV) + w;  // (the last one reads into the blocks of A)
+      direct_load(cw + n * 1024, tile + Tile::kW + n * 1024);
     }
   };
   auto fetch = [&](int buffer, int chunk) {
@@ -559,15 +573,17 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   };
   const int chunks = (s.n + kChunk - 1) / kChunk;
   if (!FULL && d.dk < 32 * KS) {
-    for (int i = threadIdx.x; i < 3 * kTileBytes / 16; i += 256) reinterpret_cast<u32x4*>(lds)[i] = u32x4{};
+    for (int i = threadIdx.x; i < 3 * Tile::kBytes / 16; i += 256) reinterpret_cast<u32x4*>(lds)[i] = u32x4{};
     __syncthreads();
   }
   // Offsets of this lane's reads in a tile. Row blocks and halves are 16-row steps, which leave the swap of the pieces as
   // it is; another k step or key block flips bits of the offset.
   const int q = l15 >> 2, pp = l15 & 3;
-  const int row_at = row_off(l15, g);           // ^ 64 ks; + 4096 b
-  const int col_at = row_off(4 * g + q, pp);    // ^ 64 (t >> 1); + 8 (t & 1), + 4096 per 16 tokens
-  const int v_at = kTileV + v_off(4 * g + q, 2 * w + (pp >> 1)) + 8 * (pp & 1);  // + 2048 b
+  const int row_at = row_off(l15, g) ^ (64 * KZ * z);         // ^ 64 ks; + 4096 b
+  const int col_at = row_off(4 * g + q, pp) ^ (64 * KZ * z);  // ^ 64 (t >> 1); + 8 (t & 1), + 4096 per 16 tokens
+  const int v_at = kTileV + Tile::off(4 * g + q, 2 * strip + (pp >> 1)) + 8 * (pp & 1);  // + kBlockV b
+  constexpr int kBlockV = 16 * 16 * Tile::kPieces;
+  char* parts = lds + 3 * Tile::kBytes + 16 * lane;           // [wave][4 tiles]
   fetch(0, 0);
   fetch(1, min(1, chunks - 1));
   Split sp[2];
@@ -575,11 +591,11 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   __syncthreads();
   int buffer = 0;
   for (int ch = 0; ch < chunks; ++ch) {
-    const char* tile = lds + buffer * kTileBytes;
+    const char* tile = lds + buffer * Tile::kBytes;
     const int free = buffer == 0 ? 2 : buffer - 1;      // was read in the step before
     const int next = min(ch + 2, chunks - 1);           // (the last one again: no branch)
     if (active) {
-      const char* cw = tile + kTileW;
+      const char* cw = tile + Tile::kW;
       auto block = [&](int b, int j) {
         return *reinterpret_cast<const f32x4*>(cw + block_at(b, j) * 1024 + l15 * 64 + 16 * g);
       };
@@ -590,9 +606,9 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
       // one another, and the splits of the next operands lie between them: the scheduling barriers keep it so.
       bf16x4 v[4];
       v[0] = read_tr4<0>(tile + v_at);
-      v[1] = read_tr4<2048>(tile + v_at);
-      v[2] = read_tr4<4096>(tile + v_at);
-      v[3] = read_tr4<6144>(tile + v_at);
+      v[1] = read_tr4<kBlockV>(tile + v_at);
+      v[2] = read_tr4<2 * kBlockV>(tile + v_at);
+      v[3] = read_tr4<3 * kBlockV>(tile + v_at);
       tr_wait(v[0], v[1]);
       tr_wait(v[2], v[3]);
       bf16x8 kf[2][4];
@@ -601,16 +617,16 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
         for (int b = 0; b < 4; ++b) kk[b] = *reinterpret_cast<const bf16x8*>(tile + (row_at ^ (64 * ks)) + 4096 * b);
       };
       rows(0, kf[0]);
-      float* keep_s = ws.at(s, blockIdx.z, ch, h, d.H) + kFixedFloats + (int64_t)(c0 / 16 + w) * strip_floats(KS) + 4 * lane;
+      float* keep_s = ws.at(s, blockIdx.z, ch, h, d.H) + kFixedFloats + (int64_t)(c0 / 16 + strip) * strip_floats(KS) + 4 * lane;
       f32x4 U[4];  // K S, then u
 #pragma unroll
       for (int b = 0; b < 4; ++b) U[b] = f32x4{0.f, 0.f, 0.f, 0.f};
       f32x4 M1[4][4], f0[4], f1[4], f3[4];  // [row block][column block]
       const float keep = *reinterpret_cast<const float*>(cw + kBlocks * 1024 + 16 * kChunk);
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
+      for (int ks = 0; ks < KZ; ++ks) {
         __builtin_amdgcn_sched_barrier(0);
-        if (ks + 1 < KS) {
+        if (ks + 1 < KZ) {
           rows(ks + 1, kf[(ks + 1) & 1]);
         } else {
 #pragma unroll
@@ -628,20 +644,32 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
         for (int i = 0; i < 12; ++i) {  // the smallest piece first
           __builtin_amdgcn_sched_barrier(0);
           U[i & 3] = mfma_bf16(kf[ks & 1][i & 3], sp[ks & 1].p(2 - i / 4), U[i & 3]);
-          if (ks + 1 < KS) split_step(sp[(ks + 1) & 1], i, S[2 * ks + 2], S[2 * ks + 3]);
+          if (ks + 1 < KZ) split_step(sp[(ks + 1) & 1], i, S[2 * ks + 2], S[2 * ks + 3]);
           // loads and stores are spread over the step: the wave would wait for a queue that is full
-          if ((12 * ks + i) % (2 * KS) == 2 * KS - 1) fetch_one(free, next, (12 * ks + i) / (2 * KS));  // 0 .. 5
+          constexpr int kEvery = 12 * KZ / (kLoads - 3);
+          const int n = 12 * ks + i;
+          if (n % kEvery == kEvery - 1 && n / kEvery < kLoads - 3) fetch_one(free, next, n / kEvery);
         }
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      if constexpr (Z == 2) {
+#pragma unroll
+        for (int b = 0; b < 4; ++b) *reinterpret_cast<f32x4*>(parts + (4 * w + b) * 1024) = U[b];
+        asm volatile("s_waitcnt lgkmcnt(0)" : : : "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" : : : "memory");
+#pragma unroll
+        for (int b = 0; b < 4; ++b) U[b] += *reinterpret_cast<const f32x4*>(parts + (4 * (w ^ 2) + b) * 1024);
       }
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
       for (int b = 0; b < 4; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) U[b][r] = f1[b][r] * (float)v[b][r] - f0[b][r] * U[b][r];
-      bf16x4 kt[2][2 * KS][2];  // transposed k: all key dims of 32 tokens
+      bf16x4 kt[2][2 * KZ][2];  // transposed k: all key dims of 32 tokens
       auto cols = [&](int hf) {
 #pragma unroll
-        for (int t = 0; t < 2 * KS; ++t) {
+        for (int t = 0; t < 2 * KZ; ++t) {
           const char* p0 = tile + (col_at ^ (64 * (t >> 1)));
           kt[hf][t][0] = hf == 0 ? (t & 1 ? read_tr4<8>(p0) : read_tr4<0>(p0))
                                  : (t & 1 ? read_tr4<8200>(p0) : read_tr4<8192>(p0));
@@ -668,36 +696,36 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
         for (int r = 0; r < 4; ++r) {
 #pragma unroll
           for (int b = j + 1; b < 4; ++b) U[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(M1[b][j][r], U[j][r], U[b], 0, 0, 0);
-          const int t = j == 0 ? r : (j == 1 ? 4 + r : 2 * KS);  // S goes out, then decays
-          if (t < 2 * KS) {
-            *reinterpret_cast<f32x4*>(keep_s + 256 * t) = S[t];
+          const int t = j == 0 ? r : (j == 1 ? 4 + r : 2 * KZ);  // S goes out, then decays
+          if (t < 2 * KZ) {
+            *reinterpret_cast<f32x4*>(keep_s + 256 * (2 * KZ * z + t)) = S[t];
             S[t] *= keep;
             __builtin_amdgcn_sched_barrier(0);
           }
         }
-        *reinterpret_cast<f32x4*>(keep_s + 256 * (2 * KS + j)) = U[j];
+        if (Z == 1 || j / 2 == z) *reinterpret_cast<f32x4*>(keep_s + 256 * (2 * KS + j)) = U[j];
         U[j] *= f3[j];
         if (j == 2) up[0].all(U[0], U[1]);
       }
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) tr_wait(kt[0][t][0], kt[0][t][1]);
+      for (int t = 0; t < 2 * KZ; ++t) tr_wait(kt[0][t][0], kt[0][t][1]);
       cols(1);
 #pragma unroll
-      for (int i = 0; i < 6 * KS; ++i) {
+      for (int i = 0; i < 6 * KZ; ++i) {
         __builtin_amdgcn_sched_barrier(0);
-        S[i % (2 * KS)] = mfma_bf16(key(0, i % (2 * KS)), up[0].p(2 - i / (2 * KS)), S[i % (2 * KS)]);
-        if (KS >= 2) split_step(up[1], i, U[2], U[3]);
-        if (i % (2 * KS) == 0) fetch_one(free, next, 6 + i / (2 * KS));
+        S[i % (2 * KZ)] = mfma_bf16(key(0, i % (2 * KZ)), up[0].p(2 - i / (2 * KZ)), S[i % (2 * KZ)]);
+        if (KZ >= 2) split_step(up[1], i, U[2], U[3]);
+        if (i % (2 * KZ) == 0) fetch_one(free, next, kLoads - 3 + i / (2 * KZ));
       }
-      if (KS < 2) up[1].all(U[2], U[3]);
+      if (KZ < 2) up[1].all(U[2], U[3]);
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) tr_wait(kt[1][t][0], kt[1][t][1]);
+      for (int t = 0; t < 2 * KZ; ++t) tr_wait(kt[1][t][0], kt[1][t][1]);
       // tiles 0 and 1 first: their sum is the first operand of the next chunk
 #pragma unroll
       for (int i = 0; i < 6; ++i) S[i & 1] = mfma_bf16(key(1, i & 1), up[1].p(2 - i / 2), S[i & 1]);
-      constexpr int R = 2 * KS - 2;  // the other tiles
+      constexpr int R = 2 * KZ - 2;  // the other tiles
 #pragma unroll
       for (int i = 0; i < 3 * R; ++i) {
         __builtin_amdgcn_sched_barrier(0);
@@ -709,9 +737,10 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
       for (int i = R > 0 ? 3 * R - 2 : 0; i < 12; ++i) split_step(sp[0], i, S[0], S[1]);
       __builtin_amdgcn_sched_barrier(0);
       // the next chunk's loads went out a step ago: all but this step's loads and stores have to be done
-      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(kLoads + 2 * KS + 4) : "memory");
+      asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(kLoads + 2 * KZ + 4 / Z) : "memory");
     } else {
       fetch(free, next);
+      if constexpr (Z == 2) __builtin_amdgcn_s_barrier();
       asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"(kLoads) : "memory");
     }
     __builtin_amdgcn_s_barrier();
@@ -720,10 +749,10 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_state_kernel(DeltaParams<b
   }
   if (ok)
 #pragma unroll
-    for (int t = 0; t < 2 * KS; ++t)
+    for (int t = 0; t < 2 * KZ; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int row = state_row(t, g, r);
+        const int row = state_row(2 * KZ * z + t, g, r);
         if (row < d.dk) st[(int64_t)row * dv + col] = S[t][r];
       }
 }
@@ -1094,12 +1123,12 @@ int launch_chunk_out(const DeltaParams<bf16>& p, const ChunkWs& ws, dim3 grid, h
 
 template <int KS, bool FULL>
 int launch_chunk_state(const DeltaParams<bf16>& p, const ChunkWs& ws, int n_seqs, hipStream_t st) {
-  constexpr int lds = 3 * kTileBytes;
+  constexpr int Z = KS > 1 ? 2 : 1, lds = 3 * ChunkTile<Z>::kBytes + (Z > 1 ? 16384 : 0), cols = 64 / Z;
   static_assert(lds <= 160 * 1024, "LDS");
   static const hipError_t attr = hipFuncSetAttribute((const void*)delta_chunk_state_kernel<KS, FULL>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   if (attr != hipSuccess) return attr;
-  hipLaunchKernelGGL((delta_chunk_state_kernel<KS, FULL>), dim3((p.d.dv + 63) / 64, p.d.H, n_seqs), dim3(256), lds, st, p,
+  hipLaunchKernelGGL((delta_chunk_state_kernel<KS, FULL>), dim3((p.d.dv + cols - 1) / cols, p.d.H, n_seqs), dim3(256), lds, st, p,
                      ws);
   return hipGetLastError();
 }
