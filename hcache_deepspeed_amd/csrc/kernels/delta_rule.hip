@@ -6,7 +6,8 @@
 //   S      = g S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q
 //   out    = o / sqrt(mean(o^2) + eps) * w * silu(gate)
 //
-// One projection row holds, column block by column block, q [G dk] | k [G dk] | v [H dv] | gate [H dv] | b [H] | a [H].
+// One projection row holds, column block by column block, q [G dk] | k [G dk] | v [H dv] | gate [H dv], another (or the same
+// one further on) b [H] | a [H].
 // A sequence's slot holds S of all heads and then the convolution's last inputs as a ring: the input of position p is
 // entry p % taps, [taps, C] with C = 2 G dk + H dv. (With taps - 1 of them in use, a step of one token reads other entries
 // than it writes, so the workgroups of heads that share a key head need no order among them.) A sequence whose `seen` is
@@ -46,7 +47,7 @@ struct DeltaDims {
   __device__ __host__ __forceinline__ int k0() const { return G * dk; }
   __device__ __host__ __forceinline__ int v0() const { return 2 * G * dk; }
   __device__ __host__ __forceinline__ int C() const { return 2 * G * dk + H * dv; }      // convolved channels
-  __device__ __host__ __forceinline__ int b0() const { return 2 * G * dk + 2 * H * dv; }
+  __device__ __host__ __forceinline__ int width() const { return 2 * G * dk + 2 * H * dv; }
   __device__ __host__ __forceinline__ int64_t states() const { return (int64_t)H * dk * dv; }
 };
 
@@ -54,6 +55,8 @@ template <typename T>
 struct DeltaParams {
   DeltaDims d;
   const T* proj;        // [tokens, d.ld]
+  const T* ba;          // [tokens, ldba]
+  int64_t ldba;
   const float* cw;      // [taps, C], the last row is the current token's
   const float* a_log;   // [H]
   const float* dt;      // [H]
@@ -95,7 +98,7 @@ template <typename T>
 __device__ __forceinline__ void write_gates(const DeltaParams<T>& p, const Seq& s, int t0, int rows) {
   for (int i = threadIdx.x; i < rows * p.d.H; i += blockDim.x) {
     const int t = s.q0 + t0 + i / p.d.H, h = i % p.d.H;
-    const T* row = p.proj + (int64_t)t * p.d.ld + p.d.b0();
+    const T* row = p.ba + (int64_t)t * p.ldba;
     float* gb = p.gb + 2 * ((int64_t)t * p.d.H + h);
     gb[0] = -expf(p.a_log[h]) * softplus_f(to_f(row[p.d.H + h]) + p.dt[h]);
     gb[1] = sigmoid_f(to_f(row[h]));
@@ -963,7 +966,8 @@ __global__ __launch_bounds__(NT, NT < 1024 ? 1 : (RPT <= 4 ? 8 : 4)) void delta_
       else if (k < d.taps && s.seen >= k) hist[k] = ring[(int64_t)(now >= k ? now - k : now - k + d.taps) * C + c_first];
     }
   }
-  const float xb = to_f(row[d.b0() + h]), xa = to_f(row[d.b0() + d.H + h]), al = p.a_log[h], dt = p.dt[h];
+  const T* ba = p.ba + (int64_t)s.q0 * p.ldba + h;
+  const float xb = to_f(ba[0]), xa = to_f(ba[d.H]), al = p.a_log[h], dt = p.dt[h];
   f32x4 S[RPT];
 #pragma unroll
   for (int r = 0; r < RPT; ++r) {
@@ -1191,7 +1195,7 @@ int launch_step(const DeltaParams<T>& p, int n_seqs, hipStream_t st) {
 
 bool dims_ok(const DeltaDims& d) {
   return d.H >= 1 && d.G >= 1 && d.H % d.G == 0 && d.dk >= 1 && d.dk <= 512 && d.dv >= 1 && d.taps >= 1 &&
-         d.taps <= 256 && d.H <= 65535 && d.ld >= (int64_t)d.b0() + 2 * d.H;
+         d.taps <= 256 && d.H <= 65535 && d.ld >= (int64_t)d.width();
 }
 
 }  // namespace
@@ -1203,17 +1207,17 @@ HDS_EXPORT int hds_delta_step_ok(int dk, int dv) {
 }
 
 // the sequences' one new token each
-HDS_EXPORT int hds_delta_step(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
+HDS_EXPORT int hds_delta_step(int dtype, const void* proj, int64_t ld, const void* ba, int64_t ldba, const float* cw, const float* a_log,
                               const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
                               const int* seq_meta, const int* seqs, void* out, int64_t ldo, int n_seqs, int H, int G,
                               int dk, int dv, int taps, float eps, hipStream_t st) {
   if (n_seqs <= 0) return 0;
   const DeltaDims d{H, G, dk, dv, taps, ld};
-  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || ldo < (int64_t)H * dv ||
+  if (!dims_ok(d) || !ba || ldba < 2 * H || n_seqs > 65535 || !state || !slots || ldo < (int64_t)H * dv ||
       slot_stride < d.states() + (int64_t)taps * d.C())
     return hipErrorInvalidValue;
 #define HDS_DX(TT)                                                                                                 \
-  return launch_step(DeltaParams<TT>{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, \
+  return launch_step(DeltaParams<TT>{d, (const TT*)proj, (const TT*)ba, ldba, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, \
                                      seqs, nullptr, nullptr, nullptr, nullptr, (TT*)out, ldo, 0, eps}, n_seqs, st)
   if (dtype == kBF16) HDS_DX(bf16);
   if (dtype == kF32) HDS_DX(float);
@@ -1231,19 +1235,19 @@ HDS_EXPORT int hds_delta_chunk_tokens() { return kChunk; }
 // Portions of at most max_new tokens. y [tokens, C], rn [tokens, 2 G] and gb [tokens, H, 2] are scratch memory with a row
 // for every token of the step. chunks: scratch memory of the scan by chunks (the sequences ascend in the step's rows; proj
 // and out rows 16-byte aligned); null: token by token, with o [tokens, H, dv] as scratch memory.
-HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const float* cw, const float* a_log,
+HDS_EXPORT int hds_delta_scan(int dtype, const void* proj, int64_t ld, const void* ba, int64_t ldba, const float* cw, const float* a_log,
                               const float* dt, const float* norm, float* state, int64_t slot_stride, const int* slots,
                               const int* seq_meta, const int* seqs, void* y, float* rn, float* gb, float* o, float* chunks,
                               void* out, int64_t ldo, int n_seqs, int max_new, int H, int G, int dk, int dv, int taps, float eps,
                               hipStream_t st) {
   if (n_seqs <= 0 || max_new <= 0) return 0;
   const DeltaDims d{H, G, dk, dv, taps, ld};
-  if (!dims_ok(d) || n_seqs > 65535 || !state || !slots || !y || !rn || !gb || ldo < (int64_t)H * dv ||
+  if (!dims_ok(d) || !ba || ldba < 2 * H || n_seqs > 65535 || !state || !slots || !y || !rn || !gb || ldo < (int64_t)H * dv ||
       slot_stride < d.states() + (int64_t)taps * d.C())
     return hipErrorInvalidValue;
 #define HDS_DX(TT)                                                                                                   \
   {                                                                                                                  \
-    const DeltaParams<TT> p{d, (const TT*)proj, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, seqs,     \
+    const DeltaParams<TT> p{d, (const TT*)proj, (const TT*)ba, ldba, cw, a_log, dt, norm, state, slot_stride, slots, seq_meta, seqs,     \
                             (TT*)y, rn, gb, o, (TT*)out, ldo, 0, eps};                                               \
     if (int e = launch_conv(p, n_seqs, max_new, st)) return e;                                                       \
     return scan(p);                                                                                                  \

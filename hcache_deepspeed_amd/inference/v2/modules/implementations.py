@@ -331,6 +331,14 @@ def _is_plain(lin):
     return isinstance(lin, BlasFPLinear)
 
 
+SPLIT_ROWS = 1024  # tokens from which on a projection may run as several products
+
+
+def _tile_rounds(rows, cols):
+    """How often the library's 256 x 256 tiles of a product go round the 256 CUs."""
+    return -(-(-(-rows // 256) * -(-cols // 256)) // 256)
+
+
 @DSMixerRegistry.register_module
 class MinGRUMixer(DSMixerBase):
     """Gated linear recurrence whose gates read the current token only (ops/gated_scan.py)."""
@@ -503,13 +511,19 @@ class HeadAttentionMixer(DSMixerBase):
 
     def forward(self, x, w, lins, out, batch, cache, state, offset):
         sh = self.shape
-        qkv = lins["in.w"](x, w["in.w"])
+        lin, in_w, n = lins["in.w"], w["in.w"], sh.qkv_width
+        gate = None
+        if sh.gate_width > 1 and x.shape[0] >= SPLIT_ROWS and _is_plain(lin) and n % 8 == 0:
+            # gates as wide as the heads: of two narrower products both are closer to the library's best
+            qkv, gate = lin(x, in_w[:n]), lin(x, in_w[n:sh.width])
+        else:
+            qkv = lin(x, in_w)
         own = qkv[:, sh.qkv_width - sh.kv_heads * sh.vdim:sh.qkv_width]
         if self.value_mix == "source":
             batch.carry["values"] = own
         first = batch.carry["values"] if self.value_mix == "mix" else None
         return head_attention(qkv, sh, w["q.norm"], w["k.norm"], w["sink"], cache, batch, self._plan(batch), out, first,
-                              w["vmix"])
+                              w["vmix"], gate)
 
 
 @DSMixerRegistry.register_module
@@ -553,8 +567,15 @@ class DeltaMixer(DSMixerBase):
         return plan
 
     def forward(self, x, w, lins, out, batch, cache, state, offset):
-        return delta_rule(lins["in.w"](x, w["in.w"]), self.shape, w["conv.w"], w["A_log"], w["dt_bias"], w["norm"],
-                          state, offset, batch, self._plan(batch), out)
+        sh, lin, in_w, T = self.shape, lins["in.w"], w["in.w"], x.shape[0]
+        n, ba = sh.main_width, None
+        if T >= SPLIT_ROWS and _is_plain(lin) and n % 8 == 0 and _tile_rounds(T, n) < _tile_rounds(T, self.in_width):
+            # the few columns of b and a would cost another round of tiles
+            proj, ba = lin(x, in_w[:n]), lin(x, in_w[n:])
+        else:
+            proj = lin(x, in_w)
+        return delta_rule(proj, sh, w["conv.w"], w["A_log"], w["dt_bias"], w["norm"], state, offset, batch,
+                          self._plan(batch), out, ba)
 
 
 @DSOutputNormRegistry.register_module

@@ -31,9 +31,13 @@ class DeltaShape:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
     @property
+    def main_width(self):
+        """Columns of the projection without b and a: q | k | v | output gate."""
+        return self.channels + self.heads * self.vdim
+
+    @property
     def width(self):
-        """Columns of the projection: q | k | v | output gate | b | a."""
-        return self.channels + self.heads * self.vdim + 2 * self.heads
+        return self.main_width + 2 * self.heads
 
     @property
     def state_floats(self):
@@ -77,19 +81,24 @@ def _chunk_floats(sh, dtype, n_tok, n_seqs):
     return (n_tok // lib.hds_delta_chunk_tokens() + n_seqs) * sh.heads * per
 
 
-def delta_rule(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch, plan, out):
-    """proj: [T, >= shape.width]; conv_w: [taps, channels], the last row is the current token's; a_log, dt_bias: [heads];
+def delta_rule(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch, plan, out, ba=None):
+    """proj: [T, >= shape.width], q | k | v | output gate | b | a; or with ``ba`` [T, >= 2 heads] (b | a) without these
+    columns. conv_w: [taps, channels], the last row is the current token's; a_log, dt_bias: [heads];
     norm_w: [vdim], all float32. ``state[slot, offset:offset + shape.state_floats]`` is read and advanced; ``out``
     [T, heads * vdim] (unit column stride)."""
+    if ba is None:
+        assert proj.shape[1] >= shape.width
+        ba = proj[:, shape.main_width:]
     if not native.use_native(proj):
-        return _delta_rule_cpu(proj, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch, out)
+        return _delta_rule_cpu(proj, ba, shape, conv_w, a_log, dt_bias, norm_w, state, offset, batch, out)
     sh, lib, dt, st = shape, native.kernels(), native.dt(proj), native.stream()
     T, dev = proj.shape[0], proj.device
-    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.dtype == proj.dtype and proj.shape[1] >= sh.width
+    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.dtype == proj.dtype and proj.shape[1] >= sh.main_width
+    assert ba.dtype == proj.dtype and ba.shape[0] == T and ba.shape[1] >= 2 * sh.heads and ba.stride(1) == 1
     assert out.shape == (T, sh.heads * sh.vdim) and conv_w.shape == (sh.taps, sh.channels) and conv_w.is_contiguous()
     assert a_log.numel() == dt_bias.numel() == sh.heads and norm_w.numel() == sh.vdim
     assert offset + sh.state_floats <= state.shape[1]
-    head = (dt, proj.data_ptr(), proj.stride(0), conv_w.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),
+    head = (dt, proj.data_ptr(), proj.stride(0), ba.data_ptr(), ba.stride(0), conv_w.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),
             norm_w.data_ptr(), state.data_ptr() + 4 * offset, state.stride(0), batch.slots.data_ptr(),
             batch.seq_meta.data_ptr())
     dims = (sh.heads, sh.kv_heads, sh.dim, sh.vdim, sh.taps, float(sh.eps), st)
@@ -114,9 +123,10 @@ def _silu(x):
     return x * torch.sigmoid(x)
 
 
-def _delta_rule_cpu(proj, sh, conv_w, a_log, dt_bias, norm_w, state, offset, batch, out):
+def _delta_rule_cpu(proj, ba, sh, conv_w, a_log, dt_bias, norm_w, state, offset, batch, out):
     H, G, d, e, C, taps = sh.heads, sh.kv_heads, sh.dim, sh.vdim, sh.channels, sh.taps
-    x, gate, b, a = proj[:, :sh.width].float().split([C, H * e, H, H], 1)
+    x, gate = proj[:, :sh.main_width].float().split([C, H * e], 1)
+    b, a = ba[:, :2 * H].float().split(H, 1)
     decay = torch.exp(-torch.exp(a_log) * torch.nn.functional.softplus(a + dt_bias, threshold=40.0))
     beta = torch.sigmoid(b)
     n_state = H * d * e

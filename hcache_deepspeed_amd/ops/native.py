@@ -45,10 +45,10 @@ _KERNEL_SIGS = {
     "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
     "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "pp" + "iii" + "s",
     "hds_delta_step_ok": "ii",
-    "hds_delta_step": "i" + "pl" + "pppp" + "pl" + "ppp" + "pl" + "iiiiii" + "f" + "s",
+    "hds_delta_step": "i" + "plpl" + "pppp" + "pl" + "ppp" + "pl" + "iiiiii" + "f" + "s",
     "hds_delta_chunk_floats": "iii",
     "hds_delta_chunk_tokens": "",
-    "hds_delta_scan": "i" + "pl" + "pppp" + "pl" + "ppp" + "ppppp" + "pl" + "i" * 7 + "f" + "s",
+    "hds_delta_scan": "i" + "plpl" + "pppp" + "pl" + "ppp" + "ppppp" + "pl" + "i" * 7 + "f" + "s",
     "hds_gemv_recur_bf16": "ppppp" + "pl" + "pp" + "iii" + "ll" + "s",
     "hds_latent_prep": "i" + "plpl" + "ppp" + "p" * 9 + "i" * 10 + "f" + "s",
     "hds_latent_decode_mfma_ok": "ii",

@@ -259,19 +259,22 @@ def head_blocks_ok(shape, dtype):
     return dtype == torch.bfloat16 and bool(native.kernels().hds_paged_attn_supported(shape.dim, shape.vdim))
 
 
-def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, values=None, mix=None):
-    """qkv: [T, >= shape.width] projection, row by row q heads | k heads | v heads | gates (consumed). q_norm / k_norm:
+def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, values=None, mix=None, gate=None):
+    """qkv: [T, >= shape.width] projection, row by row q heads | k heads | v heads | gates (consumed); or with ``gate``
+    [T, heads * gate_width] without the gates. q_norm / k_norm:
     [dim] float32 or None; sink: [heads] float32 or None; cache: [blocks, block_size, shape.row]. Appends the step's keys
     and values to ``cache`` and writes the gated heads into ``out`` [T, heads * vdim] (unit column stride). ``values``:
     [T, kv_heads * vdim] values of another layer, of which the share ``mix`` ([1] float32) goes into this layer's."""
     sh, T = shape, qkv.shape[0]
+    if sh.gated and gate is None:
+        gate = qkv[:, sh.qkv_width:sh.width]
     if not native.use_native(qkv):
-        return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values, mix)
+        return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values, mix, gate)
     lib, st, dt = native.kernels(), native.stream(), native.dt(qkv)
     bs, tab = cache.shape[1], batch.block_tables
     mb = tab.shape[1]
     assert qkv.stride(1) == 1 and out.stride(1) == 1 and cache.dtype == qkv.dtype == out.dtype
-    assert cache.shape[2] == sh.row and qkv.shape[1] >= sh.width and out.shape[1] == sh.heads * sh.vdim
+    assert cache.shape[2] == sh.row and qkv.shape[1] >= sh.qkv_width and out.shape[1] == sh.heads * sh.vdim
     native.check(
         lib.hds_head_norm_scatter(dt, qkv.data_ptr(), qkv.stride(0), native.ptr(q_norm), native.ptr(k_norm),
                                   cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(),
@@ -279,10 +282,12 @@ def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, va
                                   native.ptr(values), 0 if values is None else values.stride(0),
                                   None if values is None else mix.data_ptr(), st),
         "head_norm_scatter")
-    gate = qkv.data_ptr() + qkv.element_size() * sh.qkv_width if sh.gated else None
+    assert not sh.gated or (gate.shape == (T, sh.heads * sh.gate_width) and gate.stride(1) == 1 and gate.dtype == qkv.dtype)
+    gp, ldg = (gate.data_ptr(), gate.stride(0)) if sh.gated else (None, 0)
     assert values is None or (values.shape == (T, sh.kv_heads * sh.vdim) and values.dtype == qkv.dtype)
     fast = head_blocks_ok(sh, qkv.dtype) and qkv.stride(0) % 8 == 0 and out.stride(0) % 8 == 0 and \
-        qkv.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0
+        qkv.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0 and (gp is None or sh.gate_width == 1 or
+                                                                   (ldg % 4 == 0 and gp % 8 == 0))
     assert fast or not plan.n_atoms
     if plan.n_dec:
         n = plan.n_dec
@@ -297,19 +302,19 @@ def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, va
                                  out.stride(0), native.ptr(part_o), native.ptr(part_ml), None, native.ptr(plan.toks),
                                  batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(), mb, bs, n,
                                  sh.heads, sh.kv_heads, sh.dim, sh.vdim, splits, float(sh.scale), sh.window,
-                                 sh.chunk, float(sh.softcap), native.ptr(sink), gate, qkv.stride(0), sh.gate_width,
+                                 sh.chunk, float(sh.softcap), native.ptr(sink), gp, ldg, sh.gate_width,
                                  None, st), "paged_decode")
     if plan.n_atoms:
         native.check(
             lib.hds_paged_attn(qkv.data_ptr(), qkv.stride(0), cache.data_ptr(), out.data_ptr(), out.stride(0),
                                plan.atoms.data_ptr(), plan.n_atoms, batch.seq_meta.data_ptr(), tab.data_ptr(), mb, bs,
                                sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, sh.chunk,
-                               float(sh.softcap), native.ptr(sink), gate, qkv.stride(0), sh.gate_width, st),
+                               float(sh.softcap), native.ptr(sink), gp, ldg, sh.gate_width, st),
             "paged_attn")
     return out
 
 
-def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values=None, mix=None):
+def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values, mix, gate):
     T, H, G = qkv.shape[0], sh.heads, sh.kv_heads
 
     def normed(v, w):
@@ -321,9 +326,7 @@ def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values
     if values is not None:
         v = (1 - mix) * v + mix * values.float()
     copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
-    gate = torch.ones(T, H, 1)
-    if sh.gated:
-        gate = torch.sigmoid(qkv[:, sh.qkv_width:sh.width].float()).reshape(T, H, sh.gate_width)
+    gate = torch.sigmoid(gate.float()).reshape(T, H, sh.gate_width) if sh.gated else torch.ones(T, H, 1)
     bs = cache.shape[1]
     for s, (q0, n, seen) in enumerate(batch.seq_meta_host):
         if n == 0:

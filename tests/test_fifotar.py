@@ -255,6 +255,20 @@ def test_attention(run, name, sizes, mixed):
         close(g, _oracle_heads(sh, m, x, vals[i] if mixed else None, mix), dtype, f32=4e-5, bf16=2e-2)
 
 
+def test_projection_in_two_products(run, monkeypatch):
+    """Long steps run gates, or b and a, as a product of their own."""
+    from hcache_deepspeed_amd.inference.v2.modules import implementations
+    dev, dtype = run
+    toks = tokens_of("mixed", 150, 4)
+    calls = []
+    monkeypatch.setattr(implementations, "SPLIT_ROWS", 20)
+    monkeypatch.setattr(implementations, "_tile_rounds", lambda rows, cols: calls.append(cols) or len(calls))
+    eng = engine("mixed", run, blocks=12)
+    got, = feed(eng, [toks], [[(0, 100, 0)], [(0, 19, 100)], [(0, 31, 119)]])
+    check_logits(got, oracle_logits("mixed", toks), dtype)
+    assert len(calls) == 2 * 2 * 2
+
+
 @pytest.mark.parametrize("name", ["exact-64", "exact-128", "uneven", "12-per-key"])
 @pytest.mark.parametrize("sizes", [[1000], [90]])
 def test_attention_long_prompts(run, name, sizes):
