@@ -29,6 +29,8 @@ OPS = {
     "kv_rotary_scatter (HCache restore)": ("kernels", "hds_kv_rope_scatter"),
     "latent_attention (ragged)": ("kernels", "hds_latent_decode"),
     "gated_scan (minGRU)": ("kernels", "hds_gated_scan"),
+    "delta_rule (gated, step / by chunks)": ("kernels", "hds_delta_scan"),
+    "sandwich_norm (norms around a sublayer)": ("kernels", "hds_sandwich_norm"),
     "input_norm (norm + input convolution)": ("kernels", "hds_input_norm"),
     "residual_norm (norm on a sublayer's output)": ("kernels", "hds_residual_norm"),
     "routed experts (router, grouped / skinny products)": ("kernels", "hds_experts_skinny"),
