@@ -3,7 +3,7 @@
 //   x      = silu(conv(x))                        for the channels of q, k and v: causal, depthwise, `taps` wide
 //   q, k   = q / |q| * dk^(-1/2),  k / |k|        |x| = sqrt(sum(x^2) + 1e-6); query / key head h / (H / G)
 //   beta   = sigmoid(b),  g = exp(-exp(A) * softplus(a + dt))
-//   S      = g S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q
+//   u      = beta (v - g S^T k),  S' = g S + k u^T,  o = S'^T q
 //   out    = o / sqrt(mean(o^2) + eps) * w * silu(gate)
 //
 // One projection row holds, column block by column block, q [G dk] | k [G dk] | v [H dv] | gate [H dv], another (or the same

@@ -30,7 +30,7 @@ def softcap(z, cap):
 # gated delta rule
 # -----------------------------------------------------------------------------------------------
 def short_conv(x, w):
-    """x [T, C]; w [C, taps], the last column is the current token's."""
+    """x [T, C]; w [C, taps], the newest input in the last column."""
     T, taps = x.shape[0], w.shape[1]
     y = torch.zeros_like(x)
     for t in range(T):
