@@ -5,6 +5,8 @@
 // GeLU of csrc/transformer/gelu_kernels.cu (K6). The reference has no training SwiGLU; the
 // Llama/Mixtral training path here needs fwd+bwd.
 //
+// Also act(x) times a table's row per token (act_gather).
+//
 // Layout: gate/up are the two halves of ONE fused GEMM output row [T, 2I] (gate first), so
 // the MLP runs one GEMM for W1|W3 and this kernel reads both halves with 16-byte loads.
 // Backward writes dgate|dup into the same [T, 2I] layout, which is what the fused GEMM's
@@ -335,6 +337,25 @@ __global__ __launch_bounds__(256) void glu_fwd_t(const bf16* __restrict__ gu, bf
 }
 
 // y = act(x + bias)   (bias optional, [C])
+// y[r] = act(x[r]) * table[ids[r]]
+template <typename T, int A, int V>
+__global__ __launch_bounds__(256) void act_gather(const T* __restrict__ x, int64_t ldx, const T* __restrict__ table,
+                                                  int64_t ldt, const int64_t* __restrict__ ids, T* __restrict__ y,
+                                                  int64_t ldy, int64_t rows, int C, int vocab) {
+  const int vpr = C / V;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < rows * vpr; i += (int64_t)gridDim.x * 256) {
+    const int64_t r = i / vpr;
+    const int c = (int)(i - r * vpr) * V;
+    const int64_t id = min(max(ids[r], (int64_t)0), (int64_t)vocab - 1);
+    float v[V], e[V];
+    VecN<T, V>::load(x + r * ldx + c, v);
+    VecN<T, V>::load(table + id * ldt + c, e);
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = act_f<A>(v[j]) * e[j];
+    VecN<T, V>::store(y + r * ldy + c, v);
+  }
+}
+
 template <typename T, int A>
 __global__ __launch_bounds__(256) void bias_act_fwd(const T* __restrict__ x, const T* __restrict__ bias,
                                                     T* __restrict__ y, int64_t rows, int C) {
@@ -419,6 +440,40 @@ HDS_EXPORT int hds_glu_fwd(int dtype, int act, const void* gu, void* y, int64_t 
     dim3 grid(stream_grid(rows * (I / 8), 256)), block(256);
     DT_SWITCH(dtype, ACT_SWITCH(act, glu_fwd, T, grid, block, 0, st, (const T*)gu, (T*)y, rows, I));
   }
+  return hipGetLastError();
+}
+
+// y[r] = act(x[r]) * table[ids[r]], rows [rows, C] with row strides ldx, ldt, ldy; vocab: rows of the table
+HDS_EXPORT int hds_act_gather(int dtype, int act, const void* x, int64_t ldx, const void* table, int64_t ldt,
+                              const int64_t* ids, void* y, int64_t ldy, int64_t rows, int C, int vocab, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (C < 1 || ldx < C || ldt < C || ldy < C || vocab < 1) return hipErrorInvalidValue;
+  const bool v8 = C % 8 == 0 && ldx % 8 == 0 && ldt % 8 == 0 && ldy % 8 == 0 && (uintptr_t)x % 16 == 0 &&
+                  (uintptr_t)table % 16 == 0 && (uintptr_t)y % 16 == 0;
+  const dim3 grid(stream_grid(rows * (v8 ? C / 8 : C), 256)), block(256);
+#define HDS_AG(TT, AA)                                                                                               \
+  case AA:                                                                                                           \
+    if (v8)                                                                                                          \
+      hipLaunchKernelGGL((act_gather<TT, AA, 8>), grid, block, 0, st, (const TT*)x, ldx, (const TT*)table, ldt, ids, \
+                         (TT*)y, ldy, rows, C, vocab);                                                               \
+    else                                                                                                             \
+      hipLaunchKernelGGL((act_gather<TT, AA, 1>), grid, block, 0, st, (const TT*)x, ldx, (const TT*)table, ldt, ids, \
+                         (TT*)y, ldy, rows, C, vocab);                                                               \
+    break;
+#define HDS_AGA(TT)                                                                                                \
+  switch (act) {                                                                                                   \
+    HDS_AG(TT, kSilu) HDS_AG(TT, kGeluTanh) HDS_AG(TT, kRelu) HDS_AG(TT, kGeluErf) HDS_AG(TT, kIdentity)          \
+    default: return hipErrorInvalidValue;                                                                          \
+  }
+  if (dtype == kBF16) {
+    HDS_AGA(bf16)
+  } else if (dtype == kF32) {
+    HDS_AGA(float)
+  } else {
+    return hipErrorInvalidValue;
+  }
+#undef HDS_AGA
+#undef HDS_AG
   return hipGetLastError();
 }
 

@@ -1,10 +1,11 @@
 // Routed expert layers of the serving engine: router, choice of the experts, and the expert products of small steps.
 //
 //   z = W_router h                       (32-bit accumulation and result)
-//   s = softmax(z) over the experts and the identity experts behind them
+//   s = softmax(z) over the experts and the identity experts behind them, or sigmoid(z)
 //   c = s + correction                   (decides, does not weigh)
 //   groups of neighbours are ranked by their largest c, only the best `keep` of them take part
-//   the `top` largest c are chosen; weight = s * scale
+//   the `top` largest c are chosen; weight = s * scale, of an expert's output, or of its input: then the product's rows are
+//   multiplied with it in front of the activation
 //
 // Steps of few tokens run the experts straight from the choices (experts_skinny_kernel: every chosen expert's weights
 // are streamed once, whatever the number of tokens that chose it, the gated activation included). Longer steps sort
@@ -100,7 +101,7 @@ __device__ __forceinline__ float of_lane(float v, int l) {
 // One wave per token; lane l holds entries l + 64 q of the N = experts + identities. groups <= 64. Up to 128 entries every
 // lane ranks its own against all others (readlane, no dependent steps); more are picked one by one.
 template <int Q>
-__global__ __launch_bounds__(256) void router_select_kernel(const float* __restrict__ z, int64_t ldz,
+__global__ __launch_bounds__(256) void router_select_kernel(const float* __restrict__ z, int64_t ldz, int sigmoid,
                                                             const float* __restrict__ correction,
                                                             int* __restrict__ expert, float* __restrict__ weight, int T,
                                                             int N, int groups, int keep, int top, float scale) {
@@ -114,19 +115,28 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     s[q] = e < N ? z[(int64_t)t * ldz + e] : -INFINITY;
     m = fmaxf(m, s[q]);
   }
-  m = wave_max(m);
-  float sum = 0.f;
+  float inv = 1.f;
+  if (sigmoid) {
 #pragma unroll
-  for (int q = 0; q < Q; ++q) {
-    s[q] = lane + 64 * q < N ? expf(s[q] - m) : 0.f;
-    sum += s[q];
+    for (int q = 0; q < Q; ++q) {
+      const float e = expf(-fabsf(s[q])), r = 1.f / (1.f + e);
+      s[q] = s[q] >= 0.f ? r : e * r;
+    }
+  } else {
+    m = wave_max(m);
+    float sum = 0.f;
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+      s[q] = lane + 64 * q < N ? expf(s[q] - m) : 0.f;
+      sum += s[q];
+    }
+    inv = 1.f / wave_sum(sum);
   }
-  const float inv = 1.f / wave_sum(sum);
 #pragma unroll
   for (int q = 0; q < Q; ++q) {
     const int e = lane + 64 * q;
     s[q] *= inv;
-    c[q] = e < N ? s[q] + correction[e] : -INFINITY;
+    c[q] = e < N ? (correction != nullptr ? s[q] + correction[e] : s[q]) : -INFINITY;
     if (c[q] != c[q]) c[q] = -3.0e38f;  // rank a NaN last: every choice stays a valid index
   }
   if constexpr (Q <= 2) {
@@ -240,10 +250,11 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
 constexpr int kMaxExperts = 1024;
 
 // One workgroup. offs[E + 1]: rows of every expert; row[a] of choice a = token * k + j (identity choices: -1);
-// token[row]; the tile list (expert, first row inside the expert) for products of tm rows.
+// token[row] and, if asked, the choices' weights in the same order; the tile list (expert, first row inside the expert) for products of tm rows.
 __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict__ expert, int n, int k, int E,
                                                            int* __restrict__ offs, int* __restrict__ row,
-                                                           int* __restrict__ token, int tm, int* __restrict__ tile_e,
+                                                           int* __restrict__ token, const float* __restrict__ weight,
+                                                           float* __restrict__ row_weight, int tm, int* __restrict__ tile_e,
                                                            int* __restrict__ tile_m, int* __restrict__ n_tiles,
                                                            int max_tiles) {
   __shared__ int count[kMaxExperts], start[kMaxExperts], tiles[kMaxExperts], wsum[2][16];
@@ -314,6 +325,7 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
       if (a >= n || r[u] < 0) continue;
       row[a] = start[e[u]] + r[u];
       token[start[e[u]] + r[u]] = a / k;
+      if (row_weight != nullptr) row_weight[start[e[u]] + r[u]] = weight[a];
     }
   }
 }
@@ -339,7 +351,16 @@ struct SkinnyParams {
   bf16* outs;          // [n_sh, ldos]
   int64_t ldos;
   int n_sh, Ns, Ks;
+  int act;             // GLU: 0 silu, 5 the clamped unit
+  float limit;
+  const float* weight; // [n] or null: GLU multiplies the routed rows' products with it
 };
+
+__device__ __forceinline__ float gated_unit(float g, float u, int act, float limit) {
+  if (act == 0) return g / (1.f + __expf(-g)) * u;
+  g = fminf(g, limit);
+  return g / (1.f + __expf(-1.702f * g)) * (fminf(fmaxf(u, -limit), limit) + 1.f);
+}
 
 constexpr int kSkinnyMax = 2048;  // choices
 
@@ -432,11 +453,12 @@ __global__ __launch_bounds__(256) void experts_skinny_kernel(SkinnyParams p) {
       for (int r = 0; r < R; ++r)
 #pragma unroll
         for (int v = 0; v < 3; ++v) acc[r] += red[v][r][lane];
+      const float rw = GLU && routed && p.weight != nullptr ? p.weight[a] : 1.f;
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const int n = n0 + 4 * (lane >> 4) + q;
         float v = acc[0][q];
-        if constexpr (GLU) v = v / (1.f + __expf(-v)) * acc[R - 1][q];
+        if constexpr (GLU) v = gated_unit(v * rw, acc[R - 1][q] * rw, p.act, p.limit);
         if (n < N) out[(int64_t)a * ldo + n] = (bf16)v;
       }
     }
@@ -452,7 +474,8 @@ __global__ __launch_bounds__(256) void experts_gemm_f32_kernel(const float* __re
                                                                const int* __restrict__ offs,
                                                                const int* __restrict__ tile_e,
                                                                const int* __restrict__ tile_m,
-                                                               const int* __restrict__ n_tiles, int rows_max, int N,
+                                                               const int* __restrict__ n_tiles,
+                                                               const float* __restrict__ row_weight, int rows_max, int N,
                                                                int K) {
   const int t = blockIdx.y;
   if (t >= *n_tiles) return;
@@ -492,10 +515,11 @@ __global__ __launch_bounds__(256) void experts_gemm_f32_kernel(const float* __re
   for (int i = 0; i < 4; ++i) {
     const int r = r0 + ty * 4 + i;
     if (r >= r1) continue;
+    const float rw = row_weight != nullptr ? row_weight[r] : 1.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) y[(int64_t)r * ldy + n] = acc[i][j];
+      if (n < N) y[(int64_t)r * ldy + n] = acc[i][j] * rw;
     }
   }
 }
@@ -515,15 +539,16 @@ HDS_EXPORT int hds_router_logits(const void* x, int64_t ldx, const void* w, floa
   return hipGetLastError();
 }
 
-// N = experts + identities <= 1024, in `groups` <= 64 equal groups of which `keep` take part
-HDS_EXPORT int hds_router_select(const float* z, int64_t ldz, const float* correction, int* expert, float* weight,
+// N = experts + identities <= 1024, in `groups` <= 64 equal groups of which `keep` take part; sigmoid: scores are sigmoid(z),
+// not softmax(z); correction may be null
+HDS_EXPORT int hds_router_select(const float* z, int64_t ldz, int sigmoid, const float* correction, int* expert, float* weight,
                                  int T, int N, int groups, int keep, int top, float scale, hipStream_t st) {
   if (T <= 0) return 0;
   if (N < 1 || N > 1024 || ldz < N || groups < 1 || groups > 64 || N % groups || keep < 1 || keep > groups || top < 1 ||
       top > keep * (N / groups))
     return hipErrorInvalidValue;
 #define HDS_RS(Q)                                                                                                   \
-  hipLaunchKernelGGL(router_select_kernel<Q>, dim3((T + 3) / 4), dim3(256), 0, st, z, ldz, correction, expert,     \
+  hipLaunchKernelGGL(router_select_kernel<Q>, dim3((T + 3) / 4), dim3(256), 0, st, z, ldz, sigmoid, correction, expert, \
                      weight, T, N, groups, keep, top, scale)
   if (N <= 64) HDS_RS(1); else if (N <= 128) HDS_RS(2); else if (N <= 256) HDS_RS(4); else if (N <= 512) HDS_RS(8);
   else HDS_RS(16);
@@ -531,32 +556,34 @@ HDS_EXPORT int hds_router_select(const float* z, int64_t ldz, const float* corre
   return hipGetLastError();
 }
 
-// n = tokens * k choices; row [n], token [n], offs [E + 1], tile lists of max_tiles >= n / tm + E entries
-HDS_EXPORT int hds_expert_sort(const int* expert, int n, int k, int E, int* offs, int* row, int* token, int tm,
+// n = tokens * k choices; row [n], token [n], weight and row_weight [n] or null, offs [E + 1], tile lists of max_tiles >= n / tm + E entries
+HDS_EXPORT int hds_expert_sort(const int* expert, int n, int k, int E, int* offs, int* row, int* token,
+                               const float* weight, float* row_weight, int tm,
                                int* tile_e, int* tile_m, int* n_tiles, int max_tiles, hipStream_t st) {
   if (n <= 0) return 0;
-  if (k < 1 || E < 1 || E > kMaxExperts || tm < 1 || max_tiles < n / tm + (E < n ? E : n)) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 0, st, expert, n, k, E, offs, row, token, tm, tile_e,
+  if (k < 1 || E < 1 || E > kMaxExperts || tm < 1 || (row_weight != nullptr && weight == nullptr) || max_tiles < n / tm + (E < n ? E : n)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 0, st, expert, n, k, E, offs, row, token, weight,
+                     row_weight, tm, tile_e,
                      tile_m, n_tiles, max_tiles);
   return hipGetLastError();
 }
 
 HDS_EXPORT int hds_experts_skinny_max() { return kSkinnyMax; }
 
-// See SkinnyParams. glu: w / ws hold gate and up rows. kx: choices per row of x. K, Ks % 128 == 0; 16-B rows.
+// See SkinnyParams. glu: w / ws hold gate and up rows, act 0 (silu) or 5 (clamped, with limit). kx: choices per row of x. K, Ks % 128 == 0; 16-B rows.
 HDS_EXPORT int hds_experts_skinny(int glu, const void* x, int64_t ldx, const void* w, void* out, int64_t ldo,
                                   const int* expert, int n, int kx, int E, int N, int K, const void* xs, int64_t ldxs,
-                                  const void* ws, void* outs, int64_t ldos, int n_sh, int Ns, int Ks,
-                                  hipStream_t st) {
+                                  const void* ws, void* outs, int64_t ldos, int n_sh, int Ns, int Ks, int act,
+                                  float limit, const float* weight, hipStream_t st) {
   if (n <= 0) return 0;
   const bool sh = ws != nullptr && n_sh > 0;
-  if (n > kSkinnyMax || kx < 1 || E < 1 || N < 1 || K < 128 || K % 128 || ldx < K || ldx % 8 || ldo < N ||
+  if (n > kSkinnyMax || (act != 0 && act != 5) || kx < 1 || E < 1 || N < 1 || K < 128 || K % 128 || ldx < K || ldx % 8 || ldo < N ||
       (sh && (Ns < 1 || Ks < 128 || Ks % 128 || ldxs < Ks || ldxs % 8 || ldos < Ns)))
     return hipErrorInvalidValue;
   const int slots = n < E ? n : E;
   // n == E: a slot may be read as a choice or as an expert; both cover everything once
   SkinnyParams p{(const bf16*)x, ldx, (const bf16*)w, (bf16*)out, ldo, expert, n, kx, E, N, K, slots, (const bf16*)xs,
-                 ldxs, (const bf16*)ws, (bf16*)outs, ldos, sh ? n_sh : 0, Ns, Ks};
+                 ldxs, (const bf16*)ws, (bf16*)outs, ldos, sh ? n_sh : 0, Ns, Ks, act, limit, weight};
   const int64_t blocks = (int64_t)slots * ((N + 15) / 16) + (sh ? (Ns + 15) / 16 : 0);
   if (glu)
     hipLaunchKernelGGL(experts_skinny_kernel<true>, dim3(blocks), dim3(256), 0, st, p);
@@ -565,13 +592,14 @@ HDS_EXPORT int hds_experts_skinny(int glu, const void* x, int64_t ldx, const voi
   return hipGetLastError();
 }
 
-// rows of 64-row tiles (expert_sort with tm = 64); src: row of x for every sorted row (null: the row itself)
+// rows of 64-row tiles (expert_sort with tm = 64); src: row of x for every sorted row (null: the row itself);
+// row_weight [rows] or null multiplies the results
 HDS_EXPORT int hds_experts_gemm_f32(const float* x, int64_t ldx, const float* w, float* y, int64_t ldy, const int* src,
                                     const int* offs, const int* tile_e, const int* tile_m, const int* n_tiles,
-                                    int max_tiles, int rows, int N, int K, hipStream_t st) {
+                                    int max_tiles, const float* row_weight, int rows, int N, int K, hipStream_t st) {
   if (rows <= 0) return 0;
   if (N < 1 || K < 1 || ldx < K || ldy < N || max_tiles < 1 || max_tiles > 65535) return hipErrorInvalidValue;
   hipLaunchKernelGGL(experts_gemm_f32_kernel, dim3((N + 63) / 64, max_tiles), dim3(256), 0, st, x, ldx, w, y, ldy, src,
-                     offs, tile_e, tile_m, n_tiles, rows, N, K);
+                     offs, tile_e, tile_m, n_tiles, row_weight, rows, N, K);
   return hipGetLastError();
 }

@@ -17,8 +17,8 @@
 //     64 x 256 B tiles of attn_common.h (conflict-free ds_read_b128 A/B fragments), double-buffered:
 //     the next K tile streams in while the current one feeds the MFMAs;
 //   * options (serving, hds_experts_gemm): X rows read through an index list instead of being permuted first; W = [gate;
-//     up] with the activation silu(gate) * up in the epilogue -- a wave then holds the accumulators of the same features
-//     of both halves; a tile list made elsewhere (experts.hip);
+//     up] with the activation silu(gate) * up or the clamped unit, optionally after a factor per row, in the epilogue -- a
+//     wave then holds the accumulators of the same features of both halves; a tile list made elsewhere (experts.hip);
 //   * blockIdx.x walks N tiles fastest so the (consecutively dispatched, XCD-round-robin) blocks of one
 //     token tile share the X tile in L2 while W[e] streams.
 #include "attn_common.h"
@@ -53,7 +53,20 @@ __global__ __launch_bounds__(64) void gg_plan_kernel(const int* __restrict__ off
   if (lane == 0) *n_tiles = base < max_tiles ? base : max_tiles;
 }
 
-__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
+// epilogue of gate | up products
+struct GatedUnit {
+  const float* weight;  // [rows] or null
+  int clamped;
+  float limit;
+  __device__ __forceinline__ float factor(int row) const { return weight != nullptr ? weight[row] : 1.f; }
+  __device__ __forceinline__ float operator()(float g, float u, float w) const {
+    g *= w;
+    u *= w;
+    if (!clamped) return g / (1.f + __expf(-g)) * u;
+    g = fminf(g, limit);
+    return g / (1.f + __expf(-1.702f * g)) * (fminf(fmaxf(u, -limit), limit) + 1.f);
+  }
+};
 
 // GATHER: row r of the sorted order is x[src[r]] (n_src rows of x). GLU: w holds 2N rows per expert, gate then up.
 template <bool GATHER, bool GLU>
@@ -61,7 +74,8 @@ __global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, int
                                                  const int* __restrict__ src, int n_src, const bf16* __restrict__ w,
                                                  bf16* __restrict__ y, const int* __restrict__ offs,
                                                  const int* __restrict__ tile_e, const int* __restrict__ tile_m,
-                                                 const int* __restrict__ n_tiles, int T, int N, int K, int ldy) {
+                                                 const int* __restrict__ n_tiles, int T, int N, int K, int ldy,
+                                                 GatedUnit unit) {
   const int t = blockIdx.y;
   if (t >= *n_tiles) return;  // block-uniform exit before any barrier
   const int e = tile_e[t];
@@ -143,11 +157,12 @@ __global__ __launch_bounds__(256) void gg_kernel(const bf16* __restrict__ x, int
     if (m >= rows) continue;
     bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + (GLU ? 32 : 64) * wn;
     if constexpr (GLU) {
+      const float rw = unit.factor(row0 + m);
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         bf16x4 v;
 #pragma unroll
-        for (int q = 0; q < 4; ++q) v[q] = (bf16)silu_mul(acc[0][j][4 * g + q], acc[1][j][4 * g + q]);
+        for (int q = 0; q < 4; ++q) v[q] = (bf16)unit(acc[0][j][4 * g + q], acc[1][j][4 * g + q], rw);
         *reinterpret_cast<bf16x4*>(yr + acc_row(4 * g, h)) = v;
       }
       continue;
@@ -205,7 +220,7 @@ __global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x,
                                                      const bf16* __restrict__ w, bf16* __restrict__ y, const int* __restrict__ offs,
                                                      const int* __restrict__ tile_e, const int* __restrict__ tile_m,
                                                      const int* __restrict__ n_tiles, int T, int N, int K, int ldy,
-                                                     int ntn) {
+                                                     int ntn, GatedUnit unit) {
   // XCD-contiguous remap of the 1-D grid (bijective for any size)
   const int nwg = gridDim.x, orig = blockIdx.x;
   const int q = nwg / 8, r = nwg % 8, xcd = orig % 8;
@@ -290,13 +305,14 @@ __global__ __launch_bounds__(512) void gg_big_kernel(const bf16* __restrict__ x,
     if (m >= rows) continue;
     bf16* yr = y + (int64_t)(row0 + m) * ldy + n0 + (GLU ? 64 : 128) * wn;
     if constexpr (GLU) {
+      const float rw = unit.factor(row0 + m);
 #pragma unroll
       for (int i = 0; i < 2; ++i)
 #pragma unroll
         for (int g = 0; g < 4; ++g) {
           bf16x4 v;
 #pragma unroll
-          for (int q = 0; q < 4; ++q) v[q] = (bf16)silu_mul(acc[i][j][4 * g + q], acc[i + 2][j][4 * g + q]);
+          for (int q = 0; q < 4; ++q) v[q] = (bf16)unit(acc[i][j][4 * g + q], acc[i + 2][j][4 * g + q], rw);
           *reinterpret_cast<bf16x4*>(yr + 32 * i + acc_row(4 * g, h)) = v;
         }
       continue;
@@ -336,11 +352,12 @@ HDS_EXPORT int hds_grouped_gemm(const void* x, const void* w, void* y, const int
     const int ntn = N / BN2;
     hipLaunchKernelGGL(gg_plan_kernel<BM2>, dim3(1), dim3(64), 0, st, offs, E, T, tile_e, tile_m, n_tiles, max_tiles);
     hipLaunchKernelGGL((gg_big_kernel<false, false>), dim3(ntn * max_tiles), dim3(512), 0, st, (const bf16*)x, K,
-                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, ntn);
+                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, ntn,
+                       GatedUnit{});
   } else {
     hipLaunchKernelGGL(gg_plan_kernel<BM>, dim3(1), dim3(64), 0, st, offs, E, T, tile_e, tile_m, n_tiles, cap);
     hipLaunchKernelGGL((gg_kernel<false, false>), dim3(N / BN, cap), dim3(256), 0, st, (const bf16*)x, K,
-                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy);
+                       (const int*)nullptr, 0, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, GatedUnit{});
   }
   return hipGetLastError();
 }
@@ -350,23 +367,26 @@ HDS_EXPORT int hds_experts_gemm_tile(int T, int N, int E) { return N % BN2 == 0 
 
 // Grouped product of sorted rows with a ready tile list (tm = 128 or 256 rows, see hds_experts_gemm_tile; at most
 // max_tiles entries, the number on the device). src: row of x [n_src, ldx] for every sorted row, or null: x is sorted.
-// glu: w [E, 2N, K] is gate rows then up rows and y = silu(gate) * up. T: upper bound of the rows. K % 128 == 0; N a
+// glu: w [E, 2N, K] is gate rows then up rows and y = silu(gate) * up, or the clamped unit with its limit (act 5); weight [T]
+// or null multiplies the sorted rows' products in front of it. T: upper bound of the rows. K % 128 == 0; N a
 // multiple of the tile's columns (128, 256; half of that with glu).
 HDS_EXPORT int hds_experts_gemm(const void* x, int64_t ldx, const int* src, int n_src, const void* w, void* y, int ldy,
                                 const int* offs, const int* tile_e, const int* tile_m, const int* n_tiles,
-                                int max_tiles, int tm, int T, int N, int K, int E, int glu, hipStream_t st) {
+                                int max_tiles, int tm, int T, int N, int K, int E, int glu, int act, float limit,
+                                const float* weight, hipStream_t st) {
   if (T <= 0 || E <= 0) return 0;
+  const GatedUnit unit{weight, act == 5, limit};
   const int cols = (tm == BM2 ? BN2 : BN) / (glu ? 2 : 1);
   if ((tm != BM && tm != BM2) || N % cols || K % BK || ldx < K || ldx % 8 || ldy < N || ldy % 8 || max_tiles < 1 ||
-      max_tiles > 65535 || (src != nullptr && n_src < 1))
+      max_tiles > 65535 || (src != nullptr && n_src < 1) || (act != 0 && act != 5))
     return hipErrorInvalidValue;
 #define HDS_EG(GA, GL)                                                                                               \
   if (tm == BM2)                                                                                                     \
     hipLaunchKernelGGL((gg_big_kernel<GA, GL>), dim3(N / cols * max_tiles), dim3(512), 0, st, (const bf16*)x, ldx,  \
-                       src, n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, N / cols); \
+                       src, n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, N / cols, unit); \
   else                                                                                                               \
     hipLaunchKernelGGL((gg_kernel<GA, GL>), dim3(N / cols, max_tiles), dim3(256), 0, st, (const bf16*)x, ldx, src,  \
-                       n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy)
+                       n_src, (const bf16*)w, (bf16*)y, offs, tile_e, tile_m, n_tiles, T, N, K, ldy, unit)
   if (src != nullptr) {
     if (glu) { HDS_EG(true, true); } else { HDS_EG(true, false); }
   } else {

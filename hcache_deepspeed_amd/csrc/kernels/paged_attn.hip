@@ -21,7 +21,7 @@
 // so K/V of a kv head are read ONCE for all of its query heads -- for decode (1 token) one wave
 // serves the whole GQA group from a single pass over the sequence's KV blocks.
 //
-// Options of all attention kernels: a sliding window; chunks, runs of positions counted from the sequence's start that see
+// Options of all attention kernels: a sliding window, in front of which the sequence's first `keep` positions stay visible; chunks, runs of positions counted from the sequence's start that see
 // only themselves; a soft cap of the scores, cap * tanh(score / cap); a sink, one score per query head that joins the
 // softmax denominator but has no key and no value; an output gate, one value per token and query head (or per element of
 // the head's output) whose sigmoid multiplies it. head_norm_scatter is the counterpart of the RoPE scatter for heads that
@@ -250,7 +250,7 @@ __device__ __forceinline__ float soft_cap2(float x, float cap2, float inv2) {
   return cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(fast_exp2(x * inv2) + 1.f);
 }
 
-// the first position that position pos sees (window, chunk: 0 for none)
+// the first position that position pos sees (window, chunk: 0 for none), apart from the kept ones below `keep`
 __device__ __forceinline__ int first_key(int pos, int window, int chunk) {
   int lo = window > 0 ? max(0, pos + 1 - window) : 0;
   if (chunk > 0) lo = max(lo, pos - pos % chunk);
@@ -271,7 +271,7 @@ struct PagedParams {
   int hq, hkv;
   int dk, dv;  // read by the padded kernels only
   float scale;
-  int window, chunk;
+  int window, chunk, keep;
   float softcap;      // 0: none
   const float* sink;  // [Hq] or null
   const bf16* gate;   // [T, Hq * gw] with token stride sg, or null
@@ -329,6 +329,9 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
   const int ctx = wg_qpos_max + 1;
   const int kt_end = (ctx + BN - 1) / BN;
   const int kt_begin = bounded ? first_key(seen + row_start / G, p.window, p.chunk) / BN : 0;
+  const int kept = bounded ? min((p.keep + BN - 1) / BN, kt_begin) : 0;  // tiles of kept keys ahead of the others
+  const int n_tiles = kt_end - kt_begin + kept;
+  auto tile_at = [&](int i) { return i < kept ? i : i - kept + kt_begin; };
   auto rowp = [&](int kt, int off) {
     return [=](int row) {
       int pos = kt * BN + row;
@@ -363,16 +366,16 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
     l = 1.f;
   }
 
-  stage(0, kt_begin);
+  stage(0, tile_at(0));
   __syncthreads();
-  for (int kt = kt_begin; kt < kt_end; ++kt) {
-    const int buf = (kt - kt_begin) & 1;
+  for (int it = 0; it < n_tiles; ++it) {
+    const int buf = it & 1, kt = tile_at(it);
     const char* Kt = smem + buf * TLK;
     const char* Vt = smem + 2 * TLK + buf * TLV;
-    if (kt + 1 < kt_end) stage(buf ^ 1, kt + 1);
+    if (it + 1 < n_tiles) stage(buf ^ 1, tile_at(it + 1));
     const int k0 = kt * BN;
     bool skip = !wave_active || k0 > w_qpos_hi;
-    if (k0 + BN - 1 < w_lo) skip = true;
+    if (k0 + BN - 1 < w_lo && k0 >= p.keep) skip = true;
     if (!skip) {
       f32x16 s[2];
 #pragma unroll
@@ -395,7 +398,7 @@ __global__ __launch_bounds__(64 * NW, (atom_waves<DK, DV>())) void paged_attn_ke
         for (int r = 0; r < 16; ++r) {
           const int kp = k0 + 32 * t + acc_row(r, h);
           float x = s[t][r] * c;
-          if (kp > qpos || !row_ok || kp < lo) x = -INFINITY;
+          if (kp > qpos || !row_ok || (kp < lo && kp >= p.keep)) x = -INFINITY;
           s[t][r] = x;
           tmax = fmaxf(tmax, x);
         }
@@ -485,7 +488,7 @@ struct PagedDecodeParams {
   const int* block_tables;
   int max_blocks, block_size, hq, hkv, dk, dv, splits;
   float scale;
-  int window, chunk;
+  int window, chunk, keep;
   float softcap;      // 0: none
   const float* sink;  // [Hq] or null
   const T* gate;      // [T, Hq * gw] with token stride sg, or null
@@ -508,13 +511,16 @@ __device__ __forceinline__ DecodeToken decode_token(const PagedDecodeParams<T>& 
   return {t, p.tok_seq[t], p.tok_pos[t]};
 }
 
-// this split's keys: an equal share of what the token sees
+// this split's keys: an equal share of what the token sees, counted without the gap between the kept keys and the others
+struct DecodeKeys {
+  int j0, j1, keep, gap;
+  __device__ __forceinline__ int pos(int j) const { return j < keep ? j : j + gap; }
+};
 template <typename T>
-__device__ __forceinline__ void decode_keys(const PagedDecodeParams<T>& p, int pos, int split, int& j0, int& j1) {
-  const int lo = first_key(pos, p.window, p.chunk);
-  const int per = (pos + 1 - lo + p.splits - 1) / p.splits;
-  j0 = lo + split * per;
-  j1 = min(pos + 1, j0 + per);
+__device__ __forceinline__ DecodeKeys decode_keys(const PagedDecodeParams<T>& p, int pos, int split) {
+  const int gap = max(first_key(pos, p.window, p.chunk) - p.keep, 0), n = pos + 1 - gap;
+  const int per = (n + p.splits - 1) / p.splits;
+  return {split * per, min(n, split * per + per), p.keep, gap};
 }
 
 // factor of head h's weighted value sum whose softmax so far has maximum m and denominator l
@@ -571,8 +577,8 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int kl = lane / LPK, c = lane % LPK;
   const DecodeToken tk = decode_token(p, b);
-  int j0, j1;
-  decode_keys(p, tk.pos, split, j0, j1);
+  const DecodeKeys keys = decode_keys(p, tk.pos, split);
+  const int j0 = keys.j0, j1 = keys.j1;
   const PageTable pages(p.block_tables + (int64_t)tk.seq * p.max_blocks, p.block_size, p.max_blocks);
   const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
   // lanes past a head's size read its start: their q is zero, their value columns are not stored
@@ -601,7 +607,7 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(PagedDecodeParams<bf1
   auto fetch = [&](int j) {
     int64_t r[U];
 #pragma unroll
-    for (int u = 0; u < U; ++u) r[u] = pages.slot(min(j + u * STEP, j1 - 1)) * kv_row;
+    for (int u = 0; u < U; ++u) r[u] = pages.slot(keys.pos(min(j + u * STEP, j1 - 1))) * kv_row;
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       kn[u] = *reinterpret_cast<const bf16x8*>(kbase + r[u]);
@@ -734,11 +740,11 @@ __global__ __launch_bounds__(256) void paged_plain_kernel(PagedDecodeParams<T> p
   const int split = blockIdx.x, h = blockIdx.y, b = blockIdx.z, hk = h / (p.hq / p.hkv);
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const DecodeToken tk = decode_token(p, b);
-  int j0, j1;
-  decode_keys(p, tk.pos, split, j0, j1);
+  const DecodeKeys keys = decode_keys(p, tk.pos, split);
+  const int j0 = keys.j0, j1 = keys.j1;
   const PageTable pages(p.block_tables + (int64_t)tk.seq * p.max_blocks, p.block_size, p.max_blocks);
   const int64_t kv_row = (int64_t)p.hkv * (p.dk + p.dv);
-  auto slot = [&](int j) { return p.cache + pages.slot(j) * kv_row; };
+  auto slot = [&](int j) { return p.cache + pages.slot(keys.pos(j)) * kv_row; };
   for (int i = threadIdx.x; i < p.dk; i += 256) sq[i] = to_f(p.q[(int64_t)tk.row * p.sq + (int64_t)h * p.dk + i]);
   for (int i = threadIdx.x; i < p.dv; i += 256) acc[i] = 0.f;
   __syncthreads();
@@ -921,18 +927,18 @@ HDS_EXPORT int hds_paged_attn_supported(int dk, int dv) {
   return dk >= 8 && dv >= 8 && dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256;
 }
 
-// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]; window, chunk and softcap: 0 for none; sink [hq]
+// atoms: device int32 [n_atoms][3]; seq_meta: device int32 [n_seqs][3]; window, chunk, keep and softcap: 0 for none; sink [hq]
 // and gate [tokens, hq * gw] (gw 1 or dv) may be null
 HDS_EXPORT int hds_paged_attn(const void* q, int64_t sq, const void* cache, void* o, int64_t so, const int* atoms,
                               int n_atoms, const int* seq_meta, const int* block_tables, int max_blocks,
                               int block_size, int hq, int hkv, int dk, int dv, float scale, int window, int chunk,
-                              float softcap, const float* sink, const void* gate, int64_t sg, int gw, hipStream_t st) {
+                              int keep, float softcap, const float* sink, const void* gate, int64_t sg, int gw, hipStream_t st) {
   if (hq < 1 || hkv < 1 || hq % hkv || sq % 8 || so % 4 || !hds_paged_attn_supported(dk, dv) || window < 0 ||
-      chunk < 0 || (gate != nullptr && gw != 1 && (gw != dv || sg % 4 || (uintptr_t)gate % 8)))
+      chunk < 0 || keep < 0 || (gate != nullptr && gw != 1 && (gw != dv || sg % 4 || (uintptr_t)gate % 8)))
     return hipErrorInvalidValue;
   if (n_atoms <= 0) return 0;
   PagedParams p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, atoms, seq_meta, block_tables, max_blocks,
-                block_size, hq, hkv, dk, dv, scale, window, chunk, softcap, sink, (const bf16*)gate, sg, gw};
+                block_size, hq, hkv, dk, dv, scale, window, chunk, keep, softcap, sink, (const bf16*)gate, sg, gw};
 #define HDS_CASE(d)                                                                                    \
   if (dk == d && dv == d) {                                                                            \
     hipLaunchKernelGGL((paged_attn_kernel<d, d, 4, false>), dim3(n_atoms), dim3(256), 0, st, p);       \
@@ -973,24 +979,24 @@ HDS_EXPORT int hds_paged_decode(int dtype, int plain, const void* q, int64_t sq,
                                 float* part_o, float* part_ml, const int* seq_meta, const int* toks,
                                 const int* tok_seq, const int* tok_pos, const int* block_tables, int max_blocks,
                                 int block_size, int n, int hq, int hkv, int dk, int dv, int splits, float scale,
-                                int window, int chunk, float softcap, const float* sink, const void* gate, int64_t sg,
-                                int gw, int* counters, hipStream_t st) {
+                                int window, int chunk, int keep, float softcap, const float* sink, const void* gate,
+                                int64_t sg, int gw, int* counters, hipStream_t st) {
   if (n <= 0) return 0;
   if (hq < 1 || hkv < 1 || hq % hkv || dk < 1 || dv < 1 || splits < 1 || splits > 64 || n > 65535 ||
-      window < 0 || chunk < 0 || (gate != nullptr && gw != 1 && gw != dv) ||
+      window < 0 || chunk < 0 || keep < 0 || (gate != nullptr && gw != 1 && gw != dv) ||
       (seq_meta == nullptr && (tok_seq == nullptr || tok_pos == nullptr)) ||
       (splits > 1 && (!part_o || !part_ml)))  // <= 64: the combine kernel stages the split stats in LDS
     return hipErrorInvalidValue;
   if (dtype == kF32) {
     return launch_plain(PagedDecodeParams<float>{(const float*)q, sq, (const float*)cache, (float*)o, so, part_o,
                                                  part_ml, seq_meta, toks, tok_seq, tok_pos, block_tables, max_blocks,
-                                                 block_size, hq, hkv, dk, dv, splits, scale, window, chunk, softcap,
+                                                 block_size, hq, hkv, dk, dv, splits, scale, window, chunk, keep, softcap,
                                                  sink, (const float*)gate, sg, gw, nullptr}, n, st);
   }
   if (dtype != kBF16) return hipErrorInvalidValue;
   PagedDecodeParams<bf16> p{(const bf16*)q, sq, (const bf16*)cache, (bf16*)o, so, part_o, part_ml, seq_meta, toks,
                             tok_seq, tok_pos, block_tables, max_blocks, block_size, hq, hkv, dk, dv, splits, scale,
-                            window, chunk, softcap, sink, (const bf16*)gate, sg, gw, counters};
+                            window, chunk, keep, softcap, sink, (const bf16*)gate, sg, gw, counters};
   if (plain) {
     p.counters = nullptr;
     return launch_plain(p, n, st);

@@ -42,7 +42,7 @@ class ArchSpec:
     lm_head_bias: bool = False
     moe: Optional[dict] = None         # {num_experts, top_k, normalize, shared}
     # layers listed one by one (hybrid.py): one entry per layer with weights, {"mixer": {"type", sizes ...}, "mlp":
-    # {"ff", "act"[, "limit"]}, {"ff", "act", "shared_ff", "router": {...}} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
+    # {"ff", "act"[, "limit"]}, {"kind": "moe", "ff", "act"[, "limit"], "shared_ff", "router": {...}} or None}; loop: {"start", "stop", "times"}, layers that run several times in a row
     layers: Optional[list] = None
     loop: Optional[dict] = None
     order: Optional[list] = None       # the layer every layer run uses (None: each once, with ``loop``)
@@ -51,6 +51,8 @@ class ArchSpec:
     embed_scale: float = 1.0
     logit_scale: float = 1.0
     logit_softcap: float = 0.0         # logits <- cap * tanh(logits / cap); 0: none
+    pair_embed: Optional[dict] = None  # {"mul_prev", "mul_cur"}: a second embedding row by the previous and this token
+    token_side: int = 0                # width of every layer's own input by the token (a table beside the embedding)
     extra: dict = field(default_factory=dict)
 
     # LlamaConfig-compatible aliases used by the engine / KV cache sizing
@@ -257,9 +259,90 @@ def convert_fifotar(sd, spec):
     return out
 
 
+# ---------------------------------------------------------------------------------------------
+# Duzizen: matrix memories with exponential gates (mLSTM), and layers of two mixers side by side: attention with short
+# convolutions, norms across the heads and keys that are the values (window with kept first tokens, zero sink), and
+# retention; dense or routed feed-forwards, layer norms on both sides of every sublayer, an input of its own per layer
+# and token, a bigram embedding
+# ---------------------------------------------------------------------------------------------
+def _duzizen_attention(m):
+    if int(m["vdim"]) != int(m["dim"]):
+        raise ValueError(f"Duzizen attention: the values are the keys, but vdim {m['vdim']} is not dim {m['dim']}")
+    rot, mask = m["rot"], m.get("mask") or {}
+    sc = rot.get("scaling")
+    if sc is not None:
+        sc = {"rope_type": "llama3", "factor": float(sc["factor"]), "low_freq_factor": float(sc["low"]),
+              "high_freq_factor": float(sc["high"]), "original_max_position_embeddings": float(sc["original"])}
+    return {"type": "attention", **{k: int(m[k]) for k in ("heads", "kv_heads", "dim", "vdim", "conv")},
+            "window": int(mask.get("size") or 0), "keep": int(mask.get("keep_first") or 0), "scale": float(m["scale"]),
+            "rot_dims": int(rot["dims"]), "rope_base": float(rot["base"]), "rope_scaling": sc, "shared_values": True,
+            "norm_all": True, "zero_sink": True, "gated": False}
+
+
+def _duzizen_mixer(kind, m):
+    if kind == "mlstm":
+        return {"type": kind, **{k: int(m[k]) for k in ("heads", "dim", "vdim")}, "cap": float(m["gate_cap"])}
+    if kind == "parallel":
+        left, right = m["left"], m["right"]
+        if len(right["decay"]) != int(right["heads"]):
+            raise ValueError("Duzizen retention: one decay per head")
+        return {"type": kind, "left": _duzizen_attention(left),
+                "right": {"type": "retention", **{k: int(right[k]) for k in ("heads", "dim", "vdim")},
+                          "decay": [float(d) for d in right["decay"]], "rot_dims": int(right["rot"]["dims"]),
+                          "rope_base": float(right["rot"]["base"]), "rot_layout": "half"}}
+    raise NotImplementedError(f"Duzizen mixer {kind!r}")
+
+
+def _duzizen_mlp(mlp):
+    if mlp is None:
+        return None
+    if mlp["kind"] == "dense":
+        return {"ff": int(mlp["ff"]), "act": "gelu_tanh"}
+    if mlp["kind"] == "moe":
+        r = mlp["router"]
+        return {"kind": "moe", "ff": int(mlp["expert"]["ff"]), "act": "clamped", "limit": float(mlp["expert"]["limit"]),
+                "router": {"experts": int(r["experts"]), "top": int(r["top"]), "score": "sigmoid",
+                           "weigh_input": True}}
+    raise NotImplementedError(f"Duzizen feed-forward {mlp['kind']!r}")
+
+
+def spec_duzizen(cfg):
+    layers = [{"mixer": _duzizen_mixer(e["type"], e["mixer"]), "mlp": _duzizen_mlp(e.get("mlp"))} for e in cfg["layers"]]
+    pair = (cfg.get("embedding") or {}).get("bigram")
+    attn = [x["mixer"]["left"] for x in layers if x["mixer"]["type"] == "parallel"]
+    return ArchSpec(model_type="duzizen", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                    num_hidden_layers=len(layers), num_attention_heads=max((a["heads"] for a in attn), default=1),
+                    num_key_value_heads=max((a["kv_heads"] for a in attn), default=1),
+                    head_dim=max((a["dim"] for a in attn), default=0),
+                    intermediate_size=max((x["mlp"]["ff"] for x in layers if x["mlp"]), default=0), norm="ln",
+                    norm_eps=float(cfg["norm"]["eps"]), act="gelu_tanh", gated=True, layers=layers, norm_place="both",
+                    pair_embed={k: int(pair[k]) for k in ("mul_prev", "mul_cur")} if pair else None,
+                    token_side=int((cfg.get("token_side") or {}).get("dim") or 0))
+
+
+def convert_duzizen(sd, spec):
+    out = {"embed": sd["embed"], "pair_embed": sd.get("bigram"), "side_embed": sd.get("side.embed"),
+           "final.w": sd["final.norm"], "final.b": sd["final.norm.b"], "lm_head.w": sd["head"], "layers": []}
+    for i, e in enumerate(spec.layers):
+        p = f"l{i}."
+        L = {"mix": {k[len(p) + 4:]: v for k, v in sd.items() if k.startswith(p + "mix.")}}
+        for k in ("1", "1b", "2", "2b") if e["mlp"] is not None else ("1", "1b"):
+            L[f"ln{k}.w"], L[f"ln{k}.b"] = sd[f"{p}norm{k}"], sd[f"{p}norm{k}.b"]
+        if e["mlp"] is not None and e["mlp"].get("kind") == "moe":
+            L["experts"] = {k: torch.stack([sd[f"{p}mlp.e{x}.{k}"] for x in range(e["mlp"]["router"]["experts"])])
+                            for k in ("gate", "up", "down")}
+            L["experts"]["router"] = sd[p + "mlp.router"]
+        elif e["mlp"] is not None:
+            L.update({f"{k}.w": sd[f"{p}mlp.{k}"] for k in ("gate", "up", "down")})
+        if spec.token_side:
+            L.update({f"side.{k}.w": sd[f"{p}side.{k}"] for k in ("gate", "proj", "norm")})
+        out["layers"].append(L)
+    return out
+
+
 # config.json's "architecture" / "model_type" -> (config reader, weight converter)
 ARCHITECTURES = {"gofasun": (spec_gofasun, convert_gofasun), "buvuzen": (spec_buvuzen, convert_buvuzen),
-                 "fifotar": (spec_fifotar, convert_fifotar)}
+                 "fifotar": (spec_fifotar, convert_fifotar), "duzizen": (spec_duzizen, convert_duzizen)}
 
 
 def spec_from_hf(hf):

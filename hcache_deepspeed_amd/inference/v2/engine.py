@@ -19,7 +19,7 @@ import torch
 
 from ... import comm as dist
 from ...utils.logging import log_dist
-from .hybrid import HybridTransformer, PostNormTransformer, SandwichTransformer
+from .hybrid import HybridTransformer, MemorySandwichTransformer, PostNormTransformer, SandwichTransformer
 from .model import RaggedTransformer
 from .ragged import (BlockedKVCache, DSStateManager, DSStateManagerConfig, RaggedBatchWrapper, SequenceStatePool)
 
@@ -63,6 +63,8 @@ def transformer_class(spec):
     """The model implementation that serves an ArchSpec."""
     if spec.layers is None:
         return RaggedTransformer
+    if spec.norm_place == "both" and spec.norm == "ln":
+        return MemorySandwichTransformer
     return {"pre": HybridTransformer, "post": PostNormTransformer, "both": SandwichTransformer}[spec.norm_place]
 
 
@@ -293,6 +295,7 @@ class InferenceEngineV2:
         m = self._model
         sd = {"embed": m.embed, "pos_embed": m.pos_embed, "final.w": m.final_w, "final.b": m.final_b,
               "lm_head.w": m.lm_head, "lm_head.b": m.lm_head_b,
+              "pair_embed": getattr(m, "pair_embed", None), "side_embed": getattr(m, "side_embed", None),
               "layers": [{k: v for k, v in L.w.items() if v is not None} for L in m.layers]}
 
         from .modules.implementations import _PackedWeight
@@ -343,7 +346,7 @@ def build_hf_engine(path, engine_config=None, debug_level=None, device=None, num
     """Serving engine from a HuggingFace checkpoint directory (config.json + *.safetensors / *.bin).
 
     Supported ``model_type``: llama, mistral, mixtral, qwen, qwen2, qwen2_moe, phi, phi3, falcon, opt
-    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun, Buvuzen, Fifotar."""
+    (reference inference/v2/engine_factory.py:69-130); ``architecture``: Gofasun, Buvuzen, Fifotar, Duzizen."""
     from .arch import convert_hf, spec_from_hf
     with open(os.path.join(path, "config.json")) as f:
         hf = json.load(f)

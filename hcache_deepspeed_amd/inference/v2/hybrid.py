@@ -9,8 +9,10 @@ paged cache, batch metadata and decode graphs as :class:`model.RaggedTransformer
 * :class:`PostNormTransformer` ("post"): mixer, then expert layer, each reading the residual itself; the norm is on their
   outputs. A layer is: mixer and its output projection, norm + residual add (one kernel), router and experts, and one
   kernel that sums the experts' outputs, norms the sum and adds it.
-* :class:`SandwichTransformer` ("both"): mixer, then gated MLP, each between a norm of its input and a norm of its output.
-  One kernel between two sublayers norms the first one's output, adds it to the residual and norms the sum for the next.
+* :class:`SandwichTransformer` ("both"): mixer, then gated MLP or routed experts, each between a norm of its input and a norm
+  of its output (RMS or layer norms). One kernel between two sublayers norms the first one's output, adds it to the residual
+  and norms the sum for the next. Optionally a third sublayer without a norm of its input: the residual gates a row of the
+  token's own, one per layer (``token_side``), and a second embedding row by the previous and this token (``pair_embed``).
 
 Common to all:
 
@@ -21,10 +23,10 @@ Common to all:
 """
 import torch
 
+from ...ops.activations import act_gather
 from ...ops.experts import RouterShape
-from ...ops.output_norm import norm_rows
+from ...ops.output_norm import embed_pairs, norm_rows
 from ...ops.paged import copy_rows
-from ...ops.rope import rope_tables
 from .arch import run_order
 from .model import RaggedTransformer, _Layer
 from .modules import (DSExpertLayerConfig, DSGatedMLPConfig, DSInputNormConfig, DSLinearConfig, DSMixerConfig,
@@ -43,7 +45,8 @@ class _Run:
 
 
 # weights kept in the engine's dtype; every other float32 tensor stays float32
-_MATRICES = ("in.w", "up.w", "out.w", "down.w", "uq.w", "ukv.w", "router.w", "w13", "w2", "ws13", "ws2")
+_MATRICES = ("in.w", "up.w", "out.w", "down.w", "uq.w", "ukv.w", "router.w", "w13", "w2", "ws13", "ws2", "left.o.w",
+             "right.o.w", "side.gate.w", "side.proj.w")
 
 
 class HybridTransformer(RaggedTransformer):
@@ -74,12 +77,13 @@ class HybridTransformer(RaggedTransformer):
         for e in spec.layers:
             mix = instantiate_mixer(DSMixerConfig(e["mixer"]["type"], H, e["mixer"], spec.norm_eps, self.tp,
                                                   self.dtype), ec)
-            if hasattr(mix, "bind_tables"):
-                mix.bind_tables(*rope_tables(self.max_positions, mix.shape.rot_dims, mix.rope_base, mix.rope_scaling,
-                                             device=self.device))
+            mix.bind_positions(self.max_positions, self.device)
+            mix.bind_group(self._allreduce)
             self.mixers.append(mix)
         self._build_layers(ec)
         for lins, mix in zip(self.linears, self.mixers):
+            if mix.own_output:
+                lins.pop("out.w")
             lins.update({k: instantiate_linear(DSLinearConfig(*io), ec) for k, io in mix.extra_linears().items()})
 
     def _build_layers(self, ec):
@@ -110,7 +114,9 @@ class HybridTransformer(RaggedTransformer):
             return self._load_presharded(sd)
         t, f, r = self._t, self._f32, self.tp_rank
         self.embed, self.final_w = t(sd["embed"]), f(sd["final.w"].reshape(-1))
-        self.pos_embed = self.final_b = self.lm_head_b = None
+        self.pos_embed = self.lm_head_b = None
+        self.final_b = f(sd.get("final.b"))
+        self._load_tables(sd)
         lm = sd["lm_head.w"]
         self.vocab = lm.shape[0]
         vs = -(-self.vocab // self.tp)
@@ -123,14 +129,20 @@ class HybridTransformer(RaggedTransformer):
         for i, Ls in enumerate(sd["layers"]):
             L = _Layer()
             mw = self.mixers[i].shard(Ls["mix"], self._rows, self._cols)
-            o = mw.pop("o.w")
+            o = mw.pop("o.w", None)
             self._put(L, mw)
-            for k in ("1", "2", "1b", "2b"):
-                if Ls.get(f"ln{k}.w") is not None:
-                    L.w[f"ln{k}.w"] = f(Ls[f"ln{k}.w"].reshape(-1))
-            L.w["out.w"] = t(self._load_layer(i, L, Ls, o))
+            for k in (f"ln{n}.{kind}" for n in ("1", "2", "1b", "2b") for kind in "wb"):
+                if Ls.get(k) is not None:
+                    L.w[k] = f(Ls[k].reshape(-1))
+            o = self._load_layer(i, L, Ls, o)
+            if o is not None:
+                L.w["out.w"] = t(o)
             self._transform(L)
             self.layers.append(L)
+
+    def _load_tables(self, sd):
+        """Tables by token besides the embedding."""
+        self.pair_embed, self.side_embed = self._t(sd.get("pair_embed")), self._t(sd.get("side_embed"))
 
     def _put(self, L, weights):
         for k, v in weights.items():
@@ -149,7 +161,9 @@ class HybridTransformer(RaggedTransformer):
     def _load_presharded(self, sd):
         t, f = self._t, self._f32
         self.embed, self.final_w, self.lm_head = t(sd["embed"]), f(sd["final.w"]), t(sd["lm_head.w"])
-        self.pos_embed = self.final_b = self.lm_head_b = None
+        self.pos_embed = self.lm_head_b = None
+        self.final_b = f(sd.get("final.b"))
+        self._load_tables(sd)
         self.vocab = self.spec.vocab_size
         self.layers = []
         for Ls in sd["layers"]:
@@ -164,7 +178,7 @@ class HybridTransformer(RaggedTransformer):
             self.layers.append(L)
 
     def _plan_runs(self):
-        self.runs, off = [], 0
+        self.runs, off = [], 4 if self.spec.pair_embed else 0  # the last token, ahead of the layers' states
         self.row_widths = []
         for li in run_order(self.spec):
             mix = self.mixers[li]
@@ -330,56 +344,104 @@ class PostNormTransformer(HybridTransformer):
 
 
 class SandwichTransformer(HybridTransformer):
-    """Layers with a norm on both sides of every sublayer: x += n1b(mixer(n1(x))), x += n2b(mlp(n2(x))); the factor of the
-    residual sum is part of the gains of n1b and n2b."""
+    """Layers with a norm on both sides of every sublayer: x += n1b(mixer(n1(x))), x += n2b(ff(n2(x))); a factor of the
+    residual sum is part of the gains of n1b and n2b. With ``token_side``, behind it x += n(proj(gelu(gate x) * e)), e the
+    token's row of this layer."""
     KERNEL_SOURCES = ("act.hip", "delta_rule.hip", "gemv.hip", "latent_attn.hip", "output_norm.hip", "paged_attn.hip",
                       "paged_rows.hip")
 
     def _build_layers(self, ec):
         spec, H = self.spec, self.spec.hidden_size
-        self.norm_mod = instantiate_sandwich_norm(DSNormConfig(H, "rms", spec.norm_eps, torch.float32, self.dtype), ec)
+        self.norm_mod = instantiate_sandwich_norm(
+            DSNormConfig(H, "layer" if spec.norm == "ln" else "rms", spec.norm_eps, torch.float32, self.dtype), ec)
         for e, mix in zip(spec.layers, self.mixers):
             m = e["mlp"]
             lins = {"in.w": instantiate_linear(DSLinearConfig(H, mix.in_width), ec),
                     "out.w": instantiate_linear(DSLinearConfig(mix.out_width, H), ec)}
             mlp, ff = None, 0
-            if m is not None:
+            if m is not None and m.get("kind") == "moe":
+                mlp = instantiate_expert_layer(
+                    DSExpertLayerConfig(H, m["ff"], RouterShape(**m["router"]), m.get("shared_ff", 0), self.tp, self.dtype,
+                                        m["act"], m.get("limit", 0.0)), ec)
+            elif m is not None:
                 assert m["ff"] % self.tp == 0, "the feed-forward width must divide the tensor-parallel size"
                 ff = m["ff"] // self.tp
                 mlp = instantiate_gated_mlp(DSGatedMLPConfig(H, ff, m["act"], m.get("limit", 0.0)), ec)
                 lins["up.w"] = instantiate_linear(DSLinearConfig(H, 2 * ff), ec)
                 lins["down.w"] = instantiate_linear(DSLinearConfig(ff, H), ec)
+            if spec.token_side:
+                lins["side.gate.w"] = instantiate_linear(DSLinearConfig(H, spec.token_side), ec)
+                lins["side.proj.w"] = instantiate_linear(DSLinearConfig(spec.token_side, H), ec)
             self.mlps.append((mlp, ff))
             self.linears.append(lins)
 
     def _load_layer(self, i, L, Ls, o):
-        if self.mlps[i][0] is not None:
+        mlp, ff = self.mlps[i]
+        if "experts" in Ls:
+            self._put(L, mlp.shard(Ls["experts"], self._rows, self._cols))
+        elif mlp is not None:
             L.w["up.w"] = self._t(torch.cat([self._rows(Ls["gate.w"]), self._rows(Ls["up.w"])]))
             L.w["down.w"] = self._t(self._cols(Ls["down.w"]))
+        if self.spec.token_side:
+            L.w["side.gate.w"], L.w["side.proj.w"] = self._t(Ls["side.gate.w"]), self._t(Ls["side.proj.w"])
+            L.w["side.norm.w"] = self._f32(Ls["side.norm.w"])
         return o
 
     def _norm_state_floats(self):
         return 0
 
-    # the stream: (32-bit residual or None at the start, the last sublayer's output, the gain of its norm)
+    # the stream: (32-bit residual or None at the start, the last sublayer's output, its norm)
     def _start(self, batch):
-        self._rows_in = (self.embed, batch.input_ids, self.spec.embed_scale)
-        return None, None, None
+        spec = self.spec
+        self._rows_in = (self.embed, batch.input_ids, spec.embed_scale)
+        if not spec.pair_embed:
+            return None, None, None
+        return embed_pairs(self.embed, self.pair_embed, batch.input_ids, spec.embed_scale, spec.pair_embed["mul_prev"],
+                           spec.pair_embed["mul_cur"], self._state(), 0, batch), None, None
 
     def _final(self, stream, idx):
-        return self.norm_mod(*stream, self.final_w, embed=self._rows_in, idx=idx)[1]
+        norm = self.final_w if self.final_b is None else (self.final_w, self.final_b)
+        return self.norm_mod(*stream, norm, embed=self._rows_in, idx=idx)[1]
+
+    @staticmethod
+    def _norm_of(L, k):
+        w, b = L[f"ln{k}.w"], L[f"ln{k}.b"]
+        return w if b is None else (w, b)
 
     def _layer(self, run, stream, batch):
         i = run.layer
         L, mix, (mlp, ff), lins = self.layers[i], self.mixers[i], self.mlps[i], self.linears[i]
         T = batch.current_tokens
-        x, rows = self.norm_mod(*stream, L["ln1.w"], embed=self._rows_in)
+        x, rows = self.norm_mod(*stream, self._norm_of(L, "1"), embed=self._rows_in)
         mid = torch.empty(T, mix.out_width, dtype=self.dtype, device=self.device)
         self._mix(run, rows, mid, batch)
-        y = self._allreduce(lins["out.w"](mid, L["out.w"]))
-        if mlp is None:
-            return x, y, L["ln1b.w"]
-        x, rows = self.norm_mod(x, y, L["ln1b.w"], L["ln2.w"])
-        h = torch.empty(T, ff, dtype=self.dtype, device=self.device)
-        mlp(rows, L["up.w"], lins["up.w"], h)
-        return x, self._allreduce(lins["down.w"](h, L["down.w"])), L["ln2b.w"]
+        y, norm = mix.output(mid, L, lins, self._allreduce), self._norm_of(L, "1b")
+        if mlp is not None:
+            if ff:
+                x, rows = self.norm_mod(x, y, norm, self._norm_of(L, "2"))
+                h = torch.empty(T, ff, dtype=self.dtype, device=self.device)
+                mlp(rows, L["up.w"], lins["up.w"], h)
+                y = self._allreduce(lins["down.w"](h, L["down.w"]))
+            else:
+                x, rows = self.norm_mod(x, y, norm, self._norm_of(L, "2"), pad=mlp.row_pad())
+                y = mlp(rows, L, self.tp_rank)
+                if self.tp > 1:
+                    y = self._allreduce(mlp.total(x, y))
+            norm = self._norm_of(L, "2b")
+        if self.spec.token_side:
+            x, rows = self.norm_mod(x, y, norm, None)
+            y, norm = self._side(i, rows, batch), L["side.norm.w"]
+        return x, y, norm
+
+    def _side(self, i, rows, batch):
+        """The layer's own input of every token, gated by the residual."""
+        L, lins, n = self.layers[i], self.linears[i], self.spec.token_side
+        g = act_gather(lins["side.gate.w"](rows, L["side.gate.w"]), "gelu_tanh", self.side_embed[:, i * n:(i + 1) * n],
+                       batch.input_ids)
+        return lins["side.proj.w"](g, L["side.proj.w"])
+
+
+class MemorySandwichTransformer(SandwichTransformer):
+    """The same layers on layer norms, with matrix memories and parallel mixers (the kernels it runs on are others)."""
+    KERNEL_SOURCES = ("act.hip", "experts.hip", "gemv.hip", "grouped_gemm.hip", "head_prep.hip", "matrix_memory.hip",
+                      "output_norm.hip", "paged_attn.hip", "paged_rows.hip")

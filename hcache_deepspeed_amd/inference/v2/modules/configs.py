@@ -79,6 +79,8 @@ class DSExpertLayerConfig:
     shared_features: int = 0  # 0: no shared expert
     tp: int = 1
     input_dtype: torch.dtype = torch.bfloat16
+    activation: str = "silu"  # or "clamped"
+    limit: float = 0.0        # of the activation "clamped"
 
 
 @dataclass

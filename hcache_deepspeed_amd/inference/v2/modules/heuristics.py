@@ -73,7 +73,8 @@ def instantiate_output_norm(config: DSNormConfig, engine_config=None):
 
 
 def instantiate_sandwich_norm(config: DSNormConfig, engine_config=None):
-    return DSSandwichNormRegistry.instantiate_config(ConfigBundle("rms_sandwich", config))
+    return DSSandwichNormRegistry.instantiate_config(ConfigBundle("ln_sandwich" if config.type == "layer" else "rms_sandwich",
+                                                                   config))
 
 
 def instantiate_expert_layer(config: DSExpertLayerConfig, engine_config=None):

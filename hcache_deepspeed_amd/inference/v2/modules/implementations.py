@@ -21,13 +21,16 @@ from ....ops.gemv import glu_gemv
 from ....ops.grouped_gemm import moe_ffn_dropless
 from ....ops.input_norm import input_norm
 from ....ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
+from ....ops.matrix_memory import MemoryShape, make_memory_plan, matrix_memory
+from ....ops.matrix_memory import step_ok as memory_step_ok
 from ....ops.moe import moe_combine, moe_dispatch, topk_assign, topk_route
 from ....ops.norm import layer_norm, rms_norm
-from ....ops.output_norm import (embed_rows, padded, residual_norm, rms_rows, sandwich_norm, softcap_,
-                                 sum_experts)
-from ....ops.paged import (HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
+from ....ops.output_norm import (PairSum, embed_rows, padded, residual_norm, rms_rows, sandwich_norm, softcap_,
+                                 stream_norm, sum_experts)
+from ....ops.paged import (HeadPrep, HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
                            paged_attention)
 from ....ops.quantizer import fp6_linear, int_linear, quantize, quantize_minifloat
+from ....ops.rope import rope_tables
 from .interfaces import (DSEmbeddingBase, DSEmbeddingRegistry, DSExpertLayerBase, DSExpertLayerRegistry, DSGatedMLPBase,
                          DSGatedMLPRegistry, DSInputNormBase, DSInputNormRegistry, DSLinearBase, DSLinearRegistry,
                          DSMixerBase, DSMixerRegistry, DSMoEBase, DSMoERegistry, DSOutputNormBase, DSOutputNormRegistry,
@@ -370,6 +373,21 @@ class MinGRUMixer(DSMixerBase):
         return gated_scan(lin(x, w["in.w"]), w["z.b"], w["x.b"], out, batch, state, offset)
 
 
+def _pair_order(rot_dims, dim):
+    """Dimensions of a head whose halves i and i + rot_dims / 2 turn together, in the order the kernels turn them in."""
+    return [i for j in range(rot_dims // 2) for i in (j, j + rot_dims // 2)] + list(range(rot_dims, dim))
+
+
+def _lone_plan(kind, batch, single, make):
+    """The batch's plan of lone tokens and portions for a kind of recurrence (shared by layers of the same answer)."""
+    key = (kind, single)
+    plan = batch.plans.get(key)
+    if plan is None:
+        plan = batch.plans[key] = make(batch.seq_meta_host, batch.current_sequences, batch.max_new, single,
+                                       batch.tok_pos.device)
+    return plan
+
+
 @DSMixerRegistry.register_module
 class LatentAttentionMixer(DSMixerBase):
     """Attention over compressed K/V rows, sliding window, rotation of a shared key part, optionally queries through a
@@ -402,14 +420,13 @@ class LatentAttentionMixer(DSMixerBase):
 
     def _turned(self, w):
         """w [..., rot, in]: the rotated rows in the kernels' order."""
-        n = self.shape.rot_dims
-        if not self.half:
-            return w
-        order = [i for j in range(n // 2) for i in (j, j + n // 2)] + list(range(n, self.shape.rot))
-        return w[..., order, :]
+        return w[..., _pair_order(self.shape.rot_dims, self.shape.rot), :] if self.half else w
 
     def bind_tables(self, cos, sin):
         self.cos, self.sin = cos, sin
+
+    def bind_positions(self, positions, device):
+        self.bind_tables(*rope_tables(positions, self.shape.rot_dims, self.rope_base, self.rope_scaling, device=device))
 
     def shard(self, w, rows, cols):
         # q, uk, uv and the gate are laid out head by head: equal row slices are whole heads
@@ -459,10 +476,12 @@ class LatentAttentionMixer(DSMixerBase):
 
 @DSMixerRegistry.register_module
 class HeadAttentionMixer(DSMixerBase):
-    """Grouped-query attention without rotation: sliding window or chunks, soft cap, optional query / key norms, sink (learned
-    or of score zero), output gate per head or element, and values mixed with those of an earlier layer (``value_mix``:
-    "source" leaves its values for the later ones of the step, "mix" takes them). ops/paged.py ``head_attention``. Heads
-    are sharded over the tensor-parallel group."""
+    """Grouped-query attention: sliding window (the sequence's first ``keep`` tokens stay visible) or chunks, soft cap, sink
+    (learned or of score zero), output gate per head or element, and values mixed with those of an earlier layer
+    (``value_mix``: "source" leaves its values for the later ones of the step, "mix" takes them). Queries and keys are normed
+    head by head, if at all; or, with ``conv`` in the parameters, convolved over a few tokens, normed across all heads
+    (``norm_all``) and rotated (``rot_dims``, neighbouring pairs), and the keys as convolved may be the values
+    (``shared_values``). ops/paged.py ``head_attention``. Heads are sharded over the tensor-parallel group."""
 
     @staticmethod
     def name():
@@ -476,22 +495,40 @@ class HeadAttentionMixer(DSMixerBase):
         self.shape = HeadShape(heads=p["heads"] // tp, kv_heads=p["kv_heads"] // tp, dim=p["dim"], vdim=p["vdim"],
                                window=p["window"], scale=p["scale"], eps=config.eps, gated=p["gated"],
                                gate_width=p["vdim"] if p.get("gate_elements") else 1, chunk=p.get("chunk", 0),
-                               softcap=p.get("softcap", 0.0))
+                               softcap=p.get("softcap", 0.0), keep=p.get("keep", 0), prep="conv" in p,
+                               taps=p.get("conv", 1), rot=p.get("rot_dims", 0), shared=p.get("shared_values", False))
+        self.norm_all = p.get("norm_all", False)
+        self.rope_base, self.rope_scaling = p.get("rope_base"), p.get("rope_scaling")
+        self.tables = self.reduce = None
         self.value_mix = p.get("value_mix")
         self.zero_sink = p.get("zero_sink", False)
         self.out_width = self.shape.heads * p["vdim"]
         self.in_width = padded(self.shape.width, 8)  # 16-byte rows
         self.cache_row = self.shape.row
 
+    def state_floats(self):
+        return padded(self.shape.state_floats, 4)
+
+    def bind_positions(self, positions, device):
+        if self.shape.rot:
+            self.tables = rope_tables(positions, self.shape.rot, self.rope_base, self.rope_scaling, device=device)
+
+    def bind_group(self, reduce):
+        self.reduce = reduce
+
     def shard(self, w, rows, cols):
-        # q, k, v, g and the sink are laid out head by head: equal slices are whole heads
-        parts = [rows(w[k]) for k in (("q", "k", "v", "g") if self.shape.gated else ("q", "k", "v"))]
+        # q, k, v, g, convolutions, norms across heads and the sink are laid out head by head: equal slices are whole heads
+        names = ["q", "k"] + (["v"] if not self.shape.shared else []) + (["g"] if self.shape.gated else [])
+        parts = [rows(w[k]) for k in names]
         fill = self.in_width - self.shape.width
         if fill:
             parts.append(parts[0].new_zeros(fill, parts[0].shape[1]))
         out = {"in.w": torch.cat(parts), "o.w": cols(w["o"])}
         for k in ("q.norm", "k.norm"):
-            out[k] = w[k].float() if k in w else None
+            out[k] = (rows(w[k]) if self.norm_all else w[k]).float() if k in w else None
+        if self.shape.prep:
+            conv = [w.get("q.conv"), w.get("k.conv")]
+            out["conv.w"] = None if conv[0] is None else torch.cat([rows(c) for c in conv]).float().t().contiguous()
         out["sink"] = rows(w["sink"]).float() if "sink" in w else None
         if self.zero_sink:
             out["sink"] = torch.zeros(self.shape.heads)
@@ -518,6 +555,14 @@ class HeadAttentionMixer(DSMixerBase):
             qkv, gate = lin(x, in_w[:n]), lin(x, in_w[n:sh.width])
         else:
             qkv = lin(x, in_w)
+        return self.mix(qkv, w, out, batch, cache, state, offset, gate)
+
+    def mix(self, qkv, w, out, batch, cache, state, offset, gate=None):
+        """The projected rows (``gate``: without the gates) -> the heads' outputs."""
+        sh = self.shape
+        if sh.prep:
+            prep = HeadPrep(w["conv.w"], w["q.norm"], w["k.norm"], self.tables, state, offset, self._config.tp, self.reduce)
+            return head_attention(qkv, sh, None, None, w["sink"], cache, batch, self._plan(batch), out, gate=gate, prep=prep)
         own = qkv[:, sh.qkv_width - sh.kv_heads * sh.vdim:sh.qkv_width]
         if self.value_mix == "source":
             batch.carry["values"] = own
@@ -558,13 +603,7 @@ class DeltaMixer(DSMixerBase):
                 "A_log": rows(w["A_log"]).float(), "dt_bias": rows(w["dt_bias"]).float(), "norm": w["norm"].float()}
 
     def _plan(self, batch):
-        single = batch.tok_pos.is_cuda and step_ok(self.shape)
-        key = ("delta", single)
-        plan = batch.plans.get(key)
-        if plan is None:
-            plan = batch.plans[key] = make_delta_plan(batch.seq_meta_host, batch.current_sequences, batch.max_new, single,
-                                                      batch.tok_pos.device)
-        return plan
+        return _lone_plan("delta", batch, batch.tok_pos.is_cuda and step_ok(self.shape), make_delta_plan)
 
     def forward(self, x, w, lins, out, batch, cache, state, offset):
         sh, lin, in_w, T = self.shape, lins["in.w"], w["in.w"], x.shape[0]
@@ -576,6 +615,167 @@ class DeltaMixer(DSMixerBase):
             proj = lin(x, in_w)
         return delta_rule(proj, sh, w["conv.w"], w["A_log"], w["dt_bias"], w["norm"], state, offset, batch,
                           self._plan(batch), out, ba)
+
+
+class _MatrixMemoryMixer(DSMixerBase):
+    """Linear attention with a decaying matrix state per head (ops/matrix_memory.py). Heads are sharded over the
+    tensor-parallel group. The kernels turn neighbouring dimensions; the "half" rotation becomes that by reordering the
+    rotated rows of the query and key weights."""
+
+    def _init(self, **kind):
+        p, c = self._config.params, self._config
+        if p["heads"] % c.tp:
+            raise ValueError(f"{p['heads']} heads: not groups of equal size on {c.tp} ranks")
+        self.shape = MemoryShape(heads=p["heads"] // c.tp, dim=p["dim"], vdim=p["vdim"], eps=c.eps,
+                                 rot=p.get("rot_dims", 0), **kind)
+        self.half = p.get("rot_layout", "interleaved") == "half"
+        self.rope_base, self.rope_scaling = p.get("rope_base"), p.get("rope_scaling")
+        self.out_width = self.shape.heads * self.shape.vdim
+        self.in_width = padded(self.shape.width, 8)
+        self.tables = None
+
+    def state_floats(self):
+        return padded(self.shape.state_floats, 4)
+
+    def bind_positions(self, positions, device):
+        if self.shape.rot:
+            self.tables = rope_tables(positions, self.shape.rot, self.rope_base, self.rope_scaling, device=device)
+
+    def _turned(self, w):
+        """w [heads * dim, in]: the rotated rows of every head in the kernels' order."""
+        sh = self.shape
+        if not (sh.rot and self.half):
+            return w
+        return w.reshape(sh.heads, sh.dim, -1)[:, _pair_order(sh.rot, sh.dim)].reshape(sh.heads * sh.dim, -1)
+
+    def _extra(self, w, rows):
+        """Further weights, and the rows of the input projection behind the output gate."""
+        raise NotImplementedError
+
+    def shard(self, w, rows, cols):
+        # everything is laid out head by head: equal slices are whole heads
+        extra, gates = self._extra(w, rows)
+        parts = [self._turned(rows(w["q"])), self._turned(rows(w["k"])), rows(w["v"]), rows(w["g"])] + gates
+        fill = self.in_width - self.shape.width
+        if fill:
+            parts.append(parts[0].new_zeros(fill, parts[0].shape[1]))
+        return {"in.w": torch.cat(parts), "o.w": cols(w["o"]), **extra}
+
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
+        return self.mix(lins["in.w"](x, w["in.w"]), w, out, batch, cache, state, offset)
+
+    def mix(self, proj, w, out, batch, cache, state, offset):
+        """The projected rows -> the heads' outputs."""
+        plan = _lone_plan("memory", batch, batch.tok_pos.is_cuda and memory_step_ok(self.shape), make_memory_plan)
+        return matrix_memory(proj, self.shape, w, self.tables, state, offset, batch, plan, out)
+
+
+@DSMixerRegistry.register_module
+class MLSTMMixer(_MatrixMemoryMixer):
+    """Exponential input and forget gates with soft caps, a normalizer, a norm weight across all heads, a sigmoid gate."""
+
+    @staticmethod
+    def name():
+        return "mlstm"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        self._init(gate="sigmoid", gated=True, cap=config.params["cap"])
+
+    def _extra(self, w, rows):
+        extra = {"norm": rows(w["norm"]).float(), "i.b": rows(w["i.b"]).float(), "f.b": rows(w["f.b"]).float()}
+        return extra, [rows(w["i"]), rows(w["f"])]
+
+
+@DSMixerRegistry.register_module
+class RetentionMixer(_MatrixMemoryMixer):
+    """A fixed decay per head, rotated queries and keys, a norm without weights, a SiLU gate."""
+
+    @staticmethod
+    def name():
+        return "retention"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        self._init(gate="silu", gated=False)
+
+    def _extra(self, w, rows):
+        decay = torch.tensor(self._config.params["decay"], dtype=torch.float64).clamp(min=1e-38)
+        return {"log_decay": rows(decay.log().float()), "norm": None}, []
+
+
+class _Part:
+    """The entries of a layer's weights that share a prefix."""
+
+    def __init__(self, w, prefix):
+        self.w, self.prefix = w, prefix
+
+    def __getitem__(self, k):
+        return self.w[self.prefix + k]
+
+
+@DSMixerRegistry.register_module
+class ParallelMixer(DSMixerBase):
+    """Two mixers that read the same rows: one input projection, an output projection each, and the mean of both outputs,
+    each RMS-normed over the model width."""
+    own_output = True
+    SIDES = ("left", "right")
+
+    @staticmethod
+    def name():
+        return "parallel"
+
+    def __init__(self, config, implementation_config=None):
+        super().__init__(config, implementation_config)
+        c = config
+        self.parts = []
+        for side in self.SIDES:
+            p = c.params[side]
+            cls = DSMixerRegistry.registry[p["type"]]
+            self.parts.append(cls(type(c)(p["type"], c.model_dim, p, c.eps, c.tp, c.input_dtype), implementation_config))
+        self.in_width = sum(m.in_width for m in self.parts)
+        self.out_width = sum(m.out_width for m in self.parts)
+        if sum(m.cache_row > 0 for m in self.parts) > 1:
+            raise NotImplementedError("two cached mixers side by side")
+        self.cache_row = sum(m.cache_row for m in self.parts)
+
+    def state_floats(self):
+        return sum(m.state_floats() for m in self.parts)
+
+    def bind_positions(self, positions, device):
+        for m in self.parts:
+            m.bind_positions(positions, device)
+
+    def bind_group(self, reduce):
+        for m in self.parts:
+            m.bind_group(reduce)
+
+    def extra_linears(self):
+        return {f"{s}.o.w": (m.out_width, self._config.model_dim) for s, m in zip(self.SIDES, self.parts)}
+
+    def shard(self, w, rows, cols):
+        out, ins = {}, []
+        for side, m in zip(self.SIDES, self.parts):
+            own = m.shard({k[len(side) + 1:]: v for k, v in w.items() if k.startswith(side + ".")}, rows, cols)
+            ins.append(own.pop("in.w"))
+            out.update({f"{side}.{k}": v for k, v in own.items()})
+            out[f"{side}.out"] = w[side + ".out"].float()
+        return {"in.w": torch.cat(ins), **out}
+
+    def forward(self, x, w, lins, out, batch, cache, state, offset):
+        y = lins["in.w"](x, w["in.w"])
+        i = o = 0
+        for side, m in zip(self.SIDES, self.parts):
+            m.mix(y[:, i:i + m.in_width], _Part(w, side + "."), out[:, o:o + m.out_width], batch,
+                  cache if m.cache_row else None, state, offset)
+            i, o, offset = i + m.in_width, o + m.out_width, offset + m.state_floats()
+
+    def output(self, mid, w, lins, reduce):
+        y, o = [], 0
+        for side, m in zip(self.SIDES, self.parts):
+            y.append(reduce(lins[f"{side}.o.w"](mid[:, o:o + m.out_width], w[f"{side}.o.w"])))
+            o += m.out_width
+        return PairSum(*y, w["left.out"], w["right.out"])
 
 
 @DSOutputNormRegistry.register_module
@@ -612,13 +812,33 @@ class RmsSandwich(DSSandwichNormBase):
     def supports_config(c):
         return c.type == "rms"
 
-    def forward(self, x, delta, gain, next_gain, embed=None, idx=None):
-        return sandwich_norm(x, delta, gain, next_gain, self._config.eps, self._config.input_dtype, embed, idx)
+    def forward(self, x, delta, norm, next_norm, embed=None, idx=None, pad=1):
+        assert pad == 1
+        return sandwich_norm(x, delta, norm, next_norm, self._config.eps, self._config.input_dtype, embed, idx)
+
+
+@DSSandwichNormRegistry.register_module
+class LnSandwich(DSSandwichNormBase):
+    """32-bit residual, layer norms on both sides of every sublayer (RMS norms where only a gain is given)."""
+
+    @staticmethod
+    def name():
+        return "ln_sandwich"
+
+    @staticmethod
+    def supports_config(c):
+        return c.type == "layer"
+
+    def forward(self, x, delta, norm, next_norm, embed=None, idx=None, pad=1):
+        dt = self._config.input_dtype
+        if x is None:
+            x = embed_rows(*embed, dt)[0]
+        return stream_norm(x, delta, norm, next_norm, self._config.eps, dt, idx, pad)
 
 
 @DSExpertLayerRegistry.register_module
 class RoutedExperts(DSExpertLayerBase):
-    """Group-limited top-k experts with identity experts and a gated shared expert (ops/experts.py). Every expert's
+    """Top-k experts, optionally limited to groups, with identity experts and a gated shared expert (ops/experts.py). Every expert's
     feed-forward width is sharded over the tensor-parallel group; bf16 weights are zero-padded to the products' tile."""
 
     @staticmethod
@@ -630,6 +850,10 @@ class RoutedExperts(DSExpertLayerBase):
         config.router.check()
         if config.intermediate_features % config.tp or config.shared_features % config.tp:
             raise ValueError("the experts' widths must divide the tensor-parallel size")
+
+    def row_pad(self):
+        """What the length of the rows it reads has to be a multiple of."""
+        return PAD if self._config.input_dtype == torch.bfloat16 else 1
 
     def _fit(self, w):
         """w zero-padded at the end of its last two dimensions."""
@@ -647,13 +871,15 @@ class RoutedExperts(DSExpertLayerBase):
         fit, shared = self._fit, self._config.shared_features > 0
         router = torch.cat([w["router"], w["shared.sg"]]) if shared else w["router"]
         n = router.shape[0]
-        return {"router.w": fit(router)[:n], "router.c": w["correction"].float(),
+        correction = w["correction"].float() if "correction" in w else None
+        return {"router.w": fit(router)[:n], "router.c": correction,
                 "w13": self._gate_up(w["gate"], w["up"], rows), "w2": fit(cols(w["down"])),
                 "ws13": self._gate_up(w["shared.gate"], w["shared.up"], rows) if shared else None,
                 "ws2": fit(cols(w["shared.down"])) if shared else None}
 
     def forward(self, x, w, rank=0):
-        return routed_experts(x, w, self._config.router, identity=rank == 0)
+        c = self._config
+        return routed_experts(x, w, c.router, identity=rank == 0, act=c.activation, limit=c.limit)
 
     def total(self, x32, parts):
         return sum_experts(x32, parts, self._config.input_dtype)

@@ -42,14 +42,27 @@ class DSMixerBase(DSModuleBase):
     the paged cache; ``state_floats()``: unpaged float32 state per sequence; ``shard(weights, rows, cols)`` -> this
     rank's weights, with the input projection "in.w" and the output projection "o.w"; ``extra_linears()``: further
     products, name -> (in, out); forward(x, weights, lins, out, batch, cache, state, offset) fills ``out`` [T, out_width],
-    ``lins`` holds the linear modules by weight name, ``batch.carry`` what layers of a step hand to later ones."""
+    ``lins`` holds the linear modules by weight name, ``batch.carry`` what layers of a step hand to later ones.
+    ``bind_positions(n, device)``: tables for n positions; ``output(mid, weights, lins, reduce)``: what the layer's norm reads
+    (``reduce`` sums a product over the tensor-parallel group). A mixer of its own products (``own_output``) has no "o.w".
+    ``bind_group(reduce)``: the same sum, for what a mixer adds up over the group inside."""
     cache_row = 0
+    own_output = False
 
     def state_floats(self):
         return 0
 
     def extra_linears(self):
         return {}
+
+    def bind_positions(self, positions, device):
+        pass
+
+    def bind_group(self, reduce):
+        pass
+
+    def output(self, mid, w, lins, reduce):
+        return reduce(lins["out.w"](mid, w["out.w"]))
 
 
 class DSOutputNormBase(DSModuleBase):
@@ -58,8 +71,9 @@ class DSOutputNormBase(DSModuleBase):
 
 
 class DSSandwichNormBase(DSModuleBase):
-    """forward(x32, delta, gain, next_gain, embed, idx) -> (x32 + gain * norm(delta), next_gain * norm(of that)); x32 None:
-    the stream starts from ``embed`` (table, ids, scale); ``idx``: the second result of these rows only."""
+    """forward(x32, delta, norm, next_norm, embed, idx, pad) -> (x32 + norm(delta), next_norm(of that)); a norm is a gain, or
+    (gain, bias) of a layer norm; x32 None: the stream starts from ``embed`` (table, ids, scale); ``idx``: the second result
+    of these rows only; ``pad``: its rows zero-padded to a multiple of this."""
 
 
 class DSExpertLayerBase(DSModuleBase):

@@ -177,6 +177,21 @@ def clamped_unit(g, u, limit):
     return g * torch.sigmoid(1.702 * g) * (u + 1)
 
 
+def act_gather(x, act, table, ids):
+    """act(x) * table[ids] of rows [T, C] (any row strides), contiguous. ids: int64."""
+    T, C = x.shape
+    a = act_code(act)
+    y = torch.empty(T, C, dtype=x.dtype, device=x.device)
+    if native.use_native(x):
+        assert x.stride(1) == 1 and table.stride(1) == 1 and table.dtype == x.dtype and table.shape[1] == C
+        assert ids.dtype == torch.int64 and ids.numel() == T
+        native.check(native.kernels().hds_act_gather(native.dt(x), a, x.data_ptr(), x.stride(0), table.data_ptr(),
+                                                     table.stride(0), ids.data_ptr(), y.data_ptr(), C, T, C,
+                                                     table.shape[0], native.stream()), "act_gather")
+        return y
+    return y.copy_(_ref_act(x.float(), a) * table[ids].float())
+
+
 def glu_rows(gu, act, out, limit=0.0):
     """``glu`` without autograd into ``out`` [T, I], a (possibly strided) column block; any width. ``act`` "clamped":
     ``clamped_unit`` with ``limit``."""

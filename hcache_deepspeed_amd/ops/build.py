@@ -43,7 +43,8 @@ FILE_FLAGS = {"flash_attn.hip": ["-fno-slp-vectorize"],
               "flash_attn_w64.hip": ["-fno-slp-vectorize", "-mllvm", "-amdgpu-mfma-vgpr-form"],
               "flash_attn_bwd_w64.hip": ["-fno-slp-vectorize", "-mllvm", "-amdgpu-mfma-vgpr-form"],
               # the chunk scan works on its accumulators with vector instructions too: no moves from and to AGPRs
-              "delta_rule.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
+              "delta_rule.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
+              "matrix_memory.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
 HOST_FLAGS = ["-O3", "-fPIC", "-std=c++17", "-fopenmp", "-D__HIP_PLATFORM_AMD__", f"-I{ROCM}/include",
               "-Wall", "-Wno-unused-function", "-Wno-unused-variable"]
 

@@ -30,18 +30,26 @@ _KERNEL_SIGS = {
     "hds_input_norm": "i" + "ppppp" + "pipp" + "pipp" + "p" + "l" + "pp" + "iiiii" + "f" + "s",
     "hds_residual_norm": "i" + "ppp" + "l" + "pl" + "p" + "ii" + "f" + "s",
     "hds_sandwich_norm": "i" + "ppp" + "f" + "pl" + "ppppp" + "iii" + "f" + "s",
+    "hds_stream_norm": "ii" + "p" + "pl" + "pl" + "pp" + "pl" + "ppp" + "pl" + "pl" + "iii" + "pppp" + "pp" + "pl" + "ii" + "f" + "s",
+    "hds_embed_pairs": "i" + "ppp" + "f" + "pppp" + "l" + "p" + "iiii" + "ll" + "s",
+    "hds_act_gather": "ii" + "pl" + "pl" + "p" + "pl" + "l" + "ii" + "s",
+    "hds_memory_step_ok": "ii",
+    "hds_memory_chunk_floats": "iiii",
+    "hds_memory_chunk_tokens": "",
+    "hds_memory": "ii" + "pl" + "ppp" + "f" + "pp" + "i" + "p" + "i" + "pl" + "ppp" + "ppp" + "pl" + "ii" + "iii" + "f" + "s",
+    "hds_head_prep": "i" + "pl" + "i" * 7 + "ppppp" + "pl" + "pp" + "ii" + "ppp" + "pl" + "ppp" + "ii" + "f" + "iii" + "s",
     "hds_row_norm": "i" + "pl" + "ppl" + "ii" + "f" + "s",
     "hds_softcap": "i" + "p" + "l" + "f" + "s",
     "hds_experts_norm": "i" + "ppp" + "l" + "pp" + "pl" + "ppp" + "pl" + "pl" + "iiiii" + "f" + "s",
     "hds_embed_rows": "i" + "pp" + "f" + "pp" + "l" + "iii" + "s",
     "hds_router_logits": "pl" + "p" + "pl" + "iii" + "s",
-    "hds_router_select": "pl" + "ppp" + "iiiii" + "f" + "s",
-    "hds_expert_sort": "p" + "iii" + "ppp" + "i" + "ppp" + "i" + "s",
+    "hds_router_select": "pl" + "i" + "ppp" + "iiiii" + "f" + "s",
+    "hds_expert_sort": "p" + "iii" + "ppppp" + "i" + "ppp" + "i" + "s",
     "hds_experts_skinny_max": "",
-    "hds_experts_skinny": "i" + "pl" + "p" + "pl" + "p" + "iiiii" + "pl" + "p" + "pl" + "iii" + "s",
-    "hds_experts_gemm_f32": "pl" + "p" + "pl" + "ppppp" + "iiii" + "s",
+    "hds_experts_skinny": "i" + "pl" + "p" + "pl" + "p" + "iiiii" + "pl" + "p" + "pl" + "iii" + "i" + "f" + "p" + "s",
+    "hds_experts_gemm_f32": "pl" + "p" + "pl" + "ppppp" + "i" + "p" + "iii" + "s",
     "hds_experts_gemm_tile": "iii",
-    "hds_experts_gemm": "pl" + "pi" + "pp" + "i" + "pppp" + "iiiiiii" + "s",
+    "hds_experts_gemm": "pl" + "pi" + "pp" + "i" + "pppp" + "iiiiiii" + "i" + "f" + "p" + "s",
     "hds_norm_rows": "i" + "pppp" + "i" + "p" + "ii" + "f" + "s",
     "hds_gated_scan": "i" + "pl" + "pp" + "pl" + "pl" + "pp" + "iii" + "s",
     "hds_delta_step_ok": "ii",
@@ -86,7 +94,7 @@ _KERNEL_SIGS = {
     "hds_head_norm_scatter": "i" + "pl" + "pppppp" + "iiiiiii" + "f" + "plp" + "s",
     "hds_paged_rows": "ii" + "ppl" + "pppp" + "iiii" + "s",
     "hds_paged_attn_supported": "ii",
-    "hds_paged_attn": "pl" + "p" + "pl" + "pi" + "pp" + "i" * 6 + "f" + "ii" + "f" + "pp" + "li" + "s",
+    "hds_paged_attn": "pl" + "p" + "pl" + "pi" + "pp" + "i" * 6 + "f" + "iii" + "f" + "pp" + "li" + "s",
     "hds_paged_rows_per_atom": "",
     "hds_moe_dispatch": "i" + "pppp" + "iiii" + "s",
     "hds_moe_dispatch_bwd": "i" + "pppp" + "iiii" + "s",
@@ -133,7 +141,7 @@ _KERNEL_SIGS = {
     "hds_nhwc_bias_add": "i" + "ppppp" + "l" + "ii" + "s",
     "hds_paged_decode_supported": "ii",
     "hds_paged_decode_splits": "iii",
-    "hds_paged_decode": "ii" + "pl" + "p" + "pl" + "pp" + "ppppp" + "i" * 8 + "f" + "ii" + "f" + "pp" + "li" + "p" + "s",
+    "hds_paged_decode": "ii" + "pl" + "p" + "pl" + "pp" + "ppppp" + "i" * 8 + "f" + "iii" + "f" + "pp" + "li" + "p" + "s",
     "hds_copy_d2h": "pp" + "l" + "i" + "s",
     "hds_latent_slot_store": "p" + "l" + "pp" + "l" + "i" + "l" + "s",
     "hds_slot_advance": "p" + "i" + "s",

@@ -4,9 +4,12 @@
 plain matrix or an :class:`ops.experts.ExpertSum`, the parts of a routed expert layer's output, which the kernel sums on
 the way in. It returns the new residual and the rows the next sublayer reads: rounded to the activations' type and
 zero-padded to a multiple of ``pad`` columns (the 32-bit rows themselves where that changes nothing). ``embed_rows``
-starts the stream, ``norm_rows`` is the output norm of selected rows. ``sandwich_norm`` is the step between two sublayers
-with a norm on both sides: the residual sum of the first one's normed output and the second one's norm in one kernel.
+and ``embed_pairs`` start the stream, ``norm_rows`` is the output norm of selected rows. ``sandwich_norm`` is the step between two sublayers
+with a norm on both sides: the residual sum of the first one's normed output and the second one's norm in one kernel;
+``stream_norm`` is its general form (layer norms, a :class:`PairSum` or an ExpertSum as the output, no second norm, padded rows).
 ``rms_rows`` norms column blocks, ``softcap_`` bounds logits. CPU tensors run the torch implementations."""
+from dataclasses import dataclass
+
 import torch
 
 from . import native
@@ -86,7 +89,7 @@ def _experts_norm(x, xb, ld, gain, out, p, eps):
     native.check(
         native.kernels().hds_experts_norm(
             native.dt(p.y), x.data_ptr(), x.data_ptr(), native.ptr(xb), ld, native.ptr(gain), native.ptr(out),
-            p.y.data_ptr(), p.y.stride(0), p.expert.data_ptr(), p.weight.data_ptr(), native.ptr(p.row), native.ptr(sh),
+            p.y.data_ptr(), p.y.stride(0), p.expert.data_ptr(), native.ptr(p.weight), native.ptr(p.row), native.ptr(sh),
             0 if sh is None else sh.stride(0), None if sh is None else p.gate.data_ptr(),
             0 if sh is None else p.gate.stride(0), p.n_experts, p.expert.shape[1], int(p.identity), T, W, float(eps),
             native.stream()), "experts_norm")
@@ -112,6 +115,107 @@ def norm_rows(x, delta, idx, gain, eps, dtype=None):
 
 def _rms(x, eps):
     return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+
+@dataclass
+class PairSum:
+    """(ga * rms(a) + gb * rms(b)) / 2: two outputs of one sublayer, each normed by itself. a, b: [T, W]; gains: [W] float32."""
+    a: torch.Tensor
+    b: torch.Tensor
+    ga: torch.Tensor
+    gb: torch.Tensor
+
+    def total(self, eps):
+        return 0.5 * (self.ga * _rms(self.a.float(), eps) + self.gb * _rms(self.b.float(), eps))
+
+
+def _normed(x, norm, eps):
+    """norm: an RMS norm's gain, or (gain, bias) of a layer norm."""
+    if torch.is_tensor(norm):
+        return norm * _rms(x, eps)
+    d = x - x.mean(-1, keepdim=True)
+    return norm[0] * _rms(d, eps) + norm[1]
+
+
+def stream_norm(x, delta, norm, next_norm, eps, dtype, idx=None, pad=1):
+    """(x' = x + norm(delta), next_norm(x') in ``dtype``, zero-padded to a multiple of ``pad`` columns). x: [T, W] float32,
+    updated in place; delta: [T, W] of ``dtype``, a PairSum, an ExpertSum or None (x' = x). A norm is the gain [W] of an
+    RMS norm or (gain, bias) of a layer norm, float32; next_norm None: the rows of x' themselves. ``idx`` (int32): only these
+    rows, and the first result is None."""
+    W = x.shape[1]
+    n = x.shape[0] if idx is None else idx.numel()
+    ld = padded(W, pad)
+    same = next_norm is None and idx is None and dtype == torch.float32 and ld == W  # x' serves as the rows
+    y = None if same else torch.empty(n, ld, dtype=dtype, device=x.device)
+    pair = isinstance(delta, PairSum)
+    plain = delta is None or torch.is_tensor(delta)
+    if native.use_native(x):
+        if same and delta is None:
+            return x, x
+        assert x.is_contiguous() and x.dtype == torch.float32
+
+        def split(m):
+            w, b = (m, None) if m is None or torch.is_tensor(m) else m
+            assert all(v is None or (v.numel() == W and v.dtype == torch.float32) for v in (w, b))
+            return native.ptr(w), native.ptr(b)
+
+        first, other = (delta.a, delta.b) if pair else (delta if plain else None, None)
+        for v in (first, other):
+            assert v is None or (v.dtype == dtype and v.stride(1) == 1 and v.shape[1] == W and v.shape[0] == x.shape[0])
+        parts = [None, 0] + [None] * 4 + [0, None, 0, 0, 0, 0]
+        if not (plain or pair):
+            sh = delta.shared
+            assert delta.y.dtype == dtype and delta.expert.shape[0] == x.shape[0]
+            parts = [delta.y.data_ptr(), delta.y.stride(0), delta.expert.data_ptr(), native.ptr(delta.weight),
+                     native.ptr(delta.row), native.ptr(sh), 0 if sh is None else sh.stride(0),
+                     None if sh is None else delta.gate.data_ptr(), 0 if sh is None else delta.gate.stride(0),
+                     delta.n_experts, delta.expert.shape[1], int(delta.identity)]
+        native.check(
+            native.kernels().hds_stream_norm(
+                native.dt(dtype), 0 if plain else (1 if pair else 2), x.data_ptr(), native.ptr(first),
+                0 if first is None else first.stride(0), native.ptr(other), 0 if other is None else other.stride(0),
+                native.ptr(delta.ga if pair else None), native.ptr(delta.gb if pair else None), *parts, *split(norm),
+                *split(next_norm), native.ptr(idx), None if idx is not None or delta is None else x.data_ptr(),
+                native.ptr(y), ld, n, W, float(eps), native.stream()), "stream_norm")
+        return None if idx is not None else x, x if same else y
+    d = delta
+    if not plain:
+        d = delta.total(eps) if pair else delta.total(x)
+    h = x if idx is None else x[idx.long()]
+    if d is not None:
+        h = h + _normed((d if idx is None else d[idx.long()]).float(), norm, eps)
+    if idx is None:
+        x.copy_(h)
+    if same:
+        return x, x
+    return None if idx is not None else x, _fill(y, h if next_norm is None else _normed(h, next_norm, eps))
+
+
+def embed_pairs(embed, pairs, ids, scale, mul_prev, mul_cur, state, offset, batch):
+    """scale * embed[ids] + pairs[(previous id * mul_prev + id * mul_cur) mod buckets] in float32; pairs: [buckets + 1, W], its
+    last row for a sequence's first token. ``state[slot, offset]`` keeps a sequence's last token (as an int32)."""
+    n, W = ids.numel(), embed.shape[1]
+    buckets = pairs.shape[0] - 1
+    if native.use_native(embed):
+        x = torch.empty(n, W, dtype=torch.float32, device=embed.device)
+        assert embed.dtype == pairs.dtype and ids.dtype == torch.int64 and embed.is_contiguous() and pairs.is_contiguous()
+        native.check(
+            native.kernels().hds_embed_pairs(native.dt(embed), embed.data_ptr(), pairs.data_ptr(), ids.data_ptr(),
+                                             float(scale), batch.tok_seq.data_ptr(), batch.seq_meta.data_ptr(),
+                                             batch.slots.data_ptr(), state.data_ptr() + 4 * offset, state.stride(0),
+                                             x.data_ptr(), n, W, embed.shape[0], buckets, mul_prev, mul_cur,
+                                             native.stream()), "embed_pairs")
+        return x
+    at = torch.empty_like(ids)
+    last = state.view(torch.int32)[:, offset]
+    for s, (q0, k, seen) in enumerate(batch.seq_meta_host):
+        slot = batch.slots_host[s]
+        before = torch.cat([last[slot:slot + 1].long(), ids[q0:q0 + k - 1]])
+        at[q0:q0 + k] = (before * mul_prev + ids[q0:q0 + k] * mul_cur) % buckets
+        if seen == 0:
+            at[q0] = buckets
+        last[slot] = ids[q0 + k - 1].to(torch.int32)
+    return embed[ids].float() * scale + pairs[at].float()
 
 
 def sandwich_norm(x, delta, gain, next_gain, eps, dtype, embed=None, idx=None):

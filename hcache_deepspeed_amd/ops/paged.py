@@ -1,6 +1,7 @@
 """Paged-KV serving ops: fused RoPE + KV scatter, ragged paged attention (HIP, csrc/kernels/paged_attn.hip), and
-``head_attention``: attention with unrotated heads (optionally normed), a window or chunks, a soft cap, a sink, value mixing
-and an output gate over the same kernels.
+``head_attention``: attention with heads that are normed one by one and not rotated, or convolved, normed across the heads
+and rotated (csrc/kernels/head_prep.hip), with a window (and first tokens that stay visible) or chunks, a soft cap, a sink,
+value mixing and an output gate over the same kernels.
 
 Reference parity: inference/v2/kernels/ragged_ops/linear_blocked_kv_rotary (``LinearBlockedKVCopy``,
 ``BlockedRotaryEmbeddings``) and ragged_ops/blocked_flash (``BlockedFlashAttn``) + atom_builder.
@@ -124,13 +125,13 @@ def paged_attention(q, cache, atoms, n_atoms, seq_meta, block_tables, n_q, n_kv,
                 lib.hds_paged_decode(native.dt(q), 0, q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(),
                                      n_q * D, native.ptr(part_o), native.ptr(part_ml), seq_meta.data_ptr(), None, None,
                                      None, block_tables.data_ptr(), block_tables.shape[1], cache.shape[1], n_seqs, n_q,
-                                     n_kv, D, D, splits, float(scale), int(window), 0, 0.0, None, None, 0, 1, counters,
+                                     n_kv, D, D, splits, float(scale), int(window), 0, 0, 0.0, None, None, 0, 1, counters,
                                      native.stream()), "paged_decode")
             return o
         native.check(
             lib.hds_paged_attn(q.data_ptr(), q.stride(0), cache.data_ptr(), o.data_ptr(), n_q * D, atoms.data_ptr(),
                                n_atoms, seq_meta.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
-                               cache.shape[1], n_q, n_kv, D, D, float(scale), int(window), 0, 0.0, None, None, 0, 1,
+                               cache.shape[1], n_q, n_kv, D, D, float(scale), int(window), 0, 0, 0.0, None, None, 0, 1,
                                native.stream()), "paged_attn")
         return o
     meta = seq_meta_host if seq_meta_host is not None else seq_meta.tolist()
@@ -181,7 +182,7 @@ def copy_rows(cache, rows, seq, pos, tables, dst_row=None, to_cache=False):
 
 
 # -----------------------------------------------------------------------------------------------------------------
-# unrotated heads: norms, window, chunks, soft cap, sink, value mixing, output gate
+# heads with norms, convolutions, rotation, window, chunks, soft cap, sink, value mixing, output gate
 # -----------------------------------------------------------------------------------------------------------------
 @dataclass(frozen=True)
 class HeadShape:
@@ -196,6 +197,13 @@ class HeadShape:
     gate_width: int = 1   # .. or, vdim: one per element of the heads' outputs
     chunk: int = 0        # positions see their own run of this many, counted from the sequence's start; 0: no chunks
     softcap: float = 0.0  # 0: none
+    keep: int = 0         # of a window: the sequence's first positions, which stay visible
+    # between projection and attention (``head_prep``): a short convolution of q and k, norms over all heads of q (of k),
+    # rotation of the first ``rot`` dimensions of a head (neighbouring pairs); the keys as convolved may be the values
+    prep: bool = False
+    taps: int = 1
+    rot: int = 0
+    shared: bool = False
 
     @property
     def row(self):
@@ -204,12 +212,22 @@ class HeadShape:
     @property
     def span(self):
         """The most keys a position sees; 0: no bound."""
-        bounds = [b for b in (self.window, self.chunk) if b]
+        bounds = [b + self.keep for b in (self.window, self.chunk) if b]
         return min(bounds) if bounds else 0
 
     @property
+    def channels(self):
+        """q and k columns of the projection."""
+        return (self.heads + self.kv_heads) * self.dim
+
+    @property
     def qkv_width(self):
-        return self.heads * self.dim + self.row
+        return self.channels + (0 if self.shared else self.kv_heads * self.vdim)
+
+    @property
+    def state_floats(self):
+        """The convolution's last inputs, a ring [taps, channels]: the input of position p is entry p % taps."""
+        return self.taps * self.channels if self.taps > 1 else 0
 
     @property
     def width(self):
@@ -259,29 +277,127 @@ def head_blocks_ok(shape, dtype):
     return dtype == torch.bfloat16 and bool(native.kernels().hds_paged_attn_supported(shape.dim, shape.vdim))
 
 
-def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, values=None, mix=None, gate=None):
+@dataclass
+class HeadPrep:
+    """What ``head_prep`` works with. conv: [taps, channels] float32, the last row is the current token's, or None; norms:
+    [heads * dim] and [kv_heads * dim] float32, or None; tables: (cos, sin) [positions, rot / 2] or None;
+    ``state[slot, offset:]`` is read and advanced. total: sums the rows' sums of squares [T, 2] over the ranks that share the
+    heads, which hold ``ranks`` times as many."""
+    conv: Optional[torch.Tensor]
+    q_norm: Optional[torch.Tensor]
+    k_norm: Optional[torch.Tensor]
+    tables: Optional[tuple]
+    state: Optional[torch.Tensor]
+    offset: int
+    ranks: int = 1
+    total: Optional[callable] = None
+
+
+def head_prep(x, shape, p, cache, batch):
+    """x: [T, >= shape.qkv_width] projection, q heads | k heads (| v heads). Appends the step's keys and values to ``cache``
+    and returns the queries [T, heads * dim]."""
+    sh, T = shape, x.shape[0]
+    if not native.use_native(x):
+        return _head_prep_cpu(x, sh, p, cache, batch)
+    lib, dev = native.kernels(), x.device
+    cos, sin = p.tables if sh.rot else (None, None)
+    assert x.stride(1) == 1 and cache.dtype == x.dtype and cache.shape[2] == sh.row and x.shape[1] >= sh.qkv_width
+    assert sh.taps == 1 or (p.state is not None and p.offset + sh.state_floats <= p.state.shape[1])
+    assert p.conv is None or (p.conv.shape == (sh.taps, sh.channels) and p.conv.is_contiguous())
+    assert p.q_norm is None or (p.q_norm.numel() == sh.heads * sh.dim and p.k_norm.numel() == sh.kv_heads * sh.dim)
+    assert not sh.rot or cos.shape[1] == sh.rot // 2
+    q = torch.empty(T, sh.heads * sh.dim, dtype=x.dtype, device=dev)
+    tab = batch.block_tables
+
+    def run(out, sums):
+        native.check(
+            lib.hds_head_prep(native.dt(x), x.data_ptr(), x.stride(0), sh.heads, sh.kv_heads, sh.dim, sh.vdim, sh.taps,
+                              sh.rot, int(sh.shared), native.ptr(p.conv), native.ptr(p.q_norm), native.ptr(p.k_norm),
+                              native.ptr(cos), native.ptr(sin), q.data_ptr(), q.stride(0), cache.data_ptr(),
+                              tab.data_ptr(), tab.shape[1], cache.shape[1], batch.tok_seq.data_ptr(),
+                              batch.tok_pos.data_ptr(), batch.seq_meta.data_ptr(),
+                              None if p.state is None else p.state.data_ptr() + 4 * p.offset,
+                              0 if p.state is None else p.state.stride(0), batch.slots.data_ptr(), native.ptr(out),
+                              native.ptr(sums), p.ranks * sh.heads * sh.dim, p.ranks * sh.kv_heads * sh.dim,
+                              float(sh.eps), T, batch.current_sequences, batch.max_new, native.stream()), "head_prep")
+
+    sums = None
+    if p.ranks > 1 and p.q_norm is not None:
+        sums = torch.empty(T, 2, dtype=torch.float32, device=dev)
+        run(sums, None)
+        sums = p.total(sums)
+    run(None, sums)
+    return q
+
+
+def _head_prep_cpu(x, sh, p, cache, batch):
+    T, C, taps = x.shape[0], sh.channels, sh.taps
+    u = x[:, :C].float()
+    if p.conv is not None:
+        raw, u = u, torch.zeros(T, C)
+        for s, (q0, n, seen) in enumerate(batch.seq_meta_host):
+            ring = None
+            if taps > 1:
+                ring = p.state[batch.slots_host[s], p.offset:p.offset + sh.state_floats].view(taps, C)
+            for t in range(n):
+                pos = seen + t
+                if ring is None:
+                    u[q0 + t] = p.conv[0] * raw[q0 + t]
+                    continue
+                ring[pos % taps] = raw[q0 + t]
+                u[q0 + t] = sum(p.conv[taps - 1 - k] * ring[(pos - k) % taps] for k in range(min(taps, pos + 1)))
+    q, k = u.split([sh.heads * sh.dim, sh.kv_heads * sh.dim], 1)
+    v = k if sh.shared else x[:, C:sh.qkv_width].float()
+    if p.q_norm is not None:
+        sums = torch.stack([(q * q).sum(1), (k * k).sum(1)], 1)
+        if p.ranks > 1:
+            sums = p.total(sums)
+        q, k = (a / torch.sqrt(sums[:, j:j + 1] / (p.ranks * a.shape[1]) + sh.eps) * w
+                for j, (a, w) in enumerate(((q, p.q_norm), (k, p.k_norm))))
+    if sh.rot:
+        pos, h = batch.tok_pos.long(), sh.rot // 2
+        c, s = (t[pos][:, None, :h] for t in p.tables)
+
+        def turned(a):
+            a = a.reshape(T, -1, sh.dim).clone()
+            x0, x1 = a[..., 0:sh.rot:2].clone(), a[..., 1:sh.rot:2].clone()
+            a[..., 0:sh.rot:2], a[..., 1:sh.rot:2] = x0 * c - x1 * s, x1 * c + x0 * s
+            return a.reshape(T, -1)
+
+        q, k = turned(q), turned(k)
+    copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
+    return q.to(x.dtype)
+
+
+def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, values=None, mix=None, gate=None,
+                   prep=None):
     """qkv: [T, >= shape.width] projection, row by row q heads | k heads | v heads | gates (consumed); or with ``gate``
     [T, heads * gate_width] without the gates. q_norm / k_norm:
     [dim] float32 or None; sink: [heads] float32 or None; cache: [blocks, block_size, shape.row]. Appends the step's keys
     and values to ``cache`` and writes the gated heads into ``out`` [T, heads * vdim] (unit column stride). ``values``:
-    [T, kv_heads * vdim] values of another layer, of which the share ``mix`` ([1] float32) goes into this layer's."""
+    [T, kv_heads * vdim] values of another layer, of which the share ``mix`` ([1] float32) goes into this layer's. ``prep`` (a HeadPrep, for shapes with
+    ``prep``): q and k are convolved, normed and rotated first (q_norm, k_norm, values unused)."""
     sh, T = shape, qkv.shape[0]
     if sh.gated and gate is None:
         gate = qkv[:, sh.qkv_width:sh.width]
+    assert sh.prep == (prep is not None)
+    if prep is not None:
+        qkv = head_prep(qkv, sh, prep, cache, batch)
     if not native.use_native(qkv):
         return _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values, mix, gate)
     lib, st, dt = native.kernels(), native.stream(), native.dt(qkv)
     bs, tab = cache.shape[1], batch.block_tables
     mb = tab.shape[1]
     assert qkv.stride(1) == 1 and out.stride(1) == 1 and cache.dtype == qkv.dtype == out.dtype
-    assert cache.shape[2] == sh.row and qkv.shape[1] >= sh.qkv_width and out.shape[1] == sh.heads * sh.vdim
-    native.check(
-        lib.hds_head_norm_scatter(dt, qkv.data_ptr(), qkv.stride(0), native.ptr(q_norm), native.ptr(k_norm),
-                                  cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(),
-                                  T, mb, bs, sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.eps),
-                                  native.ptr(values), 0 if values is None else values.stride(0),
-                                  None if values is None else mix.data_ptr(), st),
-        "head_norm_scatter")
+    assert cache.shape[2] == sh.row and out.shape[1] == sh.heads * sh.vdim
+    assert qkv.shape[1] >= (sh.heads * sh.dim if sh.prep else sh.qkv_width)
+    if not sh.prep:
+        native.check(
+            lib.hds_head_norm_scatter(dt, qkv.data_ptr(), qkv.stride(0), native.ptr(q_norm), native.ptr(k_norm),
+                                      cache.data_ptr(), batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(),
+                                      tab.data_ptr(), T, mb, bs, sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.eps),
+                                      native.ptr(values), 0 if values is None else values.stride(0),
+                                      None if values is None else mix.data_ptr(), st), "head_norm_scatter")
     assert not sh.gated or (gate.shape == (T, sh.heads * sh.gate_width) and gate.stride(1) == 1 and gate.dtype == qkv.dtype)
     gp, ldg = (gate.data_ptr(), gate.stride(0)) if sh.gated else (None, 0)
     assert values is None or (values.shape == (T, sh.kv_heads * sh.vdim) and values.dtype == qkv.dtype)
@@ -302,13 +418,13 @@ def head_attention(qkv, shape, q_norm, k_norm, sink, cache, batch, plan, out, va
                                  out.stride(0), native.ptr(part_o), native.ptr(part_ml), None, native.ptr(plan.toks),
                                  batch.tok_seq.data_ptr(), batch.tok_pos.data_ptr(), tab.data_ptr(), mb, bs, n,
                                  sh.heads, sh.kv_heads, sh.dim, sh.vdim, splits, float(sh.scale), sh.window,
-                                 sh.chunk, float(sh.softcap), native.ptr(sink), gp, ldg, sh.gate_width,
+                                 sh.chunk, sh.keep, float(sh.softcap), native.ptr(sink), gp, ldg, sh.gate_width,
                                  None, st), "paged_decode")
     if plan.n_atoms:
         native.check(
             lib.hds_paged_attn(qkv.data_ptr(), qkv.stride(0), cache.data_ptr(), out.data_ptr(), out.stride(0),
                                plan.atoms.data_ptr(), plan.n_atoms, batch.seq_meta.data_ptr(), tab.data_ptr(), mb, bs,
-                               sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, sh.chunk,
+                               sh.heads, sh.kv_heads, sh.dim, sh.vdim, float(sh.scale), sh.window, sh.chunk, sh.keep,
                                float(sh.softcap), native.ptr(sink), gp, ldg, sh.gate_width, st),
             "paged_attn")
     return out
@@ -320,12 +436,15 @@ def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values
     def normed(v, w):
         return v if w is None else v / torch.sqrt((v * v).mean(-1, keepdim=True) + sh.eps) * w
 
-    q, k, v = qkv[:, :sh.qkv_width].float().split([H * sh.dim, G * sh.dim, G * sh.vdim], 1)
-    q = normed(q.reshape(T, H, sh.dim), q_norm)
-    k = normed(k.reshape(T, G, sh.dim), k_norm).reshape(T, -1)
-    if values is not None:
-        v = (1 - mix) * v + mix * values.float()
-    copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
+    if sh.prep:
+        q = qkv.float().reshape(T, H, sh.dim)
+    else:
+        q, k, v = qkv[:, :sh.qkv_width].float().split([H * sh.dim, G * sh.dim, G * sh.vdim], 1)
+        q = normed(q.reshape(T, H, sh.dim), q_norm)
+        k = normed(k.reshape(T, G, sh.dim), k_norm).reshape(T, -1)
+        if values is not None:
+            v = (1 - mix) * v + mix * values.float()
+        copy_rows(cache, torch.cat([k, v], 1), batch.tok_seq, batch.tok_pos, batch.block_tables, to_cache=True)
     gate = torch.sigmoid(gate.float()).reshape(T, H, sh.gate_width) if sh.gated else torch.ones(T, H, 1)
     bs = cache.shape[1]
     for s, (q0, n, seen) in enumerate(batch.seq_meta_host):
@@ -334,7 +453,7 @@ def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values
         lo = max(0, seen - sh.window + 1) if sh.window else 0
         if sh.chunk:
             lo = max(lo, seen - seen % sh.chunk)
-        j = torch.arange(lo, seen + n)
+        j = torch.cat([torch.arange(min(sh.keep, lo)), torch.arange(lo, seen + n)])
         rows = cache[batch.block_tables[s, j // bs].long(), j % bs].float()
         kk = rows[:, :G * sh.dim].view(-1, G, sh.dim).repeat_interleave(H // G, 1)
         vv = rows[:, G * sh.dim:].reshape(-1, G, sh.vdim).repeat_interleave(H // G, 1)
@@ -344,9 +463,9 @@ def _head_attention_cpu(qkv, sh, q_norm, k_norm, sink, cache, batch, out, values
         i = seen + torch.arange(n)
         hide = j[None] > i[:, None]
         if sh.window:
-            hide |= j[None] <= i[:, None] - sh.window
+            hide |= (j[None] <= i[:, None] - sh.window) & (j[None] >= sh.keep)
         if sh.chunk:
-            hide |= j[None] < (i - i % sh.chunk)[:, None]
+            hide |= (j[None] < (i - i % sh.chunk)[:, None]) & (j[None] >= sh.keep)
         sc = sc.masked_fill(hide[None], float("-inf"))
         if sink is not None:
             sc = torch.cat([sc, sink.view(H, 1, 1).expand(H, n, 1)], -1)
