@@ -114,7 +114,8 @@ def main():
     ap.add_argument("--serving", default=None, metavar="MODELS",
                     help="instead of the training step: prefill and decode throughput of the ragged serving engine, "
                     "comma-separated from llama, gofasun, gofasun-mingru, gofasun-latent, qwen2-moe, buvuzen, "
-                    "fifotar, fifotar-delta, fifotar-latent, fifotar-attention (one JSON line each)")
+                    "fifotar, fifotar-delta, fifotar-latent, fifotar-attention, duzizen, duzizen-mlstm, duzizen-parallel, "
+                    "duzizen-moe (one JSON line each)")
     ap.add_argument("--serving-sizes", default="2048,4096", help="layer widths of --serving")
     ap.add_argument("--serving-layers", type=int, default=8)
     ap.add_argument("--serving-prompt", type=int, default=4096)

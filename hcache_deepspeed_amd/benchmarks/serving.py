@@ -1,6 +1,6 @@
 """Prefill and decode throughput of the ragged serving engine on random weights of a real model's layer sizes: the hybrid
-designs (Gofasun, Fifotar) next to the dense Llama layout at equal width, depth, feed-forward and head count, and the
-post-norm routed design (Buvuzen) next to the Qwen2-MoE layout at equal width, depth, heads and experts
+designs (Gofasun, Fifotar, Duzizen) next to the dense Llama layout at equal width, depth, feed-forward and head count, and
+the routed designs (Buvuzen, duzizen-moe) next to the Qwen2-MoE layout at equal width, depth, heads and experts
 (``bench.py --serving``). One JSON line per measurement."""
 import json
 import time
@@ -163,6 +163,64 @@ def fifotar_model(size, layers, dev, kinds=FIFOTAR):
     return spec, convert_hf(w, spec)
 
 
+DUZIZEN = ("mlstm", "parallel")
+KEPT, SIDE, BUCKETS = 64, 256, 32768
+
+
+def duzizen_model(size, layers, dev, kinds=DUZIZEN, routed=False):
+    """A parallel layer has half of the heads in each of its mixers."""
+    from ..inference.v2.arch import convert_hf, spec_from_hf
+    W, ff, H, G = SIZES[size]
+    E, top, eff, _ = EXPERTS[size]
+    taps, h, g2 = 4, H // 2, G // 2
+    mixers = {"mlstm": {"heads": H, "dim": HEAD, "vdim": HEAD, "gate_cap": 15.0},
+              "parallel": {"left": {"heads": h, "kv_heads": g2, "dim": HEAD, "vdim": HEAD, "conv": taps, "scale": HEAD**-0.5,
+                                    "mask": {"size": WINDOW, "keep_first": KEPT},
+                                    "rot": {"base": 500000.0, "dims": ROT, "scaling": {
+                                        "factor": 8.0, "low": 1.0, "high": 4.0, "original": 4096}}},
+                           "right": {"heads": h, "dim": HEAD, "vdim": HEAD, "decay": [1 - 0.5**(5 + 0.25 * i) for i in range(h)],
+                                     "rot": {"base": 10000.0, "dims": HEAD}}}}
+    mlp = {"kind": "moe", "router": {"experts": E, "top": top}, "expert": {"ff": eff, "limit": 7.0}} if routed else \
+        {"kind": "dense", "ff": ff}
+    cfg = {"architecture": "Duzizen", "vocab": VOCAB, "width": W, "norm": {"eps": 1e-5}, "token_side": {"dim": SIDE},
+           "embedding": {"bigram": {"buckets": BUCKETS, "mul_prev": 7919, "mul_cur": 31}},
+           "layers": [{"type": kinds[i % len(kinds)], "mixer": mixers[kinds[i % len(kinds)]], "mlp": mlp}
+                      for i in range(layers)]}
+    g = torch.Generator(device=dev).manual_seed(0)
+    one, zero = torch.ones(W, device=dev), torch.zeros(W, device=dev)
+    w = {"embed": _rand(g, dev, VOCAB, W), "head": _rand(g, dev, VOCAB, W), "bigram": _rand(g, dev, BUCKETS + 1, W),
+         "side.embed": _rand(g, dev, VOCAB, SIDE * layers, scale=1.0), "final.norm": one, "final.norm.b": zero}
+    for i, e in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        for k in ("norm1", "norm1b", "norm2", "norm2b"):
+            w[p + k], w[p + k + ".b"] = one, zero
+        w[p + "side.norm"] = one
+        shapes = {"side.gate": (SIDE, W), "side.proj": (W, SIDE)}
+        if routed:
+            shapes["mlp.router"] = (E, W)
+            for x in range(E):
+                shapes.update({f"mlp.e{x}.gate": (eff, W), f"mlp.e{x}.up": (eff, W), f"mlp.e{x}.down": (W, eff)})
+        else:
+            shapes.update({"mlp.gate": (ff, W), "mlp.up": (ff, W), "mlp.down": (W, ff)})
+        if e["type"] == "mlstm":
+            shapes.update({f"mix.{k}": (H * HEAD, W) for k in "qkvg"})
+            shapes.update({"mix.o": (W, H * HEAD), "mix.i": (H, W), "mix.f": (H, W)})
+            w[p + "mix.norm"] = torch.ones(H * HEAD, device=dev)
+            w[p + "mix.i.b"], w[p + "mix.f.b"] = torch.zeros(H, device=dev), torch.full((H, ), 4.0, device=dev)
+        else:
+            for k, n in (("q", h * HEAD), ("k", g2 * HEAD)):
+                shapes[f"mix.left.{k}"] = (n, W)
+                w[f"{p}mix.left.{k}.conv"] = _rand(g, dev, n, taps, scale=0.5)
+                w[f"{p}mix.left.{k}.norm"] = torch.ones(n, device=dev)
+            shapes.update({f"mix.right.{k}": (h * HEAD, W) for k in "qkvg"})
+            shapes.update({"mix.left.o": (W, h * HEAD), "mix.right.o": (W, h * HEAD)})
+            w[p + "mix.left.out"], w[p + "mix.right.out"] = one, one
+        for k, s in shapes.items():
+            w[p + k] = _rand(g, dev, *s)
+    spec = spec_from_hf(cfg)
+    return spec, convert_hf(w, spec)
+
+
 def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
     from ..inference.v2.engine import InferenceEngineV2, RaggedInferenceEngineConfig
     if kind == "llama":
@@ -175,6 +233,9 @@ def _engine(kind, size, layers, dev, batch, max_context, max_batch_tokens):
         kinds = {"fifotar": FIFOTAR, "fifotar-delta": ("delta", ), "fifotar-latent": ("latent_attention", ),
                  "fifotar-attention": ("attention", )}[kind]
         spec, w = fifotar_model(size, layers, dev, kinds)
+    elif kind.startswith("duzizen"):
+        kinds = {"duzizen-mlstm": ("mlstm", ), "duzizen-parallel": ("parallel", )}.get(kind, DUZIZEN)
+        spec, w = duzizen_model(size, layers, dev, kinds, routed=kind == "duzizen-moe")
     else:
         kinds = {"gofasun": ("mingru", "latent_attention"), "gofasun-mingru": ("mingru", ),
                  "gofasun-latent": ("latent_attention", )}[kind]

@@ -313,11 +313,13 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
   }
   for (int a0 = tid; a0 < n; a0 += 1024 * U) {
     int e[U], r[U];
+    float wt[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       const int a = min(a0 + 1024 * u, n - 1);
       e[u] = expert[a];
       r[u] = row[a];  // written by this thread above
+      wt[u] = row_weight != nullptr ? weight[a] : 0.f;
     }
 #pragma unroll
     for (int u = 0; u < U; ++u) {
@@ -325,7 +327,7 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
       if (a >= n || r[u] < 0) continue;
       row[a] = start[e[u]] + r[u];
       token[start[e[u]] + r[u]] = a / k;
-      if (row_weight != nullptr) row_weight[start[e[u]] + r[u]] = weight[a];
+      if (row_weight != nullptr) row_weight[start[e[u]] + r[u]] = wt[u];
     }
   }
 }

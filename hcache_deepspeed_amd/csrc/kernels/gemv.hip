@@ -26,10 +26,24 @@ __device__ __forceinline__ float dot8(const bf16x8& a, const bf16x8& b, float c)
   return c;
 }
 
-template <int MAXM, int R>
+__device__ __forceinline__ float gate_f(float v, int act);
+
+// Optional last step of the kernels below (GATHER): y[m, n] = act(y[m, n]) * table[ids[m], n]
+struct Gather {
+  const bf16* table;  // [vocab, ld]
+  int64_t ld;
+  const int64_t* ids;
+  int vocab, act;
+  __device__ __forceinline__ float operator()(float v, int m, int n) const {
+    const int64_t id = min(max(ids[m], (int64_t)0), (int64_t)vocab - 1);
+    return gate_f((float)(bf16)v, act) * (float)table[id * ld + n];  // (the product rounded, as the separate kernel reads it)
+  }
+};
+
+template <int MAXM, int R, bool GATHER>
 __global__ __launch_bounds__(256) void gemv_bf16_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
                                                         const bf16* __restrict__ bias, bf16* __restrict__ y, int M,
-                                                        int N, int K, int64_t ldx, int64_t ldy) {
+                                                        int N, int K, int64_t ldx, int64_t ldy, Gather gather) {
   const int lane = threadIdx.x & 63;
   const int n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * R;
   if (n0 >= N) return;
@@ -80,6 +94,7 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const bf16* __restrict__
         float v = wave_sum(acc[r][m]);
         if (lane == 0) {
           if (bias) v += (float)bias[n0 + r];
+          if constexpr (GATHER) v = gather(v, m, n0 + r);
           y[m * ldy + n0 + r] = (bf16)v;
         }
       }
@@ -251,10 +266,10 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16* __restrict_
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-template <int U>
+template <int U, bool GATHER>
 __global__ __launch_bounds__(256) void skinny_mfma_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
                                                           const bf16* __restrict__ bias, bf16* __restrict__ y, int M,
-                                                          int N, int K, int64_t ldx, int64_t ldy) {
+                                                          int N, int K, int64_t ldx, int64_t ldy, Gather gather) {
   __shared__ f32x4 red[3][64];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int n0 = blockIdx.x * 16;
@@ -297,6 +312,7 @@ __global__ __launch_bounds__(256) void skinny_mfma_kernel(const bf16* __restrict
         if (n < N) {
           float v = acc[r];
           if (bias) v += (float)bias[n];
+          if constexpr (GATHER) v = gather(v, tok, n);
           y[(int64_t)tok * ldy + n] = (bf16)v;
         }
       }
@@ -408,14 +424,14 @@ HDS_EXPORT int hds_skinny_gemm_bf16(const void* x, const void* w, const void* bi
                                     int64_t ldx, int64_t ldy, hipStream_t st) {
   if (M < 1 || M > 16 || N < 1 || K < 128 || K % 128 || ldx % 8) return hipErrorInvalidValue;
   if (g_skinny_u == 32 && (K >> 2) % 1024 == 0)
-    hipLaunchKernelGGL(skinny_mfma_kernel<32>, dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
-                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy);
+    hipLaunchKernelGGL((skinny_mfma_kernel<32, false>), dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
+                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy, Gather{});
   else if (g_skinny_u >= 16)
-    hipLaunchKernelGGL(skinny_mfma_kernel<16>, dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
-                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy);
+    hipLaunchKernelGGL((skinny_mfma_kernel<16, false>), dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
+                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy, Gather{});
   else
-    hipLaunchKernelGGL(skinny_mfma_kernel<8>, dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
-                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy);
+    hipLaunchKernelGGL((skinny_mfma_kernel<8, false>), dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
+                       (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy, Gather{});
   return hipGetLastError();
 }
 
@@ -465,8 +481,8 @@ HDS_EXPORT int hds_gemv_bf16(const void* x, const void* w, const void* bias, voi
   if (!hds_gemv_bf16_supported(M, N, K) || ldx % 8) return hipErrorInvalidValue;
   // R = 4 rows per wave while that still leaves >= 2 waves per SIMD on 256 CUs, else 2 / 1 (parallelism)
 #define HDS_GV(MM, RR)                                                                                        \
-  hipLaunchKernelGGL((gemv_bf16_kernel<MM, RR>), dim3((N + 4 * RR - 1) / (4 * RR)), dim3(256), 0, st,        \
-                     (const bf16*)x, (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy)
+  hipLaunchKernelGGL((gemv_bf16_kernel<MM, RR, false>), dim3((N + 4 * RR - 1) / (4 * RR)), dim3(256), 0, st, \
+                     (const bf16*)x, (const bf16*)w, (const bf16*)bias, (bf16*)y, M, N, K, ldx, ldy, Gather{})
 #define HDS_GVM(RR)                                                                                           \
   if (M == 1) HDS_GV(1, RR); else if (M <= 2) HDS_GV(2, RR); else if (M <= 4) HDS_GV(4, RR); else HDS_GV(8, RR);
   if (N >= 8192) {
@@ -478,5 +494,23 @@ HDS_EXPORT int hds_gemv_bf16(const void* x, const void* w, const void* bias, voi
   }
 #undef HDS_GVM
 #undef HDS_GV
+  return hipGetLastError();
+}
+
+// y[M, N] = act(x . W^T) * table[ids[m], :N] (act: 0 silu, 1 gelu_tanh, 2 relu) for up to 16 rows: one row takes the GEMV
+// (K % 8 == 0), more the skinny GEMM (K % 128 == 0). 16-B aligned x and w.
+HDS_EXPORT int hds_gather_gemv_bf16(const void* x, const void* w, const void* table, int64_t ldt, const int64_t* ids,
+                                    int vocab, int act, void* y, int M, int N, int K, int64_t ldx, int64_t ldy,
+                                    hipStream_t st) {
+  if (M < 1 || M > 16 || N < 1 || K < 8 || K % (M == 1 ? 8 : 128) || ldx % 8 || ldx < K || ldt < N || ldy < N ||
+      vocab < 1 || act < 0 || act > 2 || table == nullptr || ids == nullptr)
+    return hipErrorInvalidValue;
+  const Gather gather{(const bf16*)table, ldt, ids, vocab, act};
+  if (M == 1)
+    hipLaunchKernelGGL((gemv_bf16_kernel<1, 1, true>), dim3((N + 3) / 4), dim3(256), 0, st, (const bf16*)x,
+                       (const bf16*)w, (const bf16*)nullptr, (bf16*)y, M, N, K, ldx, ldy, gather);
+  else
+    hipLaunchKernelGGL((skinny_mfma_kernel<16, true>), dim3((N + 15) / 16), dim3(256), 0, st, (const bf16*)x,
+                       (const bf16*)w, (const bf16*)nullptr, (bf16*)y, M, N, K, ldx, ldy, gather);
   return hipGetLastError();
 }

@@ -121,31 +121,43 @@ __device__ __forceinline__ float rotated(const MemoryParams<T>& p, const T* x, i
   return e & 1 ? v * c + u * s : v * c - u * s;
 }
 
-// eight neighbouring elements from e (a multiple of 8)
-template <typename T>
-__device__ __forceinline__ void rotated8(const MemoryParams<T>& p, const T* x, int e, int pos, float (&v)[8]) {
-  Vec8<T>::load(x + e, v);
-  if (e >= p.d.rot) return;
-  const int half = p.d.rot / 2;
-  const float* cp = p.cos_t + (int64_t)pos * half + e / 2;
-  const float* sp = p.sin_t + (int64_t)pos * half + e / 2;
+// cosines and sines of the four pairs from element e (a multiple of 8) on, at position pos
+struct Turn {
   float c[4], s[4];
-  if ((half & 3) == 0) {
-    VecN<float, 4>::load(cp, c);
-    VecN<float, 4>::load(sp, s);
-  } else {
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const bool on = e / 2 + j < half;
-      c[j] = on ? cp[j] : 1.f;
-      s[j] = on ? sp[j] : 0.f;
-    }
-  }
+};
+template <typename T>
+__device__ __forceinline__ Turn turn_of(const MemoryParams<T>& p, int e, int pos) {
+  const int half = p.d.rot / 2;
+  Turn t;
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const float a = v[2 * j], b = v[2 * j + 1];
-    v[2 * j] = a * c[j] - b * s[j];
-    v[2 * j + 1] = b * c[j] + a * s[j];
+    t.c[j] = 1.f;
+    t.s[j] = 0.f;
+  }
+  if (e >= p.d.rot) return t;
+  const float* cp = p.cos_t + (int64_t)pos * half + e / 2;
+  const float* sp = p.sin_t + (int64_t)pos * half + e / 2;
+  if ((half & 3) == 0) {
+    VecN<float, 4>::load(cp, t.c);
+    VecN<float, 4>::load(sp, t.s);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (e / 2 + j < half) {
+        t.c[j] = cp[j];
+        t.s[j] = sp[j];
+      }
+  }
+  return t;
+}
+// the elements as numbers, turned
+template <bool TURNS>
+__device__ __forceinline__ void turned(const bf16x8& x, const Turn& t, float (&v)[8]) {
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const float a = (float)x[2 * j], b = (float)x[2 * j + 1];
+    v[2 * j] = TURNS ? a * t.c[j] - b * t.s[j] : a;
+    v[2 * j + 1] = TURNS ? b * t.c[j] + a * t.s[j] : b;
   }
 }
 
@@ -495,8 +507,9 @@ __device__ __forceinline__ bf16x8 read_tokens(const bf16* tile, int ld) {
   return __builtin_shufflevector(read_tr(tile, ld), read_tr(tile + 16 * ld, ld), 0, 1, 2, 3, 4, 5, 6, 7);
 }
 
-// KT: 16-row tiles of the state a wave has (dk <= 64 KT)
-template <int KT>
+// KT: 16-row tiles of the state a wave has (dk <= 64 KT). Everything a thread reads is requested at once.
+// LPV lanes a token of v (dv <= 8 LPV).
+template <int KT, bool TURNS, int LPV>
 __global__ __launch_bounds__(256) void memory_chunk_sum_kernel(MemoryParams<bf16> p, ChunkWs ws) {
   extern __shared__ __attribute__((aligned(16))) bf16 lds[];  // k e^(..) in three planes [64][ldk], v [64][ldv]
   __shared__ float sw[kChunk];
@@ -511,6 +524,26 @@ __global__ __launch_bounds__(256) void memory_chunk_sum_kernel(MemoryParams<bf16
   const int pos0 = s.seen + chunk * kChunk;
   float* out = ws.at(s, blockIdx.z, chunk, h, d.H);
   bf16* sv = lds + 3 * kChunk * ldk;
+  // missing tokens have weight zero and repeat the last one
+  constexpr int LPK = 8 * KT, NK = 64 * LPK / 256, NV = 64 * LPV / 256;
+  const int ke = 8 * (threadIdx.x % LPK), ve = 8 * (threadIdx.x % LPV);
+  bf16x8 kx[NK], vx[NV];
+  Turn turn[NK];
+#pragma unroll
+  for (int y = 0; y < NK; ++y) {
+    const int tt = min((int)threadIdx.x / LPK + y * (256 / LPK), left - 1), e = ke;
+    kx[y] = bf16x8{};
+    if (e < dk) {
+      kx[y] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + tt) * d.ld + d.k0() + h * dk + e);
+      if (TURNS) turn[y] = turn_of(p, e, pos0 + tt);
+    }
+  }
+#pragma unroll
+  for (int y = 0; y < NV; ++y) {
+    const int tt = min((int)threadIdx.x / LPV + y * (256 / LPV), left - 1);
+    vx[y] = bf16x8{};
+    if (ve < dv) vx[y] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + tt) * d.ld + d.v0() + h * dv + ve);
+  }
   if (w == 0) {
     float f = 0.f, i = -INFINITY, G, P;
     if (lane < left) log_gates(p, t0 + lane, h, f, i);
@@ -525,27 +558,25 @@ __global__ __launch_bounds__(256) void memory_chunk_sum_kernel(MemoryParams<bf16
     }
   }
   __syncthreads();
-  // missing tokens have weight zero and repeat the last one
-  const int k8 = kp / 8, v8 = vp / 8;
-  for (int x = threadIdx.x; x < kChunk * k8; x += 256) {
-    const int t = x / k8, e = 8 * (x - t * k8);
-    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (e < dk) {
-      const int tt = min(t, left - 1);
-      rotated8(p, p.proj + (t0 + tt) * d.ld + d.k0() + h * dk, e, pos0 + tt, v);
+#pragma unroll
+  for (int y = 0; y < NK; ++y) {
+    const int t = threadIdx.x / LPK + y * (256 / LPK), e = ke;
+    if (e < kp) {
+      float v[8];
+      turned<TURNS>(kx[y], turn[y], v);
+      const float f = sw[t];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = e < dk ? v[j] * f : 0.f;
+      bf16x8 pl[3];
+      split8<3>(v, pl);
+#pragma unroll
+      for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8*>(lds + (k * kChunk + t) * ldk + e) = pl[k];
     }
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] *= sw[t];
-    bf16x8 pl[3];
-    split8<3>(v, pl);
-#pragma unroll
-    for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8*>(lds + (k * kChunk + t) * ldk + e) = pl[k];
   }
-  for (int x = threadIdx.x; x < kChunk * v8; x += 256) {
-    const int t = x / v8, e = 8 * (x - t * v8);
-    bf16x8 v = {};
-    if (e < dv) v = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + min(t, left - 1)) * d.ld + d.v0() + h * dv + e);
-    *reinterpret_cast<bf16x8*>(sv + t * ldv + e) = v;
+#pragma unroll
+  for (int y = 0; y < NV; ++y) {
+    const int t = threadIdx.x / LPV + y * (256 / LPV);
+    if (ve < vp) *reinterpret_cast<bf16x8*>(sv + t * ldv + ve) = vx[y];
   }
   __syncthreads();
   bf16x8 a[KT][2][3];
@@ -570,12 +601,12 @@ __global__ __launch_bounds__(256) void memory_chunk_sum_kernel(MemoryParams<bf16
     }
     if (c + l15 < dv)
 #pragma unroll
-      for (int r = 0; r < KT; ++r)
+      for (int r = 0; r < KT; ++r) {
+        const int row = 16 * (w + 4 * r) + 4 * g;  // (dk is a multiple of 8)
+        if (row < dk)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int row = 16 * (w + 4 * r) + 4 * g + j;
-          if (row < dk) out[(int64_t)row * dv + c + l15] = acc[r][j];
-        }
+          for (int j = 0; j < 4; ++j) (out + j * dv)[(uint32_t)(row * dv + c + l15)] = acc[r][j];
+      }
   }
   if (d.gated)
     for (int e = threadIdx.x; e < dk; e += 256) {
@@ -643,10 +674,10 @@ __device__ __forceinline__ void piece_products(F&& f) {
 // in the norm. First the 64 x 64 matrix A, wave (block of 16 queries, half of the blocks of 16 keys), then every wave takes 16
 // columns of the head.
 template <int KS, int PL, int LPU>
-__global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<bf16> p, ChunkWs ws) {
+__global__ __launch_bounds__(512, PL == 1 && LPU <= 16 ? 4 : 2) void memory_chunk_out_kernel(MemoryParams<bf16> p, ChunkWs ws) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   constexpr int ldq = 32 * KS + kPadRow, lda = kChunk + kPadRow;
-  __shared__ float rows[2][kChunk], s_alpha[kChunk], s_inv[kChunk];
+  __shared__ float rows[2][kChunk], s_alpha[kChunk], s_inv[kChunk], s_row[kChunk], s_col[kChunk], s_floor[kChunk];
   const Seq s = seq_of(p, blockIdx.z);
   const int chunk = blockIdx.x, h = blockIdx.y, left = s.n - chunk * kChunk;
   if (left <= 0) return;
@@ -661,63 +692,124 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
   bf16* sv = sa + 3 * kChunk * lda;              // [64][ldv]
   float* so = reinterpret_cast<float*>(smem);    // [64][ldo], when q and A have been read
   const float scale = 1.f / sqrtf((float)dk);
-  // rows past the end repeat the last one: they are not stored
-  for (int x = threadIdx.x; x < kChunk * 4 * KS; x += 512) {
-    const int t = x / (4 * KS), e = 8 * (x - t * 4 * KS), tt = min(t, left - 1);
-    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (e < dk) rotated8(p, p.proj + (t0 + tt) * d.ld + h * dk, e, pos0 + tt, v);
-    bf16x8 pl[PL];
-    split8<PL>(v, pl);
+  constexpr bool TURNS = PL > 1;
+  // Everything a thread reads is requested at once (the keys' cosines apart). Rows past the end repeat the last one: they are
+  // not stored.
+  constexpr int NQ = (KS + 1) / 2, NV = LPU / 8, NG = LPU / 8;
+  const int ge = 8 * (threadIdx.x % LPU);  // columns of v and of the gate
+  bf16x8 qx[NQ], vx[NV], kx[2][KS], gx[NG];
+  Turn turn[NQ];
 #pragma unroll
-    for (int k = 0; k < PL; ++k) *reinterpret_cast<bf16x8*>(sq + (k * kChunk + t) * ldq + e) = pl[k];
+  for (int y = 0; y < NQ; ++y) {
+    const int x = threadIdx.x + 512 * y, t = x / (4 * KS), e = 8 * (x - t * 4 * KS), tt = min(t, left - 1);
+    qx[y] = bf16x8{};
+    if (e < dk && t < kChunk) {
+      qx[y] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + tt) * d.ld + h * dk + e);
+      if (TURNS) turn[y] = turn_of(p, e, pos0 + tt);
+    }
   }
-  for (int x = threadIdx.x; x < kChunk * (vp / 8); x += 512) {
-    const int t = x / (vp / 8), e = 8 * (x - t * (vp / 8));
-    bf16x8 v = {};
-    if (e < dv) v = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + min(t, left - 1)) * d.ld + d.v0() + h * dv + e);
-    *reinterpret_cast<bf16x8*>(sv + t * ldv + e) = v;
-  }
-  // factors of token `lane`
-  float G, P;
   float f = 0.f, i = -INFINITY;
-  if (lane < left) log_gates(p, t0 + lane, h, f, i);
-  run_sums(f, i, G, P);
-  const float m_front = front[d.head() + 2], m = G + fmaxf(m_front, P);
-  if (w == 0) s_alpha[lane] = expf(G + m_front - m);
+  if (w == 0 && lane < left) log_gates(p, t0 + lane, h, f, i);
+  const int ib = w & 3, half = w >> 2;  // blocks of 16 queries; of 16 keys
+#pragma unroll
+  for (int y = 0; y < 2; ++y)
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int jb = half + 2 * y, e = 32 * ks + 8 * g;
+      kx[y][ks] = bf16x8{};
+      if (jb <= ib && e < dk)
+        kx[y][ks] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + min(16 * jb + l15, left - 1)) * d.ld + d.k0() + h * dk + e);
+    }
+#pragma unroll
+  for (int y = 0; y < NV; ++y) {
+    const int t = threadIdx.x / LPU + y * (512 / LPU);
+    vx[y] = bf16x8{};
+    if (ge < dv) vx[y] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + min(t, left - 1)) * d.ld + d.v0() + h * dv + ge);
+  }
+  float S0[KS][8];
+  // rows of the state in front, one of columns c .. c + 15 (rows past dk: any others, q is zero there)
+  auto state_at = [&](int c, int ks, float (&x)[8]) {
+    const uint32_t at = min(32 * ks + 8 * g, dk - 8) * dv + min(c + l15, dv - 1);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = (front + j * dv)[at];
+  };
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) state_at(16 * w, ks, S0[ks]);
+#pragma unroll
+  for (int y = 0; y < NG; ++y) {
+    const int t = threadIdx.x / LPU + y * (512 / LPU);
+    gx[y] = bf16x8{};
+    if (ge < dv) gx[y] = *reinterpret_cast<const bf16x8*>(p.proj + (t0 + min(t, left - 1)) * d.ld + d.g0() + h * dv + ge);
+  }
+#pragma unroll
+  for (int y = 0; y < NQ; ++y) {
+    const int x = threadIdx.x + 512 * y, t = x / (4 * KS), e = 8 * (x - t * 4 * KS);
+    if (t < kChunk) {
+      float v[8];
+      turned<TURNS>(qx[y], turn[y], v);
+      if (TURNS && e >= dk)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = 0.f;
+      bf16x8 pl[PL];
+      split8<PL>(v, pl);
+#pragma unroll
+      for (int k = 0; k < PL; ++k) *reinterpret_cast<bf16x8*>(sq + (k * kChunk + t) * ldq + e) = pl[k];
+    }
+  }
+#pragma unroll
+  for (int y = 0; y < NV; ++y) {
+    const int t = threadIdx.x / LPU + y * (512 / LPU);
+    if (ge < vp) *reinterpret_cast<bf16x8*>(sv + t * ldv + ge) = vx[y];
+  }
+  if (w == 0) {  // factors of token `lane`
+    float G, P;
+    run_sums(f, i, G, P);
+    const float m_front = front[d.head() + 2], m = G + fmaxf(m_front, P);
+    s_alpha[lane] = expf(G + m_front - m) * scale;
+    s_row[lane] = G - m;
+    s_col[lane] = i - G;
+    s_floor[lane] = expf(-m);
+  }
   __syncthreads();
   {
-    const int ib = w & 3, half = w >> 2;
     bf16x8 qf[KS][PL];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
       for (int k = 0; k < PL; ++k)
         qf[ks][k] = *reinterpret_cast<const bf16x8*>(sq + (k * kChunk + 16 * ib + l15) * ldq + 32 * ks + 8 * g);
-    const float mi = __shfl(m, 16 * ib + l15, 64), Gi = __shfl(G, 16 * ib + l15, 64);
-    const float Gj = i - G;  // of token `lane`
+    const float fi = s_row[16 * ib + l15];
     float sum = 0.f;
-    for (int jb = half; jb < 4; jb += 2) {
+#pragma unroll
+    for (int y = 0; y < 2; ++y) {
+      const int jb = half + 2 * y;
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       if (jb <= ib) {
         const int tt = min(16 * jb + l15, left - 1);
-        const bf16* kr = p.proj + (t0 + tt) * d.ld + d.k0() + h * dk;
+        Turn kt[KS];
+        if constexpr (TURNS)
+#pragma unroll
+          for (int ks = 0; ks < KS; ++ks) kt[ks] = turn_of(p, 32 * ks + 8 * g, pos0 + tt);
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
-          const int e = 32 * ks + 8 * g;
-          float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-          if (e < dk) rotated8(p, kr, e, pos0 + tt, v);
           bf16x8 kf[PL];
-          split8<PL>(v, kf);
+          if constexpr (TURNS) {
+            float v[8];
+            turned<true>(kx[y][ks], kt[ks], v);
+            split8<PL>(v, kf);
+          } else {
+            kf[0] = kx[y][ks];
+          }
           piece_products<PL, PL>([&](int a, int b) { acc = mfma_bf16(kf[a], qf[ks][b], acc); });
         }
       }
       // lane: query 16 ib + l15, keys 16 jb + 4 g + r
       float a[4];
+      const f32x4 fj = *reinterpret_cast<const f32x4*>(s_col + 16 * jb + 4 * g);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
+      for (int r = 0; r < 4; ++r) {  // (missing keys: a factor of zero)
         const int j = 16 * jb + 4 * g + r;
-        const float wj = __shfl(Gj, j, 64);
-        a[r] = j <= 16 * ib + l15 && j < left ? acc[r] * scale * expf(Gi + wj - mi) : 0.f;
+        a[r] = j <= 16 * ib + l15 ? acc[r] * scale * __expf(fi + fj[r]) : 0.f;
         sum += a[r];
       }
       float rest[4] = {a[0], a[1], a[2], a[3]};
@@ -747,13 +839,12 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
       for (int k = PL - 1; k >= 0; --k) q += (float)sq[(k * kChunk + t) * ldq + e];
       nq += n[e] * q;
     }
-    nq = group_sum<8>(nq) * scale * s_alpha[t] + rows[0][t] + rows[1][t];
-    const float mt = __shfl(m, t, 64);
-    if ((threadIdx.x & 7) == 0) s_inv[t] = 1.f / (fmaxf(fabsf(nq), expf(-mt)) + kFloorEps);
+    nq = group_sum<8>(nq) * s_alpha[t] + rows[0][t] + rows[1][t];
+    if ((threadIdx.x & 7) == 0) s_inv[t] = 1.f / (fmaxf(fabsf(nq), s_floor[t]) + kFloorEps);
   } else if (threadIdx.x < kChunk) {
     s_inv[threadIdx.x] = 1.f;
   }
-  constexpr int kMaxTiles = 2;  // dv <= 256
+  constexpr int kMaxTiles = LPU > 16 ? 2 : 1;  // dv <= 8 LPU
   f32x4 O[kMaxTiles][4];
 #pragma unroll
   for (int x = 0; x < kMaxTiles; ++x) {
@@ -761,21 +852,13 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
 #pragma unroll
     for (int b = 0; b < 4; ++b) O[x][b] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c >= dv) continue;
-    const float* sp = front + min(c + l15, dv - 1);
-    float nx[8];
-    auto fetch = [&](int ks) {
+    if (x > 0)
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int row = 32 * ks + 8 * g + j;
-        nx[j] = row < dk ? sp[(int64_t)row * dv] : 0.f;
-      }
-    };
-    fetch(0);
+      for (int ks = 0; ks < KS; ++ks) state_at(c, ks, S0[ks]);
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       bf16x8 sf[3];
-      split8<3>(nx, sf);
-      if (ks + 1 < KS) fetch(ks + 1);
+      split8<3>(S0[ks], sf);
 #pragma unroll
       for (int b = 0; b < 4; ++b) {
         bf16x8 qf[PL];
@@ -787,7 +870,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
     }
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
-      O[x][b] *= s_alpha[16 * b + l15] * scale;
+      O[x][b] *= s_alpha[16 * b + l15];
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         if (2 * ks > b) continue;
@@ -812,15 +895,15 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
       for (int b = 0; b < 4; ++b) *reinterpret_cast<f32x4*>(so + (16 * b + l15) * ldo + c) = O[x][b] * s_inv[16 * b + l15];
   }
   __syncthreads();
-  const int e = 8 * (threadIdx.x % LPU);
   float nw[8] = {1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f};
-  if (e < dv && p.norm != nullptr) Vec8<float>::load(p.norm + h * dv + e, nw);
-  for (int t = threadIdx.x / LPU; t < kChunk; t += 512 / LPU) {
-    const bool on = t < left && e < dv;
-    float o[8], gt[8], ss = 0.f;
+  if (ge < dv && p.norm != nullptr) Vec8<float>::load(p.norm + h * dv + ge, nw);
+#pragma unroll
+  for (int y = 0; y < NG; ++y) {
+    const int t = threadIdx.x / LPU + y * (512 / LPU);
+    const bool on = t < left && ge < dv;
+    float o[8], ss = 0.f;
     if (on) {
-      Vec8<float>::load(so + t * ldo + e, o);
-      Vec8<bf16>::load(p.proj + (t0 + t) * d.ld + d.g0() + h * dv + e, gt);
+      Vec8<float>::load(so + t * ldo + ge, o);
 #pragma unroll
       for (int x = 0; x < 8; ++x) ss += o[x] * o[x];
     }
@@ -828,8 +911,8 @@ __global__ __launch_bounds__(512, 2) void memory_chunk_out_kernel(MemoryParams<b
     if (!on) continue;
     const float rs = 1.f / sqrtf(ss / (float)dv + p.eps);
 #pragma unroll
-    for (int x = 0; x < 8; ++x) o[x] *= rs * nw[x] * gate_act<bf16>(gt[x], p.act);
-    Vec8<bf16>::store(p.out + (t0 + t) * p.ldo + h * dv + e, o);
+    for (int x = 0; x < 8; ++x) o[x] *= rs * nw[x] * gate_act<bf16>((float)gx[y][x], p.act);
+    Vec8<bf16>::store(p.out + (t0 + t) * p.ldo + h * dv + ge, o);
   }
 }
 
@@ -851,14 +934,20 @@ int allow_lds(K* kernel, int bytes) {
                            : hipSuccess;
 }
 
-template <int KT>
-int launch_chunk_sum(const MemoryParams<bf16>& p, const ChunkWs& ws, dim3 grid, hipStream_t st) {
-  static const int attr = allow_lds(memory_chunk_sum_kernel<KT>, 158 * 1024);
+template <int KT, bool TURNS, int LPV>
+int launch_chunk_sum_as(const MemoryParams<bf16>& p, const ChunkWs& ws, dim3 grid, hipStream_t st) {
+  static const int attr = allow_lds(memory_chunk_sum_kernel<KT, TURNS, LPV>, 158 * 1024);
   if (attr) return attr;
   const int kp = (p.d.dk + 15) / 16 * 16, vp = (p.d.dv + 15) / 16 * 16;
   const size_t lds = sizeof(bf16) * kChunk * (3 * (kp + kPadRow) + vp + kPadRow);
-  hipLaunchKernelGGL(memory_chunk_sum_kernel<KT>, grid, dim3(256), lds, st, p, ws);
+  hipLaunchKernelGGL((memory_chunk_sum_kernel<KT, TURNS, LPV>), grid, dim3(256), lds, st, p, ws);
   return hipGetLastError();
+}
+template <int KT, bool TURNS>
+int launch_chunk_sum(const MemoryParams<bf16>& p, const ChunkWs& ws, dim3 grid, hipStream_t st) {
+  if (p.d.dv <= 64) return launch_chunk_sum_as<KT, TURNS, 8>(p, ws, grid, st);
+  if (p.d.dv <= 128) return launch_chunk_sum_as<KT, TURNS, 16>(p, ws, grid, st);
+  return launch_chunk_sum_as<KT, TURNS, 32>(p, ws, grid, st);
 }
 
 template <int KS, int PL, int LPU>
@@ -882,11 +971,14 @@ int launch_chunk_out_as(const MemoryParams<bf16>& p, const ChunkWs& ws, dim3 gri
 int launch_chunks(const MemoryParams<bf16>& p, float* base, int n_seqs, int max_new, hipStream_t st) {
   const ChunkWs ws{base, chunk_floats(p.d.dk, p.d.dv, p.d.gated)};
   const dim3 grid((max_new + kChunk - 1) / kChunk, p.d.H, n_seqs);
-  if (int e = p.d.dk <= 64 ? launch_chunk_sum<1>(p, ws, grid, st) : launch_chunk_sum<2>(p, ws, grid, st)) return e;
+  const bool turns = p.d.rot > 0;
+  const int sum = p.d.dk <= 64 ? (turns ? launch_chunk_sum<1, true>(p, ws, grid, st) : launch_chunk_sum<1, false>(p, ws, grid, st))
+                               : (turns ? launch_chunk_sum<2, true>(p, ws, grid, st) : launch_chunk_sum<2, false>(p, ws, grid, st));
+  if (sum) return sum;
   hipLaunchKernelGGL(memory_chunk_walk_kernel, dim3((p.d.head() / 4 + 255) / 256, p.d.H, n_seqs), dim3(256), 0, st, p, ws);
   if (const hipError_t e = hipGetLastError()) return e;
   const int ks = p.d.dk <= 32 ? 1 : p.d.dk <= 64 ? 2 : 4;
-  if (p.d.rot > 0) {
+  if (turns) {
     if (ks == 1) return launch_chunk_out_as<1, 3>(p, ws, grid, st);
     if (ks == 2) return launch_chunk_out_as<2, 3>(p, ws, grid, st);
     return launch_chunk_out_as<4, 3>(p, ws, grid, st);

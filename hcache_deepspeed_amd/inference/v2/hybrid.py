@@ -25,6 +25,7 @@ import torch
 
 from ...ops.activations import act_gather
 from ...ops.experts import RouterShape
+from ...ops.gemv import gather_gemv
 from ...ops.output_norm import embed_pairs, norm_rows
 from ...ops.paged import copy_rows
 from .arch import run_order
@@ -33,7 +34,7 @@ from .modules import (DSExpertLayerConfig, DSGatedMLPConfig, DSInputNormConfig, 
                       DSNormConfig, DSUnembedConfig, instantiate_expert_layer, instantiate_gated_mlp,
                       instantiate_input_norm, instantiate_linear, instantiate_mixer, instantiate_output_norm,
                       instantiate_sandwich_norm, instantiate_unembed)
-from .modules.implementations import _PackedWeight
+from .modules.implementations import BlasFPLinear, _PackedWeight
 
 
 class _Run:
@@ -436,8 +437,10 @@ class SandwichTransformer(HybridTransformer):
     def _side(self, i, rows, batch):
         """The layer's own input of every token, gated by the residual."""
         L, lins, n = self.layers[i], self.linears[i], self.spec.token_side
-        g = act_gather(lins["side.gate.w"](rows, L["side.gate.w"]), "gelu_tanh", self.side_embed[:, i * n:(i + 1) * n],
-                       batch.input_ids)
+        gate, w, e = lins["side.gate.w"], L["side.gate.w"], self.side_embed[:, i * n:(i + 1) * n]
+        g = gather_gemv(rows, w, "gelu_tanh", e, batch.input_ids) if isinstance(gate, BlasFPLinear) else None
+        if g is None:
+            g = act_gather(gate(rows, w), "gelu_tanh", e, batch.input_ids)
         return lins["side.proj.w"](g, L["side.proj.w"])
 
 

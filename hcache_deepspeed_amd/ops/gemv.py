@@ -158,3 +158,23 @@ def glu_gemv(x2, w, act, out, limit=0.0):
                                                       w.shape[0] // 2, K,
                                                       x2.stride(0), out.stride(0), native.stream()), "glu_gemv")
     return True
+
+
+_GATHER_ACTS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
+
+
+def gather_gemv(x2, w, act, table, ids):
+    """act(x . w^T) * table[ids] of decode rows (at most 16) in one kernel, [M, N]; table: [vocab, N] with any row stride. None
+    for rows or weights the kernel does not take."""
+    if act not in _GATHER_ACTS or not torch.is_tensor(w) or x2.shape[0] > 16 or not (
+            skinny_ok(x2, w) if x2.shape[0] > 1 else gemv_ok(x2, w)):
+        return None
+    assert table.dtype == x2.dtype and table.stride(1) == 1 and table.shape[1] == w.shape[0]
+    assert ids.dtype == torch.int64 and ids.numel() == x2.shape[0]
+    M, K = x2.shape
+    y = torch.empty(M, w.shape[0], dtype=x2.dtype, device=x2.device)
+    native.check(native.kernels().hds_gather_gemv_bf16(x2.data_ptr(), w.data_ptr(), table.data_ptr(), table.stride(0),
+                                                       ids.data_ptr(), table.shape[0], _GATHER_ACTS[act], y.data_ptr(), M,
+                                                       w.shape[0], K, x2.stride(0), y.stride(0), native.stream()),
+                 "gather_gemv")
+    return y

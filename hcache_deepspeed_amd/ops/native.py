@@ -114,6 +114,7 @@ _KERNEL_SIGS = {
     "hds_gemv_bf16_supported": "iii",
     "hds_gemv_bf16": "pppp" + "iii" + "ll" + "s",
     "hds_gemv_fused_bf16": "ppp" + "f" + "pppp" + "if" + "iii" + "ll" + "s",
+    "hds_gather_gemv_bf16": "ppp" + "l" + "p" + "ii" + "p" + "iii" + "ll" + "s",
     "hds_skinny_gemm_bf16": "pppp" + "iii" + "ll" + "s",
     "hds_skinny_set_unroll": "i",
     "hds_wmix_splits": "iii",

@@ -20,6 +20,7 @@ from hcache_deepspeed_amd.inference.v2.modules import (DSExpertLayerConfig, DSGa
 from hcache_deepspeed_amd.ops import matrix_memory as memory_op
 from hcache_deepspeed_amd.ops.activations import act_gather
 from hcache_deepspeed_amd.ops.experts import ExpertSum, RouterShape, route
+from hcache_deepspeed_amd.ops.gemv import gather_gemv
 from hcache_deepspeed_amd.ops.matrix_memory import MemoryShape, make_memory_plan, matrix_memory, step_ok
 from hcache_deepspeed_amd.ops.output_norm import PairSum, embed_pairs, stream_norm
 from hcache_deepspeed_amd.ops.paged import HeadPrep, HeadShape, head_attention, head_blocks_ok, make_head_plan
@@ -579,6 +580,20 @@ def test_act_gather(run, T, C, layers):
         got = act_gather(x.to(dev)[:, :C], "gelu_tanh", table.to(dev)[:, i * C:(i + 1) * C], ids.to(dev))
         want = oracle.gelu(x[:, :C].double()) * table[ids, i * C:(i + 1) * C].double()
         close(got, want, dtype, bf16=5e-3)
+
+
+@GPU
+@pytest.mark.parametrize("M,W,C", [(1, 40, 24), (1, 4096, 256), (2, 128, 5), (7, 256, 40), (16, 1024, 72)])
+def test_gather_gemv(M, W, C):
+    """The product of decode rows with the activation and the table's row in one kernel: the same numbers as the two."""
+    print(f"gather {M} {W} {C}", flush=True)
+    x, w = (rnd(n, W, seed=s, scale=W**-0.25).to(torch.bfloat16).cuda() for n, s in ((M, 1), (C, 2)))
+    table = rnd(19, 3 * C, seed=3).to(torch.bfloat16).cuda()[:, C:2 * C]
+    ids = torch.randint(0, 19, (M, ), generator=torch.Generator().manual_seed(3))
+    got = gather_gemv(x, w, "gelu_tanh", table, ids.cuda())
+    want = oracle.gelu(x.double().cpu() @ w.double().cpu().T) * table.double().cpu()[ids]
+    close(got, want, torch.bfloat16, bf16=1e-2)
+    assert gather_gemv(x.float(), w.float(), "gelu_tanh", table.float(), ids.cuda()) is None
 
 
 @pytest.mark.parametrize("T", [1, 2, 40])
