@@ -394,8 +394,7 @@ int launch_prep(const PrepParams<T>& p, int n_seqs, int max_new, hipStream_t st)
     const dim3 grid((max_new + R - 1) / R, n_seqs);
 #define HDS_HR(NT, MM, OO) hipLaunchKernelGGL((head_prep_run_kernel<T, NT, MM, OO>), grid, dim3(NT), 0, st, p, R)
 #define HDS_HRM(NT) { if (p.taps <= 4) HDS_HR(NT, 3, 4); else HDS_HR(NT, 7, 2); }
-    if (C <= 2048) HDS_HRM(256) else if (C <= 2560) HDS_HRM(320) else if (C <= 4096) HDS_HRM(512)
-    else if (C <= 5120) HDS_HR(640, 3, 4); else HDS_HR(1024, 3, 4);
+    if (C <= 2048) HDS_HRM(256) else if (C <= 4096) HDS_HRM(512) else HDS_HR(1024, 3, 4);
 #undef HDS_HRM
 #undef HDS_HR
     return hipGetLastError();
