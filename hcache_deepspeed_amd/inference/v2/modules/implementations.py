@@ -19,6 +19,7 @@ from ....ops.experts import PAD, routed_experts
 from ....ops.gated_scan import gated_scan, recur_step, recur_step_ok
 from ....ops.gemv import glu_gemv
 from ....ops.grouped_gemm import moe_ffn_dropless
+from ....ops.head_prep import HeadPrep
 from ....ops.input_norm import input_norm
 from ....ops.latent_attention import LatentShape, can_expand, latent_attention, make_plan
 from ....ops.matrix_memory import MemoryShape, make_memory_plan, matrix_memory
@@ -27,7 +28,7 @@ from ....ops.moe import moe_combine, moe_dispatch, topk_assign, topk_route
 from ....ops.norm import layer_norm, rms_norm
 from ....ops.output_norm import (PairSum, embed_rows, padded, residual_norm, rms_rows, sandwich_norm, softcap_,
                                  stream_norm, sum_experts)
-from ....ops.paged import (HeadPrep, HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
+from ....ops.paged import (HeadShape, head_attention, head_blocks_ok, kv_rope_scatter, make_head_plan,
                            paged_attention)
 from ....ops.quantizer import fp6_linear, int_linear, quantize, quantize_minifloat
 from ....ops.rope import rope_tables

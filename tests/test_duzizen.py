@@ -21,9 +21,10 @@ from hcache_deepspeed_amd.ops import matrix_memory as memory_op
 from hcache_deepspeed_amd.ops.activations import act_gather
 from hcache_deepspeed_amd.ops.experts import ExpertSum, RouterShape, route
 from hcache_deepspeed_amd.ops.gemv import gather_gemv
+from hcache_deepspeed_amd.ops.head_prep import HeadPrep
 from hcache_deepspeed_amd.ops.matrix_memory import MemoryShape, make_memory_plan, matrix_memory, step_ok
 from hcache_deepspeed_amd.ops.output_norm import PairSum, embed_pairs, stream_norm
-from hcache_deepspeed_amd.ops.paged import HeadPrep, HeadShape, head_attention, head_blocks_ok, make_head_plan
+from hcache_deepspeed_amd.ops.paged import HeadShape, head_attention, head_blocks_ok, make_head_plan
 from hcache_deepspeed_amd.ops.rope import rope_inv_freq, rope_tables
 
 from . import duzizen_oracle as oracle
